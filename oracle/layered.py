@@ -1,0 +1,136 @@
+"""Plain numpy (float64) restatement of models whose layers are described one by one (mixer + optional feed-forward): TEST
+INFRASTRUCTURE only, slow on purpose, one function per mechanism, no code shared with the product.
+
+Weights are a dict name -> array ([out, in] for linear maps); ``cfg`` is the parsed config.json.  Every function takes whole
+sequences; ``forward`` runs a prompt from nothing, and ``forward(..., cache=...)`` is deliberately NOT offered: a test that needs
+"prompt then decode" compares the product's steps against rows of one whole-sequence run.
+"""
+from __future__ import annotations
+
+import math
+
+import numpy as np
+
+F = np.float64
+
+
+def gelu_tanh(z):
+    return 0.5 * z * (1.0 + np.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
+def sigmoid(z):
+    return 1.0 / (1.0 + np.exp(-z))
+
+
+def log_sigmoid(z):
+    return -np.logaddexp(0.0, -z)
+
+
+def rms(x, eps):
+    return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + eps)
+
+
+def layer_norm(x, w, eps):
+    mu = np.mean(x, axis=-1, keepdims=True)
+    d = x - mu
+    return d / np.sqrt(np.mean(d * d, axis=-1, keepdims=True) + eps) * w
+
+
+def bigram_rows(tokens, buckets, mul_prev, mul_cur):
+    """Row of the pair table for every position: a hash of (previous, current); the extra last row opens a sequence."""
+    return [buckets if p == 0 else (int(tokens[p - 1]) * mul_prev + int(tokens[p]) * mul_cur) % buckets for p in range(len(tokens))]
+
+
+def rope_frequencies(rot):
+    """(frequency of each pair, factor on cos and sin) with the YaRN blend when ``rot`` has a scaling entry."""
+    n, base = int(rot["dims"]), float(rot["base"])
+    f = np.array([base ** (-2.0 * i / n) for i in range(n // 2)], dtype=F)
+    sc = rot.get("scaling")
+    if not sc:
+        return f, 1.0
+    turn = lambda t: n * math.log(sc["original"] / (2 * math.pi * t)) / (2 * math.log(base))
+    lo, hi = max(math.floor(turn(sc["fast"])), 0), min(math.ceil(turn(sc["slow"])), n - 1)
+    ramp = np.clip((np.arange(n // 2) - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return f / sc["factor"] * ramp + f * (1.0 - ramp), 0.1 * math.log(sc["factor"]) + 1.0
+
+
+def rotate_pairs(x, positions, rot):
+    """x [T, ..., d]: neighbouring pairs (2i, 2i+1) of the first rot.dims values turned by position * frequency."""
+    f, mag = rope_frequencies(rot)
+    n = int(rot["dims"])
+    out = np.array(x, dtype=F)
+    ang = np.asarray(positions, dtype=F).reshape((-1,) + (1,) * (x.ndim - 1)) * f
+    c, s = np.cos(ang) * mag, np.sin(ang) * mag
+    u, v = x[..., 0:n:2], x[..., 1:n:2]
+    out[..., 0:n:2] = u * c - v * s
+    out[..., 1:n:2] = v * c + u * s
+    return out
+
+
+def latent_attention(h, w, mx, eps):
+    """h [T, width] -> [T, width]; w: the layer's mixer tensors by short name."""
+    T, H, d, r, dv, kr = len(h), mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"], mx["kv_rank"]
+    pos = np.arange(T)
+    q = (h @ w["q"].T).reshape(T, H, d + r)
+    dkv = h @ w["dkv"].T
+    c = rms(dkv[:, :kr], eps) * w["dkv.norm"]
+    k_rot = rotate_pairs(dkv[:, kr:], pos, mx["rot"])
+    q_rot = rotate_pairs(q[..., d:], pos, mx["rot"])
+    k = (c @ w["uk"].T).reshape(T, H, d)
+    v = (c @ w["uv"].T).reshape(T, H, dv)
+    gate = sigmoid(h @ w["g"].T)
+    out = np.zeros((T, H, dv), dtype=F)
+    for i in range(T):
+        for n in range(H):
+            s = (k[: i + 1, n] @ q[i, n, :d] + k_rot[: i + 1] @ q_rot[i, n]) * mx["scale"]
+            p = np.exp(s - s.max())
+            out[i, n] = (p / p.sum()) @ v[: i + 1, n] * gate[i, n]
+    return out.reshape(T, H * dv) @ w["o"].T
+
+
+def mlstm(h, w, mx, eps):
+    """The matrix memory, one token after the other, from an empty state."""
+    T, H, d, dv, cap = len(h), mx["heads"], mx["dim"], mx["vdim"], mx["gate_cap"]
+    q = (h @ w["q"].T).reshape(T, H, d) * d ** -0.5
+    k = (h @ w["k"].T).reshape(T, H, d)
+    v = (h @ w["v"].T).reshape(T, H, dv)
+    li = cap * np.tanh((h @ w["i"].T + w["i.b"]) / cap)
+    lf = log_sigmoid(cap * np.tanh((h @ w["f"].T + w["f.b"]) / cap))
+    out = np.zeros((T, H, dv), dtype=F)
+    for n in range(H):
+        S, nv, m = np.zeros((d, dv), dtype=F), np.zeros(d, dtype=F), 0.0
+        for t in range(T):
+            m2 = max(lf[t, n] + m, li[t, n])
+            a, b = math.exp(lf[t, n] + m - m2), math.exp(li[t, n] - m2)
+            m = m2
+            S = a * S + b * np.outer(k[t, n], v[t, n])
+            nv = a * nv + b * k[t, n]
+            out[t, n] = (S.T @ q[t, n]) / (max(abs(nv @ q[t, n]), math.exp(-m)) + 1e-6)
+    out = rms(out, eps).reshape(T, H * dv) * w["norm"] * sigmoid(h @ w["g"].T)
+    return out @ w["o"].T
+
+
+def dense_ff(x, w):
+    return (gelu_tanh(x @ w["gate"].T) * (x @ w["up"].T)) @ w["down"].T
+
+
+MIXERS = {"latent_attention": latent_attention, "mlstm": mlstm}
+
+
+def forward(cfg, weights, tokens, layers_out=None):
+    """Logits [T, vocab] of a whole sequence; layers_out (a list) receives the residual stream after every layer."""
+    W = {k: np.asarray(v, dtype=F) for k, v in weights.items()}
+    eps, m = cfg["norm"]["eps"], cfg["residual_mult"]
+    x = W["embed"][list(tokens)]
+    big = (cfg.get("embedding") or {}).get("bigram")
+    if big:
+        x = x + W["bigram"][bigram_rows(tokens, big["buckets"], big["mul_prev"], big["mul_cur"])]
+    for i, lay in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        sub = lambda g: {k[len(p + g):]: v for k, v in W.items() if k.startswith(p + g)}
+        x = x + m * layer_norm(MIXERS[lay["type"]](x, sub("mix."), lay["mixer"], eps), W[p + "norm1"], eps)
+        if lay["mlp"]:
+            x = x + m * layer_norm(dense_ff(x, sub("mlp.")), W[p + "norm2"], eps)
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return layer_norm(x, W["final.norm"], eps) @ W["head"].T

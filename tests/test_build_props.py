@@ -11,6 +11,7 @@ import __graft_entry__ as graft
 
 CSRC = os.path.join(graft.PKG_DIR, "csrc")
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-mllvm", "-amdgpu-kernarg-preload-count=8",
+         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
          "-Rpass-analysis=kernel-resource-usage", "--cuda-device-only", "-c"]
 
 

@@ -39,14 +39,6 @@ __global__ void valu(float* out, int iters, unsigned long long* cyc) {
       asm volatile("v_and_b32 %0, 0x0f0f0f0f, %0" : "+v"(u2)); asm volatile("v_and_b32 %0, 0x0f0f0f0f, %0" : "+v"(u3));
       asm volatile("v_lshrrev_b32 %0, 4, %0" : "+v"(u0)); asm volatile("v_lshrrev_b32 %0, 4, %0" : "+v"(u1));
       asm volatile("v_lshrrev_b32 %0, 4, %0" : "+v"(u2)); asm volatile("v_lshrrev_b32 %0, 4, %0" : "+v"(u3));
-    } else {  // v_pk_fma_f32
-      typedef float f2 __attribute__((ext_vector_type(2)));
-      f2 p0 = {a0, a1}, p1 = {a2, a3}, p2 = {a4, a5}, p3 = {a6, a7}, m = {1.0001f, 1.0001f}, c = {0.5f, 0.5f};
-      asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(p0) : "v"(m), "v"(c)); asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(p1) : "v"(m), "v"(c));
-      asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(p2) : "v"(m), "v"(c)); asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(p3) : "v"(m), "v"(c));
-      asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(p0) : "v"(m), "v"(c)); asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(p1) : "v"(m), "v"(c));
-      asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(p2) : "v"(m), "v"(c)); asm volatile("v_pk_fma_f32 %0, %0, %1, %2" : "+v"(p3) : "v"(m), "v"(c));
-      a0 = p0.x; a1 = p0.y; a2 = p1.x; a3 = p1.y; a4 = p2.x; a5 = p2.y; a6 = p3.x; a7 = p3.y;
     }
   }
   unsigned long long t1 = __builtin_amdgcn_s_memtime();
@@ -131,15 +123,14 @@ int main() {
   CK(hipMalloc(&outf, 1024 * 1024 * 4)); CK(hipMalloc(&cyc, 4096 * 8)); CK(hipMalloc(&outi, 1024 * 1024 * 16));
   const int iters = 20000;
   hipEvent_t e0, e1; CK(hipEventCreate(&e0)); CK(hipEventCreate(&e1));
-  const char* names[4] = {"v_fma_f32 (8 chains)", "v_cvt_f32_ubyteN", "v_and/v_lshr", "v_pk_fma_f32"};
+  const char* names[3] = {"v_fma_f32 (8 chains)", "v_cvt_f32_ubyteN", "v_and/v_lshr"};
   for (int wps = 1; wps <= 4; wps *= 2) {
     int threads = 256 * wps;  // one workgroup per CU, wps waves per SIMD
-    for (int kind = 0; kind < 4; kind++) {
+    for (int kind = 0; kind < 3; kind++) {
       CK(hipEventRecord(e0, 0));
       if (kind == 0) hipLaunchKernelGGL(valu<0>, dim3(256), dim3(threads), 0, 0, outf, iters, cyc);
       if (kind == 1) hipLaunchKernelGGL(valu<1>, dim3(256), dim3(threads), 0, 0, outf, iters, cyc);
       if (kind == 2) hipLaunchKernelGGL(valu<2>, dim3(256), dim3(threads), 0, 0, outf, iters, cyc);
-      if (kind == 3) hipLaunchKernelGGL(valu<3>, dim3(256), dim3(threads), 0, 0, outf, iters, cyc);
       CK(hipEventRecord(e1, 0));
       CK(hipDeviceSynchronize());
       float ms = 0; CK(hipEventElapsedTime(&ms, e0, e1));
