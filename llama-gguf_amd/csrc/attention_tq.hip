@@ -272,7 +272,7 @@ __global__ void __launch_bounds__(256) attn_tq_partial_kernel(const float* __res
   };
   // the first rows of this wave are requested NOW, ahead of the rotations (row `pos` holds stale bytes until this launch has
   // written it: read anyway — it lies inside the cache — and replaced from LDS below)
-  constexpr int kAhead = 2;
+  constexpr int kAhead = G >= 8 ? 1 : 2;   // (beside 8 heads' 128 accumulators a second row in flight spills)
   const uint32_t base0 = (sp * NW + wave) * RPW;
   unsigned long long kk0[kAhead], vv0[kAhead];
   uint32_t sg0[kAhead];
