@@ -1,0 +1,154 @@
+// layered.h — models whose layers are described one by one (lgh_layer_desc: a mixer and an optional feed-forward), on the engine's own
+// context, step function and graphs (internal).  Kernels: linear_bf16.hip (matrix products), latent_attention.hip, mlstm.hip,
+// layered_misc.hip (embedding, norms); layered.hip assembles them.
+#pragma once
+
+#include "common.h"
+
+namespace lgh {
+
+// A bf16 weight matrix [n][k] kept as it came: rows padded to a multiple of 16, columns to a multiple of 64 (zeros).  Several
+// matrices with the same input lie below one another (SEGMENTS, each starting at a multiple of 16 rows), so that one launch
+// computes them all; a "paired" matrix (feed-forward gate | up) interleaves its two halves in blocks of 16 rows.
+struct LinW {
+  uint16_t* w = nullptr;
+  uint32_t n = 0, k = 0;       // rows (all segments, padded to 16), columns that hold values
+  uint32_t kp = 0;             // row stride in elements, multiple of 64
+  bool paired = false;
+  uint32_t np() const { return (n + 15) / 16 * 16; }
+  size_t bytes() const { return (size_t)n * k * 2; }
+};
+
+// What a decode mat-vec does to its input vector before the product (every workgroup, in LDS)
+enum LinPro : int {
+  LP_COPY = 0,    // x
+  LP_RESID = 1,   // x + mult * layer_norm(y) * nw, also written to xout (the new residual stream)
+  LP_HEAD = 2,    // layer_norm of the same sum, times nw2 (final norm in front of the output projection)
+  LP_MLSTM = 3,   // matrix-memory read-out: numerators / denominators, per-head RMS norm, norm weight, sigmoid gate
+};
+struct LinMv {
+  const uint16_t* w;
+  uint32_t n, kp, k, paired;
+  float* out;                  // [n], paired: [n / 2] = gelu(gate) * up
+  const float* x;
+  const float* y;              // LP_RESID / LP_HEAD: the pending sublayer output
+  const float* nw;             // its norm weight
+  const float* nw2;
+  float* xout;
+  float eps, mult;
+  const float* num;            // LP_MLSTM: [heads][ldo] numerators, column vdim = n . q, column vdim + 1 = exp(-m)
+  const float* gate;
+  uint32_t heads, vdim, ldo;
+};
+hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st);
+constexpr uint32_t kLinMvMaxK = 36864;   // input vectors live in LDS
+
+// Matrix product of a block of tokens: out[m][n] = sum_k x[m][k] * w[n][k].  f32 = true: activations and products in 32-bit
+// (f32 matrix cores), otherwise bf16 activations with f32 accumulation.
+enum LinEpi : int {
+  LE_F32 = 0,     // out: float [M][ldo]
+  LE_ACT = 1,     // out: activation type [M][ldo]
+  LE_GEGLU = 2,   // paired weights: gelu(gate) * up as activation type [M][ldo]
+  LE_HEADS = 3,   // activation type, row n = head * hd + j of token m at out[(head * tcap + m) * ldo + j]
+  LE_HEADS_T = 4, // activation type, transposed per head: out[(head * hrows + j) * ldo + m]
+};
+struct LinGemm {
+  const uint16_t* w;
+  const void* x;               // [M][ldx], columns k..kp of every row are zero
+  void* out;
+  uint32_t n, np, kp, ldx, ldo, M;
+  uint32_t hd, hrows;          // LE_HEADS / LE_HEADS_T
+  uint64_t tcap;
+};
+hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st);
+// upload: rows [row0, row0 + rows) of a bf16 matrix; mode 0 plain, 1 first half of a pair, 2 second half of a pair
+hipError_t lin_pack_launch(const uint16_t* src, uint32_t rows, uint32_t k, uint16_t* dst, uint32_t kp, uint32_t row0, int mode, hipStream_t st);
+// per head [dim][rank] -> [rank][dimp]
+hipError_t lin_transpose_heads_launch(const uint16_t* src, uint32_t heads, uint32_t dim, uint32_t rank, uint16_t* dst, uint32_t dimp, hipStream_t st);
+hipError_t bf16_to_f32_launch(const uint16_t* src, float* dst, uint64_t n, hipStream_t st);
+
+// ---- layered_misc.hip ----
+struct EmbedArgs {
+  const uint16_t* embed;       // [vocab][width] bf16
+  const uint16_t* bigram;      // [buckets + 1][width] or NULL
+  uint32_t width, buckets;
+  uint64_t mul_prev, mul_cur;
+  int* hist;                   // token of every position (the previous token is part of the sequence's state)
+};
+hipError_t layered_embed_launch(const EmbedArgs& a, int* state, float* x, hipStream_t st);
+hipError_t layered_embed_block_launch(const EmbedArgs& a, const int* tokens, uint32_t pos0, uint32_t M, float* x, void* xa, uint32_t ldx, bool f32,
+                                      hipStream_t st);
+// x += mult * layer_norm(y) * w; also as activations
+hipError_t resid_norm_launch(float* x, const float* y, uint32_t ldy, const float* w, float eps, float mult, uint32_t width, uint32_t M, void* xa,
+                             uint32_t ldx, bool f32, hipStream_t st);
+// decode without a consumer: xout = x + mult * layer_norm(y) * w
+hipError_t resid_norm_out_launch(const float* x, const float* y, const float* w, float eps, float mult, uint32_t width, float* xout, hipStream_t st);
+// rows[i] of x, layer-normed with w, as activations
+hipError_t final_norm_rows_launch(const float* x, const int* rows, uint32_t n_rows, const float* w, float eps, uint32_t width, void* xa, uint32_t ldx,
+                                  bool f32, hipStream_t st);
+
+// ---- latent_attention.hip ----
+struct LatentShape {
+  uint32_t heads, dim, rot_dim, rot_n, vdim, rank;
+  uint32_t ldc;                // elements of a cache row: [latent rank | rotated key part rot_dim | zeros], multiple of 32
+  uint32_t dimp, rankp;        // row strides of the transposed key expansion [head][rank][dimp] and the value expansion [head * vdim][rankp]
+  uint32_t off_q, off_dkv, off_g, ldcat;   // where a token's projections lie in its row of the fused product
+  float scale, eps;
+};
+struct LatentBufs {
+  const float* cat;            // [M][ldcat]
+  const float* dkv_norm;       // [rank]
+  const float* cs;             // [max_seq][rot_n / 2][2]
+  const uint16_t *uk_t, *uv;
+  void* cache;                 // [max_seq][ldc]
+  void* qa;                    // [M * heads][ldc]: absorbed queries
+  float *part_ml, *part_acc;   // [split][M * heads][2], [split][M * heads][rank]
+};
+constexpr uint32_t kLatMaxSplits = 64;
+constexpr uint32_t kLatAbsorbRows = 1024;   // (token, head) rows the absorbed path's buffers hold
+// pos_ptr (device) or pos0: position of the first of the M tokens
+hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, bool f32, hipStream_t st);
+hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32,
+                              hipStream_t st);
+// merges the splits, expands the latent to the value and applies the head gate -> out [M][ldo] (f32 vector in decode, activations otherwise)
+hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32cache,
+                             void* out, uint32_t ldo, bool out_f32, hipStream_t st);
+uint32_t latent_key_tile(const LatentShape& s, bool f32, uint32_t M);   // keys per tile of the absorbed kernel (0: does not fit LDS)
+// expanded path (long prompts): keys and values per head
+struct LatentFlash {
+  void* q;                     // [heads][Mcap][dq]
+  void* k;                     // [heads][Tcap][dq]
+  void* vt;                    // [heads][dvp][Tcap]
+  uint32_t dq, dvp, Mcap;
+  uint64_t Tcap;
+};
+bool latent_flash_shape(const LatentShape& s, uint32_t* dq, uint32_t* dvp);
+hipError_t latent_flash_prep_launch(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, bool f32, hipStream_t st);
+hipError_t latent_flash_launch(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, bool f32, void* out,
+                               uint32_t ldo, hipStream_t st);
+
+// ---- mlstm.hip ----
+struct MlstmShape {
+  uint32_t heads, dim, vdim;
+  uint32_t lds;                // row stride of the state [head][dim][lds]: columns 0..vdim-1 = S, column vdim = n
+  uint32_t ldo;                // row stride of the numerators [M][heads][ldo]
+  uint32_t off_q, off_k, off_v, off_g, off_i, off_f, ldcat;
+  float cap, eps;
+};
+struct MlstmBufs {
+  const float* cat;            // [M][ldcat]
+  const float *bi, *bf;        // [heads]
+  const float* norm;           // [heads * vdim]
+  float* S;
+  double* m;                   // [2][heads]: the running maximum before position p lies in half p & 1
+  float* num;                  // [M][heads][ldo]
+  double *u, *mx;              // prompt blocks: [heads][Mcap]
+  float* a;                    // prompt blocks: [chunk][heads][64][64] decayed scores
+  uint32_t Mcap;
+};
+constexpr uint32_t kMlstmMaxDim = 1024;
+hipError_t mlstm_step_launch(const MlstmShape& s, const MlstmBufs& b, const int* pos_ptr, hipStream_t st);
+hipError_t mlstm_block_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t pos0, uint32_t M, hipStream_t st);
+hipError_t mlstm_out_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t M, void* out, uint32_t ldo, bool f32, hipStream_t st);
+
+}  // namespace lgh

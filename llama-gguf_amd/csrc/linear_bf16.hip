@@ -1,0 +1,340 @@
+// linear_bf16.hip — matrix products with weights kept in bf16 (layered.h): the decode mat-vec (weights streamed once, input vector
+// prepared in LDS by every workgroup: residual + layer norm, matrix-memory read-out) and the block product on the matrix cores.
+#include "layered.h"
+#include "layered_device.h"
+
+namespace lgh {
+
+// ------------------------------------------------------------------------------------------------
+// decode mat-vec: a workgroup of 4 waves owns 8 rows at a time; the waves share a row's columns (2048 per pass), every lane keeps
+// 8 rows x 16 bytes in flight.
+// ------------------------------------------------------------------------------------------------
+constexpr int kMvR = 8;
+
+// layer norm of the K values in xs (in place), times w
+__device__ __forceinline__ void ln_lds(float* xs, uint32_t K, const float* w, float eps, float* red) {
+  float s = 0.0f;
+  for (uint32_t i = threadIdx.x; i < K; i += 256) s += xs[i];
+  const float mean = block_sum(s, red) / (float)K;
+  float v = 0.0f;
+  for (uint32_t i = threadIdx.x; i < K; i += 256) { const float d = xs[i] - mean; v = __builtin_fmaf(d, d, v); }
+  const float inv = 1.0f / __builtin_sqrtf(block_sum(v, red) / (float)K + eps);
+  for (uint32_t i = threadIdx.x; i < K; i += 256) xs[i] = (xs[i] - mean) * inv * w[i];
+}
+
+template <int PRO>
+__global__ void __launch_bounds__(256) lin_mv_kernel(const LinMv a, uint32_t n_groups) {
+  extern __shared__ __attribute__((aligned(16))) float xs[];   // [kp]
+  __shared__ float red[2][4][kMvR];
+  __shared__ float bred[16];
+  const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  if (PRO == LP_COPY) {
+    for (uint32_t i = tid; i < a.k; i += 256) xs[i] = a.x[i];
+  } else if (PRO == LP_RESID || PRO == LP_HEAD) {
+    for (uint32_t i = tid; i < a.k; i += 256) xs[i] = a.y[i];
+    ln_lds(xs, a.k, a.nw, a.eps, bred);
+    for (uint32_t i = tid; i < a.k; i += 256) {
+      const float v = a.x[i] + a.mult * xs[i];
+      xs[i] = v;
+      if (blockIdx.x == 0) a.xout[i] = v;
+    }
+    if (PRO == LP_HEAD) ln_lds(xs, a.k, a.nw2, a.eps, bred);
+  } else {
+    for (uint32_t h = wave; h < a.heads; h += 4) {
+      const float* num = a.num + (size_t)h * a.ldo;
+      const float inv = 1.0f / (fmaxf(fabsf(num[a.vdim]), num[a.vdim + 1]) + 1e-6f);
+      float ss = 0.0f;
+      for (uint32_t j = lane; j < a.vdim; j += 64) { const float o = num[j] * inv; ss = __builtin_fmaf(o, o, ss); }
+      const float r = 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+      for (uint32_t j = lane; j < a.vdim; j += 64) {
+        const uint32_t e = h * a.vdim + j;
+        xs[e] = num[j] * inv * r * a.nw[e] * sigmoid_f(a.gate[e]);
+      }
+    }
+  }
+  for (uint32_t i = a.k + tid; i < a.kp; i += 256) xs[i] = 0.0f;
+  __syncthreads();
+  uint32_t par = 0;
+  for (uint32_t g = blockIdx.x; g < n_groups; g += gridDim.x, par ^= 1) {
+    // rows of this group: 8 consecutive ones, or 4 pairs (a gate row and the up row 16 below it)
+    const uint16_t* wr[kMvR];
+#pragma unroll
+    for (int r = 0; r < kMvR; r++) {
+      uint32_t row;
+      if (a.paired) { const uint32_t p = g * 4 + (r & 3); row = (p >> 4) * 32 + (p & 15) + (r >> 2) * 16; }
+      else row = g * kMvR + r;
+      wr[r] = a.w + (size_t)(row < a.n ? row : a.n - 1) * a.kp;
+    }
+    float acc[kMvR];
+#pragma unroll
+    for (int r = 0; r < kMvR; r++) acc[r] = 0.0f;
+#pragma unroll 2
+    for (uint32_t kb = tid * 8; kb < a.kp; kb += 2048) {
+      u32x4 w[kMvR];
+#pragma unroll
+      for (int r = 0; r < kMvR; r++) w[r] = ldg_nt128(wr[r] + kb);
+      const f32x4 x0 = *reinterpret_cast<const f32x4*>(xs + kb), x1 = *reinterpret_cast<const f32x4*>(xs + kb + 4);
+#pragma unroll
+      for (int r = 0; r < kMvR; r++) {
+        float s = acc[r];
+        s = __builtin_fmaf(bf_lo(w[r].x), x0.x, s); s = __builtin_fmaf(bf_hi(w[r].x), x0.y, s);
+        s = __builtin_fmaf(bf_lo(w[r].y), x0.z, s); s = __builtin_fmaf(bf_hi(w[r].y), x0.w, s);
+        s = __builtin_fmaf(bf_lo(w[r].z), x1.x, s); s = __builtin_fmaf(bf_hi(w[r].z), x1.y, s);
+        s = __builtin_fmaf(bf_lo(w[r].w), x1.z, s); s = __builtin_fmaf(bf_hi(w[r].w), x1.w, s);
+        acc[r] = s;
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < kMvR; r++) {
+      const float t = wave_sum_to_lane63(acc[r]);
+      if (lane == 63) red[par][wave][r] = t;
+    }
+    __syncthreads();
+    if (!a.paired) {
+      if (tid < kMvR) {
+        const uint32_t row = g * kMvR + tid;
+        if (row < a.n) a.out[row] = (red[par][0][tid] + red[par][1][tid]) + (red[par][2][tid] + red[par][3][tid]);
+      }
+    } else if (tid < 4) {
+      const uint32_t p = g * 4 + tid;
+      if (p < a.n / 2) {
+        const float gt = (red[par][0][tid] + red[par][1][tid]) + (red[par][2][tid] + red[par][3][tid]);
+        const float up = (red[par][0][tid + 4] + red[par][1][tid + 4]) + (red[par][2][tid + 4] + red[par][3][tid + 4]);
+        a.out[p] = gelu_tanh_f(gt) * up;
+      }
+    }
+  }
+}
+
+template <int PRO>
+static hipError_t lin_mv_go(const LinMv& a, hipStream_t st) {
+  static bool opted[64] = {};
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_mv_kernel<PRO>), 152 * 1024, opted); e != hipSuccess) return e;
+  const uint32_t groups = (a.n + kMvR - 1) / kMvR;
+  const uint32_t grid = groups < 2048u ? groups : 2048u;
+  hipLaunchKernelGGL(lin_mv_kernel<PRO>, dim3(grid), dim3(256), (size_t)a.kp * 4, st, a, groups);
+  return hipGetLastError();
+}
+
+hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st) {
+  if (!a.w || !a.out || a.n == 0 || a.kp % 64 || a.kp > kLinMvMaxK || a.k > a.kp || (a.paired && a.n % 32)) return hipErrorInvalidValue;
+  switch (pro) {
+    case LP_COPY: return a.x ? lin_mv_go<LP_COPY>(a, st) : hipErrorInvalidValue;
+    case LP_RESID: return a.x && a.y && a.nw && a.xout ? lin_mv_go<LP_RESID>(a, st) : hipErrorInvalidValue;
+    case LP_HEAD: return a.x && a.y && a.nw && a.nw2 && a.xout ? lin_mv_go<LP_HEAD>(a, st) : hipErrorInvalidValue;
+    case LP_MLSTM: return a.num && a.nw && a.gate && a.heads * a.vdim == a.k ? lin_mv_go<LP_MLSTM>(a, st) : hipErrorInvalidValue;
+  }
+  return hipErrorInvalidValue;
+}
+
+// ------------------------------------------------------------------------------------------------
+// block product.  A workgroup of 4 waves computes BN weight rows x BM tokens, k in steps of 64; both operands go global -> LDS by
+// DMA (two buffers), 16-byte chunks of a row stored at chunk ^ (row & mask) so that the 16 rows of a fragment read different banks.
+// The weights are the A operand: a lane ends up with 4 consecutive output columns of one token.
+// ------------------------------------------------------------------------------------------------
+template <class T> constexpr uint32_t act_chunks() { return 64 * sizeof(T) / 16; }   // 16-byte chunks of a row's 64 columns
+
+template <class T, int BM, int BN, int WN, int EPI>
+__global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t tiles_n, uint32_t tiles_m) {
+  constexpr int WM = 4 / WN, NT = BN / WN / 16, MT = BM / WM / 16;
+  constexpr uint32_t XC = act_chunks<T>();
+  constexpr uint32_t kWBytes = BN * 128, kXBytes = BM * XC * 16, kBuf = kWBytes + kXBytes;
+  extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
+  const uint32_t lane = threadIdx.x & 63, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
+  // consecutive tiles of one weight panel on one XCD (workgroups go round-robin over the 8 XCDs)
+  uint32_t t = blockIdx.x;
+  const uint32_t total = tiles_n * tiles_m;
+  {
+    const uint32_t q = total / 8, r = total % 8, xcd = t % 8, i = t / 8;
+    t = xcd * q + (xcd < r ? xcd : r) + i;
+  }
+  const uint32_t tn = t / tiles_m, tm = t % tiles_m;
+  const uint32_t n0 = tn * BN, m0 = tm * BM;
+  const uint32_t wn = wave % WN, wm = wave / WN;
+  const uint32_t r16 = lane & 15, g = lane >> 4;
+  const T* X = reinterpret_cast<const T*>(a.x);
+
+  auto stage = [&](uint32_t k0, uint32_t buf) {
+    uint8_t* base = smem + buf * kBuf;
+#pragma unroll
+    for (int i = 0; i < (int)(kWBytes / 4096); i++) {       // weights: 8 chunks a row, a wave instruction covers 8 rows
+      const uint32_t row = (i * 4 + wave) * 8 + (lane >> 3), ch = (lane & 7) ^ (row & 7);
+      const uint32_t n = n0 + row < a.np ? n0 + row : a.np - 1;
+      lds_dma16(a.w + (size_t)n * a.kp + k0 + ch * 8, base + (i * 4 + wave) * 1024);
+    }
+    constexpr uint32_t RPI = 64 / XC;                        // rows per wave instruction
+#pragma unroll
+    for (int i = 0; i < (int)((kXBytes / 1024 + 3) / 4); i++) {
+      const uint32_t blk = i * 4 + wave;
+      if (kXBytes / 1024 % 4 == 0 || blk < kXBytes / 1024) {
+        const uint32_t row = blk * RPI + lane / XC, ch = (lane % XC) ^ (row & (XC - 1));
+        const uint32_t m = m0 + row < a.M ? m0 + row : a.M - 1;
+        lds_dma16(X + (size_t)m * a.ldx + k0 + ch * (16 / sizeof(T)), base + kWBytes + blk * 1024);
+      }
+    }
+  };
+
+  f32x4 acc[NT][MT];
+#pragma unroll
+  for (int i = 0; i < NT; i++)
+#pragma unroll
+    for (int j = 0; j < MT; j++) acc[i][j] = (f32x4)(0.0f);
+
+  stage(0, 0);
+  __builtin_amdgcn_s_waitcnt(0x0F70);   // vmcnt(0)
+  __syncthreads();
+  const uint32_t steps = a.kp / 64;
+  for (uint32_t s = 0; s < steps; s++) {
+    const uint32_t cur = s & 1;
+    if (s + 1 < steps) stage((s + 1) * 64, cur ^ 1);
+    const uint8_t* wb = smem + cur * kBuf;
+    const uint8_t* xb = wb + kWBytes;
+    constexpr int U = 64 / Frag<T>::KU;
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      typename Frag<T>::V wf[NT], xf[MT];
+#pragma unroll
+      for (int i = 0; i < NT; i++) {
+        const uint32_t row = (wn * NT + i) * 16 + r16;
+        if constexpr (sizeof(T) == 2) {
+          wf[i] = *reinterpret_cast<const bf16x8*>(wb + row * 128 + (((uint32_t)(u * 4) + g) ^ (row & 7)) * 16);
+        } else {   // 4 bf16 values of the 16-column unit: half a chunk
+          const u32x2 h = *reinterpret_cast<const u32x2*>(wb + row * 128 + (((uint32_t)(u * 2) + (g >> 1)) ^ (row & 7)) * 16 + (g & 1) * 8);
+          f32x4 v;
+          v.x = bf_lo(h.x); v.y = bf_hi(h.x); v.z = bf_lo(h.y); v.w = bf_hi(h.y);
+          wf[i] = v;
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < MT; j++) {
+        const uint32_t row = (wm * MT + j) * 16 + r16;
+        xf[j] = Frag<T>::load(reinterpret_cast<const T*>(xb + row * (XC * 16) + (((uint32_t)(u * 4) + g) ^ (row & (XC - 1))) * 16));
+      }
+#pragma unroll
+      for (int i = 0; i < NT; i++)
+#pragma unroll
+        for (int j = 0; j < MT; j++) acc[i][j] = Frag<T>::mma(wf[i], xf[j], acc[i][j]);
+    }
+    __builtin_amdgcn_s_waitcnt(0x0F70);
+    __syncthreads();
+  }
+  // lane: token r16 of a token tile, columns 4g .. 4g + 3 of a weight tile
+#pragma unroll
+  for (int j = 0; j < MT; j++) {
+    const uint32_t m = m0 + (wm * MT + j) * 16 + r16;
+    if (m >= a.M) continue;
+    if constexpr (EPI == LE_GEGLU) {
+#pragma unroll
+      for (int i = 0; i < NT; i += 2) {
+        const uint32_t nb = n0 + (wn * NT + i) * 16;           // gate rows; the up rows follow
+        if (nb >= a.n) continue;
+        T* o = reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + nb / 2 + g * 4;
+#pragma unroll
+        for (int e = 0; e < 4; e++) o[e] = to_act<T>(gelu_tanh_f(acc[i][j][e]) * acc[i + 1][j][e]);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < NT; i++) {
+        const uint32_t nb = n0 + (wn * NT + i) * 16 + g * 4;
+        if constexpr (EPI == LE_F32) {
+          float* o = reinterpret_cast<float*>(a.out) + (size_t)m * a.ldo + nb;
+          if (nb + 4 <= a.n && (a.ldo & 3) == 0) *reinterpret_cast<f32x4*>(o) = acc[i][j];
+          else
+            for (int e = 0; e < 4; e++)
+              if (nb + e < a.n) o[e] = acc[i][j][e];
+        } else if constexpr (EPI == LE_ACT) {
+          T* o = reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + nb;
+#pragma unroll
+          for (int e = 0; e < 4; e++)
+            if (nb + e < a.n) o[e] = to_act<T>(acc[i][j][e]);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; e++) {
+            const uint32_t n = nb + e;
+            if (n >= a.n) break;
+            const uint32_t h = n / a.hd, d = n % a.hd;
+            const size_t at = EPI == LE_HEADS ? ((size_t)h * a.tcap + m) * a.ldo + d : ((size_t)h * a.hrows + d) * a.ldo + m;
+            reinterpret_cast<T*>(a.out)[at] = to_act<T>(acc[i][j][e]);
+          }
+        }
+      }
+    }
+  }
+}
+
+template <class T, int BM, int BN, int WN, int EPI>
+static hipError_t lin_gemm_go(const LinGemm& a, hipStream_t st) {
+  static bool opted[64] = {};
+  constexpr size_t lds = 2 * (BN * 128 + (size_t)BM * act_chunks<T>() * 16);
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_gemm_kernel<T, BM, BN, WN, EPI>), (int)lds, opted); e != hipSuccess) return e;
+  const uint32_t tn = (a.n + BN - 1) / BN, tm = (a.M + BM - 1) / BM;
+  hipLaunchKernelGGL((lin_gemm_kernel<T, BM, BN, WN, EPI>), dim3(tn * tm), dim3(256), lds, st, a, tn, tm);
+  return hipGetLastError();
+}
+
+template <class T, int EPI>
+static hipError_t lin_gemm_pick(const LinGemm& a, hipStream_t st) {
+  const uint32_t tn = (a.n + 127) / 128;
+  if (a.M > 64 && tn * ((a.M + 127) / 128) >= 224) return lin_gemm_go<T, 128, 128, 2, EPI>(a, st);
+  if (a.M > 32 && tn * ((a.M + 63) / 64) >= 160) return lin_gemm_go<T, 64, 128, 4, EPI>(a, st);
+  if (a.M > 16) return lin_gemm_go<T, 32, 128, 4, EPI>(a, st);
+  return lin_gemm_go<T, 16, 128, 4, EPI>(a, st);
+}
+
+hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st) {
+  const uint32_t el = f32 ? 4 : 2;
+  if (!a.w || !a.x || !a.out || a.n == 0 || a.M == 0 || a.kp % 64 || a.ldx < a.kp || (a.ldx * el) % 16 || a.np % 16 || a.n > a.np) return hipErrorInvalidValue;
+  if (epi == LE_GEGLU && a.n % 32) return hipErrorInvalidValue;
+  if ((epi == LE_HEADS || epi == LE_HEADS_T) && !a.hd) return hipErrorInvalidValue;
+#define LGH_GEMM_CASE(E) \
+  case E: return f32 ? lin_gemm_pick<float, E>(a, st) : lin_gemm_pick<__bf16, E>(a, st);
+  switch (epi) {
+    LGH_GEMM_CASE(LE_F32)
+    LGH_GEMM_CASE(LE_ACT)
+    LGH_GEMM_CASE(LE_GEGLU)
+    LGH_GEMM_CASE(LE_HEADS)
+    LGH_GEMM_CASE(LE_HEADS_T)
+  }
+#undef LGH_GEMM_CASE
+  return hipErrorInvalidValue;
+}
+
+// ------------------------------------------------------------------------------------------------
+// upload-time layouts
+// ------------------------------------------------------------------------------------------------
+__global__ void __launch_bounds__(256) lin_pack_kernel(const uint16_t* __restrict__ src, uint32_t k, uint16_t* __restrict__ dst, uint32_t kp, uint32_t row0, int mode) {
+  const uint32_t r = blockIdx.y;
+  const uint32_t row = mode == 0 ? row0 + r : row0 + (r >> 4) * 32 + (r & 15) + (mode == 2 ? 16 : 0);
+  for (uint32_t i = blockIdx.x * 256 + threadIdx.x; i < k; i += gridDim.x * 256) dst[(size_t)row * kp + i] = src[(size_t)r * k + i];
+}
+
+hipError_t lin_pack_launch(const uint16_t* src, uint32_t rows, uint32_t k, uint16_t* dst, uint32_t kp, uint32_t row0, int mode, hipStream_t st) {
+  for (uint32_t r = 0; r < rows; r += 32768) {   // (32768: a multiple of the pair block, below the grid's y limit)
+    const uint32_t c = rows - r < 32768 ? rows - r : 32768;
+    hipLaunchKernelGGL(lin_pack_kernel, dim3((k + 1023) / 1024, c), dim3(256), 0, st, src + (size_t)r * k, k, dst, kp, row0 + (mode ? 2 * r : r), mode);
+  }
+  return hipGetLastError();
+}
+
+__global__ void __launch_bounds__(256) lin_transpose_heads_kernel(const uint16_t* __restrict__ src, uint32_t dim, uint32_t rank, uint16_t* __restrict__ dst, uint32_t dimp) {
+  const uint32_t h = blockIdx.y, r = blockIdx.x;
+  for (uint32_t d = threadIdx.x; d < dim; d += 256) dst[((size_t)h * rank + r) * dimp + d] = src[((size_t)h * dim + d) * rank + r];
+}
+
+hipError_t lin_transpose_heads_launch(const uint16_t* src, uint32_t heads, uint32_t dim, uint32_t rank, uint16_t* dst, uint32_t dimp, hipStream_t st) {
+  hipLaunchKernelGGL(lin_transpose_heads_kernel, dim3(rank, heads), dim3(256), 0, st, src, dim, rank, dst, dimp);
+  return hipGetLastError();
+}
+
+__global__ void __launch_bounds__(256) bf16_to_f32_kernel(const uint16_t* __restrict__ src, float* __restrict__ dst, uint64_t n) {
+  for (uint64_t i = (uint64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (uint64_t)gridDim.x * 256) dst[i] = bf_f(src[i]);
+}
+
+hipError_t bf16_to_f32_launch(const uint16_t* src, float* dst, uint64_t n, hipStream_t st) {
+  uint64_t blocks = (n + 255) / 256;
+  if (blocks > 4096) blocks = 4096;
+  if (blocks) hipLaunchKernelGGL(bf16_to_f32_kernel, dim3((uint32_t)blocks), dim3(256), 0, st, src, dst, n);
+  return hipGetLastError();
+}
+
+}  // namespace lgh
