@@ -1,0 +1,308 @@
+// latent_attention.hip — attention over a shared low-rank latent (layered.h).  A cached position is ONE row for all heads: the normed
+// latent c (rank values) and a rotated key part.  Per head k = [W_uk c | rotated part], v = W_uv c.
+//
+//   decode and short portions ("absorbed"): q . W_uk c = (W_uk^T q) . c, so the key expansion moves to the query and the value
+//     expansion behind the weighted sum; (token, head) pairs are the rows of one product against the cached rows, read once for all heads.
+//   long portions ("expanded"): keys and values of the context are formed per head by two block products, then ordinary causal attention.
+//
+// Scores, softmax and the weighted sums are in 32-bit; operands of the matrix cores are the cache's type (bf16 or f32).
+#include "layered.h"
+#include "layered_device.h"
+
+namespace lgh {
+
+constexpr float kNegHuge = -1e30f;
+
+// token t of a block -> rotated pair i of src
+__device__ __forceinline__ void rot_pair(const float* src, const float* cs, uint32_t i, float& a, float& b) {
+  const float u = src[2 * i], v = src[2 * i + 1], c = cs[2 * i], s = cs[2 * i + 1];
+  a = u * c - v * s;
+  b = v * c + u * s;
+}
+
+// cache row of token t: RMS norm of the latent, rotation of the shared key part.  One workgroup.
+template <class T>
+__device__ __forceinline__ void latent_cache_row(const LatentShape& s, const LatentBufs& b, const float* dkv, uint32_t pos, float* red) {
+  T* row = reinterpret_cast<T*>(b.cache) + (size_t)pos * s.ldc;
+  float ss = 0.0f;
+  for (uint32_t i = threadIdx.x; i < s.rank; i += 256) ss = __builtin_fmaf(dkv[i], dkv[i], ss);
+  const float inv = 1.0f / __builtin_sqrtf(block_sum(ss, red) / (float)s.rank + s.eps);
+  for (uint32_t i = threadIdx.x; i < s.rank; i += 256) row[i] = to_act<T>(dkv[i] * inv * b.dkv_norm[i]);
+  const float* cs = b.cs + (size_t)pos * s.rot_n;
+  for (uint32_t i = threadIdx.x; i < s.rot_dim; i += 256) {
+    float v = dkv[s.rank + i];
+    if (i < s.rot_n) { float p0, p1; rot_pair(dkv + s.rank, cs, i >> 1, p0, p1); v = (i & 1) ? p1 : p0; }
+    row[s.rank + i] = to_act<T>(v);
+  }
+}
+
+// absorbed queries: grid (chunks of 64 latent rows, heads + 1, tokens); the extra head writes the cache row
+template <class T>
+__global__ void __launch_bounds__(256) latent_prep_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0) {
+  __shared__ float red[16];
+  extern __shared__ float qn[];   // [dimp]
+  const uint32_t t = blockIdx.z, h = blockIdx.y, tid = threadIdx.x;
+  const uint32_t pos = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + t;
+  const float* cat = b.cat + (size_t)t * s.ldcat;
+  if (h == s.heads) {
+    if (blockIdx.x == 0) latent_cache_row<T>(s, b, cat + s.off_dkv, pos, red);
+    return;
+  }
+  const float* q = cat + s.off_q + (size_t)h * (s.dim + s.rot_dim);
+  T* qa = reinterpret_cast<T*>(b.qa) + ((size_t)t * s.heads + h) * s.ldc;
+  for (uint32_t i = tid; i < s.dimp; i += 256) qn[i] = i < s.dim ? q[i] : 0.0f;
+  __syncthreads();
+  const uint32_t sub = tid & 15;
+  const uint16_t* W = b.uk_t + (size_t)h * s.rank * s.dimp;
+#pragma unroll
+  for (int it = 0; it < 4; it++) {
+    const uint32_t r = blockIdx.x * 64 + it * 16 + (tid >> 4);
+    float acc = 0.0f;
+    if (r < s.rank) {
+      for (uint32_t d = sub * 8; d < s.dimp; d += 128) {
+        const u32x4 w = *reinterpret_cast<const u32x4*>(W + (size_t)r * s.dimp + d);
+        const float* x = qn + d;
+        acc = __builtin_fmaf(bf_lo(w.x), x[0], acc); acc = __builtin_fmaf(bf_hi(w.x), x[1], acc);
+        acc = __builtin_fmaf(bf_lo(w.y), x[2], acc); acc = __builtin_fmaf(bf_hi(w.y), x[3], acc);
+        acc = __builtin_fmaf(bf_lo(w.z), x[4], acc); acc = __builtin_fmaf(bf_hi(w.z), x[5], acc);
+        acc = __builtin_fmaf(bf_lo(w.w), x[6], acc); acc = __builtin_fmaf(bf_hi(w.w), x[7], acc);
+      }
+    }
+    acc += dpp_f<0xB1>(acc); acc += dpp_f<0x4E>(acc); acc += dpp_f<0x141>(acc); acc += dpp_f<0x140>(acc);   // 16 lanes
+    if (r < s.rank && sub == 0) qa[r] = to_act<T>(acc);
+  }
+  if (blockIdx.x == 0) {
+    const float* cs = b.cs + (size_t)pos * s.rot_n;
+    for (uint32_t i = tid; i < s.ldc - s.rank; i += 256) {
+      float v = i < s.rot_dim ? q[s.dim + i] : 0.0f;
+      if (i < s.rot_n) { float p0, p1; rot_pair(q + s.dim, cs, i >> 1, p0, p1); v = (i & 1) ? p1 : p0; }
+      qa[s.rank + i] = to_act<T>(v);
+    }
+  }
+}
+
+hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, bool f32, hipStream_t st) {
+  if (s.dimp % 8 || s.ldc < s.rank + s.rot_dim || s.rot_n > s.rot_dim || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
+  const dim3 grid((s.rank + 63) / 64, s.heads + 1, M);
+  if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, grid, dim3(256), s.dimp * 4, st, s, b, pos_ptr, pos0);
+  else hipLaunchKernelGGL(latent_prep_kernel<__bf16>, grid, dim3(256), s.dimp * 4, st, s, b, pos_ptr, pos0);
+  return hipGetLastError();
+}
+
+// ------------------------------------------------------------------------------------------------
+// absorbed attention.  A workgroup = 16 (token, head) rows x one split of the keys x up to 512 latent columns of the output;
+// KT keys at a time in LDS.  Scores: wave w multiplies the 16 rows with keys 16 w ..; weighted sums: wave w owns a quarter of the
+// columns and takes the values straight from the key tile (the latent IS the value).
+// ------------------------------------------------------------------------------------------------
+template <class T> constexpr uint32_t lat_pad() { return 16 / sizeof(T); }   // LDS row padding: consecutive rows shift by 4 banks
+
+template <class T, int NCT>   // NCT: 16-column tiles of the output per wave
+__global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M,
+                                                          uint32_t n_splits, uint32_t KT) {
+  extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
+  const uint32_t tid = threadIdx.x, lane = tid & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
+  const uint32_t r16 = lane & 15, g = lane >> 4;
+  const uint32_t rows = M * s.heads, row0 = blockIdx.x * 16, sp = blockIdx.y, col0 = blockIdx.z * (NCT * 64);
+  const uint32_t p0 = pos_ptr ? (uint32_t)*pos_ptr : pos0;
+  const uint32_t kv = p0 + M;                                   // keys 0 .. kv - 1
+  const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles + n_splits - 1) / n_splits;
+  const uint32_t tb = sp * per, te = tb + per < tiles ? tb + per : tiles;
+  if (tb >= te) return;                                         // (the merge skips the same splits)
+  const uint32_t ldq = s.ldc + lat_pad<T>(), lds_s = KT + 4, lds_p = KT + lat_pad<T>();
+  T* Qs = reinterpret_cast<T*>(smem);                           // [16][ldq]
+  T* Cs = Qs + 16 * ldq;                                        // [KT][ldq]
+  T* Ps = Cs + KT * ldq;                                        // [16][lds_p]
+  float* Ss = reinterpret_cast<float*>(Ps + 16 * lds_p);        // [16][lds_s]
+  constexpr uint32_t PER = Frag<T>::PER, KU = Frag<T>::KU;
+  const uint32_t cpr = s.ldc / PER;                             // 16-byte chunks of a row
+  const T* qg = reinterpret_cast<const T*>(b.qa);
+  const T* cg = reinterpret_cast<const T*>(b.cache);
+  for (uint32_t i = tid; i < 16 * cpr; i += 256) {
+    const uint32_t r = i / cpr, ch = i % cpr, rr = row0 + r < rows ? row0 + r : rows - 1;
+    *reinterpret_cast<u32x4*>(Qs + r * ldq + ch * PER) = *reinterpret_cast<const u32x4*>(qg + (size_t)rr * s.ldc + ch * PER);
+  }
+  // the rows of this lane's accumulators: 4g .. 4g + 3
+  uint32_t lim[4];
+  float m[4], l[4];
+#pragma unroll
+  for (int e = 0; e < 4; e++) {
+    const uint32_t r = row0 + g * 4 + e;
+    lim[e] = p0 + (r < rows ? r : rows - 1) / s.heads + 1;      // keys this row sees
+    m[e] = kNegHuge; l[e] = 0.0f;
+  }
+  f32x4 o[NCT];
+#pragma unroll
+  for (int i = 0; i < NCT; i++) o[i] = (f32x4)(0.0f);
+  const uint32_t wc = col0 + w * NCT * 16;
+  for (uint32_t tl = tb; tl < te; tl++) {
+    const uint32_t k0 = tl * KT;
+    __syncthreads();                                            // the previous tile is used up
+    for (uint32_t i = tid; i < KT * cpr; i += 256) {
+      const uint32_t r = i / cpr, ch = i % cpr, kk = k0 + r < kv ? k0 + r : kv - 1;
+      *reinterpret_cast<u32x4*>(Cs + r * ldq + ch * PER) = *reinterpret_cast<const u32x4*>(cg + (size_t)kk * s.ldc + ch * PER);
+    }
+    __syncthreads();
+    if (w * 16 < KT) {
+      f32x4 sc = (f32x4)(0.0f);
+      const T* qa = Qs + r16 * ldq + g * PER;
+      const T* kb = Cs + (w * 16 + r16) * ldq + g * PER;
+      for (uint32_t k = 0; k < s.ldc; k += KU) sc = Frag<T>::mma(Frag<T>::load(qa + k), Frag<T>::load(kb + k), sc);
+#pragma unroll
+      for (int e = 0; e < 4; e++) Ss[(g * 4 + e) * lds_s + w * 16 + r16] = sc[e] * s.scale;
+    }
+    __syncthreads();
+    // softmax of the tile, by every wave for its own use: lane (r16, g) looks at keys r16, r16 + 16, .. of rows 4g .. 4g + 3
+    float alpha[4];
+#pragma unroll
+    for (int e = 0; e < 4; e++) {
+      float mx = m[e], sv[4];
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        const uint32_t key = r16 + j * 16;
+        sv[j] = key < KT && k0 + key < lim[e] ? Ss[(g * 4 + e) * lds_s + key] : kNegHuge;
+        mx = fmaxf(mx, sv[j]);
+      }
+      mx = fmaxf(mx, dpp_f<0xB1>(mx)); mx = fmaxf(mx, dpp_f<0x4E>(mx)); mx = fmaxf(mx, dpp_f<0x141>(mx)); mx = fmaxf(mx, dpp_f<0x140>(mx));
+      float sum = 0.0f;
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        const uint32_t key = r16 + j * 16;
+        const float p = key < KT && k0 + key < lim[e] ? expf(sv[j] - mx) : 0.0f;
+        sum += p;
+        if (w == 0 && key < KT) Ps[(g * 4 + e) * lds_p + key] = to_act<T>(p);
+      }
+      sum += dpp_f<0xB1>(sum); sum += dpp_f<0x4E>(sum); sum += dpp_f<0x141>(sum); sum += dpp_f<0x140>(sum);
+      alpha[e] = expf(m[e] - mx);
+      l[e] = l[e] * alpha[e] + sum;
+      m[e] = mx;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < NCT; i++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) o[i][e] *= alpha[e];
+    for (uint32_t k = 0; k < KT; k += KU) {
+      const typename Frag<T>::V pf = Frag<T>::load(Ps + r16 * lds_p + k + g * PER);
+#pragma unroll
+      for (int i = 0; i < NCT; i++) {
+        const uint32_t c = wc + i * 16 + r16;
+        typename Frag<T>::V vf;
+        const T* src = Cs + (k + g * PER) * ldq + (c < s.ldc ? c : s.ldc - 1);
+#pragma unroll
+        for (uint32_t e = 0; e < PER; e++) vf[e] = src[e * ldq];
+        o[i] = Frag<T>::mma(pf, vf, o[i]);
+      }
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < 4; e++) {
+    const uint32_t r = row0 + g * 4 + e;
+    if (r >= rows) continue;
+    const size_t pr = (size_t)sp * rows + r;
+    if (w == 0 && r16 == 0 && blockIdx.z == 0) { b.part_ml[pr * 2] = m[e]; b.part_ml[pr * 2 + 1] = l[e]; }
+#pragma unroll
+    for (int i = 0; i < NCT; i++) {
+      const uint32_t c = wc + i * 16 + r16;
+      if (c < s.rank) b.part_acc[pr * s.rank + c] = o[i][e];
+    }
+  }
+}
+
+static size_t latent_lds(const LatentShape& s, uint32_t KT, uint32_t el) {
+  const uint32_t pad = 16 / el, ldq = s.ldc + pad;
+  return (size_t)(16 + KT) * ldq * el + (size_t)16 * (KT + pad) * el + (size_t)16 * (KT + 4) * 4;
+}
+
+uint32_t latent_key_tile(const LatentShape& s, bool f32, uint32_t M) {
+  (void)M;
+  for (uint32_t KT : {64u, 32u, 16u}) {
+    if (!f32 && KT < 32) break;   // a bf16 unit spans 32 keys
+    if (latent_lds(s, KT, f32 ? 4 : 2) <= 155 * 1024) return KT;
+  }
+  return 0;
+}
+
+template <class T, int NCT>
+static hipError_t latent_attn_go(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, uint32_t KT,
+                                 uint32_t zs, hipStream_t st) {
+  static bool opted[64] = {};
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&latent_attn_kernel<T, NCT>), 156 * 1024, opted); e != hipSuccess) return e;
+  hipLaunchKernelGGL((latent_attn_kernel<T, NCT>), dim3((M * s.heads + 15) / 16, n_splits, zs), dim3(256), latent_lds(s, KT, sizeof(T)), st, s, b, pos_ptr,
+                     pos0, M, n_splits, KT);
+  return hipGetLastError();
+}
+
+hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32,
+                              hipStream_t st) {
+  const uint32_t KT = latent_key_tile(s, f32, M);
+  if (!KT || s.ldc % 32 || n_splits == 0 || n_splits > kLatMaxSplits || M == 0 || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
+  const uint32_t nct = (s.rank + 63) / 64;
+#define LGH_LAT_CASE(N) return f32 ? latent_attn_go<float, N>(s, b, pos_ptr, pos0, M, n_splits, KT, zs, st) : latent_attn_go<__bf16, N>(s, b, pos_ptr, pos0, M, n_splits, KT, zs, st)
+  uint32_t zs = 1;
+  if (nct <= 1) LGH_LAT_CASE(1);
+  if (nct <= 2) LGH_LAT_CASE(2);
+  if (nct <= 4) LGH_LAT_CASE(4);
+  zs = (nct + 7) / 8;
+  LGH_LAT_CASE(8);
+#undef LGH_LAT_CASE
+}
+
+// ------------------------------------------------------------------------------------------------
+// merge + value expansion + head gate: grid (chunks of 32 value rows, token * heads)
+// ------------------------------------------------------------------------------------------------
+template <class O>
+__global__ void __launch_bounds__(256) latent_out_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M,
+                                                         uint32_t n_splits, uint32_t KT, O* __restrict__ out, uint32_t ldo) {
+  extern __shared__ __attribute__((aligned(16))) float lat[];   // [rankp]
+  __shared__ float wgt[kLatMaxSplits];
+  const uint32_t tid = threadIdx.x, r = blockIdx.y, t = r / s.heads, h = r % s.heads, rows = M * s.heads;
+  const uint32_t kv = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + M;
+  const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles + n_splits - 1) / n_splits, act = (tiles + per - 1) / per;
+  if (tid < 64) {
+    const float mi = tid < act ? b.part_ml[((size_t)tid * rows + r) * 2] : kNegHuge;
+    const float li = tid < act ? b.part_ml[((size_t)tid * rows + r) * 2 + 1] : 0.0f;
+    const float mm = wave_max(mi), f = expf(mi - mm), tot = wave_sum(f * li);
+    wgt[tid] = f / tot;
+  }
+  __syncthreads();
+  for (uint32_t i = tid; i < s.rankp; i += 256) {
+    float v = 0.0f;
+    if (i < s.rank) {
+#pragma unroll 8
+      for (uint32_t sp = 0; sp < act; sp++) v = __builtin_fmaf(wgt[sp], b.part_acc[((size_t)sp * rows + r) * s.rank + i], v);
+    }
+    lat[i] = v;
+  }
+  __syncthreads();
+  const float gate = sigmoid_f(b.cat[(size_t)t * s.ldcat + s.off_g + h]);
+  const uint32_t lane = tid & 63, w = tid >> 6;
+#pragma unroll 2
+  for (int it = 0; it < 8; it++) {
+    const uint32_t v = blockIdx.x * 32 + it * 4 + w;
+    if (v >= s.vdim) break;
+    const uint16_t* W = b.uv + ((size_t)h * s.vdim + v) * s.rankp;
+    float acc = 0.0f;
+    for (uint32_t k = lane * 8; k < s.rankp; k += 512) {
+      const u32x4 wv = *reinterpret_cast<const u32x4*>(W + k);
+      const f32x4 x0 = *reinterpret_cast<const f32x4*>(lat + k), x1 = *reinterpret_cast<const f32x4*>(lat + k + 4);
+      acc = __builtin_fmaf(bf_lo(wv.x), x0.x, acc); acc = __builtin_fmaf(bf_hi(wv.x), x0.y, acc);
+      acc = __builtin_fmaf(bf_lo(wv.y), x0.z, acc); acc = __builtin_fmaf(bf_hi(wv.y), x0.w, acc);
+      acc = __builtin_fmaf(bf_lo(wv.z), x1.x, acc); acc = __builtin_fmaf(bf_hi(wv.z), x1.y, acc);
+      acc = __builtin_fmaf(bf_lo(wv.w), x1.z, acc); acc = __builtin_fmaf(bf_hi(wv.w), x1.w, acc);
+    }
+    acc = wave_sum_to_lane63(acc);
+    if (lane == 63) out[(size_t)t * ldo + h * s.vdim + v] = to_act<O>(acc * gate);
+  }
+}
+
+hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32cache,
+                             void* out, uint32_t ldo, bool out_f32, hipStream_t st) {
+  const uint32_t KT = latent_key_tile(s, f32cache, M);
+  if (!KT || s.rankp % 8 || n_splits == 0 || n_splits > kLatMaxSplits) return hipErrorInvalidValue;
+  const dim3 grid((s.vdim + 31) / 32, M * s.heads);
+  if (out_f32) hipLaunchKernelGGL(latent_out_kernel<float>, grid, dim3(256), s.rankp * 4, st, s, b, pos_ptr, pos0, M, n_splits, KT, (float*)out, ldo);
+  else hipLaunchKernelGGL(latent_out_kernel<__bf16>, grid, dim3(256), s.rankp * 4, st, s, b, pos_ptr, pos0, M, n_splits, KT, (__bf16*)out, ldo);
+  return hipGetLastError();
+}
+
+}  // namespace lgh

@@ -140,7 +140,7 @@ struct MlstmBufs {
   const float *bi, *bf;        // [heads]
   const float* norm;           // [heads * vdim]
   float* S;
-  double* m;                   // [2][heads]: the running maximum before position p lies in half p & 1
+  double* m;                   // [3][heads]: the running maximum before position p lies in part p & 1; part 2: a block's start
   float* num;                  // [M][heads][ldo]
   double *u, *mx;              // prompt blocks: [heads][Mcap]
   float* a;                    // prompt blocks: [chunk][heads][64][64] decayed scores
