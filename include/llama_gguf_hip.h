@@ -160,7 +160,10 @@ enum {
   LGH_SYM_MVQ_MIXED = 17,  /* lgh::mvq_kernel<3u> : ... Q4_K and Q6_K matrices in one launch (fused QKV of Q4_K_M) */
   LGH_SYM_MVQ_Q5K = 18,    /* lgh::mvq_kernel<4u> / <6u> : Q5_K (and Q5_K + Q6_K) */
   LGH_SYM_MVQ_Q80_Q40 = 19, /* lgh::mvq_kernel<8u> / <16u> : Q8_0 / Q4_0 */
-  LGH_SYM_PTOK = 20,       /* (unused since round 3) */
+  LGH_SYM_PTOK = 20,       /* (unused) */
+  LGH_SYM_LINEAR = 21,     /* lgh::lin_mv_kernel / lgh::lin_gemm_kernel : products over weights kept in bf16 (lgh_create_layered) */
+  LGH_SYM_LATENT = 22,     /* lgh::latent_* : attention over a shared latent */
+  LGH_SYM_MLSTM = 23,      /* lgh::mlstm_* : matrix-memory recurrence */
   LGH_SYM_COUNT = 24
 };
 
@@ -261,6 +264,48 @@ int lgh_set_kv_qjl_matrices(lgh_ctx* ctx, const float* matrices, size_t n);
  * (S r)_i >= 0, r the residual) and *residual_norm.  Bit-exact with the reference's arithmetic for the given matrix. */
 int lgh_op_tq_compress_qjl(int device, int bits, const float* x, size_t dim, const float* signs, const float* qjl_matrix, uint8_t* codes,
                            uint64_t* qjl_bits, float* residual_norm);
+
+/* A portion of the sequence with logits inside it: tokens[0..n) at the context's position, as lgh_prefill_batch feeds them (block
+ * products where the model has them, otherwise one step per token), and the logits after tokens want[0..n_want) (ascending places
+ * within the portion) -> logits_out [n_want][vocab_size]; n_want may be 0.  Portions may be cut anywhere. */
+int lgh_eval(lgh_ctx* ctx, const uint32_t* tokens, size_t n, const uint32_t* want, size_t n_want, float* logits_out);
+
+/* ---- models whose layers are described one by one: every layer has a mixer (attention or a recurrence) and, optionally, a
+ * feed-forward; sublayers read the residual stream itself and their outputs are layer-normed, x += residual_mult * norm(sublayer(x)).
+ * No reference counterpart.  The context is driven by the entry points above (GpuInference, lgh_eval, lgh_decode_greedy, ...; the
+ * cache rows and recurrent states are the context's).  Weights are bf16 and stay bf16 in HBM; tensors are uploaded by their
+ * checkpoint names (`embed`, `bigram`, `l0.mix.q`, `l0.mlp.gate`, `l0.norm1`, `final.norm`, `head`) with GGML dims (in fastest).
+ * Single stage, one sequence per context. ---- */
+enum { LGH_MIXER_LATENT_ATTENTION = 1, LGH_MIXER_MLSTM = 2 };
+enum { LGH_FF_NONE = 0, LGH_FF_GEGLU = 1 };            /* down(gelu_tanh(gate x) * (up x)) */
+enum { LGH_COMPUTE_BF16 = 0, LGH_COMPUTE_F32 = 1 };    /* operands of block products, cache rows: bf16 (f32 accumulation), or f32 throughout */
+typedef struct lgh_layer_desc {
+  uint32_t struct_size;
+  uint32_t mixer;                    /* LGH_MIXER_* */
+  uint32_t heads, dim, vdim;         /* query / key size per head (latent attention: the unrotated part), value size per head */
+  uint32_t kv_rank, rot_dim;         /* latent attention: latent size, rotated query / key part */
+  uint32_t rot_dims;                 /* leading values of the rotated part that are rotated (neighbouring pairs) */
+  uint32_t ff_kind, ff;              /* LGH_FF_*, feed-forward size */
+  double scale;                      /* latent attention: factor on the scores */
+  double rot_base;
+  double yarn_factor, yarn_original, yarn_fast, yarn_slow;   /* yarn_factor 0: plain frequencies */
+  double gate_cap;                   /* mLSTM: soft cap of the gates' pre-activations */
+} lgh_layer_desc;
+typedef struct lgh_layered_desc {
+  uint32_t struct_size;
+  uint32_t width, vocab_size, num_layers, max_seq_len;
+  uint32_t compute;                  /* LGH_COMPUTE_* */
+  int32_t device_id;
+  uint32_t flags;                    /* LGH_FLAG_NO_GRAPH, LGH_FLAG_EXACT_PREFILL, LGH_FLAG_ATTN_SPLITS_SHIFT */
+  uint32_t bigram_buckets;           /* 0: no pair embedding */
+  uint64_t bigram_mul_prev, bigram_mul_cur;
+  double norm_eps, residual_mult;
+} lgh_layered_desc;
+int lgh_create_layered(const lgh_layered_desc* desc, const lgh_layer_desc* layers, lgh_ctx** out);
+/* Residual stream after every layer, for parity tests: switched on, the next lgh_eval portions (block path) keep it;
+ * lgh_read_layers copies [num_layers][tokens of the last portion][width] f32. */
+int lgh_set_layer_tap(lgh_ctx* ctx, int on);
+int lgh_read_layers(lgh_ctx* ctx, float* out, size_t n_floats);
 
 /* ---- multi-sequence decode: the device side of BatchedEngine (src/engine_batched.rs:23-194, 200-330, 355-400) ----
  * The reference keeps one InferenceContext (KV cache + position) per ActiveSequence (engine_batched.rs:84-100, 332-353) and every

@@ -77,6 +77,8 @@ struct BatchScratch {
   hipGraphExec_t graph[kMaxBatch + 1][2] = {};        // [n_seq][0 logits only, 1 + arg-max fed back]
 };
 
+struct LayeredModel;   // layered.hip: models described layer by layer
+
 }  // namespace lgh
 
 struct lgh_ctx {
@@ -120,6 +122,7 @@ struct lgh_ctx {
   std::vector<float> tq_signs_host;
   float* tq_qjl = nullptr;                     // TurboQuantProd: [owned layer][kv head][head_dim][head_dim] QJL projection matrices (device)
   std::vector<float> tq_qjl_host;
+  lgh::LayeredModel* lm = nullptr;             // set by lgh_create_layered: layers, weights, caches and states live there
   float* kv_shift_tmp = nullptr;               // scratch of lgh_kv_shift_left (one cache tensor), allocated at first use
 };
 
@@ -161,6 +164,7 @@ int build_mv_group(lgh_ctx* c, const SegSpec* specs, int nseg, const float* norm
 int ffn_forward(lgh_ctx* c, lgh::LayerW& Lw, const FfnView& v, const float* next_nw, bool next_mfma);
 int engine_shape_check(const lgh_model_desc& d, std::string& why);   // LGH_OK, or the status lgh_create returns and why
 int dev_alloc(lgh_ctx* c, void** p, size_t bytes);
+void dev_free_tracked(lgh_ctx* c, void* p);
 LayoutInfo layout_for(int src_type);
 bool fused_type(int t);
 int upload_matrix(lgh_ctx* c, lgh::DevWeight& W, int src_type, uint32_t k, uint32_t n, uint32_t n_stack, int slot,
@@ -172,6 +176,15 @@ void xq_stale(lgh_ctx* c, const float* f32);
 int linear_any(lgh_ctx* c, int cls, const lgh::DevWeight& W, const float* x, float* out, const float* norm_w,
                const float* resid, const float* bias, int xq_next = 0, const float* xq_next_nw = nullptr);
 int drain_prof(lgh_ctx* c);
+// layered.hip, behind the entry points of engine.hip when c->lm is set
+int layered_upload(lgh_ctx* c, const char* name, uint32_t type, const uint64_t ne[4], const void* host, size_t nbytes);
+int layered_finalize(lgh_ctx* c);
+int layered_enqueue_token(lgh_ctx* c, int mode);
+bool layered_has_blocks(const lgh_ctx* c);
+int layered_block(lgh_ctx* c, const uint32_t* tokens, size_t n, const uint32_t* want, size_t n_want, float* logits_out);   // any n >= 1
+bool layered_recurrent(const lgh_ctx* c);
+uint64_t layered_step_bytes(const lgh_ctx* c);
+void layered_destroy(lgh_ctx* c);
 
 // ------------------------------------------------------------------------------------------------
 // launch recording (profiling mode: hipEvent pair per launch, on the launch stream)

@@ -54,7 +54,7 @@ int dev_alloc(lgh_ctx* c, void** p, size_t bytes) {
   return LGH_OK;
 }
 
-static void dev_free_tracked(lgh_ctx* c, void* p) {
+void dev_free_tracked(lgh_ctx* c, void* p) {
   for (auto& a : c->allocs)
     if (a == p) { a = c->allocs.back(); c->allocs.pop_back(); break; }
   (void)hipFree(p);
@@ -637,6 +637,7 @@ static int layer_forward(lgh_ctx* c, uint32_t li, const float* next_nw, bool nex
 
 // Everything one token needs, in stream order.  Used eagerly and under graph capture.
 static int enqueue_token(lgh_ctx* c, int mode) {
+  if (c->lm) return layered_enqueue_token(c, mode);
   const lgh_model_desc& d = c->d;
   int rc;
   for (auto& q : c->xqs) q.fresh = false;   // the residual stream is (re)written in f32 now (embedding / previous stage)
@@ -773,6 +774,7 @@ static int set_token(lgh_ctx* c, uint32_t token) {
 // batched prompt processing (prefill.hip)
 // ------------------------------------------------------------------------------------------------
 static bool pf_eligible(const lgh_ctx* c) {
+  if (c->lm) return false;   // (models described layer by layer have their own block path)
   const lgh_model_desc& d = c->d;
   if (d.flags & (LGH_FLAG_EXACT_PREFILL | LGH_FLAG_KV_INT8)) return false;   // (the batched path writes f32 K/V rows)
   const uint32_t QD = d.num_heads * d.head_dim, KD = d.num_kv_heads * d.head_dim, g = d.num_heads / d.num_kv_heads;
@@ -1071,6 +1073,7 @@ int lgh_upload_tensor(lgh_ctx* c, const char* name, uint32_t type, const uint64_
   if (!c || !name || !ne || !host) return LGH_INVALID_ARGUMENT;
   if (bind(c)) return fail(c, LGH_NOT_AVAILABLE, "hipSetDevice failed");
   if (c->finalized) return fail(c, LGH_INVALID_ARGUMENT, "upload after finalize");
+  if (c->lm) return layered_upload(c, name, type, ne, host, nbytes);
   const lgh_model_desc& d = c->d;
   const std::string nm(name);
   const uint64_t n0 = ne[0], n1 = ne[1] ? ne[1] : 1, n2 = ne[2] ? ne[2] : 1;
@@ -1166,6 +1169,12 @@ int lgh_finalize(lgh_ctx* c) {
   if (c->finalized) return LGH_OK;
   const lgh_model_desc& d = c->d;
   int rc;
+  if (c->lm) {
+    if ((rc = layered_finalize(c))) return rc;
+    c->finalized = true;
+    c->pos = 0;
+    return warm_kernels(c);
+  }
   if (c->first && !c->embd_raw) return fail(c, LGH_INITIALIZATION_FAILED, "missing token_embd.weight");
   if (c->last) {
     if (!c->output_norm) return fail(c, LGH_INITIALIZATION_FAILED, "missing output_norm.weight");
@@ -1340,6 +1349,7 @@ void lgh_destroy(lgh_ctx* c) {
   if (c->pf.tok_pinned) (void)hipHostFree(c->pf.tok_pinned);
   if (c->pf.tok_copied) (void)hipEventDestroy(c->pf.tok_copied);
   if (c->own_stream) (void)hipStreamDestroy(c->own_stream);
+  layered_destroy(c);
   delete c;
 }
 
@@ -1370,7 +1380,7 @@ int lgh_prefill_token(lgh_ctx* c, uint32_t token) {
   return step(c, MODE_PREFILL);
 }
 
-int lgh_prefill_is_batched(lgh_ctx* c) { return c && c->finalized && pf_eligible(c) ? 1 : 0; }
+int lgh_prefill_is_batched(lgh_ctx* c) { return c && c->finalized && (c->lm ? layered_has_blocks(c) : pf_eligible(c)) ? 1 : 0; }
 
 int lgh_stage_hidden_block_buffer(lgh_ctx* c, void** p) {
   int rc = check_ready(c);
@@ -1399,6 +1409,7 @@ int lgh_prefill_batch(lgh_ctx* c, const uint32_t* tokens, size_t n) {
   int rc = check_ready(c);
   if (rc) return rc;
   if (n && !tokens) return fail(c, LGH_INVALID_ARGUMENT, "tokens is NULL");
+  if (c->lm && n >= 2 && layered_has_blocks(c)) return lgh_eval(c, tokens, n, nullptr, 0, nullptr);
   if (n >= 2 && c->first && c->last && pf_eligible(c)) {
     if (c->pos + n > c->d.max_seq_len)
       return fail(c, LGH_INVALID_ARGUMENT, "prompt of " + std::to_string(n) + " tokens at position " + std::to_string(c->pos) + " exceeds max_seq_len");
@@ -1411,6 +1422,31 @@ int lgh_prefill_batch(lgh_ctx* c, const uint32_t* tokens, size_t n) {
   }
   for (size_t i = 0; i < n; i++)
     if ((rc = lgh_prefill_token(c, tokens[i]))) return rc;
+  HIP_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
+  return LGH_OK;
+}
+
+int lgh_eval(lgh_ctx* c, const uint32_t* tokens, size_t n, const uint32_t* want, size_t n_want, float* logits_out) {
+  int rc = check_ready(c);
+  if (rc) return rc;
+  if (!c->first || !c->last) return fail(c, LGH_INVALID_ARGUMENT, "lgh_eval needs a single-stage context");
+  if ((n && !tokens) || (n_want && (!want || !logits_out))) return fail(c, LGH_INVALID_ARGUMENT, "a pointer is NULL");
+  if (c->pos + n > c->d.max_seq_len)
+    return fail(c, LGH_INVALID_ARGUMENT, "portion of " + std::to_string(n) + " tokens at position " + std::to_string(c->pos) + " exceeds max_seq_len");
+  for (size_t i = 0; i < n; i++)
+    if (tokens[i] >= c->d.vocab_size) return fail(c, LGH_INVALID_ARGUMENT, "token id exceeds vocab size");
+  for (size_t i = 0; i < n_want; i++)
+    if (want[i] >= n || (i && want[i] <= want[i - 1])) return fail(c, LGH_INVALID_ARGUMENT, "wanted places must ascend within the portion");
+  if (c->lm && n >= 2 && layered_has_blocks(c)) return layered_block(c, tokens, n, want, n_want, logits_out);
+  // stretches without a wanted place as prompt blocks, wanted places as steps
+  size_t at = 0;
+  for (size_t i = 0; i < n_want; i++) {
+    const size_t len = want[i] - at;
+    if (len && (rc = lgh_prefill_batch(c, tokens + at, len))) return rc;
+    if ((rc = lgh_forward(c, tokens[want[i]], logits_out + i * (size_t)c->d.vocab_size))) return rc;
+    at = want[i] + 1;
+  }
+  if (at < n) return lgh_prefill_batch(c, tokens + at, n - at);
   HIP_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
   return LGH_OK;
 }
@@ -1461,6 +1497,8 @@ size_t lgh_position(const lgh_ctx* c) { return c ? c->pos : 0; }
 int lgh_kv_truncate(lgh_ctx* c, size_t new_len) {
   int rc = check_ready(c);
   if (rc) return rc;
+  if (c->lm && layered_recurrent(c) && new_len < c->pos && new_len)
+    return fail(c, LGH_UNSUPPORTED, "a recurrent state cannot be cut back to an earlier position (only to 0)");
   if (new_len < c->pos) {   // KVCache::truncate (model/mod.rs:130-134): only ever shortens
     c->pos = new_len;
     HIP_TRY(c, LGH_OPERATION_FAILED, hipMemsetD32Async((hipDeviceptr_t)(c->state + ST_NEXT), (int)c->pos, 1, c->stream));
@@ -1472,6 +1510,7 @@ int lgh_kv_shift_left(lgh_ctx* c, size_t amount) {
   int rc = check_ready(c);
   if (rc) return rc;
   const lgh_model_desc& d = c->d;
+  if (c->lm && amount && amount < c->pos) return fail(c, LGH_UNSUPPORTED, "this model's cache and states cannot drop their first positions");
   if (amount == 0 || amount >= c->pos) {   // model/mod.rs:143-146 — a shift by 0 clears the cache too
     c->pos = 0;
   } else {
@@ -1545,7 +1584,8 @@ int lgh_get_stats(lgh_ctx* c, lgh_stats* out) {
   // algorithmic bytes of one decode step at the current position
   uint64_t b = 0;
   const lgh_model_desc& d = c->d;
-  if (c->finalized) {
+  if (c->finalized && c->lm) b = layered_step_bytes(c);
+  else if (c->finalized) {
     if (c->first) b += (uint64_t)d.hidden_size * blk_bytes(c->embd_type) / blk_elems(c->embd_type);
     for (uint32_t i = c->l0; i < c->l1; i++) {
       const LayerW& L = c->layers[i];

@@ -130,6 +130,7 @@ int launch_mvb(lgh_ctx* c, int cls, const SegSpec* specs, int nseg, const float*
 
 bool batch_weights_ok(const lgh_ctx* c, std::string& why) {
   const lgh_model_desc& d = c->d;
+  if (c->lm) { why = "a model described layer by layer holds one sequence per context"; return false; }
   if (d.hidden_size % 256 || (d.num_heads * d.head_dim) % 256) { why = "hidden size and heads x head_dim must be multiples of 256"; return false; }
   if (d.use_neox_rope) { why = "NeoX RoPE is not fused into the QKV launch"; return false; }
   if (!attn_shape_has_fast_kernel(d.head_dim, d.num_heads / d.num_kv_heads)) { why = "attention shape outside the split kernels"; return false; }

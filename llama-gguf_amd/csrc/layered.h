@@ -65,7 +65,6 @@ hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st);
 hipError_t lin_pack_launch(const uint16_t* src, uint32_t rows, uint32_t k, uint16_t* dst, uint32_t kp, uint32_t row0, int mode, hipStream_t st);
 // per head [dim][rank] -> [rank][dimp]
 hipError_t lin_transpose_heads_launch(const uint16_t* src, uint32_t heads, uint32_t dim, uint32_t rank, uint16_t* dst, uint32_t dimp, hipStream_t st);
-hipError_t bf16_to_f32_launch(const uint16_t* src, float* dst, uint64_t n, hipStream_t st);
 
 // ---- layered_misc.hip ----
 struct EmbedArgs {

@@ -1,0 +1,633 @@
+// layered.hip — models whose layers are described one by one (lgh_create_layered): weight store, cache rows and recurrent states, the
+// decode launch sequence (captured in the engine's token graphs) and the block path for prompt portions.
+//
+// Decode, per token (every residual update rides in the prologue of the product that reads it):
+//   latent attention   fused q | latent | gate product -> queries absorbed, cache row written -> split attention -> merge + value
+//                      expansion + gate -> output product
+//   mLSTM              fused q | k | v | gates product -> recurrence step -> output product (read-out norm and gate in its prologue)
+//   feed-forward       gate | up product with gelu * in its epilogue -> down product
+// A sequence's state: the cache rows, the matrix memories with their running maxima, and the last token (pair embedding), kept as a
+// token history by position; a position of 0 makes every kernel ignore what is stored, so lgh_reset stays O(1).
+#include <algorithm>
+#include <cmath>
+#include <map>
+
+#include "engine.h"
+#include "layered.h"
+
+using namespace lgh;
+
+namespace lgh {
+
+constexpr uint32_t kBlockTokens = 2048;    // tokens per pass of the block path
+constexpr uint32_t kLogitRows = 128;       // wanted rows per output product
+
+struct LayeredLayer {
+  lgh_layer_desc d{};
+  LinW in, out, gu, down, uk, uv;          // mixer inputs (one product), mixer output, gate | up, down, latent expansions
+  uint16_t* uk_t = nullptr;
+  float *norm1 = nullptr, *norm2 = nullptr, *dkv_norm = nullptr, *mnorm = nullptr, *bi = nullptr, *bf = nullptr, *cs = nullptr;
+  void* cache = nullptr;
+  float* S = nullptr;
+  double* m = nullptr;
+  LatentShape ls{};
+  MlstmShape ms{};
+  bool latent() const { return d.mixer == LGH_MIXER_LATENT_ATTENTION; }
+};
+
+struct LayeredSlot {                       // where a named tensor goes
+  LinW* mat = nullptr;
+  uint32_t row0 = 0, n = 0, k = 0;
+  int mode = 0;
+  float** vec = nullptr;
+  uint16_t** raw = nullptr;
+  LayeredLayer* transpose = nullptr;
+  bool done = false;
+};
+
+struct LayeredModel {
+  lgh_layered_desc d{};
+  std::vector<LayeredLayer> layers;
+  std::map<std::string, LayeredSlot> slots;
+  uint16_t *embed = nullptr, *bigram = nullptr;
+  LinW head;
+  float* final_norm = nullptr;
+  int* hist = nullptr;
+  bool f32 = false, recurrent = false;
+  uint32_t n_sub = 0, n_splits = 1;
+  // decode
+  float *x[2] = {nullptr, nullptr}, *y = nullptr, *cat = nullptr, *ao = nullptr, *act = nullptr, *num = nullptr, *part_ml = nullptr, *part_acc = nullptr;
+  void* qa = nullptr;
+  uint32_t max_cat = 0, max_ao = 0, max_act = 0, max_num = 0;
+  // blocks
+  bool blk_ready = false;
+  uint32_t blk = 0;
+  float *bx = nullptr, *by = nullptr, *bcat = nullptr, *bnum = nullptr, *ba = nullptr, *blogits = nullptr;
+  double *bu = nullptr, *bmx = nullptr;
+  void *bxa = nullptr, *bao = nullptr, *bact = nullptr, *bla = nullptr;
+  int *btok = nullptr, *brows = nullptr;
+  // expanded attention (grown with the context)
+  LatentFlash fl{};
+  size_t fl_q_bytes = 0, fl_k_bytes = 0, fl_v_bytes = 0;
+  // layer tap
+  bool tap = false;
+  float* tap_buf = nullptr;
+  uint32_t tap_tokens = 0;
+  uint32_t el() const { return f32 ? 4 : 2; }
+};
+
+}  // namespace lgh
+
+static uint32_t up(uint32_t v, uint32_t a) { return (v + a - 1) / a * a; }
+
+#define L_TRY(c, status, expr)                                                                                    \
+  do {                                                                                                            \
+    hipError_t e__ = (expr);                                                                                      \
+    if (e__ != hipSuccess) return fail((c), (status), std::string(#expr) + ": " + hipGetErrorString(e__));        \
+  } while (0)
+
+void layered_destroy(lgh_ctx* c) {
+  delete c->lm;
+  c->lm = nullptr;
+}
+bool layered_recurrent(const lgh_ctx* c) { return c->lm->recurrent; }
+bool layered_has_blocks(const lgh_ctx* c) { return !(c->d.flags & LGH_FLAG_EXACT_PREFILL); }
+
+// What the kernels can hold, checked before anything is allocated
+static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std::string& why) {
+  if (!d.width || !d.vocab_size || !d.num_layers || !d.max_seq_len) { why = "a model dimension is zero"; return LGH_INVALID_ARGUMENT; }
+  if (d.compute > LGH_COMPUTE_F32) { why = "unknown compute type"; return LGH_INVALID_ARGUMENT; }
+  if (!(d.norm_eps >= 0.0) || !std::isfinite(d.residual_mult)) { why = "norm_eps / residual_mult"; return LGH_INVALID_ARGUMENT; }
+  if (up(d.width, 64) > 32768) { why = "width above 32768"; return LGH_UNSUPPORTED; }
+  for (uint32_t i = 0; i < d.num_layers; i++) {
+    const lgh_layer_desc& l = L[i];
+    const std::string at = "layer " + std::to_string(i) + ": ";
+    if (l.struct_size != sizeof(lgh_layer_desc)) { why = at + "descriptor size"; return LGH_INVALID_ARGUMENT; }
+    if (!l.heads || !l.dim || !l.vdim) { why = at + "a mixer dimension is zero"; return LGH_INVALID_ARGUMENT; }
+    if (l.ff_kind > LGH_FF_GEGLU || (l.ff_kind && !l.ff)) { why = at + "feed-forward"; return LGH_INVALID_ARGUMENT; }
+    if (l.ff_kind && up(l.ff, 64) > kLinMvMaxK) { why = at + "feed-forward above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
+    if (up(l.heads * l.vdim, 64) > kLinMvMaxK) { why = at + "heads * vdim above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
+    if (l.mixer == LGH_MIXER_LATENT_ATTENTION) {
+      if (!l.kv_rank || l.rot_dims > l.rot_dim || l.rot_dims % 2) { why = at + "latent attention sizes"; return LGH_INVALID_ARGUMENT; }
+      if (l.rot_dims && !(l.rot_base > 0.0)) { why = at + "rotation base"; return LGH_INVALID_ARGUMENT; }
+      LatentShape s{};
+      s.rank = l.kv_rank;
+      s.ldc = up(l.kv_rank + l.rot_dim, 32);
+      if (l.heads > kLatAbsorbRows || !latent_key_tile(s, d.compute == LGH_COMPUTE_F32, 1)) { why = at + "latent rows too large for LDS"; return LGH_UNSUPPORTED; }
+    } else if (l.mixer == LGH_MIXER_MLSTM) {
+      if (!(l.gate_cap > 0.0)) { why = at + "gate_cap"; return LGH_INVALID_ARGUMENT; }
+      if (l.dim > kMlstmMaxDim) { why = at + "matrix memory: dim above " + std::to_string(kMlstmMaxDim); return LGH_UNSUPPORTED; }
+    } else { why = at + "unknown mixer"; return LGH_UNSUPPORTED; }
+  }
+  return LGH_OK;
+}
+
+// rows of a fused product: segments one below another, each starting at a multiple of 16
+static uint32_t seg(LinW& W, uint32_t rows) {
+  const uint32_t at = up(W.n, 16);
+  W.n = at + rows;
+  return at;
+}
+
+static void add_mat(LayeredModel& m, const std::string& nm, LinW* W, uint32_t row0, uint32_t n, uint32_t k, int mode = 0) {
+  LayeredSlot s;
+  s.mat = W; s.row0 = row0; s.n = n; s.k = k; s.mode = mode;
+  m.slots[nm] = s;
+}
+static void add_vec(LayeredModel& m, const std::string& nm, float** v, uint32_t n) {
+  LayeredSlot s;
+  s.vec = v; s.n = n;
+  m.slots[nm] = s;
+}
+
+// sizes, offsets and the tensor table of every layer
+static void layered_plan(LayeredModel& m) {
+  const lgh_layered_desc& d = m.d;
+  const uint32_t W = d.width;
+  {
+    LayeredSlot s;
+    s.raw = &m.embed; s.n = d.vocab_size; s.k = W;
+    m.slots["embed"] = s;
+    if (d.bigram_buckets) { s.raw = &m.bigram; s.n = d.bigram_buckets + 1; m.slots["bigram"] = s; }
+  }
+  auto whole = [&](LinW& L, uint32_t n, uint32_t k) { L.n = n; L.k = k; L.kp = up(k, 64); };
+  for (uint32_t i = 0; i < d.num_layers; i++) {
+    LayeredLayer& L = m.layers[i];
+    const lgh_layer_desc& l = L.d;
+    const std::string p = "l" + std::to_string(i) + ".";
+    add_vec(m, p + "norm1", &L.norm1, W);
+    m.n_sub++;
+    L.in.k = W; L.in.kp = up(W, 64);
+    const uint32_t vd = l.heads * l.vdim;
+    auto in_seg = [&](const char* nm, uint32_t rows) { const uint32_t at = seg(L.in, rows); add_mat(m, p + "mix." + nm, &L.in, at, rows, W); return at; };
+    if (L.latent()) {
+      LatentShape& s = L.ls;
+      s.heads = l.heads; s.dim = l.dim; s.rot_dim = l.rot_dim; s.rot_n = l.rot_dims; s.vdim = l.vdim; s.rank = l.kv_rank;
+      s.ldc = up(l.kv_rank + l.rot_dim, 32);
+      s.dimp = up(l.dim, 8);
+      s.rankp = up(l.kv_rank, 64);
+      s.scale = (float)l.scale; s.eps = (float)d.norm_eps;
+      s.off_q = in_seg("q", l.heads * (l.dim + l.rot_dim));
+      s.off_dkv = in_seg("dkv", l.kv_rank + l.rot_dim);
+      s.off_g = in_seg("g", l.heads);
+      L.in.n = up(L.in.n, 16);
+      s.ldcat = L.in.n;
+      add_vec(m, p + "mix.dkv.norm", &L.dkv_norm, l.kv_rank);
+      whole(L.uk, l.heads * l.dim, l.kv_rank);
+      whole(L.uv, vd, l.kv_rank);
+      add_mat(m, p + "mix.uk", &L.uk, 0, L.uk.n, l.kv_rank);
+      m.slots[p + "mix.uk"].transpose = &L;
+      add_mat(m, p + "mix.uv", &L.uv, 0, vd, l.kv_rank);
+    } else {
+      MlstmShape& s = L.ms;
+      s.heads = l.heads; s.dim = l.dim; s.vdim = l.vdim;
+      s.lds = up(l.vdim + 1, 16); s.ldo = up(l.vdim + 2, 4);
+      s.cap = (float)l.gate_cap; s.eps = (float)d.norm_eps;
+      s.off_q = in_seg("q", l.heads * l.dim);
+      s.off_k = in_seg("k", l.heads * l.dim);
+      s.off_v = in_seg("v", vd);
+      s.off_g = in_seg("g", vd);
+      s.off_i = in_seg("i", l.heads);
+      s.off_f = in_seg("f", l.heads);
+      L.in.n = up(L.in.n, 16);
+      s.ldcat = L.in.n;
+      add_vec(m, p + "mix.i.b", &L.bi, l.heads);
+      add_vec(m, p + "mix.f.b", &L.bf, l.heads);
+      add_vec(m, p + "mix.norm", &L.mnorm, vd);
+      m.recurrent = true;
+      m.max_num = std::max(m.max_num, l.heads * s.ldo);
+    }
+    m.max_cat = std::max(m.max_cat, L.in.n);
+    whole(L.out, W, vd);
+    add_mat(m, p + "mix.o", &L.out, 0, W, vd);
+    m.max_ao = std::max(m.max_ao, L.out.kp);
+    if (l.ff_kind) {
+      m.n_sub++;
+      add_vec(m, p + "norm2", &L.norm2, W);
+      whole(L.gu, 2 * up(l.ff, 16), W);
+      L.gu.paired = true;
+      add_mat(m, p + "mlp.gate", &L.gu, 0, l.ff, W, 1);
+      add_mat(m, p + "mlp.up", &L.gu, 0, l.ff, W, 2);
+      whole(L.down, W, l.ff);
+      add_mat(m, p + "mlp.down", &L.down, 0, W, l.ff);
+      m.max_act = std::max(m.max_act, L.down.kp);
+    }
+  }
+  add_vec(m, "final.norm", &m.final_norm, W);
+  whole(m.head, d.vocab_size, W);
+  add_mat(m, "head", &m.head, 0, d.vocab_size, W);
+}
+
+extern "C" int lgh_create_layered(const lgh_layered_desc* desc, const lgh_layer_desc* layers, lgh_ctx** out) {
+  if (!desc || !layers || !out || desc->struct_size != sizeof(lgh_layered_desc)) return LGH_INVALID_ARGUMENT;
+  *out = nullptr;
+  if (desc->flags & LGH_FLAG_REMOVED_MASK) return LGH_UNSUPPORTED;
+  std::string why;
+  if (int rc = layered_check(*desc, layers, why)) return rc;
+  const int ndev = lgh_device_count();
+  if (ndev <= 0 || desc->device_id < 0 || desc->device_id >= ndev) return LGH_NOT_AVAILABLE;
+  lgh_ctx* c = new lgh_ctx();
+  lgh_model_desc& d = c->d;   // what the engine's shared entry points read
+  d.struct_size = sizeof(d);
+  d.hidden_size = desc->width; d.vocab_size = desc->vocab_size; d.num_layers = desc->num_layers; d.max_seq_len = desc->max_seq_len;
+  d.norm_eps = (float)desc->norm_eps; d.device_id = desc->device_id; d.flags = desc->flags & ~(uint32_t)LGH_FLAG_KV_INT8;
+  c->device = d.device_id;
+  c->l0 = 0; c->l1 = d.num_layers;
+  c->direct_attn_max_kv = 0;   // one attention structure
+  if (hipSetDevice(c->device) != hipSuccess || hipStreamCreateWithFlags(&c->own_stream, hipStreamNonBlocking) != hipSuccess) {
+    delete c;
+    return LGH_INITIALIZATION_FAILED;
+  }
+  c->stream = c->own_stream;
+  LayeredModel* m = new LayeredModel();
+  c->lm = m;
+  m->d = *desc;
+  m->f32 = desc->compute == LGH_COMPUTE_F32;
+  m->layers.resize(d.num_layers);
+  for (uint32_t i = 0; i < d.num_layers; i++) m->layers[i].d = layers[i];
+  layered_plan(*m);
+  *out = c;
+  return LGH_OK;
+}
+
+static int zeroed(lgh_ctx* c, void** p, size_t bytes, uint64_t* account) {
+  if (int rc = dev_alloc(c, p, bytes)) return rc;
+  if (bytes) L_TRY(c, LGH_OPERATION_FAILED, hipMemsetAsync(*p, 0, bytes, c->stream));
+  if (account) *account += bytes;
+  return LGH_OK;
+}
+
+int layered_upload(lgh_ctx* c, const char* name, uint32_t type, const uint64_t ne[4], const void* host, size_t nbytes) {
+  LayeredModel& m = *c->lm;
+  const std::string nm(name);
+  auto it = m.slots.find(nm);
+  if (it == m.slots.end()) return fail(c, LGH_INVALID_ARGUMENT, "unknown tensor name " + nm);
+  LayeredSlot& s = it->second;
+  const uint64_t n0 = ne[0], n1 = ne[1] ? ne[1] : 1, n2 = ne[2] ? ne[2] : 1;
+  int rc;
+  if (s.vec) {
+    if (n0 * n1 * n2 != s.n) return fail(c, LGH_SHAPE_MISMATCH, nm + ": expected " + std::to_string(s.n) + " elements");
+    if ((rc = upload_f32(c, s.vec, (int)type, s.n, host, nbytes))) return rc;
+    s.done = true;
+    return LGH_OK;
+  }
+  if (type != LGH_TYPE_BF16) return fail(c, LGH_DTYPE_MISMATCH, nm + ": matrices of this model are bf16");
+  if (n0 != s.k || n1 != s.n || n2 != 1) return fail(c, LGH_SHAPE_MISMATCH, nm + ": expected [" + std::to_string(s.k) + "," + std::to_string(s.n) + "]");
+  if (nbytes != (size_t)s.n * s.k * 2) return fail(c, LGH_SHAPE_MISMATCH, nm + ": byte size does not match its shape");
+  if (s.raw) {
+    if (!*s.raw && (rc = dev_alloc(c, (void**)s.raw, nbytes))) return rc;
+    L_TRY(c, LGH_OPERATION_FAILED, hipMemcpy(*s.raw, host, nbytes, hipMemcpyHostToDevice));
+    c->stats.weight_bytes += s.done ? 0 : nbytes;
+    s.done = true;
+    return LGH_OK;
+  }
+  LinW& W = *s.mat;
+  if (!W.w && (rc = zeroed(c, (void**)&W.w, (size_t)W.np() * W.kp * 2, nullptr))) return rc;
+  void* raw = nullptr;
+  L_TRY(c, LGH_ALLOCATION_FAILED, hipMalloc(&raw, nbytes));
+  hipError_t e = hipMemcpy(raw, host, nbytes, hipMemcpyHostToDevice);
+  if (e == hipSuccess) e = lin_pack_launch((const uint16_t*)raw, s.n, s.k, W.w, W.kp, s.row0, s.mode, c->stream);
+  if (e == hipSuccess && s.transpose) {
+    LayeredLayer& L = *s.transpose;
+    const size_t tb = (size_t)L.ls.heads * L.ls.rank * L.ls.dimp * 2;
+    if (!L.uk_t && (rc = zeroed(c, (void**)&L.uk_t, tb, nullptr))) { (void)hipFree(raw); return rc; }
+    e = lin_transpose_heads_launch((const uint16_t*)raw, L.ls.heads, L.ls.dim, L.ls.rank, L.uk_t, L.ls.dimp, c->stream);
+  }
+  if (e == hipSuccess) e = hipStreamSynchronize(c->stream);
+  (void)hipFree(raw);
+  if (e != hipSuccess) return fail(c, LGH_OPERATION_FAILED, nm + ": " + hipGetErrorString(e));
+  c->stats.weight_bytes += s.done ? 0 : nbytes;
+  s.done = true;
+  return LGH_OK;
+}
+
+// cos / sin of every position: angles in 64-bit, with the YaRN blend of frequencies when the layer asks for it
+static std::vector<float> rotation_table(const lgh_layer_desc& l, uint32_t max_seq) {
+  const uint32_t np = l.rot_dims / 2;
+  std::vector<double> f(np);
+  for (uint32_t i = 0; i < np; i++) f[i] = std::pow(l.rot_base, -2.0 * i / l.rot_dims);
+  double mag = 1.0;
+  if (l.yarn_factor > 0.0) {
+    auto turn = [&](double t) { return l.rot_dims * std::log(l.yarn_original / (2.0 * M_PI * t)) / (2.0 * std::log(l.rot_base)); };
+    const double lo = std::max(std::floor(turn(l.yarn_fast)), 0.0), hi = std::min(std::ceil(turn(l.yarn_slow)), (double)l.rot_dims - 1.0);
+    for (uint32_t i = 0; i < np; i++) {
+      const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+      f[i] = f[i] / l.yarn_factor * ramp + f[i] * (1.0 - ramp);
+    }
+    mag = 0.1 * std::log(l.yarn_factor) + 1.0;
+  }
+  std::vector<float> cs((size_t)max_seq * np * 2);
+  for (uint32_t p = 0; p < max_seq; p++)
+    for (uint32_t i = 0; i < np; i++) {
+      cs[((size_t)p * np + i) * 2] = (float)(std::cos(p * f[i]) * mag);
+      cs[((size_t)p * np + i) * 2 + 1] = (float)(std::sin(p * f[i]) * mag);
+    }
+  return cs;
+}
+
+int layered_finalize(lgh_ctx* c) {
+  LayeredModel& m = *c->lm;
+  std::string missing;
+  for (auto& s : m.slots)
+    if (!s.second.done) missing += (missing.empty() ? "" : ", ") + s.first;
+  if (!missing.empty()) return fail(c, LGH_INITIALIZATION_FAILED, "missing tensors: " + missing.substr(0, 400));
+  const lgh_layered_desc& d = m.d;
+  int rc;
+  uint32_t max_rows = 0, max_rank = 0, max_ldc = 0;
+  for (uint32_t i = 0; i < d.num_layers; i++) {
+    LayeredLayer& L = m.layers[i];
+    if (L.latent()) {
+      if ((rc = zeroed(c, &L.cache, (size_t)d.max_seq_len * L.ls.ldc * m.el(), &c->stats.kv_bytes))) return rc;
+      for (uint32_t j = 0; j < i && !L.cs; j++) {   // layers with the same rotation share its table
+        const lgh_layer_desc &a = L.d, &b = m.layers[j].d;
+        if (m.layers[j].latent() && a.rot_dims == b.rot_dims && a.rot_base == b.rot_base && a.yarn_factor == b.yarn_factor &&
+            a.yarn_original == b.yarn_original && a.yarn_fast == b.yarn_fast && a.yarn_slow == b.yarn_slow)
+          L.cs = m.layers[j].cs;
+      }
+      if (!L.cs) {
+        const std::vector<float> cs = rotation_table(L.d, d.max_seq_len);
+        if ((rc = zeroed(c, (void**)&L.cs, cs.size() * 4, &c->stats.scratch_bytes))) return rc;
+        L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
+        if (!cs.empty()) L_TRY(c, LGH_OPERATION_FAILED, hipMemcpy(L.cs, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
+      }
+      max_rows = std::max(max_rows, L.ls.heads); max_rank = std::max(max_rank, L.ls.rank); max_ldc = std::max(max_ldc, L.ls.ldc);
+    } else {
+      if ((rc = zeroed(c, (void**)&L.S, (size_t)L.ms.heads * L.ms.dim * L.ms.lds * 4, &c->stats.kv_bytes))) return rc;
+      if ((rc = zeroed(c, (void**)&L.m, (size_t)3 * L.ms.heads * 8, &c->stats.kv_bytes))) return rc;
+    }
+  }
+  uint32_t splits = (c->d.flags >> LGH_FLAG_ATTN_SPLITS_SHIFT) & 0xFFu;
+  if (!splits) splits = 256 / std::max(1u, (max_rows + 15) / 16);
+  m.n_splits = std::max(1u, std::min(splits, kLatMaxSplits));
+  // the absorbed path's rows: one token's heads in decode, several tokens' in short portions
+  const size_t rows = max_rows ? kLatAbsorbRows : 0;
+  uint64_t* sb = &c->stats.scratch_bytes;
+  struct { void** p; size_t n; } bufs[] = {
+      {(void**)&m.x[0], (size_t)d.width * 4}, {(void**)&m.x[1], (size_t)d.width * 4}, {(void**)&m.y, (size_t)up(d.width, 16) * 4},
+      {(void**)&m.cat, (size_t)m.max_cat * 4}, {(void**)&m.ao, (size_t)m.max_ao * 4}, {(void**)&m.act, (size_t)m.max_act * 4},
+      {(void**)&m.num, (size_t)m.max_num * 4}, {(void**)&m.qa, rows * max_ldc * m.el()},
+      {(void**)&m.part_ml, rows * m.n_splits * 2 * 4}, {(void**)&m.part_acc, rows * m.n_splits * max_rank * 4},
+      {(void**)&m.hist, (size_t)d.max_seq_len * 4}, {(void**)&c->logits, (size_t)d.vocab_size * 4}, {(void**)&c->state, ST_WORDS * 4},
+      {(void**)&c->amax_v, 64 * 4}, {(void**)&c->amax_i, 64 * 4}, {(void**)&c->tok_log, (size_t)d.max_seq_len * 4},
+  };
+  for (auto& b : bufs)
+    if ((rc = zeroed(c, b.p, b.n, sb))) return rc;
+  c->hidden = m.x[m.n_sub & 1];   // where the residual stream ends up: every sublayer's update swaps the two vectors
+  L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
+  return LGH_OK;
+}
+
+static EmbedArgs embed_args(const LayeredModel& m) {
+  EmbedArgs a{};
+  a.embed = m.embed; a.bigram = m.bigram; a.width = m.d.width; a.buckets = m.d.bigram_buckets;
+  a.mul_prev = m.d.bigram_mul_prev; a.mul_cur = m.d.bigram_mul_cur; a.hist = m.hist;
+  return a;
+}
+
+static LatentBufs latent_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat) {
+  LatentBufs b{};
+  b.cat = cat; b.dkv_norm = L.dkv_norm; b.cs = L.cs; b.uk_t = L.uk_t; b.uv = L.uv.w; b.cache = L.cache; b.qa = m.qa;
+  b.part_ml = m.part_ml; b.part_acc = m.part_acc;
+  return b;
+}
+static MlstmBufs mlstm_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat, float* num) {
+  MlstmBufs b{};
+  b.cat = cat; b.bi = L.bi; b.bf = L.bf; b.norm = L.mnorm; b.S = L.S; b.m = L.m; b.num = num;
+  b.u = m.bu; b.mx = m.bmx; b.a = m.ba; b.Mcap = m.blk;
+  return b;
+}
+
+// bytes of one token's attention / recurrence in a layer at the current position
+static uint64_t mixer_bytes(const lgh_ctx* c, const LayeredLayer& L) {
+  if (L.latent()) return (uint64_t)(c->pos + 1) * (L.ls.rank + L.ls.rot_dim) * c->lm->el();
+  return (uint64_t)L.ms.heads * L.ms.dim * (L.ms.vdim + 1) * 8;   // state read and written
+}
+
+int layered_enqueue_token(lgh_ctx* c, int mode) {
+  LayeredModel& m = *c->lm;
+  hipStream_t st = c->stream;
+  const int* pos = c->state + ST_POS;
+  int rc;
+  if ((rc = run_k(c, LGH_K_EMBED, LGH_SYM_EMBED, (uint64_t)m.d.width * 4, [&] { return layered_embed_launch(embed_args(m), c->state, m.x[0], st); }))) return rc;
+  uint32_t cur = 0;
+  const float* pend = nullptr;   // norm weight of the sublayer output waiting in m.y
+  auto mv = [&](int cls, const LinW& W, float* out, LinMv a, int pro) {
+    a.w = W.w; a.n = W.n; a.kp = W.kp; a.k = W.k; a.paired = W.paired; a.out = out;
+    return run_k(c, cls, LGH_SYM_LINEAR, W.bytes(), [&] { return lin_mv_launch(pro, a, st); });
+  };
+  auto mv_x = [&](int cls, const LinW& W, float* out, const float* nw2 = nullptr) -> int {   // a product that reads the residual stream
+    LinMv a{};
+    a.x = m.x[cur];
+    int pro = LP_COPY;
+    if (pend) {
+      a.y = m.y; a.nw = pend; a.nw2 = nw2; a.xout = m.x[cur ^ 1]; a.eps = (float)m.d.norm_eps; a.mult = (float)m.d.residual_mult;
+      pro = nw2 ? LP_HEAD : LP_RESID;
+      cur ^= 1;
+      pend = nullptr;
+    }
+    return mv(cls, W, out, a, pro);
+  };
+  for (LayeredLayer& L : m.layers) {
+    if ((rc = mv_x(LGH_K_QKV, L.in, m.cat))) return rc;
+    if (L.latent()) {
+      const LatentBufs b = latent_bufs(m, L, m.cat);
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, (uint64_t)L.ls.heads * L.ls.rank * L.ls.dim * 2, [&] { return latent_prep_launch(L.ls, b, pos, 0, 1, m.f32, st); }))) return rc;
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, mixer_bytes(c, L), [&] { return latent_attn_launch(L.ls, b, pos, 0, 1, m.n_splits, m.f32, st); }))) return rc;
+      if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_LATENT, L.uv.bytes(), [&] {
+             return latent_out_launch(L.ls, b, pos, 0, 1, m.n_splits, m.f32, m.ao, 0, true, st);
+           })))
+        return rc;
+      LinMv a{};
+      a.x = m.ao;
+      if ((rc = mv(LGH_K_WO, L.out, m.y, a, LP_COPY))) return rc;
+    } else {
+      const MlstmBufs b = mlstm_bufs(m, L, m.cat, m.num);
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_MLSTM, mixer_bytes(c, L), [&] { return mlstm_step_launch(L.ms, b, pos, st); }))) return rc;
+      LinMv a{};
+      a.num = m.num; a.nw = L.mnorm; a.gate = m.cat + L.ms.off_g; a.heads = L.ms.heads; a.vdim = L.ms.vdim; a.ldo = L.ms.ldo; a.eps = L.ms.eps;
+      if ((rc = mv(LGH_K_WO, L.out, m.y, a, LP_MLSTM))) return rc;
+    }
+    pend = L.norm1;
+    if (L.d.ff_kind) {
+      if ((rc = mv_x(LGH_K_GATEUP, L.gu, m.act))) return rc;
+      LinMv a{};
+      a.x = m.act;
+      if ((rc = mv(LGH_K_DOWN, L.down, m.y, a, LP_COPY))) return rc;
+      pend = L.norm2;
+    }
+  }
+  if (mode == MODE_PREFILL)
+    return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
+      return resid_norm_out_launch(m.x[cur], m.y, pend, (float)m.d.norm_eps, (float)m.d.residual_mult, m.d.width, m.x[cur ^ 1], st);
+    });
+  if ((rc = mv_x(LGH_K_OUTPUT, m.head, c->logits, m.final_norm))) return rc;
+  if (mode == MODE_GREEDY)
+    return run_k(c, LGH_K_ARGMAX, LGH_SYM_ARGMAX, (uint64_t)m.d.vocab_size * 4, [&] {
+      return argmax_launch(c->logits, m.d.vocab_size, c->amax_v, c->amax_i, c->state, c->tok_log, st);
+    });
+  return LGH_OK;
+}
+
+uint64_t layered_step_bytes(const lgh_ctx* c) {
+  const LayeredModel& m = *c->lm;
+  uint64_t b = (uint64_t)m.d.width * (m.bigram ? 4 : 2) + m.head.bytes() + (uint64_t)m.d.vocab_size * 4 + m.d.width * 4;
+  for (const LayeredLayer& L : m.layers) {
+    b += L.in.bytes() + L.out.bytes() + mixer_bytes(c, L) + (uint64_t)m.d.width * 4;
+    if (L.latent()) b += L.uk.bytes() + L.uv.bytes();
+    if (L.d.ff_kind) b += L.gu.bytes() + L.down.bytes() + (uint64_t)m.d.width * 4;
+  }
+  return b;
+}
+
+// ------------------------------------------------------------------------------------------------
+// blocks of tokens
+// ------------------------------------------------------------------------------------------------
+static int block_ensure(lgh_ctx* c) {
+  LayeredModel& m = *c->lm;
+  if (m.blk_ready) return LGH_OK;
+  const lgh_layered_desc& d = m.d;
+  m.blk = std::min(kBlockTokens, d.max_seq_len);
+  uint32_t heads = 0;
+  for (auto& L : m.layers)
+    if (!L.latent()) heads = std::max(heads, L.ms.heads);
+  const size_t B = m.blk, chunks = (B + 63) / 64, el = m.el();
+  struct { void** p; size_t n; } bufs[] = {
+      {(void**)&m.bx, B * d.width * 4}, {&m.bxa, B * up(d.width, 64) * el}, {(void**)&m.by, B * up(d.width, 4) * 4},
+      {(void**)&m.bcat, B * m.max_cat * 4}, {&m.bao, B * m.max_ao * el}, {&m.bact, B * m.max_act * el},
+      {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * B * 8}, {(void**)&m.bmx, heads * B * 8},
+      {(void**)&m.btok, B * 4}, {(void**)&m.brows, B * 4}, {&m.bla, (size_t)kLogitRows * up(d.width, 64) * el},
+      {(void**)&m.blogits, (size_t)kLogitRows * up(d.vocab_size, 4) * 4},
+  };
+  int rc;
+  for (auto& b : bufs)
+    if ((rc = zeroed(c, b.p, b.n, &c->stats.scratch_bytes))) return rc;
+  L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
+  m.blk_ready = true;
+  return LGH_OK;
+}
+
+static int block_gemm(lgh_ctx* c, int cls, const LinW& W, int epi, const void* x, uint32_t ldx, void* out, uint32_t ldo, uint32_t M) {
+  LinGemm g{};
+  g.w = W.w; g.x = x; g.out = out; g.n = W.n; g.np = W.np(); g.kp = W.kp; g.ldx = ldx; g.ldo = ldo; g.M = M;
+  return run_k(c, cls, LGH_SYM_LINEAR, W.bytes(), [&] { return lin_gemm_launch(epi, c->lm->f32, g, c->stream); });
+}
+
+static int block_latent(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) {
+  LayeredModel& m = *c->lm;
+  hipStream_t st = c->stream;
+  int rc;
+  // absorbed, as many tokens at a time as their (token, head) rows fit the buffers
+  const uint32_t step = std::max(1u, kLatAbsorbRows / L.ls.heads);
+  for (uint32_t t = 0; t < M; t += step) {
+    const uint32_t n = std::min(step, M - t), p = pos0 + t;
+    const uint32_t splits = std::max(1u, std::min(m.n_splits, 512u / ((n * L.ls.heads + 15) / 16)));
+    const LatentBufs b = latent_bufs(m, L, m.bcat + (size_t)t * L.ls.ldcat);
+    if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, 0, [&] { return latent_prep_launch(L.ls, b, nullptr, p, n, m.f32, st); }))) return rc;
+    if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, 0, [&] { return latent_attn_launch(L.ls, b, nullptr, p, n, splits, m.f32, st); }))) return rc;
+    if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_LATENT, 0, [&] {
+           return latent_out_launch(L.ls, b, nullptr, p, n, splits, m.f32, (uint8_t*)m.bao + (size_t)t * L.out.kp * m.el(), L.out.kp, m.f32, st);
+         })))
+      return rc;
+  }
+  return LGH_OK;
+}
+
+static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint32_t* want, uint32_t n_want, float* logits_out) {
+  LayeredModel& m = *c->lm;
+  const lgh_layered_desc& d = m.d;
+  hipStream_t st = c->stream;
+  const uint32_t pos0 = (uint32_t)c->pos, ldx = up(d.width, 64), ldy = up(d.width, 4);
+  const float eps = (float)d.norm_eps, mult = (float)d.residual_mult;
+  int rc;
+  L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(m.btok, tokens, (size_t)M * 4, hipMemcpyHostToDevice, st));
+  if ((rc = run_k(c, LGH_K_EMBED, LGH_SYM_EMBED, (uint64_t)M * d.width * 4, [&] {
+         return layered_embed_block_launch(embed_args(m), m.btok, pos0, M, m.bx, m.bxa, ldx, m.f32, st);
+       })))
+    return rc;
+  auto resid = [&](const float* nw) {
+    return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, (uint64_t)M * d.width * 14, [&] {
+      return resid_norm_launch(m.bx, m.by, ldy, nw, eps, mult, d.width, M, m.bxa, ldx, m.f32, st);
+    });
+  };
+  for (uint32_t li = 0; li < d.num_layers; li++) {
+    LayeredLayer& L = m.layers[li];
+    if ((rc = block_gemm(c, LGH_K_QKV, L.in, LE_F32, m.bxa, ldx, m.bcat, L.in.n, M))) return rc;
+    if (L.latent()) {
+      if ((rc = block_latent(c, L, pos0, M))) return rc;
+    } else {
+      const MlstmBufs b = mlstm_bufs(m, L, m.bcat, m.bnum);
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_MLSTM, 0, [&] { return mlstm_block_launch(L.ms, b, pos0, M, st); }))) return rc;
+      if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_MLSTM, 0, [&] { return mlstm_out_launch(L.ms, b, M, m.bao, L.out.kp, m.f32, st); }))) return rc;
+    }
+    if ((rc = block_gemm(c, LGH_K_WO, L.out, LE_F32, m.bao, L.out.kp, m.by, ldy, M))) return rc;
+    if ((rc = resid(L.norm1))) return rc;
+    if (L.d.ff_kind) {
+      if ((rc = block_gemm(c, LGH_K_GATEUP, L.gu, LE_GEGLU, m.bxa, ldx, m.bact, L.down.kp, M))) return rc;
+      if ((rc = block_gemm(c, LGH_K_DOWN, L.down, LE_F32, m.bact, L.down.kp, m.by, ldy, M))) return rc;
+      if ((rc = resid(L.norm2))) return rc;
+    }
+    if (m.tap && m.tap_tokens == M)
+      L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(m.tap_buf + (size_t)li * M * d.width, m.bx, (size_t)M * d.width * 4, hipMemcpyDeviceToDevice, st));
+  }
+  L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(c->hidden, m.bx + (size_t)(M - 1) * d.width, (size_t)d.width * 4, hipMemcpyDeviceToDevice, st));
+  const uint32_t ldl = up(d.vocab_size, 4);
+  for (uint32_t w = 0; w < n_want; w += kLogitRows) {
+    const uint32_t n = std::min(kLogitRows, n_want - w);
+    L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(m.brows, want + w, (size_t)n * 4, hipMemcpyHostToDevice, st));
+    if ((rc = run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] { return final_norm_rows_launch(m.bx, m.brows, n, m.final_norm, eps, d.width, m.bla, ldx, m.f32, st); })))
+      return rc;
+    if ((rc = block_gemm(c, LGH_K_OUTPUT, m.head, LE_F32, m.bla, ldx, m.blogits, ldl, n))) return rc;
+    L_TRY(c, LGH_OPERATION_FAILED, hipMemcpy2DAsync(logits_out + (size_t)w * d.vocab_size, (size_t)d.vocab_size * 4, m.blogits, (size_t)ldl * 4,
+                                                    (size_t)d.vocab_size * 4, n, hipMemcpyDeviceToHost, st));
+    L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(st));
+  }
+  c->pos += M;
+  c->stats.tokens_processed += M;
+  L_TRY(c, LGH_OPERATION_FAILED, hipMemsetD32Async((hipDeviceptr_t)(c->state + ST_NEXT), (int)c->pos, 1, st));
+  L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(st));   // the caller's tokens / want are free again
+  return c->profiling ? drain_prof(c) : LGH_OK;
+}
+
+int layered_block(lgh_ctx* c, const uint32_t* tokens, size_t n, const uint32_t* want, size_t n_want, float* logits_out) {
+  LayeredModel& m = *c->lm;
+  int rc = block_ensure(c);
+  if (rc) return rc;
+  if (m.tap) {
+    m.tap_tokens = 0;
+    if (m.tap_buf) dev_free_tracked(c, m.tap_buf);
+    m.tap_buf = nullptr;
+    if (n <= m.blk) {
+      if ((rc = dev_alloc(c, (void**)&m.tap_buf, (size_t)m.d.num_layers * n * m.d.width * 4))) return rc;
+      m.tap_tokens = (uint32_t)n;
+    }
+  }
+  size_t w = 0;
+  std::vector<uint32_t> local;
+  for (size_t t = 0; t < n; t += m.blk) {
+    const uint32_t M = (uint32_t)std::min<size_t>(m.blk, n - t);
+    local.clear();
+    const size_t w0 = w;
+    while (w < n_want && want[w] < t + M) local.push_back((uint32_t)(want[w++] - t));
+    if ((rc = block_pass(c, tokens + t, M, local.data(), (uint32_t)local.size(), logits_out ? logits_out + w0 * m.d.vocab_size : nullptr))) return rc;
+  }
+  return LGH_OK;
+}
+
+extern "C" int lgh_set_layer_tap(lgh_ctx* c, int on) {
+  if (!c) return LGH_INVALID_ARGUMENT;
+  if (!c->lm) return fail(c, LGH_UNSUPPORTED, "only models described layer by layer have a layer tap");
+  c->lm->tap = on != 0;
+  c->lm->tap_tokens = 0;
+  return LGH_OK;
+}
+
+extern "C" int lgh_read_layers(lgh_ctx* c, float* out, size_t n_floats) {
+  if (!c || !out) return LGH_INVALID_ARGUMENT;
+  if (!c->lm || !c->lm->tap_tokens) return fail(c, LGH_INVALID_ARGUMENT, "no portion was run with the layer tap on");
+  const size_t n = (size_t)c->lm->d.num_layers * c->lm->tap_tokens * c->lm->d.width;
+  if (n_floats != n) return fail(c, LGH_SHAPE_MISMATCH, "expected " + std::to_string(n) + " floats");
+  if (hipSetDevice(c->device) != hipSuccess) return fail(c, LGH_NOT_AVAILABLE, "hipSetDevice failed");
+  L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(out, c->lm->tap_buf, n * 4, hipMemcpyDeviceToHost, c->stream));
+  L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
+  return LGH_OK;
+}

@@ -326,15 +326,4 @@ hipError_t lin_transpose_heads_launch(const uint16_t* src, uint32_t heads, uint3
   return hipGetLastError();
 }
 
-__global__ void __launch_bounds__(256) bf16_to_f32_kernel(const uint16_t* __restrict__ src, float* __restrict__ dst, uint64_t n) {
-  for (uint64_t i = (uint64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (uint64_t)gridDim.x * 256) dst[i] = bf_f(src[i]);
-}
-
-hipError_t bf16_to_f32_launch(const uint16_t* src, float* dst, uint64_t n, hipStream_t st) {
-  uint64_t blocks = (n + 255) / 256;
-  if (blocks > 4096) blocks = 4096;
-  if (blocks) hipLaunchKernelGGL(bf16_to_f32_kernel, dim3((uint32_t)blocks), dim3(256), 0, st, src, dst, n);
-  return hipGetLastError();
-}
-
 }  // namespace lgh

@@ -36,6 +36,7 @@ ABI_SYMBOLS = (
     "lgh_pipeline_prefill_token", "lgh_pipeline_decode_greedy", "lgh_pipeline_reset", "lgh_pipeline_position", "lgh_pipeline_kv_truncate", "lgh_pipeline_stages",
     "lgh_pipeline_last_error",
     "lgh_set_kv_rotation_signs", "lgh_op_tq_compress", "lgh_set_kv_qjl_matrices", "lgh_op_tq_compress_qjl",
+    "lgh_eval", "lgh_create_layered", "lgh_set_layer_tap", "lgh_read_layers",
     "lgh_batch_create", "lgh_batch_reset", "lgh_batch_position", "lgh_batch_prefill", "lgh_forward_multi", "lgh_decode_greedy_multi",
 )
 
@@ -47,7 +48,7 @@ SYM_NAMES = ("lgh::mv_kernel<1u, 1024>", "lgh::mv_kernel<8u, 1024>", "lgh::mv_ke
              "lgh::mv_kernel<2u, 768>", "lgh::mv_kernel<4u, 512>", "lgh::mv_kernel<5u, 512>", "lgh::mv_kernel<6u, 512>",
              "lgh::mv_kernel<31u, 512>", "lgh::f32_matvec_kernel", "lgh::attn_partial_kernel", "lgh::attn_combine_kernel",
              "lgh::embed_kernel", "lgh::argmax_stage1+2", "lgh::moe_router_kernel", "other", "lgh::mvq_kernel<1u>", "lgh::mvq_kernel<2u>", "lgh::mvq_kernel<3u>", "lgh::mvq_kernel<4u>",
-             "lgh::mvq_kernel<8u>", "unused")
+             "lgh::mvq_kernel<8u>", "unused", "lgh::lin_mv / lin_gemm", "lgh::latent_*", "lgh::mlstm_*")
 FLAG_NO_GRAPH = 1
 FLAG_EXACT_PREFILL = 4   # forward_batch feeds tokens one by one (f32 throughout) instead of the batched f16 GEMM path
 KV_F32, KV_INT8, KV_FP8_E4M3, KV_FP8_E5M2 = 0, 1, 2, 3   # lgh_model_desc.kv_cache_type: f32, or QuantizedKVCache's formats (kv_quantized.rs; no CLI flag reaches them)
@@ -77,6 +78,24 @@ class ModelDesc(C.Structure):
                 + [(n, C.c_float) for n in ("norm_eps", "rope_freq_base", "rope_freq_scale")]
                 + [("device_id", C.c_int32), ("layer_begin", C.c_uint32), ("layer_end", C.c_uint32),
                    ("flags", C.c_uint32), ("kv_cache_type", C.c_uint32)])
+
+
+class LayerDesc(C.Structure):
+    """lgh_layer_desc: one layer of a model described layer by layer."""
+    _fields_ = ([(n, C.c_uint32) for n in ("struct_size", "mixer", "heads", "dim", "vdim", "kv_rank", "rot_dim", "rot_dims", "ff_kind", "ff")]
+                + [(n, C.c_double) for n in ("scale", "rot_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow", "gate_cap")])
+
+
+class LayeredDesc(C.Structure):
+    """lgh_layered_desc."""
+    _fields_ = ([(n, C.c_uint32) for n in ("struct_size", "width", "vocab_size", "num_layers", "max_seq_len", "compute")]
+                + [("device_id", C.c_int32), ("flags", C.c_uint32), ("bigram_buckets", C.c_uint32), ("bigram_mul_prev", C.c_uint64),
+                   ("bigram_mul_cur", C.c_uint64), ("norm_eps", C.c_double), ("residual_mult", C.c_double)])
+
+
+MIXER_LATENT_ATTENTION, MIXER_MLSTM = 1, 2      # LGH_MIXER_*
+FF_NONE, FF_GEGLU = 0, 1                        # LGH_FF_*
+COMPUTE_BF16, COMPUTE_F32 = 0, 1                # LGH_COMPUTE_*
 
 
 class GgufInfo(C.Structure):
@@ -162,6 +181,9 @@ def load_library() -> C.CDLL:
         "lgh_pipeline_position": (sz, [vp]), "lgh_pipeline_kv_truncate": (C.c_int, [vp, sz]), "lgh_pipeline_stages": (C.c_int, [vp]), "lgh_pipeline_last_error": (C.c_char_p, [vp]),
         "lgh_set_kv_rotation_signs": (C.c_int, [vp, vp, sz]), "lgh_op_tq_compress": (C.c_int, [C.c_int, C.c_int, vp, sz, vp, vp]),
         "lgh_set_kv_qjl_matrices": (C.c_int, [vp, vp, sz]), "lgh_op_tq_compress_qjl": (C.c_int, [C.c_int, C.c_int, vp, sz, vp, vp, vp, vp, vp]),
+        "lgh_eval": (C.c_int, [vp, vp, sz, vp, sz, vp]),
+        "lgh_create_layered": (C.c_int, [C.POINTER(LayeredDesc), C.POINTER(LayerDesc), C.POINTER(vp)]),
+        "lgh_set_layer_tap": (C.c_int, [vp, C.c_int]), "lgh_read_layers": (C.c_int, [vp, vp, sz]),
         "lgh_batch_create": (C.c_int, [vp, u32]), "lgh_batch_reset": (C.c_int, [vp, u32]), "lgh_batch_position": (sz, [vp, u32]),
         "lgh_batch_prefill": (C.c_int, [vp, u32, vp, sz]), "lgh_forward_multi": (C.c_int, [vp, vp, vp, u32, vp, vp]),
         "lgh_decode_greedy_multi": (C.c_int, [vp, vp, vp, u32, sz, vp]),
@@ -236,6 +258,26 @@ class HipGpuInference:
         return self
 
     @classmethod
+    def from_layered(cls, model, max_seq_len: int, device: int = 0, compute: int = COMPUTE_BF16, flags: int = 0, attn_splits: int = 0) -> "HipGpuInference":
+        """A model described layer by layer (layered_model.LayeredModel): `.config` with `.desc()` / `.layer_descs()` and
+        `.tensors()` yielding (name, ggml_type, ne, host bytes)."""
+        L = load_library()
+        self = cls()
+        cfg = model.config
+        d = cfg.desc()
+        d.max_seq_len, d.device_id, d.compute, d.flags = int(max_seq_len), device, compute, flags | ((attn_splits & 0xFF) << 8)
+        _chk(L.lgh_create_layered(C.byref(d), cfg.layer_descs(), C.byref(self._h)), "lgh_create_layered (sizes supported? a HIP device visible?)")
+        self.config, self.vocab_size, self.hidden_size = cfg, cfg.vocab_size, cfg.hidden_size
+        try:
+            for name, t, ne, data in model.tensors():
+                self.upload_tensor(name, t, ne, data)
+            self._call(L.lgh_finalize(self._h))
+        except Exception:
+            self.close()
+            raise
+        return self
+
+    @classmethod
     def from_gguf(cls, path: str, max_seq_len: int = 0, device: int = 0, layer_range: Optional[Sequence[int]] = None,
                   flags: int = 0) -> "HipGpuInference":
         """GGUF -> HBM direct load (lgh_load_gguf): header parsed and tensors uploaded by the library itself."""
@@ -274,6 +316,22 @@ class HipGpuInference:
     def forward_batch(self, tokens: Sequence[int]) -> None:  # gpu_only.rs:776-790 minus the final forward
         toks = np.ascontiguousarray(tokens, dtype=np.uint32)
         self._call(load_library().lgh_prefill_batch(self._h, toks.ctypes.data, toks.size))
+
+    def eval(self, tokens: Sequence[int], want: Sequence[int] = ()) -> np.ndarray:
+        """A portion of the sequence: the logits after its places `want` (ascending), [len(want), vocab]."""
+        toks, w = np.ascontiguousarray(tokens, dtype=np.uint32), np.ascontiguousarray(want, dtype=np.uint32)
+        out = np.empty((w.size, self.vocab_size), dtype=np.float32)
+        self._call(load_library().lgh_eval(self._h, toks.ctypes.data, toks.size, w.ctypes.data, w.size, out.ctypes.data))
+        return out
+
+    def set_layer_tap(self, on: bool) -> None:
+        self._call(load_library().lgh_set_layer_tap(self._h, int(on)))
+
+    def read_layers(self, n_tokens: int) -> np.ndarray:
+        """Residual stream after every layer of the last eval portion, [layers, n_tokens, width]."""
+        out = np.empty((self.config.num_layers, n_tokens, self.hidden_size), dtype=np.float32)
+        self._call(load_library().lgh_read_layers(self._h, out.ctypes.data, out.size))
+        return out
 
     def prefill_is_batched(self) -> bool:
         return bool(load_library().lgh_prefill_is_batched(self._h))

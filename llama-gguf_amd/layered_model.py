@@ -1,0 +1,217 @@
+"""Models described layer by layer: the registry of architectures, config.json, safetensors weights.
+
+A model folder holds ``config.json`` (its ``architecture`` picks the parser here) and ``model.safetensors``.  A parser turns the
+configuration into ``LayeredConfig``; every layer is a mixer (``MIXERS``) and an optional feed-forward (``FEED_FORWARDS``), each read
+by a function of its own, so another architecture made of the same parts adds one entry.  The engine takes the result through
+``HipGpuInference.from_layered``; nothing here computes.
+"""
+from __future__ import annotations
+
+import json
+import os
+from dataclasses import dataclass, field
+from typing import Iterator, List, Optional, Tuple
+
+import numpy as np
+
+from . import hip_backend as hb
+
+BF16, F32 = 30, 0        # ggml type ids
+_SAFETENSORS_TYPES = {"BF16": (BF16, 2), "F32": (F32, 4)}
+
+
+class ConfigError(ValueError):
+    """config.json asks for something no part of the engine computes, or lacks a value."""
+
+
+def _need(d: dict, key: str, where: str):
+    if not isinstance(d, dict) or key not in d:
+        raise ConfigError(f"{where}: '{key}' is missing")
+    return d[key]
+
+
+def _sizes(layer: hb.LayerDesc, mixer: dict, where: str, **fields) -> None:
+    for name, key in fields.items():
+        setattr(layer, name, int(_need(mixer, key, where)))
+
+
+def _latent_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_LATENT_ATTENTION
+    _sizes(layer, mx, where, heads="heads", dim="dim", vdim="vdim", kv_rank="kv_rank", rot_dim="rot_dim")
+    layer.scale = float(_need(mx, "scale", where))
+    rot = mx.get("rot")
+    if not rot:
+        return                                     # nothing is rotated
+    layer.rot_dims, layer.rot_base = int(_need(rot, "dims", where)), float(_need(rot, "base", where))
+    sc = rot.get("scaling")
+    if sc:
+        for f in ("factor", "original", "fast", "slow"):
+            setattr(layer, "yarn_" + f, float(_need(sc, f, where)))
+
+
+def _mlstm(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_MLSTM
+    _sizes(layer, mx, where, heads="heads", dim="dim", vdim="vdim")
+    layer.gate_cap = float(_need(mx, "gate_cap", where))
+
+
+def _dense(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
+    layer.ff_kind, layer.ff = hb.FF_GEGLU, int(_need(mlp, "ff", where))
+
+
+MIXERS = {"latent_attention": _latent_attention, "mlstm": _mlstm}
+FEED_FORWARDS = {"dense": _dense}
+
+
+@dataclass
+class LayeredConfig:
+    name: str
+    hidden_size: int
+    vocab_size: int
+    norm_eps: float
+    residual_mult: float
+    layers: List[hb.LayerDesc] = field(default_factory=list)
+    bigram: Optional[Tuple[int, int, int]] = None      # buckets, factor of the previous token, factor of the token
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def desc(self) -> hb.LayeredDesc:
+        d = hb.LayeredDesc()
+        d.struct_size = hb.C.sizeof(hb.LayeredDesc)
+        d.width, d.vocab_size, d.num_layers = self.hidden_size, self.vocab_size, self.num_layers
+        d.norm_eps, d.residual_mult = self.norm_eps, self.residual_mult
+        if self.bigram:
+            d.bigram_buckets, d.bigram_mul_prev, d.bigram_mul_cur = self.bigram
+        return d
+
+    def layer_descs(self):
+        return (hb.LayerDesc * self.num_layers)(*self.layers)
+
+    def tensor_shapes(self) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        """(name, shape) of every tensor the model needs, [out, in]."""
+        W = self.hidden_size
+        yield "embed", (self.vocab_size, W)
+        if self.bigram:
+            yield "bigram", (self.bigram[0] + 1, W)
+        for i, l in enumerate(self.layers):
+            p, vd = f"l{i}.", l.heads * l.vdim
+            yield p + "norm1", (W,)
+            if l.mixer == hb.MIXER_LATENT_ATTENTION:
+                yield p + "mix.q", (l.heads * (l.dim + l.rot_dim), W)
+                yield p + "mix.dkv", (l.kv_rank + l.rot_dim, W)
+                yield p + "mix.dkv.norm", (l.kv_rank,)
+                yield p + "mix.uk", (l.heads * l.dim, l.kv_rank)
+                yield p + "mix.uv", (vd, l.kv_rank)
+                yield p + "mix.g", (l.heads, W)
+            else:
+                yield p + "mix.q", (l.heads * l.dim, W)
+                yield p + "mix.k", (l.heads * l.dim, W)
+                yield p + "mix.v", (vd, W)
+                yield p + "mix.g", (vd, W)
+                yield p + "mix.norm", (vd,)
+                for g in ("i", "f"):
+                    yield p + "mix." + g, (l.heads, W)
+                    yield p + "mix." + g + ".b", (l.heads,)
+            yield p + "mix.o", (W, vd)
+            if l.ff_kind:
+                yield p + "norm2", (W,)
+                yield p + "mlp.gate", (l.ff, W)
+                yield p + "mlp.up", (l.ff, W)
+                yield p + "mlp.down", (W, l.ff)
+        yield "final.norm", (W,)
+        yield "head", (self.vocab_size, W)
+
+
+def _zamelix(cfg: dict) -> LayeredConfig:
+    """Latent attention and matrix-memory layers in any order, gated feed-forwards, layer norm on every sublayer's output, a hashed
+    pair embedding."""
+    where = "Zamelix"
+    out = LayeredConfig(where, int(_need(cfg, "width", where)), int(_need(cfg, "vocab", where)),
+                        float(_need(_need(cfg, "norm", where), "eps", where)), float(_need(cfg, "residual_mult", where)))
+    big = (cfg.get("embedding") or {}).get("bigram")
+    if big:
+        out.bigram = tuple(int(_need(big, k, where)) for k in ("buckets", "mul_prev", "mul_cur"))
+    for i, entry in enumerate(_need(cfg, "layers", where)):
+        at = f"{where} layer {i}"
+        layer = hb.LayerDesc()
+        layer.struct_size = hb.C.sizeof(hb.LayerDesc)
+        kind = _need(entry, "type", at)
+        if kind not in MIXERS:
+            raise ConfigError(f"{at}: unknown mixer '{kind}'")
+        MIXERS[kind](layer, _need(entry, "mixer", at), at)
+        mlp = entry.get("mlp")
+        if mlp:
+            if _need(mlp, "kind", at) not in FEED_FORWARDS:
+                raise ConfigError(f"{at}: unknown feed-forward '{mlp['kind']}'")
+            FEED_FORWARDS[mlp["kind"]](layer, mlp, at)
+        out.layers.append(layer)
+    return out
+
+
+ARCHITECTURES = {"Zamelix": _zamelix}      # config.json "architecture" -> parser
+
+
+def parse_config(cfg: dict) -> LayeredConfig:
+    arch = _need(cfg, "architecture", "config.json")
+    if arch not in ARCHITECTURES:
+        raise ConfigError(f"config.json: unknown architecture '{arch}' (known: {', '.join(sorted(ARCHITECTURES))})")
+    return ARCHITECTURES[arch](cfg)
+
+
+class SafetensorsFile:
+    """The tensors of a .safetensors file, mapped: an 8-byte little-endian header length, a JSON header, then the data."""
+
+    def __init__(self, path: str):
+        size = os.path.getsize(path)
+        with open(path, "rb") as f:
+            n = int.from_bytes(f.read(8), "little")
+            if n > size - 8:
+                raise ConfigError(f"{path}: header longer than the file")
+            self.header = json.loads(f.read(n))
+        self.header.pop("__metadata__", None)
+        self._data = np.memmap(path, dtype=np.uint8, mode="r", offset=8 + n) if size > 8 + n else np.zeros(0, np.uint8)
+
+    def get(self, name: str, shape: Tuple[int, ...]) -> Tuple[int, np.ndarray]:
+        """(ggml type, bytes) of a tensor, checked against the shape the model needs."""
+        h = self.header.get(name)
+        if h is None:
+            raise ConfigError(f"tensor '{name}' is missing")
+        if h["dtype"] not in _SAFETENSORS_TYPES:
+            raise ConfigError(f"tensor '{name}': type {h['dtype']} is not supported")
+        t, el = _SAFETENSORS_TYPES[h["dtype"]]
+        a, b = h["data_offsets"]
+        if tuple(h["shape"]) != tuple(shape) or b - a != el * int(np.prod(shape)) or a < 0 or b > self._data.size:
+            raise ConfigError(f"tensor '{name}': shape {h['shape']}, expected {list(shape)}")
+        return t, self._data[a:b]
+
+
+class LayeredModel:
+    """A configuration with its weights; `tensors()` is what `HipGpuInference.from_layered` uploads."""
+
+    def __init__(self, config: LayeredConfig, source):
+        self.config, self._source = config, source       # source.get(name, shape) -> (ggml type, bytes)
+
+    @classmethod
+    def from_dir(cls, path: str) -> "LayeredModel":
+        with open(os.path.join(path, "config.json")) as f:
+            cfg = parse_config(json.load(f))
+        return cls(cfg, SafetensorsFile(os.path.join(path, "model.safetensors")))
+
+    def tensors(self):
+        for name, shape in self.config.tensor_shapes():
+            t, data = self._source.get(name, shape)
+            yield name, t, tuple(reversed(shape)), data
+
+    def weight_bytes(self) -> int:
+        return sum(2 * int(np.prod(s)) for _, s in self.config.tensor_shapes())
+
+
+def load_model(path: str, max_seq_len: int, device: int = 0, compute: int = hb.COMPUTE_BF16, flags: int = 0) -> hb.HipGpuInference:
+    """A model folder (config.json + model.safetensors) or a .gguf file -> a ready context."""
+    if os.path.isdir(path):
+        return hb.HipGpuInference.from_layered(LayeredModel.from_dir(path), max_seq_len, device, compute, flags)
+    if compute == hb.COMPUTE_F32:
+        raise hb.BackendError(5, "GGUF models run with quantized weights and f32 activations; there is no separate 32-bit mode")
+    return hb.HipGpuInference.from_gguf(path, max_seq_len, device, flags=flags)
