@@ -122,7 +122,114 @@ def parse_args():
     ap.add_argument("--stages", type=int, default=0, help="with --inlib: stage count when it differs from --gpus (several stages on one GPU)")
     ap.add_argument("--fake-stage", action="store_true",
                     help="CPU rehearsal of the N>1 launcher and hop protocol: gloo + pipeline.FakeStage, no GPU, no engine (not a measurement)")
+    ap.add_argument("--layered", default="", metavar="SIZE[,SIZE]",
+                    help="models described layer by layer (latent attention + matrix memory) beside the Llama-style model of equal width, depth and "
+                         "feed-forward, random weights: " + ", ".join(LAYERED_SIZES) + " or all; not the headline metric")
+    ap.add_argument("--layered-only", choices=("both", "layered", "closest"), default="both", help="with --layered: run one side (for a profiler)")
+    ap.add_argument("--layered-context", type=int, default=2048, help="with --layered: prompt length")
     return ap.parse_args()
+
+
+# Layer sizes of real models: TinyLlama's, Llama-3-8B's and -70B's width / feed-forward, few layers (every second one a matrix memory without a
+# feed-forward), attention and memory sizes as published models of those widths use them.
+LAYERED_SIZES = {
+    "w2048": dict(width=2048, ff=5632, vocab=32000, layers=8, heads=16, dim=128, rot=64, vdim=128, rank=512, mheads=4, mdim=256, mvdim=512,
+                  closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),
+    "w4096": dict(width=4096, ff=14336, vocab=128256, layers=8, heads=32, dim=128, rot=64, vdim=128, rank=512, mheads=8, mdim=256, mvdim=512,
+                  closest=dict(num_heads=32, num_kv_heads=8, head_dim=128)),
+    "w8192": dict(width=8192, ff=28672, vocab=128256, layers=4, heads=64, dim=128, rot=64, vdim=128, rank=512, mheads=8, mdim=512, mvdim=1024,
+                  closest=dict(num_heads=64, num_kv_heads=8, head_dim=128)),
+}
+
+
+class RandomBf16:
+    """Random weights for a layered model: slices of one random block, scaled by 1 / sqrt(in); norm weights 1."""
+
+    def __init__(self, seed=1):
+        self.block = np.random.default_rng(seed).standard_normal(1 << 22, dtype=np.float32)
+
+    def get(self, name, shape):
+        n = int(np.prod(shape))
+        if len(shape) == 1:
+            v = np.ones(n, np.float32) if name.endswith("norm") or "norm" in name.rsplit(".", 1)[-1] else np.zeros(n, np.float32)
+            return 0, v
+        blk = ((self.block * np.float32(1.0 / np.sqrt(shape[1]))).view(np.uint32) >> 16).astype(np.uint16)
+        return 30, np.resize(np.roll(blk, len(name) * 7919), n)
+
+
+def layered_config(sz):
+    attn = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": sz["ff"]},
+            "mixer": {"heads": sz["heads"], "dim": sz["dim"], "rot_dim": sz["rot"], "vdim": sz["vdim"], "kv_rank": sz["rank"],
+                      "scale": (sz["dim"] + sz["rot"]) ** -0.5, "rot": {"base": 10000.0, "dims": sz["rot"]}}}
+    mem = {"type": "mlstm", "mlp": None, "mixer": {"heads": sz["mheads"], "dim": sz["mdim"], "vdim": sz["mvdim"], "gate_cap": 15.0}}
+    return {"architecture": "Zamelix", "width": sz["width"], "vocab": sz["vocab"], "norm": {"eps": 1e-5}, "residual_mult": 0.5,
+            "embedding": {"bigram": {"buckets": 4096, "mul_prev": 31, "mul_cur": 7}},
+            "layers": [mem if i % 2 else attn for i in range(sz["layers"])]}
+
+
+def layered_measure(eng, prompt, steps, reps):
+    """Prompt pass and greedy decode of one context: seconds per prompt, seconds per token, and the eager per-class pass."""
+    eng.forward_batch(prompt)
+    pre, dec = [], []
+    for _ in range(reps):
+        eng.reset()
+        eng.synchronize()
+        t0 = time.perf_counter()
+        eng.forward_batch(prompt)
+        eng.synchronize()
+        pre.append(time.perf_counter() - t0)
+        eng.decode_greedy(1, 4)
+        t0 = time.perf_counter()
+        eng.decode_greedy(1, steps)
+        dec.append((time.perf_counter() - t0) / steps)
+    out = {"prefill_tokens_per_s": round(len(prompt) / min(pre), 1), "prefill_ms": round(1e3 * min(pre), 3),
+           "decode_tokens_per_s": round(1.0 / min(dec), 1), "decode_us": round(1e6 * min(dec), 1)}
+    st = eng.stats()
+    out["decode_alg_bytes"] = st["step_alg_bytes"]
+    out["decode_frac_of_hbm_peak"] = round(st["step_alg_bytes"] / min(dec) / 1e9 / HBM_PEAK_GBPS, 3)
+    eng.set_profiling(True)
+    for t in range(4):
+        eng.forward_argmax(1)
+    st = eng.stats()
+    br = st["event_bracket_us"]
+    out["decode_kernels_us"] = {k: {"launches": v["launches"] / 4, "us_with_event_bracket": round(v["time_us"] / 4, 1),
+                                    "GBps": round(v["alg_bytes"] / max(v["time_us"] - br * v["launches"], 1e-3) / 1e3, 1)} for k, v in st["kernels"].items()}
+    eng.set_profiling(True)
+    eng.reset()
+    eng.forward_batch(prompt)
+    out["prefill_kernels_us"] = {k: {"launches": v["launches"], "us_with_event_bracket": round(v["time_us"], 1)} for k, v in eng.stats()["kernels"].items()}
+    eng.set_profiling(False)
+    return out
+
+
+def run_layered(args, pkg):
+    """`--layered`: prefill and decode throughput beside the Llama-style model of equal width, depth and feed-forward (Q8_0: the engine's widest
+    fused weight format)."""
+    names = list(LAYERED_SIZES) if args.layered == "all" else args.layered.split(",")
+    res, steps, n = {}, min(args.steps, 64), args.layered_context
+    for name in names:
+        sz, r = LAYERED_SIZES[name], {}
+        prompt = prompt_tokens(n, sz["vocab"])
+        cap = n + steps * (args.reps + 1) + 64
+        if args.layered_only != "closest":
+            cfg = pkg.layered_model.parse_config(layered_config(sz))
+            eng = pkg.HipGpuInference.from_layered(pkg.LayeredModel(cfg, RandomBf16()), cap)
+            r["layered"] = layered_measure(eng, prompt, steps, args.reps)
+            eng.close()
+        if args.layered_only != "layered":
+            c = pkg.ModelConfig(name="closest", hidden_size=sz["width"], intermediate_size=sz["ff"], num_layers=sz["layers"], vocab_size=sz["vocab"],
+                                max_seq_len=cap, **sz["closest"])
+            eng = pkg.HipGpuInference.from_model(pkg.SynthModel(c, mix="Q8_0"), cap)
+            r["closest"] = layered_measure(eng, prompt, steps, args.reps)
+            eng.close()
+        res[name] = r
+        print(f"# {name} done", file=sys.stderr, flush=True)
+    first = res[names[0]].get("layered") or res[names[0]]["closest"]
+    print(json.dumps({"metric": f"decode tokens/sec, layered model {names[0]} (random weights), 1 GPU", "value": first["decode_tokens_per_s"],
+                      "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 4, "ms_per_step": round(first["decode_us"] / 1e3, 4),
+                      "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16 weights and block products, f32 residual / state",
+                      "data": "synthetic", "config": {"workload": f"{n}-token prompt, then greedy decode", "sizes": {k: LAYERED_SIZES[k] for k in names}},
+                      "results": res}))
 
 
 def prompt_tokens(n: int, vocab: int):
@@ -626,7 +733,9 @@ def main():
     from importlib import import_module
     pkg.pipeline = import_module("llama_gguf_amd.pipeline")
     # LGH_BENCH_FORCE_PIPELINE=1: run the N>1 code path with however many ranks there are (a 1-rank rehearsal on a 1-GPU box)
-    if args.batch:
+    if args.layered:
+        run_layered(args, pkg)
+    elif args.batch:
         run_batch(args, pkg)
     elif args.inlib:
         run_inlib(args, pkg)
