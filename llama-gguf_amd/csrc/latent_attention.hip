@@ -253,7 +253,7 @@ hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const i
 template <class O>
 __global__ void __launch_bounds__(256) latent_out_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M,
                                                          uint32_t n_splits, uint32_t KT, O* __restrict__ out, uint32_t ldo) {
-  extern __shared__ __attribute__((aligned(16))) float lat[];   // [rankp]
+  extern __shared__ __attribute__((aligned(16))) float lat[];   // [rankp], with room for the merge's thread groups
   __shared__ float wgt[kLatMaxSplits];
   const uint32_t tid = threadIdx.x, r = blockIdx.y, t = r / s.heads, h = r % s.heads, rows = M * s.heads;
   const uint32_t kv = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + M;
@@ -265,13 +265,36 @@ __global__ void __launch_bounds__(256) latent_out_kernel(const LatentShape s, co
     wgt[tid] = f / tot;
   }
   __syncthreads();
-  for (uint32_t i = tid; i < s.rankp; i += 256) {
-    float v = 0.0f;
-    if (i < s.rank) {
+  if ((s.rank & 3) == 0) {   // 4 columns per thread, the splits dealt to as many thread groups as there are threads for
+    const uint32_t quads = s.rankp / 4, groups = quads < 256 ? 256 / quads : 1, grp = tid / quads;
+    f32x4* acc4 = reinterpret_cast<f32x4*>(lat);   // [groups][quads]
+    for (uint32_t q = quads < 256 ? tid % quads : tid; q < quads && grp < groups; q += 256) {
+      f32x4 v = (f32x4)(0.0f);
+      if (q * 4 < s.rank) {
+        const float* src = b.part_acc + (size_t)r * s.rank + q * 4;
 #pragma unroll 8
-      for (uint32_t sp = 0; sp < act; sp++) v = __builtin_fmaf(wgt[sp], b.part_acc[((size_t)sp * rows + r) * s.rank + i], v);
+        for (uint32_t sp = grp; sp < act; sp += groups) {
+          const f32x4 x = *reinterpret_cast<const f32x4*>(src + (size_t)sp * rows * s.rank);
+          const float wg = wgt[sp];
+#pragma unroll
+          for (int e = 0; e < 4; e++) v[e] = __builtin_fmaf(wg, x[e], v[e]);
+        }
+      }
+      acc4[grp * quads + q] = v;
     }
-    lat[i] = v;
+    __syncthreads();
+    for (uint32_t q = tid; q < quads; q += 256) {
+      f32x4 v = acc4[q];
+      for (uint32_t k = 1; k < groups; k++) v += acc4[k * quads + q];
+      acc4[q] = v;
+    }
+  } else {
+    for (uint32_t i = tid; i < s.rankp; i += 256) {
+      float v = 0.0f;
+      if (i < s.rank)
+        for (uint32_t sp = 0; sp < act; sp++) v = __builtin_fmaf(wgt[sp], b.part_acc[((size_t)sp * rows + r) * s.rank + i], v);
+      lat[i] = v;
+    }
   }
   __syncthreads();
   const float gate = sigmoid_f(b.cat[(size_t)t * s.ldcat + s.off_g + h]);
@@ -300,9 +323,247 @@ hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const in
   const uint32_t KT = latent_key_tile(s, f32cache, M);
   if (!KT || s.rankp % 8 || n_splits == 0 || n_splits > kLatMaxSplits) return hipErrorInvalidValue;
   const dim3 grid((s.vdim + 31) / 32, M * s.heads);
-  if (out_f32) hipLaunchKernelGGL(latent_out_kernel<float>, grid, dim3(256), s.rankp * 4, st, s, b, pos_ptr, pos0, M, n_splits, KT, (float*)out, ldo);
-  else hipLaunchKernelGGL(latent_out_kernel<__bf16>, grid, dim3(256), s.rankp * 4, st, s, b, pos_ptr, pos0, M, n_splits, KT, (__bf16*)out, ldo);
+  const size_t lds = (size_t)(s.rankp < 1024 ? 1024 : s.rankp) * 4;
+  if (out_f32) hipLaunchKernelGGL(latent_out_kernel<float>, grid, dim3(256), lds, st, s, b, pos_ptr, pos0, M, n_splits, KT, (float*)out, ldo);
+  else hipLaunchKernelGGL(latent_out_kernel<__bf16>, grid, dim3(256), lds, st, s, b, pos_ptr, pos0, M, n_splits, KT, (__bf16*)out, ldo);
   return hipGetLastError();
+}
+
+// ------------------------------------------------------------------------------------------------
+// expanded path: queries, keys and values per head
+// ------------------------------------------------------------------------------------------------
+bool latent_flash_shape(const LatentShape& s, uint32_t* dq, uint32_t* dvp) {
+  const uint32_t d = s.dim + s.rot_dim;
+  if (d > 256 || s.vdim > 256) return false;
+  *dq = d <= 64 ? 64 : d <= 128 ? 128 : d <= 192 ? 192 : 256;
+  *dvp = s.vdim <= 64 ? 64 : s.vdim <= 128 ? 128 : 256;
+  return true;
+}
+
+// the block's cache rows and queries [head][token][dq] = [unrotated | rotated | zeros]; grid (tokens)
+template <class T>
+__global__ void __launch_bounds__(256) latent_flash_prep_kernel(const LatentShape s, const LatentBufs b, T* __restrict__ q, uint32_t dq, uint32_t Mcap,
+                                                                uint32_t pos0) {
+  __shared__ float red[16];
+  const uint32_t t = blockIdx.x, pos = pos0 + t;
+  const float* cat = b.cat + (size_t)t * s.ldcat;
+  latent_cache_row<T>(s, b, cat + s.off_dkv, pos, red);
+  const float* cs = b.cs + (size_t)pos * s.rot_n;
+  const uint32_t hd = s.dim + s.rot_dim;
+  for (uint32_t i = threadIdx.x; i < s.heads * dq; i += 256) {
+    const uint32_t h = i / dq, j = i % dq;
+    const float* src = cat + s.off_q + (size_t)h * hd;
+    float v = j < hd ? src[j] : 0.0f;
+    if (j >= s.dim && j - s.dim < s.rot_n) {
+      float p0, p1;
+      rot_pair(src + s.dim, cs, (j - s.dim) >> 1, p0, p1);
+      v = ((j - s.dim) & 1) ? p1 : p0;
+    }
+    q[((size_t)h * Mcap + t) * dq + j] = to_act<T>(v);
+  }
+}
+
+// the shared rotated key part of every cached position, beside each head's own key; grid (positions)
+template <class T>
+__global__ void __launch_bounds__(256) latent_rot_spread_kernel(const LatentShape s, const T* __restrict__ cache, T* __restrict__ k, uint32_t dq, uint64_t Tcap) {
+  const uint32_t t = blockIdx.x;
+  for (uint32_t i = threadIdx.x; i < s.heads * s.rot_dim; i += 256) {
+    const uint32_t h = i / s.rot_dim, j = i % s.rot_dim;
+    k[((size_t)h * Tcap + t) * dq + s.dim + j] = cache[(size_t)t * s.ldc + s.rank + j];
+  }
+}
+
+hipError_t latent_flash_prep_launch(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, bool f32, hipStream_t st) {
+  if (M == 0 || M > f.Mcap || pos0 + M > f.Tcap) return hipErrorInvalidValue;
+  if (f32) {
+    hipLaunchKernelGGL(latent_flash_prep_kernel<float>, dim3(M), dim3(256), 0, st, s, b, (float*)f.q, f.dq, f.Mcap, pos0);
+    if (s.rot_dim) hipLaunchKernelGGL(latent_rot_spread_kernel<float>, dim3(pos0 + M), dim3(256), 0, st, s, (const float*)b.cache, (float*)f.k, f.dq, f.Tcap);
+  } else {
+    hipLaunchKernelGGL(latent_flash_prep_kernel<__bf16>, dim3(M), dim3(256), 0, st, s, b, (__bf16*)f.q, f.dq, f.Mcap, pos0);
+    if (s.rot_dim) hipLaunchKernelGGL(latent_rot_spread_kernel<__bf16>, dim3(pos0 + M), dim3(256), 0, st, s, (const __bf16*)b.cache, (__bf16*)f.k, f.dq, f.Tcap);
+  }
+  return hipGetLastError();
+}
+
+// Causal attention, everything transposed: S^T = K Q^T leaves a lane with one query's scores of keys 4g .. 4g + 3, which is the B
+// operand of O^T = V^T P^T when the value fragment's k slots are assigned the same way — the weights never leave the registers.
+// A workgroup = 4 waves = 64 * QT queries of one head; K and V^T tiles of KT keys go to LDS by DMA, two buffers.
+template <class T, int DQ, int DV>
+__global__ void __launch_bounds__(256) latent_flash_kernel(const LatentShape s, const LatentBufs b, const LatentFlash f, uint32_t pos0, uint32_t M, uint32_t nqb,
+                                                           T* __restrict__ out, uint32_t ldo) {
+  constexpr bool BF = sizeof(T) == 2;
+  constexpr int KT = BF ? 64 : 32, QT = BF ? 2 : 1, NK = KT / 16, NU = DQ / Frag<T>::KU, ND = DV / 16, NP = KT / Frag<T>::KU;
+  constexpr uint32_t XC = DQ * sizeof(T) / 16, kK = KT * XC * 16, kV = DV * 128, kBuf = kK + kV;
+  extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
+  const uint32_t lane = threadIdx.x & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)), r16 = lane & 15, g = lane >> 4;
+  const uint32_t h = blockIdx.x % s.heads, qb = nqb - 1 - blockIdx.x / s.heads;   // the longest rows first
+  const uint32_t q0 = qb * 64 * QT, qw = q0 + w * 16 * QT;
+  const uint32_t qlast = q0 + 64 * QT - 1 < M - 1 ? q0 + 64 * QT - 1 : M - 1;
+  const uint32_t tiles = (pos0 + qlast + KT) / KT;   // keys 0 .. pos0 + qlast
+  const T* K = reinterpret_cast<const T*>(f.k) + (size_t)h * f.Tcap * DQ;
+  const T* V = reinterpret_cast<const T*>(f.vt) + (size_t)h * f.dvp * f.Tcap;
+  auto stage = [&](uint32_t tl, uint32_t buf) {
+    uint8_t* base = smem + buf * kBuf;
+#pragma unroll
+    for (int i = 0; i < (int)(kK / 4096); i++) {
+      const uint32_t c = (i * 4 + w) * 64 + lane, row = c / XC, ch = (c % XC) ^ (row & 7);
+      lds_dma16(K + ((size_t)tl * KT + row) * DQ + ch * (16 / sizeof(T)), base + (i * 4 + w) * 1024);
+    }
+#pragma unroll
+    for (int i = 0; i < (int)(kV / 4096); i++) {
+      const uint32_t c = (i * 4 + w) * 64 + lane, row = c / 8, ch = (c % 8) ^ (row & 7);
+      lds_dma16(V + (size_t)row * f.Tcap + (size_t)tl * KT + ch * (16 / sizeof(T)), base + kK + (i * 4 + w) * 1024);
+    }
+  };
+  stage(0, 0);
+  typename Frag<T>::V qf[QT][NU];
+#pragma unroll
+  for (int t = 0; t < QT; t++) {
+    const uint32_t m = qw + t * 16 + r16;
+    const T* qr = reinterpret_cast<const T*>(f.q) + ((size_t)h * f.Mcap + (m < M ? m : M - 1)) * DQ + g * Frag<T>::PER;
+#pragma unroll
+    for (int u = 0; u < NU; u++) qf[t][u] = Frag<T>::load(qr + u * Frag<T>::KU);
+  }
+  f32x4 o[ND][QT];
+  float mx[QT], l[QT];
+#pragma unroll
+  for (int t = 0; t < QT; t++) {
+    mx[t] = kNegHuge; l[t] = 0.0f;
+#pragma unroll
+    for (int i = 0; i < ND; i++) o[i][t] = (f32x4)(0.0f);
+  }
+  // bf16: scores in units of log2 (one v_exp per weight); f32: natural, with the library exponential
+  const float sc = BF ? s.scale * 1.4426950408889634f : s.scale;
+  __builtin_amdgcn_s_waitcnt(0x0F70);   // vmcnt(0)
+  __syncthreads();
+  for (uint32_t tl = 0; tl < tiles; tl++) {
+    const uint32_t cur = tl & 1, k0 = tl * KT;
+    if (tl + 1 < tiles) stage(tl + 1, cur ^ 1);
+    const uint8_t* kb = smem + cur * kBuf;
+    const uint8_t* vb = kb + kK;
+    f32x4 sa[NK][QT];
+#pragma unroll
+    for (int n = 0; n < NK; n++)
+#pragma unroll
+      for (int t = 0; t < QT; t++) sa[n][t] = (f32x4)(0.0f);
+#pragma unroll
+    for (int u = 0; u < NU; u++)
+#pragma unroll
+      for (int n = 0; n < NK; n++) {
+        const uint32_t row = n * 16 + r16;
+        const typename Frag<T>::V kf = Frag<T>::load(reinterpret_cast<const T*>(kb + row * (XC * 16) + (((uint32_t)(u * 4) + g) ^ (row & 7)) * 16));
+#pragma unroll
+        for (int t = 0; t < QT; t++) sa[n][t] = Frag<T>::mma(kf, qf[t][u], sa[n][t]);
+      }
+    const bool edge = k0 + KT > pos0 + qw + 1;   // wave-uniform: some key may lie behind some query
+#pragma unroll
+    for (int t = 0; t < QT; t++) {
+      const uint32_t lim = pos0 + qw + t * 16 + r16;   // last visible key
+      float m1 = mx[t];
+#pragma unroll
+      for (int n = 0; n < NK; n++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+          float v = sa[n][t][e] * sc;
+          if (edge) v = k0 + n * 16 + g * 4 + e > lim ? kNegHuge : v;
+          sa[n][t][e] = v;
+          m1 = fmaxf(m1, v);
+        }
+      m1 = fmaxf(m1, __shfl_xor(m1, 16, 64));
+      m1 = fmaxf(m1, __shfl_xor(m1, 32, 64));
+      const float a = BF ? __builtin_amdgcn_exp2f(mx[t] - m1) : expf(mx[t] - m1);
+      float sum = 0.0f;
+#pragma unroll
+      for (int n = 0; n < NK; n++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+          const float p = BF ? __builtin_amdgcn_exp2f(sa[n][t][e] - m1) : expf(sa[n][t][e] - m1);
+          sa[n][t][e] = p;
+          sum += p;
+        }
+      l[t] = __builtin_fmaf(l[t], a, sum);
+      if (__any(m1 > mx[t])) {
+#pragma unroll
+        for (int i = 0; i < ND; i++) o[i][t] *= a;
+      }
+      mx[t] = m1;
+    }
+#pragma unroll
+    for (int u = 0; u < NP; u++) {
+      typename Frag<T>::V pf[QT];
+#pragma unroll
+      for (int t = 0; t < QT; t++) {
+        if constexpr (BF) {
+#pragma unroll
+          for (int e = 0; e < 4; e++) { pf[t][e] = (__bf16)sa[2 * u][t][e]; pf[t][4 + e] = (__bf16)sa[2 * u + 1][t][e]; }
+        } else {
+          pf[t] = sa[u][t];
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < ND; i++) {
+        const uint32_t row = i * 16 + r16;
+        typename Frag<T>::V vf;
+        if constexpr (BF) {
+          const bf16x4 a = *reinterpret_cast<const bf16x4*>(vb + row * 128 + (((uint32_t)(4 * u) + (g >> 1)) ^ (row & 7)) * 16 + (g & 1) * 8);
+          const bf16x4 c = *reinterpret_cast<const bf16x4*>(vb + row * 128 + (((uint32_t)(4 * u + 2) + (g >> 1)) ^ (row & 7)) * 16 + (g & 1) * 8);
+          vf = __builtin_shufflevector(a, c, 0, 1, 2, 3, 4, 5, 6, 7);
+        } else {
+          vf = Frag<T>::load(reinterpret_cast<const T*>(vb + row * 128 + (((uint32_t)(4 * u) + g) ^ (row & 7)) * 16));
+        }
+#pragma unroll
+        for (int t = 0; t < QT; t++) o[i][t] = Frag<T>::mma(vf, pf[t], o[i][t]);
+      }
+    }
+    __builtin_amdgcn_s_waitcnt(0x0F70);
+    __syncthreads();
+  }
+#pragma unroll
+  for (int t = 0; t < QT; t++) {
+    float lt = l[t];
+    lt += __shfl_xor(lt, 16, 64);
+    lt += __shfl_xor(lt, 32, 64);
+    const uint32_t m = qw + t * 16 + r16;
+    if (m >= M) continue;
+    const float fac = sigmoid_f(b.cat[(size_t)m * s.ldcat + s.off_g + h]) / lt;
+    T* dst = out + (size_t)m * ldo + h * s.vdim;
+#pragma unroll
+    for (int i = 0; i < ND; i++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        const uint32_t v = i * 16 + g * 4 + e;
+        if (v < s.vdim) dst[v] = to_act<T>(o[i][t][e] * fac);
+      }
+  }
+}
+
+template <class T, int DQ, int DV>
+static hipError_t latent_flash_go(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, void* out, uint32_t ldo, hipStream_t st) {
+  static bool opted[64] = {};
+  constexpr size_t KT = sizeof(T) == 2 ? 64 : 32, lds = 2 * (KT * DQ * sizeof(T) + DV * 128);
+  static_assert(lds <= 160 * 1024, "two tiles fit LDS");
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&latent_flash_kernel<T, DQ, DV>), (int)lds, opted); e != hipSuccess) return e;
+  const uint32_t QB = sizeof(T) == 2 ? 128 : 64, nqb = (M + QB - 1) / QB;
+  hipLaunchKernelGGL((latent_flash_kernel<T, DQ, DV>), dim3(nqb * s.heads), dim3(256), lds, st, s, b, f, pos0, M, nqb, (T*)out, ldo);
+  return hipGetLastError();
+}
+
+template <class T>
+static hipError_t latent_flash_pick(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, void* out, uint32_t ldo, hipStream_t st) {
+#define LGH_FLASH_CASE(Q, V) if (f.dq == Q && f.dvp == V) return latent_flash_go<T, Q, V>(s, b, f, pos0, M, out, ldo, st);
+  LGH_FLASH_CASE(64, 64) LGH_FLASH_CASE(64, 128) LGH_FLASH_CASE(64, 256)
+  LGH_FLASH_CASE(128, 64) LGH_FLASH_CASE(128, 128) LGH_FLASH_CASE(128, 256)
+  LGH_FLASH_CASE(192, 64) LGH_FLASH_CASE(192, 128) LGH_FLASH_CASE(192, 256)
+  LGH_FLASH_CASE(256, 64) LGH_FLASH_CASE(256, 128) LGH_FLASH_CASE(256, 256)
+#undef LGH_FLASH_CASE
+  return hipErrorInvalidValue;
+}
+
+hipError_t latent_flash_launch(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, bool f32, void* out, uint32_t ldo,
+                               hipStream_t st) {
+  const uint64_t KT = f32 ? 32 : 64;
+  if (M == 0 || M > f.Mcap || f.Tcap % 64 || (pos0 + M + KT - 1) / KT * KT > f.Tcap) return hipErrorInvalidValue;   // whole key tiles are read
+  return f32 ? latent_flash_pick<float>(s, b, f, pos0, M, out, ldo, st) : latent_flash_pick<__bf16>(s, b, f, pos0, M, out, ldo, st);
 }
 
 }  // namespace lgh

@@ -112,7 +112,7 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
       if (l.rot_dims && !(l.rot_base > 0.0)) { why = at + "rotation base"; return LGH_INVALID_ARGUMENT; }
       LatentShape s{};
       s.rank = l.kv_rank;
-      s.ldc = up(l.kv_rank + l.rot_dim, 32);
+      s.ldc = std::max(up(l.kv_rank + l.rot_dim, 32), up(l.kv_rank, 64));
       if (l.heads > kLatAbsorbRows || !latent_key_tile(s, d.compute == LGH_COMPUTE_F32, 1)) { why = at + "latent rows too large for LDS"; return LGH_UNSUPPORTED; }
     } else if (l.mixer == LGH_MIXER_MLSTM) {
       if (!(l.gate_cap > 0.0)) { why = at + "gate_cap"; return LGH_INVALID_ARGUMENT; }
@@ -163,7 +163,7 @@ static void layered_plan(LayeredModel& m) {
     if (L.latent()) {
       LatentShape& s = L.ls;
       s.heads = l.heads; s.dim = l.dim; s.rot_dim = l.rot_dim; s.rot_n = l.rot_dims; s.vdim = l.vdim; s.rank = l.kv_rank;
-      s.ldc = up(l.kv_rank + l.rot_dim, 32);
+      s.ldc = std::max(up(l.kv_rank + l.rot_dim, 32), up(l.kv_rank, 64));   // (a whole row is also the input row of the expansions)
       s.dimp = up(l.dim, 8);
       s.rankp = up(l.kv_rank, 64);
       s.scale = (float)l.scale; s.eps = (float)d.norm_eps;
@@ -512,10 +512,44 @@ static int block_gemm(lgh_ctx* c, int cls, const LinW& W, int epi, const void* x
   return run_k(c, cls, LGH_SYM_LINEAR, W.bytes(), [&] { return lin_gemm_launch(epi, c->lm->f32, g, c->stream); });
 }
 
+// a buffer of the expanded path, grown when the context does (zeroed: the padding of a key tile must be finite)
+static int grow(lgh_ctx* c, void** p, size_t* have, size_t need) {
+  if (*have >= need) return LGH_OK;
+  L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
+  if (*p) dev_free_tracked(c, *p);
+  c->stats.scratch_bytes -= *have;
+  *p = nullptr;
+  *have = 0;
+  if (int rc = zeroed(c, p, need, &c->stats.scratch_bytes)) return rc;
+  *have = need;
+  return LGH_OK;
+}
+
+// portions from this many tokens on form keys and values per head when the context is not much longer than they are
+constexpr uint32_t kExpandTokens = 64;
+
 static int block_latent(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) {
   LayeredModel& m = *c->lm;
   hipStream_t st = c->stream;
   int rc;
+  LatentFlash& f = m.fl;
+  if (M >= kExpandTokens && pos0 <= 64 * M && latent_flash_shape(L.ls, &f.dq, &f.dvp)) {
+    const uint32_t kv = pos0 + M, H = L.ls.heads;
+    f.Mcap = m.blk;
+    f.Tcap = up(kv, 1024);
+    if ((rc = grow(c, &f.q, &m.fl_q_bytes, (size_t)H * f.Mcap * f.dq * m.el())) || (rc = grow(c, &f.k, &m.fl_k_bytes, (size_t)H * f.Tcap * f.dq * m.el())) ||
+        (rc = grow(c, &f.vt, &m.fl_v_bytes, (size_t)H * f.dvp * f.Tcap * m.el())))
+      return rc;
+    const LatentBufs b = latent_bufs(m, L, m.bcat);
+    if ((rc = run_k(c, LGH_K_MISC, LGH_SYM_LATENT, 0, [&] { return latent_flash_prep_launch(L.ls, b, f, pos0, M, m.f32, st); }))) return rc;
+    LinGemm g{};
+    g.x = L.cache; g.ldx = L.ls.ldc; g.M = kv;
+    g.w = L.uk.w; g.n = L.uk.n; g.np = L.uk.np(); g.kp = L.uk.kp; g.out = f.k; g.ldo = f.dq; g.hd = L.ls.dim; g.tcap = f.Tcap;
+    if ((rc = run_k(c, LGH_K_ROUTER, LGH_SYM_LINEAR, L.uk.bytes(), [&] { return lin_gemm_launch(LE_HEADS, m.f32, g, st); }))) return rc;
+    g.w = L.uv.w; g.n = L.uv.n; g.np = L.uv.np(); g.kp = L.uv.kp; g.out = f.vt; g.ldo = (uint32_t)f.Tcap; g.hd = L.ls.vdim; g.hrows = f.dvp;
+    if ((rc = run_k(c, LGH_K_ROUTER, LGH_SYM_LINEAR, L.uv.bytes(), [&] { return lin_gemm_launch(LE_HEADS_T, m.f32, g, st); }))) return rc;
+    return run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, 0, [&] { return latent_flash_launch(L.ls, b, f, pos0, M, m.f32, m.bao, L.out.kp, st); });
+  }
   // absorbed, as many tokens at a time as their (token, head) rows fit the buffers
   const uint32_t step = std::max(1u, kLatAbsorbRows / L.ls.heads);
   for (uint32_t t = 0; t < M; t += step) {

@@ -247,6 +247,12 @@ __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t
 #pragma unroll
           for (int e = 0; e < 4; e++)
             if (nb + e < a.n) o[e] = to_act<T>(acc[i][j][e]);
+        } else if (EPI == LE_HEADS && (a.hd & 3) == 0 && nb + 4 <= a.n) {   // the four columns lie in one head
+          T* o = reinterpret_cast<T*>(a.out) + ((size_t)(nb / a.hd) * a.tcap + m) * a.ldo + nb % a.hd;
+          T v[4];
+#pragma unroll
+          for (int e = 0; e < 4; e++) v[e] = to_act<T>(acc[i][j][e]);
+          __builtin_memcpy(__builtin_assume_aligned(o, sizeof(v)), v, sizeof(v));
         } else {
 #pragma unroll
           for (int e = 0; e < 4; e++) {
