@@ -90,15 +90,40 @@ hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const i
 }
 
 // ------------------------------------------------------------------------------------------------
-// absorbed attention.  A workgroup = 16 (token, head) rows x one split of the keys x up to 512 latent columns of the output;
-// KT keys at a time in LDS.  Scores: wave w multiplies the 16 rows with keys 16 w ..; weighted sums: wave w owns a quarter of the
-// columns and takes the values straight from the key tile (the latent IS the value).
+// absorbed attention.  A workgroup = 16 (token, head) rows x one split of the keys x up to 512 latent columns of the output; 32 keys
+// at a time go to LDS by DMA (16-byte chunks of a row stored at chunk ^ (row & 7)).  Scores: wave w multiplies the 16 rows with keys
+// 16 (w & 1) .. over half w >> 1 of the row; weighted sums: wave w owns a quarter of the columns and takes the values straight from
+// the key tile (the latent IS the value), transposed on the way out of LDS.
 // ------------------------------------------------------------------------------------------------
-template <class T> constexpr uint32_t lat_pad() { return 16 / sizeof(T); }   // LDS row padding: consecutive rows shift by 4 banks
+constexpr uint32_t kLatKeys = 32;
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+
+// value fragment: column c0 + r16, keys kb .. (the unit's) of the tile; row stride ld elements, chunks swizzled by row & 7
+template <class T>
+__device__ __forceinline__ typename Frag<T>::V lat_value_frag(const T* tile, uint32_t ld, uint32_t kb, uint32_t c0, uint32_t r16, uint32_t g) {
+  if constexpr (sizeof(T) == 2) {   // lane i of a 16-lane group fetches 4 columns of key row i / 4 and receives 4 keys of column i
+    const uint32_t col = c0 + (r16 & 3) * 4, row = kb + g * 8 + (r16 >> 2);
+    typedef __attribute__((address_space(3))) s16x4* lds_p;
+    const T* p0 = tile + row * ld + ((col >> 3) ^ (row & 7)) * 8 + (col & 7);
+    const T* p1 = tile + (row + 4) * ld + ((col >> 3) ^ ((row + 4) & 7)) * 8 + (col & 7);
+    const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)p0), b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)p1);
+    return __builtin_bit_cast(bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
+  } else {
+    const uint32_t col = c0 + r16;
+    f32x4 v;
+#pragma unroll
+    for (uint32_t e = 0; e < 4; e++) {
+      const uint32_t row = kb + g * 4 + e;
+      v[e] = tile[row * ld + ((col >> 2) ^ (row & 7)) * 4 + (col & 3)];
+    }
+    return v;
+  }
+}
 
 template <class T, int NCT>   // NCT: 16-column tiles of the output per wave
 __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M,
-                                                          uint32_t n_splits, uint32_t KT) {
+                                                          uint32_t n_splits, uint32_t nbuf) {
+  constexpr uint32_t KT = kLatKeys, PER = Frag<T>::PER, KU = Frag<T>::KU, LP = KT + 16 / sizeof(T), LS = KT + 4;
   extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
   const uint32_t tid = threadIdx.x, lane = tid & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
   const uint32_t r16 = lane & 15, g = lane >> 4;
@@ -108,19 +133,25 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
   const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles + n_splits - 1) / n_splits;
   const uint32_t tb = sp * per, te = tb + per < tiles ? tb + per : tiles;
   if (tb >= te) return;                                         // (the merge skips the same splits)
-  const uint32_t ldq = s.ldc + lat_pad<T>(), lds_s = KT + 4, lds_p = KT + lat_pad<T>();
-  T* Qs = reinterpret_cast<T*>(smem);                           // [16][ldq]
-  T* Cs = Qs + 16 * ldq;                                        // [KT][ldq]
-  T* Ps = Cs + KT * ldq;                                        // [16][lds_p]
-  float* Ss = reinterpret_cast<float*>(Ps + 16 * lds_p);        // [16][lds_s]
-  constexpr uint32_t PER = Frag<T>::PER, KU = Frag<T>::KU;
-  const uint32_t cpr = s.ldc / PER;                             // 16-byte chunks of a row
+  const uint32_t ld = s.ldc, cpr = ld / PER;                    // 16-byte chunks of a row: a multiple of 8
+  T* Qs = reinterpret_cast<T*>(smem);                           // [16][ld]
+  T* Cs = Qs + 16 * ld;                                         // [nbuf][KT][ld]
+  T* Ps = Cs + nbuf * KT * ld;                                  // [16][LP]
+  float* Ss = reinterpret_cast<float*>(Ps + 16 * LP);           // [2][16][LS]
   const T* qg = reinterpret_cast<const T*>(b.qa);
   const T* cg = reinterpret_cast<const T*>(b.cache);
-  for (uint32_t i = tid; i < 16 * cpr; i += 256) {
-    const uint32_t r = i / cpr, ch = i % cpr, rr = row0 + r < rows ? row0 + r : rows - 1;
-    *reinterpret_cast<u32x4*>(Qs + r * ldq + ch * PER) = *reinterpret_cast<const u32x4*>(qg + (size_t)rr * s.ldc + ch * PER);
+  auto stage = [&](uint32_t tl, uint32_t buf) {
+    T* dst = Cs + buf * KT * ld;
+    for (uint32_t i = w; i < KT * cpr / 64; i += 4) {
+      const uint32_t c = i * 64 + lane, r = c / cpr, ch = (c % cpr) ^ (r & 7), kk = tl * KT + r < kv ? tl * KT + r : kv - 1;
+      lds_dma16(cg + (size_t)kk * ld + ch * PER, dst + (size_t)i * 64 * PER);
+    }
+  };
+  for (uint32_t i = w; i < 16 * cpr / 64; i += 4) {             // the queries, same layout
+    const uint32_t c = i * 64 + lane, r = c / cpr, ch = (c % cpr) ^ (r & 7), rr = row0 + r < rows ? row0 + r : rows - 1;
+    lds_dma16(qg + (size_t)rr * ld + ch * PER, Qs + (size_t)i * 64 * PER);
   }
+  stage(tb, 0);
   // the rows of this lane's accumulators: 4g .. 4g + 3
   uint32_t lim[4];
   float m[4], l[4];
@@ -133,43 +164,52 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
   f32x4 o[NCT];
 #pragma unroll
   for (int i = 0; i < NCT; i++) o[i] = (f32x4)(0.0f);
-  const uint32_t wc = col0 + w * NCT * 16;
+  const uint32_t wc = col0 + w * NCT * 16, half = cpr / 8 * (w >> 1);   // first unit of the wave's half row (4 chunks a unit)
+  const uint32_t u1 = w >> 1 ? cpr / 4 : cpr / 8;
+  __builtin_amdgcn_s_waitcnt(0x0F70);   // vmcnt(0)
+  __syncthreads();
   for (uint32_t tl = tb; tl < te; tl++) {
-    const uint32_t k0 = tl * KT;
-    __syncthreads();                                            // the previous tile is used up
-    for (uint32_t i = tid; i < KT * cpr; i += 256) {
-      const uint32_t r = i / cpr, ch = i % cpr, kk = k0 + r < kv ? k0 + r : kv - 1;
-      *reinterpret_cast<u32x4*>(Cs + r * ldq + ch * PER) = *reinterpret_cast<const u32x4*>(cg + (size_t)kk * s.ldc + ch * PER);
-    }
-    __syncthreads();
-    if (w * 16 < KT) {
-      f32x4 sc = (f32x4)(0.0f);
-      const T* qa = Qs + r16 * ldq + g * PER;
-      const T* kb = Cs + (w * 16 + r16) * ldq + g * PER;
-      for (uint32_t k = 0; k < s.ldc; k += KU) sc = Frag<T>::mma(Frag<T>::load(qa + k), Frag<T>::load(kb + k), sc);
+    const uint32_t k0 = tl * KT, cur = nbuf == 2 ? (tl - tb) & 1 : 0;
+    if (nbuf == 2 && tl + 1 < te) stage(tl + 1, cur ^ 1);
+    const T* tile = Cs + cur * KT * ld;
+    {
+      f32x4 sc = (f32x4)(0.0f), sd = (f32x4)(0.0f);
+      const T* qa = Qs + r16 * ld;
+      const T* kb = tile + ((w & 1) * 16 + r16) * ld;
+      uint32_t u = half;
+      for (; u + 2 <= u1; u += 2) {
+        const uint32_t c0 = ((u * 4 + g) ^ (r16 & 7)) * PER, c1 = ((u * 4 + 4 + g) ^ (r16 & 7)) * PER;
+        sc = Frag<T>::mma(Frag<T>::load(qa + c0), Frag<T>::load(kb + c0), sc);
+        sd = Frag<T>::mma(Frag<T>::load(qa + c1), Frag<T>::load(kb + c1), sd);
+      }
+      if (u < u1) {
+        const uint32_t c0 = ((u * 4 + g) ^ (r16 & 7)) * PER;
+        sc = Frag<T>::mma(Frag<T>::load(qa + c0), Frag<T>::load(kb + c0), sc);
+      }
+      sc += sd;
 #pragma unroll
-      for (int e = 0; e < 4; e++) Ss[(g * 4 + e) * lds_s + w * 16 + r16] = sc[e] * s.scale;
+      for (int e = 0; e < 4; e++) Ss[((w >> 1) * 16 + g * 4 + e) * LS + (w & 1) * 16 + r16] = sc[e];
     }
     __syncthreads();
-    // softmax of the tile, by every wave for its own use: lane (r16, g) looks at keys r16, r16 + 16, .. of rows 4g .. 4g + 3
+    // softmax of the tile, by every wave for its own use: lane (r16, g) looks at keys r16, r16 + 16 of rows 4g .. 4g + 3
     float alpha[4];
 #pragma unroll
     for (int e = 0; e < 4; e++) {
-      float mx = m[e], sv[4];
+      float mx = m[e], sv[2];
 #pragma unroll
-      for (int j = 0; j < 4; j++) {
-        const uint32_t key = r16 + j * 16;
-        sv[j] = key < KT && k0 + key < lim[e] ? Ss[(g * 4 + e) * lds_s + key] : kNegHuge;
+      for (int j = 0; j < 2; j++) {
+        const uint32_t key = r16 + j * 16, at = (g * 4 + e) * LS + key;
+        sv[j] = k0 + key < lim[e] ? (Ss[at] + Ss[16 * LS + at]) * s.scale : kNegHuge;
         mx = fmaxf(mx, sv[j]);
       }
       mx = fmaxf(mx, dpp_f<0xB1>(mx)); mx = fmaxf(mx, dpp_f<0x4E>(mx)); mx = fmaxf(mx, dpp_f<0x141>(mx)); mx = fmaxf(mx, dpp_f<0x140>(mx));
       float sum = 0.0f;
 #pragma unroll
-      for (int j = 0; j < 4; j++) {
+      for (int j = 0; j < 2; j++) {
         const uint32_t key = r16 + j * 16;
-        const float p = key < KT && k0 + key < lim[e] ? expf(sv[j] - mx) : 0.0f;
+        const float p = k0 + key < lim[e] ? expf(sv[j] - mx) : 0.0f;
         sum += p;
-        if (w == 0 && key < KT) Ps[(g * 4 + e) * lds_p + key] = to_act<T>(p);
+        if (w == 0) Ps[(g * 4 + e) * LP + key] = to_act<T>(p);
       }
       sum += dpp_f<0xB1>(sum); sum += dpp_f<0x4E>(sum); sum += dpp_f<0x141>(sum); sum += dpp_f<0x140>(sum);
       alpha[e] = expf(m[e] - mx);
@@ -181,18 +221,21 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
     for (int i = 0; i < NCT; i++)
 #pragma unroll
       for (int e = 0; e < 4; e++) o[i][e] *= alpha[e];
+#pragma unroll
     for (uint32_t k = 0; k < KT; k += KU) {
-      const typename Frag<T>::V pf = Frag<T>::load(Ps + r16 * lds_p + k + g * PER);
+      const typename Frag<T>::V pf = Frag<T>::load(Ps + r16 * LP + k + g * PER);
 #pragma unroll
       for (int i = 0; i < NCT; i++) {
-        const uint32_t c = wc + i * 16 + r16;
-        typename Frag<T>::V vf;
-        const T* src = Cs + (k + g * PER) * ldq + (c < s.ldc ? c : s.ldc - 1);
-#pragma unroll
-        for (uint32_t e = 0; e < PER; e++) vf[e] = src[e * ldq];
-        o[i] = Frag<T>::mma(pf, vf, o[i]);
+        const uint32_t c0 = wc + i * 16 < ld ? wc + i * 16 : ld - 16;   // (columns past the row: computed, never stored)
+        o[i] = Frag<T>::mma(pf, lat_value_frag<T>(tile, ld, k, c0, r16, g), o[i]);
       }
     }
+    if (nbuf == 1 && tl + 1 < te) {
+      __syncthreads();
+      stage(tl + 1, 0);
+    }
+    __builtin_amdgcn_s_waitcnt(0x0F70);
+    __syncthreads();
   }
 #pragma unroll
   for (int e = 0; e < 4; e++) {
@@ -208,36 +251,34 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
   }
 }
 
-static size_t latent_lds(const LatentShape& s, uint32_t KT, uint32_t el) {
-  const uint32_t pad = 16 / el, ldq = s.ldc + pad;
-  return (size_t)(16 + KT) * ldq * el + (size_t)16 * (KT + pad) * el + (size_t)16 * (KT + 4) * 4;
+static size_t latent_lds(const LatentShape& s, uint32_t nbuf, uint32_t el) {
+  return (size_t)(16 + nbuf * kLatKeys) * s.ldc * el + (size_t)16 * (kLatKeys + 16 / el) * el + (size_t)2 * 16 * (kLatKeys + 4) * 4;
 }
 
-uint32_t latent_key_tile(const LatentShape& s, bool f32, uint32_t M) {
-  (void)M;
-  for (uint32_t KT : {64u, 32u, 16u}) {
-    if (!f32 && KT < 32) break;   // a bf16 unit spans 32 keys
-    if (latent_lds(s, KT, f32 ? 4 : 2) <= 155 * 1024) return KT;
-  }
+// key tiles in flight (0: a row is too long for LDS)
+static uint32_t latent_nbuf(const LatentShape& s, bool f32) {
+  for (uint32_t n : {2u, 1u})
+    if (latent_lds(s, n, f32 ? 4 : 2) <= 155 * 1024) return n;
   return 0;
 }
+bool latent_fits(const LatentShape& s, bool f32) { return latent_nbuf(s, f32) != 0; }
 
 template <class T, int NCT>
-static hipError_t latent_attn_go(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, uint32_t KT,
+static hipError_t latent_attn_go(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, uint32_t nbuf,
                                  uint32_t zs, hipStream_t st) {
   static bool opted[64] = {};
   if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&latent_attn_kernel<T, NCT>), 156 * 1024, opted); e != hipSuccess) return e;
-  hipLaunchKernelGGL((latent_attn_kernel<T, NCT>), dim3((M * s.heads + 15) / 16, n_splits, zs), dim3(256), latent_lds(s, KT, sizeof(T)), st, s, b, pos_ptr,
-                     pos0, M, n_splits, KT);
+  hipLaunchKernelGGL((latent_attn_kernel<T, NCT>), dim3((M * s.heads + 15) / 16, n_splits, zs), dim3(256), latent_lds(s, nbuf, sizeof(T)), st, s, b, pos_ptr,
+                     pos0, M, n_splits, nbuf);
   return hipGetLastError();
 }
 
 hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32,
                               hipStream_t st) {
-  const uint32_t KT = latent_key_tile(s, f32, M);
-  if (!KT || s.ldc % 32 || n_splits == 0 || n_splits > kLatMaxSplits || M == 0 || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
+  const uint32_t nbuf = latent_nbuf(s, f32);
+  if (!nbuf || s.ldc % 64 || n_splits == 0 || n_splits > kLatMaxSplits || M == 0 || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
   const uint32_t nct = (s.rank + 63) / 64;
-#define LGH_LAT_CASE(N) return f32 ? latent_attn_go<float, N>(s, b, pos_ptr, pos0, M, n_splits, KT, zs, st) : latent_attn_go<__bf16, N>(s, b, pos_ptr, pos0, M, n_splits, KT, zs, st)
+#define LGH_LAT_CASE(N) return f32 ? latent_attn_go<float, N>(s, b, pos_ptr, pos0, M, n_splits, nbuf, zs, st) : latent_attn_go<__bf16, N>(s, b, pos_ptr, pos0, M, n_splits, nbuf, zs, st)
   uint32_t zs = 1;
   if (nct <= 1) LGH_LAT_CASE(1);
   if (nct <= 2) LGH_LAT_CASE(2);
@@ -258,6 +299,13 @@ __global__ void __launch_bounds__(256) latent_out_kernel(const LatentShape s, co
   const uint32_t tid = threadIdx.x, r = blockIdx.y, t = r / s.heads, h = r % s.heads, rows = M * s.heads;
   const uint32_t kv = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + M;
   const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles + n_splits - 1) / n_splits, act = (tiles + per - 1) / per;
+  const uint32_t lane = tid & 63, w = tid >> 6;
+  u32x4 wv0[8];   // the wave's 8 value rows, first 512 columns: requested before the merge
+#pragma unroll
+  for (int it = 0; it < 8; it++) {
+    const uint32_t v = blockIdx.x * 32 + it * 4 + w, vc = v < s.vdim ? v : s.vdim - 1, k = lane * 8 < s.rankp ? lane * 8 : 0;
+    wv0[it] = *reinterpret_cast<const u32x4*>(b.uv + ((size_t)h * s.vdim + vc) * s.rankp + k);
+  }
   if (tid < 64) {
     const float mi = tid < act ? b.part_ml[((size_t)tid * rows + r) * 2] : kNegHuge;
     const float li = tid < act ? b.part_ml[((size_t)tid * rows + r) * 2 + 1] : 0.0f;
@@ -298,15 +346,14 @@ __global__ void __launch_bounds__(256) latent_out_kernel(const LatentShape s, co
   }
   __syncthreads();
   const float gate = sigmoid_f(b.cat[(size_t)t * s.ldcat + s.off_g + h]);
-  const uint32_t lane = tid & 63, w = tid >> 6;
-#pragma unroll 2
+#pragma unroll
   for (int it = 0; it < 8; it++) {
     const uint32_t v = blockIdx.x * 32 + it * 4 + w;
-    if (v >= s.vdim) break;
+    if (v >= s.vdim) continue;
     const uint16_t* W = b.uv + ((size_t)h * s.vdim + v) * s.rankp;
     float acc = 0.0f;
     for (uint32_t k = lane * 8; k < s.rankp; k += 512) {
-      const u32x4 wv = *reinterpret_cast<const u32x4*>(W + k);
+      const u32x4 wv = k < 512 ? wv0[it] : *reinterpret_cast<const u32x4*>(W + k);
       const f32x4 x0 = *reinterpret_cast<const f32x4*>(lat + k), x1 = *reinterpret_cast<const f32x4*>(lat + k + 4);
       acc = __builtin_fmaf(bf_lo(wv.x), x0.x, acc); acc = __builtin_fmaf(bf_hi(wv.x), x0.y, acc);
       acc = __builtin_fmaf(bf_lo(wv.y), x0.z, acc); acc = __builtin_fmaf(bf_hi(wv.y), x0.w, acc);
@@ -320,8 +367,8 @@ __global__ void __launch_bounds__(256) latent_out_kernel(const LatentShape s, co
 
 hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32cache,
                              void* out, uint32_t ldo, bool out_f32, hipStream_t st) {
-  const uint32_t KT = latent_key_tile(s, f32cache, M);
-  if (!KT || s.rankp % 8 || n_splits == 0 || n_splits > kLatMaxSplits) return hipErrorInvalidValue;
+  constexpr uint32_t KT = kLatKeys;
+  if (s.rankp % 8 || n_splits == 0 || n_splits > kLatMaxSplits) return hipErrorInvalidValue;
   const dim3 grid((s.vdim + 31) / 32, M * s.heads);
   const size_t lds = (size_t)(s.rankp < 1024 ? 1024 : s.rankp) * 4;
   if (out_f32) hipLaunchKernelGGL(latent_out_kernel<float>, grid, dim3(256), lds, st, s, b, pos_ptr, pos0, M, n_splits, KT, (float*)out, ldo);

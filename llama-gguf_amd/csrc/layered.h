@@ -89,7 +89,7 @@ hipError_t final_norm_rows_launch(const float* x, const int* rows, uint32_t n_ro
 // ---- latent_attention.hip ----
 struct LatentShape {
   uint32_t heads, dim, rot_dim, rot_n, vdim, rank;
-  uint32_t ldc;                // elements of a cache row: [latent rank | rotated key part rot_dim | zeros], multiple of 32
+  uint32_t ldc;                // elements of a cache row: [latent rank | rotated key part rot_dim | zeros], multiple of 64
   uint32_t dimp, rankp;        // row strides of the transposed key expansion [head][rank][dimp] and the value expansion [head * vdim][rankp]
   uint32_t off_q, off_dkv, off_g, ldcat;   // where a token's projections lie in its row of the fused product
   float scale, eps;
@@ -112,7 +112,7 @@ hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const i
 // merges the splits, expands the latent to the value and applies the head gate -> out [M][ldo] (f32 vector in decode, activations otherwise)
 hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32cache,
                              void* out, uint32_t ldo, bool out_f32, hipStream_t st);
-uint32_t latent_key_tile(const LatentShape& s, bool f32, uint32_t M);   // keys per tile of the absorbed kernel (0: does not fit LDS)
+bool latent_fits(const LatentShape& s, bool f32);   // the absorbed kernel's tiles fit LDS
 // expanded path (long prompts): keys and values per head
 struct LatentFlash {
   void* q;                     // [heads][Mcap][dq]
@@ -139,10 +139,11 @@ struct MlstmBufs {
   const float *bi, *bf;        // [heads]
   const float* norm;           // [heads * vdim]
   float* S;
-  double* m;                   // [3][heads]: the running maximum before position p lies in part p & 1; part 2: a block's start
+  double* m;                   // [2][heads]: the running maximum before position p lies in half p & 1
   float* num;                  // [M][heads][ldo]
-  double *u, *mx;              // prompt blocks: [heads][Mcap]
-  float* a;                    // prompt blocks: [chunk][heads][64][64] decayed scores
+  double *u, *mx;              // blocks: [heads][Mcap]
+  float *dec, *wgt, *cdec;     // blocks: factors of the state kernel, [heads][Mcap] and [heads][chunks]
+  float* a;                    // blocks: [chunk][heads][64][64] decayed scores
   uint32_t Mcap;
 };
 constexpr uint32_t kMlstmMaxDim = 1024;

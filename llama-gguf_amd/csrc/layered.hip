@@ -64,6 +64,7 @@ struct LayeredModel {
   uint32_t blk = 0;
   float *bx = nullptr, *by = nullptr, *bcat = nullptr, *bnum = nullptr, *ba = nullptr, *blogits = nullptr;
   double *bu = nullptr, *bmx = nullptr;
+  float *bdec = nullptr, *bwgt = nullptr, *bcdec = nullptr;
   void *bxa = nullptr, *bao = nullptr, *bact = nullptr, *bla = nullptr;
   int *btok = nullptr, *brows = nullptr;
   // expanded attention (grown with the context)
@@ -112,8 +113,8 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
       if (l.rot_dims && !(l.rot_base > 0.0)) { why = at + "rotation base"; return LGH_INVALID_ARGUMENT; }
       LatentShape s{};
       s.rank = l.kv_rank;
-      s.ldc = std::max(up(l.kv_rank + l.rot_dim, 32), up(l.kv_rank, 64));
-      if (l.heads > kLatAbsorbRows || !latent_key_tile(s, d.compute == LGH_COMPUTE_F32, 1)) { why = at + "latent rows too large for LDS"; return LGH_UNSUPPORTED; }
+      s.ldc = up(l.kv_rank + l.rot_dim, 64);
+      if (l.heads > kLatAbsorbRows || !latent_fits(s, d.compute == LGH_COMPUTE_F32)) { why = at + "latent rows too large for LDS"; return LGH_UNSUPPORTED; }
     } else if (l.mixer == LGH_MIXER_MLSTM) {
       if (!(l.gate_cap > 0.0)) { why = at + "gate_cap"; return LGH_INVALID_ARGUMENT; }
       if (l.dim > kMlstmMaxDim) { why = at + "matrix memory: dim above " + std::to_string(kMlstmMaxDim); return LGH_UNSUPPORTED; }
@@ -163,7 +164,7 @@ static void layered_plan(LayeredModel& m) {
     if (L.latent()) {
       LatentShape& s = L.ls;
       s.heads = l.heads; s.dim = l.dim; s.rot_dim = l.rot_dim; s.rot_n = l.rot_dims; s.vdim = l.vdim; s.rank = l.kv_rank;
-      s.ldc = std::max(up(l.kv_rank + l.rot_dim, 32), up(l.kv_rank, 64));   // (a whole row is also the input row of the expansions)
+      s.ldc = up(l.kv_rank + l.rot_dim, 64);   // (a whole row is also the input row of the expansions)
       s.dimp = up(l.dim, 8);
       s.rankp = up(l.kv_rank, 64);
       s.scale = (float)l.scale; s.eps = (float)d.norm_eps;
@@ -353,7 +354,7 @@ int layered_finalize(lgh_ctx* c) {
       max_rows = std::max(max_rows, L.ls.heads); max_rank = std::max(max_rank, L.ls.rank); max_ldc = std::max(max_ldc, L.ls.ldc);
     } else {
       if ((rc = zeroed(c, (void**)&L.S, (size_t)L.ms.heads * L.ms.dim * L.ms.lds * 4, &c->stats.kv_bytes))) return rc;
-      if ((rc = zeroed(c, (void**)&L.m, (size_t)3 * L.ms.heads * 8, &c->stats.kv_bytes))) return rc;
+      if ((rc = zeroed(c, (void**)&L.m, (size_t)2 * L.ms.heads * 8, &c->stats.kv_bytes))) return rc;
     }
   }
   uint32_t splits = (c->d.flags >> LGH_FLAG_ATTN_SPLITS_SHIFT) & 0xFFu;
@@ -393,7 +394,7 @@ static LatentBufs latent_bufs(const LayeredModel& m, const LayeredLayer& L, cons
 static MlstmBufs mlstm_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat, float* num) {
   MlstmBufs b{};
   b.cat = cat; b.bi = L.bi; b.bf = L.bf; b.norm = L.mnorm; b.S = L.S; b.m = L.m; b.num = num;
-  b.u = m.bu; b.mx = m.bmx; b.a = m.ba; b.Mcap = m.blk;
+  b.u = m.bu; b.mx = m.bmx; b.dec = m.bdec; b.wgt = m.bwgt; b.cdec = m.bcdec; b.a = m.ba; b.Mcap = m.blk;
   return b;
 }
 
@@ -495,6 +496,7 @@ static int block_ensure(lgh_ctx* c) {
       {(void**)&m.bx, B * d.width * 4}, {&m.bxa, B * up(d.width, 64) * el}, {(void**)&m.by, B * up(d.width, 4) * 4},
       {(void**)&m.bcat, B * m.max_cat * 4}, {&m.bao, B * m.max_ao * el}, {&m.bact, B * m.max_act * el},
       {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * B * 8}, {(void**)&m.bmx, heads * B * 8},
+      {(void**)&m.bdec, heads * B * 4}, {(void**)&m.bwgt, heads * B * 4}, {(void**)&m.bcdec, heads * chunks * 4},
       {(void**)&m.btok, B * 4}, {(void**)&m.brows, B * 4}, {&m.bla, (size_t)kLogitRows * up(d.width, 64) * el},
       {(void**)&m.blogits, (size_t)kLogitRows * up(d.vocab_size, 4) * 4},
   };

@@ -28,6 +28,21 @@ __global__ void __launch_bounds__(256) lin_mv_kernel(const LinMv a, uint32_t n_g
   __shared__ float red[2][4][kMvR];
   __shared__ float bred[16];
   const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const uint32_t kb0 = tid * 8;
+  // row r of group g: 8 consecutive rows, or 4 pairs (a gate row and the up row 16 below it)
+  auto row_of = [&](uint32_t g, int r) -> const uint16_t* {
+    uint32_t row;
+    if (a.paired) { const uint32_t p = g * 4 + (r & 3); row = (p >> 4) * 32 + (p & 15) + (r >> 2) * 16; }
+    else row = g * kMvR + r;
+    return a.w + (size_t)(row < a.n ? row : a.n - 1) * a.kp;
+  };
+  // the weight stream runs one step (8 rows x 16 bytes per lane) ahead of the arithmetic, across groups; its first step is requested
+  // before the input vector is prepared.  Lanes past the row's end re-read its first bytes (unconditional loads) and add nothing.
+  uint32_t g = blockIdx.x, kb = kb0;
+  const uint32_t kc0 = kb0 < a.kp ? kb0 : 0;
+  u32x4 nxt[kMvR];
+#pragma unroll
+  for (int r = 0; r < kMvR; r++) nxt[r] = ldg_nt128(row_of(g, r) + kc0);
   if (PRO == LP_COPY) {
     for (uint32_t i = tid; i < a.k; i += 256) xs[i] = a.x[i];
   } else if (PRO == LP_RESID || PRO == LP_HEAD) {
@@ -42,37 +57,56 @@ __global__ void __launch_bounds__(256) lin_mv_kernel(const LinMv a, uint32_t n_g
   } else {
     for (uint32_t h = wave; h < a.heads; h += 4) {
       const float* num = a.num + (size_t)h * a.ldo;
-      const float inv = 1.0f / (fmaxf(fabsf(num[a.vdim]), num[a.vdim + 1]) + 1e-6f);
-      float ss = 0.0f;
-      for (uint32_t j = lane; j < a.vdim; j += 64) { const float o = num[j] * inv; ss = __builtin_fmaf(o, o, ss); }
-      const float r = 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
-      for (uint32_t j = lane; j < a.vdim; j += 64) {
-        const uint32_t e = h * a.vdim + j;
-        xs[e] = num[j] * inv * r * a.nw[e] * sigmoid_f(a.gate[e]);
+      const float* nw = a.nw + h * a.vdim;
+      const float* gt = a.gate + h * a.vdim;
+      const float den = num[a.vdim], em = num[a.vdim + 1];
+      if (a.vdim <= 512) {   // everything a lane needs of the head requested at once
+        float v[8], w[8], z[8];
+#pragma unroll
+        for (int j = 0; j < 8; j++) {
+          const uint32_t e = lane + j * 64, ec = e < a.vdim ? e : 0;
+          v[j] = num[ec]; w[j] = nw[ec]; z[j] = gt[ec];
+          if (e >= a.vdim) v[j] = 0.0f;
+        }
+        const float inv = 1.0f / (fmaxf(fabsf(den), em) + 1e-6f);
+        float ss = 0.0f;
+#pragma unroll
+        for (int j = 0; j < 8; j++) { v[j] *= inv; ss = __builtin_fmaf(v[j], v[j], ss); }
+        const float r = 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+#pragma unroll
+        for (int j = 0; j < 8; j++) {
+          const uint32_t e = lane + j * 64;
+          if (e < a.vdim) xs[h * a.vdim + e] = v[j] * r * w[j] * sigmoid_f(z[j]);
+        }
+      } else {
+        const float inv = 1.0f / (fmaxf(fabsf(den), em) + 1e-6f);
+        float ss = 0.0f;
+        for (uint32_t j = lane; j < a.vdim; j += 64) { const float o = num[j] * inv; ss = __builtin_fmaf(o, o, ss); }
+        const float r = 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+        for (uint32_t j = lane; j < a.vdim; j += 64) xs[h * a.vdim + j] = num[j] * inv * r * nw[j] * sigmoid_f(gt[j]);
       }
     }
   }
   for (uint32_t i = a.k + tid; i < a.kp; i += 256) xs[i] = 0.0f;
   __syncthreads();
   uint32_t par = 0;
-  for (uint32_t g = blockIdx.x; g < n_groups; g += gridDim.x, par ^= 1) {
-    // rows of this group: 8 consecutive ones, or 4 pairs (a gate row and the up row 16 below it)
-    const uint16_t* wr[kMvR];
+  float acc[kMvR];
 #pragma unroll
-    for (int r = 0; r < kMvR; r++) {
-      uint32_t row;
-      if (a.paired) { const uint32_t p = g * 4 + (r & 3); row = (p >> 4) * 32 + (p & 15) + (r >> 2) * 16; }
-      else row = g * kMvR + r;
-      wr[r] = a.w + (size_t)(row < a.n ? row : a.n - 1) * a.kp;
+  for (int r = 0; r < kMvR; r++) acc[r] = 0.0f;
+  const uint32_t passes = (a.kp + 2047) / 2048;
+  uint32_t pass = 0;
+  while (g < n_groups) {
+    u32x4 w[kMvR];
+#pragma unroll
+    for (int r = 0; r < kMvR; r++) w[r] = nxt[r];
+    const bool last = pass + 1 == passes;
+    const uint32_t gn = last ? g + gridDim.x : g, kn = last ? kb0 : kb + 2048;
+    if (gn < n_groups) {
+      const uint32_t kc = kn < a.kp ? kn : 0;
+#pragma unroll
+      for (int r = 0; r < kMvR; r++) nxt[r] = ldg_nt128(row_of(gn, r) + kc);
     }
-    float acc[kMvR];
-#pragma unroll
-    for (int r = 0; r < kMvR; r++) acc[r] = 0.0f;
-#pragma unroll 2
-    for (uint32_t kb = tid * 8; kb < a.kp; kb += 2048) {
-      u32x4 w[kMvR];
-#pragma unroll
-      for (int r = 0; r < kMvR; r++) w[r] = ldg_nt128(wr[r] + kb);
+    if (kb < a.kp) {
       const f32x4 x0 = *reinterpret_cast<const f32x4*>(xs + kb), x1 = *reinterpret_cast<const f32x4*>(xs + kb + 4);
 #pragma unroll
       for (int r = 0; r < kMvR; r++) {
@@ -84,25 +118,34 @@ __global__ void __launch_bounds__(256) lin_mv_kernel(const LinMv a, uint32_t n_g
         acc[r] = s;
       }
     }
+    if (last) {
 #pragma unroll
-    for (int r = 0; r < kMvR; r++) {
-      const float t = wave_sum_to_lane63(acc[r]);
-      if (lane == 63) red[par][wave][r] = t;
-    }
-    __syncthreads();
-    if (!a.paired) {
-      if (tid < kMvR) {
-        const uint32_t row = g * kMvR + tid;
-        if (row < a.n) a.out[row] = (red[par][0][tid] + red[par][1][tid]) + (red[par][2][tid] + red[par][3][tid]);
+      for (int r = 0; r < kMvR; r++) {
+        const float t = wave_sum_to_lane63(acc[r]);
+        if (lane == 63) red[par][wave][r] = t;
+        acc[r] = 0.0f;
       }
-    } else if (tid < 4) {
-      const uint32_t p = g * 4 + tid;
-      if (p < a.n / 2) {
-        const float gt = (red[par][0][tid] + red[par][1][tid]) + (red[par][2][tid] + red[par][3][tid]);
-        const float up = (red[par][0][tid + 4] + red[par][1][tid + 4]) + (red[par][2][tid + 4] + red[par][3][tid + 4]);
-        a.out[p] = gelu_tanh_f(gt) * up;
+      __syncthreads();
+      if (!a.paired) {
+        if (tid < kMvR) {
+          const uint32_t row = g * kMvR + tid;
+          if (row < a.n) a.out[row] = (red[par][0][tid] + red[par][1][tid]) + (red[par][2][tid] + red[par][3][tid]);
+        }
+      } else if (tid < 4) {
+        const uint32_t p = g * 4 + tid;
+        if (p < a.n / 2) {
+          const float gt = (red[par][0][tid] + red[par][1][tid]) + (red[par][2][tid] + red[par][3][tid]);
+          const float up = (red[par][0][tid + 4] + red[par][1][tid + 4]) + (red[par][2][tid + 4] + red[par][3][tid + 4]);
+          a.out[p] = gelu_tanh_f(gt) * up;
+        }
       }
+      par ^= 1;
+      pass = 0;
+    } else {
+      pass++;
     }
+    g = gn;
+    kb = kn;
   }
 }
 
@@ -111,7 +154,7 @@ static hipError_t lin_mv_go(const LinMv& a, hipStream_t st) {
   static bool opted[64] = {};
   if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_mv_kernel<PRO>), 152 * 1024, opted); e != hipSuccess) return e;
   const uint32_t groups = (a.n + kMvR - 1) / kMvR;
-  const uint32_t grid = groups < 2048u ? groups : 2048u;
+  const uint32_t rounds = (groups + 1023) / 1024, grid = (groups + rounds - 1) / rounds;   // 4 workgroups per CU, equal shares
   hipLaunchKernelGGL(lin_mv_kernel<PRO>, dim3(grid), dim3(256), (size_t)a.kp * 4, st, a, groups);
   return hipGetLastError();
 }

@@ -20,21 +20,34 @@ __device__ __forceinline__ float gate_in(float z, float cap) { return cap * tanh
 __device__ __forceinline__ float log_sigmoid_f(float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
 
 // ------------------------------------------------------------------------------------------------
-// decode: one token.  A workgroup owns 32 columns of one head's state (8 lanes x 4 columns, 32 rows at a time).
+// decode: one token.  A workgroup owns 16 columns of one head's state (4 lanes x 4 columns, 64 rows at a time).
 // ------------------------------------------------------------------------------------------------
 __global__ void __launch_bounds__(256) mlstm_step_kernel(const MlstmShape s, const MlstmBufs b, const int* __restrict__ pos_ptr) {
-  __shared__ float o_s[32][33];
-  const uint32_t h = blockIdx.y, tid = threadIdx.x, c4 = blockIdx.x * 32 + (tid & 7) * 4, r0 = tid >> 3;
+  __shared__ float o_s[4][16];
+  const uint32_t h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, c4 = blockIdx.x * 16 + (tid & 3) * 4, r0 = tid >> 2;
   const uint32_t pos = (uint32_t)*pos_ptr;
+  const float* q = b.cat + s.off_q + (size_t)h * s.dim;
+  const float* k = b.cat + s.off_k + (size_t)h * s.dim;
+  const float* v = b.cat + s.off_v + (size_t)h * s.vdim;
+  float* S = b.S + (size_t)h * s.dim * s.lds + c4;
+  f32x4 st[4];
+  float kd[4], qd[4];
+  auto fetch = [&](uint32_t d0) {   // 4 x 64 rows (rows past the end re-read the last one and are dropped)
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      const uint32_t d = d0 + i * 64 + r0, dc = d < s.dim ? d : s.dim - 1;
+      st[i] = *reinterpret_cast<const f32x4*>(S + (size_t)dc * s.lds);
+      kd[i] = k[dc];
+      qd[i] = q[dc];
+    }
+  };
+  fetch(0);
   const float iv = gate_in(b.cat[s.off_i + h] + b.bi[h], s.cap);
   const float fv = log_sigmoid_f(gate_in(b.cat[s.off_f + h] + b.bf[h], s.cap));
   const double m0 = pos ? b.m[(pos & 1) * s.heads + h] : 0.0;
   const double m1 = fmax((double)fv + m0, (double)iv);
   const float fa = expf((float)((double)fv + m0 - m1)), fb = expf((float)((double)iv - m1));
   const float qs = 1.0f / __builtin_sqrtf((float)s.dim);
-  const float* q = b.cat + s.off_q + (size_t)h * s.dim;
-  const float* k = b.cat + s.off_k + (size_t)h * s.dim;
-  const float* v = b.cat + s.off_v + (size_t)h * s.vdim;
   float vv[4], o[4];
 #pragma unroll
   for (int e = 0; e < 4; e++) {
@@ -42,30 +55,31 @@ __global__ void __launch_bounds__(256) mlstm_step_kernel(const MlstmShape s, con
     vv[e] = fb * (c < s.vdim ? v[c] : c == s.vdim ? 1.0f : 0.0f);
     o[e] = 0.0f;
   }
-  if (c4 < s.lds) {
-    float* S = b.S + (size_t)h * s.dim * s.lds + c4;
-#pragma unroll 4
-    for (uint32_t d = r0; d < s.dim; d += 32) {
-      f32x4* at = reinterpret_cast<f32x4*>(S + (size_t)d * s.lds);
-      f32x4 st = (f32x4)(0.0f);
-      if (pos) st = *at;
-      const float kd = k[d], qd = q[d] * qs;
+  for (uint32_t d0 = 0; d0 < s.dim; d0 += 256) {
+    if (d0) fetch(d0);
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      const uint32_t d = d0 + i * 64 + r0;
+      if (d >= s.dim) continue;
+      f32x4 x;
 #pragma unroll
       for (int e = 0; e < 4; e++) {
-        st[e] = __builtin_fmaf(kd, vv[e], fa * st[e]);
-        o[e] = __builtin_fmaf(st[e], qd, o[e]);
+        x[e] = __builtin_fmaf(kd[i], vv[e], pos ? fa * st[i][e] : 0.0f);   // at position 0 whatever is stored belongs to another sequence
+        o[e] = __builtin_fmaf(x[e], qd[i], o[e]);
       }
-      *at = st;
+      *reinterpret_cast<f32x4*>(S + (size_t)d * s.lds) = x;
     }
   }
 #pragma unroll
-  for (int e = 0; e < 4; e++) o_s[r0][(tid & 7) * 4 + e] = o[e];
+  for (int e = 0; e < 4; e++) {   // the 16 row slots of a wave: lanes with equal lane & 3
+    o[e] *= qs;
+    o[e] += __shfl_xor(o[e], 4, 64); o[e] += __shfl_xor(o[e], 8, 64); o[e] += __shfl_xor(o[e], 16, 64); o[e] += __shfl_xor(o[e], 32, 64);
+    if (lane < 4) o_s[tid >> 6][lane * 4 + e] = o[e];
+  }
   __syncthreads();
-  if (tid < 32) {
-    const uint32_t c = blockIdx.x * 32 + tid;
-    float t = 0.0f;
-    for (int r = 0; r < 32; r++) t += o_s[r][tid];
-    if (c <= s.vdim) b.num[(size_t)h * s.ldo + c] = t;
+  if (tid < 16) {
+    const uint32_t c = blockIdx.x * 16 + tid;
+    if (c <= s.vdim) b.num[(size_t)h * s.ldo + c] = (o_s[0][tid] + o_s[1][tid]) + (o_s[2][tid] + o_s[3][tid]);
     if (c == 0) {
       b.m[((pos + 1) & 1) * s.heads + h] = m1;
       b.num[(size_t)h * s.ldo + s.vdim + 1] = expf((float)(-m1));
@@ -75,44 +89,62 @@ __global__ void __launch_bounds__(256) mlstm_step_kernel(const MlstmShape s, con
 
 hipError_t mlstm_step_launch(const MlstmShape& s, const MlstmBufs& b, const int* pos_ptr, hipStream_t st) {
   if (s.lds % 16 || s.lds < s.vdim + 1 || s.ldo < s.vdim + 2) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(mlstm_step_kernel, dim3((s.vdim + 1 + 31) / 32, s.heads), dim3(256), 0, st, s, b, pos_ptr);
+  hipLaunchKernelGGL(mlstm_step_kernel, dim3((s.vdim + 1 + 15) / 16, s.heads), dim3(256), 0, st, s, b, pos_ptr);
   return hipGetLastError();
 }
 
 // ------------------------------------------------------------------------------------------------
-// blocks of tokens: gates.  One wave per head, 64 tokens per step: a running sum (G) and a running maximum (M) across lanes.
+// blocks of tokens: gates.  One workgroup per head; a wave takes one chunk of 64 tokens at a time (16 chunks a round) and scans it from
+// the chunk's own start — a running sum (G) and a running maximum (of u) across lanes; the chunks' offsets then follow in order.
+// Besides u and M it leaves, as f32 factors for the state kernel: dec_t = exp(M_p - M_t) / sqrt(dim), wgt_t = exp(u_t - M_e) and each
+// chunk's exp(M_p - M_e) (p: the token before the chunk, e: its last token).
 // ------------------------------------------------------------------------------------------------
-__global__ void __launch_bounds__(64) mlstm_gates_kernel(const MlstmShape s, const MlstmBufs b, uint32_t pos0, uint32_t M) {
-  const uint32_t h = blockIdx.x, lane = threadIdx.x;
+__global__ void __launch_bounds__(1024) mlstm_gates_kernel(const MlstmShape s, const MlstmBufs b, uint32_t pos0, uint32_t M) {
+  __shared__ double tot[16], top[16], G0[17], M0[17];
+  const uint32_t h = blockIdx.x, lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const double m0 = pos0 ? b.m[(pos0 & 1) * s.heads + h] : 0.0;
-  double G = 0.0, Mx = m0, mt = m0;
   const float bi = b.bi[h], bf = b.bf[h];
-  for (uint32_t t0 = 0; t0 < M; t0 += 64) {
-    const uint32_t t = t0 + lane;
+  const float qs = 1.0f / __builtin_sqrtf((float)s.dim);
+  double G = 0.0, Mx = m0;
+  for (uint32_t base = 0; base < M; base += 1024) {
+    const uint32_t t = base + w * 64 + lane;
     const bool ok = t < M;
     const float* row = b.cat + (size_t)(ok ? t : M - 1) * s.ldcat;
     const double iv = (double)gate_in(row[s.off_i + h] + bi, s.cap);
     double f = ok ? (double)log_sigmoid_f(gate_in(row[s.off_f + h] + bf, s.cap)) : 0.0;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) { const double p = __shfl_up(f, o, 64); if ((int)lane >= o) f += p; }
-    const double Gt = G + f, u = iv - Gt;
-    double mx = ok ? u : -1e300;
+    const double ul = iv - f;                     // u up to the chunk's offset
+    double mx = ok ? ul : -1e300;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) { const double p = __shfl_up(mx, o, 64); if ((int)lane >= o) mx = fmax(mx, p); }
-    mx = fmax(mx, Mx);
-    if (ok) {
-      b.u[(size_t)h * b.Mcap + t] = u;
-      b.mx[(size_t)h * b.Mcap + t] = mx;
-      b.num[((size_t)t * s.heads + h) * s.ldo + s.vdim + 1] = expf((float)(-(Gt + mx)));
+    if (lane == 63) { tot[w] = f; top[w] = mx; }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+      double g = G, m = Mx;
+      for (int i = 0; i < 16; i++) {
+        G0[i] = g; M0[i] = m;
+        m = fmax(m, top[i] - g);
+        g += tot[i];
+      }
+      G0[16] = g; M0[16] = m;
     }
-    G = __shfl(Gt, 63, 64);
-    Mx = __shfl(mx, 63, 64);
-    mt = G + Mx;
+    __syncthreads();
+    const double g0 = G0[w], mp = M0[w], me = M0[w + 1];
+    const double u = ul - g0, mt = fmax(mp, mx - g0);
+    if (ok) {
+      const size_t at = (size_t)h * b.Mcap + t;
+      b.u[at] = u;
+      b.mx[at] = mt;
+      b.dec[at] = qs * expf((float)(mp - mt));
+      b.wgt[at] = expf((float)(u - me));
+      if (lane == 0) b.cdec[(size_t)h * ((b.Mcap + 63) / 64) + t / 64] = expf((float)(mp - me));
+      b.num[((size_t)t * s.heads + h) * s.ldo + s.vdim + 1] = expf((float)(-(g0 + f + mt)));
+    }
+    G = G0[16];
+    Mx = M0[16];
   }
-  if (lane == 0) {
-    b.m[((pos0 + M) & 1) * s.heads + h] = mt;   // (for an even M the half it was read from ...
-    b.m[2 * s.heads + h] = m0;                  // ... so the state kernel finds the old value here)
-  }
+  if (threadIdx.x == 0) b.m[((pos0 + M) & 1) * s.heads + h] = G + Mx;
 }
 
 // four consecutive values p[0..3] of which the first n exist (n may be <= 0)
@@ -166,21 +198,25 @@ __global__ void __launch_bounds__(256) mlstm_scores_kernel(const MlstmShape s, c
   }
 }
 
-// the recurrence over the chunks.  A workgroup owns 16 columns of one head's state: wave w the rows of dim quarter w, as matrix-core
+// the recurrence over the chunks.  A workgroup owns 16 columns of one head's state: wave w of NW the rows NT * 16 * w .., as matrix-core
 // accumulators (NT tiles of 16 rows).  A tile's register e of lane (column r16, group g) is row 4g + e — exactly what the j = e-th
-// f32 product wants as its B operand, so the state is multiplied where it lies.
-template <int NT>
-__global__ void __launch_bounds__(256) mlstm_state_kernel(const MlstmShape s, const MlstmBufs b, uint32_t pos0, uint32_t M) {
-  __shared__ f32x4 part[4][4][64];   // [wave][token tile][lane]
+// f32 product wants as its B operand, so the state is multiplied where it lies.  The workgroups are few (one per CU and less), so the
+// next chunk's operands are requested into registers while the current one is computed (PRE; large dims have no registers for it).
+template <int NT, int NW, bool PRE>
+__global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShape s, const MlstmBufs b, uint32_t pos0, uint32_t M) {
+  __shared__ f32x4 part[2][NW][4][64];   // [chunk parity][wave][token tile][lane]
   const uint32_t h = blockIdx.y, c0 = blockIdx.x * 16, lane = threadIdx.x & 63;
   const uint32_t w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
   const uint32_t r16 = lane & 15, g = lane >> 4, c = c0 + r16;
-  const bool vec = (s.dim & 3) == 0 && (s.ldcat & 3) == 0 && (s.off_q & 3) == 0;
-  const float qs = 1.0f / __builtin_sqrtf((float)s.dim);
+  const bool vec = (s.dim & 3) == 0;
   const uint32_t dbase = w * NT * 16;
-  const double* u = b.u + (size_t)h * b.Mcap;
-  const double* mx = b.mx + (size_t)h * b.Mcap;
+  const float* dec = b.dec + (size_t)h * b.Mcap;
+  const float* wgt = b.wgt + (size_t)h * b.Mcap;
+  const float* cdec = b.cdec + (size_t)h * ((b.Mcap + 63) / 64);
   float* Sg = b.S + (size_t)h * s.dim * s.lds;
+  const float* Q = b.cat + s.off_q + (size_t)h * s.dim;
+  const float* K = b.cat + s.off_k + (size_t)h * s.dim;
+  const float* V = b.cat + s.off_v + (size_t)h * s.vdim + (c < s.vdim ? c : 0);
   f32x4 S[NT];
 #pragma unroll
   for (int i = 0; i < NT; i++)
@@ -189,82 +225,101 @@ __global__ void __launch_bounds__(256) mlstm_state_kernel(const MlstmShape s, co
       const uint32_t d = dbase + i * 16 + g * 4 + e;
       S[i][e] = pos0 && d < s.dim && c <= s.vdim ? Sg[(size_t)d * s.lds + c] : 0.0f;
     }
-  double mp = b.m[2 * s.heads + h];
-  const uint32_t nch = (M + 63) / 64;
-  for (uint32_t ch = 0; ch < nch; ch++) {
-    const uint32_t t0 = ch * 64, te = (t0 + 63 < M ? t0 + 63 : M - 1);
-    const double me = mx[te];
-    // ---- numerators: the wave's share of S^T q (its dim quarter) and of A v (its 16 source tokens)
+  struct Ops { f32x4 q[NT][4]; f32x4 k[NT][4]; f32x4 v[4], wg[4], dc[4], a[4]; float cd; };
+  // a chunk's operands: q tiles (lane: token r16 of tile j, 4 dims), k (lane: dim r16, tokens 4g ..), v, factors, the wave's score columns.
+  // Rows and dims past the end are read clamped; their weight is 0 (tokens) or their state row is never stored (dims).
+  auto fetch = [&](uint32_t ch, Ops& x) {
+    const uint32_t t0 = ch * 64;
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+      const uint32_t t = t0 + j * 16 + r16, tc = t < M ? t : M - 1;
+      const float* qr = Q + (size_t)tc * s.ldcat;
+#pragma unroll
+      for (int i = 0; i < NT; i++) {
+        const uint32_t d = dbase + i * 16 + g * 4;
+        if (vec) {
+          x.q[i][j] = *reinterpret_cast<const f32x4*>(qr + (d < s.dim ? d : 0));
+          if (d >= s.dim) x.q[i][j] = (f32x4)(0.0f);
+        } else {
+          x.q[i][j] = load4(qr + d, (int)s.dim - (int)d, false);
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        const uint32_t ts = t0 + j * 16 + g * 4 + e, tsc = ts < M ? ts : M - 1;
+        const size_t ro = (size_t)tsc * s.ldcat;
+        x.v[j][e] = c < s.vdim ? V[ro] : c == s.vdim ? 1.0f : 0.0f;
+        x.wg[j][e] = ts < M ? wgt[tsc] : 0.0f;
+        x.dc[j][e] = dec[tsc];
+#pragma unroll
+        for (int i = 0; i < NT; i++) {
+          const uint32_t d = dbase + i * 16 + r16;
+          x.k[i][j][e] = K[ro + (d < s.dim ? d : s.dim - 1)];
+        }
+      }
+      x.a[j] = w >= 4 ? (f32x4)(0.0f) : *reinterpret_cast<const f32x4*>(b.a + ((size_t)ch * s.heads + h) * 4096 + (j * 16 + r16) * 64 + w * 16 + g * 4);
+    }
+    x.cd = cdec[ch];
+  };
+  auto chunk = [&](uint32_t ch, const Ops& x) {
+    const uint32_t t0 = ch * 64;
     f32x4 o[4];
 #pragma unroll
     for (int j = 0; j < 4; j++) o[j] = (f32x4)(0.0f);
+    // numerators: the wave's share of S^T q (its rows) and of A v (16 source tokens; the first four waves)
 #pragma unroll
-    for (int i = 0; i < NT; i++) {
-      const uint32_t d = dbase + i * 16 + g * 4;
+    for (int i = 0; i < NT; i++)
 #pragma unroll
-      for (int j = 0; j < 4; j++) {
-        const uint32_t t = t0 + j * 16 + r16;
-        const f32x4 qf = load4(b.cat + (size_t)(t < M ? t : M - 1) * s.ldcat + s.off_q + (size_t)h * s.dim + d, (int)s.dim - (int)d, vec);
-        o[j] = Frag<float>::mma(qf, S[i], o[j]);
-      }
-    }
-#pragma unroll
-    for (int j = 0; j < 4; j++)
-#pragma unroll
-      for (int e = 0; e < 4; e++) {
-        const uint32_t t = t0 + j * 16 + g * 4 + e;
-        o[j][e] *= qs * expf((float)(mp - (t < M ? mx[t] : me)));
-      }
-    f32x4 vf;                                                   // v of the wave's 16 tokens: lane column c, tokens 4g .. 4g + 3
+      for (int j = 0; j < 4; j++) o[j] = Frag<float>::mma(x.q[i][j], S[i], o[j]);
+    f32x4 vw;
 #pragma unroll
     for (int e = 0; e < 4; e++) {
+      const float v = w == 0 ? x.v[0][e] : w == 1 ? x.v[1][e] : w == 2 ? x.v[2][e] : x.v[3][e];
+      vw[e] = v;
+    }
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+      o[j] *= x.dc[j];
+      if (w < 4) o[j] = Frag<float>::mma(x.a[j], vw, o[j]);   // (scores of later keys are stored as zeros)
+      part[ch & 1][w][j][lane] = o[j];
+    }
+    // the state at the chunk's end
+#pragma unroll
+    for (int i = 0; i < NT; i++) S[i] *= x.cd;
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+      const f32x4 wv = x.v[j] * x.wg[j];
+#pragma unroll
+      for (int i = 0; i < NT; i++) S[i] = Frag<float>::mma(x.k[i][j], wv, S[i]);
+    }
+    __syncthreads();
+    if (w >= 4) return;
+    f32x4 t4 = (part[ch & 1][0][w][lane] + part[ch & 1][1][w][lane]) + (part[ch & 1][2][w][lane] + part[ch & 1][3][w][lane]);
+#pragma unroll
+    for (int k = 4; k < NW; k++) t4 += part[ch & 1][k][w][lane];
+#pragma unroll
+    for (int e = 0; e < 4; e++) {   // wave w finishes token tile w
       const uint32_t t = t0 + w * 16 + g * 4 + e;
-      vf[e] = t < M ? (c < s.vdim ? b.cat[(size_t)t * s.ldcat + s.off_v + (size_t)h * s.vdim + c] : c == s.vdim ? 1.0f : 0.0f) : 0.0f;
+      if (t < M && c <= s.vdim) b.num[((size_t)t * s.heads + h) * s.ldo + c] = t4[e];
     }
-    const float* A = b.a + ((size_t)ch * s.heads + h) * 4096;
-#pragma unroll
-    for (int j = 0; j < 4; j++)
-      if (j >= (int)w) o[j] = Frag<float>::mma(*reinterpret_cast<const f32x4*>(A + (j * 16 + r16) * 64 + w * 16 + g * 4), vf, o[j]);
-#pragma unroll
-    for (int j = 0; j < 4; j++) part[w][j][lane] = o[j];
-    // ---- the state at the chunk's end
-    const float decay = expf((float)(mp - me));
-#pragma unroll
-    for (int i = 0; i < NT; i++) S[i] *= decay;
-#pragma unroll
-    for (int sj = 0; sj < 4; sj++) {
-      if (t0 + sj * 16 >= M) break;
-      f32x4 wv;
-      uint32_t tt[4];
-#pragma unroll
-      for (int e = 0; e < 4; e++) {
-        const uint32_t t = t0 + sj * 16 + g * 4 + e;
-        tt[e] = t < M ? t : M - 1;
-        const float v = c < s.vdim ? b.cat[(size_t)tt[e] * s.ldcat + s.off_v + (size_t)h * s.vdim + c] : c == s.vdim ? 1.0f : 0.0f;
-        wv[e] = t < M ? v * expf((float)(u[t] - me)) : 0.0f;
-      }
-#pragma unroll
-      for (int i = 0; i < NT; i++) {
-        const uint32_t d = dbase + i * 16 + r16;
-        f32x4 kf = (f32x4)(0.0f);
-        if (d < s.dim) {
-#pragma unroll
-          for (int e = 0; e < 4; e++) kf[e] = b.cat[(size_t)tt[e] * s.ldcat + s.off_k + (size_t)h * s.dim + d];
-        }
-        S[i] = Frag<float>::mma(kf, wv, S[i]);
-      }
+  };
+  const uint32_t nch = (M + 63) / 64;
+  if constexpr (PRE) {
+    Ops x0, x1;
+    fetch(0, x0);
+    for (uint32_t ch = 0; ch < nch; ch += 2) {
+      fetch(ch + 1 < nch ? ch + 1 : ch, x1);
+      chunk(ch, x0);
+      if (ch + 1 >= nch) break;
+      fetch(ch + 2 < nch ? ch + 2 : ch + 1, x0);
+      chunk(ch + 1, x1);
     }
-    mp = me;
-    __syncthreads();
-    {  // add the four waves' shares; wave w finishes token tile w
-      const f32x4 t4 = (part[0][w][lane] + part[1][w][lane]) + (part[2][w][lane] + part[3][w][lane]);
-#pragma unroll
-      for (int e = 0; e < 4; e++) {
-        const uint32_t t = t0 + w * 16 + g * 4 + e;
-        if (t < M && c <= s.vdim) b.num[((size_t)t * s.heads + h) * s.ldo + c] = t4[e];
-      }
+  } else {
+    Ops x;
+    for (uint32_t ch = 0; ch < nch; ch++) {
+      fetch(ch, x);
+      chunk(ch, x);
     }
-    __syncthreads();
   }
 #pragma unroll
   for (int i = 0; i < NT; i++)
@@ -278,14 +333,16 @@ __global__ void __launch_bounds__(256) mlstm_state_kernel(const MlstmShape s, co
 hipError_t mlstm_block_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t pos0, uint32_t M, hipStream_t st) {
   if (M == 0 || M > b.Mcap || s.dim > kMlstmMaxDim || s.lds < s.vdim + 1 || s.ldo < s.vdim + 2) return hipErrorInvalidValue;
   const dim3 gs((s.vdim + 1 + 15) / 16, s.heads), t(256);
-  hipLaunchKernelGGL(mlstm_gates_kernel, dim3(s.heads), dim3(64), 0, st, s, b, pos0, M);
+  hipLaunchKernelGGL(mlstm_gates_kernel, dim3(s.heads), dim3(1024), 0, st, s, b, pos0, M);
   hipLaunchKernelGGL(mlstm_scores_kernel, dim3((M + 63) / 64, s.heads), t, 0, st, s, b, M);
   const uint32_t nt = (s.dim + 63) / 64;
-  if (nt <= 1) hipLaunchKernelGGL(mlstm_state_kernel<1>, gs, t, 0, st, s, b, pos0, M);
-  else if (nt <= 2) hipLaunchKernelGGL(mlstm_state_kernel<2>, gs, t, 0, st, s, b, pos0, M);
-  else if (nt <= 4) hipLaunchKernelGGL(mlstm_state_kernel<4>, gs, t, 0, st, s, b, pos0, M);
-  else if (nt <= 8) hipLaunchKernelGGL(mlstm_state_kernel<8>, gs, t, 0, st, s, b, pos0, M);
-  else hipLaunchKernelGGL(mlstm_state_kernel<16>, gs, t, 0, st, s, b, pos0, M);
+#define LGH_STATE(N, W, P) hipLaunchKernelGGL((mlstm_state_kernel<N, W, P>), gs, dim3(W * 64), 0, st, s, b, pos0, M)
+  if (nt <= 1) LGH_STATE(1, 4, true);
+  else if (nt <= 2) LGH_STATE(2, 4, true);
+  else if (nt <= 4) LGH_STATE(4, 4, true);
+  else if (nt <= 8) LGH_STATE(4, 8, false);
+  else LGH_STATE(8, 8, false);
+#undef LGH_STATE
   return hipGetLastError();
 }
 
