@@ -135,7 +135,7 @@ struct MlstmShape {
   float cap, eps;
 };
 struct MlstmBufs {
-  const float* cat;            // [M][ldcat]
+  const float* cat;            // [M][ldcat], blocks: + kMlstmRowSlack
   const float *bi, *bf;        // [heads]
   const float* norm;           // [heads * vdim]
   float* S;
@@ -146,8 +146,9 @@ struct MlstmBufs {
   float* a;                    // blocks: [chunk][heads][64][64] decayed scores
   uint32_t Mcap;
 };
-constexpr uint32_t kMlstmMaxDim = 1024;
-hipError_t mlstm_step_launch(const MlstmShape& s, const MlstmBufs& b, const int* pos_ptr, hipStream_t st);
+constexpr uint32_t kMlstmBlockDim = 512;      // larger heads take blocks token by token
+constexpr uint32_t kMlstmRowSlack = 2048;   // floats the block kernels may read behind the last row of cat (never used)
+hipError_t mlstm_step_launch(const MlstmShape& s, const MlstmBufs& b, const int* pos_ptr, hipStream_t st, uint32_t pos0 = 0);   // pos_ptr or pos0
 hipError_t mlstm_block_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t pos0, uint32_t M, hipStream_t st);
 hipError_t mlstm_out_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t M, void* out, uint32_t ldo, bool f32, hipStream_t st);
 

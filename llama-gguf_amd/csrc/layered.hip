@@ -117,7 +117,6 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
       if (l.heads > kLatAbsorbRows || !latent_fits(s, d.compute == LGH_COMPUTE_F32)) { why = at + "latent rows too large for LDS"; return LGH_UNSUPPORTED; }
     } else if (l.mixer == LGH_MIXER_MLSTM) {
       if (!(l.gate_cap > 0.0)) { why = at + "gate_cap"; return LGH_INVALID_ARGUMENT; }
-      if (l.dim > kMlstmMaxDim) { why = at + "matrix memory: dim above " + std::to_string(kMlstmMaxDim); return LGH_UNSUPPORTED; }
     } else { why = at + "unknown mixer"; return LGH_UNSUPPORTED; }
   }
   return LGH_OK;
@@ -394,7 +393,7 @@ static LatentBufs latent_bufs(const LayeredModel& m, const LayeredLayer& L, cons
 static MlstmBufs mlstm_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat, float* num) {
   MlstmBufs b{};
   b.cat = cat; b.bi = L.bi; b.bf = L.bf; b.norm = L.mnorm; b.S = L.S; b.m = L.m; b.num = num;
-  b.u = m.bu; b.mx = m.bmx; b.dec = m.bdec; b.wgt = m.bwgt; b.cdec = m.bcdec; b.a = m.ba; b.Mcap = m.blk;
+  b.u = m.bu; b.mx = m.bmx; b.dec = m.bdec; b.wgt = m.bwgt; b.cdec = m.bcdec; b.a = m.ba; b.Mcap = up(m.blk, 64);
   return b;
 }
 
@@ -491,12 +490,12 @@ static int block_ensure(lgh_ctx* c) {
   uint32_t heads = 0;
   for (auto& L : m.layers)
     if (!L.latent()) heads = std::max(heads, L.ms.heads);
-  const size_t B = m.blk, chunks = (B + 63) / 64, el = m.el();
+  const size_t B = m.blk, chunks = (B + 63) / 64, Bc = chunks * 64, el = m.el();
   struct { void** p; size_t n; } bufs[] = {
       {(void**)&m.bx, B * d.width * 4}, {&m.bxa, B * up(d.width, 64) * el}, {(void**)&m.by, B * up(d.width, 4) * 4},
-      {(void**)&m.bcat, B * m.max_cat * 4}, {&m.bao, B * m.max_ao * el}, {&m.bact, B * m.max_act * el},
-      {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * B * 8}, {(void**)&m.bmx, heads * B * 8},
-      {(void**)&m.bdec, heads * B * 4}, {(void**)&m.bwgt, heads * B * 4}, {(void**)&m.bcdec, heads * chunks * 4},
+      {(void**)&m.bcat, (B * m.max_cat + kMlstmRowSlack) * 4}, {&m.bao, B * m.max_ao * el}, {&m.bact, B * m.max_act * el},
+      {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * Bc * 8}, {(void**)&m.bmx, heads * Bc * 8},
+      {(void**)&m.bdec, heads * Bc * 4}, {(void**)&m.bwgt, heads * Bc * 4}, {(void**)&m.bcdec, heads * chunks * 4},
       {(void**)&m.btok, B * 4}, {(void**)&m.brows, B * 4}, {&m.bla, (size_t)kLogitRows * up(d.width, 64) * el},
       {(void**)&m.blogits, (size_t)kLogitRows * up(d.vocab_size, 4) * 4},
   };

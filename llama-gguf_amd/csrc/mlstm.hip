@@ -22,10 +22,10 @@ __device__ __forceinline__ float log_sigmoid_f(float z) { return fminf(z, 0.0f) 
 // ------------------------------------------------------------------------------------------------
 // decode: one token.  A workgroup owns 16 columns of one head's state (4 lanes x 4 columns, 64 rows at a time).
 // ------------------------------------------------------------------------------------------------
-__global__ void __launch_bounds__(256) mlstm_step_kernel(const MlstmShape s, const MlstmBufs b, const int* __restrict__ pos_ptr) {
+__global__ void __launch_bounds__(256) mlstm_step_kernel(const MlstmShape s, const MlstmBufs b, const int* __restrict__ pos_ptr, uint32_t pos0) {
   __shared__ float o_s[4][16];
   const uint32_t h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, c4 = blockIdx.x * 16 + (tid & 3) * 4, r0 = tid >> 2;
-  const uint32_t pos = (uint32_t)*pos_ptr;
+  const uint32_t pos = pos_ptr ? (uint32_t)*pos_ptr : pos0;
   const float* q = b.cat + s.off_q + (size_t)h * s.dim;
   const float* k = b.cat + s.off_k + (size_t)h * s.dim;
   const float* v = b.cat + s.off_v + (size_t)h * s.vdim;
@@ -87,9 +87,9 @@ __global__ void __launch_bounds__(256) mlstm_step_kernel(const MlstmShape s, con
   }
 }
 
-hipError_t mlstm_step_launch(const MlstmShape& s, const MlstmBufs& b, const int* pos_ptr, hipStream_t st) {
+hipError_t mlstm_step_launch(const MlstmShape& s, const MlstmBufs& b, const int* pos_ptr, hipStream_t st, uint32_t pos0) {
   if (s.lds % 16 || s.lds < s.vdim + 1 || s.ldo < s.vdim + 2) return hipErrorInvalidValue;
-  hipLaunchKernelGGL(mlstm_step_kernel, dim3((s.vdim + 1 + 15) / 16, s.heads), dim3(256), 0, st, s, b, pos_ptr);
+  hipLaunchKernelGGL(mlstm_step_kernel, dim3((s.vdim + 1 + 15) / 16, s.heads), dim3(256), 0, st, s, b, pos_ptr, pos0);
   return hipGetLastError();
 }
 
@@ -132,6 +132,7 @@ __global__ void __launch_bounds__(1024) mlstm_gates_kernel(const MlstmShape s, c
     __syncthreads();
     const double g0 = G0[w], mp = M0[w], me = M0[w + 1];
     const double u = ul - g0, mt = fmax(mp, mx - g0);
+    if (!ok && t < ((M + 63) & ~63u)) b.wgt[(size_t)h * b.Mcap + t] = 0.0f;   // the rest of the last chunk
     if (ok) {
       const size_t at = (size_t)h * b.Mcap + t;
       b.u[at] = u;
@@ -147,39 +148,47 @@ __global__ void __launch_bounds__(1024) mlstm_gates_kernel(const MlstmShape s, c
   if (threadIdx.x == 0) b.m[((pos0 + M) & 1) * s.heads + h] = G + Mx;
 }
 
-// four consecutive values p[0..3] of which the first n exist (n may be <= 0)
-__device__ __forceinline__ f32x4 load4(const float* p, int n, bool vec) {
-  if (vec && n >= 4) return *reinterpret_cast<const f32x4*>(p);
-  f32x4 r = (f32x4)(0.0f);
+// Loads of the block kernels are unconditional and masks are factors (a select with a loaded operand becomes a branch around the load,
+// which then waits for it): a head's last 16-wide tile may read on into the next head's or segment's values — the row buffer has room for
+// that behind its last row — and one side of every product is multiplied by 0 there.
+template <bool VEC>   // VEC: rows and heads start at multiples of 16 bytes
+__device__ __forceinline__ f32x4 row4(const float* base, uint32_t off) {
+  const char* p = reinterpret_cast<const char*>(base) + off * 4u;
+  if constexpr (VEC) return *reinterpret_cast<const f32x4*>(p);
+  f32x4 r;
 #pragma unroll
-  for (int e = 0; e < 4; e++)
-    if (e < n) r[e] = p[e];
+  for (int e = 0; e < 4; e++) r[e] = *reinterpret_cast<const float*>(p + 4 * e);
   return r;
+}
+__device__ __forceinline__ float row1(const float* base, uint32_t off) { return *reinterpret_cast<const float*>(reinterpret_cast<const char*>(base) + off * 4u); }
+// the four values at dims d .. d + 3 of a query, zero from dim on
+__device__ __forceinline__ f32x4 keep_dims(f32x4 v, uint32_t d, uint32_t dim) {
+#pragma unroll
+  for (int e = 0; e < 4; e++) v[e] *= d + e < dim ? 1.0f : 0.0f;
+  return v;
 }
 
 // decayed scores of a chunk: A[t][s] = exp(u_s - M_t) (q_t . k_s) / sqrt(dim) for s <= t, else 0
+template <bool VEC>
 __global__ void __launch_bounds__(256) mlstm_scores_kernel(const MlstmShape s, const MlstmBufs b, uint32_t M) {
   const uint32_t ch = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, g = lane >> 4;
   const uint32_t t0 = ch * 64;
-  const bool vec = (s.dim & 3) == 0 && (s.ldcat & 3) == 0 && (s.off_q & 3) == 0 && (s.off_k & 3) == 0;
   const float qs = 1.0f / __builtin_sqrtf((float)s.dim);
   const uint32_t tq = t0 + w * 16 + r16;
-  const float* qrow = b.cat + (size_t)(tq < M ? tq : M - 1) * s.ldcat + s.off_q + (size_t)h * s.dim;
-  const float* krow[4];
+  const uint32_t qo = (tq < M ? tq : M - 1) * s.ldcat + s.off_q + h * s.dim + g * 4;
+  uint32_t ko[4];
 #pragma unroll
   for (int j = 0; j < 4; j++) {
     const uint32_t tk = t0 + j * 16 + r16;
-    krow[j] = b.cat + (size_t)(tk < M ? tk : M - 1) * s.ldcat + s.off_k + (size_t)h * s.dim;
+    ko[j] = (tk < M ? tk : M - 1) * s.ldcat + s.off_k + h * s.dim + g * 4;
   }
   f32x4 acc[4];
 #pragma unroll
   for (int j = 0; j < 4; j++) acc[j] = (f32x4)(0.0f);
   for (uint32_t d = 0; d < s.dim; d += 16) {
-    const int n = (int)s.dim - (int)(d + g * 4);
-    const f32x4 qf = load4(qrow + d + g * 4, n, vec);
+    const f32x4 qf = keep_dims(row4<VEC>(b.cat, qo + d), d + g * 4, s.dim);
 #pragma unroll
-    for (int j = 0; j < 4; j++)
-      if (j <= (int)w) acc[j] = Frag<float>::mma(qf, load4(krow[j] + d + g * 4, n, vec), acc[j]);   // (wave-uniform: later keys are masked)
+    for (int j = 0; j < 4; j++) acc[j] = Frag<float>::mma(qf, row4<VEC>(b.cat, ko[j] + d), acc[j]);
   }
   float* A = b.a + ((size_t)ch * s.heads + h) * 4096;
   const double* u = b.u + (size_t)h * b.Mcap;
@@ -202,62 +211,50 @@ __global__ void __launch_bounds__(256) mlstm_scores_kernel(const MlstmShape s, c
 // accumulators (NT tiles of 16 rows).  A tile's register e of lane (column r16, group g) is row 4g + e — exactly what the j = e-th
 // f32 product wants as its B operand, so the state is multiplied where it lies.  The workgroups are few (one per CU and less), so the
 // next chunk's operands are requested into registers while the current one is computed (PRE; large dims have no registers for it).
-template <int NT, int NW, bool PRE>
+template <int NT, int NW, bool PRE, bool VEC>
 __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShape s, const MlstmBufs b, uint32_t pos0, uint32_t M) {
   __shared__ f32x4 part[2][NW][4][64];   // [chunk parity][wave][token tile][lane]
   const uint32_t h = blockIdx.y, c0 = blockIdx.x * 16, lane = threadIdx.x & 63;
   const uint32_t w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
   const uint32_t r16 = lane & 15, g = lane >> 4, c = c0 + r16;
-  const bool vec = (s.dim & 3) == 0;
   const uint32_t dbase = w * NT * 16;
   const float* dec = b.dec + (size_t)h * b.Mcap;
   const float* wgt = b.wgt + (size_t)h * b.Mcap;
   const float* cdec = b.cdec + (size_t)h * ((b.Mcap + 63) / 64);
   float* Sg = b.S + (size_t)h * s.dim * s.lds;
-  const float* Q = b.cat + s.off_q + (size_t)h * s.dim;
-  const float* K = b.cat + s.off_k + (size_t)h * s.dim;
-  const float* V = b.cat + s.off_v + (size_t)h * s.vdim + (c < s.vdim ? c : 0);
+  const uint32_t qo = s.off_q + h * s.dim + dbase + g * 4, ko = s.off_k + h * s.dim + dbase + r16, vo = s.off_v + h * s.vdim + (c < s.vdim ? c : 0);
+  const float vpad = c == s.vdim ? 1.0f : 0.0f, vmask = c < s.vdim ? 1.0f : 0.0f;
+  const bool ragged = s.dim != NT * NW * 16;   // rows past dim: never stored, kept 0
   f32x4 S[NT];
 #pragma unroll
   for (int i = 0; i < NT; i++)
 #pragma unroll
     for (int e = 0; e < 4; e++) {
       const uint32_t d = dbase + i * 16 + g * 4 + e;
-      S[i][e] = pos0 && d < s.dim && c <= s.vdim ? Sg[(size_t)d * s.lds + c] : 0.0f;
+      const bool ok = d < s.dim && c <= s.vdim;
+      const float v = Sg[ok ? (size_t)d * s.lds + c : 0];
+      S[i][e] = pos0 && ok ? v : 0.0f;
     }
   struct Ops { f32x4 q[NT][4]; f32x4 k[NT][4]; f32x4 v[4], wg[4], dc[4], a[4]; float cd; };
   // a chunk's operands: q tiles (lane: token r16 of tile j, 4 dims), k (lane: dim r16, tokens 4g ..), v, factors, the wave's score columns.
-  // Rows and dims past the end are read clamped; their weight is 0 (tokens) or their state row is never stored (dims).
+  // Tokens past the end re-read the last one: their weight is 0 and their numerators are not stored.
   auto fetch = [&](uint32_t ch, Ops& x) {
     const uint32_t t0 = ch * 64;
 #pragma unroll
     for (int j = 0; j < 4; j++) {
-      const uint32_t t = t0 + j * 16 + r16, tc = t < M ? t : M - 1;
-      const float* qr = Q + (size_t)tc * s.ldcat;
+      const uint32_t t = t0 + j * 16 + r16, ro = (t < M ? t : M - 1) * s.ldcat + qo;
 #pragma unroll
-      for (int i = 0; i < NT; i++) {
-        const uint32_t d = dbase + i * 16 + g * 4;
-        if (vec) {
-          x.q[i][j] = *reinterpret_cast<const f32x4*>(qr + (d < s.dim ? d : 0));
-          if (d >= s.dim) x.q[i][j] = (f32x4)(0.0f);
-        } else {
-          x.q[i][j] = load4(qr + d, (int)s.dim - (int)d, false);
-        }
-      }
+      for (int i = 0; i < NT; i++) x.q[i][j] = row4<VEC>(b.cat, ro + i * 16);
 #pragma unroll
       for (int e = 0; e < 4; e++) {
-        const uint32_t ts = t0 + j * 16 + g * 4 + e, tsc = ts < M ? ts : M - 1;
-        const size_t ro = (size_t)tsc * s.ldcat;
-        x.v[j][e] = c < s.vdim ? V[ro] : c == s.vdim ? 1.0f : 0.0f;
-        x.wg[j][e] = ts < M ? wgt[tsc] : 0.0f;
-        x.dc[j][e] = dec[tsc];
+        const uint32_t ts = t0 + j * 16 + g * 4 + e, tsc = ts < M ? ts : M - 1, so = tsc * s.ldcat;
+        x.v[j][e] = __builtin_fmaf(row1(b.cat, so + vo), vmask, vpad);
+        x.wg[j][e] = row1(wgt, ts);   // (0 behind the block's last token)
+        x.dc[j][e] = row1(dec, tsc);
 #pragma unroll
-        for (int i = 0; i < NT; i++) {
-          const uint32_t d = dbase + i * 16 + r16;
-          x.k[i][j][e] = K[ro + (d < s.dim ? d : s.dim - 1)];
-        }
+        for (int i = 0; i < NT; i++) x.k[i][j][e] = row1(b.cat, so + ko + i * 16);
       }
-      x.a[j] = w >= 4 ? (f32x4)(0.0f) : *reinterpret_cast<const f32x4*>(b.a + ((size_t)ch * s.heads + h) * 4096 + (j * 16 + r16) * 64 + w * 16 + g * 4);
+      x.a[j] = *reinterpret_cast<const f32x4*>(b.a + ((size_t)ch * s.heads + h) * 4096 + (j * 16 + r16) * 64 + (w & 3) * 16 + g * 4);
     }
     x.cd = cdec[ch];
   };
@@ -291,6 +288,12 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
       const f32x4 wv = x.v[j] * x.wg[j];
 #pragma unroll
       for (int i = 0; i < NT; i++) S[i] = Frag<float>::mma(x.k[i][j], wv, S[i]);
+    }
+    if (ragged) {
+#pragma unroll
+      for (int i = 0; i < NT; i++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) S[i][e] *= dbase + i * 16 + g * 4 + e < s.dim ? 1.0f : 0.0f;
     }
     __syncthreads();
     if (w >= 4) return;
@@ -331,17 +334,32 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
 }
 
 hipError_t mlstm_block_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t pos0, uint32_t M, hipStream_t st) {
-  if (M == 0 || M > b.Mcap || s.dim > kMlstmMaxDim || s.lds < s.vdim + 1 || s.ldo < s.vdim + 2) return hipErrorInvalidValue;
+  if (M == 0 || M > b.Mcap || b.Mcap % 64 || s.lds < s.vdim + 1 || s.ldo < s.vdim + 2) return hipErrorInvalidValue;
+  if (s.dim > kMlstmBlockDim) {   // a head's rows do not fit the block kernel's registers: the recurrence itself, token by token
+    for (uint32_t t = 0; t < M; t++) {
+      MlstmBufs r = b;
+      r.cat += (size_t)t * s.ldcat;
+      r.num += (size_t)t * s.heads * s.ldo;
+      if (hipError_t e = mlstm_step_launch(s, r, nullptr, st, pos0 + t); e != hipSuccess) return e;
+    }
+    return hipSuccess;
+  }
   const dim3 gs((s.vdim + 1 + 15) / 16, s.heads), t(256);
   hipLaunchKernelGGL(mlstm_gates_kernel, dim3(s.heads), dim3(1024), 0, st, s, b, pos0, M);
-  hipLaunchKernelGGL(mlstm_scores_kernel, dim3((M + 63) / 64, s.heads), t, 0, st, s, b, M);
+  const bool vec = (s.dim & 3) == 0 && (s.ldcat & 3) == 0 && (s.off_q & 3) == 0 && (s.off_k & 3) == 0;
+  const dim3 gq((M + 63) / 64, s.heads);
+  if (vec) hipLaunchKernelGGL(mlstm_scores_kernel<true>, gq, t, 0, st, s, b, M);
+  else hipLaunchKernelGGL(mlstm_scores_kernel<false>, gq, t, 0, st, s, b, M);
   const uint32_t nt = (s.dim + 63) / 64;
-#define LGH_STATE(N, W, P) hipLaunchKernelGGL((mlstm_state_kernel<N, W, P>), gs, dim3(W * 64), 0, st, s, b, pos0, M)
+#define LGH_STATE(N, W, P)                                                                                      \
+  do {                                                                                                          \
+    if (vec) hipLaunchKernelGGL((mlstm_state_kernel<N, W, P, true>), gs, dim3(W * 64), 0, st, s, b, pos0, M);   \
+    else hipLaunchKernelGGL((mlstm_state_kernel<N, W, P, false>), gs, dim3(W * 64), 0, st, s, b, pos0, M);      \
+  } while (0)
   if (nt <= 1) LGH_STATE(1, 4, true);
   else if (nt <= 2) LGH_STATE(2, 4, true);
   else if (nt <= 4) LGH_STATE(4, 4, true);
-  else if (nt <= 8) LGH_STATE(4, 8, false);
-  else LGH_STATE(8, 8, false);
+  else LGH_STATE(4, 8, false);
 #undef LGH_STATE
   return hipGetLastError();
 }
