@@ -143,6 +143,7 @@ struct MlstmBufs {
   float* num;                  // [M][heads][ldo]
   double *u, *mx;              // blocks: [heads][Mcap]
   float *dec, *wgt, *cdec;     // blocks: factors of the state kernel, [heads][Mcap] and [heads][chunks]
+  float* nk;                   // blocks: [chunk][heads][dim]: a chunk's contribution to n, then n before the chunk
   float* a;                    // blocks: [chunk][heads][64][64] decayed scores
   uint32_t Mcap;
 };

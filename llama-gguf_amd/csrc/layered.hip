@@ -64,7 +64,7 @@ struct LayeredModel {
   uint32_t blk = 0;
   float *bx = nullptr, *by = nullptr, *bcat = nullptr, *bnum = nullptr, *ba = nullptr, *blogits = nullptr;
   double *bu = nullptr, *bmx = nullptr;
-  float *bdec = nullptr, *bwgt = nullptr, *bcdec = nullptr;
+  float *bdec = nullptr, *bwgt = nullptr, *bcdec = nullptr, *bnk = nullptr;
   void *bxa = nullptr, *bao = nullptr, *bact = nullptr, *bla = nullptr;
   int *btok = nullptr, *brows = nullptr;
   // expanded attention (grown with the context)
@@ -393,7 +393,7 @@ static LatentBufs latent_bufs(const LayeredModel& m, const LayeredLayer& L, cons
 static MlstmBufs mlstm_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat, float* num) {
   MlstmBufs b{};
   b.cat = cat; b.bi = L.bi; b.bf = L.bf; b.norm = L.mnorm; b.S = L.S; b.m = L.m; b.num = num;
-  b.u = m.bu; b.mx = m.bmx; b.dec = m.bdec; b.wgt = m.bwgt; b.cdec = m.bcdec; b.a = m.ba; b.Mcap = up(m.blk, 64);
+  b.u = m.bu; b.mx = m.bmx; b.dec = m.bdec; b.wgt = m.bwgt; b.cdec = m.bcdec; b.a = m.ba; b.nk = m.bnk; b.Mcap = up(m.blk, 64);
   return b;
 }
 
@@ -487,15 +487,15 @@ static int block_ensure(lgh_ctx* c) {
   if (m.blk_ready) return LGH_OK;
   const lgh_layered_desc& d = m.d;
   m.blk = std::min(kBlockTokens, d.max_seq_len);
-  uint32_t heads = 0;
+  uint32_t heads = 0, hdim = 0;
   for (auto& L : m.layers)
-    if (!L.latent()) heads = std::max(heads, L.ms.heads);
+    if (!L.latent()) { heads = std::max(heads, L.ms.heads); hdim = std::max(hdim, L.ms.heads * L.ms.dim); }
   const size_t B = m.blk, chunks = (B + 63) / 64, Bc = chunks * 64, el = m.el();
   struct { void** p; size_t n; } bufs[] = {
       {(void**)&m.bx, B * d.width * 4}, {&m.bxa, B * up(d.width, 64) * el}, {(void**)&m.by, B * up(d.width, 4) * 4},
       {(void**)&m.bcat, (B * m.max_cat + kMlstmRowSlack) * 4}, {&m.bao, B * m.max_ao * el}, {&m.bact, B * m.max_act * el},
       {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * Bc * 8}, {(void**)&m.bmx, heads * Bc * 8},
-      {(void**)&m.bdec, heads * Bc * 4}, {(void**)&m.bwgt, heads * Bc * 4}, {(void**)&m.bcdec, heads * chunks * 4},
+      {(void**)&m.bdec, heads * Bc * 4}, {(void**)&m.bwgt, heads * Bc * 4}, {(void**)&m.bcdec, heads * chunks * 4}, {(void**)&m.bnk, chunks * hdim * 4},
       {(void**)&m.btok, B * 4}, {(void**)&m.brows, B * 4}, {&m.bla, (size_t)kLogitRows * up(d.width, 64) * el},
       {(void**)&m.blogits, (size_t)kLogitRows * up(d.vocab_size, 4) * 4},
   };

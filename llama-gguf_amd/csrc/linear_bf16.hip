@@ -6,56 +6,81 @@
 namespace lgh {
 
 // ------------------------------------------------------------------------------------------------
-// decode mat-vec: a workgroup of 4 waves owns 8 rows at a time; the waves share a row's columns (2048 per pass), every lane keeps
-// 8 rows x 16 bytes in flight.
+// decode mat-vec: one workgroup of 16 waves per CU, so that preparing the input vector (layer norm, read-out) costs a CU once.  A team
+// of `ks` waves takes 4 rows at a time and shares their columns; every lane keeps two passes of 4 rows x 16 bytes in flight, across row
+// groups, and the first of them are requested before the input vector is prepared.
 // ------------------------------------------------------------------------------------------------
-constexpr int kMvR = 8;
+constexpr int kMvR = 4;
+constexpr uint32_t kMvThreads = 1024;
 
 // layer norm of the K values in xs (in place), times w
 __device__ __forceinline__ void ln_lds(float* xs, uint32_t K, const float* w, float eps, float* red) {
   float s = 0.0f;
-  for (uint32_t i = threadIdx.x; i < K; i += 256) s += xs[i];
+  for (uint32_t i = threadIdx.x; i < K; i += kMvThreads) s += xs[i];
   const float mean = block_sum(s, red) / (float)K;
   float v = 0.0f;
-  for (uint32_t i = threadIdx.x; i < K; i += 256) { const float d = xs[i] - mean; v = __builtin_fmaf(d, d, v); }
+  for (uint32_t i = threadIdx.x; i < K; i += kMvThreads) { const float d = xs[i] - mean; v = __builtin_fmaf(d, d, v); }
   const float inv = 1.0f / __builtin_sqrtf(block_sum(v, red) / (float)K + eps);
-  for (uint32_t i = threadIdx.x; i < K; i += 256) xs[i] = (xs[i] - mean) * inv * w[i];
+  for (uint32_t i = threadIdx.x; i < K; i += kMvThreads) xs[i] = (xs[i] - mean) * inv * w[i];
 }
 
-template <int PRO>
-__global__ void __launch_bounds__(256) lin_mv_kernel(const LinMv a, uint32_t n_groups) {
-  extern __shared__ __attribute__((aligned(16))) float xs[];   // [kp]
-  __shared__ float red[2][4][kMvR];
-  __shared__ float bred[16];
-  const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const uint32_t kb0 = tid * 8;
-  // row r of group g: 8 consecutive rows, or 4 pairs (a gate row and the up row 16 below it)
-  auto row_of = [&](uint32_t g, int r) -> const uint16_t* {
-    uint32_t row;
-    if (a.paired) { const uint32_t p = g * 4 + (r & 3); row = (p >> 4) * 32 + (p & 15) + (r >> 2) * 16; }
-    else row = g * kMvR + r;
-    return a.w + (size_t)(row < a.n ? row : a.n - 1) * a.kp;
-  };
-  // the weight stream runs one step (8 rows x 16 bytes per lane) ahead of the arithmetic, across groups; its first step is requested
-  // before the input vector is prepared.  Lanes past the row's end re-read its first bytes (unconditional loads) and add nothing.
-  uint32_t g = blockIdx.x, kb = kb0;
-  const uint32_t kc0 = kb0 < a.kp ? kb0 : 0;
-  u32x4 nxt[kMvR];
+// row r of group g: 4 consecutive rows, or 2 pairs (a gate row and the up row 16 below it)
+__device__ __forceinline__ const uint16_t* mv_row(const LinMv& a, uint32_t g, int r) {
+  uint32_t row;
+  if (a.paired) { const uint32_t p = g * 2 + (r & 1); row = (p >> 4) * 32 + (p & 15) + (r >> 1) * 16; }
+  else row = g * kMvR + r;
+  return a.w + (size_t)(row < a.n ? row : a.n - 1) * a.kp;
+}
+struct MvW { u32x4 w[kMvR]; };
+// lanes past the row's end re-read its first bytes (unconditional loads) and add nothing
+__device__ __forceinline__ void mv_fetch(const LinMv& a, uint32_t g, uint32_t kb, MvW& o) {
+  const uint32_t kc = kb < a.kp ? kb : 0;
 #pragma unroll
-  for (int r = 0; r < kMvR; r++) nxt[r] = ldg_nt128(row_of(g, r) + kc0);
+  for (int r = 0; r < kMvR; r++) o.w[r] = ldg_nt128(mv_row(a, g, r) + kc);
+}
+__device__ __forceinline__ void mv_acc(const MvW& o, f32x4 x0, f32x4 x1, float* acc) {
+#pragma unroll
+  for (int r = 0; r < kMvR; r++) {
+    const u32x4 w = o.w[r];
+    float s = acc[r];
+    s = __builtin_fmaf(bf_lo(w.x), x0.x, s); s = __builtin_fmaf(bf_hi(w.x), x0.y, s);
+    s = __builtin_fmaf(bf_lo(w.y), x0.z, s); s = __builtin_fmaf(bf_hi(w.y), x0.w, s);
+    s = __builtin_fmaf(bf_lo(w.z), x1.x, s); s = __builtin_fmaf(bf_hi(w.z), x1.y, s);
+    s = __builtin_fmaf(bf_lo(w.w), x1.z, s); s = __builtin_fmaf(bf_hi(w.w), x1.w, s);
+    acc[r] = s;
+  }
+}
+template <int PRO>
+__global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint32_t n_groups, uint32_t ks) {
+  extern __shared__ __attribute__((aligned(16))) float xs[];   // [kp]
+  __shared__ float red[2][16][kMvR];
+  __shared__ float bred[16];
+  const uint32_t tid = threadIdx.x, lane = tid & 63, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
+  const uint32_t team = wave / ks, sub = wave % ks, teams = 16 / ks;
+  const uint32_t kb0 = (sub * 64 + lane) * 8, kstep = ks * 512, passes = (a.kp + kstep - 1) / kstep;
+  const uint32_t gstep = gridDim.x * teams;
+  uint32_t g = blockIdx.x + gridDim.x * team;
+  uint32_t gf = g, pf = 0;   // the next pass to request
+  MvW n0, n1;
+  auto request = [&](MvW& o) {
+    if (gf < n_groups) mv_fetch(a, gf, kb0 + pf * kstep, o);
+    if (++pf == passes) { pf = 0; gf += gstep; }
+  };
+  request(n0);
+  request(n1);
   if (PRO == LP_COPY) {
-    for (uint32_t i = tid; i < a.k; i += 256) xs[i] = a.x[i];
+    for (uint32_t i = tid; i < a.k; i += kMvThreads) xs[i] = a.x[i];
   } else if (PRO == LP_RESID || PRO == LP_HEAD) {
-    for (uint32_t i = tid; i < a.k; i += 256) xs[i] = a.y[i];
+    for (uint32_t i = tid; i < a.k; i += kMvThreads) xs[i] = a.y[i];
     ln_lds(xs, a.k, a.nw, a.eps, bred);
-    for (uint32_t i = tid; i < a.k; i += 256) {
+    for (uint32_t i = tid; i < a.k; i += kMvThreads) {
       const float v = a.x[i] + a.mult * xs[i];
       xs[i] = v;
       if (blockIdx.x == 0) a.xout[i] = v;
     }
     if (PRO == LP_HEAD) ln_lds(xs, a.k, a.nw2, a.eps, bred);
   } else {
-    for (uint32_t h = wave; h < a.heads; h += 4) {
+    for (uint32_t h = wave; h < a.heads; h += 16) {
       const float* num = a.num + (size_t)h * a.ldo;
       const float* nw = a.nw + h * a.vdim;
       const float* gt = a.gate + h * a.vdim;
@@ -87,65 +112,45 @@ __global__ void __launch_bounds__(256) lin_mv_kernel(const LinMv a, uint32_t n_g
       }
     }
   }
-  for (uint32_t i = a.k + tid; i < a.kp; i += 256) xs[i] = 0.0f;
+  for (uint32_t i = a.k + tid; i < a.kp; i += kMvThreads) xs[i] = 0.0f;
   __syncthreads();
-  uint32_t par = 0;
-  float acc[kMvR];
-#pragma unroll
-  for (int r = 0; r < kMvR; r++) acc[r] = 0.0f;
-  const uint32_t passes = (a.kp + 2047) / 2048;
-  uint32_t pass = 0;
-  while (g < n_groups) {
-    u32x4 w[kMvR];
-#pragma unroll
-    for (int r = 0; r < kMvR; r++) w[r] = nxt[r];
-    const bool last = pass + 1 == passes;
-    const uint32_t gn = last ? g + gridDim.x : g, kn = last ? kb0 : kb + 2048;
-    if (gn < n_groups) {
-      const uint32_t kc = kn < a.kp ? kn : 0;
-#pragma unroll
-      for (int r = 0; r < kMvR; r++) nxt[r] = ldg_nt128(row_of(gn, r) + kc);
-    }
-    if (kb < a.kp) {
-      const f32x4 x0 = *reinterpret_cast<const f32x4*>(xs + kb), x1 = *reinterpret_cast<const f32x4*>(xs + kb + 4);
-#pragma unroll
-      for (int r = 0; r < kMvR; r++) {
-        float s = acc[r];
-        s = __builtin_fmaf(bf_lo(w[r].x), x0.x, s); s = __builtin_fmaf(bf_hi(w[r].x), x0.y, s);
-        s = __builtin_fmaf(bf_lo(w[r].y), x0.z, s); s = __builtin_fmaf(bf_hi(w[r].y), x0.w, s);
-        s = __builtin_fmaf(bf_lo(w[r].z), x1.x, s); s = __builtin_fmaf(bf_hi(w[r].z), x1.y, s);
-        s = __builtin_fmaf(bf_lo(w[r].w), x1.z, s); s = __builtin_fmaf(bf_hi(w[r].w), x1.w, s);
-        acc[r] = s;
+  const uint32_t rounds = (n_groups + gstep - 1) / gstep;   // the same for every wave: the teams meet at a barrier when ks > 1
+  for (uint32_t rd = 0; rd < rounds; rd++, g += gstep) {
+    float acc[kMvR] = {0.0f, 0.0f, 0.0f, 0.0f};
+    if (g < n_groups) {
+      for (uint32_t p = 0; p < passes; p++) {
+        const MvW cur = n0;
+        n0 = n1;
+        request(n1);
+        const uint32_t kb = kb0 + p * kstep;
+        if (kb < a.kp) mv_acc(cur, *reinterpret_cast<const f32x4*>(xs + kb), *reinterpret_cast<const f32x4*>(xs + kb + 4), acc);
       }
-    }
-    if (last) {
 #pragma unroll
-      for (int r = 0; r < kMvR; r++) {
-        const float t = wave_sum_to_lane63(acc[r]);
-        if (lane == 63) red[par][wave][r] = t;
-        acc[r] = 0.0f;
+      for (int r = 0; r < kMvR; r++) acc[r] = wave_sum_to_lane63(acc[r]);
+    }
+    if (ks > 1) {
+      if (lane == 63) {
+#pragma unroll
+        for (int r = 0; r < kMvR; r++) red[rd & 1][wave][r] = acc[r];
       }
       __syncthreads();
-      if (!a.paired) {
-        if (tid < kMvR) {
-          const uint32_t row = g * kMvR + tid;
-          if (row < a.n) a.out[row] = (red[par][0][tid] + red[par][1][tid]) + (red[par][2][tid] + red[par][3][tid]);
-        }
-      } else if (tid < 4) {
-        const uint32_t p = g * 4 + tid;
-        if (p < a.n / 2) {
-          const float gt = (red[par][0][tid] + red[par][1][tid]) + (red[par][2][tid] + red[par][3][tid]);
-          const float up = (red[par][0][tid + 4] + red[par][1][tid + 4]) + (red[par][2][tid + 4] + red[par][3][tid + 4]);
-          a.out[p] = gelu_tanh_f(gt) * up;
-        }
+      if (sub == 0 && lane == 63) {
+#pragma unroll
+        for (int r = 0; r < kMvR; r++)
+          for (uint32_t k = 1; k < ks; k++) acc[r] += red[rd & 1][wave + k][r];
       }
-      par ^= 1;
-      pass = 0;
-    } else {
-      pass++;
     }
-    g = gn;
-    kb = kn;
+    if (sub == 0 && lane == 63 && g < n_groups) {
+      if (!a.paired) {
+#pragma unroll
+        for (int r = 0; r < kMvR; r++)
+          if (g * kMvR + r < a.n) a.out[g * kMvR + r] = acc[r];
+      } else {
+#pragma unroll
+        for (int r = 0; r < 2; r++)
+          if (g * 2 + r < a.n / 2) a.out[g * 2 + r] = gelu_tanh_f(acc[r]) * acc[r + 2];
+      }
+    }
   }
 }
 
@@ -154,8 +159,10 @@ static hipError_t lin_mv_go(const LinMv& a, hipStream_t st) {
   static bool opted[64] = {};
   if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_mv_kernel<PRO>), 152 * 1024, opted); e != hipSuccess) return e;
   const uint32_t groups = (a.n + kMvR - 1) / kMvR;
-  const uint32_t rounds = (groups + 1023) / 1024, grid = (groups + rounds - 1) / rounds;   // 4 workgroups per CU, equal shares
-  hipLaunchKernelGGL(lin_mv_kernel<PRO>, dim3(grid), dim3(256), (size_t)a.kp * 4, st, a, groups);
+  uint32_t ks = 1;   // waves per team: enough teams for the groups of a CU, and at least a full pass of columns per wave
+  while (ks < 8 && (uint64_t)groups * ks * 2 <= kNumCU * 16 && a.kp >= 1024 * ks) ks *= 2;
+  const uint32_t teams = 16 / ks, want = (groups + teams - 1) / teams;
+  hipLaunchKernelGGL(lin_mv_kernel<PRO>, dim3(want < kNumCU ? want : kNumCU), dim3(kMvThreads), (size_t)a.kp * 4, st, a, groups, ks);
   return hipGetLastError();
 }
 

@@ -3,7 +3,8 @@
 // With log forget gates f_t, log input gates i_t and the running maximum m_t = max(f_t + m_(t-1), i_t):
 //   S_t = exp(f_t + m_(t-1) - m_t) S_(t-1) + exp(i_t - m_t) k_t v_t^T,   n_t the same with k_t alone,
 //   o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6).
-// n is kept as one more column of S (a value of constant 1), so a state is [head][dim][vdim + 1].
+// n is kept as one more column of S (a value of constant 1), so a state is [head][dim][vdim + 1]; the block kernels take it apart (the
+// state kernel's workgroups are one per CU at common sizes, a 16-column tile of n alone would be a second round).
 //
 // Blocks of tokens use the recurrence's closed form.  With G_t = f_1 + .. + f_t (from the block's start), u_s = i_s - G_s and
 // M_t = max(m_0, max_(s<=t) u_s):  m_t = G_t + M_t, the weight of token s in S_t is exp(u_s - M_t) and that of the state before the
@@ -139,7 +140,7 @@ __global__ void __launch_bounds__(1024) mlstm_gates_kernel(const MlstmShape s, c
       b.mx[at] = mt;
       b.dec[at] = qs * expf((float)(mp - mt));
       b.wgt[at] = expf((float)(u - me));
-      if (lane == 0) b.cdec[(size_t)h * ((b.Mcap + 63) / 64) + t / 64] = expf((float)(mp - me));
+      if (lane == 0) b.cdec[(size_t)h * (b.Mcap / 64) + t / 64] = expf((float)(mp - me));
       b.num[((size_t)t * s.heads + h) * s.ldo + s.vdim + 1] = expf((float)(-(g0 + f + mt)));
     }
     G = G0[16];
@@ -190,6 +191,16 @@ __global__ void __launch_bounds__(256) mlstm_scores_kernel(const MlstmShape s, c
 #pragma unroll
     for (int j = 0; j < 4; j++) acc[j] = Frag<float>::mma(qf, row4<VEC>(b.cat, ko[j] + d), acc[j]);
   }
+  {  // the chunk's contribution to n: sum_s exp(u_s - M_e) k_s
+    const uint32_t rows = M - t0 < 64 ? M - t0 : 64;
+    const float* wg = b.wgt + (size_t)h * b.Mcap + t0;
+    for (uint32_t d = threadIdx.x; d < s.dim; d += 256) {
+      float n = 0.0f;
+#pragma unroll 8
+      for (uint32_t r = 0; r < rows; r++) n = __builtin_fmaf(wg[r], row1(b.cat, (t0 + r) * s.ldcat + s.off_k + h * s.dim + d), n);
+      b.nk[((size_t)ch * s.heads + h) * s.dim + d] = n;
+    }
+  }
   float* A = b.a + ((size_t)ch * s.heads + h) * 4096;
   const double* u = b.u + (size_t)h * b.Mcap;
   const double* mx = b.mx + (size_t)h * b.Mcap;
@@ -207,6 +218,31 @@ __global__ void __launch_bounds__(256) mlstm_scores_kernel(const MlstmShape s, c
   }
 }
 
+// n before every chunk (in place of the chunks' contributions) and after the last
+__global__ void __launch_bounds__(256) mlstm_n_kernel(const MlstmShape s, const MlstmBufs b, uint32_t pos0, uint32_t M) {
+  const uint32_t h = blockIdx.y, d = blockIdx.x * 256 + threadIdx.x, nch = (M + 63) / 64;
+  if (d >= s.dim) return;
+  float* Sn = b.S + ((size_t)h * s.dim + d) * s.lds + s.vdim;
+  const float* cdec = b.cdec + (size_t)h * (b.Mcap / 64);
+  float n = pos0 ? *Sn : 0.0f;
+  for (uint32_t c0 = 0; c0 < nch; c0 += 8) {
+    float k[8], f[8];
+#pragma unroll
+    for (uint32_t i = 0; i < 8; i++) {
+      const uint32_t ch = c0 + i < nch ? c0 + i : nch - 1;
+      k[i] = b.nk[((size_t)ch * s.heads + h) * s.dim + d];
+      f[i] = cdec[ch];
+    }
+#pragma unroll
+    for (uint32_t i = 0; i < 8; i++)
+      if (c0 + i < nch) {
+        b.nk[((size_t)(c0 + i) * s.heads + h) * s.dim + d] = n;
+        n = __builtin_fmaf(f[i], n, k[i]);
+      }
+  }
+  *Sn = n;
+}
+
 // the recurrence over the chunks.  A workgroup owns 16 columns of one head's state: wave w of NW the rows NT * 16 * w .., as matrix-core
 // accumulators (NT tiles of 16 rows).  A tile's register e of lane (column r16, group g) is row 4g + e — exactly what the j = e-th
 // f32 product wants as its B operand, so the state is multiplied where it lies.  The workgroups are few (one per CU and less), so the
@@ -220,10 +256,9 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
   const uint32_t dbase = w * NT * 16;
   const float* dec = b.dec + (size_t)h * b.Mcap;
   const float* wgt = b.wgt + (size_t)h * b.Mcap;
-  const float* cdec = b.cdec + (size_t)h * ((b.Mcap + 63) / 64);
+  const float* cdec = b.cdec + (size_t)h * (b.Mcap / 64);
   float* Sg = b.S + (size_t)h * s.dim * s.lds;
   const uint32_t qo = s.off_q + h * s.dim + dbase + g * 4, ko = s.off_k + h * s.dim + dbase + r16, vo = s.off_v + h * s.vdim + (c < s.vdim ? c : 0);
-  const float vpad = c == s.vdim ? 1.0f : 0.0f, vmask = c < s.vdim ? 1.0f : 0.0f;
   const bool ragged = s.dim != NT * NW * 16;   // rows past dim: never stored, kept 0
   f32x4 S[NT];
 #pragma unroll
@@ -231,7 +266,7 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
 #pragma unroll
     for (int e = 0; e < 4; e++) {
       const uint32_t d = dbase + i * 16 + g * 4 + e;
-      const bool ok = d < s.dim && c <= s.vdim;
+      const bool ok = d < s.dim && c < s.vdim;
       const float v = Sg[ok ? (size_t)d * s.lds + c : 0];
       S[i][e] = pos0 && ok ? v : 0.0f;
     }
@@ -248,7 +283,7 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
 #pragma unroll
       for (int e = 0; e < 4; e++) {
         const uint32_t ts = t0 + j * 16 + g * 4 + e, tsc = ts < M ? ts : M - 1, so = tsc * s.ldcat;
-        x.v[j][e] = __builtin_fmaf(row1(b.cat, so + vo), vmask, vpad);
+        x.v[j][e] = row1(b.cat, so + vo);   // (columns past vdim: computed, never stored)
         x.wg[j][e] = row1(wgt, ts);   // (0 behind the block's last token)
         x.dc[j][e] = row1(dec, tsc);
 #pragma unroll
@@ -303,7 +338,7 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
 #pragma unroll
     for (int e = 0; e < 4; e++) {   // wave w finishes token tile w
       const uint32_t t = t0 + w * 16 + g * 4 + e;
-      if (t < M && c <= s.vdim) b.num[((size_t)t * s.heads + h) * s.ldo + c] = t4[e];
+      if (t < M && c < s.vdim) b.num[((size_t)t * s.heads + h) * s.ldo + c] = t4[e];
     }
   };
   const uint32_t nch = (M + 63) / 64;
@@ -329,7 +364,7 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
 #pragma unroll
     for (int e = 0; e < 4; e++) {
       const uint32_t d = dbase + i * 16 + g * 4 + e;
-      if (d < s.dim && c <= s.vdim) Sg[(size_t)d * s.lds + c] = S[i][e];
+      if (d < s.dim && c < s.vdim) Sg[(size_t)d * s.lds + c] = S[i][e];
     }
 }
 
@@ -344,12 +379,13 @@ hipError_t mlstm_block_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t 
     }
     return hipSuccess;
   }
-  const dim3 gs((s.vdim + 1 + 15) / 16, s.heads), t(256);
+  const dim3 gs((s.vdim + 15) / 16, s.heads), t(256);
   hipLaunchKernelGGL(mlstm_gates_kernel, dim3(s.heads), dim3(1024), 0, st, s, b, pos0, M);
   const bool vec = (s.dim & 3) == 0 && (s.ldcat & 3) == 0 && (s.off_q & 3) == 0 && (s.off_k & 3) == 0;
   const dim3 gq((M + 63) / 64, s.heads);
   if (vec) hipLaunchKernelGGL(mlstm_scores_kernel<true>, gq, t, 0, st, s, b, M);
   else hipLaunchKernelGGL(mlstm_scores_kernel<false>, gq, t, 0, st, s, b, M);
+  hipLaunchKernelGGL(mlstm_n_kernel, dim3((s.dim + 255) / 256, s.heads), t, 0, st, s, b, pos0, M);
   const uint32_t nt = (s.dim + 63) / 64;
 #define LGH_STATE(N, W, P)                                                                                      \
   do {                                                                                                          \
@@ -372,7 +408,18 @@ __global__ void __launch_bounds__(256) mlstm_out_kernel(const MlstmShape s, cons
   const uint32_t t = blockIdx.x, lane = threadIdx.x & 63;
   for (uint32_t h = threadIdx.x >> 6; h < s.heads; h += 4) {
     const float* num = b.num + ((size_t)t * s.heads + h) * s.ldo;
-    const float inv = 1.0f / (fmaxf(fabsf(num[s.vdim]), num[s.vdim + 1]) + 1e-6f);
+    float den;
+    if (s.dim > kMlstmBlockDim) {
+      den = num[s.vdim];
+    } else {   // n . q = exp(M_p - M_t) n_p . q + the row sum of the decayed scores
+      const size_t chh = (size_t)(t / 64) * s.heads + h;
+      const float* q = b.cat + (size_t)t * s.ldcat + s.off_q + (size_t)h * s.dim;
+      const float* n = b.nk + chh * s.dim;
+      float dot = 0.0f;
+      for (uint32_t d = lane; d < s.dim; d += 64) dot = __builtin_fmaf(q[d], n[d], dot);
+      den = wave_sum(__builtin_fmaf(dot, b.dec[(size_t)h * b.Mcap + t], b.a[chh * 4096 + (t & 63) * 64 + lane]));
+    }
+    const float inv = 1.0f / (fmaxf(fabsf(den), num[s.vdim + 1]) + 1e-6f);
     float ss = 0.0f;
     for (uint32_t j = lane; j < s.vdim; j += 64) { const float o = num[j] * inv; ss = __builtin_fmaf(o, o, ss); }
     const float r = 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)s.vdim + s.eps);
