@@ -11,7 +11,7 @@
 
 namespace lgh {
 
-constexpr float kNegHuge = -1e30f;
+constexpr float kNegHuge = -1e30f, kLog2e = 1.4426950408889634f;
 
 // token t of a block -> rotated pair i of src
 __device__ __forceinline__ void rot_pair(const float* src, const float* cs, uint32_t i, float& a, float& b) {
@@ -161,6 +161,9 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
     lim[e] = p0 + (r < rows ? r : rows - 1) / s.heads + 1;      // keys this row sees
     m[e] = kNegHuge; l[e] = 0.0f;
   }
+  // bf16: scores in units of log2 (one v_exp per weight); f32: natural, with the library exponential
+  const float scl = sizeof(T) == 2 ? s.scale * kLog2e : s.scale;
+  auto ex = [](float x) { return sizeof(T) == 2 ? __builtin_amdgcn_exp2f(x) : expf(x); };
   f32x4 o[NCT];
 #pragma unroll
   for (int i = 0; i < NCT; i++) o[i] = (f32x4)(0.0f);
@@ -177,12 +180,19 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
       const T* qa = Qs + r16 * ld;
       const T* kb = tile + ((w & 1) * 16 + r16) * ld;
       uint32_t u = half;
-      for (; u + 2 <= u1; u += 2) {
-        const uint32_t c0 = ((u * 4 + g) ^ (r16 & 7)) * PER, c1 = ((u * 4 + 4 + g) ^ (r16 & 7)) * PER;
-        sc = Frag<T>::mma(Frag<T>::load(qa + c0), Frag<T>::load(kb + c0), sc);
-        sd = Frag<T>::mma(Frag<T>::load(qa + c1), Frag<T>::load(kb + c1), sd);
+      for (; u + 3 <= u1; u += 3) {   // three units' fragments requested together, two accumulation chains
+        typename Frag<T>::V qf[3], kf[3];
+#pragma unroll
+        for (int i = 0; i < 3; i++) {
+          const uint32_t c = (((u + i) * 4 + g) ^ (r16 & 7)) * PER;
+          qf[i] = Frag<T>::load(qa + c);
+          kf[i] = Frag<T>::load(kb + c);
+        }
+        sc = Frag<T>::mma(qf[0], kf[0], sc);
+        sd = Frag<T>::mma(qf[1], kf[1], sd);
+        sc = Frag<T>::mma(qf[2], kf[2], sc);
       }
-      if (u < u1) {
+      for (; u < u1; u++) {
         const uint32_t c0 = ((u * 4 + g) ^ (r16 & 7)) * PER;
         sc = Frag<T>::mma(Frag<T>::load(qa + c0), Frag<T>::load(kb + c0), sc);
       }
@@ -199,7 +209,7 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
 #pragma unroll
       for (int j = 0; j < 2; j++) {
         const uint32_t key = r16 + j * 16, at = (g * 4 + e) * LS + key;
-        sv[j] = k0 + key < lim[e] ? (Ss[at] + Ss[16 * LS + at]) * s.scale : kNegHuge;
+        sv[j] = k0 + key < lim[e] ? (Ss[at] + Ss[16 * LS + at]) * scl : kNegHuge;
         mx = fmaxf(mx, sv[j]);
       }
       mx = fmaxf(mx, dpp_f<0xB1>(mx)); mx = fmaxf(mx, dpp_f<0x4E>(mx)); mx = fmaxf(mx, dpp_f<0x141>(mx)); mx = fmaxf(mx, dpp_f<0x140>(mx));
@@ -207,12 +217,12 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
 #pragma unroll
       for (int j = 0; j < 2; j++) {
         const uint32_t key = r16 + j * 16;
-        const float p = k0 + key < lim[e] ? expf(sv[j] - mx) : 0.0f;
+        const float p = k0 + key < lim[e] ? ex(sv[j] - mx) : 0.0f;
         sum += p;
         if (w == 0) Ps[(g * 4 + e) * LP + key] = to_act<T>(p);
       }
       sum += dpp_f<0xB1>(sum); sum += dpp_f<0x4E>(sum); sum += dpp_f<0x141>(sum); sum += dpp_f<0x140>(sum);
-      alpha[e] = expf(m[e] - mx);
+      alpha[e] = ex(m[e] - mx);
       l[e] = l[e] * alpha[e] + sum;
       m[e] = mx;
     }
@@ -242,7 +252,7 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
     const uint32_t r = row0 + g * 4 + e;
     if (r >= rows) continue;
     const size_t pr = (size_t)sp * rows + r;
-    if (w == 0 && r16 == 0 && blockIdx.z == 0) { b.part_ml[pr * 2] = m[e]; b.part_ml[pr * 2 + 1] = l[e]; }
+    if (w == 0 && r16 == 0 && blockIdx.z == 0) { b.part_ml[pr * 2] = sizeof(T) == 2 ? m[e] * (1.0f / kLog2e) : m[e]; b.part_ml[pr * 2 + 1] = l[e]; }
 #pragma unroll
     for (int i = 0; i < NCT; i++) {
       const uint32_t c = wc + i * 16 + r16;
@@ -289,66 +299,79 @@ hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const i
 }
 
 // ------------------------------------------------------------------------------------------------
-// merge + value expansion + head gate: grid (chunks of 32 value rows, token * heads)
+// merge + value expansion + head gate: grid (chunks of 32 value rows, token * heads).  The value rows and the first partial sums are
+// requested before the merge weights are known: the kernel is a handful of memory round trips long.
 // ------------------------------------------------------------------------------------------------
+constexpr int kOutB = 16;   // partial sums in flight per thread
+
 template <class O>
-__global__ void __launch_bounds__(256) latent_out_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M,
-                                                         uint32_t n_splits, uint32_t KT, O* __restrict__ out, uint32_t ldo) {
+__global__ void __launch_bounds__(512) latent_out_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M,
+                                                         uint32_t n_splits, O* __restrict__ out, uint32_t ldo) {
   extern __shared__ __attribute__((aligned(16))) float lat[];   // [rankp], with room for the merge's thread groups
   __shared__ float wgt[kLatMaxSplits];
   const uint32_t tid = threadIdx.x, r = blockIdx.y, t = r / s.heads, h = r % s.heads, rows = M * s.heads;
   const uint32_t kv = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + M;
-  const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles + n_splits - 1) / n_splits, act = (tiles + per - 1) / per;
+  const uint32_t tiles = (kv + kLatKeys - 1) / kLatKeys, per = (tiles + n_splits - 1) / n_splits, act = (tiles + per - 1) / per;
   const uint32_t lane = tid & 63, w = tid >> 6;
-  u32x4 wv0[8];   // the wave's 8 value rows, first 512 columns: requested before the merge
+  const float mi = lane < act ? b.part_ml[((size_t)lane * rows + r) * 2] : kNegHuge;
+  const float li = lane < act ? b.part_ml[((size_t)lane * rows + r) * 2 + 1] : 0.0f;
+  u32x4 wv0[4];   // the wave's 4 value rows, first 512 columns
 #pragma unroll
-  for (int it = 0; it < 8; it++) {
-    const uint32_t v = blockIdx.x * 32 + it * 4 + w, vc = v < s.vdim ? v : s.vdim - 1, k = lane * 8 < s.rankp ? lane * 8 : 0;
+  for (int it = 0; it < 4; it++) {
+    const uint32_t v = blockIdx.x * 32 + it * 8 + w, vc = v < s.vdim ? v : s.vdim - 1, k = lane * 8 < s.rankp ? lane * 8 : 0;
     wv0[it] = *reinterpret_cast<const u32x4*>(b.uv + ((size_t)h * s.vdim + vc) * s.rankp + k);
   }
-  if (tid < 64) {
-    const float mi = tid < act ? b.part_ml[((size_t)tid * rows + r) * 2] : kNegHuge;
-    const float li = tid < act ? b.part_ml[((size_t)tid * rows + r) * 2 + 1] : 0.0f;
-    const float mm = wave_max(mi), f = expf(mi - mm), tot = wave_sum(f * li);
-    wgt[tid] = f / tot;
-  }
-  __syncthreads();
-  if ((s.rank & 3) == 0) {   // 4 columns per thread, the splits dealt to as many thread groups as there are threads for
-    const uint32_t quads = s.rankp / 4, groups = quads < 256 ? 256 / quads : 1, grp = tid / quads;
-    f32x4* acc4 = reinterpret_cast<f32x4*>(lat);   // [groups][quads]
-    for (uint32_t q = quads < 256 ? tid % quads : tid; q < quads && grp < groups; q += 256) {
-      f32x4 v = (f32x4)(0.0f);
-      if (q * 4 < s.rank) {
-        const float* src = b.part_acc + (size_t)r * s.rank + q * 4;
-#pragma unroll 8
-        for (uint32_t sp = grp; sp < act; sp += groups) {
-          const f32x4 x = *reinterpret_cast<const f32x4*>(src + (size_t)sp * rows * s.rank);
-          const float wg = wgt[sp];
+  // 4 columns per thread, the splits dealt to as many thread groups as there are threads for
+  const uint32_t quads = s.rankp / 4, groups = quads < 512 ? 512 / quads : 1, grp = tid / quads < groups ? tid / quads : 0;
+  const bool vec = (s.rank & 3) == 0;
+  auto fetch = [&](uint32_t sp, uint32_t q) -> f32x4 {   // clamped: the loads are unconditional
+    const float* src = b.part_acc + ((size_t)(sp < act ? sp : act - 1) * rows + r) * s.rank;
+    if (vec) return *reinterpret_cast<const f32x4*>(src + (q * 4 < s.rank ? q * 4 : 0));
+    f32x4 v;
 #pragma unroll
-          for (int e = 0; e < 4; e++) v[e] = __builtin_fmaf(wg, x[e], v[e]);
-        }
-      }
-      acc4[grp * quads + q] = v;
-    }
-    __syncthreads();
-    for (uint32_t q = tid; q < quads; q += 256) {
-      f32x4 v = acc4[q];
-      for (uint32_t k = 1; k < groups; k++) v += acc4[k * quads + q];
-      acc4[q] = v;
-    }
-  } else {
-    for (uint32_t i = tid; i < s.rankp; i += 256) {
-      float v = 0.0f;
-      if (i < s.rank)
-        for (uint32_t sp = 0; sp < act; sp++) v = __builtin_fmaf(wgt[sp], b.part_acc[((size_t)sp * rows + r) * s.rank + i], v);
-      lat[i] = v;
-    }
+    for (uint32_t e = 0; e < 4; e++) v[e] = src[q * 4 + e < s.rank ? q * 4 + e : 0];
+    return v;
+  };
+  f32x4 first[kOutB];
+  const uint32_t q0 = quads < 512 ? tid % quads : tid;
+#pragma unroll
+  for (int i = 0; i < kOutB; i++) first[i] = fetch(grp + i * groups, q0 < quads ? q0 : 0);
+  {
+    const float mm = wave_max(mi), f = expf(mi - mm), tot = wave_sum(f * li);
+    if (w == 0) wgt[lane] = f / tot;   // (inactive splits: 0)
   }
   __syncthreads();
+  f32x4* acc4 = reinterpret_cast<f32x4*>(lat);   // [groups][quads]
+  for (uint32_t q = q0; q < quads && tid / quads < groups; q += 512) {
+    f32x4 v = (f32x4)(0.0f);
+    for (uint32_t sp = grp; sp < act; sp += groups * kOutB) {
+#pragma unroll
+      for (int i = 0; i < kOutB; i++) {
+        const uint32_t k = sp + i * groups;
+        const f32x4 x = q == q0 && sp == grp ? first[i] : fetch(k, q);
+        const float wg = k < act ? wgt[k] : 0.0f;
+#pragma unroll
+        for (int e = 0; e < 4; e++) v[e] = __builtin_fmaf(wg, x[e], v[e]);
+      }
+    }
+#pragma unroll
+    for (uint32_t e = 0; e < 4; e++)
+      if (q * 4 + e >= s.rank) v[e] = 0.0f;
+    acc4[grp * quads + q] = v;
+  }
+  __syncthreads();
+  if (groups > 1) {
+    f32x4 v = (f32x4)(0.0f);
+    if (tid < quads)
+      for (uint32_t k = 0; k < groups; k++) v += acc4[k * quads + tid];
+    __syncthreads();
+    if (tid < quads) acc4[tid] = v;
+    __syncthreads();
+  }
   const float gate = sigmoid_f(b.cat[(size_t)t * s.ldcat + s.off_g + h]);
 #pragma unroll
-  for (int it = 0; it < 8; it++) {
-    const uint32_t v = blockIdx.x * 32 + it * 4 + w;
+  for (int it = 0; it < 4; it++) {
+    const uint32_t v = blockIdx.x * 32 + it * 8 + w;
     if (v >= s.vdim) continue;
     const uint16_t* W = b.uv + ((size_t)h * s.vdim + v) * s.rankp;
     float acc = 0.0f;
@@ -365,14 +388,12 @@ __global__ void __launch_bounds__(256) latent_out_kernel(const LatentShape s, co
   }
 }
 
-hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32cache,
-                             void* out, uint32_t ldo, bool out_f32, hipStream_t st) {
-  constexpr uint32_t KT = kLatKeys;
+hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, void* out, uint32_t ldo, bool out_f32, hipStream_t st) {
   if (s.rankp % 8 || n_splits == 0 || n_splits > kLatMaxSplits) return hipErrorInvalidValue;
-  const dim3 grid((s.vdim + 31) / 32, M * s.heads);
-  const size_t lds = (size_t)(s.rankp < 1024 ? 1024 : s.rankp) * 4;
-  if (out_f32) hipLaunchKernelGGL(latent_out_kernel<float>, grid, dim3(256), lds, st, s, b, pos_ptr, pos0, M, n_splits, KT, (float*)out, ldo);
-  else hipLaunchKernelGGL(latent_out_kernel<__bf16>, grid, dim3(256), lds, st, s, b, pos_ptr, pos0, M, n_splits, KT, (__bf16*)out, ldo);
+  const dim3 grid((s.vdim + 31) / 32, M * s.heads), th(512);
+  const size_t lds = (size_t)(s.rankp < 2048 ? 2048 : s.rankp) * 4;
+  if (out_f32) hipLaunchKernelGGL(latent_out_kernel<float>, grid, th, lds, st, s, b, pos_ptr, pos0, M, n_splits, (float*)out, ldo);
+  else hipLaunchKernelGGL(latent_out_kernel<__bf16>, grid, th, lds, st, s, b, pos_ptr, pos0, M, n_splits, (__bf16*)out, ldo);
   return hipGetLastError();
 }
 
@@ -480,7 +501,7 @@ __global__ void __launch_bounds__(256) latent_flash_kernel(const LatentShape s, 
     for (int i = 0; i < ND; i++) o[i][t] = (f32x4)(0.0f);
   }
   // bf16: scores in units of log2 (one v_exp per weight); f32: natural, with the library exponential
-  const float sc = BF ? s.scale * 1.4426950408889634f : s.scale;
+  const float sc = BF ? s.scale * kLog2e : s.scale;
   __builtin_amdgcn_s_waitcnt(0x0F70);   // vmcnt(0)
   __syncthreads();
   for (uint32_t tl = 0; tl < tiles; tl++) {

@@ -110,8 +110,7 @@ hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const i
 hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32,
                               hipStream_t st);
 // merges the splits, expands the latent to the value and applies the head gate -> out [M][ldo] (f32 vector in decode, activations otherwise)
-hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32cache,
-                             void* out, uint32_t ldo, bool out_f32, hipStream_t st);
+hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, void* out, uint32_t ldo, bool out_f32, hipStream_t st);
 bool latent_fits(const LatentShape& s, bool f32);   // the absorbed kernel's tiles fit LDS
 // expanded path (long prompts): keys and values per head
 struct LatentFlash {

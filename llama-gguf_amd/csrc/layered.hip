@@ -434,7 +434,7 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, (uint64_t)L.ls.heads * L.ls.rank * L.ls.dim * 2, [&] { return latent_prep_launch(L.ls, b, pos, 0, 1, m.f32, st); }))) return rc;
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, mixer_bytes(c, L), [&] { return latent_attn_launch(L.ls, b, pos, 0, 1, m.n_splits, m.f32, st); }))) return rc;
       if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_LATENT, L.uv.bytes(), [&] {
-             return latent_out_launch(L.ls, b, pos, 0, 1, m.n_splits, m.f32, m.ao, 0, true, st);
+             return latent_out_launch(L.ls, b, pos, 0, 1, m.n_splits, m.ao, 0, true, st);
            })))
         return rc;
       LinMv a{};
@@ -560,7 +560,7 @@ static int block_latent(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) 
     if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, 0, [&] { return latent_prep_launch(L.ls, b, nullptr, p, n, m.f32, st); }))) return rc;
     if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, 0, [&] { return latent_attn_launch(L.ls, b, nullptr, p, n, splits, m.f32, st); }))) return rc;
     if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_LATENT, 0, [&] {
-           return latent_out_launch(L.ls, b, nullptr, p, n, splits, m.f32, (uint8_t*)m.bao + (size_t)t * L.out.kp * m.el(), L.out.kp, m.f32, st);
+           return latent_out_launch(L.ls, b, nullptr, p, n, splits, (uint8_t*)m.bao + (size_t)t * L.out.kp * m.el(), L.out.kp, m.f32, st);
          })))
       return rc;
   }
