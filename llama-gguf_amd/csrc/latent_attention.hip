@@ -91,29 +91,30 @@ hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const i
 
 // ------------------------------------------------------------------------------------------------
 // absorbed attention.  A workgroup = 16 (token, head) rows x one split of the keys x up to 512 latent columns of the output; 32 keys
-// at a time go to LDS by DMA (16-byte chunks of a row stored at chunk ^ (row & 7)).  Scores: wave w multiplies the 16 rows with keys
-// 16 (w & 1) .. over half w >> 1 of the row; weighted sums: wave w owns a quarter of the columns and takes the values straight from
+// at a time go to LDS by DMA (16-byte chunks of a row stored at chunk ^ (row & 7)).  Everything transposed, as in the expanded kernel
+// below: S^T = C Q^T leaves a lane with one row's scores of 8 keys, which is the B operand of O^T = C^T P^T.  Every wave forms all the
+// scores (cheaper than exchanging them: one barrier per tile) and owns a quarter of the columns, whose values it takes straight from
 // the key tile (the latent IS the value), transposed on the way out of LDS.
 // ------------------------------------------------------------------------------------------------
 constexpr uint32_t kLatKeys = 32;
 typedef short s16x4 __attribute__((ext_vector_type(4)));
 
-// value fragment: column c0 + r16, keys kb .. (the unit's) of the tile; row stride ld elements, chunks swizzled by row & 7
+// value fragment of k slots (lane group g, j): bf16: keys 4g + j of the tile's first 16 rows (j < 4) and of its second 16 (j >= 4);
+// f32: keys 4g + j of rows 16 n ..; column c0 + r16.  ld: row stride in elements.
 template <class T>
-__device__ __forceinline__ typename Frag<T>::V lat_value_frag(const T* tile, uint32_t ld, uint32_t kb, uint32_t c0, uint32_t r16, uint32_t g) {
+__device__ __forceinline__ typename Frag<T>::V lat_value_frag(const T* tile, uint32_t ld, int n, uint32_t c0, uint32_t r16, uint32_t g) {
   if constexpr (sizeof(T) == 2) {   // lane i of a 16-lane group fetches 4 columns of key row i / 4 and receives 4 keys of column i
-    const uint32_t col = c0 + (r16 & 3) * 4, row = kb + g * 8 + (r16 >> 2);
+    const uint32_t col = c0 + (r16 & 3) * 4, row = g * 4 + (r16 >> 2);
     typedef __attribute__((address_space(3))) s16x4* lds_p;
-    const T* p0 = tile + row * ld + ((col >> 3) ^ (row & 7)) * 8 + (col & 7);
-    const T* p1 = tile + (row + 4) * ld + ((col >> 3) ^ ((row + 4) & 7)) * 8 + (col & 7);
-    const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)p0), b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)p1);
+    const T* p0 = tile + row * ld + ((col >> 3) ^ (row & 7)) * 8 + (col & 7);   // row + 16 has the same low bits
+    const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)p0), b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)(p0 + 16 * ld));
     return __builtin_bit_cast(bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
   } else {
     const uint32_t col = c0 + r16;
     f32x4 v;
 #pragma unroll
     for (uint32_t e = 0; e < 4; e++) {
-      const uint32_t row = kb + g * 4 + e;
+      const uint32_t row = n * 16 + g * 4 + e;
       v[e] = tile[row * ld + ((col >> 2) ^ (row & 7)) * 4 + (col & 3)];
     }
     return v;
@@ -123,9 +124,11 @@ __device__ __forceinline__ typename Frag<T>::V lat_value_frag(const T* tile, uin
 template <class T, int NCT>   // NCT: 16-column tiles of the output per wave
 __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M,
                                                           uint32_t n_splits, uint32_t nbuf) {
-  constexpr uint32_t KT = kLatKeys, PER = Frag<T>::PER, KU = Frag<T>::KU, LP = KT + 16 / sizeof(T), LS = KT + 4;
+  constexpr bool BF = sizeof(T) == 2;
+  constexpr uint32_t KT = kLatKeys, PER = Frag<T>::PER;
+  constexpr int QU = (NCT * 64 + 64) / Frag<T>::KU;             // units of a query row kept in registers (a longer row's rest is read from LDS)
   extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
-  const uint32_t tid = threadIdx.x, lane = tid & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
+  const uint32_t lane = threadIdx.x & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
   const uint32_t r16 = lane & 15, g = lane >> 4;
   const uint32_t rows = M * s.heads, row0 = blockIdx.x * 16, sp = blockIdx.y, col0 = blockIdx.z * (NCT * 64);
   const uint32_t p0 = pos_ptr ? (uint32_t)*pos_ptr : pos0;
@@ -133,141 +136,160 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
   const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles + n_splits - 1) / n_splits;
   const uint32_t tb = sp * per, te = tb + per < tiles ? tb + per : tiles;
   if (tb >= te) return;                                         // (the merge skips the same splits)
-  const uint32_t ld = s.ldc, cpr = ld / PER;                    // 16-byte chunks of a row: a multiple of 8
+  const uint32_t ld = s.ldc, cpr = ld / PER, nu = cpr / 4;      // 16-byte chunks (a multiple of 8) and units of a row
   T* Qs = reinterpret_cast<T*>(smem);                           // [16][ld]
   T* Cs = Qs + 16 * ld;                                         // [nbuf][KT][ld]
-  T* Ps = Cs + nbuf * KT * ld;                                  // [16][LP]
-  float* Ss = reinterpret_cast<float*>(Ps + 16 * LP);           // [2][16][LS]
   const T* qg = reinterpret_cast<const T*>(b.qa);
   const T* cg = reinterpret_cast<const T*>(b.cache);
+  const uint32_t cs_addr = (uint32_t)__builtin_amdgcn_readfirstlane((int)lds_addr_of(Cs)), qs_addr = (uint32_t)__builtin_amdgcn_readfirstlane((int)lds_addr_of(Qs));
+  // this lane's first 16-byte chunk of a tile, and the step to its next one (4 waves x 64 lanes further)
+  const uint32_t sr0 = (w * 64 + lane) / cpr, sc0 = (w * 64 + lane) % cpr, dr = 256 / cpr, dc = 256 % cpr;
   auto stage = [&](uint32_t tl, uint32_t buf) {
-    T* dst = Cs + buf * KT * ld;
+    const uint32_t dst = cs_addr + buf * KT * ld * (uint32_t)sizeof(T);
+    uint32_t r = sr0, ch = sc0;
     for (uint32_t i = w; i < KT * cpr / 64; i += 4) {
-      const uint32_t c = i * 64 + lane, r = c / cpr, ch = (c % cpr) ^ (r & 7), kk = tl * KT + r < kv ? tl * KT + r : kv - 1;
-      lds_dma16(cg + (size_t)kk * ld + ch * PER, dst + (size_t)i * 64 * PER);
+      const uint32_t kk = tl * KT + r < kv ? tl * KT + r : kv - 1;
+      lds_dma16_untracked(cg + (size_t)kk * ld + (ch ^ (r & 7)) * PER, dst + i * 1024);
+      r += dr;
+      ch += dc;
+      if (ch >= cpr) { ch -= cpr; r++; }
     }
   };
   for (uint32_t i = w; i < 16 * cpr / 64; i += 4) {             // the queries, same layout
     const uint32_t c = i * 64 + lane, r = c / cpr, ch = (c % cpr) ^ (r & 7), rr = row0 + r < rows ? row0 + r : rows - 1;
-    lds_dma16(qg + (size_t)rr * ld + ch * PER, Qs + (size_t)i * 64 * PER);
+    lds_dma16_untracked(qg + (size_t)rr * ld + ch * PER, qs_addr + i * 1024);
   }
-  stage(tb, 0);
-  // the rows of this lane's accumulators: 4g .. 4g + 3
-  uint32_t lim[4];
-  float m[4], l[4];
-#pragma unroll
-  for (int e = 0; e < 4; e++) {
-    const uint32_t r = row0 + g * 4 + e;
-    lim[e] = p0 + (r < rows ? r : rows - 1) / s.heads + 1;      // keys this row sees
-    m[e] = kNegHuge; l[e] = 0.0f;
-  }
+  // nbuf - 1 tiles are under way ahead of the one in use (a wave's share of a tile: cpr / 8 DMA instructions)
+  const uint32_t ahead = nbuf > 1 ? nbuf - 1 : 1;
+  for (uint32_t i = 0; i < ahead && tb + i < te; i++) stage(tb + i, i);
+  const uint32_t row = row0 + r16 < rows ? row0 + r16 : rows - 1;   // this lane's (token, head) row
+  const uint32_t lim = p0 + row / s.heads + 1;                  // keys it sees
   // bf16: scores in units of log2 (one v_exp per weight); f32: natural, with the library exponential
-  const float scl = sizeof(T) == 2 ? s.scale * kLog2e : s.scale;
-  auto ex = [](float x) { return sizeof(T) == 2 ? __builtin_amdgcn_exp2f(x) : expf(x); };
+  const float scl = BF ? s.scale * kLog2e : s.scale;
+  auto ex = [](float x) { return BF ? __builtin_amdgcn_exp2f(x) : expf(x); };
+  float m = kNegHuge, l = 0.0f;
   f32x4 o[NCT];
 #pragma unroll
   for (int i = 0; i < NCT; i++) o[i] = (f32x4)(0.0f);
-  const uint32_t wc = col0 + w * NCT * 16, half = cpr / 8 * (w >> 1);   // first unit of the wave's half row (4 chunks a unit)
-  const uint32_t u1 = w >> 1 ? cpr / 4 : cpr / 8;
-  __builtin_amdgcn_s_waitcnt(0x0F70);   // vmcnt(0)
+  const uint32_t wc = col0 + w * NCT * 16;
+  wait_vm(ahead > 1 && tb + 1 < te ? cpr / 8 : 0);
   __syncthreads();
+  auto chunk_at = [&](uint32_t u) { return ((u * 4 + g) ^ (r16 & 7)) * PER; };
+  typename Frag<T>::V qr[QU];
+#pragma unroll
+  for (int u = 0; u < QU; u++) {
+    qr[u] = Frag<T>::load(Qs + r16 * ld + chunk_at((uint32_t)u < nu ? u : 0));
+    if ((uint32_t)u >= nu) qr[u] = Frag<T>::zero();   // (a shorter row: its first unit again, times 0 — no branches between the loads)
+  }
   for (uint32_t tl = tb; tl < te; tl++) {
-    const uint32_t k0 = tl * KT, cur = nbuf == 2 ? (tl - tb) & 1 : 0;
-    if (nbuf == 2 && tl + 1 < te) stage(tl + 1, cur ^ 1);
+    const uint32_t k0 = tl * KT, cur = (tl - tb) % nbuf;
+    if (nbuf > 1 && tl + ahead < te) stage(tl + ahead, (tl - tb + ahead) % nbuf);
     const T* tile = Cs + cur * KT * ld;
-    {
-      f32x4 sc = (f32x4)(0.0f), sd = (f32x4)(0.0f);
-      const T* qa = Qs + r16 * ld;
-      const T* kb = tile + ((w & 1) * 16 + r16) * ld;
-      uint32_t u = half;
-      for (; u + 3 <= u1; u += 3) {   // three units' fragments requested together, two accumulation chains
-        typename Frag<T>::V qf[3], kf[3];
+    const T* ka = tile + r16 * ld;
+    f32x4 sa[2] = {(f32x4)(0.0f), (f32x4)(0.0f)};
+    // two units' key fragments are read while the two before them are multiplied
+    typename Frag<T>::V kf[2][4];
+    auto read2 = [&](int u, typename Frag<T>::V* k) {
 #pragma unroll
-        for (int i = 0; i < 3; i++) {
-          const uint32_t c = (((u + i) * 4 + g) ^ (r16 & 7)) * PER;
-          qf[i] = Frag<T>::load(qa + c);
-          kf[i] = Frag<T>::load(kb + c);
-        }
-        sc = Frag<T>::mma(qf[0], kf[0], sc);
-        sd = Frag<T>::mma(qf[1], kf[1], sd);
-        sc = Frag<T>::mma(qf[2], kf[2], sc);
+      for (int i = 0; i < 2; i++) {
+        const uint32_t c = chunk_at((uint32_t)(u + i) < nu ? u + i : 0);
+        k[2 * i] = Frag<T>::load(ka + c);
+        k[2 * i + 1] = Frag<T>::load(ka + 16 * ld + c);
       }
-      for (; u < u1; u++) {
-        const uint32_t c0 = ((u * 4 + g) ^ (r16 & 7)) * PER;
-        sc = Frag<T>::mma(Frag<T>::load(qa + c0), Frag<T>::load(kb + c0), sc);
-      }
-      sc += sd;
+    };
+    static_assert(QU % 2 == 0, "units in pairs");
+    read2(0, kf[0]);
 #pragma unroll
-      for (int e = 0; e < 4; e++) Ss[((w >> 1) * 16 + g * 4 + e) * LS + (w & 1) * 16 + r16] = sc[e];
+    for (int u = 0; u < QU; u += 2) {
+      if (u + 2 < QU) read2(u + 2, kf[(u / 2 + 1) & 1]);
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int i = 0; i < 2; i++) {
+        sa[0] = Frag<T>::mma(kf[(u / 2) & 1][2 * i], qr[u + i], sa[0]);
+        sa[1] = Frag<T>::mma(kf[(u / 2) & 1][2 * i + 1], qr[u + i], sa[1]);
+      }
     }
-    __syncthreads();
-    // softmax of the tile, by every wave for its own use: lane (r16, g) looks at keys r16, r16 + 16 of rows 4g .. 4g + 3
-    float alpha[4];
+    for (uint32_t u = QU; u < nu; u++) {
+      const uint32_t c = chunk_at(u);
+      const typename Frag<T>::V q = Frag<T>::load(Qs + r16 * ld + c);
+      sa[0] = Frag<T>::mma(Frag<T>::load(ka + c), q, sa[0]);
+      sa[1] = Frag<T>::mma(Frag<T>::load(ka + 16 * ld + c), q, sa[1]);
+    }
+    float m1 = m;
 #pragma unroll
-    for (int e = 0; e < 4; e++) {
-      float mx = m[e], sv[2];
+    for (int n = 0; n < 2; n++)
 #pragma unroll
-      for (int j = 0; j < 2; j++) {
-        const uint32_t key = r16 + j * 16, at = (g * 4 + e) * LS + key;
-        sv[j] = k0 + key < lim[e] ? (Ss[at] + Ss[16 * LS + at]) * scl : kNegHuge;
-        mx = fmaxf(mx, sv[j]);
+      for (int e = 0; e < 4; e++) {
+        const float v = k0 + n * 16 + g * 4 + e < lim ? sa[n][e] * scl : kNegHuge;
+        sa[n][e] = v;
+        m1 = fmaxf(m1, v);
       }
-      mx = fmaxf(mx, dpp_f<0xB1>(mx)); mx = fmaxf(mx, dpp_f<0x4E>(mx)); mx = fmaxf(mx, dpp_f<0x141>(mx)); mx = fmaxf(mx, dpp_f<0x140>(mx));
-      float sum = 0.0f;
+    m1 = fmaxf(m1, __shfl_xor(m1, 16, 64));
+    m1 = fmaxf(m1, __shfl_xor(m1, 32, 64));
+    const float alpha = ex(m - m1);
+    float sum = 0.0f;
 #pragma unroll
-      for (int j = 0; j < 2; j++) {
-        const uint32_t key = r16 + j * 16;
-        const float p = k0 + key < lim[e] ? ex(sv[j] - mx) : 0.0f;
+    for (int n = 0; n < 2; n++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        const float p = k0 + n * 16 + g * 4 + e < lim ? ex(sa[n][e] - m1) : 0.0f;
+        sa[n][e] = p;
         sum += p;
-        if (w == 0) Ps[(g * 4 + e) * LP + key] = to_act<T>(p);
       }
-      sum += dpp_f<0xB1>(sum); sum += dpp_f<0x4E>(sum); sum += dpp_f<0x141>(sum); sum += dpp_f<0x140>(sum);
-      alpha[e] = ex(m[e] - mx);
-      l[e] = l[e] * alpha[e] + sum;
-      m[e] = mx;
+    l = __builtin_fmaf(l, alpha, sum);   // this lane's keys only; added up at the end
+    if (__any(m1 > m)) {
+#pragma unroll
+      for (int i = 0; i < NCT; i++) o[i] *= alpha;
     }
-    __syncthreads();
+    m = m1;
+    if constexpr (BF) {
+      bf16x8 pf;
 #pragma unroll
-    for (int i = 0; i < NCT; i++)
-#pragma unroll
-      for (int e = 0; e < 4; e++) o[i][e] *= alpha[e];
-#pragma unroll
-    for (uint32_t k = 0; k < KT; k += KU) {
-      const typename Frag<T>::V pf = Frag<T>::load(Ps + r16 * LP + k + g * PER);
+      for (int e = 0; e < 4; e++) { pf[e] = (__bf16)sa[0][e]; pf[4 + e] = (__bf16)sa[1][e]; }
 #pragma unroll
       for (int i = 0; i < NCT; i++) {
         const uint32_t c0 = wc + i * 16 < ld ? wc + i * 16 : ld - 16;   // (columns past the row: computed, never stored)
-        o[i] = Frag<T>::mma(pf, lat_value_frag<T>(tile, ld, k, c0, r16, g), o[i]);
+        o[i] = Frag<T>::mma(lat_value_frag<T>(tile, ld, 0, c0, r16, g), pf, o[i]);
       }
+    } else {
+#pragma unroll
+      for (int n = 0; n < 2; n++)
+#pragma unroll
+        for (int i = 0; i < NCT; i++) {
+          const uint32_t c0 = wc + i * 16 < ld ? wc + i * 16 : ld - 16;
+          o[i] = Frag<T>::mma(lat_value_frag<T>(tile, ld, n, c0, r16, g), sa[n], o[i]);
+        }
     }
     if (nbuf == 1 && tl + 1 < te) {
       __syncthreads();
       stage(tl + 1, 0);
     }
-    __builtin_amdgcn_s_waitcnt(0x0F70);
+    wait_vm(tl + 2 < te && nbuf > 2 ? cpr / 8 : 0);   // the next tile has arrived; the one after it may be under way
     __syncthreads();
   }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (row0 + r16 >= rows) return;
+  const size_t pr = (size_t)sp * rows + row0 + r16;
+  if (w == 0 && g == 0 && blockIdx.z == 0) { b.part_ml[pr * 2] = BF ? m * (1.0f / kLog2e) : m; b.part_ml[pr * 2 + 1] = l; }
 #pragma unroll
-  for (int e = 0; e < 4; e++) {
-    const uint32_t r = row0 + g * 4 + e;
-    if (r >= rows) continue;
-    const size_t pr = (size_t)sp * rows + r;
-    if (w == 0 && r16 == 0 && blockIdx.z == 0) { b.part_ml[pr * 2] = sizeof(T) == 2 ? m[e] * (1.0f / kLog2e) : m[e]; b.part_ml[pr * 2 + 1] = l[e]; }
-#pragma unroll
-    for (int i = 0; i < NCT; i++) {
-      const uint32_t c = wc + i * 16 + r16;
-      if (c < s.rank) b.part_acc[pr * s.rank + c] = o[i][e];
-    }
+  for (int i = 0; i < NCT; i++) {
+    const uint32_t c = wc + i * 16 + g * 4;
+    float* dst = b.part_acc + pr * s.rank + c;
+    if (c + 4 <= s.rank && (s.rank & 3) == 0) *reinterpret_cast<f32x4*>(dst) = o[i];
+    else
+      for (uint32_t e = 0; e < 4; e++)
+        if (c + e < s.rank) dst[e] = o[i][e];
   }
 }
 
 static size_t latent_lds(const LatentShape& s, uint32_t nbuf, uint32_t el) {
-  return (size_t)(16 + nbuf * kLatKeys) * s.ldc * el + (size_t)16 * (kLatKeys + 16 / el) * el + (size_t)2 * 16 * (kLatKeys + 4) * 4;
+  return (size_t)(16 + nbuf * kLatKeys) * s.ldc * el;
 }
 
 // key tiles in flight (0: a row is too long for LDS)
 static uint32_t latent_nbuf(const LatentShape& s, bool f32) {
-  for (uint32_t n : {2u, 1u})
+  for (uint32_t n : {3u, 2u, 1u})
     if (latent_lds(s, n, f32 ? 4 : 2) <= 155 * 1024) return n;
   return 0;
 }
@@ -313,8 +335,14 @@ __global__ void __launch_bounds__(512) latent_out_kernel(const LatentShape s, co
   const uint32_t kv = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + M;
   const uint32_t tiles = (kv + kLatKeys - 1) / kLatKeys, per = (tiles + n_splits - 1) / n_splits, act = (tiles + per - 1) / per;
   const uint32_t lane = tid & 63, w = tid >> 6;
-  const float mi = lane < act ? b.part_ml[((size_t)lane * rows + r) * 2] : kNegHuge;
-  const float li = lane < act ? b.part_ml[((size_t)lane * rows + r) * 2 + 1] : 0.0f;
+  static_assert(kLatMaxSplits == 128, "two splits per lane");
+  float mi[2], li[2];
+#pragma unroll
+  for (uint32_t k = 0; k < 2; k++) {
+    const uint32_t sp = lane + k * 64, spc = sp < act ? sp : act - 1;
+    mi[k] = b.part_ml[((size_t)spc * rows + r) * 2];
+    li[k] = b.part_ml[((size_t)spc * rows + r) * 2 + 1] * (sp < act ? 1.0f : 0.0f);   // (an inactive split repeats the last one with weight 0)
+  }
   u32x4 wv0[4];   // the wave's 4 value rows, first 512 columns
 #pragma unroll
   for (int it = 0; it < 4; it++) {
@@ -337,8 +365,8 @@ __global__ void __launch_bounds__(512) latent_out_kernel(const LatentShape s, co
 #pragma unroll
   for (int i = 0; i < kOutB; i++) first[i] = fetch(grp + i * groups, q0 < quads ? q0 : 0);
   {
-    const float mm = wave_max(mi), f = expf(mi - mm), tot = wave_sum(f * li);
-    if (w == 0) wgt[lane] = f / tot;   // (inactive splits: 0)
+    const float mm = wave_max(fmaxf(mi[0], mi[1])), f0 = expf(mi[0] - mm), f1 = expf(mi[1] - mm), tot = wave_sum(f0 * li[0] + f1 * li[1]);
+    if (w == 0) { wgt[lane] = f0 / tot; wgt[lane + 64] = f1 / tot; }
   }
   __syncthreads();
   f32x4* acc4 = reinterpret_cast<f32x4*>(lat);   // [groups][quads]

@@ -103,7 +103,7 @@ struct LatentBufs {
   void* qa;                    // [M * heads][ldc]: absorbed queries
   float *part_ml, *part_acc;   // [split][M * heads][2], [split][M * heads][rank]
 };
-constexpr uint32_t kLatMaxSplits = 64;
+constexpr uint32_t kLatMaxSplits = 128;
 constexpr uint32_t kLatAbsorbRows = 1024;   // (token, head) rows the absorbed path's buffers hold
 // pos_ptr (device) or pos0: position of the first of the M tokens
 hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, bool f32, hipStream_t st);

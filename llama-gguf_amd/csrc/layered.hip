@@ -357,7 +357,8 @@ int layered_finalize(lgh_ctx* c) {
     }
   }
   uint32_t splits = (c->d.flags >> LGH_FLAG_ATTN_SPLITS_SHIFT) & 0xFFu;
-  if (!splits) splits = 256 / std::max(1u, (max_rows + 15) / 16);
+  // enough splits that a long context's workgroups cover the chip; no more, since every split's partial sums are merged
+  if (!splits) splits = std::min(512 / std::max(1u, (max_rows + 15) / 16), std::min(std::max(d.max_seq_len / 128, 64u), kLatMaxSplits));
   m.n_splits = std::max(1u, std::min(splits, kLatMaxSplits));
   // the absorbed path's rows: one token's heads in decode, several tokens' in short portions
   const size_t rows = max_rows ? kLatAbsorbRows : 0;

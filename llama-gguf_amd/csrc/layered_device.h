@@ -62,4 +62,26 @@ __device__ __forceinline__ void lds_dma16(const void* g, void* lds) {
   __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)g, (__attribute__((address_space(3))) void*)lds, 16, 0, 0);
 }
 
+// The same through inline assembly, for kernels whose LDS reads the compiler's wait-count pass does not tell apart from the DMA's
+// target (transposed reads): it does not see these loads, and the kernel waits for them itself with wait_vm.
+__device__ __forceinline__ void lds_dma16_untracked(const void* g, uint32_t lds_addr) {
+  uint32_t keep;
+  asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
+               : "=&s"(keep) : "v"(g), "s"(lds_addr) : "memory");
+}
+__device__ __forceinline__ uint32_t lds_addr_of(const void* p) {
+  return (uint32_t)(uintptr_t)(const __attribute__((address_space(3))) uint8_t*)(const uint8_t*)p;
+}
+// all but the last n vector-memory operations have completed (n = 1 .. 20; any other n waits for all)
+__device__ __forceinline__ void wait_vm(uint32_t n) {
+  switch (n) {
+#define LGH_WAIT_VM(N) case N: __builtin_amdgcn_s_waitcnt(0x0F70 | (N & 15) | ((N >> 4) << 14)); break;
+    LGH_WAIT_VM(1) LGH_WAIT_VM(2) LGH_WAIT_VM(3) LGH_WAIT_VM(4) LGH_WAIT_VM(5) LGH_WAIT_VM(6) LGH_WAIT_VM(7) LGH_WAIT_VM(8) LGH_WAIT_VM(9)
+    LGH_WAIT_VM(10) LGH_WAIT_VM(11) LGH_WAIT_VM(12) LGH_WAIT_VM(13) LGH_WAIT_VM(14) LGH_WAIT_VM(15) LGH_WAIT_VM(16) LGH_WAIT_VM(17)
+    LGH_WAIT_VM(18) LGH_WAIT_VM(19) LGH_WAIT_VM(20)
+#undef LGH_WAIT_VM
+    default: __builtin_amdgcn_s_waitcnt(0x0F70);
+  }
+}
+
 }  // namespace lgh
