@@ -9,6 +9,8 @@
 #include "layered.h"
 #include "layered_device.h"
 
+#include <algorithm>
+
 namespace lgh {
 
 constexpr float kNegHuge = -1e30f, kLog2e = 1.4426950408889634f;
@@ -94,7 +96,8 @@ hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const i
 // at a time go to LDS by DMA (16-byte chunks of a row stored at chunk ^ (row & 7)).  Everything transposed, as in the expanded kernel
 // below: S^T = C Q^T leaves a lane with one row's scores of 8 keys, which is the B operand of O^T = C^T P^T.  Every wave forms all the
 // scores (cheaper than exchanging them: one barrier per tile) and owns a quarter of the columns, whose values it takes straight from
-// the key tile (the latent IS the value), transposed on the way out of LDS.
+// the key tile (the latent IS the value), transposed on the way out of LDS.  With bf16 rows two TEAMS of 4 waves take alternate tiles —
+// a tile is a chain of short dependent steps, the other team's fill it — and are merged at the end.
 // ------------------------------------------------------------------------------------------------
 constexpr uint32_t kLatKeys = 32;
 typedef short s16x4 __attribute__((ext_vector_type(4)));
@@ -121,14 +124,18 @@ __device__ __forceinline__ typename Frag<T>::V lat_value_frag(const T* tile, uin
   }
 }
 
-template <class T, int NCT>   // NCT: 16-column tiles of the output per wave
-__global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M,
-                                                          uint32_t n_splits, uint32_t nbuf) {
+template <class T> constexpr int lat_teams() { return sizeof(T) == 2 ? 2 : 1; }   // (f32 query rows leave no registers for a second wave per SIMD)
+template <class T, int NCT> constexpr int lat_units() { return (NCT * 64 + 64) / Frag<T>::KU; }   // units of a query row kept in registers
+
+// NCT: 16-column tiles of the output per wave; nbuf: tile buffers per team; q_alias: the queries pass through the last buffer
+template <class T, int NCT>
+__global__ void __launch_bounds__(256 * lat_teams<T>()) latent_attn_kernel(const LatentShape s, const LatentBufs b, const int* __restrict__ pos_ptr, uint32_t pos0,
+                                                                           uint32_t M, uint32_t n_splits, uint32_t nbuf, uint32_t q_alias) {
   constexpr bool BF = sizeof(T) == 2;
   constexpr uint32_t KT = kLatKeys, PER = Frag<T>::PER;
-  constexpr int QU = (NCT * 64 + 64) / Frag<T>::KU;             // units of a query row kept in registers (a longer row's rest is read from LDS)
+  constexpr int QU = lat_units<T, NCT>(), TM = lat_teams<T>();  // (a longer query row's rest is read from LDS)
   extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
-  const uint32_t lane = threadIdx.x & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
+  const uint32_t lane = threadIdx.x & 63, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)), w = wave & 3, team = wave >> 2;
   const uint32_t r16 = lane & 15, g = lane >> 4;
   const uint32_t rows = M * s.heads, row0 = blockIdx.x * 16, sp = blockIdx.y, col0 = blockIdx.z * (NCT * 64);
   const uint32_t p0 = pos_ptr ? (uint32_t)*pos_ptr : pos0;
@@ -137,8 +144,9 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
   const uint32_t tb = sp * per, te = tb + per < tiles ? tb + per : tiles;
   if (tb >= te) return;                                         // (the merge skips the same splits)
   const uint32_t ld = s.ldc, cpr = ld / PER, nu = cpr / 4;      // 16-byte chunks (a multiple of 8) and units of a row
-  T* Qs = reinterpret_cast<T*>(smem);                           // [16][ld]
-  T* Cs = Qs + 16 * ld;                                         // [nbuf][KT][ld]
+  T* Cs = reinterpret_cast<T*>(smem) + (q_alias ? 0 : 16 * ld); // [team][nbuf][KT][ld]
+  T* Qs = q_alias ? Cs + (TM * nbuf - 1) * KT * ld : reinterpret_cast<T*>(smem);   // [16][ld]
+  Cs += team * nbuf * KT * ld;
   const T* qg = reinterpret_cast<const T*>(b.qa);
   const T* cg = reinterpret_cast<const T*>(b.cache);
   const uint32_t cs_addr = (uint32_t)__builtin_amdgcn_readfirstlane((int)lds_addr_of(Cs)), qs_addr = (uint32_t)__builtin_amdgcn_readfirstlane((int)lds_addr_of(Qs));
@@ -155,13 +163,14 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
       if (ch >= cpr) { ch -= cpr; r++; }
     }
   };
-  for (uint32_t i = w; i < 16 * cpr / 64; i += 4) {             // the queries, same layout
+  for (uint32_t i = wave; i < 16 * cpr / 64; i += 4 * TM) {     // the queries, same layout
     const uint32_t c = i * 64 + lane, r = c / cpr, ch = (c % cpr) ^ (r & 7), rr = row0 + r < rows ? row0 + r : rows - 1;
     lds_dma16_untracked(qg + (size_t)rr * ld + ch * PER, qs_addr + i * 1024);
   }
   // nbuf - 1 tiles are under way ahead of the one in use (a wave's share of a tile: cpr / 8 DMA instructions)
   const uint32_t ahead = nbuf > 1 ? nbuf - 1 : 1;
-  for (uint32_t i = 0; i < ahead && tb + i < te; i++) stage(tb + i, i);
+  const uint32_t t_first = tb + team;
+  for (uint32_t i = 0; i < ahead && t_first + i * TM < te; i++) stage(t_first + i * TM, i);
   const uint32_t row = row0 + r16 < rows ? row0 + r16 : rows - 1;   // this lane's (token, head) row
   const uint32_t lim = p0 + row / s.heads + 1;                  // keys it sees
   // bf16: scores in units of log2 (one v_exp per weight); f32: natural, with the library exponential
@@ -172,7 +181,7 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
 #pragma unroll
   for (int i = 0; i < NCT; i++) o[i] = (f32x4)(0.0f);
   const uint32_t wc = col0 + w * NCT * 16;
-  wait_vm(ahead > 1 && tb + 1 < te ? cpr / 8 : 0);
+  wait_vm(ahead > 1 && t_first + TM < te ? cpr / 8 : 0);
   __syncthreads();
   auto chunk_at = [&](uint32_t u) { return ((u * 4 + g) ^ (r16 & 7)) * PER; };
   typename Frag<T>::V qr[QU];
@@ -181,9 +190,13 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
     qr[u] = Frag<T>::load(Qs + r16 * ld + chunk_at((uint32_t)u < nu ? u : 0));
     if ((uint32_t)u >= nu) qr[u] = Frag<T>::zero();   // (a shorter row: its first unit again, times 0 — no branches between the loads)
   }
-  for (uint32_t tl = tb; tl < te; tl++) {
-    const uint32_t k0 = tl * KT, cur = (tl - tb) % nbuf;
-    if (nbuf > 1 && tl + ahead < te) stage(tl + ahead, (tl - tb + ahead) % nbuf);
+  if (q_alias) __syncthreads();   // the queries' buffer is free
+  const uint32_t rounds = (te - tb + TM - 1) / TM;
+  uint32_t cur = 0;
+  for (uint32_t rd = 0; rd < rounds; rd++, cur = cur + 1 < nbuf ? cur + 1 : 0) {
+    const uint32_t tl = t_first + rd * TM, k0 = tl * KT;
+    if (nbuf > 1 && tl + ahead * TM < te) stage(tl + ahead * TM, cur + ahead < nbuf ? cur + ahead : cur + ahead - nbuf);
+    if (tl < te) {   // (the last round may have a tile for the first team only)
     const T* tile = Cs + cur * KT * ld;
     const T* ka = tile + r16 * ld;
     f32x4 sa[2] = {(f32x4)(0.0f), (f32x4)(0.0f)};
@@ -260,15 +273,37 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
           o[i] = Frag<T>::mma(lat_value_frag<T>(tile, ld, n, c0, r16, g), sa[n], o[i]);
         }
     }
-    if (nbuf == 1 && tl + 1 < te) {
-      __syncthreads();
-      stage(tl + 1, 0);
     }
-    wait_vm(tl + 2 < te && nbuf > 2 ? cpr / 8 : 0);   // the next tile has arrived; the one after it may be under way
+    if (nbuf == 1) {
+      __syncthreads();
+      if (tl + TM < te) stage(tl + TM, 0);
+    }
+    wait_vm(tl + 2 * TM < te && nbuf > 2 ? cpr / 8 : 0);   // the next tile has arrived; the one after it may be under way
     __syncthreads();
   }
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
+  if constexpr (TM == 2) {   // the second team's share, lane by lane
+    f32x4* mo = reinterpret_cast<f32x4*>(smem);                  // [wave][NCT][lane]
+    float* mm = reinterpret_cast<float*>(mo + 4 * NCT * 64);     // [wave][2][lane]
+    if (team == 1) {
+#pragma unroll
+      for (int i = 0; i < NCT; i++) mo[(w * NCT + i) * 64 + lane] = o[i];
+      mm[w * 128 + lane] = m;
+      mm[w * 128 + 64 + lane] = l;
+    }
+    __syncthreads();
+    if (team == 1) return;
+    const float om = mm[w * 128 + lane], ol = mm[w * 128 + 64 + lane], mn = fmaxf(m, om), a0 = ex(m - mn), a1 = ex(om - mn);
+    l = l * a0 + ol * a1;
+    m = mn;
+#pragma unroll
+    for (int i = 0; i < NCT; i++) {
+      const f32x4 x = mo[(w * NCT + i) * 64 + lane];
+#pragma unroll
+      for (int e = 0; e < 4; e++) o[i][e] = o[i][e] * a0 + x[e] * a1;
+    }
+  }
   if (row0 + r16 >= rows) return;
   const size_t pr = (size_t)sp * rows + row0 + r16;
   if (w == 0 && g == 0 && blockIdx.z == 0) { b.part_ml[pr * 2] = BF ? m * (1.0f / kLog2e) : m; b.part_ml[pr * 2 + 1] = l; }
@@ -283,34 +318,37 @@ __global__ void __launch_bounds__(256) latent_attn_kernel(const LatentShape s, c
   }
 }
 
-static size_t latent_lds(const LatentShape& s, uint32_t nbuf, uint32_t el) {
-  return (size_t)(16 + nbuf * kLatKeys) * s.ldc * el;
+// how a shape's tiles lie in LDS (bytes 0: a row is too long)
+struct LatentPlan { uint32_t nbuf, q_alias; size_t bytes; };
+static LatentPlan latent_plan(const LatentShape& s, bool f32) {
+  const uint32_t el = f32 ? 4 : 2, teams = f32 ? lat_teams<float>() : lat_teams<__bf16>();
+  const size_t row = (size_t)s.ldc * el, tile = kLatKeys * row, merge = 34 * 1024 + 1024;
+  const uint32_t nct = (s.rank + 63) / 64, c = nct <= 1 ? 1 : nct <= 2 ? 2 : nct <= 4 ? 4 : 8;   // the kernel's column tiles per wave
+  const bool in_regs = s.ldc <= c * 64 + 64;                                                 // the whole query row stays in registers
+  for (uint32_t n : {3u, 2u, 1u}) {
+    if (16 * row + teams * n * tile <= 155 * 1024) return {n, 0u, std::max(16 * row + teams * n * tile, merge)};
+    if (n > 1 && in_regs && teams * n * tile <= 155 * 1024) return {n, 1u, std::max(teams * n * tile, merge)};
+  }
+  return {0, 0, 0};
 }
-
-// key tiles in flight (0: a row is too long for LDS)
-static uint32_t latent_nbuf(const LatentShape& s, bool f32) {
-  for (uint32_t n : {3u, 2u, 1u})
-    if (latent_lds(s, n, f32 ? 4 : 2) <= 155 * 1024) return n;
-  return 0;
-}
-bool latent_fits(const LatentShape& s, bool f32) { return latent_nbuf(s, f32) != 0; }
+bool latent_fits(const LatentShape& s, bool f32) { return latent_plan(s, f32).bytes != 0; }
 
 template <class T, int NCT>
-static hipError_t latent_attn_go(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, uint32_t nbuf,
+static hipError_t latent_attn_go(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, const LatentPlan& pl,
                                  uint32_t zs, hipStream_t st) {
   static bool opted[64] = {};
   if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&latent_attn_kernel<T, NCT>), 156 * 1024, opted); e != hipSuccess) return e;
-  hipLaunchKernelGGL((latent_attn_kernel<T, NCT>), dim3((M * s.heads + 15) / 16, n_splits, zs), dim3(256), latent_lds(s, nbuf, sizeof(T)), st, s, b, pos_ptr,
-                     pos0, M, n_splits, nbuf);
+  hipLaunchKernelGGL((latent_attn_kernel<T, NCT>), dim3((M * s.heads + 15) / 16, n_splits, zs), dim3(256 * lat_teams<T>()), pl.bytes, st, s, b, pos_ptr,
+                     pos0, M, n_splits, pl.nbuf, pl.q_alias);
   return hipGetLastError();
 }
 
 hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32,
                               hipStream_t st) {
-  const uint32_t nbuf = latent_nbuf(s, f32);
-  if (!nbuf || s.ldc % 64 || n_splits == 0 || n_splits > kLatMaxSplits || M == 0 || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
+  const LatentPlan pl = latent_plan(s, f32);
+  if (!pl.bytes || s.ldc % 64 || n_splits == 0 || n_splits > kLatMaxSplits || M == 0 || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
   const uint32_t nct = (s.rank + 63) / 64;
-#define LGH_LAT_CASE(N) return f32 ? latent_attn_go<float, N>(s, b, pos_ptr, pos0, M, n_splits, nbuf, zs, st) : latent_attn_go<__bf16, N>(s, b, pos_ptr, pos0, M, n_splits, nbuf, zs, st)
+#define LGH_LAT_CASE(N) return f32 ? latent_attn_go<float, N>(s, b, pos_ptr, pos0, M, n_splits, pl, zs, st) : latent_attn_go<__bf16, N>(s, b, pos_ptr, pos0, M, n_splits, pl, zs, st)
   uint32_t zs = 1;
   if (nct <= 1) LGH_LAT_CASE(1);
   if (nct <= 2) LGH_LAT_CASE(2);
