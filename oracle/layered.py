@@ -74,8 +74,8 @@ def latent_attention(h, w, mx, eps):
     q = (h @ w["q"].T).reshape(T, H, d + r)
     dkv = h @ w["dkv"].T
     c = rms(dkv[:, :kr], eps) * w["dkv.norm"]
-    k_rot = rotate_pairs(dkv[:, kr:], pos, mx["rot"])
-    q_rot = rotate_pairs(q[..., d:], pos, mx["rot"])
+    turn = lambda x: rotate_pairs(x, pos, mx["rot"]) if mx.get("rot") else x
+    k_rot, q_rot = turn(dkv[:, kr:]), turn(q[..., d:])
     k = (c @ w["uk"].T).reshape(T, H, d)
     v = (c @ w["uv"].T).reshape(T, H, dv)
     gate = sigmoid(h @ w["g"].T)
