@@ -130,6 +130,7 @@ typedef struct lgh_ctx lgh_ctx;
 enum {
   LGH_K_EMBED = 0, LGH_K_QKV = 1, LGH_K_ATTN = 2, LGH_K_ATTN_COMBINE = 3, LGH_K_WO = 4, LGH_K_GATEUP = 5,
   LGH_K_DOWN = 6, LGH_K_ROUTER = 7, LGH_K_OUTPUT = 8, LGH_K_ARGMAX = 9, LGH_K_MISC = 10,
+  LGH_K_EXPAND = 12,  /* latent attention, long portions: keys and values per head */
   LGH_K_TOKEN = 11,   /* (unused since round 3: was the persistent token kernel) */
   LGH_K_COUNT = 16
 };

@@ -543,13 +543,13 @@ static int block_latent(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) 
         (rc = grow(c, &f.vt, &m.fl_v_bytes, (size_t)H * f.dvp * f.Tcap * m.el())))
       return rc;
     const LatentBufs b = latent_bufs(m, L, m.bcat);
-    if ((rc = run_k(c, LGH_K_MISC, LGH_SYM_LATENT, 0, [&] { return latent_flash_prep_launch(L.ls, b, f, pos0, M, m.f32, st); }))) return rc;
+    if ((rc = run_k(c, LGH_K_EXPAND, LGH_SYM_LATENT, 0, [&] { return latent_flash_prep_launch(L.ls, b, f, pos0, M, m.f32, st); }))) return rc;
     LinGemm g{};
     g.x = L.cache; g.ldx = L.ls.ldc; g.M = kv;
     g.w = L.uk.w; g.n = L.uk.n; g.np = L.uk.np(); g.kp = L.uk.kp; g.out = f.k; g.ldo = f.dq; g.hd = L.ls.dim; g.tcap = f.Tcap;
-    if ((rc = run_k(c, LGH_K_ROUTER, LGH_SYM_LINEAR, L.uk.bytes(), [&] { return lin_gemm_launch(LE_HEADS, m.f32, g, st); }))) return rc;
+    if ((rc = run_k(c, LGH_K_EXPAND, LGH_SYM_LINEAR, L.uk.bytes(), [&] { return lin_gemm_launch(LE_HEADS, m.f32, g, st); }))) return rc;
     g.w = L.uv.w; g.n = L.uv.n; g.np = L.uv.np(); g.kp = L.uv.kp; g.out = f.vt; g.ldo = (uint32_t)f.Tcap; g.hd = L.ls.vdim; g.hrows = f.dvp;
-    if ((rc = run_k(c, LGH_K_ROUTER, LGH_SYM_LINEAR, L.uv.bytes(), [&] { return lin_gemm_launch(LE_HEADS_T, m.f32, g, st); }))) return rc;
+    if ((rc = run_k(c, LGH_K_EXPAND, LGH_SYM_LINEAR, L.uv.bytes(), [&] { return lin_gemm_launch(LE_HEADS_T, m.f32, g, st); }))) return rc;
     return run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, 0, [&] { return latent_flash_launch(L.ls, b, f, pos0, M, m.f32, m.bao, L.out.kp, st); });
   }
   // absorbed, as many tokens at a time as their (token, head) rows fit the buffers

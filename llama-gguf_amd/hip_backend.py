@@ -40,7 +40,7 @@ ABI_SYMBOLS = (
     "lgh_batch_create", "lgh_batch_reset", "lgh_batch_position", "lgh_batch_prefill", "lgh_forward_multi", "lgh_decode_greedy_multi",
 )
 
-K_NAMES = ("embed", "qkv", "attn", "attn_combine", "wo", "gate_up", "down", "router", "output", "argmax", "misc", "token")
+K_NAMES = ("embed", "qkv", "attn", "attn_combine", "wo", "gate_up", "down", "router", "output", "argmax", "misc", "token", "expand")
 K_COUNT = 16
 SYM_COUNT = 24
 # kernel symbols as rocprofv3 prints them (LGH_SYM_* order)

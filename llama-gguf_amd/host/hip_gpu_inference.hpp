@@ -63,6 +63,16 @@ class HipGpuInference {
     g.check(lgh_finalize(h));
     return g;
   }
+  // a model described layer by layer (lgh_create_layered)
+  static HipGpuInference from_layered(const lgh_layered_desc& desc, const std::vector<lgh_layer_desc>& layers, const std::vector<HostTensor>& tensors) {
+    lgh_ctx* h = nullptr;
+    if (layers.size() != desc.num_layers) throw std::invalid_argument("one descriptor per layer");
+    if (int rc = lgh_create_layered(&desc, layers.data(), &h)) throw BackendError(rc, "lgh_create_layered");
+    HipGpuInference g(h, desc.vocab_size);
+    for (const HostTensor& t : tensors) g.check(lgh_upload_tensor(h, t.name.c_str(), t.ggml_type, t.ne, t.data, t.nbytes));
+    g.check(lgh_finalize(h));
+    return g;
+  }
   HipGpuInference(HipGpuInference&& o) noexcept : h_(o.h_), vocab_(o.vocab_) { o.h_ = nullptr; }
   HipGpuInference& operator=(HipGpuInference&& o) noexcept {
     if (this != &o) { lgh_destroy(h_); h_ = o.h_; vocab_ = o.vocab_; o.h_ = nullptr; }
@@ -80,6 +90,14 @@ class HipGpuInference {
   void prefill_token(uint32_t token_id) { check(lgh_prefill_token(h_, token_id)); }
   // GpuOnlyInference::forward_batch minus the final forward (gpu_only.rs:776-790); batched f16-GEMM path when the model allows
   void forward_batch(const std::vector<uint32_t>& tokens) { check(lgh_prefill_batch(h_, tokens.data(), tokens.size())); }
+  // a portion of the sequence with the logits after its places `want` (ascending): [want.size()][vocab]
+  std::vector<std::vector<float>> eval(const std::vector<uint32_t>& tokens, const std::vector<uint32_t>& want) {
+    std::vector<float> flat(want.size() * (size_t)vocab_);
+    check(lgh_eval(h_, tokens.data(), tokens.size(), want.data(), want.size(), flat.data()));
+    std::vector<std::vector<float>> out(want.size());
+    for (size_t i = 0; i < want.size(); i++) out[i].assign(flat.begin() + i * vocab_, flat.begin() + (i + 1) * vocab_);
+    return out;
+  }
   bool prefill_is_batched() { return lgh_prefill_is_batched(h_) != 0; }
   void kv_truncate(size_t new_len) { check(lgh_kv_truncate(h_, new_len)); }        // KVCache::truncate (model/mod.rs:130-134)
   void kv_shift_left(size_t amount) { check(lgh_kv_shift_left(h_, amount)); }      // KVCache::shift_left (model/mod.rs:142-172)
