@@ -522,15 +522,21 @@ hipError_t latent_flash_prep_launch(const LatentShape& s, const LatentBufs& b, c
 // Causal attention, everything transposed: S^T = K Q^T leaves a lane with one query's scores of keys 4g .. 4g + 3, which is the B
 // operand of O^T = V^T P^T when the value fragment's k slots are assigned the same way — the weights never leave the registers.
 // A workgroup = 4 waves = 64 * QT queries of one head; K and V^T tiles of KT keys go to LDS by DMA, two buffers.
+// two workgroups per CU where their tiles fit LDS
+template <class T, int DQ, int DV> constexpr size_t flash_lds() { return 2 * ((sizeof(T) == 2 ? 64 : 32) * (size_t)DQ * sizeof(T) + (size_t)DV * 128); }
+template <class T, int DQ, int DV> constexpr int flash_wgs() { return 2 * flash_lds<T, DQ, DV>() <= 160 * 1024 && DV <= 128 ? 2 : 1; }
+
 template <class T, int DQ, int DV>
-__global__ void __launch_bounds__(256) latent_flash_kernel(const LatentShape s, const LatentBufs b, const LatentFlash f, uint32_t pos0, uint32_t M, uint32_t nqb,
+__global__ void __launch_bounds__(256, (flash_wgs<T, DQ, DV>())) latent_flash_kernel(const LatentShape s, const LatentBufs b, const LatentFlash f, uint32_t pos0, uint32_t M, uint32_t nqb,
                                                            T* __restrict__ out, uint32_t ldo) {
   constexpr bool BF = sizeof(T) == 2;
   constexpr int KT = BF ? 64 : 32, QT = BF ? 2 : 1, NK = KT / 16, NU = DQ / Frag<T>::KU, ND = DV / 16, NP = KT / Frag<T>::KU;
   constexpr uint32_t XC = DQ * sizeof(T) / 16, kK = KT * XC * 16, kV = DV * 128, kBuf = kK + kV;
   extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
   const uint32_t lane = threadIdx.x & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)), r16 = lane & 15, g = lane >> 4;
-  const uint32_t h = blockIdx.x % s.heads, qb = nqb - 1 - blockIdx.x / s.heads;   // the longest rows first
+  // the longest rows first, and of the second half of the grid the shortest first: workgroups i and i + half, which share a CU when the
+  // whole grid is resident, then have equal work together
+  const uint32_t h = blockIdx.x % s.heads, qi = blockIdx.x / s.heads, hi = (nqb + 1) / 2, qb = qi < hi ? nqb - 1 - qi : qi - hi;
   const uint32_t q0 = qb * 64 * QT, qw = q0 + w * 16 * QT;
   const uint32_t qlast = q0 + 64 * QT - 1 < M - 1 ? q0 + 64 * QT - 1 : M - 1;
   const uint32_t tiles = (pos0 + qlast + KT) / KT;   // keys 0 .. pos0 + qlast
@@ -589,29 +595,35 @@ __global__ void __launch_bounds__(256) latent_flash_kernel(const LatentShape s, 
 #pragma unroll
         for (int t = 0; t < QT; t++) sa[n][t] = Frag<T>::mma(kf, qf[t][u], sa[n][t]);
       }
-    const bool edge = k0 + KT > pos0 + qw + 1;   // wave-uniform: some key may lie behind some query
+    if (k0 + KT > pos0 + qw + 1) {   // wave-uniform: some key may lie behind some query
+      asm volatile("");              // (kept a branch: most tiles have no masks to apply)
 #pragma unroll
-    for (int t = 0; t < QT; t++) {
-      const uint32_t lim = pos0 + qw + t * 16 + r16;   // last visible key
+      for (int t = 0; t < QT; t++) {
+        const uint32_t lim = pos0 + qw + t * 16 + r16;   // last visible key
+#pragma unroll
+        for (int n = 0; n < NK; n++)
+#pragma unroll
+          for (int e = 0; e < 4; e++) sa[n][t][e] = k0 + n * 16 + g * 4 + e > lim ? kNegHuge : sa[n][t][e];
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < QT; t++) {   // maxima of the raw scores; the scale goes into the exponent's multiply-add
       float m1 = mx[t];
 #pragma unroll
       for (int n = 0; n < NK; n++)
 #pragma unroll
-        for (int e = 0; e < 4; e++) {
-          float v = sa[n][t][e] * sc;
-          if (edge) v = k0 + n * 16 + g * 4 + e > lim ? kNegHuge : v;
-          sa[n][t][e] = v;
-          m1 = fmaxf(m1, v);
-        }
+        for (int e = 0; e < 4; e++) m1 = fmaxf(m1, sa[n][t][e]);
       m1 = fmaxf(m1, __shfl_xor(m1, 16, 64));
       m1 = fmaxf(m1, __shfl_xor(m1, 32, 64));
-      const float a = BF ? __builtin_amdgcn_exp2f(mx[t] - m1) : expf(mx[t] - m1);
+      const float off = -m1 * sc;
+      auto weight = [&](float v) { const float x = __builtin_fmaf(v, sc, off); return BF ? __builtin_amdgcn_exp2f(x) : expf((v - m1) * sc); };
+      const float a = weight(mx[t]);
       float sum = 0.0f;
 #pragma unroll
       for (int n = 0; n < NK; n++)
 #pragma unroll
         for (int e = 0; e < 4; e++) {
-          const float p = BF ? __builtin_amdgcn_exp2f(sa[n][t][e] - m1) : expf(sa[n][t][e] - m1);
+          const float p = weight(sa[n][t][e]);
           sa[n][t][e] = p;
           sum += p;
         }
@@ -674,7 +686,7 @@ __global__ void __launch_bounds__(256) latent_flash_kernel(const LatentShape s, 
 template <class T, int DQ, int DV>
 static hipError_t latent_flash_go(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, void* out, uint32_t ldo, hipStream_t st) {
   static bool opted[64] = {};
-  constexpr size_t KT = sizeof(T) == 2 ? 64 : 32, lds = 2 * (KT * DQ * sizeof(T) + DV * 128);
+  constexpr size_t lds = flash_lds<T, DQ, DV>();
   static_assert(lds <= 160 * 1024, "two tiles fit LDS");
   if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&latent_flash_kernel<T, DQ, DV>), (int)lds, opted); e != hipSuccess) return e;
   const uint32_t QB = sizeof(T) == 2 ? 128 : 64, nqb = (M + QB - 1) / QB;
