@@ -137,7 +137,7 @@ __global__ void __launch_bounds__(256 * lat_teams<T>()) latent_attn_kernel(const
   extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
   const uint32_t lane = threadIdx.x & 63, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)), w = wave & 3, team = wave >> 2;
   const uint32_t r16 = lane & 15, g = lane >> 4;
-  const uint32_t rows = M * s.heads, row0 = blockIdx.x * 16, sp = blockIdx.y, col0 = blockIdx.z * (NCT * 64);
+  const uint32_t rows = M * s.heads, row0 = blockIdx.y * 16, sp = blockIdx.x, col0 = blockIdx.z * (NCT * 64);   // (a split's row tiles on one XCD when the splits are a multiple of 8)
   const uint32_t p0 = pos_ptr ? (uint32_t)*pos_ptr : pos0;
   const uint32_t kv = p0 + M;                                   // keys 0 .. kv - 1
   const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles + n_splits - 1) / n_splits;
@@ -338,7 +338,7 @@ static hipError_t latent_attn_go(const LatentShape& s, const LatentBufs& b, cons
                                  uint32_t zs, hipStream_t st) {
   static bool opted[64] = {};
   if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&latent_attn_kernel<T, NCT>), 156 * 1024, opted); e != hipSuccess) return e;
-  hipLaunchKernelGGL((latent_attn_kernel<T, NCT>), dim3((M * s.heads + 15) / 16, n_splits, zs), dim3(256 * lat_teams<T>()), pl.bytes, st, s, b, pos_ptr,
+  hipLaunchKernelGGL((latent_attn_kernel<T, NCT>), dim3(n_splits, (M * s.heads + 15) / 16, zs), dim3(256 * lat_teams<T>()), pl.bytes, st, s, b, pos_ptr,
                      pos0, M, n_splits, pl.nbuf, pl.q_alias);
   return hipGetLastError();
 }
