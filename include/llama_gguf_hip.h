@@ -131,6 +131,7 @@ enum {
   LGH_K_EMBED = 0, LGH_K_QKV = 1, LGH_K_ATTN = 2, LGH_K_ATTN_COMBINE = 3, LGH_K_WO = 4, LGH_K_GATEUP = 5,
   LGH_K_DOWN = 6, LGH_K_ROUTER = 7, LGH_K_OUTPUT = 8, LGH_K_ARGMAX = 9, LGH_K_MISC = 10,
   LGH_K_EXPAND = 12,  /* latent attention, long portions: keys and values per head */
+  LGH_K_EXPERTS = 13, /* gate | up products of the routed experts (models described layer by layer) */
   LGH_K_TOKEN = 11,   /* (unused since round 3: was the persistent token kernel) */
   LGH_K_COUNT = 16
 };
@@ -165,7 +166,8 @@ enum {
   LGH_SYM_LINEAR = 21,     /* lgh::lin_mv_kernel / lgh::lin_gemm_kernel : products over weights kept in bf16 (lgh_create_layered) */
   LGH_SYM_LATENT = 22,     /* lgh::latent_* : attention over a shared latent */
   LGH_SYM_MLSTM = 23,      /* lgh::mlstm_* : matrix-memory recurrence */
-  LGH_SYM_COUNT = 24
+  LGH_SYM_TIED = 24,       /* lgh::tied_* : attention whose values are its keys */
+  LGH_SYM_COUNT = 25
 };
 
 typedef struct lgh_stats {
@@ -272,13 +274,20 @@ int lgh_op_tq_compress_qjl(int device, int bits, const float* x, size_t dim, con
 int lgh_eval(lgh_ctx* ctx, const uint32_t* tokens, size_t n, const uint32_t* want, size_t n_want, float* logits_out);
 
 /* ---- models whose layers are described one by one: every layer has a mixer (attention or a recurrence) and, optionally, a
- * feed-forward; sublayers read the residual stream itself and their outputs are layer-normed, x += residual_mult * norm(sublayer(x)).
+ * feed-forward.  How sublayers and the residual stream meet is the model's residual form:
+ *   LGH_RESIDUAL_POST_LN       sublayers read the stream itself, x += residual_mult * layer_norm(sublayer(x)) * w
+ *   LGH_RESIDUAL_SANDWICH_DYT  h = dyt(x); h += conv(h); x += residual_mult * dyt'(sublayer(h)), where dyt(x) = tanh(alpha x) * w + b and
+ *                              conv is a causal convolution over conv_taps positions, one filter per channel (0 taps: none)
  * No reference counterpart.  The context is driven by the entry points above (GpuInference, lgh_eval, lgh_decode_greedy, ...; the
  * cache rows and recurrent states are the context's).  Weights are bf16 and stay bf16 in HBM; tensors are uploaded by their
- * checkpoint names (`embed`, `bigram`, `l0.mix.q`, `l0.mlp.gate`, `l0.norm1`, `final.norm`, `head`) with GGML dims (in fastest).
+ * checkpoint names (`embed`, `bigram`, `l0.mix.q`, `l0.mlp.gate`, `l0.mlp.e0.gate`, `l0.norm1`, `l0.norm1.alpha`, `l0.canon1`, `final.norm`,
+ * `head`) with GGML dims (in fastest; a scalar has one element).
  * Single stage, one sequence per context. ---- */
-enum { LGH_MIXER_LATENT_ATTENTION = 1, LGH_MIXER_MLSTM = 2 };
+enum { LGH_MIXER_LATENT_ATTENTION = 1, LGH_MIXER_MLSTM = 2,
+       LGH_MIXER_TIED_ATTENTION = 3 };                 /* grouped heads, values = keys before their norm, no rotation; window, sinks, distance bias */
+enum { LGH_RESIDUAL_POST_LN = 0, LGH_RESIDUAL_SANDWICH_DYT = 1 };
 enum { LGH_FF_NONE = 0, LGH_FF_GEGLU = 1 };            /* down(gelu_tanh(gate x) * (up x)) */
+enum { LGH_FF_MOE = 2 };                               /* routed experts down(silu(gate x) * (up x)), sigmoid scores; optionally a shared one */
 enum { LGH_COMPUTE_BF16 = 0, LGH_COMPUTE_F32 = 1 };    /* operands of block products, cache rows: bf16 (f32 accumulation), or f32 throughout */
 typedef struct lgh_layer_desc {
   uint32_t struct_size;
@@ -286,11 +295,16 @@ typedef struct lgh_layer_desc {
   uint32_t heads, dim, vdim;         /* query / key size per head (latent attention: the unrotated part), value size per head */
   uint32_t kv_rank, rot_dim;         /* latent attention: latent size, rotated query / key part */
   uint32_t rot_dims;                 /* leading values of the rotated part that are rotated (neighbouring pairs) */
-  uint32_t ff_kind, ff;              /* LGH_FF_*, feed-forward size */
-  double scale;                      /* latent attention: factor on the scores */
+  uint32_t ff_kind, ff;              /* LGH_FF_*, feed-forward size (mixture: of one expert) */
+  uint32_t kv_heads;                 /* tied attention: key heads; query head h uses h / (heads / kv_heads) */
+  uint32_t window, keep_first;       /* tied attention: position i sees j <= i with i - j < window (0: no limit) or j < keep_first */
+  uint32_t experts, top;             /* mixture: experts, and how many a token uses */
+  uint32_t shared_ff;                /* mixture: size of the expert every token uses (0: none) */
+  double scale;                      /* attention: factor on the scores */
   double rot_base;
   double yarn_factor, yarn_original, yarn_fast, yarn_slow;   /* yarn_factor 0: plain frequencies */
   double gate_cap;                   /* mLSTM: soft cap of the gates' pre-activations */
+  double score_cap;                  /* tied attention: soft cap of the scores (0: none) */
 } lgh_layer_desc;
 typedef struct lgh_layered_desc {
   uint32_t struct_size;
@@ -301,6 +315,8 @@ typedef struct lgh_layered_desc {
   uint32_t bigram_buckets;           /* 0: no pair embedding */
   uint64_t bigram_mul_prev, bigram_mul_cur;
   double norm_eps, residual_mult;
+  uint32_t residual;                 /* LGH_RESIDUAL_* */
+  uint32_t conv_taps;
 } lgh_layered_desc;
 int lgh_create_layered(const lgh_layered_desc* desc, const lgh_layer_desc* layers, lgh_ctx** out);
 /* Residual stream after every layer, for parity tests: switched on, the next lgh_eval portions (block path) keep it;

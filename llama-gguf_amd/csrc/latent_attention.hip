@@ -100,29 +100,6 @@ hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const i
 // a tile is a chain of short dependent steps, the other team's fill it — and are merged at the end.
 // ------------------------------------------------------------------------------------------------
 constexpr uint32_t kLatKeys = 32;
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-
-// value fragment of k slots (lane group g, j): bf16: keys 4g + j of the tile's first 16 rows (j < 4) and of its second 16 (j >= 4);
-// f32: keys 4g + j of rows 16 n ..; column c0 + r16.  ld: row stride in elements.
-template <class T>
-__device__ __forceinline__ typename Frag<T>::V lat_value_frag(const T* tile, uint32_t ld, int n, uint32_t c0, uint32_t r16, uint32_t g) {
-  if constexpr (sizeof(T) == 2) {   // lane i of a 16-lane group fetches 4 columns of key row i / 4 and receives 4 keys of column i
-    const uint32_t col = c0 + (r16 & 3) * 4, row = g * 4 + (r16 >> 2);
-    typedef __attribute__((address_space(3))) s16x4* lds_p;
-    const T* p0 = tile + row * ld + ((col >> 3) ^ (row & 7)) * 8 + (col & 7);   // row + 16 has the same low bits
-    const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)p0), b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)(p0 + 16 * ld));
-    return __builtin_bit_cast(bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
-  } else {
-    const uint32_t col = c0 + r16;
-    f32x4 v;
-#pragma unroll
-    for (uint32_t e = 0; e < 4; e++) {
-      const uint32_t row = n * 16 + g * 4 + e;
-      v[e] = tile[row * ld + ((col >> 2) ^ (row & 7)) * 4 + (col & 3)];
-    }
-    return v;
-  }
-}
 
 template <class T> constexpr int lat_teams() { return sizeof(T) == 2 ? 2 : 1; }   // (f32 query rows leave no registers for a second wave per SIMD)
 template <class T, int NCT> constexpr int lat_units() { return (NCT * 64 + 64) / Frag<T>::KU; }   // units of a query row kept in registers
@@ -262,7 +239,7 @@ __global__ void __launch_bounds__(256 * lat_teams<T>()) latent_attn_kernel(const
 #pragma unroll
       for (int i = 0; i < NCT; i++) {
         const uint32_t c0 = wc + i * 16 < ld ? wc + i * 16 : ld - 16;   // (columns past the row: computed, never stored)
-        o[i] = Frag<T>::mma(lat_value_frag<T>(tile, ld, 0, c0, r16, g), pf, o[i]);
+        o[i] = Frag<T>::mma(tile_value_frag<T>(tile, ld, 0, c0, r16, g), pf, o[i]);
       }
     } else {
 #pragma unroll
@@ -270,7 +247,7 @@ __global__ void __launch_bounds__(256 * lat_teams<T>()) latent_attn_kernel(const
 #pragma unroll
         for (int i = 0; i < NCT; i++) {
           const uint32_t c0 = wc + i * 16 < ld ? wc + i * 16 : ld - 16;
-          o[i] = Frag<T>::mma(lat_value_frag<T>(tile, ld, n, c0, r16, g), sa[n], o[i]);
+          o[i] = Frag<T>::mma(tile_value_frag<T>(tile, ld, n, c0, r16, g), sa[n], o[i]);
         }
     }
     }

@@ -1,6 +1,6 @@
 // layered.h — models whose layers are described one by one (lgh_layer_desc: a mixer and an optional feed-forward), on the engine's own
-// context, step function and graphs (internal).  Kernels: linear_bf16.hip (matrix products), latent_attention.hip, mlstm.hip,
-// layered_misc.hip (embedding, norms); layered.hip assembles them.
+// context, step function and graphs (internal).  Kernels: linear_bf16.hip (matrix products), latent_attention.hip, tied_attention.hip,
+// mlstm.hip, moe_route.hip (routing of the experts), layered_misc.hip (embedding, norms, residual updates); layered.hip assembles them.
 #pragma once
 
 #include "common.h"
@@ -19,6 +19,24 @@ struct LinW {
   size_t bytes() const { return (size_t)n * k * 2; }
 };
 
+// ---- residual form LGH_RESIDUAL_SANDWICH_DYT: h = dyt(x), h += conv(h), x += mult * dyt'(sublayer(h)); all of it per channel ----
+struct DytW { const float *w = nullptr, *b = nullptr, *alpha = nullptr; };     // tanh(alpha v) * w + b
+struct ConvW {                 // causal convolution, one filter per channel
+  const float* w = nullptr;    // [width][taps], the last tap at the token itself
+  float* hist = nullptr;       // [taps - 1][width]: the input at position p lies in row p % (taps - 1) until position p + taps - 1 replaces it
+  uint32_t taps = 0;           // 0: no convolution
+};
+struct PostUpdate {            // a token's residual update and the next sublayer's input (decode: in the epilogue of the product before it)
+  const float* x = nullptr;    // residual stream, updated to xout (may be the same vector)
+  float* xout = nullptr;
+  DytW post, next;
+  ConvW conv;
+  float* hout = nullptr;
+  const int* pos = nullptr;    // device word: the token's position
+  float mult = 1.0f;
+  uint32_t width = 0;
+};
+
 // What a decode mat-vec does to its input vector before the product (every workgroup, in LDS)
 enum LinPro : int {
   LP_COPY = 0,    // x
@@ -26,10 +44,19 @@ enum LinPro : int {
   LP_HEAD = 2,    // layer_norm of the same sum, times nw2 (final norm in front of the output projection)
   LP_MLSTM = 3,   // matrix-memory read-out: numerators / denominators, per-head RMS norm, norm weight, sigmoid gate
 };
+// Which weights its rows come from
+enum LinSrc : int {
+  LS_PLAIN = 0,
+  LS_TWO = 1,      // w, and below it w2 (plain rows, same input) -> out2; w may be absent
+  LS_EXPERTS = 2,  // the top experts of `logits` (every workgroup ranks them), their gate | up pairs; the input is weighted by the expert's score
+  LS_MOE_DOWN = 3, // input [shared | expert | expert ..]: a row is a row of w (shared, absent: kps = 0) followed by the same row of every chosen expert
+};
+enum LinAct : uint32_t { LA_GELU = 0, LA_SILU = 1 };
 struct LinMv {
   const uint16_t* w;
-  uint32_t n, kp, k, paired;
-  float* out;                  // [n], paired: [n / 2] = gelu(gate) * up
+  uint32_t n, kp, k, paired;   // paired: 0 or 1
+  float* out;                  // [n], paired: [n / 2] = act(gate) * up
+  uint32_t act;                // LinAct
   const float* x;
   const float* y;              // LP_RESID / LP_HEAD: the pending sublayer output
   const float* nw;             // its norm weight
@@ -39,8 +66,18 @@ struct LinMv {
   const float* num;            // LP_MLSTM: [heads][ldo] numerators, column vdim = n . q, column vdim + 1 = exp(-m)
   const float* gate;
   uint32_t heads, vdim, ldo;
+  const uint16_t* w2;          // LS_TWO: second matrix; LS_EXPERTS / LS_MOE_DOWN: the experts, one below the other
+  float* out2;
+  uint32_t n2;
+  const float* logits;         // LS_EXPERTS: [experts] router logits
+  uint32_t experts, top;
+  int* sel;                    // [top] chosen experts: written by LS_EXPERTS, read by LS_MOE_DOWN
+  uint64_t stride;             // elements between two experts
+  uint32_t kps, kpe;           // LS_MOE_DOWN: columns of the shared part and of an expert; LS_EXPERTS: an expert's outputs lie kpe apart
+  PostUpdate post;             // post.xout set: rows are not stored but update the residual stream
 };
-hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st);
+hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st, int src = LS_PLAIN);
+constexpr uint32_t kMaxExperts = 1024, kMaxTop = 64;
 constexpr uint32_t kLinMvMaxK = 36864;   // input vectors live in LDS
 
 // Matrix product of a block of tokens: out[m][n] = sum_k x[m][k] * w[n][k].  f32 = true: activations and products in 32-bit
@@ -51,6 +88,16 @@ enum LinEpi : int {
   LE_GEGLU = 2,   // paired weights: gelu(gate) * up as activation type [M][ldo]
   LE_HEADS = 3,   // activation type, row n = head * hd + j of token m at out[(head * tcap + m) * ldo + j]
   LE_HEADS_T = 4, // activation type, transposed per head: out[(head * hrows + j) * ldo + m]
+  LE_SWIGLU = 5,  // paired weights: silu(gate) * up as activation type [M][ldo]
+};
+// rows grouped by expert: row tile i takes rows tile_row[i] .. of the group tile_e[i] (-1: no tile), which ends at seg[group + 1]; that
+// group's weights lie `stride` elements per group behind w
+struct LinGroup {
+  const int *seg = nullptr, *tile_e = nullptr, *tile_row = nullptr;
+  const int* src = nullptr;        // row of x of every row (NULL: the same row)
+  const float* scale = nullptr;    // factor of every row's input (LE_SWIGLU)
+  uint64_t stride = 0;
+  uint32_t tiles = 0, bm = 0;      // row tiles (upper bound) and their height
 };
 struct LinGemm {
   const uint16_t* w;
@@ -59,8 +106,10 @@ struct LinGemm {
   uint32_t n, np, kp, ldx, ldo, M;
   uint32_t hd, hrows;          // LE_HEADS / LE_HEADS_T
   uint64_t tcap;
+  LinGroup grp;
 };
 hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st);
+uint32_t lin_group_rows(uint32_t rows, uint32_t groups);   // height of a grouped product's row tiles for this many rows over this many groups
 // upload: rows [row0, row0 + rows) of a bf16 matrix; mode 0 plain, 1 first half of a pair, 2 second half of a pair
 hipError_t lin_pack_launch(const uint16_t* src, uint32_t rows, uint32_t k, uint16_t* dst, uint32_t kp, uint32_t row0, int mode, hipStream_t st);
 // per head [dim][rank] -> [rank][dimp]
@@ -74,7 +123,8 @@ struct EmbedArgs {
   uint64_t mul_prev, mul_cur;
   int* hist;                   // token of every position (the previous token is part of the sequence's state)
 };
-hipError_t layered_embed_launch(const EmbedArgs& a, int* state, float* x, hipStream_t st);
+// post (may be NULL): also the first sublayer's input, LGH_RESIDUAL_SANDWICH_DYT
+hipError_t layered_embed_launch(const EmbedArgs& a, int* state, float* x, const PostUpdate* post, hipStream_t st);
 hipError_t layered_embed_block_launch(const EmbedArgs& a, const int* tokens, uint32_t pos0, uint32_t M, float* x, void* xa, uint32_t ldx, bool f32,
                                       hipStream_t st);
 // x += mult * layer_norm(y) * w; also as activations
@@ -85,6 +135,72 @@ hipError_t resid_norm_out_launch(const float* x, const float* y, const float* w,
 // rows[i] of x, layer-normed with w, as activations
 hipError_t final_norm_rows_launch(const float* x, const int* rows, uint32_t n_rows, const float* w, float eps, uint32_t width, void* xa, uint32_t ldx,
                                   bool f32, hipStream_t st);
+hipError_t final_dyt_rows_launch(const float* x, const int* rows, uint32_t n_rows, const DytW& n, uint32_t width, void* xa, uint32_t ldx, bool f32, hipStream_t st);
+
+// LGH_RESIDUAL_SANDWICH_DYT over a block: v = x + mult * dyt(y), y = `y` (may be NULL) plus a token's rows of `pairs` in slot order;
+// v -> xout (another buffer than x; NULL without a sublayer output: v = x), the next sublayer's input -> xa (NULL: none).  The inputs of
+// the convolution at the block's last taps - 1 positions go to `tail` [taps - 1][width], row i = i positions before the last.
+struct DytBlock {
+  const float* x;
+  float* xout;
+  const float* y;
+  uint32_t ldy;
+  const float* pairs;          // [M * top][ldp], with slot[t * top + s] = the row of token t's s-th expert; NULL: none
+  const int* slot;
+  uint32_t ldp, top;
+  DytW post, next;
+  ConvW conv;
+  float* tail;
+  void* xa;
+  uint32_t ldx, width, M, pos0;
+  float mult;
+};
+hipError_t dyt_block_launch(const DytBlock& a, bool f32, hipStream_t st);
+// after a block: tails [n_sub][taps - 1][width] -> histories [n_sub][taps - 1][width] (row of position p: p % (taps - 1))
+hipError_t conv_store_launch(const float* tails, float* hists, uint32_t n_sub, uint32_t taps, uint32_t width, uint32_t pos0, uint32_t M, hipStream_t st);
+// y[t] += a token's rows of `pairs` in slot order (a mixture in front of LGH_RESIDUAL_POST_LN); add = false: y[t] = the rows' sum
+hipError_t pair_sum_launch(float* y, uint32_t ldy, const float* pairs, uint32_t ldp, const int* slot, uint32_t top, uint32_t width, uint32_t M, bool add, hipStream_t st);
+
+// ---- moe_route.hip: a block's tokens to their experts ----
+struct MoeRoute {
+  const float* logits;         // [M][ldl]
+  uint32_t ldl, M, experts, top, bm;
+  int* sel;                    // [M * top] chosen experts, largest score first
+  float* w;                    // [M * top] their scores
+  int *seg, *tile_e, *tile_row;   // LinGroup, row tiles of bm rows
+  int *slot;                   // [M * top]: row of the pair
+  int *src;                    // [M * top]: token of the row
+  float* roww;                 // [M * top]: score of the row
+  uint32_t tiles;              // entries of tile_e / tile_row
+};
+uint32_t moe_max_tiles(uint32_t rows, uint32_t experts, uint32_t bm);
+hipError_t moe_route_launch(const MoeRoute& a, hipStream_t st);
+
+// ---- tied_attention.hip: grouped heads, values = keys before their norm ----
+struct TiedShape {
+  uint32_t heads, kv_heads, dim, dp;   // dp: row stride of the cache, multiple of 64
+  uint32_t off_q, off_k, ldcat;
+  uint32_t window, keep;               // i sees j <= i with i - j < window or j < keep
+  uint64_t rows;                       // cache rows per key head, multiple of 64
+  float scale, cap, eps;               // cap 0: none
+};
+struct TiedBufs {
+  const float* cat;                    // [M][ldcat]
+  const float *qn, *kn, *temp, *sink;  // norm weights [heads * dim], [kv_heads * dim]; per head
+  void* cache;                         // [kv_heads][rows][dp]: keys as projected
+  float* kinv;                         // [rows]: 1 / rms over all of a position's keys
+  void* q;                             // blocks: [heads][Mcap][dp], norm weights (of the key too), temp and scale in them
+  uint32_t Mcap;
+  float *part_ml, *part_acc;           // [split][M * heads][2], [split][M * heads][dim]
+};
+constexpr uint32_t kTiedMaxSplits = 128, kTiedShort = 16, kTiedMaxDim = 256;   // portions up to kTiedShort tokens take the decode kernel
+uint32_t tied_splits(const TiedShape& s, uint32_t max_seq, uint32_t M, bool f32, uint32_t forced);
+// one token (own = true: its key is taken from cat and written to the cache) or M tokens whose keys are in the cache
+hipError_t tied_attn_launch(const TiedShape& s, const TiedBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, bool own, uint32_t n_splits, bool f32, hipStream_t st);
+hipError_t tied_merge_launch(const TiedShape& s, const TiedBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32, void* out, uint32_t ldo,
+                             bool out_f32, hipStream_t st);
+hipError_t tied_prep_launch(const TiedShape& s, const TiedBufs& b, uint32_t pos0, uint32_t M, bool f32, hipStream_t st);
+hipError_t tied_flash_launch(const TiedShape& s, const TiedBufs& b, uint32_t pos0, uint32_t M, bool f32, void* out, uint32_t ldo, hipStream_t st);
 
 // ---- latent_attention.hip ----
 struct LatentShape {

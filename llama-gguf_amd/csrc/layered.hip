@@ -5,9 +5,14 @@
 //   latent attention   fused q | latent | gate product -> queries absorbed, cache row written -> split attention -> merge + value
 //                      expansion + gate -> output product
 //   mLSTM              fused q | k | v | gates product -> recurrence step -> output product (read-out norm and gate in its prologue)
+//   tied attention     fused q | k product -> split attention (norms of q and k in its prologue, cache row written) -> merge -> output product
 //   feed-forward       gate | up product with gelu * in its epilogue -> down product
-// A sequence's state: the cache rows, the matrix memories with their running maxima, and the last token (pair embedding), kept as a
-// token history by position; a position of 0 makes every kernel ignore what is stored, so lgh_reset stays O(1).
+//   mixture            shared gate | up + router product -> the chosen experts' gate | up (every workgroup ranks the scores) -> one down
+//                      product over [shared | experts]
+// With squashing norms (LGH_RESIDUAL_SANDWICH_DYT) everything between two sublayers is per channel: it rides in the EPILOGUE of the
+// product that finishes a channel, and no norm is computed more than once.
+// A sequence's state: the cache rows, the matrix memories with their running maxima, the convolutions' last inputs, and the last token
+// (pair embedding), kept as a token history by position; a position of 0 makes every kernel ignore what is stored, so lgh_reset stays O(1).
 #include <algorithm>
 #include <cmath>
 #include <map>
@@ -21,10 +26,16 @@ namespace lgh {
 
 constexpr uint32_t kBlockTokens = 2048;    // tokens per pass of the block path
 constexpr uint32_t kLogitRows = 128;       // wanted rows per output product
+constexpr uint32_t kMaxConvTaps = 64;
 
 struct LayeredLayer {
   lgh_layer_desc d{};
-  LinW in, out, gu, down, uk, uv;          // mixer inputs (one product), mixer output, gate | up, down, latent expansions
+  LinW in, out, gu, down, uk, uv;          // mixer inputs (one product), mixer output, gate | up, down (mixture: of the shared expert), latent expansions
+  LinW router, egu, edown;                 // mixture: router, the experts' gate | up and down, `egu_rows` and `edown_rows` rows each
+  uint32_t egu_rows = 0, edown_rows = 0;
+  float *qn = nullptr, *kn = nullptr, *temp = nullptr, *sink = nullptr, *kinv = nullptr;
+  uint32_t splits = 1;
+  TiedShape ts{};
   uint16_t* uk_t = nullptr;
   float *norm1 = nullptr, *norm2 = nullptr, *dkv_norm = nullptr, *mnorm = nullptr, *bi = nullptr, *bf = nullptr, *cs = nullptr;
   void* cache = nullptr;
@@ -33,6 +44,16 @@ struct LayeredLayer {
   LatentShape ls{};
   MlstmShape ms{};
   bool latent() const { return d.mixer == LGH_MIXER_LATENT_ATTENTION; }
+  bool mlstm() const { return d.mixer == LGH_MIXER_MLSTM; }
+  bool tied() const { return d.mixer == LGH_MIXER_TIED_ATTENTION; }
+  bool moe() const { return d.ff_kind == LGH_FF_MOE; }
+  uint32_t act_cols() const { return moe() ? down.kp + d.top * edown.kp : down.kp; }   // inputs of the down product
+};
+
+struct LayeredNorm { float *w = nullptr, *b = nullptr, *alpha = nullptr; };
+struct LayeredSub {                        // LGH_RESIDUAL_SANDWICH_DYT: what surrounds a sublayer
+  LayeredNorm pre, post;
+  float* conv = nullptr;
 };
 
 struct LayeredSlot {                       // where a named tensor goes
@@ -52,9 +73,27 @@ struct LayeredModel {
   uint16_t *embed = nullptr, *bigram = nullptr;
   LinW head;
   float* final_norm = nullptr;
-  int* hist = nullptr;
+  int* tokens = nullptr;                   // token of every position
   bool f32 = false, recurrent = false;
+  uint32_t forced_splits = 0;              // LGH_FLAG_ATTN_SPLITS_SHIFT
   uint32_t n_sub = 0, n_splits = 1;
+  // LGH_RESIDUAL_SANDWICH_DYT
+  std::vector<LayeredSub> subs;
+  LayeredNorm final_dyt;
+  float *h = nullptr, *hist = nullptr, *tails = nullptr;   // a sublayer's input (decode); the convolutions' histories and a block's last inputs
+  bool dyt() const { return d.residual == LGH_RESIDUAL_SANDWICH_DYT; }
+  size_t hist_floats() const { return d.conv_taps > 1 ? (size_t)n_sub * (d.conv_taps - 1) * d.width : 0; }
+  // mixtures
+  float* rlogits = nullptr;
+  int* sel = nullptr;
+  uint32_t max_experts = 0, max_top = 0, max_pair_act = 0;   // (the last: top * columns of an expert)
+  float *brl = nullptr, *bpair = nullptr, *bselw = nullptr, *broww = nullptr;
+  int *bsel = nullptr, *bseg = nullptr, *btile_e = nullptr, *btile_row = nullptr, *bslot = nullptr, *bsrc = nullptr;
+  void* bpact = nullptr;
+  // tied attention's queries of a block
+  uint32_t max_tied_q = 0;                 // heads * row
+  size_t max_tied_rows = 0, max_tied_acc = 0;   // partial sums: (token, head) rows * splits, and times the head size
+  void* btq = nullptr;
   // decode
   float *x[2] = {nullptr, nullptr}, *y = nullptr, *cat = nullptr, *ao = nullptr, *act = nullptr, *num = nullptr, *part_ml = nullptr, *part_acc = nullptr;
   void* qa = nullptr;
@@ -62,6 +101,7 @@ struct LayeredModel {
   // blocks
   bool blk_ready = false;
   uint32_t blk = 0;
+  float *bx2 = nullptr;                    // LGH_RESIDUAL_SANDWICH_DYT: the stream's second buffer
   float *bx = nullptr, *by = nullptr, *bcat = nullptr, *bnum = nullptr, *ba = nullptr, *blogits = nullptr;
   double *bu = nullptr, *bmx = nullptr;
   float *bdec = nullptr, *bwgt = nullptr, *bcdec = nullptr, *bnk = nullptr;
@@ -91,7 +131,7 @@ void layered_destroy(lgh_ctx* c) {
   delete c->lm;
   c->lm = nullptr;
 }
-bool layered_recurrent(const lgh_ctx* c) { return c->lm->recurrent; }
+bool layered_recurrent(const lgh_ctx* c) { return c->lm->recurrent || c->lm->d.conv_taps > 1; }
 bool layered_has_blocks(const lgh_ctx* c) { return !(c->d.flags & LGH_FLAG_EXACT_PREFILL); }
 
 // What the kernels can hold, checked before anything is allocated
@@ -100,13 +140,19 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
   if (d.compute > LGH_COMPUTE_F32) { why = "unknown compute type"; return LGH_INVALID_ARGUMENT; }
   if (!(d.norm_eps >= 0.0) || !std::isfinite(d.residual_mult)) { why = "norm_eps / residual_mult"; return LGH_INVALID_ARGUMENT; }
   if (up(d.width, 64) > 32768) { why = "width above 32768"; return LGH_UNSUPPORTED; }
+  if (d.residual > LGH_RESIDUAL_SANDWICH_DYT) { why = "unknown residual form"; return LGH_UNSUPPORTED; }
+  if (d.conv_taps > kMaxConvTaps || (d.conv_taps && d.residual != LGH_RESIDUAL_SANDWICH_DYT)) { why = "convolution taps"; return LGH_UNSUPPORTED; }
   for (uint32_t i = 0; i < d.num_layers; i++) {
     const lgh_layer_desc& l = L[i];
     const std::string at = "layer " + std::to_string(i) + ": ";
     if (l.struct_size != sizeof(lgh_layer_desc)) { why = at + "descriptor size"; return LGH_INVALID_ARGUMENT; }
     if (!l.heads || !l.dim || !l.vdim) { why = at + "a mixer dimension is zero"; return LGH_INVALID_ARGUMENT; }
-    if (l.ff_kind > LGH_FF_GEGLU || (l.ff_kind && !l.ff)) { why = at + "feed-forward"; return LGH_INVALID_ARGUMENT; }
-    if (l.ff_kind && up(l.ff, 64) > kLinMvMaxK) { why = at + "feed-forward above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
+    if (l.ff_kind > LGH_FF_MOE || (l.ff_kind && !l.ff)) { why = at + "feed-forward"; return LGH_INVALID_ARGUMENT; }
+    if (l.ff_kind == LGH_FF_MOE) {
+      if (!l.experts || !l.top || l.top > l.experts) { why = at + "experts"; return LGH_INVALID_ARGUMENT; }
+      if (l.experts > kMaxExperts || l.top > kMaxTop) { why = at + "more than " + std::to_string(kMaxExperts) + " experts or " + std::to_string(kMaxTop) + " per token"; return LGH_UNSUPPORTED; }
+      if ((uint64_t)up(l.shared_ff, 64) + (uint64_t)l.top * up(l.ff, 64) > kLinMvMaxK) { why = at + "a token's experts together above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
+    } else if (l.ff_kind && up(l.ff, 64) > kLinMvMaxK) { why = at + "feed-forward above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
     if (up(l.heads * l.vdim, 64) > kLinMvMaxK) { why = at + "heads * vdim above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
     if (l.mixer == LGH_MIXER_LATENT_ATTENTION) {
       if (!l.kv_rank || l.rot_dims > l.rot_dim || l.rot_dims % 2) { why = at + "latent attention sizes"; return LGH_INVALID_ARGUMENT; }
@@ -115,6 +161,9 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
       s.rank = l.kv_rank;
       s.ldc = up(l.kv_rank + l.rot_dim, 64);
       if (l.heads > kLatAbsorbRows || !latent_fits(s, d.compute == LGH_COMPUTE_F32)) { why = at + "latent rows too large for LDS"; return LGH_UNSUPPORTED; }
+    } else if (l.mixer == LGH_MIXER_TIED_ATTENTION) {
+      if (!l.kv_heads || l.heads % l.kv_heads || l.vdim != l.dim || !(l.score_cap >= 0.0)) { why = at + "tied attention sizes"; return LGH_INVALID_ARGUMENT; }
+      if (up(l.dim, 64) > kTiedMaxDim) { why = at + "heads above " + std::to_string(kTiedMaxDim); return LGH_UNSUPPORTED; }
     } else if (l.mixer == LGH_MIXER_MLSTM) {
       if (!(l.gate_cap > 0.0)) { why = at + "gate_cap"; return LGH_INVALID_ARGUMENT; }
     } else { why = at + "unknown mixer"; return LGH_UNSUPPORTED; }
@@ -140,6 +189,23 @@ static void add_vec(LayeredModel& m, const std::string& nm, float** v, uint32_t 
   m.slots[nm] = s;
 }
 
+// a norm of LGH_RESIDUAL_SANDWICH_DYT: weight, bias and the factor inside
+static void add_dyt(LayeredModel& m, const std::string& nm, LayeredNorm& n) {
+  add_vec(m, nm, &n.w, m.d.width);
+  add_vec(m, nm + ".b", &n.b, m.d.width);
+  add_vec(m, nm + ".alpha", &n.alpha, 1);
+}
+// the norms around a sublayer ("1": mixer, "2": feed-forward)
+static void add_sub(LayeredModel& m, const std::string& p, const char* which, float** post_ln) {
+  m.n_sub++;
+  if (!m.dyt()) { add_vec(m, p + "norm" + which, post_ln, m.d.width); return; }
+  m.subs.emplace_back();                   // (never grows beyond what was reserved: the slots keep addresses)
+  LayeredSub& s = m.subs.back();
+  add_dyt(m, p + "norm" + which, s.pre);
+  add_dyt(m, p + "norm" + which + "b", s.post);
+  if (m.d.conv_taps) add_vec(m, p + "canon" + which, &s.conv, m.d.width * m.d.conv_taps);
+}
+
 // sizes, offsets and the tensor table of every layer
 static void layered_plan(LayeredModel& m) {
   const lgh_layered_desc& d = m.d;
@@ -151,12 +217,12 @@ static void layered_plan(LayeredModel& m) {
     if (d.bigram_buckets) { s.raw = &m.bigram; s.n = d.bigram_buckets + 1; m.slots["bigram"] = s; }
   }
   auto whole = [&](LinW& L, uint32_t n, uint32_t k) { L.n = n; L.k = k; L.kp = up(k, 64); };
+  m.subs.reserve(2 * (size_t)d.num_layers);
   for (uint32_t i = 0; i < d.num_layers; i++) {
     LayeredLayer& L = m.layers[i];
     const lgh_layer_desc& l = L.d;
     const std::string p = "l" + std::to_string(i) + ".";
-    add_vec(m, p + "norm1", &L.norm1, W);
-    m.n_sub++;
+    add_sub(m, p, "1", &L.norm1);
     L.in.k = W; L.in.kp = up(W, 64);
     const uint32_t vd = l.heads * l.vdim;
     auto in_seg = [&](const char* nm, uint32_t rows) { const uint32_t at = seg(L.in, rows); add_mat(m, p + "mix." + nm, &L.in, at, rows, W); return at; };
@@ -178,6 +244,27 @@ static void layered_plan(LayeredModel& m) {
       add_mat(m, p + "mix.uk", &L.uk, 0, L.uk.n, l.kv_rank);
       m.slots[p + "mix.uk"].transpose = &L;
       add_mat(m, p + "mix.uv", &L.uv, 0, vd, l.kv_rank);
+    } else if (L.tied()) {
+      TiedShape& s = L.ts;
+      s.heads = l.heads; s.kv_heads = l.kv_heads; s.dim = l.dim; s.dp = up(l.dim, 64);
+      s.window = l.window ? l.window : 0xFFFFFFFFu; s.keep = l.keep_first;
+      s.rows = up(d.max_seq_len, 64);
+      s.scale = (float)l.scale; s.cap = (float)l.score_cap; s.eps = (float)d.norm_eps;
+      s.off_q = in_seg("q", vd);
+      s.off_k = in_seg("k", l.kv_heads * l.dim);
+      L.in.n = up(L.in.n, 16);
+      s.ldcat = L.in.n;
+      add_vec(m, p + "mix.q.norm", &L.qn, vd);
+      add_vec(m, p + "mix.k.norm", &L.kn, l.kv_heads * l.dim);
+      add_vec(m, p + "mix.temp", &L.temp, l.heads);
+      add_vec(m, p + "mix.sink", &L.sink, l.heads);
+      L.splits = tied_splits(s, d.max_seq_len, 1, m.f32, m.forced_splits);
+      for (uint32_t t = 1; t <= kTiedShort; t++) {
+        const size_t rows = (size_t)t * l.heads * tied_splits(s, d.max_seq_len, t, m.f32, m.forced_splits);
+        m.max_tied_rows = std::max(m.max_tied_rows, rows);
+        m.max_tied_acc = std::max(m.max_tied_acc, rows * l.dim);
+      }
+      m.max_tied_q = std::max(m.max_tied_q, l.heads * s.dp);
     } else {
       MlstmShape& s = L.ms;
       s.heads = l.heads; s.dim = l.dim; s.vdim = l.vdim;
@@ -201,9 +288,35 @@ static void layered_plan(LayeredModel& m) {
     whole(L.out, W, vd);
     add_mat(m, p + "mix.o", &L.out, 0, W, vd);
     m.max_ao = std::max(m.max_ao, L.out.kp);
-    if (l.ff_kind) {
-      m.n_sub++;
-      add_vec(m, p + "norm2", &L.norm2, W);
+    if (L.moe()) {
+      add_sub(m, p, "2", &L.norm2);
+      whole(L.router, l.experts, W);
+      add_mat(m, p + "mlp.router", &L.router, 0, l.experts, W);
+      L.egu_rows = 2 * up(l.ff, 16);
+      L.edown_rows = up(W, 16);
+      whole(L.egu, l.experts * L.egu_rows, W);
+      L.egu.paired = true;
+      whole(L.edown, l.experts * L.edown_rows, l.ff);
+      for (uint32_t e = 0; e < l.experts; e++) {
+        const std::string pe = p + "mlp.e" + std::to_string(e) + ".";
+        add_mat(m, pe + "gate", &L.egu, e * L.egu_rows, l.ff, W, 1);
+        add_mat(m, pe + "up", &L.egu, e * L.egu_rows, l.ff, W, 2);
+        add_mat(m, pe + "down", &L.edown, e * L.edown_rows, W, l.ff);
+      }
+      if (l.shared_ff) {
+        whole(L.gu, 2 * up(l.shared_ff, 16), W);
+        L.gu.paired = true;
+        add_mat(m, p + "mlp.shared.gate", &L.gu, 0, l.shared_ff, W, 1);
+        add_mat(m, p + "mlp.shared.up", &L.gu, 0, l.shared_ff, W, 2);
+        whole(L.down, W, l.shared_ff);
+        add_mat(m, p + "mlp.shared.down", &L.down, 0, W, l.shared_ff);
+      }
+      m.max_act = std::max(m.max_act, L.act_cols());
+      m.max_experts = std::max(m.max_experts, l.experts);
+      m.max_top = std::max(m.max_top, l.top);
+      m.max_pair_act = std::max(m.max_pair_act, l.top * L.edown.kp);
+    } else if (l.ff_kind) {
+      add_sub(m, p, "2", &L.norm2);
       whole(L.gu, 2 * up(l.ff, 16), W);
       L.gu.paired = true;
       add_mat(m, p + "mlp.gate", &L.gu, 0, l.ff, W, 1);
@@ -213,7 +326,8 @@ static void layered_plan(LayeredModel& m) {
       m.max_act = std::max(m.max_act, L.down.kp);
     }
   }
-  add_vec(m, "final.norm", &m.final_norm, W);
+  if (m.dyt()) add_dyt(m, "final.norm", m.final_dyt);
+  else add_vec(m, "final.norm", &m.final_norm, W);
   whole(m.head, d.vocab_size, W);
   add_mat(m, "head", &m.head, 0, d.vocab_size, W);
 }
@@ -243,6 +357,7 @@ extern "C" int lgh_create_layered(const lgh_layered_desc* desc, const lgh_layer_
   c->lm = m;
   m->d = *desc;
   m->f32 = desc->compute == LGH_COMPUTE_F32;
+  m->forced_splits = (desc->flags >> LGH_FLAG_ATTN_SPLITS_SHIFT) & 0xFFu;
   m->layers.resize(d.num_layers);
   for (uint32_t i = 0; i < d.num_layers; i++) m->layers[i].d = layers[i];
   layered_plan(*m);
@@ -351,12 +466,15 @@ int layered_finalize(lgh_ctx* c) {
         if (!cs.empty()) L_TRY(c, LGH_OPERATION_FAILED, hipMemcpy(L.cs, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
       }
       max_rows = std::max(max_rows, L.ls.heads); max_rank = std::max(max_rank, L.ls.rank); max_ldc = std::max(max_ldc, L.ls.ldc);
+    } else if (L.tied()) {
+      if ((rc = zeroed(c, &L.cache, (size_t)L.ts.kv_heads * L.ts.rows * L.ts.dp * m.el(), &c->stats.kv_bytes))) return rc;
+      if ((rc = zeroed(c, (void**)&L.kinv, (size_t)L.ts.rows * 4, &c->stats.kv_bytes))) return rc;
     } else {
       if ((rc = zeroed(c, (void**)&L.S, (size_t)L.ms.heads * L.ms.dim * L.ms.lds * 4, &c->stats.kv_bytes))) return rc;
       if ((rc = zeroed(c, (void**)&L.m, (size_t)2 * L.ms.heads * 8, &c->stats.kv_bytes))) return rc;
     }
   }
-  uint32_t splits = (c->d.flags >> LGH_FLAG_ATTN_SPLITS_SHIFT) & 0xFFu;
+  uint32_t splits = m.forced_splits;
   // enough splits that a long context's workgroups cover the chip; no more, since every split's partial sums are merged
   if (!splits) splits = std::min(512 / std::max(1u, (max_rows + 15) / 16), std::min(std::max(d.max_seq_len / 128, 64u), kLatMaxSplits));
   m.n_splits = std::max(1u, std::min(splits, kLatMaxSplits));
@@ -367,13 +485,15 @@ int layered_finalize(lgh_ctx* c) {
       {(void**)&m.x[0], (size_t)d.width * 4}, {(void**)&m.x[1], (size_t)d.width * 4}, {(void**)&m.y, (size_t)up(d.width, 16) * 4},
       {(void**)&m.cat, (size_t)m.max_cat * 4}, {(void**)&m.ao, (size_t)m.max_ao * 4}, {(void**)&m.act, (size_t)m.max_act * 4},
       {(void**)&m.num, (size_t)m.max_num * 4}, {(void**)&m.qa, rows * max_ldc * m.el()},
-      {(void**)&m.part_ml, rows * m.n_splits * 2 * 4}, {(void**)&m.part_acc, rows * m.n_splits * max_rank * 4},
-      {(void**)&m.hist, (size_t)d.max_seq_len * 4}, {(void**)&c->logits, (size_t)d.vocab_size * 4}, {(void**)&c->state, ST_WORDS * 4},
+      {(void**)&m.part_ml, std::max(rows * m.n_splits, m.max_tied_rows) * 2 * 4}, {(void**)&m.part_acc, std::max(rows * m.n_splits * max_rank, m.max_tied_acc) * 4},
+      {(void**)&m.tokens, (size_t)d.max_seq_len * 4}, {(void**)&m.h, m.dyt() ? (size_t)up(d.width, 16) * 4 : 0}, {(void**)&m.hist, m.hist_floats() * 4},
+      {(void**)&m.rlogits, (size_t)m.max_experts * 4}, {(void**)&m.sel, (size_t)m.max_top * 4}, {(void**)&c->logits, (size_t)d.vocab_size * 4}, {(void**)&c->state, ST_WORDS * 4},
       {(void**)&c->amax_v, 64 * 4}, {(void**)&c->amax_i, 64 * 4}, {(void**)&c->tok_log, (size_t)d.max_seq_len * 4},
   };
   for (auto& b : bufs)
     if ((rc = zeroed(c, b.p, b.n, sb))) return rc;
-  c->hidden = m.x[m.n_sub & 1];   // where the residual stream ends up: every sublayer's update swaps the two vectors
+  // where the residual stream ends up: every sublayer's update swaps the two vectors; channel by channel it stays in place
+  c->hidden = m.dyt() ? m.x[0] : m.x[m.n_sub & 1];
   L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
   return LGH_OK;
 }
@@ -381,7 +501,7 @@ int layered_finalize(lgh_ctx* c) {
 static EmbedArgs embed_args(const LayeredModel& m) {
   EmbedArgs a{};
   a.embed = m.embed; a.bigram = m.bigram; a.width = m.d.width; a.buckets = m.d.bigram_buckets;
-  a.mul_prev = m.d.bigram_mul_prev; a.mul_cur = m.d.bigram_mul_cur; a.hist = m.hist;
+  a.mul_prev = m.d.bigram_mul_prev; a.mul_cur = m.d.bigram_mul_cur; a.hist = m.tokens;
   return a;
 }
 
@@ -398,8 +518,42 @@ static MlstmBufs mlstm_bufs(const LayeredModel& m, const LayeredLayer& L, const 
   return b;
 }
 
+static TiedBufs tied_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat) {
+  TiedBufs b{};
+  b.cat = cat; b.qn = L.qn; b.kn = L.kn; b.temp = L.temp; b.sink = L.sink; b.cache = L.cache; b.kinv = L.kinv;
+  b.part_ml = m.part_ml; b.part_acc = m.part_acc;
+  return b;
+}
+static DytW dyt_w(const LayeredNorm& n) {
+  DytW r;
+  r.w = n.w; r.b = n.b; r.alpha = n.alpha;
+  return r;
+}
+// the convolution in front of sublayer i
+static ConvW conv_w(const LayeredModel& m, uint32_t i) {
+  ConvW r;
+  if (!m.d.conv_taps) return r;
+  r.w = m.subs[i].conv; r.taps = m.d.conv_taps;
+  r.hist = m.d.conv_taps > 1 ? m.hist + (size_t)i * (m.d.conv_taps - 1) * m.d.width : nullptr;
+  return r;
+}
+// decode: what the product that ends sublayer i does to the stream, up to the input of sublayer i + 1 (the last one: of the output projection)
+static PostUpdate post_update(const lgh_ctx* c, int i) {
+  const LayeredModel& m = *c->lm;
+  PostUpdate p;
+  p.x = m.x[0]; p.xout = m.x[0]; p.hout = m.h; p.pos = c->state + ST_POS; p.mult = (float)m.d.residual_mult; p.width = m.d.width;
+  if (i >= 0) p.post = dyt_w(m.subs[i].post);
+  if (i + 1 < (int)m.n_sub) { p.next = dyt_w(m.subs[i + 1].pre); p.conv = conv_w(m, i + 1); }
+  else p.next = dyt_w(m.final_dyt);
+  return p;
+}
+
 // bytes of one token's attention / recurrence in a layer at the current position
 static uint64_t mixer_bytes(const lgh_ctx* c, const LayeredLayer& L) {
+  if (L.tied()) {
+    const uint64_t p = c->pos + 1, w = std::min<uint64_t>(p, L.ts.window), n = w + std::min<uint64_t>(L.ts.keep, p - w);
+    return n * ((uint64_t)L.ts.kv_heads * L.ts.dim * c->lm->el() + 4);
+  }
   if (L.latent()) return (uint64_t)(c->pos + 1) * (L.ls.rank + L.ls.rot_dim) * c->lm->el();
   return (uint64_t)L.ms.heads * L.ms.dim * (L.ms.vdim + 1) * 8;   // state read and written
 }
@@ -409,16 +563,25 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
   hipStream_t st = c->stream;
   const int* pos = c->state + ST_POS;
   int rc;
-  if ((rc = run_k(c, LGH_K_EMBED, LGH_SYM_EMBED, (uint64_t)m.d.width * 4, [&] { return layered_embed_launch(embed_args(m), c->state, m.x[0], st); }))) return rc;
+  if ((rc = run_k(c, LGH_K_EMBED, LGH_SYM_EMBED, (uint64_t)m.d.width * 4, [&] {
+         const PostUpdate first = m.dyt() ? post_update(c, -1) : PostUpdate();
+         return layered_embed_launch(embed_args(m), c->state, m.x[0], m.dyt() ? &first : nullptr, st);
+       })))
+    return rc;
   uint32_t cur = 0;
+  int sub = 0;
   const float* pend = nullptr;   // norm weight of the sublayer output waiting in m.y
   auto mv = [&](int cls, const LinW& W, float* out, LinMv a, int pro) {
     a.w = W.w; a.n = W.n; a.kp = W.kp; a.k = W.k; a.paired = W.paired; a.out = out;
     return run_k(c, cls, LGH_SYM_LINEAR, W.bytes(), [&] { return lin_mv_launch(pro, a, st); });
   };
-  auto mv_x = [&](int cls, const LinW& W, float* out, const float* nw2 = nullptr) -> int {   // a product that reads the residual stream
-    LinMv a{};
-    a.x = m.x[cur];
+  auto mv_end = [&](int cls, const LinW& W, LinMv a, int pro, float* norm) {   // the product that ends a sublayer
+    if (m.dyt()) a.post = post_update(c, sub++);
+    else pend = norm;
+    return mv(cls, W, m.y, a, pro);
+  };
+  auto read = [&](LinMv& a, const float* nw2 = nullptr) -> int {   // a product's input: the residual stream, or what was made of it
+    a.x = m.dyt() ? m.h : m.x[cur];
     int pro = LP_COPY;
     if (pend) {
       a.y = m.y; a.nw = pend; a.nw2 = nw2; a.xout = m.x[cur ^ 1]; a.eps = (float)m.d.norm_eps; a.mult = (float)m.d.residual_mult;
@@ -426,6 +589,11 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
       cur ^= 1;
       pend = nullptr;
     }
+    return pro;
+  };
+  auto mv_x = [&](int cls, const LinW& W, float* out, const float* nw2 = nullptr) {
+    LinMv a{};
+    const int pro = read(a, nw2);
     return mv(cls, W, out, a, pro);
   };
   for (LayeredLayer& L : m.layers) {
@@ -440,23 +608,46 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
         return rc;
       LinMv a{};
       a.x = m.ao;
-      if ((rc = mv(LGH_K_WO, L.out, m.y, a, LP_COPY))) return rc;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
+    } else if (L.tied()) {
+      const TiedBufs b = tied_bufs(m, L, m.cat);
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_TIED, mixer_bytes(c, L), [&] { return tied_attn_launch(L.ts, b, pos, 0, 1, true, L.splits, m.f32, st); }))) return rc;
+      if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_TIED, 0, [&] { return tied_merge_launch(L.ts, b, pos, 0, 1, L.splits, m.f32, m.ao, 0, true, st); }))) return rc;
+      LinMv a{};
+      a.x = m.ao;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
     } else {
       const MlstmBufs b = mlstm_bufs(m, L, m.cat, m.num);
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_MLSTM, mixer_bytes(c, L), [&] { return mlstm_step_launch(L.ms, b, pos, st); }))) return rc;
       LinMv a{};
       a.num = m.num; a.nw = L.mnorm; a.gate = m.cat + L.ms.off_g; a.heads = L.ms.heads; a.vdim = L.ms.vdim; a.ldo = L.ms.ldo; a.eps = L.ms.eps;
-      if ((rc = mv(LGH_K_WO, L.out, m.y, a, LP_MLSTM))) return rc;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_MLSTM, L.norm1))) return rc;
     }
-    pend = L.norm1;
-    if (L.d.ff_kind) {
+    if (L.moe()) {
+      LinMv a{};                           // shared gate | up (when there is one) and the router
+      const int pro = read(a);
+      a.w = L.gu.w; a.n = L.gu.n; a.paired = L.gu.paired; a.kp = L.router.kp; a.k = L.router.k; a.act = LA_SILU; a.out = m.act;
+      a.w2 = L.router.w; a.n2 = L.router.n; a.out2 = m.rlogits;
+      if ((rc = run_k(c, LGH_K_GATEUP, LGH_SYM_LINEAR, L.gu.bytes() + L.router.bytes(), [&] { return lin_mv_launch(pro, a, st, LS_TWO); }))) return rc;
+      LinMv e{};                           // the chosen experts' gate | up
+      e.x = m.dyt() ? m.h : m.x[cur];
+      e.w2 = L.egu.w; e.n = L.egu_rows; e.paired = 1; e.kp = L.egu.kp; e.k = L.egu.k; e.act = LA_SILU; e.out = m.act + L.down.kp;
+      e.logits = m.rlogits; e.experts = L.d.experts; e.top = L.d.top; e.sel = m.sel; e.stride = (uint64_t)L.egu_rows * L.egu.kp; e.kpe = L.edown.kp;
+      if ((rc = run_k(c, LGH_K_EXPERTS, LGH_SYM_LINEAR, L.egu.bytes() / L.d.experts * L.d.top, [&] { return lin_mv_launch(LP_COPY, e, st, LS_EXPERTS); }))) return rc;
+      LinMv o{};
+      o.x = m.act; o.w = L.down.w; o.n = m.d.width; o.kp = o.k = L.act_cols(); o.kps = L.down.kp; o.out = m.y;
+      o.w2 = L.edown.w; o.top = L.d.top; o.sel = m.sel; o.stride = (uint64_t)L.edown_rows * L.edown.kp; o.kpe = L.edown.kp;
+      if (m.dyt()) o.post = post_update(c, sub++);
+      else pend = L.norm2;
+      if ((rc = run_k(c, LGH_K_DOWN, LGH_SYM_LINEAR, L.down.bytes() + L.edown.bytes() / L.d.experts * L.d.top, [&] { return lin_mv_launch(LP_COPY, o, st, LS_MOE_DOWN); }))) return rc;
+    } else if (L.d.ff_kind) {
       if ((rc = mv_x(LGH_K_GATEUP, L.gu, m.act))) return rc;
       LinMv a{};
       a.x = m.act;
-      if ((rc = mv(LGH_K_DOWN, L.down, m.y, a, LP_COPY))) return rc;
-      pend = L.norm2;
+      if ((rc = mv_end(LGH_K_DOWN, L.down, a, LP_COPY, L.norm2))) return rc;
     }
   }
+  if (mode == MODE_PREFILL && m.dyt()) return LGH_OK;
   if (mode == MODE_PREFILL)
     return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
       return resid_norm_out_launch(m.x[cur], m.y, pend, (float)m.d.norm_eps, (float)m.d.residual_mult, m.d.width, m.x[cur ^ 1], st);
@@ -476,6 +667,7 @@ uint64_t layered_step_bytes(const lgh_ctx* c) {
     b += L.in.bytes() + L.out.bytes() + mixer_bytes(c, L) + (uint64_t)m.d.width * 4;
     if (L.latent()) b += L.uk.bytes() + L.uv.bytes();
     if (L.d.ff_kind) b += L.gu.bytes() + L.down.bytes() + (uint64_t)m.d.width * 4;
+    if (L.moe()) b += L.router.bytes() + (L.egu.bytes() + L.edown.bytes()) / L.d.experts * L.d.top;
   }
   return b;
 }
@@ -490,13 +682,19 @@ static int block_ensure(lgh_ctx* c) {
   m.blk = std::min(kBlockTokens, d.max_seq_len);
   uint32_t heads = 0, hdim = 0;
   for (auto& L : m.layers)
-    if (!L.latent()) { heads = std::max(heads, L.ms.heads); hdim = std::max(hdim, L.ms.heads * L.ms.dim); }
+    if (L.mlstm()) { heads = std::max(heads, L.ms.heads); hdim = std::max(hdim, L.ms.heads * L.ms.dim); }
+  const size_t moe_tiles = moe_max_tiles(m.blk * m.max_top, std::max(m.max_experts, 1u), 16);
   const size_t B = m.blk, chunks = (B + 63) / 64, Bc = chunks * 64, el = m.el();
   struct { void** p; size_t n; } bufs[] = {
       {(void**)&m.bx, B * d.width * 4}, {&m.bxa, B * up(d.width, 64) * el}, {(void**)&m.by, B * up(d.width, 4) * 4},
       {(void**)&m.bcat, (B * m.max_cat + kMlstmRowSlack) * 4}, {&m.bao, B * m.max_ao * el}, {&m.bact, B * m.max_act * el},
       {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * Bc * 8}, {(void**)&m.bmx, heads * Bc * 8},
       {(void**)&m.bdec, heads * Bc * 4}, {(void**)&m.bwgt, heads * Bc * 4}, {(void**)&m.bcdec, heads * chunks * 4}, {(void**)&m.bnk, chunks * hdim * 4},
+      {(void**)&m.bx2, m.dyt() ? B * d.width * 4 : 0}, {(void**)&m.tails, m.hist_floats() * 4}, {&m.btq, B * m.max_tied_q * el},
+      {(void**)&m.brl, B * up(m.max_experts, 4) * 4}, {(void**)&m.bpair, B * m.max_top * up(d.width, 4) * 4}, {&m.bpact, B * m.max_pair_act * el},
+      {(void**)&m.bsel, B * m.max_top * 4}, {(void**)&m.bselw, B * m.max_top * 4}, {(void**)&m.bslot, B * m.max_top * 4}, {(void**)&m.bsrc, B * m.max_top * 4},
+      {(void**)&m.broww, B * m.max_top * 4}, {(void**)&m.bseg, (size_t)(m.max_experts + 1) * 4}, {(void**)&m.btile_e, m.max_top ? moe_tiles * 4 : 0},
+      {(void**)&m.btile_row, m.max_top ? moe_tiles * 4 : 0},
       {(void**)&m.btok, B * 4}, {(void**)&m.brows, B * 4}, {&m.bla, (size_t)kLogitRows * up(d.width, 64) * el},
       {(void**)&m.blogits, (size_t)kLogitRows * up(d.vocab_size, 4) * 4},
   };
@@ -568,6 +766,47 @@ static int block_latent(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) 
   return LGH_OK;
 }
 
+static int block_tied(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) {
+  LayeredModel& m = *c->lm;
+  hipStream_t st = c->stream;
+  int rc;
+  TiedBufs b = tied_bufs(m, L, m.bcat);
+  const bool flash = M > kTiedShort;
+  if (flash) { b.q = m.btq; b.Mcap = m.blk; }
+  if ((rc = run_k(c, LGH_K_EXPAND, LGH_SYM_TIED, 0, [&] { return tied_prep_launch(L.ts, b, pos0, M, m.f32, st); }))) return rc;
+  if (flash) return run_k(c, LGH_K_ATTN, LGH_SYM_TIED, 0, [&] { return tied_flash_launch(L.ts, b, pos0, M, m.f32, m.bao, L.out.kp, st); });
+  const uint32_t splits = tied_splits(L.ts, m.d.max_seq_len, M, m.f32, m.forced_splits);
+  if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_TIED, 0, [&] { return tied_attn_launch(L.ts, b, nullptr, pos0, M, false, splits, m.f32, st); }))) return rc;
+  return run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_TIED, 0, [&] { return tied_merge_launch(L.ts, b, nullptr, pos0, M, splits, m.f32, m.bao, L.out.kp, m.f32, st); });
+}
+
+// routed experts of a block: the pairs' outputs -> m.bpair, rows m.bslot; the shared expert -> m.by
+static int block_moe(lgh_ctx* c, LayeredLayer& L, uint32_t ldx, uint32_t ldy, uint32_t M) {
+  LayeredModel& m = *c->lm;
+  hipStream_t st = c->stream;
+  int rc;
+  const uint32_t E = L.d.experts, rows = M * L.d.top;
+  if ((rc = block_gemm(c, LGH_K_ROUTER, L.router, LE_F32, m.bxa, ldx, m.brl, up(E, 4), M))) return rc;
+  MoeRoute r{};
+  r.logits = m.brl; r.ldl = up(E, 4); r.M = M; r.experts = E; r.top = L.d.top; r.bm = lin_group_rows(rows, std::min(rows, E));
+  r.sel = m.bsel; r.w = m.bselw; r.seg = m.bseg; r.tile_e = m.btile_e; r.tile_row = m.btile_row; r.slot = m.bslot; r.src = m.bsrc; r.roww = m.broww;
+  r.tiles = moe_max_tiles(rows, E, r.bm);
+  if ((rc = run_k(c, LGH_K_ROUTER, LGH_SYM_OTHER, 0, [&] { return moe_route_launch(r, st); }))) return rc;
+  LinGemm g{};
+  g.grp.seg = r.seg; g.grp.tile_e = r.tile_e; g.grp.tile_row = r.tile_row; g.grp.tiles = r.tiles; g.grp.bm = r.bm;
+  g.w = L.egu.w; g.n = g.np = L.egu_rows; g.kp = L.egu.kp; g.M = rows; g.x = m.bxa; g.ldx = ldx; g.out = m.bpact; g.ldo = L.edown.kp;
+  g.grp.src = r.src; g.grp.scale = r.roww; g.grp.stride = (uint64_t)L.egu_rows * L.egu.kp;
+  if ((rc = run_k(c, LGH_K_EXPERTS, LGH_SYM_LINEAR, L.egu.bytes(), [&] { return lin_gemm_launch(LE_SWIGLU, m.f32, g, st); }))) return rc;
+  g.w = L.edown.w; g.n = m.d.width; g.np = L.edown_rows; g.kp = L.edown.kp; g.x = m.bpact; g.ldx = L.edown.kp; g.out = m.bpair; g.ldo = ldy;
+  g.grp.src = nullptr; g.grp.scale = nullptr; g.grp.stride = (uint64_t)L.edown_rows * L.edown.kp;
+  if ((rc = run_k(c, LGH_K_DOWN, LGH_SYM_LINEAR, L.edown.bytes(), [&] { return lin_gemm_launch(LE_F32, m.f32, g, st); }))) return rc;
+  if (L.d.shared_ff) {
+    if ((rc = block_gemm(c, LGH_K_GATEUP, L.gu, LE_SWIGLU, m.bxa, ldx, m.bact, L.down.kp, M))) return rc;
+    if ((rc = block_gemm(c, LGH_K_DOWN, L.down, LE_F32, m.bact, L.down.kp, m.by, ldy, M))) return rc;
+  }
+  return LGH_OK;
+}
+
 static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint32_t* want, uint32_t n_want, float* logits_out) {
   LayeredModel& m = *c->lm;
   const lgh_layered_desc& d = m.d;
@@ -580,7 +819,32 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
          return layered_embed_block_launch(embed_args(m), m.btok, pos0, M, m.bx, m.bxa, ldx, m.f32, st);
        })))
     return rc;
-  auto resid = [&](const float* nw) {
+  float* xs = m.bx;                        // the residual stream
+  uint32_t sub = 0;
+  // LGH_RESIDUAL_SANDWICH_DYT: the sublayer's output into the stream, then the next sublayer's input; from_embed: the latter alone
+  auto resid_dyt = [&](bool from_embed, const LayeredLayer* moe) {
+    DytBlock b{};
+    b.x = xs; b.width = d.width; b.M = M; b.pos0 = pos0; b.mult = mult; b.ldx = ldx;
+    if (!from_embed) {
+      b.xout = xs == m.bx ? m.bx2 : m.bx;
+      b.post = dyt_w(m.subs[sub++].post);
+      if (!moe || moe->d.shared_ff) { b.y = m.by; b.ldy = ldy; }
+      if (moe) { b.pairs = m.bpair; b.ldp = ldy; b.slot = m.bslot; b.top = moe->d.top; }
+      xs = b.xout;
+    }
+    if (sub < m.n_sub) {
+      b.next = dyt_w(m.subs[sub].pre); b.conv = conv_w(m, sub); b.xa = m.bxa;
+      b.tail = m.hist_floats() ? m.tails + (size_t)sub * (d.conv_taps - 1) * d.width : nullptr;
+    }
+    return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, (uint64_t)M * d.width * 14, [&] { return dyt_block_launch(b, m.f32, st); });
+  };
+  if (m.dyt() && (rc = resid_dyt(true, nullptr))) return rc;
+  auto resid = [&](const float* nw, const LayeredLayer* moe = nullptr) -> int {
+    if (m.dyt()) return resid_dyt(false, moe);
+    if (moe && (rc = run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
+                  return pair_sum_launch(m.by, ldy, m.bpair, ldy, m.bslot, moe->d.top, d.width, M, moe->d.shared_ff != 0, st);
+                })))
+      return rc;
     return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, (uint64_t)M * d.width * 14, [&] {
       return resid_norm_launch(m.bx, m.by, ldy, nw, eps, mult, d.width, M, m.bxa, ldx, m.f32, st);
     });
@@ -590,6 +854,8 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
     if ((rc = block_gemm(c, LGH_K_QKV, L.in, LE_F32, m.bxa, ldx, m.bcat, L.in.n, M))) return rc;
     if (L.latent()) {
       if ((rc = block_latent(c, L, pos0, M))) return rc;
+    } else if (L.tied()) {
+      if ((rc = block_tied(c, L, pos0, M))) return rc;
     } else {
       const MlstmBufs b = mlstm_bufs(m, L, m.bcat, m.bnum);
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_MLSTM, 0, [&] { return mlstm_block_launch(L.ms, b, pos0, M, st); }))) return rc;
@@ -597,20 +863,30 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
     }
     if ((rc = block_gemm(c, LGH_K_WO, L.out, LE_F32, m.bao, L.out.kp, m.by, ldy, M))) return rc;
     if ((rc = resid(L.norm1))) return rc;
-    if (L.d.ff_kind) {
+    if (L.moe()) {
+      if ((rc = block_moe(c, L, ldx, ldy, M))) return rc;
+      if ((rc = resid(L.norm2, &L))) return rc;
+    } else if (L.d.ff_kind) {
       if ((rc = block_gemm(c, LGH_K_GATEUP, L.gu, LE_GEGLU, m.bxa, ldx, m.bact, L.down.kp, M))) return rc;
       if ((rc = block_gemm(c, LGH_K_DOWN, L.down, LE_F32, m.bact, L.down.kp, m.by, ldy, M))) return rc;
       if ((rc = resid(L.norm2))) return rc;
     }
     if (m.tap && m.tap_tokens == M)
-      L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(m.tap_buf + (size_t)li * M * d.width, m.bx, (size_t)M * d.width * 4, hipMemcpyDeviceToDevice, st));
+      L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(m.tap_buf + (size_t)li * M * d.width, xs, (size_t)M * d.width * 4, hipMemcpyDeviceToDevice, st));
   }
-  L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(c->hidden, m.bx + (size_t)(M - 1) * d.width, (size_t)d.width * 4, hipMemcpyDeviceToDevice, st));
+  L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(c->hidden, xs + (size_t)(M - 1) * d.width, (size_t)d.width * 4, hipMemcpyDeviceToDevice, st));
+  if (m.hist_floats() && (rc = run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
+                            return conv_store_launch(m.tails, m.hist, m.n_sub, d.conv_taps, d.width, pos0, M, st);
+                          })))
+    return rc;
   const uint32_t ldl = up(d.vocab_size, 4);
   for (uint32_t w = 0; w < n_want; w += kLogitRows) {
     const uint32_t n = std::min(kLogitRows, n_want - w);
     L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(m.brows, want + w, (size_t)n * 4, hipMemcpyHostToDevice, st));
-    if ((rc = run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] { return final_norm_rows_launch(m.bx, m.brows, n, m.final_norm, eps, d.width, m.bla, ldx, m.f32, st); })))
+    if ((rc = run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
+           return m.dyt() ? final_dyt_rows_launch(xs, m.brows, n, dyt_w(m.final_dyt), d.width, m.bla, ldx, m.f32, st)
+                          : final_norm_rows_launch(xs, m.brows, n, m.final_norm, eps, d.width, m.bla, ldx, m.f32, st);
+         })))
       return rc;
     if ((rc = block_gemm(c, LGH_K_OUTPUT, m.head, LE_F32, m.bla, ldx, m.blogits, ldl, n))) return rc;
     L_TRY(c, LGH_OPERATION_FAILED, hipMemcpy2DAsync(logits_out + (size_t)w * d.vocab_size, (size_t)d.vocab_size * 4, m.blogits, (size_t)ldl * 4,

@@ -3,6 +3,7 @@
 #pragma once
 
 #include "device_utils.h"
+#include "layered.h"
 
 namespace lgh {
 
@@ -19,6 +20,86 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
   return 0.5f * z * (1.0f + tanhf(inner));
 }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+
+// tanh: its odd series up to 1/4 (next term below 1e-7 of the value), beyond it 1 - 2 / (exp(2x) + 1); 1e-6 of the value everywhere
+__device__ __forceinline__ float tanh_series(float x) {
+  const float z = x * x;
+  float s = __builtin_fmaf(z, 62.0f / 2835.0f, -17.0f / 315.0f);
+  s = __builtin_fmaf(z, s, 2.0f / 15.0f);
+  s = __builtin_fmaf(z, s, -1.0f / 3.0f);
+  return __builtin_fmaf(x * z, s, x);
+}
+__device__ __forceinline__ float tanh_f(float x) {
+  const float e = __builtin_amdgcn_exp2f(x * 2.8853900817779268f);
+  const float far = __builtin_fmaf(-2.0f, __builtin_amdgcn_rcpf(e + 1.0f), 1.0f);
+  return fabsf(x) < 0.25f ? tanh_series(x) : far;
+}
+
+// what is not a number ranks last, so that every place is taken
+__device__ __forceinline__ float rank_key(float z) { return z == z ? z : -INFINITY; }
+
+// The `top` largest of E logits in LDS (padded with -inf to a multiple of 4), the first of equals first: expert e's place is the number of
+// experts before it.  One thread per expert; sel[place], w[place] = its score.
+__device__ __forceinline__ void rank_experts(const float* z, uint32_t E, uint32_t top, int* sel, float* w) {
+  for (uint32_t e = threadIdx.x; e < E; e += blockDim.x) {
+    const float v = z[e];
+    uint32_t place = 0;
+    for (uint32_t j = 0; j < E; j += 4) {
+      const f32x4 q = *reinterpret_cast<const f32x4*>(z + j);
+#pragma unroll
+      for (uint32_t i = 0; i < 4; i++) place += q[i] > v || (q[i] == v && j + i < e) ? 1u : 0u;
+    }
+    if (place < top) { sel[place] = (int)e; w[place] = sigmoid_f(v); }
+  }
+}
+
+// ---- residual form LGH_RESIDUAL_SANDWICH_DYT, one channel ----
+__device__ __forceinline__ float dyt_f(float v, float alpha, float w, float b) { return __builtin_fmaf(tanh_f(alpha * v), w, b); }
+
+// the convolution's taps before position p; nothing lies before position 0
+__device__ __forceinline__ float conv_past(const ConvW& cv, uint32_t width, uint32_t c, int p) {
+  float s = 0.0f;
+  for (uint32_t j0 = 1; j0 < cv.taps; j0 += 4) {
+    float w[4], h[4];
+#pragma unroll
+    for (uint32_t i = 0; i < 4; i++) {   // clamped: the loads are unconditional
+      const uint32_t j = j0 + i;
+      const bool ok = j < cv.taps && (int)j <= p;
+      const uint32_t row = ok ? (uint32_t)(p - (int)j) % (cv.taps - 1) : 0u;
+      w[i] = cv.w[(size_t)c * cv.taps + (ok ? cv.taps - 1 - j : 0u)];
+      h[i] = cv.hist[(size_t)row * width + c];
+      w[i] = ok ? w[i] : 0.0f;
+    }
+#pragma unroll
+    for (uint32_t i = 0; i < 4; i++) s = __builtin_fmaf(w[i], h[i], s);
+  }
+  return s;
+}
+// what the residual update of a channel needs besides the sublayer's output
+struct PostIn { float x, pw, pb, nw, nb, past, wl; };
+__device__ __forceinline__ PostIn post_fetch(const PostUpdate& a, uint32_t c, int p) {
+  PostIn r;
+  r.x = a.x ? a.x[c] : 0.0f;
+  r.pw = a.post.w[c]; r.pb = a.post.b[c];
+  r.nw = a.next.w[c]; r.nb = a.next.b[c];
+  const bool cv = a.conv.taps != 0;
+  r.wl = cv ? a.conv.w[(size_t)c * a.conv.taps + a.conv.taps - 1] : 0.0f;
+  r.past = cv ? conv_past(a.conv, a.width, c, p) : 0.0f;
+  return r;
+}
+// stream value v of channel c at position p -> the next sublayer's input
+__device__ __forceinline__ void post_input(const PostUpdate& a, const PostIn& r, uint32_t c, int p, float v, float nalpha) {
+  const float h = dyt_f(v, nalpha, r.nw, r.nb);
+  if (a.conv.taps > 1) a.conv.hist[(size_t)((uint32_t)p % (a.conv.taps - 1)) * a.width + c] = h;
+  a.hout[c] = h + __builtin_fmaf(r.wl, h, r.past);
+}
+__device__ __forceinline__ void post_finish(const PostUpdate& a, const PostIn& r, uint32_t c, int p, float y, float palpha, float nalpha) {
+  const float v = __builtin_fmaf(a.mult, dyt_f(y, palpha, r.pw, r.pb), r.x);
+  a.xout[c] = v;
+  post_input(a, r, c, p, v, nalpha);
+}
 
 // sum over a workgroup of up to 16 waves; every thread gets the result.  red: 16 floats of LDS, free again after the call.
 __device__ __forceinline__ float block_sum(float v, float* red) {
@@ -56,6 +137,29 @@ template <> struct Frag<float> {
 };
 
 template <class T> __device__ __forceinline__ T to_act(float v) { return (T)v; }
+
+// value fragment from a tile of keys (rows of `ld` elements, 16-byte chunks stored at chunk ^ (row & 7)); k slots (lane group g, j):
+// bf16: keys 4g + j of the tile's first 16 rows (j < 4) and of its second 16 (j >= 4); f32: keys 4g + j of rows 16 n ..; column c0 + r16.
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+template <class T>
+__device__ __forceinline__ typename Frag<T>::V tile_value_frag(const T* tile, uint32_t ld, int n, uint32_t c0, uint32_t r16, uint32_t g) {
+  if constexpr (sizeof(T) == 2) {   // lane i of a 16-lane group fetches 4 columns of key row i / 4 and receives 4 keys of column i
+    const uint32_t col = c0 + (r16 & 3) * 4, row = g * 4 + (r16 >> 2);
+    typedef __attribute__((address_space(3))) s16x4* lds_p;
+    const T* p0 = tile + row * ld + ((col >> 3) ^ (row & 7)) * 8 + (col & 7);   // row + 16 has the same low bits
+    const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)p0), b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_p)(p0 + 16 * ld));
+    return __builtin_bit_cast(bf16x8, __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7));
+  } else {
+    const uint32_t col = c0 + r16;
+    f32x4 v;
+#pragma unroll
+    for (uint32_t e = 0; e < 4; e++) {
+      const uint32_t row = n * 16 + g * 4 + e;
+      v[e] = tile[row * ld + ((col >> 2) ^ (row & 7)) * 4 + (col & 3)];
+    }
+    return v;
+  }
+}
 
 // 16 bytes per lane from global memory straight into LDS; lane l's bytes land at lds + 16 l (lds: wave-uniform)
 __device__ __forceinline__ void lds_dma16(const void* g, void* lds) {

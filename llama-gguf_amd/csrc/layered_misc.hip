@@ -1,4 +1,5 @@
-// layered_misc.hip — embedding (with the pair table), residual + layer norm, final norm of the models of layered.h.
+// layered_misc.hip — embedding (with the pair table), residual updates of both forms (layer norm; squashing norms with a short
+// convolution), final norm of the models of layered.h.
 #include "layered.h"
 #include "layered_device.h"
 
@@ -10,8 +11,9 @@ __device__ __forceinline__ uint64_t bigram_row(const EmbedArgs& a, uint32_t pos,
   return ((uint64_t)prev * a.mul_prev + (uint64_t)cur * a.mul_cur) % a.buckets;
 }
 
-// One decode token: advances the position words, notes the token in the history, writes the residual stream.  One workgroup.
-__global__ void __launch_bounds__(1024) layered_embed_kernel(const EmbedArgs a, int* state, float* __restrict__ x) {
+// One decode token: advances the position words, notes the token in the history, writes the residual stream (and, with `post`, the first
+// sublayer's input).  One workgroup.
+__global__ void __launch_bounds__(1024) layered_embed_kernel(const EmbedArgs a, int* state, float* __restrict__ x, const PostUpdate post, int with_post) {
   const int p = state[ST_NEXT];
   const uint32_t tok = (uint32_t)state[ST_TOKEN];
   const uint32_t prev = p > 0 && a.bigram ? (uint32_t)a.hist[p - 1] : 0u;
@@ -23,11 +25,23 @@ __global__ void __launch_bounds__(1024) layered_embed_kernel(const EmbedArgs a, 
   }
   const uint16_t* e = a.embed + (size_t)tok * a.width;
   const uint16_t* b = a.bigram ? a.bigram + bigram_row(a, (uint32_t)p, prev, tok) * a.width : nullptr;
-  for (uint32_t i = threadIdx.x; i < a.width; i += blockDim.x) x[i] = b ? bf_f(e[i]) + bf_f(b[i]) : bf_f(e[i]);
+  const float alpha = with_post ? *post.next.alpha : 0.0f;
+  for (uint32_t i = threadIdx.x; i < a.width; i += blockDim.x) {
+    const float v = b ? bf_f(e[i]) + bf_f(b[i]) : bf_f(e[i]);
+    x[i] = v;
+    if (with_post) {
+      PostIn r;
+      r.nw = post.next.w[i]; r.nb = post.next.b[i];
+      r.wl = post.conv.taps ? post.conv.w[(size_t)i * post.conv.taps + post.conv.taps - 1] : 0.0f;
+      r.past = post.conv.taps ? conv_past(post.conv, post.width, i, p) : 0.0f;
+      post_input(post, r, i, p, v, alpha);
+    }
+  }
 }
 
-hipError_t layered_embed_launch(const EmbedArgs& a, int* state, float* x, hipStream_t st) {
-  hipLaunchKernelGGL(layered_embed_kernel, dim3(1), dim3(1024), 0, st, a, state, x);
+hipError_t layered_embed_launch(const EmbedArgs& a, int* state, float* x, const PostUpdate* post, hipStream_t st) {
+  if (post && (post->width != a.width || !post->hout || !post->next.w || !post->next.b || !post->next.alpha)) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(layered_embed_kernel, dim3(1), dim3(1024), 0, st, a, state, x, post ? *post : PostUpdate(), post ? 1 : 0);
   return hipGetLastError();
 }
 
@@ -121,6 +135,172 @@ hipError_t final_norm_rows_launch(const float* x, const int* rows, uint32_t n_ro
                                   bool f32, hipStream_t st) {
   if (f32) hipLaunchKernelGGL(final_norm_rows_kernel<float>, dim3(n_rows), dim3(256), 0, st, x, rows, w, eps, width, (float*)xa, ldx);
   else hipLaunchKernelGGL(final_norm_rows_kernel<__bf16>, dim3(n_rows), dim3(256), 0, st, x, rows, w, eps, width, (__bf16*)xa, ldx);
+  return hipGetLastError();
+}
+
+template <class T>
+__global__ void __launch_bounds__(256) final_dyt_rows_kernel(const float* __restrict__ x, const int* __restrict__ rows, const DytW n, uint32_t width, T* __restrict__ xa,
+                                                             uint32_t ldx) {
+  const float* r = x + (size_t)rows[blockIdx.x] * width;
+  const float alpha = *n.alpha;
+  for (uint32_t i = threadIdx.x; i < width; i += 256) xa[(size_t)blockIdx.x * ldx + i] = to_act<T>(dyt_f(r[i], alpha, n.w[i], n.b[i]));
+}
+
+hipError_t final_dyt_rows_launch(const float* x, const int* rows, uint32_t n_rows, const DytW& n, uint32_t width, void* xa, uint32_t ldx, bool f32, hipStream_t st) {
+  if (f32) hipLaunchKernelGGL(final_dyt_rows_kernel<float>, dim3(n_rows), dim3(256), 0, st, x, rows, n, width, (float*)xa, ldx);
+  else hipLaunchKernelGGL(final_dyt_rows_kernel<__bf16>, dim3(n_rows), dim3(256), 0, st, x, rows, n, width, (__bf16*)xa, ldx);
+  return hipGetLastError();
+}
+
+// ------------------------------------------------------------------------------------------------
+// LGH_RESIDUAL_SANDWICH_DYT over a block.  A wave = 64 * V channels of kDytTokens tokens, walked in order; the convolution's inputs of the
+// last taps positions lie in LDS, every thread its own channels (no barriers).  The taps - 1 tokens before a wave's first are formed again
+// from the stream before the update, the ones before the block come from the history.
+// ------------------------------------------------------------------------------------------------
+constexpr int kDytTokens = 16;
+
+template <int V> struct VecF { float v[V]; };
+template <int V> __device__ __forceinline__ VecF<V> load_vec(const float* p) {
+  VecF<V> r;
+  if constexpr (V == 4) { const f32x4 q = *reinterpret_cast<const f32x4*>(p); r.v[0] = q.x; r.v[1] = q.y; r.v[2] = q.z; r.v[3] = q.w; }
+  else r.v[0] = p[0];
+  return r;
+}
+template <int V> __device__ __forceinline__ void store_vec(float* p, const VecF<V>& a) {
+  if constexpr (V == 4) { f32x4 q; q.x = a.v[0]; q.y = a.v[1]; q.z = a.v[2]; q.w = a.v[3]; *reinterpret_cast<f32x4*>(p) = q; }
+  else p[0] = a.v[0];
+}
+
+// y of one token's channels: the sublayer's output plus its experts' rows
+template <int V> __device__ __forceinline__ VecF<V> add_pairs(VecF<V> y, const float* pairs, uint32_t ldp, const int* slot, uint32_t top, uint32_t c) {
+  for (uint32_t s = 0; s < top; s++) {
+    const VecF<V> p = load_vec<V>(pairs + (size_t)slot[s] * ldp + c);
+#pragma unroll
+    for (int i = 0; i < V; i++) y.v[i] += p.v[i];
+  }
+  return y;
+}
+
+template <class T, int V>
+__global__ void __launch_bounds__(256) dyt_block_kernel(const DytBlock a) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];   // [taps][256][V] inputs, [taps][256][V] filters
+  const uint32_t tid = threadIdx.x, lane = tid & 63, c0 = (blockIdx.x * 64 + lane) * V;
+  const int t0 = (int)((blockIdx.y * 4 + (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6))) * kDytTokens);
+  if (t0 >= (int)a.M) return;
+  const int t1 = t0 + kDytTokens < (int)a.M ? t0 + kDytTokens : (int)a.M;
+  const bool live = c0 < a.width;
+  const uint32_t c = live ? c0 : 0, W = a.width;
+  const int taps = (int)a.conv.taps, back = taps ? taps - 1 : 0;
+  const bool upd = a.xout != nullptr, nxt = a.xa != nullptr;
+  float* ring = lds + tid * V;
+  float* filt = ring + (size_t)taps * 256 * V;
+  for (int j = 0; j < taps; j++)
+#pragma unroll
+    for (int i = 0; i < V; i++) filt[j * 256 * V + i] = a.conv.w[(size_t)(c + i) * taps + j];
+  VecF<V> pw, pb, nw, nb;
+  float pal = 0.0f, nal = 0.0f;
+  if (upd) { pw = load_vec<V>(a.post.w + c); pb = load_vec<V>(a.post.b + c); pal = *a.post.alpha; }
+  if (nxt) { nw = load_vec<V>(a.next.w + c); nb = load_vec<V>(a.next.b + c); nal = *a.next.alpha; }
+  auto fetch_x = [&](int t) { return load_vec<V>(a.x + (size_t)(t < 0 ? 0 : t) * W + c); };
+  auto fetch_y = [&](int t) {
+    VecF<V> y;
+#pragma unroll
+    for (int i = 0; i < V; i++) y.v[i] = 0.0f;
+    if (upd && a.y) y = load_vec<V>(a.y + (size_t)(t < 0 ? 0 : t) * a.ldy + c);
+    if (upd && a.pairs && t >= 0) y = add_pairs<V>(y, a.pairs, a.ldp, a.slot + (size_t)t * a.top, a.top, c);
+    return y;
+  };
+  const int first = nxt ? t0 - back : t0;
+  VecF<V> xn = fetch_x(first), yn = fetch_y(first);
+  int at = 0;                                       // ring row of token t
+  for (int t = first; t < t1; t++) {
+    VecF<V> v = xn, h;
+    const VecF<V> y = yn;
+    if (t + 1 < t1) { xn = fetch_x(t + 1); yn = fetch_y(t + 1); }
+    if (t < 0) {                                    // before the block
+      const int p = (int)a.pos0 + t;
+#pragma unroll
+      for (int i = 0; i < V; i++) h.v[i] = 0.0f;
+      if (p >= 0) h = load_vec<V>(a.conv.hist + (size_t)(p % back) * W + c);
+    } else {
+      if (upd) {
+#pragma unroll
+        for (int i = 0; i < V; i++) v.v[i] = __builtin_fmaf(a.mult, dyt_f(y.v[i], pal, pw.v[i], pb.v[i]), v.v[i]);
+        if (t >= t0 && live) store_vec<V>(a.xout + (size_t)t * W + c, v);
+      }
+      if (!nxt) continue;
+#pragma unroll
+      for (int i = 0; i < V; i++) h.v[i] = dyt_f(v.v[i], nal, nw.v[i], nb.v[i]);
+    }
+    if (taps) store_vec<V>(ring + at * 256 * V, h);
+    if (t >= t0) {
+      VecF<V> o = h;
+      int r = at + 1 < taps ? at + 1 : 0;           // the oldest input
+      for (int j = 0; j < taps; j++) {
+        const VecF<V> q = load_vec<V>(ring + r * 256 * V), w = load_vec<V>(filt + j * 256 * V);
+#pragma unroll
+        for (int i = 0; i < V; i++) o.v[i] = __builtin_fmaf(w.v[i], q.v[i], o.v[i]);
+        r = r + 1 < taps ? r + 1 : 0;
+      }
+      if (live) {
+        T* dst = reinterpret_cast<T*>(a.xa) + (size_t)t * a.ldx + c;
+        T q[V];
+#pragma unroll
+        for (int i = 0; i < V; i++) q[i] = to_act<T>(o.v[i]);
+        __builtin_memcpy(__builtin_assume_aligned(dst, sizeof(q)), q, sizeof(q));
+        if (t >= (int)a.M - back) store_vec<V>(a.tail + (size_t)((int)a.M - 1 - t) * W + c, h);
+      }
+    }
+    at = at + 1 < taps ? at + 1 : 0;
+  }
+}
+
+template <class T, int V>
+static hipError_t dyt_block_go(const DytBlock& a, hipStream_t st) {
+  static bool opted[64] = {};
+  const size_t lds = (size_t)a.conv.taps * 2 * 256 * V * 4;
+  if (lds > 156 * 1024) return hipErrorInvalidValue;
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&dyt_block_kernel<T, V>), 156 * 1024, opted); e != hipSuccess) return e;
+  hipLaunchKernelGGL((dyt_block_kernel<T, V>), dim3((a.width + 64 * V - 1) / (64 * V), (a.M + 4 * kDytTokens - 1) / (4 * kDytTokens)), dim3(256), lds, st, a);
+  return hipGetLastError();
+}
+
+hipError_t dyt_block_launch(const DytBlock& a, bool f32, hipStream_t st) {
+  const bool upd = a.xout != nullptr, nxt = a.xa != nullptr;
+  if (!a.x || a.M == 0 || (!upd && !nxt) || a.xout == a.x || (upd && (!(a.y || a.pairs) || !a.post.w || !a.post.b || !a.post.alpha)) ||
+      (a.pairs && !a.slot) || (nxt && (!a.next.w || !a.next.b || !a.next.alpha || a.ldx < a.width)) || (a.conv.taps && !a.conv.w) ||
+      (a.conv.taps > 1 && (!a.conv.hist || !a.tail)) || (!nxt && a.conv.taps))
+    return hipErrorInvalidValue;
+  const bool v4 = a.width % 4 == 0 && (!a.y || a.ldy % 4 == 0) && (!a.pairs || a.ldp % 4 == 0) && (!nxt || a.ldx % 4 == 0) && a.conv.taps <= 16;
+  if (v4) return f32 ? dyt_block_go<float, 4>(a, st) : dyt_block_go<__bf16, 4>(a, st);
+  return f32 ? dyt_block_go<float, 1>(a, st) : dyt_block_go<__bf16, 1>(a, st);
+}
+
+__global__ void __launch_bounds__(256) conv_store_kernel(const float* __restrict__ tails, float* __restrict__ hists, uint32_t back, uint32_t width, uint32_t last) {
+  const uint32_t c = blockIdx.x * 256 + threadIdx.x, i = blockIdx.y, k = blockIdx.z;
+  if (c < width) hists[((size_t)k * back + (last - i) % back) * width + c] = tails[((size_t)k * back + i) * width + c];
+}
+
+hipError_t conv_store_launch(const float* tails, float* hists, uint32_t n_sub, uint32_t taps, uint32_t width, uint32_t pos0, uint32_t M, hipStream_t st) {
+  if (taps < 2 || M == 0) return hipErrorInvalidValue;
+  const uint32_t back = taps - 1;
+  hipLaunchKernelGGL(conv_store_kernel, dim3((width + 255) / 256, M < back ? M : back, n_sub), dim3(256), 0, st, tails, hists, back, width, pos0 + M - 1);
+  return hipGetLastError();
+}
+
+__global__ void __launch_bounds__(256) pair_sum_kernel(float* __restrict__ y, uint32_t ldy, const float* __restrict__ pairs, uint32_t ldp, const int* __restrict__ slot,
+                                                       uint32_t top, uint32_t width, int add) {
+  const uint32_t t = blockIdx.x;
+  for (uint32_t c = threadIdx.x; c < width; c += 256) {
+    VecF<1> v;
+    v.v[0] = add ? y[(size_t)t * ldy + c] : 0.0f;
+    y[(size_t)t * ldy + c] = add_pairs<1>(v, pairs, ldp, slot + (size_t)t * top, top, c).v[0];
+  }
+}
+
+hipError_t pair_sum_launch(float* y, uint32_t ldy, const float* pairs, uint32_t ldp, const int* slot, uint32_t top, uint32_t width, uint32_t M, bool add, hipStream_t st) {
+  if (!y || !pairs || !slot || M == 0) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(pair_sum_kernel, dim3(M), dim3(256), 0, st, y, ldy, pairs, ldp, slot, top, width, add ? 1 : 0);
   return hipGetLastError();
 }
 

@@ -25,18 +25,51 @@ __device__ __forceinline__ void ln_lds(float* xs, uint32_t K, const float* w, fl
 }
 
 // row r of group g: 4 consecutive rows, or 2 pairs (a gate row and the up row 16 below it)
+__device__ __forceinline__ uint32_t mv_row_of(uint32_t paired, uint32_t g, int r) {
+  if (paired) { const uint32_t p = g * 2 + (r & 1); return (p >> 4) * 32 + (p & 15) + (r >> 1) * 16; }
+  return g * kMvR + r;
+}
 __device__ __forceinline__ const uint16_t* mv_row(const LinMv& a, uint32_t g, int r) {
-  uint32_t row;
-  if (a.paired) { const uint32_t p = g * 2 + (r & 1); row = (p >> 4) * 32 + (p & 15) + (r >> 1) * 16; }
-  else row = g * kMvR + r;
+  const uint32_t row = mv_row_of(a.paired, g, r);
   return a.w + (size_t)(row < a.n ? row : a.n - 1) * a.kp;
 }
 struct MvW { u32x4 w[kMvR]; };
-// lanes past the row's end re-read its first bytes (unconditional loads) and add nothing
-__device__ __forceinline__ void mv_fetch(const LinMv& a, uint32_t g, uint32_t kb, MvW& o) {
+// lanes past the row's end re-read its first bytes (unconditional loads) and add nothing.  g1: groups of the first matrix (LS_TWO) or of
+// one expert (LS_EXPERTS); sel: the chosen experts, in LDS
+template <int SRC>
+__device__ __forceinline__ void mv_fetch(const LinMv& a, uint32_t g, uint32_t kb, uint32_t g1, const int* sel, MvW& o) {
   const uint32_t kc = kb < a.kp ? kb : 0;
+  if (SRC == LS_TWO && g >= g1) {
 #pragma unroll
-  for (int r = 0; r < kMvR; r++) o.w[r] = ldg_nt128(mv_row(a, g, r) + kc);
+    for (int r = 0; r < kMvR; r++) {
+      const uint32_t row = (g - g1) * kMvR + r;
+      o.w[r] = ldg_nt128(a.w2 + (size_t)(row < a.n2 ? row : a.n2 - 1) * a.kp + kc);
+    }
+  } else if (SRC == LS_EXPERTS) {
+    const uint32_t slot = g / g1, gl = g - slot * g1;
+    const uint16_t* w = a.w2 + (size_t)__builtin_amdgcn_readfirstlane(sel[slot]) * a.stride + kc;
+#pragma unroll
+    for (int r = 0; r < kMvR; r++) {
+      const uint32_t row = mv_row_of(1, gl, r);
+      o.w[r] = ldg_nt128(w + (size_t)(row < a.n ? row : a.n - 1) * a.kp);
+    }
+  } else if (SRC == LS_MOE_DOWN) {
+    const uint16_t* w = a.w + kc;
+    uint32_t ld = a.kps;
+    if (kc >= a.kps) {
+      const uint32_t q = kc - a.kps, s = q / a.kpe;
+      w = a.w2 + (size_t)sel[s] * a.stride + (q - s * a.kpe);
+      ld = a.kpe;
+    }
+#pragma unroll
+    for (int r = 0; r < kMvR; r++) {
+      const uint32_t row = g * kMvR + r;
+      o.w[r] = ldg_nt128(w + (size_t)(row < a.n ? row : a.n - 1) * ld);
+    }
+  } else {
+#pragma unroll
+    for (int r = 0; r < kMvR; r++) o.w[r] = ldg_nt128(mv_row(a, g, r) + kc);
+  }
 }
 __device__ __forceinline__ void mv_acc(const MvW& o, f32x4 x0, f32x4 x1, float* acc) {
 #pragma unroll
@@ -50,11 +83,17 @@ __device__ __forceinline__ void mv_acc(const MvW& o, f32x4 x0, f32x4 x1, float* 
     acc[r] = s;
   }
 }
-template <int PRO>
-__global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint32_t n_groups, uint32_t ks) {
+__device__ __forceinline__ float mv_act(uint32_t act, float z) { return act == LA_SILU ? silu_f(z) : gelu_tanh_f(z); }
+
+template <int PRO, int SRC, bool POST>
+__global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint32_t n_groups, uint32_t ks, uint32_t g1) {
+  constexpr bool MOE = SRC == LS_EXPERTS || SRC == LS_MOE_DOWN;
   extern __shared__ __attribute__((aligned(16))) float xs[];   // [kp]
   __shared__ float red[2][16][kMvR];
   __shared__ float bred[16];
+  __shared__ __attribute__((aligned(16))) float zs[SRC == LS_EXPERTS ? kMaxExperts : 4];
+  __shared__ int sel[MOE ? kMaxTop : 1];
+  __shared__ float selw[SRC == LS_EXPERTS ? kMaxTop : 1];
   const uint32_t tid = threadIdx.x, lane = tid & 63, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
   const uint32_t team = wave / ks, sub = wave % ks, teams = 16 / ks;
   const uint32_t kb0 = (sub * 64 + lane) * 8, kstep = ks * 512, passes = (a.kp + kstep - 1) / kstep;
@@ -63,11 +102,19 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
   uint32_t gf = g, pf = 0;   // the next pass to request
   MvW n0, n1;
   auto request = [&](MvW& o) {
-    if (gf < n_groups) mv_fetch(a, gf, kb0 + pf * kstep, o);
+    if (gf < n_groups) mv_fetch<SRC>(a, gf, kb0 + pf * kstep, g1, sel, o);
     if (++pf == passes) { pf = 0; gf += gstep; }
   };
-  request(n0);
-  request(n1);
+  if (!MOE) { request(n0); request(n1); }
+  int pos = 0;
+  float palpha = 0.0f, nalpha = 0.0f;
+  if (POST) { pos = *a.post.pos; palpha = *a.post.post.alpha; nalpha = *a.post.next.alpha; }
+  if (SRC == LS_EXPERTS) {
+    const uint32_t ep = (a.experts + 3) & ~3u;
+    for (uint32_t e = tid; e < ep; e += kMvThreads) zs[e] = e < a.experts ? rank_key(a.logits[e]) : -INFINITY;
+  }
+  if (SRC == LS_MOE_DOWN)
+    for (uint32_t e = tid; e < a.top; e += kMvThreads) sel[e] = a.sel[e];
   if (PRO == LP_COPY) {
     for (uint32_t i = tid; i < a.k; i += kMvThreads) xs[i] = a.x[i];
   } else if (PRO == LP_RESID || PRO == LP_HEAD) {
@@ -114,9 +161,18 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
   }
   for (uint32_t i = a.k + tid; i < a.kp; i += kMvThreads) xs[i] = 0.0f;
   __syncthreads();
+  if (SRC == LS_EXPERTS) {
+    rank_experts(zs, a.experts, a.top, sel, selw);
+    __syncthreads();
+    if (blockIdx.x == 0 && tid < a.top) a.sel[tid] = sel[tid];
+  }
+  if (MOE) { request(n0); request(n1); }
   const uint32_t rounds = (n_groups + gstep - 1) / gstep;   // the same for every wave: the teams meet at a barrier when ks > 1
   for (uint32_t rd = 0; rd < rounds; rd++, g += gstep) {
     float acc[kMvR] = {0.0f, 0.0f, 0.0f, 0.0f};
+    const uint32_t ch = g * kMvR + (lane & 3);   // POST: the channel this lane finishes
+    PostIn pi;
+    if (POST && sub == 0) pi = post_fetch(a.post, ch < a.n ? ch : a.n - 1, pos);
     if (g < n_groups) {
       for (uint32_t p = 0; p < passes; p++) {
         const MvW cur = n0;
@@ -140,7 +196,29 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
           for (uint32_t k = 1; k < ks; k++) acc[r] += red[rd & 1][wave + k][r];
       }
     }
-    if (sub == 0 && lane == 63 && g < n_groups) {
+    if constexpr (POST) {
+      if (sub == 0 && g < n_groups) {
+        float y[kMvR];
+#pragma unroll
+        for (int r = 0; r < kMvR; r++) y[r] = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, acc[r]), 63));
+        const float v = (lane & 2) ? ((lane & 1) ? y[3] : y[2]) : ((lane & 1) ? y[1] : y[0]);
+        if (lane < kMvR && ch < a.n) post_finish(a.post, pi, ch, pos, v, palpha, nalpha);
+      }
+    } else if (SRC == LS_EXPERTS) {
+      if (sub == 0 && lane == 63 && g < n_groups) {
+        const uint32_t slot = g / g1, gl = g - slot * g1;
+        const float w = selw[slot];
+#pragma unroll
+        for (int r = 0; r < 2; r++)
+          if (gl * 2 + r < a.n / 2) a.out[(size_t)slot * a.kpe + gl * 2 + r] = mv_act(a.act, w * acc[r]) * (w * acc[r + 2]);
+      }
+    } else if (SRC == LS_TWO && g >= g1) {
+      if (sub == 0 && lane == 63 && g < n_groups) {
+#pragma unroll
+        for (int r = 0; r < kMvR; r++)
+          if ((g - g1) * kMvR + r < a.n2) a.out2[(g - g1) * kMvR + r] = acc[r];
+      }
+    } else if (sub == 0 && lane == 63 && g < n_groups) {
       if (!a.paired) {
 #pragma unroll
         for (int r = 0; r < kMvR; r++)
@@ -148,31 +226,60 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
       } else {
 #pragma unroll
         for (int r = 0; r < 2; r++)
-          if (g * 2 + r < a.n / 2) a.out[g * 2 + r] = gelu_tanh_f(acc[r]) * acc[r + 2];
+          if (g * 2 + r < a.n / 2) a.out[g * 2 + r] = mv_act(a.act, acc[r]) * acc[r + 2];
       }
     }
   }
 }
 
-template <int PRO>
-static hipError_t lin_mv_go(const LinMv& a, hipStream_t st) {
+template <int PRO, int SRC, bool POST>
+static hipError_t lin_mv_run(const LinMv& a, hipStream_t st) {
   static bool opted[64] = {};
-  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_mv_kernel<PRO>), 152 * 1024, opted); e != hipSuccess) return e;
-  const uint32_t groups = (a.n + kMvR - 1) / kMvR;
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_mv_kernel<PRO, SRC, POST>), 152 * 1024, opted); e != hipSuccess) return e;
+  const uint32_t g1 = (a.n + kMvR - 1) / kMvR;
+  const uint32_t groups = SRC == LS_TWO ? g1 + (a.n2 + kMvR - 1) / kMvR : SRC == LS_EXPERTS ? g1 * a.top : g1;
   uint32_t ks = 1;   // waves per team: enough teams for the groups of a CU, and at least a full pass of columns per wave
   while (ks < 8 && (uint64_t)groups * ks * 2 <= kNumCU * 16 && a.kp >= 1024 * ks) ks *= 2;
   const uint32_t teams = 16 / ks, want = (groups + teams - 1) / teams;
-  hipLaunchKernelGGL(lin_mv_kernel<PRO>, dim3(want < kNumCU ? want : kNumCU), dim3(kMvThreads), (size_t)a.kp * 4, st, a, groups, ks);
+  hipLaunchKernelGGL((lin_mv_kernel<PRO, SRC, POST>), dim3(want < kNumCU ? want : kNumCU), dim3(kMvThreads), (size_t)a.kp * 4, st, a, groups, ks, g1);
   return hipGetLastError();
 }
+template <int PRO, int SRC>
+static hipError_t lin_mv_post(const LinMv& a, hipStream_t st) {
+  if (!a.post.xout) return lin_mv_run<PRO, SRC, false>(a, st);
+  const PostUpdate& p = a.post;
+  if (a.paired || p.width != a.n || !p.x || !p.hout || !p.pos || !p.post.w || !p.post.b || !p.post.alpha || !p.next.w || !p.next.b || !p.next.alpha ||
+      (p.conv.taps && !p.conv.w) || (p.conv.taps > 1 && !p.conv.hist))
+    return hipErrorInvalidValue;
+  return lin_mv_run<PRO, SRC, true>(a, st);
+}
+template <int PRO>
+static hipError_t lin_mv_go(const LinMv& a, int src, hipStream_t st) {
+  if (src == LS_TWO) return a.post.xout || !a.w2 || !a.out2 || a.n2 == 0 ? hipErrorInvalidValue : lin_mv_run<PRO, LS_TWO, false>(a, st);
+  return src != LS_PLAIN || a.post.xout ? hipErrorInvalidValue : lin_mv_run<PRO, LS_PLAIN, false>(a, st);
+}
 
-hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st) {
-  if (!a.w || !a.out || a.n == 0 || a.kp % 64 || a.kp > kLinMvMaxK || a.k > a.kp || (a.paired && a.n % 32)) return hipErrorInvalidValue;
+hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st, int src) {
+  if ((a.n && src != LS_EXPERTS && !a.w && !(src == LS_MOE_DOWN && a.kps == 0)) || (a.n && !a.out && !a.post.xout) || (a.n == 0 && src != LS_TWO) || a.kp % 64 ||
+      a.kp > kLinMvMaxK || a.k > a.kp || (a.paired && a.n % 32))
+    return hipErrorInvalidValue;
+  if (src == LS_EXPERTS || src == LS_MOE_DOWN) {
+    if (pro != LP_COPY || !a.x || !a.w2 || !a.sel || a.top == 0 || a.top > kMaxTop || a.kpe % 64) return hipErrorInvalidValue;
+    if (src == LS_EXPERTS) {
+      if (!a.paired || !a.logits || !a.out || a.experts > kMaxExperts || a.top > a.experts || a.kpe < a.n / 2) return hipErrorInvalidValue;
+      return lin_mv_run<LP_COPY, LS_EXPERTS, false>(a, st);
+    }
+    if (a.paired || a.kps % 64 || a.kpe == 0 || a.kp != a.kps + a.top * a.kpe) return hipErrorInvalidValue;
+    return lin_mv_post<LP_COPY, LS_MOE_DOWN>(a, st);
+  }
   switch (pro) {
-    case LP_COPY: return a.x ? lin_mv_go<LP_COPY>(a, st) : hipErrorInvalidValue;
-    case LP_RESID: return a.x && a.y && a.nw && a.xout ? lin_mv_go<LP_RESID>(a, st) : hipErrorInvalidValue;
-    case LP_HEAD: return a.x && a.y && a.nw && a.nw2 && a.xout ? lin_mv_go<LP_HEAD>(a, st) : hipErrorInvalidValue;
-    case LP_MLSTM: return a.num && a.nw && a.gate && a.heads * a.vdim == a.k ? lin_mv_go<LP_MLSTM>(a, st) : hipErrorInvalidValue;
+    case LP_COPY:
+      if (!a.x) return hipErrorInvalidValue;
+      return src == LS_PLAIN ? lin_mv_post<LP_COPY, LS_PLAIN>(a, st) : lin_mv_go<LP_COPY>(a, src, st);
+    case LP_RESID: return a.x && a.y && a.nw && a.xout ? lin_mv_go<LP_RESID>(a, src, st) : hipErrorInvalidValue;
+    case LP_HEAD: return a.x && a.y && a.nw && a.nw2 && a.xout && src == LS_PLAIN && !a.post.xout ? lin_mv_run<LP_HEAD, LS_PLAIN, false>(a, st) : hipErrorInvalidValue;
+    case LP_MLSTM:
+      return a.num && a.nw && a.gate && a.heads * a.vdim == a.k && src == LS_PLAIN ? lin_mv_post<LP_MLSTM, LS_PLAIN>(a, st) : hipErrorInvalidValue;
   }
   return hipErrorInvalidValue;
 }
@@ -184,7 +291,7 @@ hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st) {
 // ------------------------------------------------------------------------------------------------
 template <class T> constexpr uint32_t act_chunks() { return 64 * sizeof(T) / 16; }   // 16-byte chunks of a row's 64 columns
 
-template <class T, int BM, int BN, int WN, int EPI>
+template <class T, int BM, int BN, int WN, int EPI, bool GRP>
 __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t tiles_n, uint32_t tiles_m) {
   constexpr int WM = 4 / WN, NT = BN / WN / 16, MT = BM / WM / 16;
   constexpr uint32_t XC = act_chunks<T>();
@@ -199,26 +306,44 @@ __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t
     t = xcd * q + (xcd < r ? xcd : r) + i;
   }
   const uint32_t tn = t / tiles_m, tm = t % tiles_m;
-  const uint32_t n0 = tn * BN, m0 = tm * BM;
+  const uint32_t n0 = tn * BN;
+  uint32_t m0 = tm * BM, m_end = a.M;   // rows of this tile
+  const uint16_t* W = a.w;
+  if constexpr (GRP) {
+    const int e = a.grp.tile_e[tm];
+    if (e < 0) return;
+    m0 = (uint32_t)a.grp.tile_row[tm];
+    m_end = (uint32_t)a.grp.seg[e + 1];
+    W += (size_t)e * a.grp.stride;
+  }
   const uint32_t wn = wave % WN, wm = wave / WN;
   const uint32_t r16 = lane & 15, g = lane >> 4;
   const T* X = reinterpret_cast<const T*>(a.x);
 
+  constexpr uint32_t RPI = 64 / XC;                          // rows of x per wave instruction
+  constexpr int NX = (int)((kXBytes / 1024 + 3) / 4);
+  uint32_t xrow[GRP ? NX : 1];                               // grouped: where this lane's rows lie
+  if constexpr (GRP) {
+#pragma unroll
+    for (int i = 0; i < NX; i++) {
+      const uint32_t r = m0 + (i * 4 + wave) * RPI + lane / XC, m = r < m_end ? r : m_end - 1;
+      xrow[i] = a.grp.src ? (uint32_t)a.grp.src[m] : m;
+    }
+  }
   auto stage = [&](uint32_t k0, uint32_t buf) {
     uint8_t* base = smem + buf * kBuf;
 #pragma unroll
     for (int i = 0; i < (int)(kWBytes / 4096); i++) {       // weights: 8 chunks a row, a wave instruction covers 8 rows
       const uint32_t row = (i * 4 + wave) * 8 + (lane >> 3), ch = (lane & 7) ^ (row & 7);
       const uint32_t n = n0 + row < a.np ? n0 + row : a.np - 1;
-      lds_dma16(a.w + (size_t)n * a.kp + k0 + ch * 8, base + (i * 4 + wave) * 1024);
+      lds_dma16(W + (size_t)n * a.kp + k0 + ch * 8, base + (i * 4 + wave) * 1024);
     }
-    constexpr uint32_t RPI = 64 / XC;                        // rows per wave instruction
 #pragma unroll
-    for (int i = 0; i < (int)((kXBytes / 1024 + 3) / 4); i++) {
+    for (int i = 0; i < NX; i++) {
       const uint32_t blk = i * 4 + wave;
       if (kXBytes / 1024 % 4 == 0 || blk < kXBytes / 1024) {
         const uint32_t row = blk * RPI + lane / XC, ch = (lane % XC) ^ (row & (XC - 1));
-        const uint32_t m = m0 + row < a.M ? m0 + row : a.M - 1;
+        const uint32_t m = GRP ? xrow[GRP ? i : 0] : m0 + row < a.M ? m0 + row : a.M - 1;
         lds_dma16(X + (size_t)m * a.ldx + k0 + ch * (16 / sizeof(T)), base + kWBytes + blk * 1024);
       }
     }
@@ -272,15 +397,19 @@ __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t
 #pragma unroll
   for (int j = 0; j < MT; j++) {
     const uint32_t m = m0 + (wm * MT + j) * 16 + r16;
-    if (m >= a.M) continue;
-    if constexpr (EPI == LE_GEGLU) {
+    if (m >= m_end) continue;
+    if constexpr (EPI == LE_GEGLU || EPI == LE_SWIGLU) {
+      const float in = GRP ? a.grp.scale[m] : 1.0f;            // factor of the row's input
 #pragma unroll
       for (int i = 0; i < NT; i += 2) {
         const uint32_t nb = n0 + (wn * NT + i) * 16;           // gate rows; the up rows follow
         if (nb >= a.n) continue;
         T* o = reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + nb / 2 + g * 4;
 #pragma unroll
-        for (int e = 0; e < 4; e++) o[e] = to_act<T>(gelu_tanh_f(acc[i][j][e]) * acc[i + 1][j][e]);
+        for (int e = 0; e < 4; e++) {
+          const float gt = GRP ? in * acc[i][j][e] : acc[i][j][e], u = GRP ? in * acc[i + 1][j][e] : acc[i + 1][j][e];
+          o[e] = to_act<T>((EPI == LE_SWIGLU ? silu_f(gt) : gelu_tanh_f(gt)) * u);
+        }
       }
     } else {
 #pragma unroll
@@ -318,13 +447,13 @@ __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t
   }
 }
 
-template <class T, int BM, int BN, int WN, int EPI>
+template <class T, int BM, int BN, int WN, int EPI, bool GRP = false>
 static hipError_t lin_gemm_go(const LinGemm& a, hipStream_t st) {
   static bool opted[64] = {};
   constexpr size_t lds = 2 * (BN * 128 + (size_t)BM * act_chunks<T>() * 16);
-  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_gemm_kernel<T, BM, BN, WN, EPI>), (int)lds, opted); e != hipSuccess) return e;
-  const uint32_t tn = (a.n + BN - 1) / BN, tm = (a.M + BM - 1) / BM;
-  hipLaunchKernelGGL((lin_gemm_kernel<T, BM, BN, WN, EPI>), dim3(tn * tm), dim3(256), lds, st, a, tn, tm);
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_gemm_kernel<T, BM, BN, WN, EPI, GRP>), (int)lds, opted); e != hipSuccess) return e;
+  const uint32_t tn = (a.n + BN - 1) / BN, tm = GRP ? a.grp.tiles : (a.M + BM - 1) / BM;
+  hipLaunchKernelGGL((lin_gemm_kernel<T, BM, BN, WN, EPI, GRP>), dim3(tn * tm), dim3(256), lds, st, a, tn, tm);
   return hipGetLastError();
 }
 
@@ -337,10 +466,31 @@ static hipError_t lin_gemm_pick(const LinGemm& a, hipStream_t st) {
   return lin_gemm_go<T, 16, 128, 4, EPI>(a, st);
 }
 
+uint32_t lin_group_rows(uint32_t rows, uint32_t groups) {
+  const uint32_t avg = rows / groups;
+  return avg > 96 ? 128 : avg > 40 ? 64 : avg > 16 ? 32 : 16;
+}
+template <class T, int EPI>
+static hipError_t lin_gemm_group(const LinGemm& a, hipStream_t st) {
+  switch (a.grp.bm) {
+    case 128: return lin_gemm_go<T, 128, 128, 2, EPI, true>(a, st);
+    case 64: return lin_gemm_go<T, 64, 128, 4, EPI, true>(a, st);
+    case 32: return lin_gemm_go<T, 32, 128, 4, EPI, true>(a, st);
+    case 16: return lin_gemm_go<T, 16, 128, 4, EPI, true>(a, st);
+  }
+  return hipErrorInvalidValue;
+}
+
 hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st) {
   const uint32_t el = f32 ? 4 : 2;
   if (!a.w || !a.x || !a.out || a.n == 0 || a.M == 0 || a.kp % 64 || a.ldx < a.kp || (a.ldx * el) % 16 || a.np % 16 || a.n > a.np) return hipErrorInvalidValue;
-  if (epi == LE_GEGLU && a.n % 32) return hipErrorInvalidValue;
+  if ((epi == LE_GEGLU || epi == LE_SWIGLU) && a.n % 32) return hipErrorInvalidValue;
+  if (a.grp.tiles) {
+    if (!a.grp.seg || !a.grp.tile_e || !a.grp.tile_row || (epi == LE_SWIGLU && !a.grp.scale)) return hipErrorInvalidValue;
+    if (epi == LE_SWIGLU) return f32 ? lin_gemm_group<float, LE_SWIGLU>(a, st) : lin_gemm_group<__bf16, LE_SWIGLU>(a, st);
+    if (epi == LE_F32) return f32 ? lin_gemm_group<float, LE_F32>(a, st) : lin_gemm_group<__bf16, LE_F32>(a, st);
+    return hipErrorInvalidValue;
+  }
   if ((epi == LE_HEADS || epi == LE_HEADS_T) && !a.hd) return hipErrorInvalidValue;
 #define LGH_GEMM_CASE(E) \
   case E: return f32 ? lin_gemm_pick<float, E>(a, st) : lin_gemm_pick<__bf16, E>(a, st);
@@ -350,6 +500,7 @@ hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st) 
     LGH_GEMM_CASE(LE_GEGLU)
     LGH_GEMM_CASE(LE_HEADS)
     LGH_GEMM_CASE(LE_HEADS_T)
+    LGH_GEMM_CASE(LE_SWIGLU)
   }
 #undef LGH_GEMM_CASE
   return hipErrorInvalidValue;

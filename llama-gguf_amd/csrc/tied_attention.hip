@@ -1,0 +1,593 @@
+// tied_attention.hip — grouped softmax attention whose values are its keys (layered.h): the value of a position is its key as projected,
+// the key is that row divided by the root mean square of ALL the position's key heads, times a norm weight.  So a position is cached once,
+// unnormed, beside one factor (kinv); the norm weights of queries and keys, the head's temperature and the scale go into the query.
+//
+//   score(i, j) = cap * tanh(q_i . k_j * kinv_j / cap) - 2^(-8 (h + 1) / heads) * (i - j),   j <= i and (i - j < window or j < keep)
+//
+// and the softmax's denominator has one more term, exp(sink_h).  Scores, softmax and sums are in 32-bit, in units of log2.
+//
+//   decode and short portions: a workgroup = one key head x one share of the visible keys; a lane holds 16 bytes of a few keys' rows in
+//     registers, for the score and for the weighted sum; only visible keys are touched (kept ones and the window, counted through).
+//   prompt portions: causal flash attention in the transposed form of the latent kernel, the key tile serving as the value tile.
+#include <algorithm>
+
+#include "layered.h"
+#include "layered_device.h"
+
+namespace lgh {
+
+constexpr float kTiedNeg = -1e30f, kTiedLog2e = 1.4426950408889634f;
+
+// cap * tanh(x / cap) in units of log2 (cap 0: x)
+struct CapF {
+  float cap, inv, lim, out;   // 1 / cap, a quarter of cap, cap * log2(e)
+  __device__ __forceinline__ explicit CapF(float c) : cap(c), inv(c > 0.0f ? 1.0f / c : 0.0f), lim(c > 0.0f ? 0.25f * c : INFINITY), out(c > 0.0f ? c * kTiedLog2e : kTiedLog2e) {}
+  __device__ __forceinline__ float small(float x) const { return cap > 0.0f ? tanh_series(x * inv) * out : x * kTiedLog2e; }   // |x| < lim
+  __device__ __forceinline__ float any(float x) const { return cap > 0.0f ? tanh_f(x * inv) * out : x * kTiedLog2e; }
+};
+__device__ __forceinline__ float tied_slope(uint32_t h, uint32_t heads) {   // in units of log2
+  return exp2f(-8.0f * (float)(h + 1) / (float)heads) * kTiedLog2e;
+}
+
+// the keys position i sees, counted through: v < nk are the kept ones, the others lie from lo on
+struct TiedSeen { uint32_t lo, nk, total; };
+__device__ __host__ __forceinline__ TiedSeen tied_seen(const TiedShape& s, uint32_t i) {
+  TiedSeen r;
+  r.lo = i + 1 > s.window ? i + 1 - s.window : 0;
+  r.nk = s.keep < r.lo ? s.keep : r.lo;
+  r.total = r.nk + i + 1 - r.lo;
+  return r;
+}
+
+// lanes that share a key row in the decode kernel
+__host__ __device__ constexpr uint32_t tied_lanes(uint32_t dp, uint32_t el) {
+  return dp * el <= 128 ? 8 : dp * el <= 256 ? 16 : dp * el <= 512 ? 32 : 64;
+}
+constexpr uint32_t kTiedBatch = 4;   // key rows a lane has in flight
+__host__ __device__ constexpr uint32_t tied_round(uint32_t lanes) { return 4 * kTiedBatch * (64 / lanes); }   // keys of a workgroup per round
+
+// sum over `N` neighbouring lanes, every one of them gets it
+template <uint32_t N> __device__ __forceinline__ float lanes_sum(float v) {
+  v += dpp_f<0xB1>(v); v += dpp_f<0x4E>(v); v += dpp_f<0x141>(v);
+  if constexpr (N >= 16) v += dpp_f<0x140>(v);
+  if constexpr (N >= 32) v += __shfl_xor(v, 16, 64);
+  if constexpr (N >= 64) v += __shfl_xor(v, 32, 64);
+  return v;
+}
+
+template <class T, int PER> __device__ __forceinline__ void unpack_row(const u32x4& w, float* f) {
+  if constexpr (sizeof(T) == 2) {
+    f[0] = bf_lo(w.x); f[1] = bf_hi(w.x); f[2] = bf_lo(w.y); f[3] = bf_hi(w.y);
+    f[4] = bf_lo(w.z); f[5] = bf_hi(w.z); f[6] = bf_lo(w.w); f[7] = bf_hi(w.w);
+  } else {
+    f[0] = __uint_as_float(w.x); f[1] = __uint_as_float(w.y); f[2] = __uint_as_float(w.z); f[3] = __uint_as_float(w.w);
+  }
+}
+
+// grid (splits, kv heads * chunks of HQ query heads, tokens)
+template <class T, uint32_t LPK, int HQ, bool OWN>
+__global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const TiedBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits) {
+  constexpr int PER = 16 / sizeof(T), NB = kTiedBatch;
+  constexpr uint32_t GPW = 64 / LPK, HALF = GPW > 1 ? 32 : 64;      // key groups of a wave; lanes left after folding its halves
+  __shared__ float red[16];
+  __shared__ float ml[2][4 * GPW][HQ];
+  extern __shared__ __attribute__((aligned(16))) float accs[];      // [4 waves][HQ][HALF][PER]
+  const uint32_t tid = threadIdx.x, lane = tid & 63, w = tid >> 6, grp = lane / LPK, sub = lane % LPK;
+  const uint32_t gq = s.heads / s.kv_heads, chunks = (gq + HQ - 1) / HQ, g = blockIdx.y / chunks, h0 = g * gq + (blockIdx.y % chunks) * HQ;
+  const uint32_t hn = (g + 1) * gq - h0 < (uint32_t)HQ ? (g + 1) * gq - h0 : (uint32_t)HQ, z = blockIdx.z, sp = blockIdx.x;
+  const uint32_t pos = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + z;
+  const TiedSeen seen = tied_seen(s, pos);
+  constexpr uint32_t KR = tied_round(LPK);
+  const uint32_t rounds = (seen.total + KR - 1) / KR, per = (rounds + n_splits - 1) / n_splits;
+  const uint32_t rb = sp * per, re = rb + per < rounds ? rb + per : rounds;
+  if (rb >= re) return;                                             // (the merge skips the same splits)
+  const float* cat = b.cat + (size_t)z * s.ldcat;
+  T* cache = reinterpret_cast<T*>(b.cache) + (size_t)g * s.rows * s.dp;
+  const uint32_t d0 = sub * PER, dc = d0 < s.dp ? d0 : 0;
+  u32x4 kraw[NB];
+  float kin[NB];
+  uint32_t kp[NB];
+  auto fetch = [&](uint32_t r) {
+#pragma unroll
+    for (int i = 0; i < NB; i++) {
+      const uint32_t v = (r * 4 + w) * (NB * GPW) + i * GPW + grp, vc = v < seen.total ? v : seen.total - 1;
+      const uint32_t p = vc < seen.nk ? vc : seen.lo + vc - seen.nk;
+      kp[i] = v < seen.total ? p : 0xFFFFFFFFu;
+      kraw[i] = *reinterpret_cast<const u32x4*>(cache + (size_t)p * s.dp + dc);
+      kin[i] = b.kinv[p];
+    }
+  };
+  fetch(rb);
+  // this token's norms; its key row where this workgroup has it
+  const bool owner = OWN && re == rounds;
+  float sq = 0.0f, sk = 0.0f;
+  for (uint32_t i = tid; i < s.heads * s.dim; i += 256) { const float v = cat[s.off_q + i]; sq = __builtin_fmaf(v, v, sq); }
+  if (owner)
+    for (uint32_t i = tid; i < s.kv_heads * s.dim; i += 256) { const float v = cat[s.off_k + i]; sk = __builtin_fmaf(v, v, sk); }
+  float q[HQ][PER], own[PER], own_inv = 0.0f, slope[HQ];
+#pragma unroll
+  for (int h = 0; h < HQ; h++) {
+    const uint32_t hh = h0 + ((uint32_t)h < hn ? h : 0);
+    const float f = s.scale * b.temp[hh];
+    slope[h] = tied_slope(hh, s.heads);
+#pragma unroll
+    for (int e = 0; e < PER; e++) {
+      const uint32_t d = d0 + e, dd = d < s.dim ? d : 0;
+      const float v = cat[s.off_q + hh * s.dim + dd] * b.qn[hh * s.dim + dd] * (b.kn[g * s.dim + dd] * f);
+      q[h][e] = d < s.dim ? v : 0.0f;
+    }
+  }
+  if (owner) {
+#pragma unroll
+    for (int e = 0; e < PER; e++) {
+      const uint32_t d = d0 + e;
+      own[e] = (float)to_act<T>(d < s.dim ? cat[s.off_k + g * s.dim + d] : 0.0f);
+    }
+  }
+  const float qinv = 1.0f / __builtin_sqrtf(block_sum(sq, red) / (float)(s.heads * s.dim) + s.eps);
+  if (owner) {
+    own_inv = 1.0f / __builtin_sqrtf(block_sum(sk, red) / (float)(s.kv_heads * s.dim) + s.eps);
+    if (blockIdx.y % chunks == 0 && tid < LPK && d0 < s.dp) {       // the cache row
+      T row[PER];
+#pragma unroll
+      for (int e = 0; e < PER; e++) row[e] = to_act<T>(own[e]);
+      __builtin_memcpy(__builtin_assume_aligned(cache + (size_t)pos * s.dp + d0, 16), row, 16);
+      if (blockIdx.y == 0 && tid == 0) b.kinv[pos] = own_inv;
+    }
+  }
+#pragma unroll
+  for (int h = 0; h < HQ; h++)
+#pragma unroll
+    for (int e = 0; e < PER; e++) q[h][e] *= qinv;
+  const CapF cap(s.cap);
+  float m[HQ], l[HQ], o[HQ][PER];
+#pragma unroll
+  for (int h = 0; h < HQ; h++) {
+    m[h] = kTiedNeg; l[h] = 0.0f;
+#pragma unroll
+    for (int e = 0; e < PER; e++) o[h][e] = 0.0f;
+  }
+  for (uint32_t r = rb; r < re; r++) {
+    u32x4 cur[NB];
+    float ci[NB], sc[NB][HQ];
+    uint32_t cp[NB];
+#pragma unroll
+    for (int i = 0; i < NB; i++) { cur[i] = kraw[i]; ci[i] = kin[i]; cp[i] = kp[i]; }
+    if (r + 1 < re) fetch(r + 1);
+    auto row_of = [&](int i, float* kf) {
+      unpack_row<T, PER>(cur[i], kf);
+      if (OWN && owner && cp[i] == pos) {
+#pragma unroll
+        for (int e = 0; e < PER; e++) kf[e] = own[e];
+      }
+    };
+#pragma unroll
+    for (int i = 0; i < NB; i++) {
+      float kf[PER];
+      row_of(i, kf);
+      const float inv = OWN && owner && cp[i] == pos ? own_inv : ci[i];
+      const bool ok = cp[i] != 0xFFFFFFFFu;
+      const float dist = (float)(pos - (ok ? cp[i] : pos));
+#pragma unroll
+      for (int h = 0; h < HQ; h++) {
+        float t = 0.0f;
+#pragma unroll
+        for (int e = 0; e < PER; e++) t = __builtin_fmaf(q[h][e], kf[e], t);
+        t = cap.any(lanes_sum<LPK>(t) * inv);
+        sc[i][h] = ok ? __builtin_fmaf(-slope[h], dist, t) : kTiedNeg;
+      }
+    }
+#pragma unroll
+    for (int h = 0; h < HQ; h++) {
+      float m1 = m[h];
+#pragma unroll
+      for (int i = 0; i < NB; i++) m1 = fmaxf(m1, sc[i][h]);
+      const float a = __builtin_amdgcn_exp2f(m[h] - m1);
+      l[h] *= a;
+#pragma unroll
+      for (int e = 0; e < PER; e++) o[h][e] *= a;
+      m[h] = m1;
+#pragma unroll
+      for (int i = 0; i < NB; i++) {
+        const float p = cp[i] != 0xFFFFFFFFu ? __builtin_amdgcn_exp2f(sc[i][h] - m1) : 0.0f;
+        sc[i][h] = p;
+        l[h] += p;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < NB; i++) {
+      float kf[PER];
+      row_of(i, kf);
+#pragma unroll
+      for (int h = 0; h < HQ; h++)
+#pragma unroll
+        for (int e = 0; e < PER; e++) o[h][e] = __builtin_fmaf(sc[i][h], kf[e], o[h][e]);
+    }
+  }
+  // the key groups' shares: maxima first, then the sums on a common scale
+  if (sub == 0) {
+#pragma unroll
+    for (int h = 0; h < HQ; h++) ml[0][w * GPW + grp][h] = m[h];
+  }
+  __syncthreads();
+  float mx[HQ];
+#pragma unroll
+  for (int h = 0; h < HQ; h++) {
+    mx[h] = ml[0][0][h];
+    for (uint32_t i = 1; i < 4 * GPW; i++) mx[h] = fmaxf(mx[h], ml[0][i][h]);
+    const float a = __builtin_amdgcn_exp2f(m[h] - mx[h]);
+    if (sub == 0) ml[1][w * GPW + grp][h] = l[h] * a;
+#pragma unroll
+    for (int e = 0; e < PER; e++) {
+      float v = o[h][e] * a;
+      if constexpr (GPW > 1) v += __shfl_xor(v, 32, 64);
+      if (lane < HALF) accs[((w * HQ + h) * HALF + lane) * PER + e] = v;
+    }
+  }
+  __syncthreads();
+  const size_t rows = (size_t)M * s.heads, r0 = (size_t)sp * rows + (size_t)z * s.heads + h0;
+  if (tid < hn) {
+    float lt = 0.0f;
+    for (uint32_t i = 0; i < 4 * GPW; i++) lt += ml[1][i][tid];
+    b.part_ml[(r0 + tid) * 2] = mx[0];
+    for (uint32_t h = 1; h < (uint32_t)HQ; h++)
+      if (tid == h) b.part_ml[(r0 + tid) * 2] = mx[h];
+    b.part_ml[(r0 + tid) * 2 + 1] = lt;
+  }
+  for (uint32_t i = tid; i < hn * s.dim; i += 256) {
+    const uint32_t h = i / s.dim, d = i % s.dim, ln = d / PER, e = d % PER;
+    float v = 0.0f;
+    for (uint32_t k = 0; k < 4; k++)
+      for (uint32_t x = ln; x < HALF; x += LPK) v += accs[((k * HQ + h) * HALF + x) * PER + e];
+    b.part_acc[(r0 + h) * s.dim + d] = v;
+  }
+}
+
+template <class T, uint32_t LPK, int HQ, bool OWN>
+static hipError_t tied_attn_go(const TiedShape& s, const TiedBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, hipStream_t st) {
+  const uint32_t gq = s.heads / s.kv_heads, chunks = (gq + HQ - 1) / HQ;
+  const size_t lds = (size_t)4 * HQ * (64 / LPK > 1 ? 32 : 64) * (16 / sizeof(T)) * 4;
+  hipLaunchKernelGGL((tied_attn_kernel<T, LPK, HQ, OWN>), dim3(n_splits, s.kv_heads * chunks, M), dim3(256), lds, st, s, b, pos_ptr, pos0, M, n_splits);
+  return hipGetLastError();
+}
+template <class T, uint32_t LPK>
+static hipError_t tied_attn_pick(const TiedShape& s, const TiedBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, bool own, uint32_t n_splits, hipStream_t st) {
+  const uint32_t gq = s.heads / s.kv_heads;
+#define LGH_TIED_CASE(N) return own ? tied_attn_go<T, LPK, N, true>(s, b, pos_ptr, pos0, M, n_splits, st) : tied_attn_go<T, LPK, N, false>(s, b, pos_ptr, pos0, M, n_splits, st)
+  if (gq == 1) LGH_TIED_CASE(1);
+  if (gq == 2) LGH_TIED_CASE(2);
+  LGH_TIED_CASE(4);
+#undef LGH_TIED_CASE
+}
+static bool tied_ok(const TiedShape& s) {
+  return s.heads && s.kv_heads && s.heads % s.kv_heads == 0 && s.dim && s.dim <= s.dp && s.dp % 64 == 0 && s.dp <= kTiedMaxDim && s.window && s.rows % 64 == 0;
+}
+
+hipError_t tied_attn_launch(const TiedShape& s, const TiedBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, bool own, uint32_t n_splits, bool f32, hipStream_t st) {
+  if (!tied_ok(s) || M == 0 || M > kTiedShort || (own && M != 1) || n_splits == 0 || n_splits > kTiedMaxSplits || (!pos_ptr && pos0 + M > s.rows)) return hipErrorInvalidValue;
+  switch (tied_lanes(s.dp, f32 ? 4 : 2)) {
+    case 8: return f32 ? hipErrorInvalidValue : tied_attn_pick<__bf16, 8>(s, b, pos_ptr, pos0, M, own, n_splits, st);
+    case 16: return f32 ? tied_attn_pick<float, 16>(s, b, pos_ptr, pos0, M, own, n_splits, st) : tied_attn_pick<__bf16, 16>(s, b, pos_ptr, pos0, M, own, n_splits, st);
+    case 32: return f32 ? tied_attn_pick<float, 32>(s, b, pos_ptr, pos0, M, own, n_splits, st) : tied_attn_pick<__bf16, 32>(s, b, pos_ptr, pos0, M, own, n_splits, st);
+    case 64: return f32 ? tied_attn_pick<float, 64>(s, b, pos_ptr, pos0, M, own, n_splits, st) : hipErrorInvalidValue;
+  }
+  return hipErrorInvalidValue;
+}
+
+// shares of the keys that fill the chip; not more than there are rounds of keys
+uint32_t tied_splits(const TiedShape& s, uint32_t max_seq, uint32_t M, bool f32, uint32_t forced) {
+  const uint32_t gq = s.heads / s.kv_heads, hq = gq <= 2 ? gq : 4, wgs = s.kv_heads * ((gq + hq - 1) / hq) * M;
+  const uint32_t kr = tied_round(tied_lanes(s.dp, f32 ? 4 : 2)), rounds = (tied_seen(s, max_seq - 1).total + kr - 1) / kr;
+  const uint32_t want = forced ? forced : std::max(1u, 512 / wgs);
+  return std::min(std::min(want, kTiedMaxSplits), std::max(rounds, 1u));
+}
+
+// the shares of the keys put together, the sink's term; grid (heads, tokens)
+template <class O>
+__global__ void __launch_bounds__(256) tied_merge_kernel(const TiedShape s, const TiedBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits,
+                                                         uint32_t kr, O* __restrict__ out, uint32_t ldo) {
+  __shared__ float part[256];
+  __shared__ float wgt[kTiedMaxSplits];
+  static_assert(kTiedMaxSplits == 128, "two splits per lane");
+  const uint32_t tid = threadIdx.x, lane = tid & 63, h = blockIdx.x, t = blockIdx.y;
+  const uint32_t pos = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + t;
+  const uint32_t rounds = (tied_seen(s, pos).total + kr - 1) / kr, per = (rounds + n_splits - 1) / n_splits, act = (rounds + per - 1) / per;
+  const size_t rows = (size_t)M * s.heads, r = (size_t)t * s.heads + h;
+  float mi[2], li[2];
+#pragma unroll
+  for (uint32_t k = 0; k < 2; k++) {
+    const uint32_t i = lane + k * 64, ic = i < act ? i : act - 1;
+    mi[k] = b.part_ml[(ic * rows + r) * 2];
+    li[k] = b.part_ml[(ic * rows + r) * 2 + 1] * (i < act ? 1.0f : 0.0f);
+  }
+  const float sink = b.sink[h] * kTiedLog2e;
+  // columns x groups of splits; the first partial sums are requested before the weights are known
+  const uint32_t cols = s.dim < 256 ? s.dim : 256, groups = 256 / cols, grp = tid / cols;
+  constexpr int F = 8;
+  float first[F];
+  const uint32_t c0 = tid % cols;
+#pragma unroll
+  for (int i = 0; i < F; i++) {
+    const uint32_t k = grp + i * groups;
+    first[i] = b.part_acc[((k < act ? k : act - 1) * rows + r) * s.dim + c0];
+  }
+  if (tid < 64) {
+    const float mm = fmaxf(wave_max(fmaxf(mi[0], mi[1])), sink);
+    const float f0 = __builtin_amdgcn_exp2f(mi[0] - mm), f1 = __builtin_amdgcn_exp2f(mi[1] - mm);
+    const float tot = wave_sum(f0 * li[0] + f1 * li[1]) + __builtin_amdgcn_exp2f(sink - mm);
+    wgt[lane] = f0 / tot; wgt[lane + 64] = f1 / tot;
+  }
+  __syncthreads();
+  float v = 0.0f;
+  if (grp < groups) {
+#pragma unroll
+    for (int i = 0; i < F; i++) {
+      const uint32_t k = grp + i * groups;
+      v = __builtin_fmaf(k < act ? wgt[k] : 0.0f, first[i], v);
+    }
+    for (uint32_t k = grp + F * groups; k < act; k += groups) v = __builtin_fmaf(wgt[k], b.part_acc[(k * rows + r) * s.dim + c0], v);
+  }
+  part[tid] = v;
+  __syncthreads();
+  if (tid < cols) {
+    for (uint32_t k = 1; k < groups; k++) v += part[tid + k * cols];
+    out[(size_t)t * ldo + h * s.dim + tid] = to_act<O>(v);
+  }
+}
+
+hipError_t tied_merge_launch(const TiedShape& s, const TiedBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32, void* out, uint32_t ldo,
+                             bool out_f32, hipStream_t st) {
+  if (!tied_ok(s) || n_splits == 0 || n_splits > kTiedMaxSplits || M == 0) return hipErrorInvalidValue;
+  const uint32_t kr = tied_round(tied_lanes(s.dp, f32 ? 4 : 2));
+  if (out_f32) hipLaunchKernelGGL(tied_merge_kernel<float>, dim3(s.heads, M), dim3(256), 0, st, s, b, pos_ptr, pos0, M, n_splits, kr, (float*)out, ldo);
+  else hipLaunchKernelGGL(tied_merge_kernel<__bf16>, dim3(s.heads, M), dim3(256), 0, st, s, b, pos_ptr, pos0, M, n_splits, kr, (__bf16*)out, ldo);
+  return hipGetLastError();
+}
+
+// a block's cache rows, key factors and queries; grid (tokens)
+template <class T>
+__global__ void __launch_bounds__(256) tied_prep_kernel(const TiedShape s, const TiedBufs b, uint32_t pos0) {
+  __shared__ float red[16];
+  const uint32_t t = blockIdx.x, pos = pos0 + t, tid = threadIdx.x, nq = s.heads * s.dim, nk = s.kv_heads * s.dim, gq = s.heads / s.kv_heads;
+  const float* cat = b.cat + (size_t)t * s.ldcat;
+  float sq = 0.0f, sk = 0.0f;
+  for (uint32_t i = tid; i < nq; i += 256) { const float v = cat[s.off_q + i]; sq = __builtin_fmaf(v, v, sq); }
+  for (uint32_t i = tid; i < nk; i += 256) {
+    const float v = cat[s.off_k + i];
+    sk = __builtin_fmaf(v, v, sk);
+    reinterpret_cast<T*>(b.cache)[((size_t)(i / s.dim) * s.rows + pos) * s.dp + i % s.dim] = to_act<T>(v);
+  }
+  const float qinv = 1.0f / __builtin_sqrtf(block_sum(sq, red) / (float)nq + s.eps) * s.scale;
+  const float kinv = 1.0f / __builtin_sqrtf(block_sum(sk, red) / (float)nk + s.eps);
+  if (tid == 0) b.kinv[pos] = kinv;
+  if (!b.q) return;
+  T* q = reinterpret_cast<T*>(b.q);
+  for (uint32_t i = tid; i < s.heads * s.dp; i += 256) {
+    const uint32_t h = i / s.dp, d = i % s.dp, dd = d < s.dim ? d : 0;
+    const float v = cat[s.off_q + h * s.dim + dd] * b.qn[h * s.dim + dd] * (b.kn[h / gq * s.dim + dd] * (qinv * b.temp[h]));
+    q[((size_t)h * b.Mcap + t) * s.dp + d] = to_act<T>(d < s.dim ? v : 0.0f);
+  }
+}
+
+hipError_t tied_prep_launch(const TiedShape& s, const TiedBufs& b, uint32_t pos0, uint32_t M, bool f32, hipStream_t st) {
+  if (!tied_ok(s) || M == 0 || (b.q && M > b.Mcap) || pos0 + M > s.rows) return hipErrorInvalidValue;
+  if (f32) hipLaunchKernelGGL(tied_prep_kernel<float>, dim3(M), dim3(256), 0, st, s, b, pos0);
+  else hipLaunchKernelGGL(tied_prep_kernel<__bf16>, dim3(M), dim3(256), 0, st, s, b, pos0);
+  return hipGetLastError();
+}
+
+// ------------------------------------------------------------------------------------------------
+// prompt portions.  A workgroup = 4 waves = 64 * QT queries of one head; S^T = K Q^T leaves a lane with one query's scores of keys
+// 4g .. 4g + 3, which is the operand of O^T = K^T P^T, whose key fragments come out of the same LDS tile by transposed reads.  Tiles of KT
+// keys go to LDS by DMA, two buffers: first the kept tiles in front of the window, then the tiles from the first query's window on.
+// ------------------------------------------------------------------------------------------------
+template <class T> constexpr int tied_kt() { return sizeof(T) == 2 ? 64 : 32; }
+template <class T, int DQ> constexpr size_t tied_lds() { return 2 * (size_t)tied_kt<T>() * DQ * sizeof(T); }
+template <class T, int DQ> constexpr int tied_wgs() { return DQ <= 128 ? 2 : 1; }
+
+template <class T, int DQ>
+__global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(const TiedShape s, const TiedBufs b, uint32_t pos0, uint32_t M, uint32_t nqb, T* __restrict__ out,
+                                                                              uint32_t ldo) {
+  constexpr bool BF = sizeof(T) == 2;
+  constexpr int KT = tied_kt<T>(), QT = BF ? 2 : 1, NK = KT / 16, NU = DQ / Frag<T>::KU, ND = DQ / 16;
+  constexpr uint32_t XC = DQ * sizeof(T) / 16, kBuf = KT * XC * 16;
+  extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
+  const uint32_t lane = threadIdx.x & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)), r16 = lane & 15, g = lane >> 4;
+  // the longest rows first, and of the second half of the grid the shortest first (workgroups i and i + half share a CU when all are resident)
+  const uint32_t h = blockIdx.x % s.heads, qi = blockIdx.x / s.heads, hi = (nqb + 1) / 2, qb = qi < hi ? nqb - 1 - qi : qi - hi;
+  const uint32_t q0 = qb * 64 * QT, qw = q0 + w * 16 * QT, qlast = q0 + 64 * QT - 1 < M - 1 ? q0 + 64 * QT - 1 : M - 1;
+  const uint32_t ifirst = pos0 + q0, lo = ifirst + 1 > s.window ? ifirst + 1 - s.window : 0, tw = lo / KT;
+  const uint32_t kt = (s.keep + KT - 1) / KT, nkt = kt < tw ? kt : tw;                // kept tiles in front of the window's first one
+  const uint32_t tiles = nkt + (pos0 + qlast) / KT + 1 - tw;
+  const T* K = reinterpret_cast<const T*>(b.cache) + (size_t)(h / (s.heads / s.kv_heads)) * s.rows * DQ;
+  const uint32_t lds0 = (uint32_t)__builtin_amdgcn_readfirstlane((int)lds_addr_of(smem));
+  auto tile_at = [&](uint32_t i) { return i < nkt ? i : tw + i - nkt; };
+  auto stage = [&](uint32_t tl, uint32_t buf) {
+#pragma unroll
+    for (int i = 0; i < (int)(kBuf / 4096); i++) {
+      const uint32_t c = (i * 4 + w) * 64 + lane, row = c / XC, ch = (c % XC) ^ (row & 7);
+      lds_dma16_untracked(K + ((size_t)tl * KT + row) * DQ + ch * (16 / sizeof(T)), lds0 + buf * kBuf + (i * 4 + w) * 1024);
+    }
+  };
+  f32x4 kin[NK];
+  auto factors = [&](uint32_t tl) {
+#pragma unroll
+    for (int n = 0; n < NK; n++) kin[n] = *reinterpret_cast<const f32x4*>(b.kinv + (size_t)tl * KT + n * 16 + g * 4);
+  };
+  factors(tile_at(0));
+  stage(tile_at(0), 0);
+  typename Frag<T>::V qf[QT][NU];
+#pragma unroll
+  for (int t = 0; t < QT; t++) {
+    const uint32_t m = qw + t * 16 + r16;
+    const T* qr = reinterpret_cast<const T*>(b.q) + ((size_t)h * b.Mcap + (m < M ? m : M - 1)) * DQ + g * Frag<T>::PER;
+#pragma unroll
+    for (int u = 0; u < NU; u++) qf[t][u] = Frag<T>::load(qr + u * Frag<T>::KU);
+  }
+  f32x4 o[ND][QT];
+  float mx[QT], l[QT];
+#pragma unroll
+  for (int t = 0; t < QT; t++) {
+    mx[t] = kTiedNeg; l[t] = 0.0f;
+#pragma unroll
+    for (int i = 0; i < ND; i++) o[i][t] = (f32x4)(0.0f);
+  }
+  const CapF cap(s.cap);
+  const float slope = tied_slope(h, s.heads);
+  const uint32_t iw0 = pos0 + qw, iw1 = iw0 + 16 * QT - 1;      // this wave's queries
+  wait_vm(0);
+  __syncthreads();
+  for (uint32_t it = 0; it < tiles; it++) {
+    const uint32_t cur = it & 1, k0 = tile_at(it) * KT, k1 = k0 + KT - 1;
+    f32x4 kc[NK];
+#pragma unroll
+    for (int n = 0; n < NK; n++) kc[n] = kin[n];
+    if (it + 1 < tiles) {
+      factors(tile_at(it + 1));
+      stage(tile_at(it + 1), cur ^ 1);
+    }
+    // (wave-uniform) no query of this wave sees the tile / every one sees all of it
+    const bool none = k0 > iw1 || (iw0 > k1 && iw0 - k1 >= s.window && k0 >= s.keep);
+    const bool full = k1 <= iw0 && (iw1 - k0 < s.window || k1 < s.keep);
+    if (!none) {
+      const T* tile = reinterpret_cast<const T*>(smem + cur * kBuf);
+      f32x4 sa[NK][QT];
+#pragma unroll
+      for (int n = 0; n < NK; n++)
+#pragma unroll
+        for (int t = 0; t < QT; t++) sa[n][t] = (f32x4)(0.0f);
+#pragma unroll
+      for (int u = 0; u < NU; u++)
+#pragma unroll
+        for (int n = 0; n < NK; n++) {
+          const uint32_t row = n * 16 + r16;
+          const typename Frag<T>::V kf = Frag<T>::load(tile + row * DQ + (((uint32_t)(u * 4) + g) ^ (row & 7)) * Frag<T>::PER);
+#pragma unroll
+          for (int t = 0; t < QT; t++) sa[n][t] = Frag<T>::mma(kf, qf[t][u], sa[n][t]);
+        }
+      float top = 0.0f;
+#pragma unroll
+      for (int t = 0; t < QT; t++)
+#pragma unroll
+        for (int n = 0; n < NK; n++)
+#pragma unroll
+          for (int e = 0; e < 4; e++) {
+            sa[n][t][e] *= kc[n][e];
+            top = fmaxf(top, fabsf(sa[n][t][e]));
+          }
+      const bool large = __any(!(top < cap.lim));
+#pragma unroll
+      for (int t = 0; t < QT; t++) {
+        const uint32_t i = iw0 + t * 16 + r16;
+        const float off = slope * ((float)(int)(k0 + g * 4 - i));    // - slope * (i - j) of the lane's first key
+#pragma unroll
+        for (int n = 0; n < NK; n++)
+#pragma unroll
+          for (int e = 0; e < 4; e++) {
+            const float x = sa[n][t][e];
+            sa[n][t][e] = __builtin_fmaf(slope, (float)(n * 16 + e), off) + (large ? cap.any(x) : cap.small(x));
+          }
+        if (!full) {
+          asm volatile("");              // (kept a branch: most tiles have no masks to apply)
+#pragma unroll
+          for (int n = 0; n < NK; n++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+              const uint32_t j = k0 + n * 16 + g * 4 + e;
+              sa[n][t][e] = j <= i && (i - j < s.window || j < s.keep) ? sa[n][t][e] : kTiedNeg;
+            }
+        }
+        float m1 = mx[t];
+#pragma unroll
+        for (int n = 0; n < NK; n++)
+#pragma unroll
+          for (int e = 0; e < 4; e++) m1 = fmaxf(m1, sa[n][t][e]);
+        m1 = fmaxf(m1, __shfl_xor(m1, 16, 64));
+        m1 = fmaxf(m1, __shfl_xor(m1, 32, 64));
+        // (a query that has seen nothing yet weighs masked keys; the factor of its first visible tile takes that to 0)
+        const float a = __builtin_amdgcn_exp2f(mx[t] - m1);
+        float sum = 0.0f;
+#pragma unroll
+        for (int n = 0; n < NK; n++)
+#pragma unroll
+          for (int e = 0; e < 4; e++) {
+            const float p = __builtin_amdgcn_exp2f(sa[n][t][e] - m1);
+            sa[n][t][e] = p;
+            sum += p;
+          }
+        l[t] = __builtin_fmaf(l[t], a, sum);
+        if (__any(m1 > mx[t])) {
+#pragma unroll
+          for (int d = 0; d < ND; d++) o[d][t] *= a;
+        }
+        mx[t] = m1;
+      }
+      if constexpr (BF) {
+#pragma unroll
+        for (int u = 0; u < KT / 32; u++) {
+          bf16x8 pf[QT];
+#pragma unroll
+          for (int t = 0; t < QT; t++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) { pf[t][e] = (__bf16)sa[2 * u][t][e]; pf[t][4 + e] = (__bf16)sa[2 * u + 1][t][e]; }
+#pragma unroll
+          for (int d = 0; d < ND; d++) {
+            const bf16x8 vf = tile_value_frag<T>(tile + u * 32 * DQ, DQ, 0, d * 16, r16, g);
+#pragma unroll
+            for (int t = 0; t < QT; t++) o[d][t] = Frag<T>::mma(vf, pf[t], o[d][t]);
+          }
+        }
+      } else {
+#pragma unroll
+        for (int n = 0; n < NK; n++)
+#pragma unroll
+          for (int d = 0; d < ND; d++) {
+            const f32x4 vf = tile_value_frag<T>(tile, DQ, n, d * 16, r16, g);
+#pragma unroll
+            for (int t = 0; t < QT; t++) o[d][t] = Frag<T>::mma(vf, sa[n][t], o[d][t]);
+          }
+      }
+    }
+    wait_vm(0);
+    __syncthreads();
+  }
+  const float sink = b.sink[h] * kTiedLog2e;
+#pragma unroll
+  for (int t = 0; t < QT; t++) {
+    float lt = l[t];
+    lt += __shfl_xor(lt, 16, 64);
+    lt += __shfl_xor(lt, 32, 64);
+    const uint32_t m = qw + t * 16 + r16;
+    if (m >= M) continue;
+    const float mm = fmaxf(mx[t], sink), a = __builtin_amdgcn_exp2f(mx[t] - mm), fac = a / (lt * a + __builtin_amdgcn_exp2f(sink - mm));
+    T* dst = out + (size_t)m * ldo + h * s.dim;
+#pragma unroll
+    for (int d = 0; d < ND; d++)
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        const uint32_t v = d * 16 + g * 4 + e;
+        if (v < s.dim) dst[v] = to_act<T>(o[d][t][e] * fac);
+      }
+  }
+}
+
+template <class T, int DQ>
+static hipError_t tied_flash_go(const TiedShape& s, const TiedBufs& b, uint32_t pos0, uint32_t M, void* out, uint32_t ldo, hipStream_t st) {
+  static bool opted[64] = {};
+  constexpr size_t lds = tied_lds<T, DQ>();
+  static_assert(lds <= 160 * 1024, "two tiles fit LDS");
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&tied_flash_kernel<T, DQ>), (int)lds, opted); e != hipSuccess) return e;
+  const uint32_t QB = sizeof(T) == 2 ? 128 : 64, nqb = (M + QB - 1) / QB;
+  hipLaunchKernelGGL((tied_flash_kernel<T, DQ>), dim3(nqb * s.heads), dim3(256), lds, st, s, b, pos0, M, nqb, (T*)out, ldo);
+  return hipGetLastError();
+}
+
+hipError_t tied_flash_launch(const TiedShape& s, const TiedBufs& b, uint32_t pos0, uint32_t M, bool f32, void* out, uint32_t ldo, hipStream_t st) {
+  if (!tied_ok(s) || !b.q || M == 0 || M > b.Mcap || (uint64_t)(pos0 + M + 63) / 64 * 64 > s.rows) return hipErrorInvalidValue;   // whole key tiles are read
+#define LGH_FLASH_CASE(Q) if (s.dp == Q) return f32 ? tied_flash_go<float, Q>(s, b, pos0, M, out, ldo, st) : tied_flash_go<__bf16, Q>(s, b, pos0, M, out, ldo, st);
+  LGH_FLASH_CASE(64) LGH_FLASH_CASE(128) LGH_FLASH_CASE(192) LGH_FLASH_CASE(256)
+#undef LGH_FLASH_CASE
+  return hipErrorInvalidValue;
+}
+
+}  // namespace lgh

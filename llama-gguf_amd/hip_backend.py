@@ -40,15 +40,15 @@ ABI_SYMBOLS = (
     "lgh_batch_create", "lgh_batch_reset", "lgh_batch_position", "lgh_batch_prefill", "lgh_forward_multi", "lgh_decode_greedy_multi",
 )
 
-K_NAMES = ("embed", "qkv", "attn", "attn_combine", "wo", "gate_up", "down", "router", "output", "argmax", "misc", "token", "expand")
+K_NAMES = ("embed", "qkv", "attn", "attn_combine", "wo", "gate_up", "down", "router", "output", "argmax", "misc", "token", "expand", "experts")
 K_COUNT = 16
-SYM_COUNT = 24
+SYM_COUNT = 25
 # kernel symbols as rocprofv3 prints them (LGH_SYM_* order)
 SYM_NAMES = ("lgh::mv_kernel<1u, 1024>", "lgh::mv_kernel<8u, 1024>", "lgh::mv_kernel<16u, 1024>",
              "lgh::mv_kernel<2u, 768>", "lgh::mv_kernel<4u, 512>", "lgh::mv_kernel<5u, 512>", "lgh::mv_kernel<6u, 512>",
              "lgh::mv_kernel<31u, 512>", "lgh::f32_matvec_kernel", "lgh::attn_partial_kernel", "lgh::attn_combine_kernel",
              "lgh::embed_kernel", "lgh::argmax_stage1+2", "lgh::moe_router_kernel", "other", "lgh::mvq_kernel<1u>", "lgh::mvq_kernel<2u>", "lgh::mvq_kernel<3u>", "lgh::mvq_kernel<4u>",
-             "lgh::mvq_kernel<8u>", "unused", "lgh::lin_mv / lin_gemm", "lgh::latent_*", "lgh::mlstm_*")
+             "lgh::mvq_kernel<8u>", "unused", "lgh::lin_mv / lin_gemm", "lgh::latent_*", "lgh::mlstm_*", "lgh::tied_*")
 FLAG_NO_GRAPH = 1
 FLAG_EXACT_PREFILL = 4   # forward_batch feeds tokens one by one (f32 throughout) instead of the batched f16 GEMM path
 KV_F32, KV_INT8, KV_FP8_E4M3, KV_FP8_E5M2 = 0, 1, 2, 3   # lgh_model_desc.kv_cache_type: f32, or QuantizedKVCache's formats (kv_quantized.rs; no CLI flag reaches them)
@@ -82,19 +82,21 @@ class ModelDesc(C.Structure):
 
 class LayerDesc(C.Structure):
     """lgh_layer_desc: one layer of a model described layer by layer."""
-    _fields_ = ([(n, C.c_uint32) for n in ("struct_size", "mixer", "heads", "dim", "vdim", "kv_rank", "rot_dim", "rot_dims", "ff_kind", "ff")]
-                + [(n, C.c_double) for n in ("scale", "rot_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow", "gate_cap")])
+    _fields_ = ([(n, C.c_uint32) for n in ("struct_size", "mixer", "heads", "dim", "vdim", "kv_rank", "rot_dim", "rot_dims", "ff_kind", "ff",
+                                         "kv_heads", "window", "keep_first", "experts", "top", "shared_ff")]
+                + [(n, C.c_double) for n in ("scale", "rot_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow", "gate_cap", "score_cap")])
 
 
 class LayeredDesc(C.Structure):
     """lgh_layered_desc."""
     _fields_ = ([(n, C.c_uint32) for n in ("struct_size", "width", "vocab_size", "num_layers", "max_seq_len", "compute")]
                 + [("device_id", C.c_int32), ("flags", C.c_uint32), ("bigram_buckets", C.c_uint32), ("bigram_mul_prev", C.c_uint64),
-                   ("bigram_mul_cur", C.c_uint64), ("norm_eps", C.c_double), ("residual_mult", C.c_double)])
+                   ("bigram_mul_cur", C.c_uint64), ("norm_eps", C.c_double), ("residual_mult", C.c_double), ("residual", C.c_uint32), ("conv_taps", C.c_uint32)])
 
 
-MIXER_LATENT_ATTENTION, MIXER_MLSTM = 1, 2      # LGH_MIXER_*
-FF_NONE, FF_GEGLU = 0, 1                        # LGH_FF_*
+MIXER_LATENT_ATTENTION, MIXER_MLSTM, MIXER_TIED_ATTENTION = 1, 2, 3      # LGH_MIXER_*
+FF_NONE, FF_GEGLU, FF_MOE = 0, 1, 2             # LGH_FF_*
+RESIDUAL_POST_LN, RESIDUAL_SANDWICH_DYT = 0, 1  # LGH_RESIDUAL_*
 COMPUTE_BF16, COMPUTE_F32 = 0, 1                # LGH_COMPUTE_*
 
 

@@ -55,12 +55,37 @@ def _mlstm(layer: hb.LayerDesc, mx: dict, where: str) -> None:
     layer.gate_cap = float(_need(mx, "gate_cap", where))
 
 
+def _tied_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_TIED_ATTENTION
+    _sizes(layer, mx, where, heads="heads", kv_heads="kv_heads", dim="dim")
+    layer.vdim = int(mx.get("vdim") or layer.dim)
+    if layer.vdim != layer.dim:
+        raise ConfigError(f"{where}: values are keys, 'vdim' {layer.vdim} differs from 'dim' {layer.dim}")
+    if not layer.kv_heads or layer.heads % layer.kv_heads:
+        raise ConfigError(f"{where}: {layer.heads} heads do not divide into {layer.kv_heads} key heads")
+    layer.scale = float(_need(mx, "scale", where))
+    layer.score_cap = float(mx.get("softcap") or 0.0)
+    mask = mx.get("mask")
+    if mask:
+        layer.window, layer.keep_first = int(_need(mask, "size", where)), int(mask.get("keep_first") or 0)
+        if layer.window < 1:
+            raise ConfigError(f"{where}: a window of {layer.window} positions")
+
+
 def _dense(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
     layer.ff_kind, layer.ff = hb.FF_GEGLU, int(_need(mlp, "ff", where))
 
 
-MIXERS = {"latent_attention": _latent_attention, "mlstm": _mlstm}
-FEED_FORWARDS = {"dense": _dense}
+def _moe(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
+    layer.ff_kind, layer.ff = hb.FF_MOE, int(_need(_need(mlp, "expert", where), "ff", where))
+    router = _need(mlp, "router", where)
+    layer.experts, layer.top = int(_need(router, "experts", where)), int(_need(router, "top", where))
+    if mlp.get("shared"):
+        layer.shared_ff = int(_need(mlp["shared"], "ff", where))
+
+
+MIXERS = {"latent_attention": _latent_attention, "mlstm": _mlstm, "attention": _tied_attention}
+FEED_FORWARDS = {"dense": _dense, "moe": _moe}
 
 
 @dataclass
@@ -72,6 +97,8 @@ class LayeredConfig:
     residual_mult: float
     layers: List[hb.LayerDesc] = field(default_factory=list)
     bigram: Optional[Tuple[int, int, int]] = None      # buckets, factor of the previous token, factor of the token
+    residual: int = hb.RESIDUAL_POST_LN
+    conv_taps: int = 0
 
     @property
     def num_layers(self) -> int:
@@ -82,6 +109,7 @@ class LayeredConfig:
         d.struct_size = hb.C.sizeof(hb.LayeredDesc)
         d.width, d.vocab_size, d.num_layers = self.hidden_size, self.vocab_size, self.num_layers
         d.norm_eps, d.residual_mult = self.norm_eps, self.residual_mult
+        d.residual, d.conv_taps = self.residual, self.conv_taps
         if self.bigram:
             d.bigram_buckets, d.bigram_mul_prev, d.bigram_mul_cur = self.bigram
         return d
@@ -89,15 +117,30 @@ class LayeredConfig:
     def layer_descs(self):
         return (hb.LayerDesc * self.num_layers)(*self.layers)
 
+    def _norm_shapes(self, name: str) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        yield name, (self.hidden_size,)
+        if self.residual == hb.RESIDUAL_SANDWICH_DYT:
+            yield name + ".b", (self.hidden_size,)
+            yield name + ".alpha", ()
+
+    def _sublayer_shapes(self, p: str, which: int) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        """What surrounds a layer's mixer (1) or feed-forward (2)."""
+        yield from self._norm_shapes(f"{p}norm{which}")
+        if self.residual == hb.RESIDUAL_SANDWICH_DYT:
+            yield from self._norm_shapes(f"{p}norm{which}b")
+        if self.conv_taps:
+            yield f"{p}canon{which}", (self.hidden_size, self.conv_taps)
+
     def tensor_shapes(self) -> Iterator[Tuple[str, Tuple[int, ...]]]:
         """(name, shape) of every tensor the model needs, [out, in]."""
         W = self.hidden_size
+        ff = lambda p, n: ((p + "gate", (n, W)), (p + "up", (n, W)), (p + "down", (W, n)))
         yield "embed", (self.vocab_size, W)
         if self.bigram:
             yield "bigram", (self.bigram[0] + 1, W)
         for i, l in enumerate(self.layers):
             p, vd = f"l{i}.", l.heads * l.vdim
-            yield p + "norm1", (W,)
+            yield from self._sublayer_shapes(p, 1)
             if l.mixer == hb.MIXER_LATENT_ATTENTION:
                 yield p + "mix.q", (l.heads * (l.dim + l.rot_dim), W)
                 yield p + "mix.dkv", (l.kv_rank + l.rot_dim, W)
@@ -105,6 +148,12 @@ class LayeredConfig:
                 yield p + "mix.uk", (l.heads * l.dim, l.kv_rank)
                 yield p + "mix.uv", (vd, l.kv_rank)
                 yield p + "mix.g", (l.heads, W)
+            elif l.mixer == hb.MIXER_TIED_ATTENTION:
+                for n, rows in (("q", vd), ("k", l.kv_heads * l.dim)):
+                    yield p + "mix." + n, (rows, W)
+                    yield p + "mix." + n + ".norm", (rows,)
+                yield p + "mix.temp", (l.heads,)
+                yield p + "mix.sink", (l.heads,)
             else:
                 yield p + "mix.q", (l.heads * l.dim, W)
                 yield p + "mix.k", (l.heads * l.dim, W)
@@ -116,11 +165,16 @@ class LayeredConfig:
                     yield p + "mix." + g + ".b", (l.heads,)
             yield p + "mix.o", (W, vd)
             if l.ff_kind:
-                yield p + "norm2", (W,)
-                yield p + "mlp.gate", (l.ff, W)
-                yield p + "mlp.up", (l.ff, W)
-                yield p + "mlp.down", (W, l.ff)
-        yield "final.norm", (W,)
+                yield from self._sublayer_shapes(p, 2)
+            if l.ff_kind == hb.FF_MOE:
+                yield p + "mlp.router", (l.experts, W)
+                for e in range(l.experts):
+                    yield from ff(f"{p}mlp.e{e}.", l.ff)
+                if l.shared_ff:
+                    yield from ff(p + "mlp.shared.", l.shared_ff)
+            elif l.ff_kind:
+                yield from ff(p + "mlp.", l.ff)
+        yield from self._norm_shapes("final.norm")
         yield "head", (self.vocab_size, W)
 
 
@@ -133,6 +187,25 @@ def _zamelix(cfg: dict) -> LayeredConfig:
     big = (cfg.get("embedding") or {}).get("bigram")
     if big:
         out.bigram = tuple(int(_need(big, k, where)) for k in ("buckets", "mul_prev", "mul_cur"))
+    _layers(out, cfg, where)
+    return out
+
+
+def _pubopel(cfg: dict) -> LayeredConfig:
+    """Windowed attention whose values are its keys, mixtures of experts, squashing norms before and after every sublayer, a short causal
+    convolution in front of it."""
+    where = "Pubopel"
+    out = LayeredConfig(where, int(_need(cfg, "width", where)), int(_need(cfg, "vocab", where)),
+                        float(_need(_need(cfg, "norm", where), "eps", where)), 1.0, residual=hb.RESIDUAL_SANDWICH_DYT)
+    out.conv_taps = int(_need(_need(cfg, "canon", where), "taps", where))
+    if out.conv_taps < 1:
+        raise ConfigError(f"{where}: a convolution of {out.conv_taps} taps")
+    _layers(out, cfg, where)
+    return out
+
+
+def _layers(out: LayeredConfig, cfg: dict, where: str) -> None:
+    """The 'layers' list: a mixer and an optional feed-forward each."""
     for i, entry in enumerate(_need(cfg, "layers", where)):
         at = f"{where} layer {i}"
         layer = hb.LayerDesc()
@@ -147,10 +220,9 @@ def _zamelix(cfg: dict) -> LayeredConfig:
                 raise ConfigError(f"{at}: unknown feed-forward '{mlp['kind']}'")
             FEED_FORWARDS[mlp["kind"]](layer, mlp, at)
         out.layers.append(layer)
-    return out
 
 
-ARCHITECTURES = {"Zamelix": _zamelix}      # config.json "architecture" -> parser
+ARCHITECTURES = {"Zamelix": _zamelix, "Pubopel": _pubopel}      # config.json "architecture" -> parser
 
 
 def parse_config(cfg: dict) -> LayeredConfig:
@@ -202,7 +274,7 @@ class LayeredModel:
     def tensors(self):
         for name, shape in self.config.tensor_shapes():
             t, data = self._source.get(name, shape)
-            yield name, t, tuple(reversed(shape)), data
+            yield name, t, tuple(reversed(shape)) or (1,), data
 
     def weight_bytes(self) -> int:
         return sum(2 * int(np.prod(s)) for _, s in self.config.tensor_shapes())

@@ -110,15 +110,122 @@ def mlstm(h, w, mx, eps):
     return out @ w["o"].T
 
 
+def visible_keys(i, mask):
+    """Positions that position i sees: all up to itself, or the last ``size`` of them and the sequence's first ``keep_first``."""
+    if not mask:
+        return list(range(i + 1))
+    return [j for j in range(i + 1) if i - j < mask["size"] or j < mask.get("keep_first", 0)]
+
+
+def head_slope(h, heads):
+    """What a unit of distance costs head h."""
+    return 2.0 ** (-8.0 * (h + 1) / heads)
+
+
+def soft_cap(s, cap):
+    return cap * np.tanh(s / cap) if cap else s
+
+
+def sink_softmax(s, sink):
+    """Weights of the scores s when the denominator has one more term, exp(sink)."""
+    m = max(s.max(), sink)
+    p = np.exp(s - m)
+    return p / (p.sum() + math.exp(sink - m))
+
+
+def tied_attention(h, w, mx, eps):
+    """Grouped attention whose values are its keys as they were projected; queries and keys are normed over all heads at once."""
+    T, H, G, d = len(h), mx["heads"], mx["kv_heads"], mx["dim"]
+    q = (rms(h @ w["q"].T, eps) * w["q.norm"]).reshape(T, H, d)
+    v = (h @ w["k"].T).reshape(T, G, d)
+    k = (rms(h @ w["k"].T, eps) * w["k.norm"]).reshape(T, G, d)
+    out = np.zeros((T, H, d), dtype=F)
+    for i in range(T):
+        seen = visible_keys(i, mx.get("mask"))
+        for n in range(H):
+            g = n // (H // G)
+            s = soft_cap((k[seen, g] @ q[i, n]) * mx["scale"] * w["temp"][n], mx.get("softcap"))
+            s = s - head_slope(n, H) * (i - np.array(seen, dtype=F))
+            out[i, n] = sink_softmax(s, w["sink"][n]) @ v[seen, g]
+    return out.reshape(T, H * d) @ w["o"].T
+
+
+def silu(z):
+    return z * sigmoid(z)
+
+
 def dense_ff(x, w):
     return (gelu_tanh(x @ w["gate"].T) * (x @ w["up"].T)) @ w["down"].T
 
 
-MIXERS = {"latent_attention": latent_attention, "mlstm": mlstm}
+def expert(x, w, name):
+    return (silu(x @ w[name + ".gate"].T) * (x @ w[name + ".up"].T)) @ w[name + ".down"].T
+
+
+def route(z, top):
+    """(expert, weight) of the ``top`` largest scores, largest first; the weights are the scores."""
+    s = sigmoid(z)
+    order = sorted(range(len(z)), key=lambda e: (-z[e], e))[:top]
+    return [(e, s[e]) for e in order]
+
+
+def moe_ff(x, w, mlp):
+    """Every token through its experts, each of which reads the token times its weight; a shared expert beside them."""
+    out = np.zeros_like(x)
+    for t, z in enumerate(x @ w["router"].T):
+        for e, g in route(z, mlp["router"]["top"]):
+            out[t] += expert(g * x[t], w, f"e{e}")
+    return out + expert(x, w, "shared") if mlp.get("shared") else out
+
+
+def dyt(x, w, b, alpha):
+    """A norm without statistics: a squashed multiple of every value."""
+    return np.tanh(alpha * x) * w + b
+
+
+def causal_conv(h, w):
+    """Every channel's own filter over time, w [width, taps], the last tap at the token itself; nothing before the first token."""
+    out = np.zeros_like(h)
+    taps = w.shape[1]
+    for t in range(len(h)):
+        for j in range(taps):
+            if t - taps + 1 + j >= 0:
+                out[t] += w[:, j] * h[t - taps + 1 + j]
+    return out
+
+
+MIXERS = {"latent_attention": latent_attention, "mlstm": mlstm, "attention": tied_attention}
+
+
+def feed_forward(x, w, mlp):
+    return moe_ff(x, w, mlp) if mlp["kind"] == "moe" else dense_ff(x, w)
+
+
+def forward_sandwich(cfg, weights, tokens, layers_out=None):
+    """Squashing norms before and after every sublayer, whose input is the normed stream plus a short causal convolution of it."""
+    W = {k: np.asarray(v, dtype=F) for k, v in weights.items()}
+    eps = cfg["norm"]["eps"]
+    norm = lambda v, name: dyt(v, W[name], W[name + ".b"], W[name + ".alpha"])
+    x = W["embed"][list(tokens)]
+    for i, lay in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        sub = lambda g: {k[len(p + g):]: v for k, v in W.items() if k.startswith(p + g)}
+
+        def read(n):
+            h = norm(x, f"{p}norm{n}")
+            return h + causal_conv(h, W[f"{p}canon{n}"])
+        x = x + norm(MIXERS[lay["type"]](read(1), sub("mix."), lay["mixer"], eps), p + "norm1b")
+        if lay["mlp"]:
+            x = x + norm(feed_forward(read(2), sub("mlp."), lay["mlp"]), p + "norm2b")
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return norm(x, "final.norm") @ W["head"].T
 
 
 def forward(cfg, weights, tokens, layers_out=None):
     """Logits [T, vocab] of a whole sequence; layers_out (a list) receives the residual stream after every layer."""
+    if "canon" in cfg:
+        return forward_sandwich(cfg, weights, tokens, layers_out)
     W = {k: np.asarray(v, dtype=F) for k, v in weights.items()}
     eps, m = cfg["norm"]["eps"], cfg["residual_mult"]
     x = W["embed"][list(tokens)]
@@ -130,7 +237,7 @@ def forward(cfg, weights, tokens, layers_out=None):
         sub = lambda g: {k[len(p + g):]: v for k, v in W.items() if k.startswith(p + g)}
         x = x + m * layer_norm(MIXERS[lay["type"]](x, sub("mix."), lay["mixer"], eps), W[p + "norm1"], eps)
         if lay["mlp"]:
-            x = x + m * layer_norm(dense_ff(x, sub("mlp.")), W[p + "norm2"], eps)
+            x = x + m * layer_norm(feed_forward(x, sub("mlp."), lay["mlp"]), W[p + "norm2"], eps)
         if layers_out is not None:
             layers_out.append(x.copy())
     return layer_norm(x, W["final.norm"], eps) @ W["head"].T
