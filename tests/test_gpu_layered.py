@@ -14,30 +14,7 @@ import layered_cases as lc
 from oracle import layered as lo
 
 pytestmark = pytest.mark.gpu
-TOL = {"f32": 2e-5, "bf16": 3e-2}
-DTYPES = ("f32", "bf16")
-
-
-def make(pkg, cfg, dtype, max_seq=256, seed=0, weights=None, **kw):
-    parsed = pkg.layered_model.parse_config(cfg)
-    W = weights if weights is not None else lc.Weights(parsed, seed)
-    hb = pkg.hip_backend
-    eng = pkg.HipGpuInference.from_layered(pkg.LayeredModel(parsed, W), max_seq, compute=hb.COMPUTE_F32 if dtype == "f32" else hb.COMPUTE_BF16, **kw)
-    return eng, W
-
-
-def check(got, want, dtype, what=""):
-    """f32: every row.  bf16: every row but the few whose read-out nearly cancels before its RMS norm, which magnifies the rounding of the
-    operands (the same rows are the worst of the f32 run, 20 times above the rest)."""
-    err = lc.row_error(got, want)
-    if dtype == "bf16" and len(err) >= 40:
-        assert err.max() <= 0.4, f"{what}: row {int(err.argmax())} off by {err.max():.2e}"
-        err = np.sort(err)[: int(0.96 * len(err))]
-    assert err.max() <= TOL[dtype], f"{what}: row {int(err.argmax())} of {len(err)} off by {err.max():.2e} (limit {TOL[dtype]:.0e})"
-
-
-def stepwise(eng, toks):
-    return np.array([eng.forward(int(t)) for t in toks])
+TOL, DTYPES, make, check, stepwise = lc.TOL, lc.DTYPES, lc.make, lc.check, lc.stepwise
 
 
 # every mechanism alone, and sizes at and around the kernels' granules: 1, not a multiple of 4 / 16 / 32 / 64, above a tile

@@ -210,3 +210,122 @@ def test_bench_sizes_are_models_the_registry_takes(pkg):
         shapes = dict(p.tensor_shapes())
         t, data = bench.RandomBf16().get("l0.mix.o", (8, 16))
         assert t == 30 and data.size == 128 and shapes["head"] == (sz["vocab"], sz["width"])
+
+
+# ---- the Pubopel design ----
+def test_visible_keys_and_slopes():
+    assert lo.visible_keys(3, None) == [0, 1, 2, 3]
+    assert lo.visible_keys(9, {"size": 3, "keep_first": 2}) == [0, 1, 7, 8, 9]
+    assert lo.visible_keys(2, {"size": 3, "keep_first": 5}) == [0, 1, 2] and lo.visible_keys(4, {"size": 1}) == [4]
+    assert lo.head_slope(7, 8) == pytest.approx(2.0 ** -8) and lo.head_slope(0, 8) == 0.5 and lo.head_slope(2, 3) == pytest.approx(2.0 ** -8)
+
+
+def test_sink_is_one_more_key_without_a_value():
+    s = np.array([0.3, -1.0, 2.0])
+    e = np.exp(np.append(s, 0.7))
+    assert lo.sink_softmax(s, 0.7) == pytest.approx(e[:3] / e.sum())
+    assert lo.sink_softmax(s, -np.inf).sum() == pytest.approx(1.0) and lo.sink_softmax(s, 900.0).sum() == pytest.approx(0.0)
+
+
+def test_soft_cap():
+    s = np.array([-1e4, -0.01, 0.0, 0.01, 1e4])
+    assert lo.soft_cap(s, 5.0) == pytest.approx([-5.0, -0.01, 0.0, 0.01, 5.0], rel=1e-5) and np.array_equal(lo.soft_cap(s, None), s)
+
+
+def test_tied_attention_equals_an_explicit_matrix_form():
+    """All positions at once with mask matrices, keys normed beforehand, heads repeated over their group."""
+    rng = np.random.default_rng(6)
+    T, Wd, H, G, d, mx = 13, 21, 6, 2, 5, None
+    mx = lc.tied(heads=H, kv_heads=G, dim=d, window=4, keep=2, cap=2.5, scale=0.8)["mixer"]
+    shapes = {"q": (H * d, Wd), "k": (G * d, Wd), "q.norm": (H * d,), "k.norm": (G * d,), "temp": (H,), "sink": (H,), "o": (Wd, H * d)}
+    w = {k: rng.standard_normal(s) for k, s in shapes.items()}
+    h = rng.standard_normal((T, Wd))
+    q, k = h @ w["q"].T, h @ w["k"].T
+    v = np.repeat(k.reshape(T, G, d), H // G, axis=1)
+    n = lambda x, g: x / np.sqrt((x * x).mean(-1, keepdims=True) + 1e-5) * g
+    q, kn = n(q, w["q.norm"]).reshape(T, H, d), np.repeat(n(k, w["k.norm"]).reshape(T, G, d), H // G, axis=1)
+    s = 2.5 * np.tanh(np.einsum("ihd,jhd->hij", q, kn) * 0.8 * w["temp"][:, None, None] / 2.5)
+    dist = np.arange(T)[:, None] - np.arange(T)[None]
+    s = s - (2.0 ** (-8.0 * np.arange(1, H + 1) / H))[:, None, None] * dist
+    s[:, (dist < 0) | ((dist >= 4) & (np.arange(T)[None] >= 2))] = -np.inf
+    e = np.exp(s)
+    out = np.einsum("hij,jhd->ihd", e / (e.sum(-1, keepdims=True) + np.exp(w["sink"])[:, None, None]), v)
+    assert np.allclose(lo.tied_attention(h, w, mx, 1e-5), out.reshape(T, -1) @ w["o"].T)
+
+
+def test_mixture_weights_the_experts_input():
+    rng = np.random.default_rng(7)
+    mlp = lc.moe(experts=5, top=2, ff=6, shared=4)
+    w = {"router": rng.standard_normal((5, 8))}
+    for n, f in [(f"e{i}", 6) for i in range(5)] + [("shared", 4)]:
+        w.update({n + ".gate": rng.standard_normal((f, 8)), n + ".up": rng.standard_normal((f, 8)), n + ".down": rng.standard_normal((8, f))})
+    x = rng.standard_normal((3, 8))
+    ex = lambda n, v: w[n + ".down"] @ ((w[n + ".gate"] @ v) / (1 + np.exp(-(w[n + ".gate"] @ v))) * (w[n + ".up"] @ v))
+    for t in range(3):
+        s = 1 / (1 + np.exp(-(w["router"] @ x[t])))
+        best = np.argsort(-s)[:2]
+        assert np.allclose(lo.moe_ff(x, w, mlp)[t], sum(ex(f"e{e}", s[e] * x[t]) for e in best) + ex("shared", x[t]))
+    assert [e for e, _ in lo.route(np.array([1.0, 3.0, 3.0, 2.0]), 3)] == [1, 2, 3]
+
+
+def test_convolution_and_squashing_norm():
+    h = np.array([[1.0, 10.0], [2.0, 20.0], [3.0, 30.0]])
+    w = np.array([[1.0, 2.0, 3.0], [0.0, 0.0, 1.0]])
+    assert lo.causal_conv(h, w).tolist() == [[3.0, 10.0], [8.0, 20.0], [14.0, 30.0]]
+    assert lo.dyt(np.array([0.0, 1e3]), np.array([2.0, 2.0]), np.array([0.5, 0.5]), 0.7).tolist() == [0.5, 2.5]
+
+
+def test_a_pubopel_sequence_does_not_see_its_future(pkg):
+    cfg = lc.sandwich([lc.tied(window=5, mlp=lc.moe()), lc.tied(window=0)], taps=4)
+    W = lc.Weights(pkg.layered_model.parse_config(cfg))
+    t = lc.tokens(14, cfg["vocab"])
+    assert np.allclose(lo.forward(cfg, W, t)[:9], lo.forward(cfg, W, t[:9]))
+
+
+def test_parse_pubopel_reads_every_size_and_constant(pkg):
+    hb = pkg.hip_backend
+    cfg = lc.sandwich([lc.tied(heads=9, kv_heads=3, dim=17, window=21, keep=5, scale=0.3, cap=11.0, mlp=lc.moe(7, 3, 19, 23)), lc.tied(window=0, cap=0)], eps=2e-6, taps=5)
+    p = pkg.layered_model.parse_config(cfg)
+    a, b = p.layers
+    assert (a.mixer, a.heads, a.kv_heads, a.dim, a.vdim, a.window, a.keep_first, a.scale, a.score_cap) == (hb.MIXER_TIED_ATTENTION, 9, 3, 17, 17, 21, 5, 0.3, 11.0)
+    assert (a.ff_kind, a.experts, a.top, a.ff, a.shared_ff) == (hb.FF_MOE, 7, 3, 19, 23)
+    assert (b.window, b.keep_first, b.score_cap, b.ff_kind) == (0, 0, 0.0, hb.FF_NONE)
+    d = p.desc()
+    assert (d.width, d.vocab_size, d.norm_eps, d.residual_mult, d.residual, d.conv_taps) == (88, 150, 2e-6, 1.0, hb.RESIDUAL_SANDWICH_DYT, 5)
+    shapes = dict(p.tensor_shapes())
+    assert shapes["l0.norm2b.alpha"] == () and shapes["l0.canon2"] == (88, 5) and shapes["l0.mlp.e6.down"] == (88, 19) and shapes["l0.mix.k.norm"] == (51,)
+    assert "l1.norm2" not in shapes and "l1.canon2" not in shapes and "l0.mlp.e7.up" not in shapes and shapes["final.norm.b"] == (88,)
+
+
+@pytest.mark.parametrize("break_it", [
+    lambda c: c.pop("canon"), lambda c: c["canon"].update(taps=0), lambda c: c["layers"][0]["mixer"].pop("kv_heads"), lambda c: c["layers"][0]["mixer"].update(vdim=8),
+    lambda c: c["layers"][0]["mixer"].update(kv_heads=4), lambda c: c["layers"][0]["mixer"]["mask"].update(size=0), lambda c: c["layers"][0]["mixer"].pop("scale"),
+    lambda c: c["layers"][0]["mlp"].pop("expert"), lambda c: c["layers"][0]["mlp"]["router"].pop("top"), lambda c: c["norm"].pop("eps")])
+def test_unusable_pubopel_configurations_are_refused(pkg, break_it):
+    c = lc.sandwich([lc.tied(mlp=lc.moe())])
+    break_it(c)
+    with pytest.raises(pkg.layered_model.ConfigError):
+        pkg.layered_model.parse_config(c)
+
+
+def test_scalars_in_a_model_folder(pkg, tmp_path):
+    cfg = lc.sandwich([lc.tied(mlp=lc.moe())])
+    W = lc.Weights(pkg.layered_model.parse_config(cfg))
+    lc.write_dir(tmp_path, cfg, W)
+    got = {name: (ne, data.tobytes()) for name, _, ne, data in pkg.LayeredModel.from_dir(str(tmp_path)).tensors()}
+    assert got.keys() == W.keys()
+    ne, raw = got["l0.norm1.alpha"]
+    assert ne == (1,) and (np.frombuffer(raw, "<u2").astype(np.uint32) << 16).view(np.float32)[0] == W["l0.norm1.alpha"]
+
+
+def test_create_refuses_unusable_experts_and_heads(pkg):
+    hb, parse = pkg.hip_backend, pkg.layered_model.parse_config
+
+    def status(cfg):
+        with pytest.raises(pkg.BackendError) as ei:
+            hb.HipGpuInference.from_layered(pkg.LayeredModel(parse(cfg), lc.Weights(parse(cfg))), 16)
+        return ei.value.variant
+    assert status(lc.sandwich([lc.tied(mlp=lc.moe(experts=2, top=3))])) == "InvalidArgument"
+    assert status(lc.sandwich([lc.tied(heads=1, kv_heads=1, dim=300)])) == "Unsupported"
+    assert status(lc.sandwich([lc.tied(mlp=lc.moe(experts=1, top=1, ff=8, shared=40000))], width=4, vocab=8)) == "Unsupported"
+    assert status(lc.sandwich([lc.tied()], taps=65)) == "Unsupported"
