@@ -123,8 +123,8 @@ def parse_args():
     ap.add_argument("--fake-stage", action="store_true",
                     help="CPU rehearsal of the N>1 launcher and hop protocol: gloo + pipeline.FakeStage, no GPU, no engine (not a measurement)")
     ap.add_argument("--layered", default="", metavar="SIZE[,SIZE]",
-                    help="models described layer by layer (latent attention + matrix memory) beside the Llama-style model of equal width, depth and "
-                         "feed-forward, random weights: " + ", ".join(LAYERED_SIZES) + " or all; not the headline metric")
+                    help="models described layer by layer (w*: latent attention + matrix memory; p*: windowed tied attention + mixtures) beside the "
+                         "Llama-style model of equal width, depth and feed-forward, random weights: " + ", ".join(LAYERED_SIZES) + " or all; not the headline metric")
     ap.add_argument("--layered-only", choices=("both", "layered", "closest"), default="both", help="with --layered: run one side (for a profiler)")
     ap.add_argument("--layered-context", type=int, default=2048, help="with --layered: prompt length")
     return ap.parse_args()
@@ -139,25 +139,39 @@ LAYERED_SIZES = {
                   closest=dict(num_heads=32, num_kv_heads=8, head_dim=128)),
     "w8192": dict(width=8192, ff=28672, vocab=128256, layers=4, heads=64, dim=128, rot=64, vdim=128, rank=512, mheads=8, mdim=512, mvdim=1024,
                   closest=dict(num_heads=64, num_kv_heads=8, head_dim=128)),
+    # mixtures of experts under windowed attention; closest: the Llama-style mixture with the same heads, experts and experts per token
+    "p2048": dict(design="Pubopel", width=2048, ff=2816, vocab=32000, layers=8, heads=32, kv_heads=4, dim=64, window=1024, experts=8, top=2, shared=2816,
+                  closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),
+    "p4096": dict(design="Pubopel", width=4096, ff=4096, vocab=32000, layers=4, heads=32, kv_heads=8, dim=128, window=4096, experts=8, top=2, shared=4096,
+                  closest=dict(num_heads=32, num_kv_heads=8, head_dim=128)),
+    "p2048e": dict(design="Pubopel", width=2048, ff=768, vocab=32000, layers=8, heads=32, kv_heads=4, dim=64, window=1024, experts=64, top=6, shared=1536,
+                   closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),   # (the closest model takes prompts of this one token by token)
+    "p8192": dict(design="Pubopel", width=8192, ff=8192, vocab=32000, layers=2, heads=64, kv_heads=8, dim=128, window=4096, experts=8, top=2, shared=8192,
+                  closest=dict(num_heads=64, num_kv_heads=8, head_dim=128)),
 }
 
 
 class RandomBf16:
-    """Random weights for a layered model: slices of one random block, scaled by 1 / sqrt(in); norm weights 1."""
+    """Random weights for a layered model: slices of one random block, scaled by 1 / sqrt(in); norm weights and temperatures 1."""
 
     def __init__(self, seed=1):
-        self.block = np.random.default_rng(seed).standard_normal(1 << 22, dtype=np.float32)
+        self.block, self.scaled = np.random.default_rng(seed).standard_normal(1 << 22, dtype=np.float32), {}
 
     def get(self, name, shape):
         n = int(np.prod(shape))
-        if len(shape) == 1:
-            v = np.ones(n, np.float32) if name.endswith("norm") or "norm" in name.rsplit(".", 1)[-1] else np.zeros(n, np.float32)
-            return 0, v
-        blk = ((self.block * np.float32(1.0 / np.sqrt(shape[1]))).view(np.uint32) >> 16).astype(np.uint16)
-        return 30, np.resize(np.roll(blk, len(name) * 7919), n)
+        if len(shape) <= 1:
+            return 0, np.full(n, 0.5 if not shape else 1.0 if "norm" in name.rsplit(".", 1)[-1] or name.endswith("temp") else 0.0, np.float32)
+        if shape[1] not in self.scaled:
+            self.scaled[shape[1]] = ((self.block * np.float32(1.0 / np.sqrt(shape[1]))).view(np.uint32) >> 16).astype(np.uint16)
+        return 30, np.resize(np.roll(self.scaled[shape[1]], len(name) * 7919), n)
 
 
 def layered_config(sz):
+    if sz.get("design") == "Pubopel":
+        layer = {"type": "attention", "mlp": {"kind": "moe", "expert": {"ff": sz["ff"]}, "router": {"experts": sz["experts"], "top": sz["top"]}, "shared": {"ff": sz["shared"]}},
+                 "mixer": {"heads": sz["heads"], "kv_heads": sz["kv_heads"], "dim": sz["dim"], "vdim": sz["dim"], "scale": sz["dim"] ** -0.5, "softcap": 30.0,
+                           "mask": {"size": sz["window"], "keep_first": 4}}}
+        return {"architecture": "Pubopel", "width": sz["width"], "vocab": sz["vocab"], "norm": {"eps": 1e-5}, "canon": {"taps": 4}, "layers": [layer] * sz["layers"]}
     attn = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": sz["ff"]},
             "mixer": {"heads": sz["heads"], "dim": sz["dim"], "rot_dim": sz["rot"], "vdim": sz["vdim"], "kv_rank": sz["rank"],
                       "scale": (sz["dim"] + sz["rot"]) ** -0.5, "rot": {"base": 10000.0, "dims": sz["rot"]}}}
@@ -217,8 +231,9 @@ def run_layered(args, pkg):
             r["layered"] = layered_measure(eng, prompt, steps, args.reps)
             eng.close()
         if args.layered_only != "layered":
+            moe = dict(num_experts=sz["experts"], num_experts_per_token=sz["top"], expert_intermediate_size=sz["ff"]) if "experts" in sz else {}
             c = pkg.ModelConfig(name="closest", hidden_size=sz["width"], intermediate_size=sz["ff"], num_layers=sz["layers"], vocab_size=sz["vocab"],
-                                max_seq_len=cap, **sz["closest"])
+                                max_seq_len=cap, **sz["closest"], **moe)
             eng = pkg.HipGpuInference.from_model(pkg.SynthModel(c, mix="Q8_0"), cap)
             r["closest"] = layered_measure(eng, prompt, steps, args.reps)
             eng.close()

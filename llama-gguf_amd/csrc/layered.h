@@ -163,8 +163,9 @@ hipError_t pair_sum_launch(float* y, uint32_t ldy, const float* pairs, uint32_t 
 
 // ---- moe_route.hip: a block's tokens to their experts ----
 struct MoeRoute {
-  const float* logits;         // [M][ldl]
-  uint32_t ldl, M, experts, top, bm;
+  const void* x;               // [M][ldx]
+  const uint16_t* router;      // [experts][kp]
+  uint32_t ldx, kp, M, experts, top, bm;
   int* sel;                    // [M * top] chosen experts, largest score first
   float* w;                    // [M * top] their scores
   int *seg, *tile_e, *tile_row;   // LinGroup, row tiles of bm rows
@@ -174,7 +175,7 @@ struct MoeRoute {
   uint32_t tiles;              // entries of tile_e / tile_row
 };
 uint32_t moe_max_tiles(uint32_t rows, uint32_t experts, uint32_t bm);
-hipError_t moe_route_launch(const MoeRoute& a, hipStream_t st);
+hipError_t moe_route_launch(const MoeRoute& a, bool f32, hipStream_t st);   // router product, scores, groups
 
 // ---- tied_attention.hip: grouped heads, values = keys before their norm ----
 struct TiedShape {

@@ -87,7 +87,7 @@ struct LayeredModel {
   float* rlogits = nullptr;
   int* sel = nullptr;
   uint32_t max_experts = 0, max_top = 0, max_pair_act = 0;   // (the last: top * columns of an expert)
-  float *brl = nullptr, *bpair = nullptr, *bselw = nullptr, *broww = nullptr;
+  float *bpair = nullptr, *bselw = nullptr, *broww = nullptr;
   int *bsel = nullptr, *bseg = nullptr, *btile_e = nullptr, *btile_row = nullptr, *bslot = nullptr, *bsrc = nullptr;
   void* bpact = nullptr;
   // tied attention's queries of a block
@@ -691,7 +691,7 @@ static int block_ensure(lgh_ctx* c) {
       {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * Bc * 8}, {(void**)&m.bmx, heads * Bc * 8},
       {(void**)&m.bdec, heads * Bc * 4}, {(void**)&m.bwgt, heads * Bc * 4}, {(void**)&m.bcdec, heads * chunks * 4}, {(void**)&m.bnk, chunks * hdim * 4},
       {(void**)&m.bx2, m.dyt() ? B * d.width * 4 : 0}, {(void**)&m.tails, m.hist_floats() * 4}, {&m.btq, B * m.max_tied_q * el},
-      {(void**)&m.brl, B * up(m.max_experts, 4) * 4}, {(void**)&m.bpair, B * m.max_top * up(d.width, 4) * 4}, {&m.bpact, B * m.max_pair_act * el},
+      {(void**)&m.bpair, B * m.max_top * up(d.width, 4) * 4}, {&m.bpact, B * m.max_pair_act * el},
       {(void**)&m.bsel, B * m.max_top * 4}, {(void**)&m.bselw, B * m.max_top * 4}, {(void**)&m.bslot, B * m.max_top * 4}, {(void**)&m.bsrc, B * m.max_top * 4},
       {(void**)&m.broww, B * m.max_top * 4}, {(void**)&m.bseg, (size_t)(m.max_experts + 1) * 4}, {(void**)&m.btile_e, m.max_top ? moe_tiles * 4 : 0},
       {(void**)&m.btile_row, m.max_top ? moe_tiles * 4 : 0},
@@ -786,12 +786,11 @@ static int block_moe(lgh_ctx* c, LayeredLayer& L, uint32_t ldx, uint32_t ldy, ui
   hipStream_t st = c->stream;
   int rc;
   const uint32_t E = L.d.experts, rows = M * L.d.top;
-  if ((rc = block_gemm(c, LGH_K_ROUTER, L.router, LE_F32, m.bxa, ldx, m.brl, up(E, 4), M))) return rc;
   MoeRoute r{};
-  r.logits = m.brl; r.ldl = up(E, 4); r.M = M; r.experts = E; r.top = L.d.top; r.bm = lin_group_rows(rows, std::min(rows, E));
+  r.x = m.bxa; r.ldx = ldx; r.router = L.router.w; r.kp = L.router.kp; r.M = M; r.experts = E; r.top = L.d.top; r.bm = lin_group_rows(rows, std::min(rows, E));
   r.sel = m.bsel; r.w = m.bselw; r.seg = m.bseg; r.tile_e = m.btile_e; r.tile_row = m.btile_row; r.slot = m.bslot; r.src = m.bsrc; r.roww = m.broww;
   r.tiles = moe_max_tiles(rows, E, r.bm);
-  if ((rc = run_k(c, LGH_K_ROUTER, LGH_SYM_OTHER, 0, [&] { return moe_route_launch(r, st); }))) return rc;
+  if ((rc = run_k(c, LGH_K_ROUTER, LGH_SYM_OTHER, 0, [&] { return moe_route_launch(r, m.f32, st); }))) return rc;
   LinGemm g{};
   g.grp.seg = r.seg; g.grp.tile_e = r.tile_e; g.grp.tile_row = r.tile_row; g.grp.tiles = r.tiles; g.grp.bm = r.bm;
   g.w = L.egu.w; g.n = g.np = L.egu_rows; g.kp = L.egu.kp; g.M = rows; g.x = m.bxa; g.ldx = ldx; g.out = m.bpact; g.ldo = L.edown.kp;

@@ -7,6 +7,7 @@
 
 namespace lgh {
 
+typedef float f32x2 __attribute__((ext_vector_type(2)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
 
@@ -41,59 +42,65 @@ __device__ __forceinline__ float tanh_f(float x) {
 __device__ __forceinline__ float rank_key(float z) { return z == z ? z : -INFINITY; }
 
 // The `top` largest of E logits in LDS (padded with -inf to a multiple of 4), the first of equals first: expert e's place is the number of
-// experts before it.  One thread per expert; sel[place], w[place] = its score.
-__device__ __forceinline__ void rank_experts(const float* z, uint32_t E, uint32_t top, int* sel, float* w) {
-  for (uint32_t e = threadIdx.x; e < E; e += blockDim.x) {
-    const float v = z[e];
-    uint32_t place = 0;
-    for (uint32_t j = 0; j < E; j += 4) {
-      const f32x4 q = *reinterpret_cast<const f32x4*>(z + j);
+// experts before it; sel[place], w[place] = its score.  One thread per expert.
+__device__ __forceinline__ void rank_expert(const float* z, uint32_t E, uint32_t top, uint32_t e, int* sel, float* w) {
+  const float v = z[e];
+  uint32_t place = 0;
+  for (uint32_t j = 0; j < E; j += 4) {
+    const f32x4 q = *reinterpret_cast<const f32x4*>(z + j);
 #pragma unroll
-      for (uint32_t i = 0; i < 4; i++) place += q[i] > v || (q[i] == v && j + i < e) ? 1u : 0u;
-    }
-    if (place < top) { sel[place] = (int)e; w[place] = sigmoid_f(v); }
+    for (uint32_t i = 0; i < 4; i++) place += q[i] > v || (q[i] == v && j + i < e) ? 1u : 0u;
   }
+  if (place < top) { sel[place] = (int)e; w[place] = sigmoid_f(v); }
 }
 
 // ---- residual form LGH_RESIDUAL_SANDWICH_DYT, one channel ----
 __device__ __forceinline__ float dyt_f(float v, float alpha, float w, float b) { return __builtin_fmaf(tanh_f(alpha * v), w, b); }
 
-// the convolution's taps before position p; nothing lies before position 0
-__device__ __forceinline__ float conv_past(const ConvW& cv, uint32_t width, uint32_t c, int p) {
-  float s = 0.0f;
-  for (uint32_t j0 = 1; j0 < cv.taps; j0 += 4) {
-    float w[4], h[4];
+// four of the convolution's taps before position p (wave-uniform), requested but not used yet; nothing lies before position 0
+struct ConvIn { float w[4], h[4]; };
+__device__ __forceinline__ void conv_fetch(const ConvW& cv, uint32_t width, uint32_t c, int p, uint32_t j0, ConvIn& o) {
 #pragma unroll
-    for (uint32_t i = 0; i < 4; i++) {   // clamped: the loads are unconditional
-      const uint32_t j = j0 + i;
-      const bool ok = j < cv.taps && (int)j <= p;
-      const uint32_t row = ok ? (uint32_t)(p - (int)j) % (cv.taps - 1) : 0u;
-      w[i] = cv.w[(size_t)c * cv.taps + (ok ? cv.taps - 1 - j : 0u)];
-      h[i] = cv.hist[(size_t)row * width + c];
-      w[i] = ok ? w[i] : 0.0f;
-    }
-#pragma unroll
-    for (uint32_t i = 0; i < 4; i++) s = __builtin_fmaf(w[i], h[i], s);
+  for (uint32_t i = 0; i < 4; i++) {   // clamped: the loads are unconditional
+    const uint32_t j = j0 + i;
+    const bool ok = j < cv.taps && (int)j <= p;
+    const uint32_t row = ok ? (uint32_t)(p - (int)j) % (cv.taps - 1) : 0u;
+    o.w[i] = cv.w[(size_t)c * cv.taps + (ok ? cv.taps - 1 - j : 0u)];
+    o.h[i] = cv.hist[(size_t)row * width + c];
   }
+}
+__device__ __forceinline__ float conv_use(const ConvW& cv, const ConvIn& in, int p, uint32_t j0, float s) {
+#pragma unroll
+  for (uint32_t i = 0; i < 4; i++) s = __builtin_fmaf(j0 + i < cv.taps && (int)(j0 + i) <= p ? in.w[i] : 0.0f, in.h[i], s);
   return s;
 }
 // what the residual update of a channel needs besides the sublayer's output
-struct PostIn { float x, pw, pb, nw, nb, past, wl; };
-__device__ __forceinline__ PostIn post_fetch(const PostUpdate& a, uint32_t c, int p) {
-  PostIn r;
-  r.x = a.x ? a.x[c] : 0.0f;
-  r.pw = a.post.w[c]; r.pb = a.post.b[c];
+struct PostIn { float x, pw, pb, nw, nb, wl; ConvIn in; };
+__device__ __forceinline__ void post_fetch_next(const PostUpdate& a, uint32_t c, int p, PostIn& r) {
   r.nw = a.next.w[c]; r.nb = a.next.b[c];
-  const bool cv = a.conv.taps != 0;
-  r.wl = cv ? a.conv.w[(size_t)c * a.conv.taps + a.conv.taps - 1] : 0.0f;
-  r.past = cv ? conv_past(a.conv, a.width, c, p) : 0.0f;
-  return r;
+  if (a.conv.taps) r.wl = a.conv.w[(size_t)c * a.conv.taps + a.conv.taps - 1];
+  if (a.conv.taps > 1) conv_fetch(a.conv, a.width, c, p, 1, r.in);
+}
+__device__ __forceinline__ void post_fetch(const PostUpdate& a, uint32_t c, int p, PostIn& r) {
+  r.x = a.x[c];
+  r.pw = a.post.w[c]; r.pb = a.post.b[c];
+  post_fetch_next(a, c, p, r);
 }
 // stream value v of channel c at position p -> the next sublayer's input
 __device__ __forceinline__ void post_input(const PostUpdate& a, const PostIn& r, uint32_t c, int p, float v, float nalpha) {
   const float h = dyt_f(v, nalpha, r.nw, r.nb);
-  if (a.conv.taps > 1) a.conv.hist[(size_t)((uint32_t)p % (a.conv.taps - 1)) * a.width + c] = h;
-  a.hout[c] = h + __builtin_fmaf(r.wl, h, r.past);
+  float o = h;
+  if (a.conv.taps) o = __builtin_fmaf(r.wl, h, o);
+  if (a.conv.taps > 1) {
+    o = conv_use(a.conv, r.in, p, 1, o);
+    for (uint32_t j = 5; j < a.conv.taps; j += 4) {
+      ConvIn in;
+      conv_fetch(a.conv, a.width, c, p, j, in);
+      o = conv_use(a.conv, in, p, j, o);
+    }
+    a.conv.hist[(size_t)((uint32_t)p % (a.conv.taps - 1)) * a.width + c] = h;
+  }
+  a.hout[c] = o;
 }
 __device__ __forceinline__ void post_finish(const PostUpdate& a, const PostIn& r, uint32_t c, int p, float y, float palpha, float nalpha) {
   const float v = __builtin_fmaf(a.mult, dyt_f(y, palpha, r.pw, r.pb), r.x);

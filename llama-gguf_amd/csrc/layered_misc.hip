@@ -14,8 +14,8 @@ __device__ __forceinline__ uint64_t bigram_row(const EmbedArgs& a, uint32_t pos,
 // One decode token: advances the position words, notes the token in the history, writes the residual stream (and, with `post`, the first
 // sublayer's input).  One workgroup.
 __global__ void __launch_bounds__(1024) layered_embed_kernel(const EmbedArgs a, int* state, float* __restrict__ x, const PostUpdate post, int with_post) {
-  const int p = state[ST_NEXT];
-  const uint32_t tok = (uint32_t)state[ST_TOKEN];
+  const int p = __builtin_amdgcn_readfirstlane(state[ST_NEXT]);
+  const uint32_t tok = (uint32_t)__builtin_amdgcn_readfirstlane(state[ST_TOKEN]);
   const uint32_t prev = p > 0 && a.bigram ? (uint32_t)a.hist[p - 1] : 0u;
   __syncthreads();
   if (threadIdx.x == 0) {
@@ -26,15 +26,22 @@ __global__ void __launch_bounds__(1024) layered_embed_kernel(const EmbedArgs a, 
   const uint16_t* e = a.embed + (size_t)tok * a.width;
   const uint16_t* b = a.bigram ? a.bigram + bigram_row(a, (uint32_t)p, prev, tok) * a.width : nullptr;
   const float alpha = with_post ? *post.next.alpha : 0.0f;
-  for (uint32_t i = threadIdx.x; i < a.width; i += blockDim.x) {
-    const float v = b ? bf_f(e[i]) + bf_f(b[i]) : bf_f(e[i]);
-    x[i] = v;
-    if (with_post) {
-      PostIn r;
-      r.nw = post.next.w[i]; r.nb = post.next.b[i];
-      r.wl = post.conv.taps ? post.conv.w[(size_t)i * post.conv.taps + post.conv.taps - 1] : 0.0f;
-      r.past = post.conv.taps ? conv_past(post.conv, post.width, i, p) : 0.0f;
-      post_input(post, r, i, p, v, alpha);
+  constexpr uint32_t U = 4;   // channels a thread has in flight
+  for (uint32_t i0 = threadIdx.x; i0 < a.width; i0 += U * 1024) {
+    PostIn r[U];
+    float v[U];
+#pragma unroll
+    for (uint32_t u = 0; u < U; u++) {
+      const uint32_t i = i0 + u * 1024 < a.width ? i0 + u * 1024 : i0;
+      v[u] = b ? bf_f(e[i]) + bf_f(b[i]) : bf_f(e[i]);
+      if (with_post) post_fetch_next(post, i, p, r[u]);
+    }
+#pragma unroll
+    for (uint32_t u = 0; u < U; u++) {
+      const uint32_t i = i0 + u * 1024;
+      if (i >= a.width) break;
+      x[i] = v[u];
+      if (with_post) post_input(post, r[u], i, p, v[u], alpha);
     }
   }
 }
@@ -163,11 +170,13 @@ template <int V> struct VecF { float v[V]; };
 template <int V> __device__ __forceinline__ VecF<V> load_vec(const float* p) {
   VecF<V> r;
   if constexpr (V == 4) { const f32x4 q = *reinterpret_cast<const f32x4*>(p); r.v[0] = q.x; r.v[1] = q.y; r.v[2] = q.z; r.v[3] = q.w; }
+  else if constexpr (V == 2) { const f32x2 q = *reinterpret_cast<const f32x2*>(p); r.v[0] = q.x; r.v[1] = q.y; }
   else r.v[0] = p[0];
   return r;
 }
 template <int V> __device__ __forceinline__ void store_vec(float* p, const VecF<V>& a) {
   if constexpr (V == 4) { f32x4 q; q.x = a.v[0]; q.y = a.v[1]; q.z = a.v[2]; q.w = a.v[3]; *reinterpret_cast<f32x4*>(p) = q; }
+  else if constexpr (V == 2) { f32x2 q; q.x = a.v[0]; q.y = a.v[1]; *reinterpret_cast<f32x2*>(p) = q; }
   else p[0] = a.v[0];
 }
 
@@ -271,8 +280,9 @@ hipError_t dyt_block_launch(const DytBlock& a, bool f32, hipStream_t st) {
       (a.pairs && !a.slot) || (nxt && (!a.next.w || !a.next.b || !a.next.alpha || a.ldx < a.width)) || (a.conv.taps && !a.conv.w) ||
       (a.conv.taps > 1 && (!a.conv.hist || !a.tail)) || (!nxt && a.conv.taps))
     return hipErrorInvalidValue;
-  const bool v4 = a.width % 4 == 0 && (!a.y || a.ldy % 4 == 0) && (!a.pairs || a.ldp % 4 == 0) && (!nxt || a.ldx % 4 == 0) && a.conv.taps <= 16;
-  if (v4) return f32 ? dyt_block_go<float, 4>(a, st) : dyt_block_go<__bf16, 4>(a, st);
+  const bool even = a.width % 4 == 0 && (!a.y || a.ldy % 4 == 0) && (!a.pairs || a.ldp % 4 == 0) && (!nxt || a.ldx % 4 == 0) && a.conv.taps <= 16;
+  if (even && (uint64_t)a.width * a.M <= 1u << 24) return f32 ? dyt_block_go<float, 2>(a, st) : dyt_block_go<__bf16, 2>(a, st);   // (enough waves)
+  if (even) return f32 ? dyt_block_go<float, 4>(a, st) : dyt_block_go<__bf16, 4>(a, st);
   return f32 ? dyt_block_go<float, 1>(a, st) : dyt_block_go<__bf16, 1>(a, st);
 }
 

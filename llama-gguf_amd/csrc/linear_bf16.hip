@@ -108,7 +108,7 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
   if (!MOE) { request(n0); request(n1); }
   int pos = 0;
   float palpha = 0.0f, nalpha = 0.0f;
-  if (POST) { pos = *a.post.pos; palpha = *a.post.post.alpha; nalpha = *a.post.next.alpha; }
+  if (POST) { pos = __builtin_amdgcn_readfirstlane(*a.post.pos); palpha = *a.post.post.alpha; nalpha = *a.post.next.alpha; }
   if (SRC == LS_EXPERTS) {
     const uint32_t ep = (a.experts + 3) & ~3u;
     for (uint32_t e = tid; e < ep; e += kMvThreads) zs[e] = e < a.experts ? rank_key(a.logits[e]) : -INFINITY;
@@ -162,7 +162,7 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
   for (uint32_t i = a.k + tid; i < a.kp; i += kMvThreads) xs[i] = 0.0f;
   __syncthreads();
   if (SRC == LS_EXPERTS) {
-    rank_experts(zs, a.experts, a.top, sel, selw);
+    for (uint32_t e = tid; e < a.experts; e += kMvThreads) rank_expert(zs, a.experts, a.top, e, sel, selw);
     __syncthreads();
     if (blockIdx.x == 0 && tid < a.top) a.sel[tid] = sel[tid];
   }
@@ -172,7 +172,7 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
     float acc[kMvR] = {0.0f, 0.0f, 0.0f, 0.0f};
     const uint32_t ch = g * kMvR + (lane & 3);   // POST: the channel this lane finishes
     PostIn pi;
-    if (POST && sub == 0) pi = post_fetch(a.post, ch < a.n ? ch : a.n - 1, pos);
+    if (POST && sub == 0) post_fetch(a.post, ch < a.n ? ch : a.n - 1, pos, pi);
     if (g < n_groups) {
       for (uint32_t p = 0; p < passes; p++) {
         const MvW cur = n0;

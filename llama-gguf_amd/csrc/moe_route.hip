@@ -5,12 +5,59 @@
 
 namespace lgh {
 
-__global__ void __launch_bounds__(256) moe_topk_kernel(const MoeRoute a) {
-  __shared__ __attribute__((aligned(16))) float z[kMaxExperts];
-  const uint32_t t = blockIdx.x, ep = (a.experts + 3) & ~3u;
-  for (uint32_t e = threadIdx.x; e < ep; e += 256) z[e] = e < a.experts ? rank_key(a.logits[(size_t)t * a.ldl + e]) : -INFINITY;
-  __syncthreads();
-  rank_experts(z, a.experts, a.top, a.sel + (size_t)t * a.top, a.w + (size_t)t * a.top);
+// Router logits of 16 tokens and their largest scores.  8 waves share the columns; 64 experts at a time (the weights are the A operand: a
+// lane ends up with 4 consecutive experts of one token), partial sums meet in LDS.
+constexpr uint32_t kRouteTokens = 16, kRouteWaves = 8, kRouteTiles = 4;
+
+template <class T>
+__global__ void __launch_bounds__(512) moe_topk_kernel(const MoeRoute a) {
+  __shared__ float red[kRouteWaves][kRouteTiles * 16][kRouteTokens];
+  extern __shared__ __attribute__((aligned(16))) float z[];   // [tokens][ep]
+  const uint32_t tid = threadIdx.x, lane = tid & 63, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6)), r16 = lane & 15, g = lane >> 4;
+  const uint32_t t0 = blockIdx.x * kRouteTokens, ep = (a.experts + 3) & ~3u, m = t0 + r16 < a.M ? t0 + r16 : a.M - 1;
+  const T* x = reinterpret_cast<const T*>(a.x) + (size_t)m * a.ldx + g * Frag<T>::PER;
+  for (uint32_t e0 = 0; e0 < a.experts; e0 += kRouteTiles * 16) {
+    f32x4 acc[kRouteTiles];
+    const uint16_t* w[kRouteTiles];
+#pragma unroll
+    for (uint32_t n = 0; n < kRouteTiles; n++) {
+      acc[n] = (f32x4)(0.0f);
+      const uint32_t row = e0 + n * 16 + r16;
+      w[n] = a.router + (size_t)(row < a.experts ? row : a.experts - 1) * a.kp + g * Frag<T>::PER;
+    }
+#pragma unroll 4
+    for (uint32_t k = wave * Frag<T>::KU; k < a.kp; k += kRouteWaves * Frag<T>::KU) {
+      const typename Frag<T>::V xf = Frag<T>::load(x + k);
+#pragma unroll
+      for (uint32_t n = 0; n < kRouteTiles; n++) {
+        typename Frag<T>::V wf;
+        if constexpr (sizeof(T) == 2) {
+          wf = *reinterpret_cast<const bf16x8*>(w[n] + k);
+        } else {
+          const u32x2 h = *reinterpret_cast<const u32x2*>(w[n] + k);
+          wf.x = bf_lo(h.x); wf.y = bf_hi(h.x); wf.z = bf_lo(h.y); wf.w = bf_hi(h.y);
+        }
+        acc[n] = Frag<T>::mma(wf, xf, acc[n]);
+      }
+    }
+#pragma unroll
+    for (uint32_t n = 0; n < kRouteTiles; n++)
+#pragma unroll
+      for (uint32_t e = 0; e < 4; e++) red[wave][n * 16 + g * 4 + e][r16] = acc[n][e];
+    __syncthreads();
+    for (uint32_t i = tid; i < kRouteTiles * 16 * kRouteTokens; i += 512) {
+      const uint32_t e = i / kRouteTokens, t = i % kRouteTokens;
+      float v = 0.0f;
+#pragma unroll
+      for (uint32_t k = 0; k < kRouteWaves; k++) v += red[k][e][t];
+      if (e0 + e < ep) z[t * ep + e0 + e] = e0 + e < a.experts ? rank_key(v) : -INFINITY;
+    }
+    __syncthreads();
+  }
+  for (uint32_t i = tid; i < kRouteTokens * a.experts; i += 512) {
+    const uint32_t t = i / a.experts;
+    if (t0 + t < a.M) rank_expert(z + t * ep, a.experts, a.top, i % a.experts, a.sel + (size_t)(t0 + t) * a.top, a.w + (size_t)(t0 + t) * a.top);
+  }
 }
 
 // one workgroup: sizes of the groups, their first rows and row tiles, then a row for every pair
@@ -55,11 +102,20 @@ __global__ void __launch_bounds__(1024) moe_group_rows_kernel(const MoeRoute a) 
 
 uint32_t moe_max_tiles(uint32_t rows, uint32_t experts, uint32_t bm) { return rows / bm + (rows < experts ? rows : experts); }
 
-hipError_t moe_route_launch(const MoeRoute& a, hipStream_t st) {
+hipError_t moe_route_launch(const MoeRoute& a, bool f32, hipStream_t st) {
   static_assert(kMaxExperts == 1024, "one thread per expert");
-  if (a.M == 0 || a.top == 0 || a.top > a.experts || a.top > kMaxTop || a.experts > kMaxExperts || a.bm == 0 || a.tiles < moe_max_tiles(a.M * a.top, a.experts, a.bm))
+  static bool o32[64] = {}, o16[64] = {};
+  if (!a.x || !a.router || a.kp % 64 || a.ldx < a.kp || a.M == 0 || a.top == 0 || a.top > a.experts || a.top > kMaxTop || a.experts > kMaxExperts || a.bm == 0 || a.tiles < moe_max_tiles(a.M * a.top, a.experts, a.bm))
     return hipErrorInvalidValue;
-  hipLaunchKernelGGL(moe_topk_kernel, dim3(a.M), dim3(256), 0, st, a);
+  const size_t lds = (size_t)kRouteTokens * ((a.experts + 3) & ~3u) * 4;
+  const dim3 grid((a.M + kRouteTokens - 1) / kRouteTokens);
+  if (f32) {
+    if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&moe_topk_kernel<float>), 64 * 1024, o32); e != hipSuccess) return e;
+    hipLaunchKernelGGL(moe_topk_kernel<float>, grid, dim3(512), lds, st, a);
+  } else {
+    if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&moe_topk_kernel<__bf16>), 64 * 1024, o16); e != hipSuccess) return e;
+    hipLaunchKernelGGL(moe_topk_kernel<__bf16>, grid, dim3(512), lds, st, a);
+  }
   hipLaunchKernelGGL(moe_group_rows_kernel, dim3(1), dim3(1024), 0, st, a);
   return hipGetLastError();
 }

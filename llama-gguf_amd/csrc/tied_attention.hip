@@ -18,12 +18,20 @@ namespace lgh {
 
 constexpr float kTiedNeg = -1e30f, kTiedLog2e = 1.4426950408889634f;
 
-// cap * tanh(x / cap) in units of log2 (cap 0: x)
+// cap * tanh(x / cap) in units of log2, of u = x / cap (cap 0: x itself, of u = x); the queries carry the factor 1 / cap
+__device__ __forceinline__ float cap_unit(float cap) { return cap > 0.0f ? 1.0f / cap : 1.0f; }
 struct CapF {
-  float cap, inv, lim, out;   // 1 / cap, a quarter of cap, cap * log2(e)
-  __device__ __forceinline__ explicit CapF(float c) : cap(c), inv(c > 0.0f ? 1.0f / c : 0.0f), lim(c > 0.0f ? 0.25f * c : INFINITY), out(c > 0.0f ? c * kTiedLog2e : kTiedLog2e) {}
-  __device__ __forceinline__ float small(float x) const { return cap > 0.0f ? tanh_series(x * inv) * out : x * kTiedLog2e; }   // |x| < lim
-  __device__ __forceinline__ float any(float x) const { return cap > 0.0f ? tanh_f(x * inv) * out : x * kTiedLog2e; }
+  float lim, c0, c1, c2, c3, c4;   // the series of tanh (up to |u| < lim) times cap * log2(e)
+  __device__ __forceinline__ explicit CapF(float cap) {
+    const float o = cap > 0.0f ? cap * kTiedLog2e : kTiedLog2e, k = cap > 0.0f ? o : 0.0f;
+    lim = cap > 0.0f ? 0.25f : INFINITY;
+    c0 = o; c1 = k * (-1.0f / 3.0f); c2 = k * (2.0f / 15.0f); c3 = k * (-17.0f / 315.0f); c4 = k * (62.0f / 2835.0f);
+  }
+  __device__ __forceinline__ float small(float u, float add) const {   // |u| < lim
+    const float z = u * u;
+    return __builtin_fmaf(u, __builtin_fmaf(z, __builtin_fmaf(z, __builtin_fmaf(z, __builtin_fmaf(z, c4, c3), c2), c1), c0), add);
+  }
+  __device__ __forceinline__ float any(float u, float add) const { return fabsf(u) < lim ? small(u, add) : __builtin_fmaf(tanh_f(u), c0, add); }
 };
 __device__ __forceinline__ float tied_slope(uint32_t h, uint32_t heads) {   // in units of log2
   return exp2f(-8.0f * (float)(h + 1) / (float)heads) * kTiedLog2e;
@@ -64,13 +72,51 @@ template <class T, int PER> __device__ __forceinline__ void unpack_row(const u32
   }
 }
 
+// PER values of a head's row from d0 on, 0 behind its end; vec: rows start and end at multiples of 4
+template <int PER> __device__ __forceinline__ void row_chunk(const float* p, uint32_t d0, uint32_t dim, bool vec, float* o) {
+  if (vec) {
+#pragma unroll
+    for (int i = 0; i < PER; i += 4) {
+      const f32x4 v = *reinterpret_cast<const f32x4*>(p + (d0 + i < dim ? d0 + i : 0));
+#pragma unroll
+      for (int e = 0; e < 4; e++) o[i + e] = d0 + i < dim ? v[e] : 0.0f;
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < PER; e++) {
+      const float v = p[d0 + e < dim ? d0 + e : 0];
+      o[e] = d0 + e < dim ? v : 0.0f;
+    }
+  }
+}
+// a thread's share (of 256) of the sum of n squares
+__device__ __forceinline__ float squares(const float* p, uint32_t n) {
+  float s = 0.0f;
+  if (n & 3) {
+    for (uint32_t i = threadIdx.x; i < n; i += 256) s = __builtin_fmaf(p[i], p[i], s);
+    return s;
+  }
+  for (uint32_t i0 = threadIdx.x * 4; i0 < n; i0 += 4096) {
+    f32x4 v[4];
+#pragma unroll
+    for (uint32_t u = 0; u < 4; u++) v[u] = *reinterpret_cast<const f32x4*>(p + (i0 + u * 1024 < n ? i0 + u * 1024 : i0));
+#pragma unroll
+    for (uint32_t u = 0; u < 4; u++) {
+      const float keep = i0 + u * 1024 < n ? 1.0f : 0.0f;
+#pragma unroll
+      for (int e = 0; e < 4; e++) s = __builtin_fmaf(v[u][e] * keep, v[u][e], s);
+    }
+  }
+  return s;
+}
+
 // grid (splits, kv heads * chunks of HQ query heads, tokens)
 template <class T, uint32_t LPK, int HQ, bool OWN>
 __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const TiedBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits) {
   constexpr int PER = 16 / sizeof(T), NB = kTiedBatch;
   constexpr uint32_t GPW = 64 / LPK, HALF = GPW > 1 ? 32 : 64;      // key groups of a wave; lanes left after folding its halves
   __shared__ float red[16];
-  __shared__ float ml[2][4 * GPW][HQ];
+  __shared__ float ml[2][4][HQ];
   extern __shared__ __attribute__((aligned(16))) float accs[];      // [4 waves][HQ][HALF][PER]
   const uint32_t tid = threadIdx.x, lane = tid & 63, w = tid >> 6, grp = lane / LPK, sub = lane % LPK;
   const uint32_t gq = s.heads / s.kv_heads, chunks = (gq + HQ - 1) / HQ, g = blockIdx.y / chunks, h0 = g * gq + (blockIdx.y % chunks) * HQ;
@@ -100,30 +146,27 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
   fetch(rb);
   // this token's norms; its key row where this workgroup has it
   const bool owner = OWN && re == rounds;
-  float sq = 0.0f, sk = 0.0f;
-  for (uint32_t i = tid; i < s.heads * s.dim; i += 256) { const float v = cat[s.off_q + i]; sq = __builtin_fmaf(v, v, sq); }
-  if (owner)
-    for (uint32_t i = tid; i < s.kv_heads * s.dim; i += 256) { const float v = cat[s.off_k + i]; sk = __builtin_fmaf(v, v, sk); }
-  float q[HQ][PER], own[PER], own_inv = 0.0f, slope[HQ];
+  float q[HQ][PER], kn[PER], own[PER], own_inv = 0.0f, slope[HQ];
+  const bool vec = (s.dim & 3) == 0;
+  auto chunk = [&](const float* p, float* o) { row_chunk<PER>(p, d0, s.dim, vec, o); };   // (values past the head's end: 0)
+  chunk(b.kn + g * s.dim, kn);
 #pragma unroll
   for (int h = 0; h < HQ; h++) {
     const uint32_t hh = h0 + ((uint32_t)h < hn ? h : 0);
-    const float f = s.scale * b.temp[hh];
+    float w[PER];
+    chunk(cat + s.off_q + hh * s.dim, q[h]);
+    chunk(b.qn + hh * s.dim, w);
+    const float f = s.scale * cap_unit(s.cap) * b.temp[hh];
     slope[h] = tied_slope(hh, s.heads);
 #pragma unroll
-    for (int e = 0; e < PER; e++) {
-      const uint32_t d = d0 + e, dd = d < s.dim ? d : 0;
-      const float v = cat[s.off_q + hh * s.dim + dd] * b.qn[hh * s.dim + dd] * (b.kn[g * s.dim + dd] * f);
-      q[h][e] = d < s.dim ? v : 0.0f;
-    }
+    for (int e = 0; e < PER; e++) q[h][e] *= w[e] * (kn[e] * f);
   }
   if (owner) {
+    chunk(cat + s.off_k + g * s.dim, own);
 #pragma unroll
-    for (int e = 0; e < PER; e++) {
-      const uint32_t d = d0 + e;
-      own[e] = (float)to_act<T>(d < s.dim ? cat[s.off_k + g * s.dim + d] : 0.0f);
-    }
+    for (int e = 0; e < PER; e++) own[e] = (float)to_act<T>(own[e]);
   }
+  const float sq = squares(cat + s.off_q, s.heads * s.dim), sk = owner ? squares(cat + s.off_k, s.kv_heads * s.dim) : 0.0f;
   const float qinv = 1.0f / __builtin_sqrtf(block_sum(sq, red) / (float)(s.heads * s.dim) + s.eps);
   if (owner) {
     own_inv = 1.0f / __builtin_sqrtf(block_sum(sk, red) / (float)(s.kv_heads * s.dim) + s.eps);
@@ -173,8 +216,8 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
         float t = 0.0f;
 #pragma unroll
         for (int e = 0; e < PER; e++) t = __builtin_fmaf(q[h][e], kf[e], t);
-        t = cap.any(lanes_sum<LPK>(t) * inv);
-        sc[i][h] = ok ? __builtin_fmaf(-slope[h], dist, t) : kTiedNeg;
+        t = cap.any(lanes_sum<LPK>(t) * inv, -slope[h] * dist);
+        sc[i][h] = ok ? t : kTiedNeg;
       }
     }
 #pragma unroll
@@ -205,18 +248,23 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
     }
   }
   // the key groups' shares: maxima first, then the sums on a common scale
-  if (sub == 0) {
-#pragma unroll
-    for (int h = 0; h < HQ; h++) ml[0][w * GPW + grp][h] = m[h];
-  }
-  __syncthreads();
   float mx[HQ];
 #pragma unroll
   for (int h = 0; h < HQ; h++) {
-    mx[h] = ml[0][0][h];
-    for (uint32_t i = 1; i < 4 * GPW; i++) mx[h] = fmaxf(mx[h], ml[0][i][h]);
+    mx[h] = m[h];
+#pragma unroll
+    for (uint32_t d = LPK; d < 64; d *= 2) mx[h] = fmaxf(mx[h], __shfl_xor(mx[h], d, 64));
+    if (lane == 0) ml[0][w][h] = mx[h];
+  }
+  __syncthreads();
+#pragma unroll
+  for (int h = 0; h < HQ; h++) {
+    mx[h] = fmaxf(fmaxf(ml[0][0][h], ml[0][1][h]), fmaxf(ml[0][2][h], ml[0][3][h]));
     const float a = __builtin_amdgcn_exp2f(m[h] - mx[h]);
-    if (sub == 0) ml[1][w * GPW + grp][h] = l[h] * a;
+    float lw = l[h] * a;
+#pragma unroll
+    for (uint32_t d = LPK; d < 64; d *= 2) lw += __shfl_xor(lw, d, 64);
+    if (lane == 0) ml[1][w][h] = lw;
 #pragma unroll
     for (int e = 0; e < PER; e++) {
       float v = o[h][e] * a;
@@ -227,8 +275,7 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
   __syncthreads();
   const size_t rows = (size_t)M * s.heads, r0 = (size_t)sp * rows + (size_t)z * s.heads + h0;
   if (tid < hn) {
-    float lt = 0.0f;
-    for (uint32_t i = 0; i < 4 * GPW; i++) lt += ml[1][i][tid];
+    const float lt = (ml[1][0][tid] + ml[1][1][tid]) + (ml[1][2][tid] + ml[1][3][tid]);
     b.part_ml[(r0 + tid) * 2] = mx[0];
     for (uint32_t h = 1; h < (uint32_t)HQ; h++)
       if (tid == h) b.part_ml[(r0 + tid) * 2] = mx[h];
@@ -237,8 +284,10 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
   for (uint32_t i = tid; i < hn * s.dim; i += 256) {
     const uint32_t h = i / s.dim, d = i % s.dim, ln = d / PER, e = d % PER;
     float v = 0.0f;
+#pragma unroll
     for (uint32_t k = 0; k < 4; k++)
-      for (uint32_t x = ln; x < HALF; x += LPK) v += accs[((k * HQ + h) * HALF + x) * PER + e];
+#pragma unroll
+      for (uint32_t x = 0; x < HALF; x += LPK) v += accs[((k * HQ + h) * HALF + x + ln) * PER + e];
     b.part_acc[(r0 + h) * s.dim + d] = v;
   }
 }
@@ -296,9 +345,10 @@ __global__ void __launch_bounds__(256) tied_merge_kernel(const TiedShape s, cons
   float mi[2], li[2];
 #pragma unroll
   for (uint32_t k = 0; k < 2; k++) {
-    const uint32_t i = lane + k * 64, ic = i < act ? i : act - 1;
-    mi[k] = b.part_ml[(ic * rows + r) * 2];
-    li[k] = b.part_ml[(ic * rows + r) * 2 + 1] * (i < act ? 1.0f : 0.0f);
+    const uint32_t i = lane + k * 64, ic = i < n_splits ? i : n_splits - 1;   // (what the inactive shares hold is not used: the loads need no position)
+    const f32x2 v = *reinterpret_cast<const f32x2*>(b.part_ml + (ic * rows + r) * 2);
+    mi[k] = i < act ? v.x : kTiedNeg;
+    li[k] = i < act ? v.y : 0.0f;
   }
   const float sink = b.sink[h] * kTiedLog2e;
   // columns x groups of splits; the first partial sums are requested before the weights are known
@@ -309,7 +359,7 @@ __global__ void __launch_bounds__(256) tied_merge_kernel(const TiedShape s, cons
 #pragma unroll
   for (int i = 0; i < F; i++) {
     const uint32_t k = grp + i * groups;
-    first[i] = b.part_acc[((k < act ? k : act - 1) * rows + r) * s.dim + c0];
+    first[i] = b.part_acc[((k < n_splits ? k : n_splits - 1) * rows + r) * s.dim + c0];
   }
   if (tid < 64) {
     const float mm = fmaxf(wave_max(fmaxf(mi[0], mi[1])), sink);
@@ -323,7 +373,7 @@ __global__ void __launch_bounds__(256) tied_merge_kernel(const TiedShape s, cons
 #pragma unroll
     for (int i = 0; i < F; i++) {
       const uint32_t k = grp + i * groups;
-      v = __builtin_fmaf(k < act ? wgt[k] : 0.0f, first[i], v);
+      if (k < act) v = __builtin_fmaf(wgt[k], first[i], v);
     }
     for (uint32_t k = grp + F * groups; k < act; k += groups) v = __builtin_fmaf(wgt[k], b.part_acc[(k * rows + r) * s.dim + c0], v);
   }
@@ -344,35 +394,50 @@ hipError_t tied_merge_launch(const TiedShape& s, const TiedBufs& b, const int* p
   return hipGetLastError();
 }
 
-// a block's cache rows, key factors and queries; grid (tokens)
-template <class T>
+// a block's cache rows, key factors and queries; grid (tokens).  V: 4 where heads have a multiple of 4 values
+template <class T, int V>
 __global__ void __launch_bounds__(256) tied_prep_kernel(const TiedShape s, const TiedBufs b, uint32_t pos0) {
   __shared__ float red[16];
   const uint32_t t = blockIdx.x, pos = pos0 + t, tid = threadIdx.x, nq = s.heads * s.dim, nk = s.kv_heads * s.dim, gq = s.heads / s.kv_heads;
   const float* cat = b.cat + (size_t)t * s.ldcat;
-  float sq = 0.0f, sk = 0.0f;
-  for (uint32_t i = tid; i < nq; i += 256) { const float v = cat[s.off_q + i]; sq = __builtin_fmaf(v, v, sq); }
-  for (uint32_t i = tid; i < nk; i += 256) {
-    const float v = cat[s.off_k + i];
-    sk = __builtin_fmaf(v, v, sk);
-    reinterpret_cast<T*>(b.cache)[((size_t)(i / s.dim) * s.rows + pos) * s.dp + i % s.dim] = to_act<T>(v);
-  }
-  const float qinv = 1.0f / __builtin_sqrtf(block_sum(sq, red) / (float)nq + s.eps) * s.scale;
+  struct Val { float v[V]; };
+  auto load = [](const float* p) {
+    Val r;
+    if constexpr (V == 4) { const f32x4 q = *reinterpret_cast<const f32x4*>(p); r.v[0] = q.x; r.v[1] = q.y; r.v[2] = q.z; r.v[3] = q.w; }
+    else r.v[0] = p[0];
+    return r;
+  };
+  auto store = [](T* p, const Val& a) {
+    T o[V];
+#pragma unroll
+    for (int i = 0; i < V; i++) o[i] = to_act<T>(a.v[i]);
+    __builtin_memcpy(__builtin_assume_aligned(p, sizeof(o)), o, sizeof(o));
+  };
+  for (uint32_t i = tid * V; i < nk; i += 256 * V)
+    store(reinterpret_cast<T*>(b.cache) + ((size_t)(i / s.dim) * s.rows + pos) * s.dp + i % s.dim, load(cat + s.off_k + i));
+  const float sk = squares(cat + s.off_k, nk), sq = squares(cat + s.off_q, nq);
   const float kinv = 1.0f / __builtin_sqrtf(block_sum(sk, red) / (float)nk + s.eps);
   if (tid == 0) b.kinv[pos] = kinv;
   if (!b.q) return;
-  T* q = reinterpret_cast<T*>(b.q);
-  for (uint32_t i = tid; i < s.heads * s.dp; i += 256) {
+  const float qinv = 1.0f / __builtin_sqrtf(block_sum(sq, red) / (float)nq + s.eps) * s.scale * cap_unit(s.cap);
+  for (uint32_t i = tid * V; i < s.heads * s.dp; i += 256 * V) {
     const uint32_t h = i / s.dp, d = i % s.dp, dd = d < s.dim ? d : 0;
-    const float v = cat[s.off_q + h * s.dim + dd] * b.qn[h * s.dim + dd] * (b.kn[h / gq * s.dim + dd] * (qinv * b.temp[h]));
-    q[((size_t)h * b.Mcap + t) * s.dp + d] = to_act<T>(d < s.dim ? v : 0.0f);
+    const Val q = load(cat + s.off_q + h * s.dim + dd), qn = load(b.qn + h * s.dim + dd), kn = load(b.kn + h / gq * s.dim + dd);
+    const float f = d < s.dim ? qinv * b.temp[h] : 0.0f;
+    Val o;
+#pragma unroll
+    for (int e = 0; e < V; e++) o.v[e] = q.v[e] * qn.v[e] * (kn.v[e] * f);
+    store(reinterpret_cast<T*>(b.q) + ((size_t)h * b.Mcap + t) * s.dp + d, o);
   }
 }
 
 hipError_t tied_prep_launch(const TiedShape& s, const TiedBufs& b, uint32_t pos0, uint32_t M, bool f32, hipStream_t st) {
   if (!tied_ok(s) || M == 0 || (b.q && M > b.Mcap) || pos0 + M > s.rows) return hipErrorInvalidValue;
-  if (f32) hipLaunchKernelGGL(tied_prep_kernel<float>, dim3(M), dim3(256), 0, st, s, b, pos0);
-  else hipLaunchKernelGGL(tied_prep_kernel<__bf16>, dim3(M), dim3(256), 0, st, s, b, pos0);
+  const bool v4 = s.dim % 4 == 0;
+  if (f32 && v4) hipLaunchKernelGGL((tied_prep_kernel<float, 4>), dim3(M), dim3(256), 0, st, s, b, pos0);
+  else if (f32) hipLaunchKernelGGL((tied_prep_kernel<float, 1>), dim3(M), dim3(256), 0, st, s, b, pos0);
+  else if (v4) hipLaunchKernelGGL((tied_prep_kernel<__bf16, 4>), dim3(M), dim3(256), 0, st, s, b, pos0);
+  else hipLaunchKernelGGL((tied_prep_kernel<__bf16, 1>), dim3(M), dim3(256), 0, st, s, b, pos0);
   return hipGetLastError();
 }
 
@@ -383,13 +448,14 @@ hipError_t tied_prep_launch(const TiedShape& s, const TiedBufs& b, uint32_t pos0
 // ------------------------------------------------------------------------------------------------
 template <class T> constexpr int tied_kt() { return sizeof(T) == 2 ? 64 : 32; }
 template <class T, int DQ> constexpr size_t tied_lds() { return 2 * (size_t)tied_kt<T>() * DQ * sizeof(T); }
+template <class T, int DQ> constexpr int tied_qt() { return sizeof(T) == 2 && DQ <= 192 ? 2 : 1; }   // 16-query tiles per wave
 template <class T, int DQ> constexpr int tied_wgs() { return DQ <= 128 ? 2 : 1; }
 
 template <class T, int DQ>
 __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(const TiedShape s, const TiedBufs b, uint32_t pos0, uint32_t M, uint32_t nqb, T* __restrict__ out,
                                                                               uint32_t ldo) {
   constexpr bool BF = sizeof(T) == 2;
-  constexpr int KT = tied_kt<T>(), QT = BF ? 2 : 1, NK = KT / 16, NU = DQ / Frag<T>::KU, ND = DQ / 16;
+  constexpr int KT = tied_kt<T>(), QT = tied_qt<T, DQ>(), NK = KT / 16, NU = DQ / Frag<T>::KU, ND = DQ / 16;
   constexpr uint32_t XC = DQ * sizeof(T) / 16, kBuf = KT * XC * 16;
   extern __shared__ __attribute__((aligned(16))) uint8_t smem[];
   const uint32_t lane = threadIdx.x & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)), r16 = lane & 15, g = lane >> 4;
@@ -434,6 +500,11 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
   }
   const CapF cap(s.cap);
   const float slope = tied_slope(h, s.heads);
+  f32x4 bias[NK];                                               // slope * (place in the tile) of this lane's keys
+#pragma unroll
+  for (int n = 0; n < NK; n++)
+#pragma unroll
+    for (int e = 0; e < 4; e++) bias[n][e] = slope * (float)(n * 16 + g * 4 + e);
   const uint32_t iw0 = pos0 + qw, iw1 = iw0 + 16 * QT - 1;      // this wave's queries
   wait_vm(0);
   __syncthreads();
@@ -475,18 +546,26 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
             sa[n][t][e] *= kc[n][e];
             top = fmaxf(top, fabsf(sa[n][t][e]));
           }
-      const bool large = __any(!(top < cap.lim));
+      if (__any(!(top < cap.lim))) {
+        asm volatile("");              // (kept a branch: scores come near the cap now and then)
+#pragma unroll
+        for (int t = 0; t < QT; t++)
+#pragma unroll
+          for (int n = 0; n < NK; n++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) sa[n][t][e] = cap.any(sa[n][t][e], bias[n][e]);
+      } else {
+#pragma unroll
+        for (int t = 0; t < QT; t++)
+#pragma unroll
+          for (int n = 0; n < NK; n++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) sa[n][t][e] = cap.small(sa[n][t][e], bias[n][e]);
+      }
 #pragma unroll
       for (int t = 0; t < QT; t++) {
         const uint32_t i = iw0 + t * 16 + r16;
-        const float off = slope * ((float)(int)(k0 + g * 4 - i));    // - slope * (i - j) of the lane's first key
-#pragma unroll
-        for (int n = 0; n < NK; n++)
-#pragma unroll
-          for (int e = 0; e < 4; e++) {
-            const float x = sa[n][t][e];
-            sa[n][t][e] = __builtin_fmaf(slope, (float)(n * 16 + e), off) + (large ? cap.any(x) : cap.small(x));
-          }
+        const float off = slope * (float)(int)(k0 - i);      // what the tile's place adds to every score of this lane's query
         if (!full) {
           asm volatile("");              // (kept a branch: most tiles have no masks to apply)
 #pragma unroll
@@ -497,13 +576,14 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
               sa[n][t][e] = j <= i && (i - j < s.window || j < s.keep) ? sa[n][t][e] : kTiedNeg;
             }
         }
-        float m1 = mx[t];
+        float m1 = kTiedNeg;
 #pragma unroll
         for (int n = 0; n < NK; n++)
 #pragma unroll
           for (int e = 0; e < 4; e++) m1 = fmaxf(m1, sa[n][t][e]);
         m1 = fmaxf(m1, __shfl_xor(m1, 16, 64));
-        m1 = fmaxf(m1, __shfl_xor(m1, 32, 64));
+        m1 = fmaxf(fmaxf(m1, __shfl_xor(m1, 32, 64)) + off, mx[t]);
+        const float rel = m1 - off;
         // (a query that has seen nothing yet weighs masked keys; the factor of its first visible tile takes that to 0)
         const float a = __builtin_amdgcn_exp2f(mx[t] - m1);
         float sum = 0.0f;
@@ -511,7 +591,7 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
         for (int n = 0; n < NK; n++)
 #pragma unroll
           for (int e = 0; e < 4; e++) {
-            const float p = __builtin_amdgcn_exp2f(sa[n][t][e] - m1);
+            const float p = __builtin_amdgcn_exp2f(sa[n][t][e] - rel);
             sa[n][t][e] = p;
             sum += p;
           }
@@ -577,7 +657,7 @@ static hipError_t tied_flash_go(const TiedShape& s, const TiedBufs& b, uint32_t 
   constexpr size_t lds = tied_lds<T, DQ>();
   static_assert(lds <= 160 * 1024, "two tiles fit LDS");
   if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&tied_flash_kernel<T, DQ>), (int)lds, opted); e != hipSuccess) return e;
-  const uint32_t QB = sizeof(T) == 2 ? 128 : 64, nqb = (M + QB - 1) / QB;
+  const uint32_t QB = 64 * tied_qt<T, DQ>(), nqb = (M + QB - 1) / QB;
   hipLaunchKernelGGL((tied_flash_kernel<T, DQ>), dim3(nqb * s.heads), dim3(256), lds, st, s, b, pos0, M, nqb, (T*)out, ldo);
   return hipGetLastError();
 }

@@ -131,7 +131,7 @@ def test_a_key_just_inside_and_just_outside(pkg, gpu, dtype, window, keep, n):
     W["embed"][[KA, KB], 2] = 3.0
     W["embed"][KA, 1], W["embed"][KB, 1] = 3.0, -3.0
     W["l0.norm1"][:3], W["l0.norm1.b"][:3], W["l0.canon1"][:3] = 1.0, 0.0, 0.0
-    W["l0.norm1.b"][:] *= 0.1                       # (what all tokens share would drown the question)
+    W["l0.norm1.b"][:] = lc.bf16(W["l0.norm1.b"] * 0.1)   # (what all tokens share would drown the question)
     W["l0.mix.q"][:, 0] = 0.0
     W["l0.mix.q"][16, :] = 0.0
     W["l0.mix.q"][16, 0] = 8.0                      # head 1 (the one that minds distance least) asks in its first value
