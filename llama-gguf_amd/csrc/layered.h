@@ -195,6 +195,7 @@ struct TiedBufs {
   float *part_ml, *part_acc;           // [split][M * heads][2], [split][M * heads][dim]
 };
 constexpr uint32_t kTiedMaxSplits = 128, kTiedShort = 16, kTiedMaxDim = 256;   // portions up to kTiedShort tokens take the decode kernel
+uint32_t tied_keys_per_round(const TiedShape& s, bool f32);   // keys of a workgroup per round of the decode kernel
 uint32_t tied_splits(const TiedShape& s, uint32_t max_seq, uint32_t M, bool f32, uint32_t forced);
 // one token (own = true: its key is taken from cat and written to the cache) or M tokens whose keys are in the cache
 hipError_t tied_attn_launch(const TiedShape& s, const TiedBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, bool own, uint32_t n_splits, bool f32, hipStream_t st);

@@ -210,22 +210,33 @@ __global__ void __launch_bounds__(256) dyt_block_kernel(const DytBlock a) {
   float pal = 0.0f, nal = 0.0f;
   if (upd) { pw = load_vec<V>(a.post.w + c); pb = load_vec<V>(a.post.b + c); pal = *a.post.alpha; }
   if (nxt) { nw = load_vec<V>(a.next.w + c); nb = load_vec<V>(a.next.b + c); nal = *a.next.alpha; }
-  auto fetch_x = [&](int t) { return load_vec<V>(a.x + (size_t)(t < 0 ? 0 : t) * W + c); };
-  auto fetch_y = [&](int t) {
-    VecF<V> y;
+  // a group of tokens requested while the one before it is worked on: the stream, the sublayer's output, its first two experts' rows
+  constexpr int G = 4, P = 2;
+  struct Group { VecF<V> x[G], y[G], p[G][P]; };
+  const int n_pairs = upd && a.pairs ? (int)a.top : 0;
+  auto request = [&](int t, Group& o) {
 #pragma unroll
-    for (int i = 0; i < V; i++) y.v[i] = 0.0f;
-    if (upd && a.y) y = load_vec<V>(a.y + (size_t)(t < 0 ? 0 : t) * a.ldy + c);
-    if (upd && a.pairs && t >= 0) y = add_pairs<V>(y, a.pairs, a.ldp, a.slot + (size_t)t * a.top, a.top, c);
-    return y;
+    for (int g = 0; g < G; g++) {
+      const size_t tc = (size_t)(t + g < 0 ? 0 : t + g < t1 ? t + g : t1 - 1);
+      o.x[g] = load_vec<V>(a.x + tc * W + c);
+      if (upd && a.y) o.y[g] = load_vec<V>(a.y + tc * a.ldy + c);
+#pragma unroll
+      for (int k = 0; k < P; k++)
+        if (k < n_pairs) o.p[g][k] = load_vec<V>(a.pairs + (size_t)a.slot[tc * a.top + k] * a.ldp + c);
+    }
   };
   const int first = nxt ? t0 - back : t0;
-  VecF<V> xn = fetch_x(first), yn = fetch_y(first);
+  Group nx;
+  request(first, nx);
   int at = 0;                                       // ring row of token t
-  for (int t = first; t < t1; t++) {
-    VecF<V> v = xn, h;
-    const VecF<V> y = yn;
-    if (t + 1 < t1) { xn = fetch_x(t + 1); yn = fetch_y(t + 1); }
+  for (int tg = first; tg < t1; tg += G) {
+   const Group cu = nx;
+   if (tg + G < t1) request(tg + G, nx);
+#pragma unroll
+   for (int g = 0; g < G; g++) {
+    const int t = tg + g;
+    if (t >= t1) break;
+    VecF<V> v = cu.x[g], h, y;
     if (t < 0) {                                    // before the block
       const int p = (int)a.pos0 + t;
 #pragma unroll
@@ -233,6 +244,14 @@ __global__ void __launch_bounds__(256) dyt_block_kernel(const DytBlock a) {
       if (p >= 0) h = load_vec<V>(a.conv.hist + (size_t)(p % back) * W + c);
     } else {
       if (upd) {
+#pragma unroll
+        for (int i = 0; i < V; i++) y.v[i] = a.y ? cu.y[g].v[i] : 0.0f;
+#pragma unroll
+        for (int k = 0; k < P; k++)
+          if (k < n_pairs)
+#pragma unroll
+            for (int i = 0; i < V; i++) y.v[i] += cu.p[g][k].v[i];
+        if (n_pairs > P) y = add_pairs<V>(y, a.pairs, a.ldp, a.slot + (size_t)t * a.top + P, a.top - P, c);
 #pragma unroll
         for (int i = 0; i < V; i++) v.v[i] = __builtin_fmaf(a.mult, dyt_f(y.v[i], pal, pw.v[i], pb.v[i]), v.v[i]);
         if (t >= t0 && live) store_vec<V>(a.xout + (size_t)t * W + c, v);
@@ -261,6 +280,7 @@ __global__ void __launch_bounds__(256) dyt_block_kernel(const DytBlock a) {
       }
     }
     at = at + 1 < taps ? at + 1 : 0;
+   }
   }
 }
 

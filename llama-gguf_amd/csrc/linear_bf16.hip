@@ -240,8 +240,7 @@ static hipError_t lin_mv_run(const LinMv& a, hipStream_t st) {
   const uint32_t groups = SRC == LS_TWO ? g1 + (a.n2 + kMvR - 1) / kMvR : SRC == LS_EXPERTS ? g1 * a.top : g1;
   uint32_t ks = 1;   // waves per team: enough teams for the groups of a CU, and at least a full pass of columns per wave
   while (ks < 8 && (uint64_t)groups * ks * 2 <= kNumCU * 16 && a.kp >= 1024 * ks) ks *= 2;
-  const uint32_t teams = 16 / ks, want = (groups + teams - 1) / teams;
-  hipLaunchKernelGGL((lin_mv_kernel<PRO, SRC, POST>), dim3(want < kNumCU ? want : kNumCU), dim3(kMvThreads), (size_t)a.kp * 4, st, a, groups, ks, g1);
+  hipLaunchKernelGGL((lin_mv_kernel<PRO, SRC, POST>), dim3(groups < kNumCU ? groups : kNumCU), dim3(kMvThreads), (size_t)a.kp * 4, st, a, groups, ks, g1);
   return hipGetLastError();
 }
 template <int PRO, int SRC>

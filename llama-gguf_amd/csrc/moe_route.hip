@@ -5,11 +5,11 @@
 
 namespace lgh {
 
-// Router logits of 16 tokens and their largest scores.  8 waves share the columns; 64 experts at a time (the weights are the A operand: a
+// Router logits of 16 tokens and their largest scores.  8 waves share the columns; kRouteTiles * 16 experts at a time (the weights are the A operand: a
 // lane ends up with 4 consecutive experts of one token), partial sums meet in LDS.
-constexpr uint32_t kRouteTokens = 16, kRouteWaves = 8, kRouteTiles = 4;
+constexpr uint32_t kRouteTokens = 16, kRouteWaves = 8;
 
-template <class T>
+template <class T, uint32_t kRouteTiles>
 __global__ void __launch_bounds__(512) moe_topk_kernel(const MoeRoute a) {
   __shared__ float red[kRouteWaves][kRouteTiles * 16][kRouteTokens];
   extern __shared__ __attribute__((aligned(16))) float z[];   // [tokens][ep]
@@ -25,7 +25,7 @@ __global__ void __launch_bounds__(512) moe_topk_kernel(const MoeRoute a) {
       const uint32_t row = e0 + n * 16 + r16;
       w[n] = a.router + (size_t)(row < a.experts ? row : a.experts - 1) * a.kp + g * Frag<T>::PER;
     }
-#pragma unroll 4
+#pragma unroll (kRouteTiles == 1 ? 8 : 4)
     for (uint32_t k = wave * Frag<T>::KU; k < a.kp; k += kRouteWaves * Frag<T>::KU) {
       const typename Frag<T>::V xf = Frag<T>::load(x + k);
 #pragma unroll
@@ -109,12 +109,15 @@ hipError_t moe_route_launch(const MoeRoute& a, bool f32, hipStream_t st) {
     return hipErrorInvalidValue;
   const size_t lds = (size_t)kRouteTokens * ((a.experts + 3) & ~3u) * 4;
   const dim3 grid((a.M + kRouteTokens - 1) / kRouteTokens);
-  if (f32) {
-    if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&moe_topk_kernel<float>), 64 * 1024, o32); e != hipSuccess) return e;
-    hipLaunchKernelGGL(moe_topk_kernel<float>, grid, dim3(512), lds, st, a);
+  if (a.experts <= 16) {
+    if (f32) hipLaunchKernelGGL((moe_topk_kernel<float, 1>), grid, dim3(512), lds, st, a);
+    else hipLaunchKernelGGL((moe_topk_kernel<__bf16, 1>), grid, dim3(512), lds, st, a);
+  } else if (f32) {
+    if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&moe_topk_kernel<float, 4>), 64 * 1024, o32); e != hipSuccess) return e;
+    hipLaunchKernelGGL((moe_topk_kernel<float, 4>), grid, dim3(512), lds, st, a);
   } else {
-    if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&moe_topk_kernel<__bf16>), 64 * 1024, o16); e != hipSuccess) return e;
-    hipLaunchKernelGGL(moe_topk_kernel<__bf16>, grid, dim3(512), lds, st, a);
+    if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&moe_topk_kernel<__bf16, 4>), 64 * 1024, o16); e != hipSuccess) return e;
+    hipLaunchKernelGGL((moe_topk_kernel<__bf16, 4>), grid, dim3(512), lds, st, a);
   }
   hipLaunchKernelGGL(moe_group_rows_kernel, dim3(1), dim3(1024), 0, st, a);
   return hipGetLastError();

@@ -89,23 +89,28 @@ template <int PER> __device__ __forceinline__ void row_chunk(const float* p, uin
     }
   }
 }
-// a thread's share (of 256) of the sum of n squares
-__device__ __forceinline__ float squares(const float* p, uint32_t n) {
-  float s = 0.0f;
-  if (n & 3) {
-    for (uint32_t i = threadIdx.x; i < n; i += 256) s = __builtin_fmaf(p[i], p[i], s);
-    return s;
+// a thread's share (of 256) of the sum of n squares; its first 16 values requested by `squares_fetch`
+struct Squares { f32x4 v[4]; };
+__device__ __forceinline__ void squares_fetch(const float* p, uint32_t n, uint32_t i0, Squares& o) {
+#pragma unroll
+  for (uint32_t u = 0; u < 4; u++) {
+    const uint32_t i = i0 + u * 1024;
+    if ((n & 3) == 0) { o.v[u] = *reinterpret_cast<const f32x4*>(p + (i < n ? i : 0)); continue; }
+#pragma unroll
+    for (uint32_t e = 0; e < 4; e++) o.v[u][e] = p[i + e < n ? i + e : 0];
   }
+}
+__device__ __forceinline__ float squares(const float* p, uint32_t n, Squares in) {
+  float s = 0.0f;
   for (uint32_t i0 = threadIdx.x * 4; i0 < n; i0 += 4096) {
-    f32x4 v[4];
+    if (i0 >= 4096) squares_fetch(p, n, i0, in);
 #pragma unroll
-    for (uint32_t u = 0; u < 4; u++) v[u] = *reinterpret_cast<const f32x4*>(p + (i0 + u * 1024 < n ? i0 + u * 1024 : i0));
+    for (uint32_t u = 0; u < 4; u++)
 #pragma unroll
-    for (uint32_t u = 0; u < 4; u++) {
-      const float keep = i0 + u * 1024 < n ? 1.0f : 0.0f;
-#pragma unroll
-      for (int e = 0; e < 4; e++) s = __builtin_fmaf(v[u][e] * keep, v[u][e], s);
-    }
+      for (uint32_t e = 0; e < 4; e++) {
+        const float x = i0 + u * 1024 + e < n ? in.v[u][e] : 0.0f;
+        s = __builtin_fmaf(x, x, s);
+      }
   }
   return s;
 }
@@ -146,6 +151,9 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
   fetch(rb);
   // this token's norms; its key row where this workgroup has it
   const bool owner = OWN && re == rounds;
+  Squares vq, vk;
+  squares_fetch(cat + s.off_q, s.heads * s.dim, tid * 4, vq);
+  if (owner) squares_fetch(cat + s.off_k, s.kv_heads * s.dim, tid * 4, vk);
   float q[HQ][PER], kn[PER], own[PER], own_inv = 0.0f, slope[HQ];
   const bool vec = (s.dim & 3) == 0;
   auto chunk = [&](const float* p, float* o) { row_chunk<PER>(p, d0, s.dim, vec, o); };   // (values past the head's end: 0)
@@ -166,7 +174,7 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
 #pragma unroll
     for (int e = 0; e < PER; e++) own[e] = (float)to_act<T>(own[e]);
   }
-  const float sq = squares(cat + s.off_q, s.heads * s.dim), sk = owner ? squares(cat + s.off_k, s.kv_heads * s.dim) : 0.0f;
+  const float sq = squares(cat + s.off_q, s.heads * s.dim, vq), sk = owner ? squares(cat + s.off_k, s.kv_heads * s.dim, vk) : 0.0f;
   const float qinv = 1.0f / __builtin_sqrtf(block_sum(sq, red) / (float)(s.heads * s.dim) + s.eps);
   if (owner) {
     own_inv = 1.0f / __builtin_sqrtf(block_sum(sk, red) / (float)(s.kv_heads * s.dim) + s.eps);
@@ -192,7 +200,7 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
   }
   for (uint32_t r = rb; r < re; r++) {
     u32x4 cur[NB];
-    float ci[NB], sc[NB][HQ];
+    float ci[NB], sc[NB][HQ], bias[NB], top = 0.0f;
     uint32_t cp[NB];
 #pragma unroll
     for (int i = 0; i < NB; i++) { cur[i] = kraw[i]; ci[i] = kin[i]; cp[i] = kp[i]; }
@@ -216,10 +224,27 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
         float t = 0.0f;
 #pragma unroll
         for (int e = 0; e < PER; e++) t = __builtin_fmaf(q[h][e], kf[e], t);
-        t = cap.any(lanes_sum<LPK>(t) * inv, -slope[h] * dist);
-        sc[i][h] = ok ? t : kTiedNeg;
+        sc[i][h] = lanes_sum<LPK>(t) * inv;
+        top = fmaxf(top, fabsf(sc[i][h]));
       }
+      bias[i] = dist;
     }
+    if (__any(!(top < cap.lim))) {
+      asm volatile("");                        // (kept a branch: scores come near the cap now and then)
+#pragma unroll
+      for (int i = 0; i < NB; i++)
+#pragma unroll
+        for (int h = 0; h < HQ; h++) sc[i][h] = cap.any(sc[i][h], -slope[h] * bias[i]);
+    } else {
+#pragma unroll
+      for (int i = 0; i < NB; i++)
+#pragma unroll
+        for (int h = 0; h < HQ; h++) sc[i][h] = cap.small(sc[i][h], -slope[h] * bias[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < NB; i++)
+#pragma unroll
+      for (int h = 0; h < HQ; h++) sc[i][h] = cp[i] != 0xFFFFFFFFu ? sc[i][h] : kTiedNeg;
 #pragma unroll
     for (int h = 0; h < HQ; h++) {
       float m1 = m[h];
@@ -266,10 +291,14 @@ __global__ void __launch_bounds__(256) tied_attn_kernel(const TiedShape s, const
     for (uint32_t d = LPK; d < 64; d *= 2) lw += __shfl_xor(lw, d, 64);
     if (lane == 0) ml[1][w][h] = lw;
 #pragma unroll
-    for (int e = 0; e < PER; e++) {
-      float v = o[h][e] * a;
-      if constexpr (GPW > 1) v += __shfl_xor(v, 32, 64);
-      if (lane < HALF) accs[((w * HQ + h) * HALF + lane) * PER + e] = v;
+    for (int e = 0; e < PER; e += 4) {
+      f32x4 v;
+#pragma unroll
+      for (int k = 0; k < 4; k++) {
+        v[k] = o[h][e + k] * a;
+        if constexpr (GPW > 1) v[k] += __shfl_xor(v[k], 32, 64);
+      }
+      if (lane < HALF) *reinterpret_cast<f32x4*>(accs + ((w * HQ + h) * HALF + lane) * PER + e) = v;
     }
   }
   __syncthreads();
@@ -323,74 +352,95 @@ hipError_t tied_attn_launch(const TiedShape& s, const TiedBufs& b, const int* po
   return hipErrorInvalidValue;
 }
 
+uint32_t tied_keys_per_round(const TiedShape& s, bool f32) { return tied_round(tied_lanes(s.dp, f32 ? 4 : 2)); }
+
 // shares of the keys that fill the chip; not more than there are rounds of keys
 uint32_t tied_splits(const TiedShape& s, uint32_t max_seq, uint32_t M, bool f32, uint32_t forced) {
   const uint32_t gq = s.heads / s.kv_heads, hq = gq <= 2 ? gq : 4, wgs = s.kv_heads * ((gq + hq - 1) / hq) * M;
-  const uint32_t kr = tied_round(tied_lanes(s.dp, f32 ? 4 : 2)), rounds = (tied_seen(s, max_seq - 1).total + kr - 1) / kr;
+  const uint32_t kr = tied_keys_per_round(s, f32), rounds = (tied_seen(s, max_seq - 1).total + kr - 1) / kr;
   const uint32_t want = forced ? forced : std::max(1u, 512 / wgs);
   return std::min(std::min(want, kTiedMaxSplits), std::max(rounds, 1u));
 }
 
-// the shares of the keys put together, the sink's term; grid (heads, tokens)
-template <class O>
+// the shares of the keys put together, the sink's term; grid (heads, tokens).  V: 4 where heads have a multiple of 4 values
+template <class O, int V>
 __global__ void __launch_bounds__(256) tied_merge_kernel(const TiedShape s, const TiedBufs b, const int* __restrict__ pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits,
                                                          uint32_t kr, O* __restrict__ out, uint32_t ldo) {
-  __shared__ float part[256];
+  struct Val { float v[V]; };
+  __shared__ Val part[256];
   __shared__ float wgt[kTiedMaxSplits];
   static_assert(kTiedMaxSplits == 128, "two splits per lane");
   const uint32_t tid = threadIdx.x, lane = tid & 63, h = blockIdx.x, t = blockIdx.y;
   const uint32_t pos = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + t;
   const uint32_t rounds = (tied_seen(s, pos).total + kr - 1) / kr, per = (rounds + n_splits - 1) / n_splits, act = (rounds + per - 1) / per;
   const size_t rows = (size_t)M * s.heads, r = (size_t)t * s.heads + h;
-  float mi[2], li[2];
+  // (what the inactive shares hold is not used: the loads need no position)
+  f32x2 ml[2];
 #pragma unroll
   for (uint32_t k = 0; k < 2; k++) {
-    const uint32_t i = lane + k * 64, ic = i < n_splits ? i : n_splits - 1;   // (what the inactive shares hold is not used: the loads need no position)
-    const f32x2 v = *reinterpret_cast<const f32x2*>(b.part_ml + (ic * rows + r) * 2);
-    mi[k] = i < act ? v.x : kTiedNeg;
-    li[k] = i < act ? v.y : 0.0f;
+    const uint32_t i = lane + k * 64;
+    ml[k] = *reinterpret_cast<const f32x2*>(b.part_ml + ((i < n_splits ? i : n_splits - 1) * rows + r) * 2);
   }
   const float sink = b.sink[h] * kTiedLog2e;
   // columns x groups of splits; the first partial sums are requested before the weights are known
-  const uint32_t cols = s.dim < 256 ? s.dim : 256, groups = 256 / cols, grp = tid / cols;
+  const uint32_t cols = (s.dim + V - 1) / V, groups = 256 / cols, grp = tid / cols, c0 = tid % cols * V;
+  auto load = [&](uint32_t k) {
+    Val x;
+    const float* p = b.part_acc + (k * rows + r) * s.dim + c0;
+    if constexpr (V == 4) { const f32x4 q = *reinterpret_cast<const f32x4*>(p); x.v[0] = q.x; x.v[1] = q.y; x.v[2] = q.z; x.v[3] = q.w; }
+    else x.v[0] = p[0];
+    return x;
+  };
   constexpr int F = 8;
-  float first[F];
-  const uint32_t c0 = tid % cols;
+  Val first[F], v;
 #pragma unroll
-  for (int i = 0; i < F; i++) {
-    const uint32_t k = grp + i * groups;
-    first[i] = b.part_acc[((k < n_splits ? k : n_splits - 1) * rows + r) * s.dim + c0];
-  }
+  for (int i = 0; i < F; i++) first[i] = load(grp + i * groups < n_splits ? grp + i * groups : n_splits - 1);
   if (tid < 64) {
-    const float mm = fmaxf(wave_max(fmaxf(mi[0], mi[1])), sink);
-    const float f0 = __builtin_amdgcn_exp2f(mi[0] - mm), f1 = __builtin_amdgcn_exp2f(mi[1] - mm);
-    const float tot = wave_sum(f0 * li[0] + f1 * li[1]) + __builtin_amdgcn_exp2f(sink - mm);
+    const float m0 = lane < act ? ml[0].x : kTiedNeg, m1 = lane + 64 < act ? ml[1].x : kTiedNeg;
+    const float mm = fmaxf(wave_max(fmaxf(m0, m1)), sink);
+    const float f0 = __builtin_amdgcn_exp2f(m0 - mm), f1 = __builtin_amdgcn_exp2f(m1 - mm);
+    const float l0 = lane < act ? f0 * ml[0].y : 0.0f, l1 = lane + 64 < act ? f1 * ml[1].y : 0.0f;
+    const float tot = wave_sum(l0 + l1) + __builtin_amdgcn_exp2f(sink - mm);
     wgt[lane] = f0 / tot; wgt[lane + 64] = f1 / tot;
   }
   __syncthreads();
-  float v = 0.0f;
+#pragma unroll
+  for (int j = 0; j < V; j++) v.v[j] = 0.0f;
   if (grp < groups) {
 #pragma unroll
     for (int i = 0; i < F; i++) {
       const uint32_t k = grp + i * groups;
-      if (k < act) v = __builtin_fmaf(wgt[k], first[i], v);
+      if (k < act)
+#pragma unroll
+        for (int j = 0; j < V; j++) v.v[j] = __builtin_fmaf(wgt[k], first[i].v[j], v.v[j]);
     }
-    for (uint32_t k = grp + F * groups; k < act; k += groups) v = __builtin_fmaf(wgt[k], b.part_acc[(k * rows + r) * s.dim + c0], v);
+    for (uint32_t k = grp + F * groups; k < act; k += groups) {
+      const Val x = load(k);
+#pragma unroll
+      for (int j = 0; j < V; j++) v.v[j] = __builtin_fmaf(wgt[k], x.v[j], v.v[j]);
+    }
   }
   part[tid] = v;
   __syncthreads();
   if (tid < cols) {
-    for (uint32_t k = 1; k < groups; k++) v += part[tid + k * cols];
-    out[(size_t)t * ldo + h * s.dim + tid] = to_act<O>(v);
+    for (uint32_t k = 1; k < groups; k++)
+#pragma unroll
+      for (int j = 0; j < V; j++) v.v[j] += part[tid + k * cols].v[j];
+#pragma unroll
+    for (int j = 0; j < V; j++) out[(size_t)t * ldo + h * s.dim + c0 + j] = to_act<O>(v.v[j]);
   }
 }
 
 hipError_t tied_merge_launch(const TiedShape& s, const TiedBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32, void* out, uint32_t ldo,
                              bool out_f32, hipStream_t st) {
   if (!tied_ok(s) || n_splits == 0 || n_splits > kTiedMaxSplits || M == 0) return hipErrorInvalidValue;
-  const uint32_t kr = tied_round(tied_lanes(s.dp, f32 ? 4 : 2));
-  if (out_f32) hipLaunchKernelGGL(tied_merge_kernel<float>, dim3(s.heads, M), dim3(256), 0, st, s, b, pos_ptr, pos0, M, n_splits, kr, (float*)out, ldo);
-  else hipLaunchKernelGGL(tied_merge_kernel<__bf16>, dim3(s.heads, M), dim3(256), 0, st, s, b, pos_ptr, pos0, M, n_splits, kr, (__bf16*)out, ldo);
+  const uint32_t kr = tied_keys_per_round(s, f32);
+  const dim3 grid(s.heads, M);
+  const bool v4 = s.dim % 4 == 0;
+  if (out_f32 && v4) hipLaunchKernelGGL((tied_merge_kernel<float, 4>), grid, dim3(256), 0, st, s, b, pos_ptr, pos0, M, n_splits, kr, (float*)out, ldo);
+  else if (out_f32) hipLaunchKernelGGL((tied_merge_kernel<float, 1>), grid, dim3(256), 0, st, s, b, pos_ptr, pos0, M, n_splits, kr, (float*)out, ldo);
+  else if (v4) hipLaunchKernelGGL((tied_merge_kernel<__bf16, 4>), grid, dim3(256), 0, st, s, b, pos_ptr, pos0, M, n_splits, kr, (__bf16*)out, ldo);
+  else hipLaunchKernelGGL((tied_merge_kernel<__bf16, 1>), grid, dim3(256), 0, st, s, b, pos_ptr, pos0, M, n_splits, kr, (__bf16*)out, ldo);
   return hipGetLastError();
 }
 
@@ -413,9 +463,12 @@ __global__ void __launch_bounds__(256) tied_prep_kernel(const TiedShape s, const
     for (int i = 0; i < V; i++) o[i] = to_act<T>(a.v[i]);
     __builtin_memcpy(__builtin_assume_aligned(p, sizeof(o)), o, sizeof(o));
   };
+  Squares vq, vk;
+  squares_fetch(cat + s.off_q, nq, tid * 4, vq);
+  squares_fetch(cat + s.off_k, nk, tid * 4, vk);
   for (uint32_t i = tid * V; i < nk; i += 256 * V)
     store(reinterpret_cast<T*>(b.cache) + ((size_t)(i / s.dim) * s.rows + pos) * s.dp + i % s.dim, load(cat + s.off_k + i));
-  const float sk = squares(cat + s.off_k, nk), sq = squares(cat + s.off_q, nq);
+  const float sk = squares(cat + s.off_k, nk, vk), sq = squares(cat + s.off_q, nq, vq);
   const float kinv = 1.0f / __builtin_sqrtf(block_sum(sk, red) / (float)nk + s.eps);
   if (tid == 0) b.kinv[pos] = kinv;
   if (!b.q) return;
