@@ -31,6 +31,10 @@ struct CapF {
     const float z = u * u;
     return __builtin_fmaf(u, __builtin_fmaf(z, __builtin_fmaf(z, __builtin_fmaf(z, __builtin_fmaf(z, c4, c3), c2), c1), c0), add);
   }
+  __device__ __forceinline__ float small_bf(float u, float add) const {   // to 4e-7 of the score: keys and queries are bf16
+    const float z = u * u;
+    return __builtin_fmaf(u, __builtin_fmaf(z, __builtin_fmaf(z, __builtin_fmaf(z, c3, c2), c1), c0), add);
+  }
   __device__ __forceinline__ float any(float u, float add) const { return fabsf(u) < lim ? small(u, add) : __builtin_fmaf(tanh_f(u), c0, add); }
 };
 __device__ __forceinline__ float tied_slope(uint32_t h, uint32_t heads) {   // in units of log2
@@ -580,6 +584,7 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
       for (int n = 0; n < NK; n++)
 #pragma unroll
         for (int t = 0; t < QT; t++) sa[n][t] = (f32x4)(0.0f);
+      __builtin_amdgcn_s_setprio(1);   // products ahead of the other waves' softmax
 #pragma unroll
       for (int u = 0; u < NU; u++)
 #pragma unroll
@@ -589,6 +594,7 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
 #pragma unroll
           for (int t = 0; t < QT; t++) sa[n][t] = Frag<T>::mma(kf, qf[t][u], sa[n][t]);
         }
+      __builtin_amdgcn_s_setprio(0);
       float top = 0.0f;
 #pragma unroll
       for (int t = 0; t < QT; t++)
@@ -613,7 +619,7 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
 #pragma unroll
           for (int n = 0; n < NK; n++)
 #pragma unroll
-            for (int e = 0; e < 4; e++) sa[n][t][e] = cap.small(sa[n][t][e], bias[n][e]);
+            for (int e = 0; e < 4; e++) sa[n][t][e] = BF ? cap.small_bf(sa[n][t][e], bias[n][e]) : cap.small(sa[n][t][e], bias[n][e]);
       }
 #pragma unroll
       for (int t = 0; t < QT; t++) {
@@ -635,10 +641,19 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
 #pragma unroll
           for (int e = 0; e < 4; e++) m1 = fmaxf(m1, sa[n][t][e]);
         m1 = fmaxf(m1, __shfl_xor(m1, 16, 64));
-        m1 = fmaxf(fmaxf(m1, __shfl_xor(m1, 32, 64)) + off, mx[t]);
-        const float rel = m1 - off;
+        m1 = fmaxf(m1, __shfl_xor(m1, 32, 64)) + off;
+        // the reference follows the maximum once it has risen by more than 2^8: weights stay far from overflow, most tiles rescale nothing; each
+        // query by itself, so that its rounding does not depend on its neighbours
         // (a query that has seen nothing yet weighs masked keys; the factor of its first visible tile takes that to 0)
-        const float a = __builtin_amdgcn_exp2f(mx[t] - m1);
+        if (__any(m1 > mx[t] + 8.0f)) {
+          asm volatile("");
+          const float m2 = m1 > mx[t] + 8.0f ? m1 : mx[t], a = __builtin_amdgcn_exp2f(mx[t] - m2);
+          mx[t] = m2;
+          l[t] *= a;
+#pragma unroll
+          for (int d = 0; d < ND; d++) o[d][t] *= a;
+        }
+        const float rel = mx[t] - off;
         float sum = 0.0f;
 #pragma unroll
         for (int n = 0; n < NK; n++)
@@ -648,13 +663,9 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
             sa[n][t][e] = p;
             sum += p;
           }
-        l[t] = __builtin_fmaf(l[t], a, sum);
-        if (__any(m1 > mx[t])) {
-#pragma unroll
-          for (int d = 0; d < ND; d++) o[d][t] *= a;
-        }
-        mx[t] = m1;
+        l[t] += sum;
       }
+      __builtin_amdgcn_s_setprio(1);
       if constexpr (BF) {
 #pragma unroll
         for (int u = 0; u < KT / 32; u++) {
@@ -680,6 +691,7 @@ __global__ void __launch_bounds__(256, (tied_wgs<T, DQ>())) tied_flash_kernel(co
             for (int t = 0; t < QT; t++) o[d][t] = Frag<T>::mma(vf, sa[n][t], o[d][t]);
           }
       }
+      __builtin_amdgcn_s_setprio(0);
     }
     wait_vm(0);
     __syncthreads();
