@@ -182,10 +182,15 @@ template <int V> __device__ __forceinline__ void store_vec(float* p, const VecF<
 
 // y of one token's channels: the sublayer's output plus its experts' rows
 template <int V> __device__ __forceinline__ VecF<V> add_pairs(VecF<V> y, const float* pairs, uint32_t ldp, const int* slot, uint32_t top, uint32_t c) {
-  for (uint32_t s = 0; s < top; s++) {
-    const VecF<V> p = load_vec<V>(pairs + (size_t)slot[s] * ldp + c);
+  for (uint32_t s = 0; s < top; s += 4) {   // four rows in flight
+    VecF<V> p[4];
 #pragma unroll
-    for (int i = 0; i < V; i++) y.v[i] += p.v[i];
+    for (uint32_t k = 0; k < 4; k++) p[k] = load_vec<V>(pairs + (size_t)slot[s + k < top ? s + k : s] * ldp + c);
+#pragma unroll
+    for (uint32_t k = 0; k < 4; k++)
+      if (s + k < top)
+#pragma unroll
+        for (int i = 0; i < V; i++) y.v[i] += p[k].v[i];
   }
   return y;
 }

@@ -66,7 +66,15 @@ __global__ void __launch_bounds__(1024) moe_group_rows_kernel(const MoeRoute a) 
   const uint32_t tid = threadIdx.x, pairs = a.M * a.top;
   cnt[tid] = 0;
   __syncthreads();
-  for (uint32_t p = tid; p < pairs; p += 1024) atomicAdd(&cnt[a.sel[p]], 1);
+  constexpr uint32_t U = 8;   // pairs a thread has in flight
+  for (uint32_t p0 = tid; p0 < pairs; p0 += U * 1024) {
+    int e[U];
+#pragma unroll
+    for (uint32_t u = 0; u < U; u++) e[u] = a.sel[p0 + u * 1024 < pairs ? p0 + u * 1024 : p0];
+#pragma unroll
+    for (uint32_t u = 0; u < U; u++)
+      if (p0 + u * 1024 < pairs) atomicAdd(&cnt[e[u]], 1);
+  }
   __syncthreads();
   const int n = cnt[tid], nt = (n + (int)a.bm - 1) / (int)a.bm;
   row0[tid] = n;
@@ -92,11 +100,24 @@ __global__ void __launch_bounds__(1024) moe_group_rows_kernel(const MoeRoute a) 
   for (uint32_t i = used + tid; i < a.tiles; i += 1024) { a.tile_e[i] = -1; a.tile_row[i] = 0; }
   cnt[tid] = first;
   __syncthreads();
-  for (uint32_t p = tid; p < pairs; p += 1024) {
-    const int r = atomicAdd(&cnt[a.sel[p]], 1);
-    a.slot[p] = r;
-    a.src[r] = (int)(p / a.top);
-    a.roww[r] = a.w[p];
+  for (uint32_t p0 = tid; p0 < pairs; p0 += U * 1024) {
+    int e[U];
+    float w[U];
+#pragma unroll
+    for (uint32_t u = 0; u < U; u++) {
+      const uint32_t p = p0 + u * 1024 < pairs ? p0 + u * 1024 : p0;
+      e[u] = a.sel[p];
+      w[u] = a.w[p];
+    }
+#pragma unroll
+    for (uint32_t u = 0; u < U; u++) {
+      const uint32_t p = p0 + u * 1024;
+      if (p >= pairs) break;
+      const int r = atomicAdd(&cnt[e[u]], 1);
+      a.slot[p] = r;
+      a.src[r] = (int)(p / a.top);
+      a.roww[r] = w[u];
+    }
   }
 }
 
