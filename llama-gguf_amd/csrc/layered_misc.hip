@@ -235,57 +235,57 @@ __global__ void __launch_bounds__(256) dyt_block_kernel(const DytBlock a) {
   request(first, nx);
   int at = 0;                                       // ring row of token t
   for (int tg = first; tg < t1; tg += G) {
-   const Group cu = nx;
-   if (tg + G < t1) request(tg + G, nx);
+    const Group cu = nx;
+    if (tg + G < t1) request(tg + G, nx);
 #pragma unroll
-   for (int g = 0; g < G; g++) {
-    const int t = tg + g;
-    if (t >= t1) break;
-    VecF<V> v = cu.x[g], h, y;
-    if (t < 0) {                                    // before the block
-      const int p = (int)a.pos0 + t;
+    for (int g = 0; g < G; g++) {
+      const int t = tg + g;
+      if (t >= t1) break;
+      VecF<V> v = cu.x[g], h, y;
+      if (t < 0) {                                    // before the block
+        const int p = (int)a.pos0 + t;
 #pragma unroll
-      for (int i = 0; i < V; i++) h.v[i] = 0.0f;
-      if (p >= 0) h = load_vec<V>(a.conv.hist + (size_t)(p % back) * W + c);
-    } else {
-      if (upd) {
+        for (int i = 0; i < V; i++) h.v[i] = 0.0f;
+        if (p >= 0) h = load_vec<V>(a.conv.hist + (size_t)(p % back) * W + c);
+      } else {
+        if (upd) {
 #pragma unroll
-        for (int i = 0; i < V; i++) y.v[i] = a.y ? cu.y[g].v[i] : 0.0f;
+          for (int i = 0; i < V; i++) y.v[i] = a.y ? cu.y[g].v[i] : 0.0f;
 #pragma unroll
-        for (int k = 0; k < P; k++)
-          if (k < n_pairs)
+          for (int k = 0; k < P; k++)
+            if (k < n_pairs)
 #pragma unroll
-            for (int i = 0; i < V; i++) y.v[i] += cu.p[g][k].v[i];
-        if (n_pairs > P) y = add_pairs<V>(y, a.pairs, a.ldp, a.slot + (size_t)t * a.top + P, a.top - P, c);
+              for (int i = 0; i < V; i++) y.v[i] += cu.p[g][k].v[i];
+          if (n_pairs > P) y = add_pairs<V>(y, a.pairs, a.ldp, a.slot + (size_t)t * a.top + P, a.top - P, c);
 #pragma unroll
-        for (int i = 0; i < V; i++) v.v[i] = __builtin_fmaf(a.mult, dyt_f(y.v[i], pal, pw.v[i], pb.v[i]), v.v[i]);
-        if (t >= t0 && live) store_vec<V>(a.xout + (size_t)t * W + c, v);
+          for (int i = 0; i < V; i++) v.v[i] = __builtin_fmaf(a.mult, dyt_f(y.v[i], pal, pw.v[i], pb.v[i]), v.v[i]);
+          if (t >= t0 && live) store_vec<V>(a.xout + (size_t)t * W + c, v);
+        }
+        if (!nxt) continue;
+#pragma unroll
+        for (int i = 0; i < V; i++) h.v[i] = dyt_f(v.v[i], nal, nw.v[i], nb.v[i]);
       }
-      if (!nxt) continue;
+      if (taps) store_vec<V>(ring + at * 256 * V, h);
+      if (t >= t0) {
+        VecF<V> o = h;
+        int r = at + 1 < taps ? at + 1 : 0;           // the oldest input
+        for (int j = 0; j < taps; j++) {
+          const VecF<V> q = load_vec<V>(ring + r * 256 * V), w = load_vec<V>(filt + j * 256 * V);
 #pragma unroll
-      for (int i = 0; i < V; i++) h.v[i] = dyt_f(v.v[i], nal, nw.v[i], nb.v[i]);
+          for (int i = 0; i < V; i++) o.v[i] = __builtin_fmaf(w.v[i], q.v[i], o.v[i]);
+          r = r + 1 < taps ? r + 1 : 0;
+        }
+        if (live) {
+          T* dst = reinterpret_cast<T*>(a.xa) + (size_t)t * a.ldx + c;
+          T q[V];
+#pragma unroll
+          for (int i = 0; i < V; i++) q[i] = to_act<T>(o.v[i]);
+          __builtin_memcpy(__builtin_assume_aligned(dst, sizeof(q)), q, sizeof(q));
+          if (t >= (int)a.M - back) store_vec<V>(a.tail + (size_t)((int)a.M - 1 - t) * W + c, h);
+        }
+      }
+      at = at + 1 < taps ? at + 1 : 0;
     }
-    if (taps) store_vec<V>(ring + at * 256 * V, h);
-    if (t >= t0) {
-      VecF<V> o = h;
-      int r = at + 1 < taps ? at + 1 : 0;           // the oldest input
-      for (int j = 0; j < taps; j++) {
-        const VecF<V> q = load_vec<V>(ring + r * 256 * V), w = load_vec<V>(filt + j * 256 * V);
-#pragma unroll
-        for (int i = 0; i < V; i++) o.v[i] = __builtin_fmaf(w.v[i], q.v[i], o.v[i]);
-        r = r + 1 < taps ? r + 1 : 0;
-      }
-      if (live) {
-        T* dst = reinterpret_cast<T*>(a.xa) + (size_t)t * a.ldx + c;
-        T q[V];
-#pragma unroll
-        for (int i = 0; i < V; i++) q[i] = to_act<T>(o.v[i]);
-        __builtin_memcpy(__builtin_assume_aligned(dst, sizeof(q)), q, sizeof(q));
-        if (t >= (int)a.M - back) store_vec<V>(a.tail + (size_t)((int)a.M - 1 - t) * W + c, h);
-      }
-    }
-    at = at + 1 < taps ? at + 1 : 0;
-   }
   }
 }
 
