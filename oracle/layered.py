@@ -194,11 +194,150 @@ def causal_conv(h, w):
     return out
 
 
-MIXERS = {"latent_attention": latent_attention, "mlstm": mlstm, "attention": tied_attention}
+def softplus(z):
+    return np.logaddexp(0.0, z)
+
+
+def linear(x, w, name):
+    """A projection, with its bias where there is one."""
+    y = x @ w[name].T
+    return y + w[name + ".b"] if name + ".b" in w else y
+
+
+def block_diagonal(u, m, b):
+    """u [T, n * s] in n parts, each through its own square matrix m [n, s, s] with bias b [n, s]."""
+    n, s = m.shape[0], m.shape[1]
+    parts = [u[:, i * s:(i + 1) * s] @ m[i].T + b[i] for i in range(n)]
+    return np.concatenate(parts, axis=1)
+
+
+def linear_recurrence(a, x):
+    """S_t = a_t S_(t-1) + x_t per channel, from nothing; all S [T, channels]."""
+    S, out = np.zeros(a.shape[1], dtype=F), np.zeros_like(a)
+    for t in range(len(a)):
+        S = a[t] * S + x[t]
+        out[t] = S
+    return out
+
+
+def rglru(h, w, mx, eps):
+    """A gated linear recurrence per channel behind a short convolution, beside a gelu branch."""
+    y = gelu_tanh(linear(h, w, "y"))
+    u = causal_conv(linear(h, w, "x"), w["conv"]) + w["conv.b"]
+    r = sigmoid(block_diagonal(u, w["ra"], w["ra.b"]))
+    i = sigmoid(block_diagonal(u, w["ri"], w["ri.b"]))
+    log_a = -8.0 * r * softplus(w["lam"])
+    S = linear_recurrence(np.exp(log_a), np.sqrt(-np.expm1(2.0 * log_a)) * i * u)
+    return (S * y) @ w["o"].T
+
+
+def chunk_keys(i, size):
+    """Positions that position i sees when the sequence is cut into chunks of `size` (0: not cut) from position 0 on."""
+    return list(range(i // size * size if size else 0, i + 1))
+
+
+def gated_attention(h, w, mx, eps):
+    """Grouped attention with its own values; queries and keys normed per head and then rotated; keys of the own chunk; the output gated element
+    by element before its projection."""
+    T, H, G, d, dv = len(h), mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+    pos = np.arange(T)
+    q = rms(linear(h, w, "q").reshape(T, H, d), eps) * w["q.norm"]
+    k = rms(linear(h, w, "k").reshape(T, G, d), eps) * w["k.norm"]
+    v = linear(h, w, "v").reshape(T, G, dv)
+    if mx.get("rot"):
+        q, k = rotate_pairs(q, pos, mx["rot"]), rotate_pairs(k, pos, mx["rot"])
+    size = mx["mask"]["size"] if mx.get("mask") else 0
+    out = np.zeros((T, H, dv), dtype=F)
+    for i in range(T):
+        seen = chunk_keys(i, size)
+        for n in range(H):
+            g = n // (H // G)
+            s = (k[seen, g] @ q[i, n]) * mx["scale"]
+            p = np.exp(s - s.max())
+            out[i, n] = (p / p.sum()) @ v[seen, g]
+    return (out.reshape(T, H * dv) * sigmoid(h @ w["g"].T)) @ w["o"].T
+
+
+def gated_linear_attention(h, w, mx, eps):
+    """A matrix state per head whose rows (key channels) decay each at its own rate, one token after the other."""
+    T, H, d, dv = len(h), mx["heads"], mx["dim"], mx["vdim"]
+    q = (h @ w["q"].T).reshape(T, H, d) * d ** -0.5
+    k = (h @ w["k"].T).reshape(T, H, d)
+    v = (h @ w["v"].T).reshape(T, H, dv)
+    z = (h @ w["a1"].T) @ w["a2"].T + w["a2.b"]
+    alpha = np.exp(log_sigmoid(z) / mx["tau"]).reshape(T, H, d)
+    out = np.zeros((T, H, dv), dtype=F)
+    for n in range(H):
+        S = np.zeros((d, dv), dtype=F)
+        for t in range(T):
+            S = alpha[t, n][:, None] * S + np.outer(k[t, n], v[t, n])
+            out[t, n] = S.T @ q[t, n]
+    o = rms(out, eps) * w["norm"]
+    return (o.reshape(T, H * dv) * silu(h @ w["g"].T)) @ w["o"].T
+
+
+def parallel(h, w, mx, eps):
+    """Attention and linear attention side by side on the same input."""
+    side = lambda s: {k[len(s):]: v for k, v in w.items() if k.startswith(s)}
+    return (mx["left_scale"] * gated_attention(h, side("left."), mx["left"], eps)
+            + mx["right_scale"] * gated_linear_attention(h, side("right."), mx["right"], eps))
+
+
+def clamped_expert(x, w, name, limit):
+    g = np.minimum(x @ w[name + ".gate"].T, limit)
+    u = np.clip(x @ w[name + ".up"].T, -limit, limit)
+    return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w[name + ".down"].T
+
+
+def route_groups(z, correction, router):
+    """(expert, weight) of a token: softmax scores; the choice by corrected scores among the best groups of neighbours; the weights are the plain
+    scores of the chosen ones, divided by their sum."""
+    s = np.exp(z - z.max())
+    s = s / s.sum()
+    c = s + correction
+    n, keep = router["groups"]["count"], router["groups"]["keep"]
+    size = len(z) // n
+    best = sorted(range(n), key=lambda g: (-c[g * size:(g + 1) * size].max(), g))[:keep]
+    open_ = [e for e in range(len(z)) if e // size in best]
+    chosen = sorted(open_, key=lambda e: (-c[e], e))[: router["top"]]
+    total = sum(s[e] for e in chosen) + 1e-20
+    return [(e, s[e] / total) for e in chosen]
+
+
+def grouped_moe_ff(x, w, mlp):
+    """Weighted sum of the chosen experts' outputs; the last `identity` router outputs hand the input back."""
+    out = np.zeros_like(x)
+    for t, z in enumerate(x @ w["router"].T):
+        for e, g in route_groups(z, w["correction"], mlp["router"]):
+            out[t] += g * (x[t] if e >= mlp["router"]["experts"] else clamped_expert(x[t], w, f"e{e}", mlp["expert"]["limit"]))
+    return out
+
+
+MIXERS = {"latent_attention": latent_attention, "mlstm": mlstm, "attention": tied_attention, "rglru": rglru, "parallel": parallel,
+          "gated_attention": gated_attention, "gla": gated_linear_attention}
 
 
 def feed_forward(x, w, mlp):
-    return moe_ff(x, w, mlp) if mlp["kind"] == "moe" else dense_ff(x, w)
+    if mlp["kind"] != "moe":
+        return dense_ff(x, w)
+    return grouped_moe_ff(x, w, mlp) if "groups" in mlp["router"] else moe_ff(x, w, mlp)
+
+
+def forward_pre_norm(cfg, weights, tokens, layers_out=None):
+    """Sublayers read the RMS-normed stream and add to it; the output projection is the embedding table."""
+    W = {k: np.asarray(v, dtype=F) for k, v in weights.items()}
+    eps = cfg["norm"]["eps"]
+    norm = lambda v, name: rms(v, eps) * (1.0 + W[name])
+    x = W["embed"][list(tokens)]
+    for i, lay in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        sub = lambda g: {k[len(p + g):]: v for k, v in W.items() if k.startswith(p + g)}
+        x = x + MIXERS[lay["type"]](norm(x, p + "norm1"), sub("mix."), lay["mixer"], eps)
+        if lay["mlp"]:
+            x = x + feed_forward(norm(x, p + "norm2"), sub("mlp."), lay["mlp"])
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return norm(x, "final.norm") @ W["embed"].T * cfg["logit_scale"]
 
 
 def forward_sandwich(cfg, weights, tokens, layers_out=None):
@@ -226,6 +365,8 @@ def forward(cfg, weights, tokens, layers_out=None):
     """Logits [T, vocab] of a whole sequence; layers_out (a list) receives the residual stream after every layer."""
     if "canon" in cfg:
         return forward_sandwich(cfg, weights, tokens, layers_out)
+    if "logit_scale" in cfg:
+        return forward_pre_norm(cfg, weights, tokens, layers_out)
     W = {k: np.asarray(v, dtype=F) for k, v in weights.items()}
     eps, m = cfg["norm"]["eps"], cfg["residual_mult"]
     x = W["embed"][list(tokens)]
