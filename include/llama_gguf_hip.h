@@ -167,7 +167,10 @@ enum {
   LGH_SYM_LATENT = 22,     /* lgh::latent_* : attention over a shared latent */
   LGH_SYM_MLSTM = 23,      /* lgh::mlstm_* : matrix-memory recurrence */
   LGH_SYM_TIED = 24,       /* lgh::tied_* : attention whose values are its keys */
-  LGH_SYM_COUNT = 25
+  LGH_SYM_GATTN = 25,      /* lgh::gattn_* : attention with gated values; gated linear attention where it runs beside it */
+  LGH_SYM_GLA = 26,        /* lgh::gla_* : gated linear attention */
+  LGH_SYM_GLRU = 27,       /* lgh::glru_* : gated linear recurrence per channel */
+  LGH_SYM_COUNT = 28
 };
 
 typedef struct lgh_stats {
@@ -278,16 +281,26 @@ int lgh_eval(lgh_ctx* ctx, const uint32_t* tokens, size_t n, const uint32_t* wan
  *   LGH_RESIDUAL_POST_LN       sublayers read the stream itself, x += residual_mult * layer_norm(sublayer(x)) * w
  *   LGH_RESIDUAL_SANDWICH_DYT  h = dyt(x); h += conv(h); x += residual_mult * dyt'(sublayer(h)), where dyt(x) = tanh(alpha x) * w + b and
  *                              conv is a causal convolution over conv_taps positions, one filter per channel (0 taps: none)
+ *   LGH_RESIDUAL_PRE_RMS       x += residual_mult * sublayer(rms_norm(x) * (1 + w))
  * No reference counterpart.  The context is driven by the entry points above (GpuInference, lgh_eval, lgh_decode_greedy, ...; the
  * cache rows and recurrent states are the context's).  Weights are bf16 and stay bf16 in HBM; tensors are uploaded by their
  * checkpoint names (`embed`, `bigram`, `l0.mix.q`, `l0.mlp.gate`, `l0.mlp.e0.gate`, `l0.norm1`, `l0.norm1.alpha`, `l0.canon1`, `final.norm`,
  * `head`) with GGML dims (in fastest; a scalar has one element).
  * Single stage, one sequence per context. ---- */
 enum { LGH_MIXER_LATENT_ATTENTION = 1, LGH_MIXER_MLSTM = 2,
-       LGH_MIXER_TIED_ATTENTION = 3 };                 /* grouped heads, values = keys before their norm, no rotation; window, sinks, distance bias */
-enum { LGH_RESIDUAL_POST_LN = 0, LGH_RESIDUAL_SANDWICH_DYT = 1 };
+       LGH_MIXER_TIED_ATTENTION = 3,                   /* grouped heads, values = keys before their norm, no rotation; window, sinks, distance bias */
+       LGH_MIXER_GATED_ATTENTION = 4,                  /* grouped heads, biases, norms per head, rotation, chunks; the output gated value by value */
+       LGH_MIXER_GLA = 5,                              /* gated linear attention: a matrix state whose rows decay each at its own rate */
+       LGH_MIXER_PARALLEL = 6,                         /* left_scale * gated attention + right_scale * gated linear attention, same input */
+       LGH_MIXER_GLRU = 7 };                           /* gated linear recurrence per channel behind a short convolution, times a gelu branch */
+enum { LGH_RESIDUAL_POST_LN = 0, LGH_RESIDUAL_SANDWICH_DYT = 1, LGH_RESIDUAL_PRE_RMS = 2 };
 enum { LGH_FF_NONE = 0, LGH_FF_GEGLU = 1 };            /* down(gelu_tanh(gate x) * (up x)) */
 enum { LGH_FF_MOE = 2 };                               /* routed experts down(silu(gate x) * (up x)), sigmoid scores; optionally a shared one */
+/* how a mixture's experts are chosen and weighted: sigmoid scores, the score multiplies the expert's input; or softmax scores, the choice by
+ * score + correction among the best groups of neighbours, the chosen scores divided by their sum multiply the experts' outputs */
+enum { LGH_ROUTER_SIGMOID = 0, LGH_ROUTER_SOFTMAX_GROUPS = 1 };
+enum { LGH_EXPERT_SWIGLU = 0,                          /* silu(gate) * up */
+       LGH_EXPERT_CLAMPED = 1 };                       /* g = min(gate, limit), u = clamp(up, -limit, limit): g * sigmoid(1.702 g) * (u + 1) */
 enum { LGH_COMPUTE_BF16 = 0, LGH_COMPUTE_F32 = 1 };    /* operands of block products, cache rows: bf16 (f32 accumulation), or f32 throughout */
 typedef struct lgh_layer_desc {
   uint32_t struct_size;
@@ -296,15 +309,24 @@ typedef struct lgh_layer_desc {
   uint32_t kv_rank, rot_dim;         /* latent attention: latent size, rotated query / key part */
   uint32_t rot_dims;                 /* leading values of the rotated part that are rotated (neighbouring pairs) */
   uint32_t ff_kind, ff;              /* LGH_FF_*, feed-forward size (mixture: of one expert) */
-  uint32_t kv_heads;                 /* tied attention: key heads; query head h uses h / (heads / kv_heads) */
+  uint32_t kv_heads;                 /* tied, gated attention: key heads; query head h uses h / (heads / kv_heads) */
   uint32_t window, keep_first;       /* tied attention: position i sees j <= i with i - j < window (0: no limit) or j < keep_first */
   uint32_t experts, top;             /* mixture: experts, and how many a token uses */
   uint32_t shared_ff;                /* mixture: size of the expert every token uses (0: none) */
+  uint32_t router_form, expert_form; /* mixture: LGH_ROUTER_*, LGH_EXPERT_* */
+  uint32_t groups, keep_groups;      /* LGH_ROUTER_SOFTMAX_GROUPS: groups of neighbours, and how many of them stay open */
+  uint32_t identity;                 /* LGH_ROUTER_SOFTMAX_GROUPS: further router outputs behind the experts whose expert is its input */
+  uint32_t chunk;                    /* gated attention: position i sees j <= i of the same chunk of this many positions (0: one chunk) */
+  uint32_t taps;                     /* linear recurrence: positions of its convolution; heads = diagonal blocks, dim = vdim = their size */
+  uint32_t gla_heads, gla_dim, gla_vdim, gla_rank;   /* gated linear attention; gla_rank: inner size of the decay's projection */
   double scale;                      /* attention: factor on the scores */
   double rot_base;
   double yarn_factor, yarn_original, yarn_fast, yarn_slow;   /* yarn_factor 0: plain frequencies */
   double gate_cap;                   /* mLSTM: soft cap of the gates' pre-activations */
   double score_cap;                  /* tied attention: soft cap of the scores (0: none) */
+  double expert_limit;               /* LGH_EXPERT_CLAMPED */
+  double gla_tau;                    /* gated linear attention: decay = sigmoid(z)^(1 / tau) */
+  double left_scale, right_scale;    /* LGH_MIXER_PARALLEL */
 } lgh_layer_desc;
 typedef struct lgh_layered_desc {
   uint32_t struct_size;
@@ -317,6 +339,9 @@ typedef struct lgh_layered_desc {
   double norm_eps, residual_mult;
   uint32_t residual;                 /* LGH_RESIDUAL_* */
   uint32_t conv_taps;
+  uint32_t tied_head;                /* 1: the output projection is the embedding table (no tensor `head`) */
+  uint32_t reserved;
+  double logit_scale;                /* factor on the logits (0: 1) */
 } lgh_layered_desc;
 int lgh_create_layered(const lgh_layered_desc* desc, const lgh_layer_desc* layers, lgh_ctx** out);
 /* Residual stream after every layer, for parity tests: switched on, the next lgh_eval portions (block path) keep it;

@@ -1,6 +1,6 @@
 // layered.h — models whose layers are described one by one (lgh_layer_desc: a mixer and an optional feed-forward), on the engine's own
 // context, step function and graphs (internal).  Kernels: linear_bf16.hip (matrix products), latent_attention.hip, tied_attention.hip,
-// mlstm.hip, moe_route.hip (routing of the experts), layered_misc.hip (embedding, norms, residual updates); layered.hip assembles them.
+// gated_attention.hip, mlstm.hip, gla.hip, glru.hip, moe_route.hip (routing of the experts), layered_misc.hip (embedding, norms, residual updates); layered.hip assembles them.
 #pragma once
 
 #include "common.h"
@@ -43,6 +43,7 @@ enum LinPro : int {
   LP_RESID = 1,   // x + mult * layer_norm(y) * nw, also written to xout (the new residual stream)
   LP_HEAD = 2,    // layer_norm of the same sum, times nw2 (final norm in front of the output projection)
   LP_MLSTM = 3,   // matrix-memory read-out: numerators / denominators, per-head RMS norm, norm weight, sigmoid gate
+  LP_PRE = 4,     // v = x + mult * y (y may be absent), also written to xout; rms_norm(v) * (1 + nw2) * in_scale, also written to hout
 };
 // Which weights its rows come from
 enum LinSrc : int {
@@ -51,7 +52,13 @@ enum LinSrc : int {
   LS_EXPERTS = 2,  // the top experts of `logits` (every workgroup ranks them), their gate | up pairs; the input is weighted by the expert's score
   LS_MOE_DOWN = 3, // input [shared | expert | expert ..]: a row is a row of w (shared, absent: kps = 0) followed by the same row of every chosen expert
 };
-enum LinAct : uint32_t { LA_GELU = 0, LA_SILU = 1 };
+enum LinAct : uint32_t { LA_GELU = 0, LA_SILU = 1, LA_CLAMPED = 2 };   // act(gate) * up; LA_CLAMPED: clamped_glu_f
+// how a token's experts are chosen (LGH_ROUTER_*)
+struct RouteForm {
+  uint32_t form = LGH_ROUTER_SIGMOID;
+  uint32_t groups = 1, keep = 1, identity = 0;
+  const float* correction = nullptr;   // [experts + identity]
+};
 struct LinMv {
   const uint16_t* w;
   uint32_t n, kp, k, paired;   // paired: 0 or 1
@@ -62,7 +69,10 @@ struct LinMv {
   const float* nw;             // its norm weight
   const float* nw2;
   float* xout;
-  float eps, mult;
+  float eps, mult, in_scale;
+  const float* bias;           // [n], unpaired rows (NULL: none)
+  float* hout;                 // LP_PRE: the input vector (NULL: not kept)
+  float limit;                 // LA_CLAMPED
   const float* num;            // LP_MLSTM: [heads][ldo] numerators, column vdim = n . q, column vdim + 1 = exp(-m)
   const float* gate;
   uint32_t heads, vdim, ldo;
@@ -73,11 +83,15 @@ struct LinMv {
   uint32_t experts, top;
   int* sel;                    // [top] chosen experts: written by LS_EXPERTS, read by LS_MOE_DOWN
   uint64_t stride;             // elements between two experts
+  RouteForm route;             // LS_EXPERTS (a form other than sigmoid scores weights the experts' outputs, with `logits` [experts + identity])
+  float* selw;                 // [top] weights of the chosen: written by LS_EXPERTS; LS_MOE_DOWN: those of identity experts multiply id_x
+  const float* id_x;           // LS_MOE_DOWN: what identity experts hand back (NULL: there are none)
   uint32_t kps, kpe;           // LS_MOE_DOWN: columns of the shared part and of an expert; LS_EXPERTS: an expert's outputs lie kpe apart
   PostUpdate post;             // post.xout set: rows are not stored but update the residual stream
 };
+bool route_ok(const RouteForm& f, uint32_t outputs, uint32_t top);   // LGH_ROUTER_SOFTMAX_GROUPS
 hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st, int src = LS_PLAIN);
-constexpr uint32_t kMaxExperts = 1024, kMaxTop = 64;
+constexpr uint32_t kMaxExperts = 1024, kMaxTop = 64, kMaxRouted = 512;   // (the last: router outputs of LGH_ROUTER_SOFTMAX_GROUPS)
 constexpr uint32_t kLinMvMaxK = 36864;   // input vectors live in LDS
 
 // Matrix product of a block of tokens: out[m][n] = sum_k x[m][k] * w[n][k].  f32 = true: activations and products in 32-bit
@@ -89,13 +103,15 @@ enum LinEpi : int {
   LE_HEADS = 3,   // activation type, row n = head * hd + j of token m at out[(head * tcap + m) * ldo + j]
   LE_HEADS_T = 4, // activation type, transposed per head: out[(head * hrows + j) * ldo + m]
   LE_SWIGLU = 5,  // paired weights: silu(gate) * up as activation type [M][ldo]
+  LE_CLAMPED = 6, // grouped rows, paired weights: scale * clamped_glu_f(gate, up) as activation type [M][ldo]
 };
 // rows grouped by expert: row tile i takes rows tile_row[i] .. of the group tile_e[i] (-1: no tile), which ends at seg[group + 1]; that
 // group's weights lie `stride` elements per group behind w
 struct LinGroup {
   const int *seg = nullptr, *tile_e = nullptr, *tile_row = nullptr;
   const int* src = nullptr;        // row of x of every row (NULL: the same row)
-  const float* scale = nullptr;    // factor of every row's input (LE_SWIGLU)
+  const float* scale = nullptr;    // factor of every row's input (LE_SWIGLU) or output (LE_CLAMPED)
+  float limit = 0.0f;              // LE_CLAMPED
   uint64_t stride = 0;
   uint32_t tiles = 0, bm = 0;      // row tiles (upper bound) and their height
 };
@@ -106,6 +122,7 @@ struct LinGemm {
   uint32_t n, np, kp, ldx, ldo, M;
   uint32_t hd, hrows;          // LE_HEADS / LE_HEADS_T
   uint64_t tcap;
+  const float* bias;           // LE_F32: [n] (NULL: none)
   LinGroup grp;
 };
 hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st);
@@ -119,7 +136,7 @@ hipError_t lin_transpose_heads_launch(const uint16_t* src, uint32_t heads, uint3
 struct EmbedArgs {
   const uint16_t* embed;       // [vocab][width] bf16
   const uint16_t* bigram;      // [buckets + 1][width] or NULL
-  uint32_t width, buckets;
+  uint32_t width, buckets, ld; // ld: row stride of the embedding table
   uint64_t mul_prev, mul_cur;
   int* hist;                   // token of every position (the previous token is part of the sequence's state)
 };
@@ -161,6 +178,25 @@ hipError_t conv_store_launch(const float* tails, float* hists, uint32_t n_sub, u
 // y[t] += a token's rows of `pairs` in slot order (a mixture in front of LGH_RESIDUAL_POST_LN); add = false: y[t] = the rows' sum
 hipError_t pair_sum_launch(float* y, uint32_t ldy, const float* pairs, uint32_t ldp, const int* slot, uint32_t top, uint32_t width, uint32_t M, bool add, hipStream_t st);
 
+// LGH_RESIDUAL_PRE_RMS over a block: x += mult * (y + a token's rows of `pairs` in slot order); a slot of -1 stands for selw * (the sublayer's
+// input, still in xa).  rms_norm(x) * (1 + nw) -> xa (nw NULL: not wanted).  y and pairs may be NULL.
+struct PreBlock {
+  float* x;
+  const float* y;
+  const float* pairs;
+  const int* slot;
+  const float* selw;
+  const float* nw;
+  void* xa;
+  uint32_t ldy, ldp, top, ldx, width, M;
+  float eps, mult;
+};
+hipError_t pre_block_launch(const PreBlock& a, bool f32, hipStream_t st);
+// decode without a consumer: xout = x + mult * y
+hipError_t resid_add_launch(const float* x, const float* y, float mult, uint32_t width, float* xout, hipStream_t st);
+hipError_t final_rms_rows_launch(const float* x, const int* rows, uint32_t n_rows, const float* w, float eps, float scale, uint32_t width, void* xa, uint32_t ldx,
+                                 bool f32, hipStream_t st);
+
 // ---- moe_route.hip: a block's tokens to their experts ----
 struct MoeRoute {
   const void* x;               // [M][ldx]
@@ -173,6 +209,7 @@ struct MoeRoute {
   int *src;                    // [M * top]: token of the row
   float* roww;                 // [M * top]: score of the row
   uint32_t tiles;              // entries of tile_e / tile_row
+  RouteForm route;             // (the chosen ones from `experts` on are identity experts: their slot is -1)
 };
 uint32_t moe_max_tiles(uint32_t rows, uint32_t experts, uint32_t bm);
 hipError_t moe_route_launch(const MoeRoute& a, bool f32, hipStream_t st);   // router product, scores, groups
@@ -203,6 +240,79 @@ hipError_t tied_merge_launch(const TiedShape& s, const TiedBufs& b, const int* p
                              bool out_f32, hipStream_t st);
 hipError_t tied_prep_launch(const TiedShape& s, const TiedBufs& b, uint32_t pos0, uint32_t M, bool f32, hipStream_t st);
 hipError_t tied_flash_launch(const TiedShape& s, const TiedBufs& b, uint32_t pos0, uint32_t M, bool f32, void* out, uint32_t ldo, hipStream_t st);
+
+// ---- gla.hip: gated linear attention, S_t = diag(alpha_t) S_(t-1) + k_t v_t^T per head, out S_t^T q_t ----
+struct GlaShape {
+  uint32_t heads, dim, vdim, rank;     // rank: inner size of the decay's projection
+  uint32_t lds, ldo;                   // row strides: state [head][dim][lds], outputs before their norm [M][heads][ldo]
+  uint32_t off_q, off_k, off_v, off_g, off_a, ldcat;
+  uint32_t a2_ld;
+  float tau, eps, out_scale;
+};
+struct GlaBufs {
+  const float* cat;                    // [M][ldcat], blocks: + kMlstmRowSlack
+  const uint16_t* a2;                  // [heads * dim][a2_ld]
+  const float *a2b, *norm;             // [heads * dim], [vdim]
+  float* S;
+  float* num;                          // [M][heads][ldo]
+  float* qk;                           // blocks: [Mcap][2 * heads * dim] decayed queries | keys, + kMlstmRowSlack
+  float* dec;                          // blocks: [chunk][heads * dim] a chunk's whole decay, + kMlstmRowSlack
+  float* a;                            // blocks: [chunk][heads][64][64] decayed scores
+  uint32_t Mcap;
+};
+hipError_t gla_step_launch(const GlaShape& s, const GlaBufs& b, const int* pos_ptr, uint32_t pos0, hipStream_t st);
+hipError_t gla_block_launch(const GlaShape& s, const GlaBufs& b, uint32_t pos0, uint32_t M, hipStream_t st);
+// per-head RMS norm, norm weight, silu gate, out_scale -> columns of out
+hipError_t gla_out_launch(const GlaShape& s, const GlaBufs& b, uint32_t M, void* out, uint32_t ldo, bool f32, hipStream_t st);
+
+// ---- gated_attention.hip: grouped heads with values of their own ----
+struct GattnShape {
+  uint32_t heads, kv_heads, dim, vdim, dp, vp;   // dp, vp: row strides of the caches, multiples of 64
+  uint32_t off_q, off_k, off_v, off_g, ldcat;
+  uint32_t chunk;                      // i sees j <= i with j / chunk == i / chunk
+  uint32_t rot_n;                      // leading values of a head that are rotated
+  uint64_t rows;                       // cache rows per key head, multiple of 64
+  float scale, eps, out_scale;
+};
+struct GattnBufs {
+  const float* cat;                    // [M][ldcat]
+  const float *qn, *kn, *cs;           // norm weights [dim]; [max_seq][rot_n / 2][2]
+  void *kc, *vc;                       // [kv_heads][rows][dp | vp]: keys normed and rotated, values
+  void* q;                             // blocks: [heads][Mcap][dp]
+  uint32_t Mcap;
+  float *part_ml, *part_acc;           // [split][M * heads][2], [split][M * heads][vdim]
+};
+constexpr uint32_t kGattnShort = 16, kGattnMaxDim = 512, kGattnFlashDim = 256;
+uint32_t gattn_splits(const GattnShape& s, uint32_t max_seq, uint32_t M, bool f32, uint32_t forced);
+// one token (own = true: its key and value are taken from cat and written to the cache) or M tokens whose rows are in the cache; gla (may be
+// NULL, own only): a step of gated linear attention in the same launch
+hipError_t gattn_attn_launch(const GattnShape& s, const GattnBufs& b, const GlaShape* gs, const GlaBufs* gb, const int* pos_ptr, uint32_t pos0, uint32_t M, bool own,
+                             uint32_t n_splits, bool f32, hipStream_t st);
+// the shares put together, gated -> out; gla: its read-out behind them, from column gla_col on (decode)
+hipError_t gattn_merge_launch(const GattnShape& s, const GattnBufs& b, const GlaShape* gs, const GlaBufs* gb, uint32_t gla_col, const int* pos_ptr, uint32_t pos0,
+                              uint32_t M, uint32_t n_splits, bool f32, void* out, uint32_t ldo, bool out_f32, hipStream_t st);
+hipError_t gattn_prep_launch(const GattnShape& s, const GattnBufs& b, uint32_t pos0, uint32_t M, bool f32, hipStream_t st);
+hipError_t gattn_flash_launch(const GattnShape& s, const GattnBufs& b, uint32_t pos0, uint32_t M, bool f32, void* out, uint32_t ldo, hipStream_t st);
+
+// ---- glru.hip: S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t per channel ----
+struct GlruShape {
+  uint32_t width, blocks, bs, taps;    // bs: channels of a diagonal block
+  uint32_t off_y, off_x, ldcat;
+  uint32_t gate_rows, gate_kp;         // gates [block][gate_rows][gate_kp]: r and i interleaved in blocks of 16 rows
+};
+struct GlruBufs {
+  const float* cat;                    // [M][ldcat]
+  const float *conv, *conv_b;          // [width][taps], [width]
+  const uint16_t* gates;
+  const float *rb, *ib, *lam;          // [width]
+  float* S;                            // [width]
+  float* hist;                         // [taps][width]: the convolution's input at position p lies in row p % taps
+  float *a, *x;                        // blocks: [M][width] factors and inputs of the recurrence
+  float* sum;                          // blocks: [chunk][width][2] a chunk of 64 tokens as one factor and one input
+  float* s0;                           // blocks: [width] state before the block
+};
+hipError_t glru_step_launch(const GlruShape& s, const GlruBufs& b, const int* pos_ptr, float* out, hipStream_t st);
+hipError_t glru_block_launch(const GlruShape& s, const GlruBufs& b, uint32_t pos0, uint32_t M, bool f32, void* out, uint32_t ldo, hipStream_t st);
 
 // ---- latent_attention.hip ----
 struct LatentShape {
@@ -249,6 +359,7 @@ struct MlstmShape {
   uint32_t lds;                // row stride of the state [head][dim][lds]: columns 0..vdim-1 = S, column vdim = n
   uint32_t ldo;                // row stride of the numerators [M][heads][ldo]
   uint32_t off_q, off_k, off_v, off_g, off_i, off_f, ldcat;
+  uint32_t ldqk;               // row stride of the queries and keys of a block (qk)
   float cap, eps;
 };
 struct MlstmBufs {
@@ -262,12 +373,16 @@ struct MlstmBufs {
   float *dec, *wgt, *cdec;     // blocks: factors of the state kernel, [heads][Mcap] and [heads][chunks]
   float* nk;                   // blocks: [chunk][heads][dim]: a chunk's contribution to n, then n before the chunk
   float* a;                    // blocks: [chunk][heads][64][64] decayed scores
+  const float* qk;             // blocks: queries and keys (off_q, off_k; rows of ldqk)
+  const float* rowdec;         // mlstm_state_launch with a decay per state row: [chunk][heads * dim]
   uint32_t Mcap;
 };
 constexpr uint32_t kMlstmBlockDim = 512;      // larger heads take blocks token by token
 constexpr uint32_t kMlstmRowSlack = 2048;   // floats the block kernels may read behind the last row of cat (never used)
 hipError_t mlstm_step_launch(const MlstmShape& s, const MlstmBufs& b, const int* pos_ptr, hipStream_t st, uint32_t pos0 = 0);   // pos_ptr or pos0
 hipError_t mlstm_block_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t pos0, uint32_t M, hipStream_t st);
+// a block's recurrence over its chunks alone; rowdec set: queries and keys carry their decays, every state row has its own decay per chunk
+hipError_t mlstm_state_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t pos0, uint32_t M, hipStream_t st);
 hipError_t mlstm_out_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t M, void* out, uint32_t ldo, bool f32, hipStream_t st);
 
 }  // namespace lgh

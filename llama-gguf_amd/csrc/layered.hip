@@ -6,12 +6,16 @@
 //                      expansion + gate -> output product
 //   mLSTM              fused q | k | v | gates product -> recurrence step -> output product (read-out norm and gate in its prologue)
 //   tied attention     fused q | k product -> split attention (norms of q and k in its prologue, cache row written) -> merge -> output product
+//   gated attention    fused q | k | v | gate product -> split attention (norms and rotation in its prologue, cache rows written) -> merge + gate ->
+//                      output product; a gated linear attention beside it steps and is read out in the same launches, one output product for both
+//   linear recurrence  fused y | x product -> convolution, gates and recurrence step -> output product
 //   feed-forward       gate | up product with gelu * in its epilogue -> down product
 //   mixture            shared gate | up + router product -> the chosen experts' gate | up (every workgroup ranks the scores) -> one down
 //                      product over [shared | experts]
+// With norms in front of the sublayers (LGH_RESIDUAL_PRE_RMS) the prologue of the product that reads the stream updates and norms it.
 // With squashing norms (LGH_RESIDUAL_SANDWICH_DYT) everything between two sublayers is per channel: it rides in the EPILOGUE of the
 // product that finishes a channel, and no norm is computed more than once.
-// A sequence's state: the cache rows, the matrix memories with their running maxima, the convolutions' last inputs, and the last token
+// A sequence's state: the cache rows, the matrix memories with their running maxima, the linear recurrences, the convolutions' last inputs, and the last token
 // (pair embedding), kept as a token history by position; a position of 0 makes every kernel ignore what is stored, so lgh_reset stays O(1).
 #include <algorithm>
 #include <cmath>
@@ -27,6 +31,7 @@ namespace lgh {
 constexpr uint32_t kBlockTokens = 2048;    // tokens per pass of the block path
 constexpr uint32_t kLogitRows = 128;       // wanted rows per output product
 constexpr uint32_t kMaxConvTaps = 64;
+constexpr uint32_t kMaxRecTaps = 64;
 
 struct LayeredLayer {
   lgh_layer_desc d{};
@@ -36,6 +41,14 @@ struct LayeredLayer {
   float *qn = nullptr, *kn = nullptr, *temp = nullptr, *sink = nullptr, *kinv = nullptr;
   uint32_t splits = 1;
   TiedShape ts{};
+  GattnShape gs{};
+  GlaShape as{};
+  GlruShape rs{};
+  LinW a2, gates;                          // linear attention: the decay's second factor; linear recurrence: its gates' diagonal blocks
+  float *in_bias = nullptr, *a2b = nullptr, *gnorm = nullptr, *conv = nullptr, *conv_b = nullptr, *rb = nullptr, *ib = nullptr, *lam = nullptr, *correction = nullptr;
+  float *rS = nullptr, *rhist = nullptr;
+  void* vcache = nullptr;
+  uint32_t gla_col = 0;                    // where the linear attention's values lie in the output product's input
   uint16_t* uk_t = nullptr;
   float *norm1 = nullptr, *norm2 = nullptr, *dkv_norm = nullptr, *mnorm = nullptr, *bi = nullptr, *bf = nullptr, *cs = nullptr;
   void* cache = nullptr;
@@ -46,7 +59,17 @@ struct LayeredLayer {
   bool latent() const { return d.mixer == LGH_MIXER_LATENT_ATTENTION; }
   bool mlstm() const { return d.mixer == LGH_MIXER_MLSTM; }
   bool tied() const { return d.mixer == LGH_MIXER_TIED_ATTENTION; }
+  bool gattn() const { return d.mixer == LGH_MIXER_GATED_ATTENTION || d.mixer == LGH_MIXER_PARALLEL; }
+  bool gla() const { return d.mixer == LGH_MIXER_GLA || d.mixer == LGH_MIXER_PARALLEL; }
+  bool glru() const { return d.mixer == LGH_MIXER_GLRU; }
+  bool rotated() const { return latent() || gattn(); }
   bool moe() const { return d.ff_kind == LGH_FF_MOE; }
+  RouteForm route() const {
+    RouteForm r;
+    r.form = d.router_form;
+    if (r.form == LGH_ROUTER_SOFTMAX_GROUPS) { r.groups = d.groups; r.keep = d.keep_groups; r.identity = d.identity; r.correction = correction; }
+    return r;
+  }
   uint32_t act_cols() const { return moe() ? down.kp + d.top * edown.kp : down.kp; }   // inputs of the down product
 };
 
@@ -61,6 +84,9 @@ struct LayeredSlot {                       // where a named tensor goes
   uint32_t row0 = 0, n = 0, k = 0;
   int mode = 0;
   float** vec = nullptr;
+  uint32_t off = 0, total = 0;             // vec: this tensor's place in a vector of `total` values (0: the tensor is the vector)
+  uint32_t col0 = 0, parts = 1;            // mat: first column; equal parts, each of `stride` rows
+  uint32_t stride = 0;
   uint16_t** raw = nullptr;
   LayeredLayer* transpose = nullptr;
   bool done = false;
@@ -82,15 +108,17 @@ struct LayeredModel {
   LayeredNorm final_dyt;
   float *h = nullptr, *hist = nullptr, *tails = nullptr;   // a sublayer's input (decode); the convolutions' histories and a block's last inputs
   bool dyt() const { return d.residual == LGH_RESIDUAL_SANDWICH_DYT; }
+  bool pre() const { return d.residual == LGH_RESIDUAL_PRE_RMS; }
   size_t hist_floats() const { return d.conv_taps > 1 ? (size_t)n_sub * (d.conv_taps - 1) * d.width : 0; }
   // mixtures
   float* rlogits = nullptr;
   int* sel = nullptr;
+  float* selw = nullptr;
   uint32_t max_experts = 0, max_top = 0, max_pair_act = 0;   // (the last: top * columns of an expert)
   float *bpair = nullptr, *bselw = nullptr, *broww = nullptr;
   int *bsel = nullptr, *bseg = nullptr, *btile_e = nullptr, *btile_row = nullptr, *bslot = nullptr, *bsrc = nullptr;
   void* bpact = nullptr;
-  // tied attention's queries of a block
+  // tied and gated attention's queries of a block
   uint32_t max_tied_q = 0;                 // heads * row
   size_t max_tied_rows = 0, max_tied_acc = 0;   // partial sums: (token, head) rows * splits, and times the head size
   void* btq = nullptr;
@@ -104,6 +132,8 @@ struct LayeredModel {
   float *bx2 = nullptr;                    // LGH_RESIDUAL_SANDWICH_DYT: the stream's second buffer
   float *bx = nullptr, *by = nullptr, *bcat = nullptr, *bnum = nullptr, *ba = nullptr, *blogits = nullptr;
   double *bu = nullptr, *bmx = nullptr;
+  float *brec = nullptr, *brsum = nullptr, *bqk = nullptr, *bgdec = nullptr;   // linear recurrence: factors | inputs, tiles; linear attention
+  uint32_t max_rec = 0, max_gla = 0;       // channels of a recurrence; heads * dim of a linear attention
   float *bdec = nullptr, *bwgt = nullptr, *bcdec = nullptr, *bnk = nullptr;
   void *bxa = nullptr, *bao = nullptr, *bact = nullptr, *bla = nullptr;
   int *btok = nullptr, *brows = nullptr;
@@ -140,20 +170,33 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
   if (d.compute > LGH_COMPUTE_F32) { why = "unknown compute type"; return LGH_INVALID_ARGUMENT; }
   if (!(d.norm_eps >= 0.0) || !std::isfinite(d.residual_mult)) { why = "norm_eps / residual_mult"; return LGH_INVALID_ARGUMENT; }
   if (up(d.width, 64) > 32768) { why = "width above 32768"; return LGH_UNSUPPORTED; }
-  if (d.residual > LGH_RESIDUAL_SANDWICH_DYT) { why = "unknown residual form"; return LGH_UNSUPPORTED; }
+  if (d.tied_head > 1 || !std::isfinite(d.logit_scale)) { why = "output projection"; return LGH_INVALID_ARGUMENT; }
+  if (d.logit_scale != 0.0 && d.logit_scale != 1.0 && d.residual != LGH_RESIDUAL_PRE_RMS) { why = "a factor on the logits"; return LGH_UNSUPPORTED; }
+  if (d.residual > LGH_RESIDUAL_PRE_RMS) { why = "unknown residual form"; return LGH_UNSUPPORTED; }
   if (d.conv_taps > kMaxConvTaps || (d.conv_taps && d.residual != LGH_RESIDUAL_SANDWICH_DYT)) { why = "convolution taps"; return LGH_UNSUPPORTED; }
   for (uint32_t i = 0; i < d.num_layers; i++) {
     const lgh_layer_desc& l = L[i];
     const std::string at = "layer " + std::to_string(i) + ": ";
     if (l.struct_size != sizeof(lgh_layer_desc)) { why = at + "descriptor size"; return LGH_INVALID_ARGUMENT; }
-    if (!l.heads || !l.dim || !l.vdim) { why = at + "a mixer dimension is zero"; return LGH_INVALID_ARGUMENT; }
+    if (l.mixer != LGH_MIXER_GLA && (!l.heads || !l.dim || !l.vdim)) { why = at + "a mixer dimension is zero"; return LGH_INVALID_ARGUMENT; }
     if (l.ff_kind > LGH_FF_MOE || (l.ff_kind && !l.ff)) { why = at + "feed-forward"; return LGH_INVALID_ARGUMENT; }
     if (l.ff_kind == LGH_FF_MOE) {
-      if (!l.experts || !l.top || l.top > l.experts) { why = at + "experts"; return LGH_INVALID_ARGUMENT; }
+      if (l.router_form > LGH_ROUTER_SOFTMAX_GROUPS || l.expert_form > LGH_EXPERT_CLAMPED) { why = at + "router or expert form"; return LGH_UNSUPPORTED; }
+      const bool grp = l.router_form == LGH_ROUTER_SOFTMAX_GROUPS;
+      if (!grp && l.identity) { why = at + "identity experts"; return LGH_UNSUPPORTED; }
+      if (!l.experts || !l.top || l.top > l.experts + l.identity) { why = at + "experts"; return LGH_INVALID_ARGUMENT; }
+      if (grp) {
+        const uint32_t n = l.experts + l.identity;
+        if (n > kMaxRouted) { why = at + "more than " + std::to_string(kMaxRouted) + " router outputs"; return LGH_UNSUPPORTED; }
+        if (!l.groups || n % l.groups || !l.keep_groups || l.keep_groups > l.groups || l.keep_groups * (n / l.groups) < l.top) { why = at + "groups of experts"; return LGH_INVALID_ARGUMENT; }
+        if (l.identity && d.residual != LGH_RESIDUAL_PRE_RMS) { why = at + "identity experts need a norm in front of the sublayer"; return LGH_UNSUPPORTED; }
+        if (l.expert_form != LGH_EXPERT_CLAMPED || l.shared_ff) { why = at + "softmax routing takes clamped experts, none of them shared"; return LGH_UNSUPPORTED; }
+      } else if (l.expert_form != LGH_EXPERT_SWIGLU) { why = at + "clamped experts take softmax routing"; return LGH_UNSUPPORTED; }
       if (l.experts > kMaxExperts || l.top > kMaxTop) { why = at + "more than " + std::to_string(kMaxExperts) + " experts or " + std::to_string(kMaxTop) + " per token"; return LGH_UNSUPPORTED; }
       if ((uint64_t)up(l.shared_ff, 64) + (uint64_t)l.top * up(l.ff, 64) > kLinMvMaxK) { why = at + "a token's experts together above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
     } else if (l.ff_kind && up(l.ff, 64) > kLinMvMaxK) { why = at + "feed-forward above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
-    if (up(l.heads * l.vdim, 64) > kLinMvMaxK) { why = at + "heads * vdim above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
+    const bool ga = l.mixer == LGH_MIXER_GATED_ATTENTION || l.mixer == LGH_MIXER_PARALLEL, la = l.mixer == LGH_MIXER_GLA || l.mixer == LGH_MIXER_PARALLEL;
+    if ((uint64_t)(l.mixer == LGH_MIXER_GLA ? 0 : up(l.heads * l.vdim, 64)) + (la ? up(l.gla_heads * l.gla_vdim, 64) : 0) > kLinMvMaxK) { why = at + "heads * vdim above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
     if (l.mixer == LGH_MIXER_LATENT_ATTENTION) {
       if (!l.kv_rank || l.rot_dims > l.rot_dim || l.rot_dims % 2) { why = at + "latent attention sizes"; return LGH_INVALID_ARGUMENT; }
       if (l.rot_dims && !(l.rot_base > 0.0)) { why = at + "rotation base"; return LGH_INVALID_ARGUMENT; }
@@ -164,6 +207,16 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
     } else if (l.mixer == LGH_MIXER_TIED_ATTENTION) {
       if (!l.kv_heads || l.heads % l.kv_heads || l.vdim != l.dim || !(l.score_cap >= 0.0)) { why = at + "tied attention sizes"; return LGH_INVALID_ARGUMENT; }
       if (up(l.dim, 64) > kTiedMaxDim) { why = at + "heads above " + std::to_string(kTiedMaxDim); return LGH_UNSUPPORTED; }
+    } else if (ga || la) {
+      if (ga) {
+        if (!l.kv_heads || l.heads % l.kv_heads || l.rot_dims > l.dim || l.rot_dims % 2 || (l.rot_dims && !(l.rot_base > 0.0))) { why = at + "gated attention sizes"; return LGH_INVALID_ARGUMENT; }
+        if (up(l.dim, 64) > kGattnMaxDim || up(l.vdim, 64) > kGattnMaxDim) { why = at + "heads above " + std::to_string(kGattnMaxDim); return LGH_UNSUPPORTED; }
+      }
+      if (la && (!l.gla_heads || !l.gla_dim || !l.gla_vdim || !l.gla_rank || !(l.gla_tau > 0.0))) { why = at + "linear attention sizes"; return LGH_INVALID_ARGUMENT; }
+      if (!std::isfinite(l.left_scale) || !std::isfinite(l.right_scale)) { why = at + "scales of the two sides"; return LGH_INVALID_ARGUMENT; }
+    } else if (l.mixer == LGH_MIXER_GLRU) {
+      if (l.vdim != l.dim || !l.taps) { why = at + "linear recurrence sizes"; return LGH_INVALID_ARGUMENT; }
+      if (l.taps > kMaxRecTaps) { why = at + "convolution taps"; return LGH_UNSUPPORTED; }
     } else if (l.mixer == LGH_MIXER_MLSTM) {
       if (!(l.gate_cap > 0.0)) { why = at + "gate_cap"; return LGH_INVALID_ARGUMENT; }
     } else { why = at + "unknown mixer"; return LGH_UNSUPPORTED; }
@@ -187,6 +240,12 @@ static void add_vec(LayeredModel& m, const std::string& nm, float** v, uint32_t 
   LayeredSlot s;
   s.vec = v; s.n = n;
   m.slots[nm] = s;
+}
+// part of a fused product's bias, at its rows
+static void add_bias(LayeredModel& m, const std::string& nm, float** v, uint32_t off, uint32_t n, uint32_t total) {
+  add_vec(m, nm, v, n);
+  m.slots[nm].off = off;
+  m.slots[nm].total = total;
 }
 
 // a norm of LGH_RESIDUAL_SANDWICH_DYT: weight, bias and the factor inside
@@ -213,7 +272,7 @@ static void layered_plan(LayeredModel& m) {
   {
     LayeredSlot s;
     s.raw = &m.embed; s.n = d.vocab_size; s.k = W;
-    m.slots["embed"] = s;
+    if (!d.tied_head) m.slots["embed"] = s;
     if (d.bigram_buckets) { s.raw = &m.bigram; s.n = d.bigram_buckets + 1; m.slots["bigram"] = s; }
   }
   auto whole = [&](LinW& L, uint32_t n, uint32_t k) { L.n = n; L.k = k; L.kp = up(k, 64); };
@@ -224,7 +283,7 @@ static void layered_plan(LayeredModel& m) {
     const std::string p = "l" + std::to_string(i) + ".";
     add_sub(m, p, "1", &L.norm1);
     L.in.k = W; L.in.kp = up(W, 64);
-    const uint32_t vd = l.heads * l.vdim;
+    const uint32_t vd = l.mixer == LGH_MIXER_GLA ? 0 : l.heads * l.vdim;
     auto in_seg = [&](const char* nm, uint32_t rows) { const uint32_t at = seg(L.in, rows); add_mat(m, p + "mix." + nm, &L.in, at, rows, W); return at; };
     if (L.latent()) {
       LatentShape& s = L.ls;
@@ -265,6 +324,88 @@ static void layered_plan(LayeredModel& m) {
         m.max_tied_acc = std::max(m.max_tied_acc, rows * l.dim);
       }
       m.max_tied_q = std::max(m.max_tied_q, l.heads * s.dp);
+    } else if (L.glru()) {
+      GlruShape& s = L.rs;
+      s.width = vd; s.blocks = l.heads; s.bs = l.dim; s.taps = l.taps;
+      s.off_y = in_seg("y", vd);
+      s.off_x = in_seg("x", vd);
+      L.in.n = up(L.in.n, 16);
+      s.ldcat = L.in.n;
+      add_bias(m, p + "mix.y.b", &L.in_bias, s.off_y, vd, L.in.n);
+      add_bias(m, p + "mix.x.b", &L.in_bias, s.off_x, vd, L.in.n);
+      add_vec(m, p + "mix.conv", &L.conv, vd * l.taps);
+      add_vec(m, p + "mix.conv.b", &L.conv_b, vd);
+      s.gate_rows = 2 * up(l.dim, 16);
+      whole(L.gates, l.heads * s.gate_rows, l.dim);
+      s.gate_kp = L.gates.kp;
+      for (int i = 0; i < 2; i++) {
+        const std::string nm = p + (i ? "mix.ri" : "mix.ra");
+        add_mat(m, nm, &L.gates, 0, vd, l.dim, 1 + i);
+        m.slots[nm].parts = l.heads;
+        m.slots[nm].stride = s.gate_rows;
+        add_vec(m, nm + ".b", i ? &L.ib : &L.rb, vd);
+      }
+      add_vec(m, p + "mix.lam", &L.lam, vd);
+      m.recurrent = true;
+      m.max_rec = std::max(m.max_rec, vd);
+    } else if (L.gattn() || L.gla()) {
+      const bool par = l.mixer == LGH_MIXER_PARALLEL;
+      const std::string left = par ? "left." : "", right = par ? "right." : "", pl = p + "mix." + left, pr = p + "mix." + right;
+      if (L.gattn()) {
+        GattnShape& s = L.gs;
+        s.heads = l.heads; s.kv_heads = l.kv_heads; s.dim = l.dim; s.vdim = l.vdim; s.dp = up(l.dim, 64); s.vp = up(l.vdim, 64);
+        s.chunk = l.chunk ? l.chunk : 0xFFFFFFFFu; s.rot_n = l.rot_dims;
+        s.rows = up(d.max_seq_len, 64);
+        s.scale = (float)l.scale; s.eps = (float)d.norm_eps; s.out_scale = par ? (float)l.left_scale : 1.0f;
+        s.off_q = in_seg((left + "q").c_str(), l.heads * l.dim);
+        s.off_k = in_seg((left + "k").c_str(), l.kv_heads * l.dim);
+        s.off_v = in_seg((left + "v").c_str(), l.kv_heads * l.vdim);
+        s.off_g = in_seg((left + "g").c_str(), vd);
+        add_vec(m, pl + "q.norm", &L.qn, l.dim);
+        add_vec(m, pl + "k.norm", &L.kn, l.dim);
+        L.splits = gattn_splits(s, d.max_seq_len, 1, m.f32, m.forced_splits);
+        for (uint32_t t = 1; t <= kGattnShort; t++) {
+          const size_t rows = (size_t)t * l.heads * gattn_splits(s, d.max_seq_len, t, m.f32, m.forced_splits);
+          m.max_tied_rows = std::max(m.max_tied_rows, rows);
+          m.max_tied_acc = std::max(m.max_tied_acc, rows * l.vdim);
+        }
+        if (s.dp <= kGattnFlashDim) m.max_tied_q = std::max(m.max_tied_q, l.heads * s.dp);
+      }
+      if (L.gla()) {
+        GlaShape& s = L.as;
+        s.heads = l.gla_heads; s.dim = l.gla_dim; s.vdim = l.gla_vdim; s.rank = l.gla_rank;
+        s.lds = up(s.vdim, 16); s.ldo = up(s.vdim, 4);
+        s.tau = (float)l.gla_tau; s.eps = (float)d.norm_eps; s.out_scale = par ? (float)l.right_scale : 1.0f;
+        s.off_q = in_seg((right + "q").c_str(), s.heads * s.dim);
+        s.off_k = in_seg((right + "k").c_str(), s.heads * s.dim);
+        s.off_v = in_seg((right + "v").c_str(), s.heads * s.vdim);
+        s.off_g = in_seg((right + "g").c_str(), s.heads * s.vdim);
+        s.off_a = in_seg((right + "a1").c_str(), s.rank);
+        whole(L.a2, s.heads * s.dim, s.rank);
+        s.a2_ld = L.a2.kp;
+        add_mat(m, pr + "a2", &L.a2, 0, L.a2.n, s.rank);
+        add_vec(m, pr + "a2.b", &L.a2b, L.a2.n);
+        add_vec(m, pr + "norm", &L.gnorm, s.vdim);
+        m.recurrent = true;
+        m.max_num = std::max(m.max_num, s.heads * s.ldo);
+        m.max_gla = std::max(m.max_gla, s.heads * s.dim);
+      }
+      L.in.n = up(L.in.n, 16);
+      L.gs.ldcat = L.as.ldcat = L.in.n;
+      if (L.gattn()) {
+        add_bias(m, pl + "q.b", &L.in_bias, L.gs.off_q, l.heads * l.dim, L.in.n);
+        add_bias(m, pl + "k.b", &L.in_bias, L.gs.off_k, l.kv_heads * l.dim, L.in.n);
+        add_bias(m, pl + "v.b", &L.in_bias, L.gs.off_v, l.kv_heads * l.vdim, L.in.n);
+      }
+      // both sides' output projections side by side: one product
+      L.gla_col = up(vd, 64);
+      const uint32_t cols = L.gla() ? L.gla_col + L.as.heads * L.as.vdim : vd;
+      whole(L.out, W, cols);
+      if (L.gattn()) add_mat(m, pl + "o", &L.out, 0, W, vd);
+      if (L.gla()) {
+        add_mat(m, pr + "o", &L.out, 0, W, L.as.heads * L.as.vdim);
+        m.slots[pr + "o"].col0 = L.gla_col;
+      }
     } else {
       MlstmShape& s = L.ms;
       s.heads = l.heads; s.dim = l.dim; s.vdim = l.vdim;
@@ -277,7 +418,7 @@ static void layered_plan(LayeredModel& m) {
       s.off_i = in_seg("i", l.heads);
       s.off_f = in_seg("f", l.heads);
       L.in.n = up(L.in.n, 16);
-      s.ldcat = L.in.n;
+      s.ldcat = s.ldqk = L.in.n;
       add_vec(m, p + "mix.i.b", &L.bi, l.heads);
       add_vec(m, p + "mix.f.b", &L.bf, l.heads);
       add_vec(m, p + "mix.norm", &L.mnorm, vd);
@@ -285,13 +426,16 @@ static void layered_plan(LayeredModel& m) {
       m.max_num = std::max(m.max_num, l.heads * s.ldo);
     }
     m.max_cat = std::max(m.max_cat, L.in.n);
-    whole(L.out, W, vd);
-    add_mat(m, p + "mix.o", &L.out, 0, W, vd);
+    if (!L.out.n) {
+      whole(L.out, W, vd);
+      add_mat(m, p + "mix.o", &L.out, 0, W, vd);
+    }
     m.max_ao = std::max(m.max_ao, L.out.kp);
     if (L.moe()) {
       add_sub(m, p, "2", &L.norm2);
-      whole(L.router, l.experts, W);
-      add_mat(m, p + "mlp.router", &L.router, 0, l.experts, W);
+      whole(L.router, l.experts + l.identity, W);
+      add_mat(m, p + "mlp.router", &L.router, 0, L.router.n, W);
+      if (l.router_form == LGH_ROUTER_SOFTMAX_GROUPS) add_vec(m, p + "mlp.correction", &L.correction, L.router.n);
       L.egu_rows = 2 * up(l.ff, 16);
       L.edown_rows = up(W, 16);
       whole(L.egu, l.experts * L.egu_rows, W);
@@ -312,7 +456,7 @@ static void layered_plan(LayeredModel& m) {
         add_mat(m, p + "mlp.shared.down", &L.down, 0, W, l.shared_ff);
       }
       m.max_act = std::max(m.max_act, L.act_cols());
-      m.max_experts = std::max(m.max_experts, l.experts);
+      m.max_experts = std::max(m.max_experts, l.experts + l.identity);
       m.max_top = std::max(m.max_top, l.top);
       m.max_pair_act = std::max(m.max_pair_act, l.top * L.edown.kp);
     } else if (l.ff_kind) {
@@ -329,7 +473,7 @@ static void layered_plan(LayeredModel& m) {
   if (m.dyt()) add_dyt(m, "final.norm", m.final_dyt);
   else add_vec(m, "final.norm", &m.final_norm, W);
   whole(m.head, d.vocab_size, W);
-  add_mat(m, "head", &m.head, 0, d.vocab_size, W);
+  add_mat(m, d.tied_head ? "embed" : "head", &m.head, 0, d.vocab_size, W);
 }
 
 extern "C" int lgh_create_layered(const lgh_layered_desc* desc, const lgh_layer_desc* layers, lgh_ctx** out) {
@@ -382,12 +526,18 @@ int layered_upload(lgh_ctx* c, const char* name, uint32_t type, const uint64_t n
   int rc;
   if (s.vec) {
     if (n0 * n1 * n2 != s.n) return fail(c, LGH_SHAPE_MISMATCH, nm + ": expected " + std::to_string(s.n) + " elements");
-    if ((rc = upload_f32(c, s.vec, (int)type, s.n, host, nbytes))) return rc;
+    if (s.total) {                           // a part of a vector that several tensors share
+      if (!*s.vec && (rc = zeroed(c, (void**)s.vec, (size_t)s.total * 4, nullptr))) return rc;
+      L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
+      float* at = *s.vec + s.off;
+      if ((rc = upload_f32(c, &at, (int)type, s.n, host, nbytes))) return rc;
+      c->stats.weight_bytes += s.done ? 0 : (uint64_t)s.n * 4;
+    } else if ((rc = upload_f32(c, s.vec, (int)type, s.n, host, nbytes))) return rc;
     s.done = true;
     return LGH_OK;
   }
   if (type != LGH_TYPE_BF16) return fail(c, LGH_DTYPE_MISMATCH, nm + ": matrices of this model are bf16");
-  if (n0 != s.k || n1 != s.n || n2 != 1) return fail(c, LGH_SHAPE_MISMATCH, nm + ": expected [" + std::to_string(s.k) + "," + std::to_string(s.n) + "]");
+  if (n0 != s.k || n1 != s.n / s.parts || n2 != s.parts) return fail(c, LGH_SHAPE_MISMATCH, nm + ": expected [" + std::to_string(s.k) + "," + std::to_string(s.n) + "]");
   if (nbytes != (size_t)s.n * s.k * 2) return fail(c, LGH_SHAPE_MISMATCH, nm + ": byte size does not match its shape");
   if (s.raw) {
     if (!*s.raw && (rc = dev_alloc(c, (void**)s.raw, nbytes))) return rc;
@@ -401,7 +551,8 @@ int layered_upload(lgh_ctx* c, const char* name, uint32_t type, const uint64_t n
   void* raw = nullptr;
   L_TRY(c, LGH_ALLOCATION_FAILED, hipMalloc(&raw, nbytes));
   hipError_t e = hipMemcpy(raw, host, nbytes, hipMemcpyHostToDevice);
-  if (e == hipSuccess) e = lin_pack_launch((const uint16_t*)raw, s.n, s.k, W.w, W.kp, s.row0, s.mode, c->stream);
+  for (uint32_t i = 0; i < s.parts && e == hipSuccess; i++)
+    e = lin_pack_launch((const uint16_t*)raw + (size_t)i * (s.n / s.parts) * s.k, s.n / s.parts, s.k, W.w + s.col0, W.kp, s.row0 + i * s.stride, s.mode, c->stream);
   if (e == hipSuccess && s.transpose) {
     LayeredLayer& L = *s.transpose;
     const size_t tb = (size_t)L.ls.heads * L.ls.rank * L.ls.dimp * 2;
@@ -451,11 +602,10 @@ int layered_finalize(lgh_ctx* c) {
   uint32_t max_rows = 0, max_rank = 0, max_ldc = 0;
   for (uint32_t i = 0; i < d.num_layers; i++) {
     LayeredLayer& L = m.layers[i];
-    if (L.latent()) {
-      if ((rc = zeroed(c, &L.cache, (size_t)d.max_seq_len * L.ls.ldc * m.el(), &c->stats.kv_bytes))) return rc;
+    if (L.rotated()) {
       for (uint32_t j = 0; j < i && !L.cs; j++) {   // layers with the same rotation share its table
         const lgh_layer_desc &a = L.d, &b = m.layers[j].d;
-        if (m.layers[j].latent() && a.rot_dims == b.rot_dims && a.rot_base == b.rot_base && a.yarn_factor == b.yarn_factor &&
+        if (m.layers[j].rotated() && a.rot_dims == b.rot_dims && a.rot_base == b.rot_base && a.yarn_factor == b.yarn_factor &&
             a.yarn_original == b.yarn_original && a.yarn_fast == b.yarn_fast && a.yarn_slow == b.yarn_slow)
           L.cs = m.layers[j].cs;
       }
@@ -465,10 +615,22 @@ int layered_finalize(lgh_ctx* c) {
         L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
         if (!cs.empty()) L_TRY(c, LGH_OPERATION_FAILED, hipMemcpy(L.cs, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
       }
+    }
+    if (L.latent()) {
+      if ((rc = zeroed(c, &L.cache, (size_t)d.max_seq_len * L.ls.ldc * m.el(), &c->stats.kv_bytes))) return rc;
       max_rows = std::max(max_rows, L.ls.heads); max_rank = std::max(max_rank, L.ls.rank); max_ldc = std::max(max_ldc, L.ls.ldc);
     } else if (L.tied()) {
       if ((rc = zeroed(c, &L.cache, (size_t)L.ts.kv_heads * L.ts.rows * L.ts.dp * m.el(), &c->stats.kv_bytes))) return rc;
       if ((rc = zeroed(c, (void**)&L.kinv, (size_t)L.ts.rows * 4, &c->stats.kv_bytes))) return rc;
+    } else if (L.glru()) {
+      if ((rc = zeroed(c, (void**)&L.rS, (size_t)L.rs.width * 4, &c->stats.kv_bytes))) return rc;
+      if ((rc = zeroed(c, (void**)&L.rhist, (size_t)L.rs.taps * L.rs.width * 4, &c->stats.kv_bytes))) return rc;
+    } else if (L.gattn() || L.gla()) {
+      if (L.gattn()) {
+        if ((rc = zeroed(c, &L.cache, (size_t)L.gs.kv_heads * L.gs.rows * L.gs.dp * m.el(), &c->stats.kv_bytes))) return rc;
+        if ((rc = zeroed(c, &L.vcache, (size_t)L.gs.kv_heads * L.gs.rows * L.gs.vp * m.el(), &c->stats.kv_bytes))) return rc;
+      }
+      if (L.gla() && (rc = zeroed(c, (void**)&L.S, (size_t)L.as.heads * L.as.dim * L.as.lds * 4, &c->stats.kv_bytes))) return rc;
     } else {
       if ((rc = zeroed(c, (void**)&L.S, (size_t)L.ms.heads * L.ms.dim * L.ms.lds * 4, &c->stats.kv_bytes))) return rc;
       if ((rc = zeroed(c, (void**)&L.m, (size_t)2 * L.ms.heads * 8, &c->stats.kv_bytes))) return rc;
@@ -486,7 +648,8 @@ int layered_finalize(lgh_ctx* c) {
       {(void**)&m.cat, (size_t)m.max_cat * 4}, {(void**)&m.ao, (size_t)m.max_ao * 4}, {(void**)&m.act, (size_t)m.max_act * 4},
       {(void**)&m.num, (size_t)m.max_num * 4}, {(void**)&m.qa, rows * max_ldc * m.el()},
       {(void**)&m.part_ml, std::max(rows * m.n_splits, m.max_tied_rows) * 2 * 4}, {(void**)&m.part_acc, std::max(rows * m.n_splits * max_rank, m.max_tied_acc) * 4},
-      {(void**)&m.tokens, (size_t)d.max_seq_len * 4}, {(void**)&m.h, m.dyt() ? (size_t)up(d.width, 16) * 4 : 0}, {(void**)&m.hist, m.hist_floats() * 4},
+      {(void**)&m.selw, (size_t)m.max_top * 4},
+      {(void**)&m.tokens, (size_t)d.max_seq_len * 4}, {(void**)&m.h, m.dyt() || m.pre() ? (size_t)up(d.width, 16) * 4 : 0}, {(void**)&m.hist, m.hist_floats() * 4},
       {(void**)&m.rlogits, (size_t)m.max_experts * 4}, {(void**)&m.sel, (size_t)m.max_top * 4}, {(void**)&c->logits, (size_t)d.vocab_size * 4}, {(void**)&c->state, ST_WORDS * 4},
       {(void**)&c->amax_v, 64 * 4}, {(void**)&c->amax_i, 64 * 4}, {(void**)&c->tok_log, (size_t)d.max_seq_len * 4},
   };
@@ -500,7 +663,7 @@ int layered_finalize(lgh_ctx* c) {
 
 static EmbedArgs embed_args(const LayeredModel& m) {
   EmbedArgs a{};
-  a.embed = m.embed; a.bigram = m.bigram; a.width = m.d.width; a.buckets = m.d.bigram_buckets;
+  a.embed = m.d.tied_head ? m.head.w : m.embed; a.ld = m.d.tied_head ? m.head.kp : m.d.width; a.bigram = m.bigram; a.width = m.d.width; a.buckets = m.d.bigram_buckets;
   a.mul_prev = m.d.bigram_mul_prev; a.mul_cur = m.d.bigram_mul_cur; a.hist = m.tokens;
   return a;
 }
@@ -515,6 +678,25 @@ static MlstmBufs mlstm_bufs(const LayeredModel& m, const LayeredLayer& L, const 
   MlstmBufs b{};
   b.cat = cat; b.bi = L.bi; b.bf = L.bf; b.norm = L.mnorm; b.S = L.S; b.m = L.m; b.num = num;
   b.u = m.bu; b.mx = m.bmx; b.dec = m.bdec; b.wgt = m.bwgt; b.cdec = m.bcdec; b.a = m.ba; b.nk = m.bnk; b.Mcap = up(m.blk, 64);
+  b.qk = cat;
+  return b;
+}
+static GattnBufs gattn_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat) {
+  GattnBufs b{};
+  b.cat = cat; b.qn = L.qn; b.kn = L.kn; b.cs = L.cs; b.kc = L.cache; b.vc = L.vcache;
+  b.part_ml = m.part_ml; b.part_acc = m.part_acc;
+  return b;
+}
+static GlaBufs gla_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat, float* num) {
+  GlaBufs b{};
+  b.cat = cat; b.a2 = L.a2.w; b.a2b = L.a2b; b.norm = L.gnorm; b.S = L.S; b.num = num;
+  b.qk = m.bqk; b.dec = m.bgdec; b.a = m.ba; b.Mcap = up(m.blk, 64);
+  return b;
+}
+static GlruBufs glru_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat) {
+  GlruBufs b{};
+  b.cat = cat; b.conv = L.conv; b.conv_b = L.conv_b; b.gates = L.gates.w; b.rb = L.rb; b.ib = L.ib; b.lam = L.lam; b.S = L.rS; b.hist = L.rhist;
+  b.a = m.brec; b.x = m.brec ? m.brec + (size_t)m.blk * m.max_rec : nullptr; b.sum = m.brsum; b.s0 = m.brsum ? m.brsum + (size_t)((m.blk + 63) / 64) * m.max_rec * 2 : nullptr;
   return b;
 }
 
@@ -554,6 +736,13 @@ static uint64_t mixer_bytes(const lgh_ctx* c, const LayeredLayer& L) {
     const uint64_t p = c->pos + 1, w = std::min<uint64_t>(p, L.ts.window), n = w + std::min<uint64_t>(L.ts.keep, p - w);
     return n * ((uint64_t)L.ts.kv_heads * L.ts.dim * c->lm->el() + 4);
   }
+  if (L.glru()) return L.gates.bytes() + (uint64_t)L.rs.width * (L.rs.taps * 2 + 7) * 4;
+  if (L.gattn() || L.gla()) {
+    uint64_t b = 0;
+    if (L.gattn()) b += (uint64_t)(c->pos + 1 - c->pos / L.gs.chunk * L.gs.chunk) * L.gs.kv_heads * (L.gs.dim + L.gs.vdim) * c->lm->el();
+    if (L.gla()) b += (uint64_t)L.as.heads * L.as.dim * L.as.vdim * 8 + L.a2.bytes();
+    return b;
+  }
   if (L.latent()) return (uint64_t)(c->pos + 1) * (L.ls.rank + L.ls.rot_dim) * c->lm->el();
   return (uint64_t)L.ms.heads * L.ms.dim * (L.ms.vdim + 1) * 8;   // state read and written
 }
@@ -570,7 +759,7 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
     return rc;
   uint32_t cur = 0;
   int sub = 0;
-  const float* pend = nullptr;   // norm weight of the sublayer output waiting in m.y
+  const float* pend = nullptr;   // norm weight of the sublayer output waiting in m.y (LGH_RESIDUAL_PRE_RMS: any)
   auto mv = [&](int cls, const LinW& W, float* out, LinMv a, int pro) {
     a.w = W.w; a.n = W.n; a.kp = W.kp; a.k = W.k; a.paired = W.paired; a.out = out;
     return run_k(c, cls, LGH_SYM_LINEAR, W.bytes(), [&] { return lin_mv_launch(pro, a, st); });
@@ -580,9 +769,19 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
     else pend = norm;
     return mv(cls, W, m.y, a, pro);
   };
-  auto read = [&](LinMv& a, const float* nw2 = nullptr) -> int {   // a product's input: the residual stream, or what was made of it
+  // a product's input: the residual stream, or what was made of it.  pre: the sublayer's norm in front (LGH_RESIDUAL_PRE_RMS); nw2: the final norm
+  auto read = [&](LinMv& a, const float* pre, const float* nw2 = nullptr) -> int {
     a.x = m.dyt() ? m.h : m.x[cur];
     int pro = LP_COPY;
+    if (m.pre()) {
+      a.nw2 = nw2 ? nw2 : pre; a.eps = (float)m.d.norm_eps; a.mult = (float)m.d.residual_mult; a.in_scale = nw2 && m.d.logit_scale != 0.0 ? (float)m.d.logit_scale : 1.0f;
+      if (pend) {
+        a.y = m.y; a.xout = m.x[cur ^ 1];
+        cur ^= 1;
+        pend = nullptr;
+      }
+      return LP_PRE;
+    }
     if (pend) {
       a.y = m.y; a.nw = pend; a.nw2 = nw2; a.xout = m.x[cur ^ 1]; a.eps = (float)m.d.norm_eps; a.mult = (float)m.d.residual_mult;
       pro = nw2 ? LP_HEAD : LP_RESID;
@@ -591,13 +790,14 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
     }
     return pro;
   };
-  auto mv_x = [&](int cls, const LinW& W, float* out, const float* nw2 = nullptr) {
+  auto mv_x = [&](int cls, const LinW& W, float* out, const float* pre, const float* nw2 = nullptr, const float* bias = nullptr) {
     LinMv a{};
-    const int pro = read(a, nw2);
+    a.bias = bias;
+    const int pro = read(a, pre, nw2);
     return mv(cls, W, out, a, pro);
   };
   for (LayeredLayer& L : m.layers) {
-    if ((rc = mv_x(LGH_K_QKV, L.in, m.cat))) return rc;
+    if ((rc = mv_x(LGH_K_QKV, L.in, m.cat, L.norm1, nullptr, L.in_bias))) return rc;
     if (L.latent()) {
       const LatentBufs b = latent_bufs(m, L, m.cat);
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, (uint64_t)L.ls.heads * L.ls.rank * L.ls.dim * 2, [&] { return latent_prep_launch(L.ls, b, pos, 0, 1, m.f32, st); }))) return rc;
@@ -616,6 +816,29 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
       LinMv a{};
       a.x = m.ao;
       if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
+    } else if (L.glru()) {
+      const GlruBufs b = glru_bufs(m, L, m.cat);
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GLRU, mixer_bytes(c, L), [&] { return glru_step_launch(L.rs, b, pos, m.ao, st); }))) return rc;
+      LinMv a{};
+      a.x = m.ao;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
+    } else if (L.gattn() || L.gla()) {
+      const GattnBufs b = gattn_bufs(m, L, m.cat);
+      const GlaBufs g = gla_bufs(m, L, m.cat, m.num);
+      const GlaShape* as = L.gla() ? &L.as : nullptr;
+      if (L.gattn()) {
+        if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GATTN, mixer_bytes(c, L), [&] { return gattn_attn_launch(L.gs, b, as, &g, pos, 0, 1, true, L.splits, m.f32, st); }))) return rc;
+        if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_GATTN, 0, [&] {
+               return gattn_merge_launch(L.gs, b, as, &g, L.gla_col, pos, 0, 1, L.splits, m.f32, m.ao, 0, true, st);
+             })))
+          return rc;
+      } else {
+        if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GLA, mixer_bytes(c, L), [&] { return gla_step_launch(L.as, g, pos, 0, st); }))) return rc;
+        if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_GLA, 0, [&] { return gla_out_launch(L.as, g, 1, m.ao, L.out.kp, true, st); }))) return rc;
+      }
+      LinMv a{};
+      a.x = m.ao;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
     } else {
       const MlstmBufs b = mlstm_bufs(m, L, m.cat, m.num);
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_MLSTM, mixer_bytes(c, L), [&] { return mlstm_step_launch(L.ms, b, pos, st); }))) return rc;
@@ -624,35 +847,41 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
       if ((rc = mv_end(LGH_K_WO, L.out, a, LP_MLSTM, L.norm1))) return rc;
     }
     if (L.moe()) {
+      const RouteForm route = L.route();
       LinMv a{};                           // shared gate | up (when there is one) and the router
-      const int pro = read(a);
+      const int pro = read(a, L.norm2);
+      if (m.pre()) a.hout = m.h;
       a.w = L.gu.w; a.n = L.gu.n; a.paired = L.gu.paired; a.kp = L.router.kp; a.k = L.router.k; a.act = LA_SILU; a.out = m.act;
       a.w2 = L.router.w; a.n2 = L.router.n; a.out2 = m.rlogits;
       if ((rc = run_k(c, LGH_K_GATEUP, LGH_SYM_LINEAR, L.gu.bytes() + L.router.bytes(), [&] { return lin_mv_launch(pro, a, st, LS_TWO); }))) return rc;
       LinMv e{};                           // the chosen experts' gate | up
-      e.x = m.dyt() ? m.h : m.x[cur];
-      e.w2 = L.egu.w; e.n = L.egu_rows; e.paired = 1; e.kp = L.egu.kp; e.k = L.egu.k; e.act = LA_SILU; e.out = m.act + L.down.kp;
+      e.x = m.dyt() || m.pre() ? m.h : m.x[cur];
+      e.w2 = L.egu.w; e.n = L.egu_rows; e.paired = 1; e.kp = L.egu.kp; e.k = L.egu.k; e.act = L.d.expert_form == LGH_EXPERT_CLAMPED ? LA_CLAMPED : LA_SILU; e.limit = (float)L.d.expert_limit; e.out = m.act + L.down.kp;
+      e.route = route; e.selw = m.selw;
       e.logits = m.rlogits; e.experts = L.d.experts; e.top = L.d.top; e.sel = m.sel; e.stride = (uint64_t)L.egu_rows * L.egu.kp; e.kpe = L.edown.kp;
       if ((rc = run_k(c, LGH_K_EXPERTS, LGH_SYM_LINEAR, L.egu.bytes() / L.d.experts * L.d.top, [&] { return lin_mv_launch(LP_COPY, e, st, LS_EXPERTS); }))) return rc;
       LinMv o{};
       o.x = m.act; o.w = L.down.w; o.n = m.d.width; o.kp = o.k = L.act_cols(); o.kps = L.down.kp; o.out = m.y;
+      o.experts = L.d.experts; o.selw = m.selw; o.id_x = route.identity ? m.h : nullptr;
       o.w2 = L.edown.w; o.top = L.d.top; o.sel = m.sel; o.stride = (uint64_t)L.edown_rows * L.edown.kp; o.kpe = L.edown.kp;
       if (m.dyt()) o.post = post_update(c, sub++);
       else pend = L.norm2;
       if ((rc = run_k(c, LGH_K_DOWN, LGH_SYM_LINEAR, L.down.bytes() + L.edown.bytes() / L.d.experts * L.d.top, [&] { return lin_mv_launch(LP_COPY, o, st, LS_MOE_DOWN); }))) return rc;
     } else if (L.d.ff_kind) {
-      if ((rc = mv_x(LGH_K_GATEUP, L.gu, m.act))) return rc;
+      if ((rc = mv_x(LGH_K_GATEUP, L.gu, m.act, L.norm2))) return rc;
       LinMv a{};
       a.x = m.act;
       if ((rc = mv_end(LGH_K_DOWN, L.down, a, LP_COPY, L.norm2))) return rc;
     }
   }
   if (mode == MODE_PREFILL && m.dyt()) return LGH_OK;
+  if (mode == MODE_PREFILL && m.pre())
+    return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] { return resid_add_launch(m.x[cur], m.y, (float)m.d.residual_mult, m.d.width, m.x[cur ^ 1], st); });
   if (mode == MODE_PREFILL)
     return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
       return resid_norm_out_launch(m.x[cur], m.y, pend, (float)m.d.norm_eps, (float)m.d.residual_mult, m.d.width, m.x[cur ^ 1], st);
     });
-  if ((rc = mv_x(LGH_K_OUTPUT, m.head, c->logits, m.final_norm))) return rc;
+  if ((rc = mv_x(LGH_K_OUTPUT, m.head, c->logits, nullptr, m.final_norm))) return rc;
   if (mode == MODE_GREEDY)
     return run_k(c, LGH_K_ARGMAX, LGH_SYM_ARGMAX, (uint64_t)m.d.vocab_size * 4, [&] {
       return argmax_launch(c->logits, m.d.vocab_size, c->amax_v, c->amax_i, c->state, c->tok_log, st);
@@ -683,6 +912,7 @@ static int block_ensure(lgh_ctx* c) {
   uint32_t heads = 0, hdim = 0;
   for (auto& L : m.layers)
     if (L.mlstm()) { heads = std::max(heads, L.ms.heads); hdim = std::max(hdim, L.ms.heads * L.ms.dim); }
+    else if (L.gla()) heads = std::max(heads, L.as.heads);
   const size_t moe_tiles = moe_max_tiles(m.blk * m.max_top, std::max(m.max_experts, 1u), 16);
   const size_t B = m.blk, chunks = (B + 63) / 64, Bc = chunks * 64, el = m.el();
   struct { void** p; size_t n; } bufs[] = {
@@ -690,6 +920,8 @@ static int block_ensure(lgh_ctx* c) {
       {(void**)&m.bcat, (B * m.max_cat + kMlstmRowSlack) * 4}, {&m.bao, B * m.max_ao * el}, {&m.bact, B * m.max_act * el},
       {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * Bc * 8}, {(void**)&m.bmx, heads * Bc * 8},
       {(void**)&m.bdec, heads * Bc * 4}, {(void**)&m.bwgt, heads * Bc * 4}, {(void**)&m.bcdec, heads * chunks * 4}, {(void**)&m.bnk, chunks * hdim * 4},
+      {(void**)&m.brec, B * m.max_rec * 2 * 4}, {(void**)&m.brsum, (chunks * 2 + 1) * m.max_rec * 4},
+      {(void**)&m.bqk, m.max_gla ? (Bc * m.max_gla * 2 + kMlstmRowSlack) * 4 : 0}, {(void**)&m.bgdec, m.max_gla ? (chunks * m.max_gla + kMlstmRowSlack) * 4 : 0},
       {(void**)&m.bx2, m.dyt() ? B * d.width * 4 : 0}, {(void**)&m.tails, m.hist_floats() * 4}, {&m.btq, B * m.max_tied_q * el},
       {(void**)&m.bpair, B * m.max_top * up(d.width, 4) * 4}, {&m.bpact, B * m.max_pair_act * el},
       {(void**)&m.bsel, B * m.max_top * 4}, {(void**)&m.bselw, B * m.max_top * 4}, {(void**)&m.bslot, B * m.max_top * 4}, {(void**)&m.bsrc, B * m.max_top * 4},
@@ -706,8 +938,9 @@ static int block_ensure(lgh_ctx* c) {
   return LGH_OK;
 }
 
-static int block_gemm(lgh_ctx* c, int cls, const LinW& W, int epi, const void* x, uint32_t ldx, void* out, uint32_t ldo, uint32_t M) {
+static int block_gemm(lgh_ctx* c, int cls, const LinW& W, int epi, const void* x, uint32_t ldx, void* out, uint32_t ldo, uint32_t M, const float* bias = nullptr) {
   LinGemm g{};
+  g.bias = bias;
   g.w = W.w; g.x = x; g.out = out; g.n = W.n; g.np = W.np(); g.kp = W.kp; g.ldx = ldx; g.ldo = ldo; g.M = M;
   return run_k(c, cls, LGH_SYM_LINEAR, W.bytes(), [&] { return lin_gemm_launch(epi, c->lm->f32, g, c->stream); });
 }
@@ -780,6 +1013,38 @@ static int block_tied(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) {
   return run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_TIED, 0, [&] { return tied_merge_launch(L.ts, b, nullptr, pos0, M, splits, m.f32, m.bao, L.out.kp, m.f32, st); });
 }
 
+// gated attention and / or gated linear attention of a block, side by side in the output product's input
+static int block_gattn(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) {
+  LayeredModel& m = *c->lm;
+  hipStream_t st = c->stream;
+  int rc;
+  if (L.gattn()) {
+    GattnBufs b = gattn_bufs(m, L, m.bcat);
+    const bool flash = M > kGattnShort && L.gs.dp <= kGattnFlashDim;
+    if (flash) { b.q = m.btq; b.Mcap = m.blk; }
+    if ((rc = run_k(c, LGH_K_EXPAND, LGH_SYM_GATTN, 0, [&] { return gattn_prep_launch(L.gs, b, pos0, M, m.f32, st); }))) return rc;
+    if (flash) {
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GATTN, 0, [&] { return gattn_flash_launch(L.gs, b, pos0, M, m.f32, m.bao, L.out.kp, st); }))) return rc;
+    } else {
+      for (uint32_t t = 0; t < M; t += kGattnShort) {
+        const uint32_t n = std::min(kGattnShort, M - t), splits = gattn_splits(L.gs, m.d.max_seq_len, n, m.f32, m.forced_splits);
+        b.cat = m.bcat + (size_t)t * L.gs.ldcat;
+        if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GATTN, 0, [&] { return gattn_attn_launch(L.gs, b, nullptr, nullptr, nullptr, pos0 + t, n, false, splits, m.f32, st); }))) return rc;
+        if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_GATTN, 0, [&] {
+               return gattn_merge_launch(L.gs, b, nullptr, nullptr, 0, nullptr, pos0 + t, n, splits, m.f32, (uint8_t*)m.bao + (size_t)t * L.out.kp * m.el(), L.out.kp, m.f32, st);
+             })))
+          return rc;
+      }
+    }
+  }
+  if (L.gla()) {
+    const GlaBufs g = gla_bufs(m, L, m.bcat, m.bnum);
+    if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GLA, 0, [&] { return gla_block_launch(L.as, g, pos0, M, st); }))) return rc;
+    if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_GLA, 0, [&] { return gla_out_launch(L.as, g, M, (uint8_t*)m.bao + (size_t)L.gla_col * m.el(), L.out.kp, m.f32, st); }))) return rc;
+  }
+  return LGH_OK;
+}
+
 // routed experts of a block: the pairs' outputs -> m.bpair, rows m.bslot; the shared expert -> m.by
 static int block_moe(lgh_ctx* c, LayeredLayer& L, uint32_t ldx, uint32_t ldy, uint32_t M) {
   LayeredModel& m = *c->lm;
@@ -790,12 +1055,15 @@ static int block_moe(lgh_ctx* c, LayeredLayer& L, uint32_t ldx, uint32_t ldy, ui
   r.x = m.bxa; r.ldx = ldx; r.router = L.router.w; r.kp = L.router.kp; r.M = M; r.experts = E; r.top = L.d.top; r.bm = lin_group_rows(rows, std::min(rows, E));
   r.sel = m.bsel; r.w = m.bselw; r.seg = m.bseg; r.tile_e = m.btile_e; r.tile_row = m.btile_row; r.slot = m.bslot; r.src = m.bsrc; r.roww = m.broww;
   r.tiles = moe_max_tiles(rows, E, r.bm);
+  r.route = L.route();
   if ((rc = run_k(c, LGH_K_ROUTER, LGH_SYM_OTHER, 0, [&] { return moe_route_launch(r, m.f32, st); }))) return rc;
   LinGemm g{};
   g.grp.seg = r.seg; g.grp.tile_e = r.tile_e; g.grp.tile_row = r.tile_row; g.grp.tiles = r.tiles; g.grp.bm = r.bm;
   g.w = L.egu.w; g.n = g.np = L.egu_rows; g.kp = L.egu.kp; g.M = rows; g.x = m.bxa; g.ldx = ldx; g.out = m.bpact; g.ldo = L.edown.kp;
   g.grp.src = r.src; g.grp.scale = r.roww; g.grp.stride = (uint64_t)L.egu_rows * L.egu.kp;
-  if ((rc = run_k(c, LGH_K_EXPERTS, LGH_SYM_LINEAR, L.egu.bytes(), [&] { return lin_gemm_launch(LE_SWIGLU, m.f32, g, st); }))) return rc;
+  g.grp.limit = (float)L.d.expert_limit;
+  const int epi = L.d.expert_form == LGH_EXPERT_CLAMPED ? LE_CLAMPED : LE_SWIGLU;
+  if ((rc = run_k(c, LGH_K_EXPERTS, LGH_SYM_LINEAR, L.egu.bytes(), [&] { return lin_gemm_launch(epi, m.f32, g, st); }))) return rc;
   g.w = L.edown.w; g.n = m.d.width; g.np = L.edown_rows; g.kp = L.edown.kp; g.x = m.bpact; g.ldx = L.edown.kp; g.out = m.bpair; g.ldo = ldy;
   g.grp.src = nullptr; g.grp.scale = nullptr; g.grp.stride = (uint64_t)L.edown_rows * L.edown.kp;
   if ((rc = run_k(c, LGH_K_DOWN, LGH_SYM_LINEAR, L.edown.bytes(), [&] { return lin_gemm_launch(LE_F32, m.f32, g, st); }))) return rc;
@@ -838,7 +1106,18 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
     return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, (uint64_t)M * d.width * 14, [&] { return dyt_block_launch(b, m.f32, st); });
   };
   if (m.dyt() && (rc = resid_dyt(true, nullptr))) return rc;
+  // LGH_RESIDUAL_PRE_RMS: the sublayer's output into the stream, then its norm in front of the next sublayer (nw NULL: there is none)
+  auto resid_pre = [&](const float* nw, bool from_embed, const LayeredLayer* moe) {
+    PreBlock b{};
+    b.x = m.bx; b.width = d.width; b.M = M; b.mult = mult; b.eps = eps; b.nw = nw; b.xa = m.bxa; b.ldx = ldx;
+    if (!from_embed && (!moe || moe->d.shared_ff)) { b.y = m.by; b.ldy = ldy; }
+    if (moe) { b.pairs = m.bpair; b.ldp = ldy; b.slot = m.bslot; b.selw = m.bselw; b.top = moe->d.top; }
+    return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, (uint64_t)M * d.width * 14, [&] { return pre_block_launch(b, m.f32, st); });
+  };
+  if (m.pre() && (rc = resid_pre(m.layers[0].norm1, true, nullptr))) return rc;
+  const float* next = nullptr;             // the norm in front of the sublayer that follows
   auto resid = [&](const float* nw, const LayeredLayer* moe = nullptr) -> int {
+    if (m.pre()) return resid_pre(next, false, moe);
     if (m.dyt()) return resid_dyt(false, moe);
     if (moe && (rc = run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
                   return pair_sum_launch(m.by, ldy, m.bpair, ldy, m.bslot, moe->d.top, d.width, M, moe->d.shared_ff != 0, st);
@@ -850,18 +1129,26 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
   };
   for (uint32_t li = 0; li < d.num_layers; li++) {
     LayeredLayer& L = m.layers[li];
-    if ((rc = block_gemm(c, LGH_K_QKV, L.in, LE_F32, m.bxa, ldx, m.bcat, L.in.n, M))) return rc;
+    const float* after = li + 1 < d.num_layers ? m.layers[li + 1].norm1 : nullptr;
+    if ((rc = block_gemm(c, LGH_K_QKV, L.in, LE_F32, m.bxa, ldx, m.bcat, L.in.n, M, L.in_bias))) return rc;
     if (L.latent()) {
       if ((rc = block_latent(c, L, pos0, M))) return rc;
     } else if (L.tied()) {
       if ((rc = block_tied(c, L, pos0, M))) return rc;
+    } else if (L.glru()) {
+      const GlruBufs b = glru_bufs(m, L, m.bcat);
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GLRU, 0, [&] { return glru_block_launch(L.rs, b, pos0, M, m.f32, m.bao, L.out.kp, st); }))) return rc;
+    } else if (L.gattn() || L.gla()) {
+      if ((rc = block_gattn(c, L, pos0, M))) return rc;
     } else {
       const MlstmBufs b = mlstm_bufs(m, L, m.bcat, m.bnum);
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_MLSTM, 0, [&] { return mlstm_block_launch(L.ms, b, pos0, M, st); }))) return rc;
       if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_MLSTM, 0, [&] { return mlstm_out_launch(L.ms, b, M, m.bao, L.out.kp, m.f32, st); }))) return rc;
     }
     if ((rc = block_gemm(c, LGH_K_WO, L.out, LE_F32, m.bao, L.out.kp, m.by, ldy, M))) return rc;
+    next = L.d.ff_kind ? L.norm2 : after;
     if ((rc = resid(L.norm1))) return rc;
+    next = after;
     if (L.moe()) {
       if ((rc = block_moe(c, L, ldx, ldy, M))) return rc;
       if ((rc = resid(L.norm2, &L))) return rc;
@@ -883,6 +1170,7 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
     const uint32_t n = std::min(kLogitRows, n_want - w);
     L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(m.brows, want + w, (size_t)n * 4, hipMemcpyHostToDevice, st));
     if ((rc = run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
+           if (m.pre()) return final_rms_rows_launch(xs, m.brows, n, m.final_norm, eps, d.logit_scale != 0.0 ? (float)d.logit_scale : 1.0f, d.width, m.bla, ldx, m.f32, st);
            return m.dyt() ? final_dyt_rows_launch(xs, m.brows, n, dyt_w(m.final_dyt), d.width, m.bla, ldx, m.f32, st)
                           : final_norm_rows_launch(xs, m.brows, n, m.final_norm, eps, d.width, m.bla, ldx, m.f32, st);
          })))

@@ -23,6 +23,13 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float log_sigmoid_f(float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
+__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
+// a gated unit with both halves clamped (LGH_EXPERT_CLAMPED)
+__device__ __forceinline__ float clamped_glu_f(float gate, float up, float limit) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g * sigmoid_f(1.702f * g) * (u + 1.0f);
+}
 
 // tanh: its odd series up to 1/4 (next term below 1e-7 of the value), beyond it 1 - 2 / (exp(2x) + 1); 1e-6 of the value everywhere
 __device__ __forceinline__ float tanh_series(float x) {
@@ -52,6 +59,60 @@ __device__ __forceinline__ void rank_expert(const float* z, uint32_t E, uint32_t
     for (uint32_t i = 0; i < 4; i++) place += q[i] > v || (q[i] == v && j + i < e) ? 1u : 0u;
   }
   if (place < top) { sel[place] = (int)e; w[place] = sigmoid_f(v); }
+}
+
+// LGH_ROUTER_SOFTMAX_GROUPS for T tokens by a whole workgroup.  z [T][ep] (LDS, ep = E rounded up to 4): logits, scores afterwards; c [T][ep],
+// gm [T][groups] LDS scratch; sel, w [T][top]: the chosen ones, largest choice score first, and their weights.  Ends with a barrier.
+__device__ __forceinline__ void route_groups(float* z, float* c, float* gm, uint32_t T, uint32_t E, uint32_t ep, uint32_t top, const RouteForm& f, int* sel, float* w) {
+  const uint32_t tid = threadIdx.x, nt = blockDim.x, lane = tid & 63, wave = tid >> 6, nw = nt >> 6;
+  for (uint32_t t = wave; t < T; t += nw) {
+    float m = -INFINITY, s = 0.0f;
+    for (uint32_t e = lane; e < E; e += 64) m = fmaxf(m, rank_key(z[t * ep + e]));
+    m = wave_max(m);
+    for (uint32_t e = lane; e < E; e += 64) { const float p = expf(rank_key(z[t * ep + e]) - m); z[t * ep + e] = p; s += p; }
+    const float inv = 1.0f / wave_sum(s);
+    for (uint32_t e = lane; e < ep; e += 64) {
+      const float p = e < E ? z[t * ep + e] * inv : 0.0f;
+      z[t * ep + e] = p;
+      c[t * ep + e] = e < E ? rank_key(p + f.correction[e]) : -INFINITY;
+    }
+  }
+  __syncthreads();
+  const uint32_t gs = E / f.groups;
+  for (uint32_t i = tid; i < T * f.groups; i += nt) {
+    const float* p = c + i / f.groups * ep + i % f.groups * gs;
+    float m = p[0];
+    for (uint32_t e = 1; e < gs; e++) m = fmaxf(m, p[e]);
+    gm[i] = m;
+  }
+  __syncthreads();
+  for (uint32_t i = tid; i < T * E; i += nt) {   // (a group's members all find the same place for it)
+    const uint32_t t = i / E, e = i % E, g = e / gs;
+    const float* q = gm + t * f.groups;
+    uint32_t place = 0;
+    for (uint32_t j = 0; j < f.groups; j++) place += q[j] > q[g] || (q[j] == q[g] && j < g) ? 1u : 0u;
+    if (place >= f.keep) c[t * ep + e] = -INFINITY;
+  }
+  __syncthreads();
+  for (uint32_t i = tid; i < T * E; i += nt) {
+    const uint32_t t = i / E, e = i % E;
+    const float v = c[t * ep + e];
+    uint32_t place = 0;
+    for (uint32_t j = 0; j < E; j += 4) {
+      const f32x4 q = *reinterpret_cast<const f32x4*>(c + t * ep + j);
+#pragma unroll
+      for (uint32_t k = 0; k < 4; k++) place += q[k] > v || (q[k] == v && j + k < e) ? 1u : 0u;
+    }
+    if (place < top) sel[t * top + place] = (int)e;
+  }
+  __syncthreads();
+  for (uint32_t i = tid; i < T * top; i += nt) {
+    const uint32_t t = i / top;
+    float s = 0.0f;
+    for (uint32_t k = 0; k < top; k++) s += z[t * ep + sel[t * top + k]];
+    w[i] = z[t * ep + sel[i]] / (s + 1e-20f);
+  }
+  __syncthreads();
 }
 
 // ---- residual form LGH_RESIDUAL_SANDWICH_DYT, one channel ----
@@ -106,6 +167,25 @@ __device__ __forceinline__ void post_finish(const PostUpdate& a, const PostIn& r
   const float v = __builtin_fmaf(a.mult, dyt_f(y, palpha, r.pw, r.pb), r.x);
   a.xout[c] = v;
   post_input(a, r, c, p, v, nalpha);
+}
+
+// sum over `N` neighbouring lanes, every one of them gets it
+template <uint32_t N> __device__ __forceinline__ float lanes_sum(float v) {
+  v += dpp_f<0xB1>(v); v += dpp_f<0x4E>(v); v += dpp_f<0x141>(v);
+  if constexpr (N >= 16) v += dpp_f<0x140>(v);
+  if constexpr (N >= 32) v += __shfl_xor(v, 16, 64);
+  if constexpr (N >= 64) v += __shfl_xor(v, 32, 64);
+  return v;
+}
+
+// 16 bytes of a cache row as floats
+template <class T, int PER> __device__ __forceinline__ void unpack_row(const u32x4& w, float* f) {
+  if constexpr (sizeof(T) == 2) {
+    f[0] = bf_lo(w.x); f[1] = bf_hi(w.x); f[2] = bf_lo(w.y); f[3] = bf_hi(w.y);
+    f[4] = bf_lo(w.z); f[5] = bf_hi(w.z); f[6] = bf_lo(w.w); f[7] = bf_hi(w.w);
+  } else {
+    f[0] = __uint_as_float(w.x); f[1] = __uint_as_float(w.y); f[2] = __uint_as_float(w.z); f[3] = __uint_as_float(w.w);
+  }
 }
 
 // sum over a workgroup of up to 16 waves; every thread gets the result.  red: 16 floats of LDS, free again after the call.

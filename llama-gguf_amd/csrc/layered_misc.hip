@@ -1,5 +1,5 @@
-// layered_misc.hip — embedding (with the pair table), residual updates of both forms (layer norm; squashing norms with a short
-// convolution), final norm of the models of layered.h.
+// layered_misc.hip — embedding (with the pair table), residual updates of all forms (layer norm; squashing norms with a short
+// convolution; RMS norm in front of a sublayer), final norm of the models of layered.h.
 #include "layered.h"
 #include "layered_device.h"
 
@@ -23,7 +23,7 @@ __global__ void __launch_bounds__(1024) layered_embed_kernel(const EmbedArgs a, 
     state[ST_NEXT] = p + 1;
     a.hist[p] = (int)tok;
   }
-  const uint16_t* e = a.embed + (size_t)tok * a.width;
+  const uint16_t* e = a.embed + (size_t)tok * a.ld;
   const uint16_t* b = a.bigram ? a.bigram + bigram_row(a, (uint32_t)p, prev, tok) * a.width : nullptr;
   const float alpha = with_post ? *post.next.alpha : 0.0f;
   constexpr uint32_t U = 4;   // channels a thread has in flight
@@ -57,7 +57,7 @@ __global__ void __launch_bounds__(256) layered_embed_block_kernel(const EmbedArg
                                                                   T* __restrict__ xa, uint32_t ldx) {
   const uint32_t t = blockIdx.x, pos = pos0 + t;
   const uint32_t tok = (uint32_t)tokens[t];
-  const uint16_t* e = a.embed + (size_t)tok * a.width;
+  const uint16_t* e = a.embed + (size_t)tok * a.ld;
   const uint16_t* b = nullptr;
   if (a.bigram) {
     const uint32_t prev = t ? (uint32_t)tokens[t - 1] : pos ? (uint32_t)a.hist[pos - 1] : 0u;   // this launch writes hist[pos0 ..] only
@@ -156,6 +156,34 @@ __global__ void __launch_bounds__(256) final_dyt_rows_kernel(const float* __rest
 hipError_t final_dyt_rows_launch(const float* x, const int* rows, uint32_t n_rows, const DytW& n, uint32_t width, void* xa, uint32_t ldx, bool f32, hipStream_t st) {
   if (f32) hipLaunchKernelGGL(final_dyt_rows_kernel<float>, dim3(n_rows), dim3(256), 0, st, x, rows, n, width, (float*)xa, ldx);
   else hipLaunchKernelGGL(final_dyt_rows_kernel<__bf16>, dim3(n_rows), dim3(256), 0, st, x, rows, n, width, (__bf16*)xa, ldx);
+  return hipGetLastError();
+}
+
+template <class T>
+__global__ void __launch_bounds__(256) final_rms_rows_kernel(const float* __restrict__ x, const int* __restrict__ rows, const float* __restrict__ w, float eps, float scale,
+                                                             uint32_t width, T* __restrict__ xa, uint32_t ldx) {
+  __shared__ float red[16];
+  const float* r = x + (size_t)rows[blockIdx.x] * width;
+  float q = 0.0f;
+  for (uint32_t i = threadIdx.x; i < width; i += 256) q = __builtin_fmaf(r[i], r[i], q);
+  const float inv = 1.0f / __builtin_sqrtf(block_sum(q, red) / (float)width + eps) * scale;
+  for (uint32_t i = threadIdx.x; i < width; i += 256) xa[(size_t)blockIdx.x * ldx + i] = to_act<T>(r[i] * inv * (1.0f + w[i]));
+}
+
+hipError_t final_rms_rows_launch(const float* x, const int* rows, uint32_t n_rows, const float* w, float eps, float scale, uint32_t width, void* xa, uint32_t ldx,
+                                 bool f32, hipStream_t st) {
+  if (f32) hipLaunchKernelGGL(final_rms_rows_kernel<float>, dim3(n_rows), dim3(256), 0, st, x, rows, w, eps, scale, width, (float*)xa, ldx);
+  else hipLaunchKernelGGL(final_rms_rows_kernel<__bf16>, dim3(n_rows), dim3(256), 0, st, x, rows, w, eps, scale, width, (__bf16*)xa, ldx);
+  return hipGetLastError();
+}
+
+__global__ void __launch_bounds__(256) resid_add_kernel(const float* __restrict__ x, const float* __restrict__ y, float mult, uint32_t width, float* __restrict__ xout) {
+  const uint32_t i = blockIdx.x * 256 + threadIdx.x;
+  if (i < width) xout[i] = __builtin_fmaf(mult, y[i], x[i]);
+}
+
+hipError_t resid_add_launch(const float* x, const float* y, float mult, uint32_t width, float* xout, hipStream_t st) {
+  hipLaunchKernelGGL(resid_add_kernel, dim3((width + 255) / 256), dim3(256), 0, st, x, y, mult, width, xout);
   return hipGetLastError();
 }
 
@@ -309,6 +337,79 @@ hipError_t dyt_block_launch(const DytBlock& a, bool f32, hipStream_t st) {
   if (even && (uint64_t)a.width * a.M <= 1u << 24) return f32 ? dyt_block_go<float, 2>(a, st) : dyt_block_go<__bf16, 2>(a, st);   // (enough waves)
   if (even) return f32 ? dyt_block_go<float, 4>(a, st) : dyt_block_go<__bf16, 4>(a, st);
   return f32 ? dyt_block_go<float, 1>(a, st) : dyt_block_go<__bf16, 1>(a, st);
+}
+
+// ------------------------------------------------------------------------------------------------
+// LGH_RESIDUAL_PRE_RMS over a block: a workgroup per token, the new stream row in LDS between the sum of its squares and its use
+// ------------------------------------------------------------------------------------------------
+template <class T, int V>
+__global__ void __launch_bounds__(256) pre_block_kernel(const PreBlock a) {
+  extern __shared__ __attribute__((aligned(16))) float row[];
+  __shared__ float red[16];
+  const uint32_t t = blockIdx.x;
+  float* x = a.x + (size_t)t * a.width;
+  T* xa = reinterpret_cast<T*>(a.xa) + (size_t)t * a.ldx;
+  const int* slot = a.slot + (size_t)t * a.top;
+  float q = 0.0f, id_w = 0.0f;
+  if (a.pairs)
+    for (uint32_t s = 0; s < a.top; s++) id_w += slot[s] < 0 ? a.selw[(size_t)t * a.top + s] : 0.0f;
+  for (uint32_t c = threadIdx.x * V; c < a.width; c += 256 * V) {
+    VecF<V> v = load_vec<V>(x + c), y;
+#pragma unroll
+    for (int i = 0; i < V; i++) y.v[i] = 0.0f;
+    if (a.y) y = load_vec<V>(a.y + (size_t)t * a.ldy + c);
+    if (a.pairs) {
+      for (uint32_t s = 0; s < a.top; s += 4) {   // four rows in flight
+        VecF<V> p[4];
+        float f[4];
+#pragma unroll
+        for (uint32_t k = 0; k < 4; k++) {
+          const int r = slot[s + k < a.top ? s + k : s];
+          f[k] = s + k < a.top && r >= 0 ? 1.0f : 0.0f;
+          p[k] = load_vec<V>(a.pairs + (size_t)(r >= 0 ? r : 0) * a.ldp + c);
+        }
+#pragma unroll
+        for (uint32_t k = 0; k < 4; k++)
+          if (f[k] != 0.0f)
+#pragma unroll
+            for (int i = 0; i < V; i++) y.v[i] += p[k].v[i];
+      }
+      if (id_w != 0.0f)
+#pragma unroll
+        for (int i = 0; i < V; i++) y.v[i] = __builtin_fmaf(id_w, (float)xa[c + i], y.v[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < V; i++) {
+      v.v[i] = __builtin_fmaf(a.mult, y.v[i], v.v[i]);
+      q = __builtin_fmaf(v.v[i], v.v[i], q);
+    }
+    store_vec<V>(row + c, v);
+    if (a.y || a.pairs) store_vec<V>(x + c, v);
+  }
+  if (!a.nw) return;
+  const float inv = 1.0f / __builtin_sqrtf(block_sum(q, red) / (float)a.width + a.eps);
+  for (uint32_t c = threadIdx.x * V; c < a.width; c += 256 * V) {   // (every thread its own channels again)
+    const VecF<V> v = load_vec<V>(row + c), w = load_vec<V>(a.nw + c);
+    T o[V];
+#pragma unroll
+    for (int i = 0; i < V; i++) o[i] = to_act<T>(v.v[i] * inv * (1.0f + w.v[i]));
+    __builtin_memcpy(__builtin_assume_aligned(xa + c, sizeof(o)), o, sizeof(o));
+  }
+}
+
+template <class T, int V>
+static hipError_t pre_block_go(const PreBlock& a, hipStream_t st) {
+  static bool opted[64] = {};
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&pre_block_kernel<T, V>), kNormMaxWidth * 4, opted); e != hipSuccess) return e;
+  hipLaunchKernelGGL((pre_block_kernel<T, V>), dim3(a.M), dim3(256), (size_t)a.width * 4, st, a);
+  return hipGetLastError();
+}
+
+hipError_t pre_block_launch(const PreBlock& a, bool f32, hipStream_t st) {
+  if (!a.x || !a.xa || a.M == 0 || a.width == 0 || a.width > kNormMaxWidth || a.ldx < a.width || (a.pairs && (!a.slot || !a.selw || a.top == 0))) return hipErrorInvalidValue;
+  const bool v4 = a.width % 4 == 0 && (!a.y || a.ldy % 4 == 0) && (!a.pairs || a.ldp % 4 == 0) && a.ldx % 4 == 0;
+  if (v4) return f32 ? pre_block_go<float, 4>(a, st) : pre_block_go<__bf16, 4>(a, st);
+  return f32 ? pre_block_go<float, 1>(a, st) : pre_block_go<__bf16, 1>(a, st);
 }
 
 __global__ void __launch_bounds__(256) conv_store_kernel(const float* __restrict__ tails, float* __restrict__ hists, uint32_t back, uint32_t width, uint32_t last) {

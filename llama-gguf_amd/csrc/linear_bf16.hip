@@ -46,8 +46,13 @@ __device__ __forceinline__ void mv_fetch(const LinMv& a, uint32_t g, uint32_t kb
       o.w[r] = ldg_nt128(a.w2 + (size_t)(row < a.n2 ? row : a.n2 - 1) * a.kp + kc);
     }
   } else if (SRC == LS_EXPERTS) {
-    const uint32_t slot = g / g1, gl = g - slot * g1;
-    const uint16_t* w = a.w2 + (size_t)__builtin_amdgcn_readfirstlane(sel[slot]) * a.stride + kc;
+    const uint32_t slot = g / g1, gl = g - slot * g1, ex = (uint32_t)__builtin_amdgcn_readfirstlane(sel[slot]);
+    if (ex >= a.experts) {   // (an identity expert has no rows)
+#pragma unroll
+      for (int r = 0; r < kMvR; r++) o.w[r] = (u32x4)(0u);
+      return;
+    }
+    const uint16_t* w = a.w2 + (size_t)ex * a.stride + kc;
 #pragma unroll
     for (int r = 0; r < kMvR; r++) {
       const uint32_t row = mv_row_of(1, gl, r);
@@ -58,6 +63,11 @@ __device__ __forceinline__ void mv_fetch(const LinMv& a, uint32_t g, uint32_t kb
     uint32_t ld = a.kps;
     if (kc >= a.kps) {
       const uint32_t q = kc - a.kps, s = q / a.kpe;
+      if ((uint32_t)sel[s] >= a.experts) {
+#pragma unroll
+        for (int r = 0; r < kMvR; r++) o.w[r] = (u32x4)(0u);
+        return;
+      }
       w = a.w2 + (size_t)sel[s] * a.stride + (q - s * a.kpe);
       ld = a.kpe;
     }
@@ -83,7 +93,10 @@ __device__ __forceinline__ void mv_acc(const MvW& o, f32x4 x0, f32x4 x1, float* 
     acc[r] = s;
   }
 }
-__device__ __forceinline__ float mv_act(uint32_t act, float z) { return act == LA_SILU ? silu_f(z) : gelu_tanh_f(z); }
+__device__ __forceinline__ float mv_glu(const LinMv& a, float gate, float up) {
+  if (a.act == LA_CLAMPED) return clamped_glu_f(gate, up, a.limit);
+  return (a.act == LA_SILU ? silu_f(gate) : gelu_tanh_f(gate)) * up;
+}
 
 template <int PRO, int SRC, bool POST>
 __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint32_t n_groups, uint32_t ks, uint32_t g1) {
@@ -92,6 +105,8 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
   __shared__ float red[2][16][kMvR];
   __shared__ float bred[16];
   __shared__ __attribute__((aligned(16))) float zs[SRC == LS_EXPERTS ? kMaxExperts : 4];
+  __shared__ __attribute__((aligned(16))) float zc[SRC == LS_EXPERTS ? 2 * kMaxRouted : 4];   // choice scores, groups
+  __shared__ float id_w;
   __shared__ int sel[MOE ? kMaxTop : 1];
   __shared__ float selw[SRC == LS_EXPERTS ? kMaxTop : 1];
   const uint32_t tid = threadIdx.x, lane = tid & 63, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
@@ -110,13 +125,45 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
   float palpha = 0.0f, nalpha = 0.0f;
   if (POST) { pos = __builtin_amdgcn_readfirstlane(*a.post.pos); palpha = *a.post.post.alpha; nalpha = *a.post.next.alpha; }
   if (SRC == LS_EXPERTS) {
-    const uint32_t ep = (a.experts + 3) & ~3u;
-    for (uint32_t e = tid; e < ep; e += kMvThreads) zs[e] = e < a.experts ? rank_key(a.logits[e]) : -INFINITY;
+    const uint32_t ne = a.experts + a.route.identity, ep = (ne + 3) & ~3u;
+    for (uint32_t e = tid; e < ep; e += kMvThreads) zs[e] = e < ne ? rank_key(a.logits[e]) : -INFINITY;
   }
   if (SRC == LS_MOE_DOWN)
     for (uint32_t e = tid; e < a.top; e += kMvThreads) sel[e] = a.sel[e];
   if (PRO == LP_COPY) {
     for (uint32_t i = tid; i < a.k; i += kMvThreads) xs[i] = a.x[i];
+  } else if (PRO == LP_PRE) {
+    constexpr uint32_t U = 4;   // channels a thread has in flight, their norm weights with them
+    float s = 0.0f, nw[U];
+    for (uint32_t i0 = tid; i0 < a.k; i0 += U * kMvThreads) {
+      float v[U], y[U];
+#pragma unroll
+      for (uint32_t u = 0; u < U; u++) {
+        const uint32_t i = i0 + u * kMvThreads, ic = i < a.k ? i : a.k - 1;
+        v[u] = a.x[ic];
+        y[u] = a.y ? a.y[ic] : 0.0f;
+        if (i0 == tid) nw[u] = a.nw2[ic];
+      }
+#pragma unroll
+      for (uint32_t u = 0; u < U; u++) {
+        const uint32_t i = i0 + u * kMvThreads;
+        if (i >= a.k) break;
+        const float x = __builtin_fmaf(a.mult, y[u], v[u]);
+        xs[i] = x;
+        if (a.y && blockIdx.x == 0) a.xout[i] = x;
+        s = __builtin_fmaf(x, x, s);
+      }
+    }
+    const float inv = 1.0f / __builtin_sqrtf(block_sum(s, bred) / (float)a.k + a.eps) * a.in_scale;
+    for (uint32_t i0 = tid; i0 < a.k; i0 += U * kMvThreads)
+#pragma unroll
+      for (uint32_t u = 0; u < U; u++) {
+        const uint32_t i = i0 + u * kMvThreads;
+        if (i >= a.k) break;
+        const float h = xs[i] * inv * (1.0f + (i0 == tid ? nw[u] : a.nw2[i]));
+        xs[i] = h;
+        if (a.hout && blockIdx.x == 0) a.hout[i] = h;
+      }
   } else if (PRO == LP_RESID || PRO == LP_HEAD) {
     for (uint32_t i = tid; i < a.k; i += kMvThreads) xs[i] = a.y[i];
     ln_lds(xs, a.k, a.nw, a.eps, bred);
@@ -162,9 +209,26 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
   for (uint32_t i = a.k + tid; i < a.kp; i += kMvThreads) xs[i] = 0.0f;
   __syncthreads();
   if (SRC == LS_EXPERTS) {
-    for (uint32_t e = tid; e < a.experts; e += kMvThreads) rank_expert(zs, a.experts, a.top, e, sel, selw);
+    if (a.route.form == LGH_ROUTER_SIGMOID) {
+      for (uint32_t e = tid; e < a.experts; e += kMvThreads) rank_expert(zs, a.experts, a.top, e, sel, selw);
+      __syncthreads();
+    } else {
+      const uint32_t ne = a.experts + a.route.identity;
+      route_groups(zs, zc, zc + kMaxRouted, 1, ne, (ne + 3) & ~3u, a.top, a.route, sel, selw);
+    }
+    if (blockIdx.x == 0 && tid < a.top) {
+      a.sel[tid] = sel[tid];
+      if (a.selw) a.selw[tid] = selw[tid];
+    }
+  }
+  if (SRC == LS_MOE_DOWN) {
+    if (tid == 0) {
+      float s = 0.0f;
+      if (a.id_x)
+        for (uint32_t t = 0; t < a.top; t++) s += (uint32_t)sel[t] >= a.experts ? a.selw[t] : 0.0f;
+      id_w = s;
+    }
     __syncthreads();
-    if (blockIdx.x == 0 && tid < a.top) a.sel[tid] = sel[tid];
   }
   if (MOE) { request(n0); request(n1); }
   const uint32_t rounds = (n_groups + gstep - 1) / gstep;   // the same for every wave: the teams meet at a barrier when ks > 1
@@ -207,10 +271,10 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
     } else if (SRC == LS_EXPERTS) {
       if (sub == 0 && lane == 63 && g < n_groups) {
         const uint32_t slot = g / g1, gl = g - slot * g1;
-        const float w = selw[slot];
+        const float win = a.route.form == LGH_ROUTER_SIGMOID ? selw[slot] : 1.0f, wout = a.route.form == LGH_ROUTER_SIGMOID ? 1.0f : selw[slot];
 #pragma unroll
         for (int r = 0; r < 2; r++)
-          if (gl * 2 + r < a.n / 2) a.out[(size_t)slot * a.kpe + gl * 2 + r] = mv_act(a.act, w * acc[r]) * (w * acc[r + 2]);
+          if (gl * 2 + r < a.n / 2) a.out[(size_t)slot * a.kpe + gl * 2 + r] = wout * mv_glu(a, win * acc[r], win * acc[r + 2]);
       }
     } else if (SRC == LS_TWO && g >= g1) {
       if (sub == 0 && lane == 63 && g < n_groups) {
@@ -222,11 +286,17 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
       if (!a.paired) {
 #pragma unroll
         for (int r = 0; r < kMvR; r++)
-          if (g * kMvR + r < a.n) a.out[g * kMvR + r] = acc[r];
+          if (g * kMvR + r < a.n) {
+            const uint32_t n = g * kMvR + r;
+            float v = acc[r];
+            if (a.bias) v += a.bias[n];
+            if (SRC == LS_MOE_DOWN && a.id_x) v = __builtin_fmaf(id_w, a.id_x[n], v);
+            a.out[n] = v;
+          }
       } else {
 #pragma unroll
         for (int r = 0; r < 2; r++)
-          if (g * 2 + r < a.n / 2) a.out[g * 2 + r] = mv_act(a.act, acc[r]) * acc[r + 2];
+          if (g * 2 + r < a.n / 2) a.out[g * 2 + r] = mv_glu(a, acc[r], acc[r + 2]);
       }
     }
   }
@@ -235,7 +305,7 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
 template <int PRO, int SRC, bool POST>
 static hipError_t lin_mv_run(const LinMv& a, hipStream_t st) {
   static bool opted[64] = {};
-  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_mv_kernel<PRO, SRC, POST>), 152 * 1024, opted); e != hipSuccess) return e;
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&lin_mv_kernel<PRO, SRC, POST>), (SRC == LS_EXPERTS ? 140 : 152) * 1024, opted); e != hipSuccess) return e;
   const uint32_t g1 = (a.n + kMvR - 1) / kMvR;
   const uint32_t groups = SRC == LS_TWO ? g1 + (a.n2 + kMvR - 1) / kMvR : SRC == LS_EXPERTS ? g1 * a.top : g1;
   uint32_t ks = 1;   // waves per team: enough teams for the groups of a CU, and at least a full pass of columns per wave
@@ -258,17 +328,25 @@ static hipError_t lin_mv_go(const LinMv& a, int src, hipStream_t st) {
   return src != LS_PLAIN || a.post.xout ? hipErrorInvalidValue : lin_mv_run<PRO, LS_PLAIN, false>(a, st);
 }
 
+bool route_ok(const RouteForm& f, uint32_t outputs, uint32_t top) {
+  return f.form == LGH_ROUTER_SOFTMAX_GROUPS && f.correction && outputs <= kMaxRouted && f.groups && outputs % f.groups == 0 && f.keep && f.keep <= f.groups &&
+         top && (uint64_t)f.keep * (outputs / f.groups) >= top && f.identity < outputs;
+}
+
 hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st, int src) {
+  if (a.bias && (a.paired || a.post.xout)) return hipErrorInvalidValue;
   if ((a.n && src != LS_EXPERTS && !a.w && !(src == LS_MOE_DOWN && a.kps == 0)) || (a.n && !a.out && !a.post.xout) || (a.n == 0 && src != LS_TWO) || a.kp % 64 ||
       a.kp > kLinMvMaxK || a.k > a.kp || (a.paired && a.n % 32))
     return hipErrorInvalidValue;
   if (src == LS_EXPERTS || src == LS_MOE_DOWN) {
     if (pro != LP_COPY || !a.x || !a.w2 || !a.sel || a.top == 0 || a.top > kMaxTop || a.kpe % 64) return hipErrorInvalidValue;
     if (src == LS_EXPERTS) {
-      if (!a.paired || !a.logits || !a.out || a.experts > kMaxExperts || a.top > a.experts || a.kpe < a.n / 2) return hipErrorInvalidValue;
+      const uint32_t ne = a.experts + a.route.identity;
+      if (!a.paired || !a.logits || !a.out || ne > kMaxExperts || a.top > ne || a.kpe < a.n / 2) return hipErrorInvalidValue;
+      if (a.route.form == LGH_ROUTER_SIGMOID ? a.route.identity != 0 : !route_ok(a.route, ne, a.top) || !a.selw) return hipErrorInvalidValue;
       return lin_mv_run<LP_COPY, LS_EXPERTS, false>(a, st);
     }
-    if (a.paired || a.kps % 64 || a.kpe == 0 || a.kp != a.kps + a.top * a.kpe) return hipErrorInvalidValue;
+    if (a.paired || a.kps % 64 || a.kpe == 0 || a.kp != a.kps + a.top * a.kpe || !a.experts || (a.id_x && (!a.selw || a.post.xout))) return hipErrorInvalidValue;
     return lin_mv_post<LP_COPY, LS_MOE_DOWN>(a, st);
   }
   switch (pro) {
@@ -277,6 +355,7 @@ hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st, int src) {
       return src == LS_PLAIN ? lin_mv_post<LP_COPY, LS_PLAIN>(a, st) : lin_mv_go<LP_COPY>(a, src, st);
     case LP_RESID: return a.x && a.y && a.nw && a.xout ? lin_mv_go<LP_RESID>(a, src, st) : hipErrorInvalidValue;
     case LP_HEAD: return a.x && a.y && a.nw && a.nw2 && a.xout && src == LS_PLAIN && !a.post.xout ? lin_mv_run<LP_HEAD, LS_PLAIN, false>(a, st) : hipErrorInvalidValue;
+    case LP_PRE: return a.x && a.nw2 && (!a.y || a.xout) ? lin_mv_go<LP_PRE>(a, src, st) : hipErrorInvalidValue;
     case LP_MLSTM:
       return a.num && a.nw && a.gate && a.heads * a.vdim == a.k && src == LS_PLAIN ? lin_mv_post<LP_MLSTM, LS_PLAIN>(a, st) : hipErrorInvalidValue;
   }
@@ -397,7 +476,7 @@ __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t
   for (int j = 0; j < MT; j++) {
     const uint32_t m = m0 + (wm * MT + j) * 16 + r16;
     if (m >= m_end) continue;
-    if constexpr (EPI == LE_GEGLU || EPI == LE_SWIGLU) {
+    if constexpr (EPI == LE_GEGLU || EPI == LE_SWIGLU || EPI == LE_CLAMPED) {
       const float in = GRP ? a.grp.scale[m] : 1.0f;            // factor of the row's input
 #pragma unroll
       for (int i = 0; i < NT; i += 2) {
@@ -406,6 +485,7 @@ __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t
         T* o = reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + nb / 2 + g * 4;
 #pragma unroll
         for (int e = 0; e < 4; e++) {
+          if constexpr (EPI == LE_CLAMPED) { o[e] = to_act<T>(in * clamped_glu_f(acc[i][j][e], acc[i + 1][j][e], a.grp.limit)); continue; }
           const float gt = GRP ? in * acc[i][j][e] : acc[i][j][e], u = GRP ? in * acc[i + 1][j][e] : acc[i + 1][j][e];
           o[e] = to_act<T>((EPI == LE_SWIGLU ? silu_f(gt) : gelu_tanh_f(gt)) * u);
         }
@@ -416,6 +496,10 @@ __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t
         const uint32_t nb = n0 + (wn * NT + i) * 16 + g * 4;
         if constexpr (EPI == LE_F32) {
           float* o = reinterpret_cast<float*>(a.out) + (size_t)m * a.ldo + nb;
+          if (a.bias) {
+#pragma unroll
+            for (int e = 0; e < 4; e++) acc[i][j][e] += a.bias[nb + e < a.n ? nb + e : a.n - 1];
+          }
           if (nb + 4 <= a.n && (a.ldo & 3) == 0) *reinterpret_cast<f32x4*>(o) = acc[i][j];
           else
             for (int e = 0; e < 4; e++)
@@ -483,10 +567,11 @@ static hipError_t lin_gemm_group(const LinGemm& a, hipStream_t st) {
 hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st) {
   const uint32_t el = f32 ? 4 : 2;
   if (!a.w || !a.x || !a.out || a.n == 0 || a.M == 0 || a.kp % 64 || a.ldx < a.kp || (a.ldx * el) % 16 || a.np % 16 || a.n > a.np) return hipErrorInvalidValue;
-  if ((epi == LE_GEGLU || epi == LE_SWIGLU) && a.n % 32) return hipErrorInvalidValue;
+  if ((epi == LE_GEGLU || epi == LE_SWIGLU || epi == LE_CLAMPED) && a.n % 32) return hipErrorInvalidValue;
   if (a.grp.tiles) {
-    if (!a.grp.seg || !a.grp.tile_e || !a.grp.tile_row || (epi == LE_SWIGLU && !a.grp.scale)) return hipErrorInvalidValue;
+    if (!a.grp.seg || !a.grp.tile_e || !a.grp.tile_row || ((epi == LE_SWIGLU || epi == LE_CLAMPED) && !a.grp.scale)) return hipErrorInvalidValue;
     if (epi == LE_SWIGLU) return f32 ? lin_gemm_group<float, LE_SWIGLU>(a, st) : lin_gemm_group<__bf16, LE_SWIGLU>(a, st);
+    if (epi == LE_CLAMPED) return f32 ? lin_gemm_group<float, LE_CLAMPED>(a, st) : lin_gemm_group<__bf16, LE_CLAMPED>(a, st);
     if (epi == LE_F32) return f32 ? lin_gemm_group<float, LE_F32>(a, st) : lin_gemm_group<__bf16, LE_F32>(a, st);
     return hipErrorInvalidValue;
   }

@@ -18,7 +18,6 @@
 namespace lgh {
 
 __device__ __forceinline__ float gate_in(float z, float cap) { return cap * tanhf(z / cap); }
-__device__ __forceinline__ float log_sigmoid_f(float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
 
 // ------------------------------------------------------------------------------------------------
 // decode: one token.  A workgroup owns 16 columns of one head's state (4 lanes x 4 columns, 64 rows at a time).
@@ -247,7 +246,8 @@ __global__ void __launch_bounds__(256) mlstm_n_kernel(const MlstmShape s, const 
 // accumulators (NT tiles of 16 rows).  A tile's register e of lane (column r16, group g) is row 4g + e — exactly what the j = e-th
 // f32 product wants as its B operand, so the state is multiplied where it lies.  The workgroups are few (one per CU and less), so the
 // next chunk's operands are requested into registers while the current one is computed (PRE; large dims have no registers for it).
-template <int NT, int NW, bool PRE, bool VEC>
+// ROWS: queries and keys carry their decays already, and the state's rows decay each at its own rate (rowdec).
+template <int NT, int NW, bool PRE, bool VEC, bool ROWS>
 __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShape s, const MlstmBufs b, uint32_t pos0, uint32_t M) {
   __shared__ f32x4 part[2][NW][4][64];   // [chunk parity][wave][token tile][lane]
   const uint32_t h = blockIdx.y, c0 = blockIdx.x * 16, lane = threadIdx.x & 63;
@@ -256,7 +256,7 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
   const uint32_t dbase = w * NT * 16;
   const float* dec = b.dec + (size_t)h * b.Mcap;
   const float* wgt = b.wgt + (size_t)h * b.Mcap;
-  const float* cdec = b.cdec + (size_t)h * (b.Mcap / 64);
+  const float* cdec = ROWS ? nullptr : b.cdec + (size_t)h * (b.Mcap / 64);
   float* Sg = b.S + (size_t)h * s.dim * s.lds;
   const uint32_t qo = s.off_q + h * s.dim + dbase + g * 4, ko = s.off_k + h * s.dim + dbase + r16, vo = s.off_v + h * s.vdim + (c < s.vdim ? c : 0);
   const bool ragged = s.dim != NT * NW * 16;   // rows past dim: never stored, kept 0
@@ -270,28 +270,35 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
       const float v = Sg[ok ? (size_t)d * s.lds + c : 0];
       S[i][e] = pos0 && ok ? v : 0.0f;
     }
-  struct Ops { f32x4 q[NT][4]; f32x4 k[NT][4]; f32x4 v[4], wg[4], dc[4], a[4]; float cd; };
+  struct Ops { f32x4 q[NT][4]; f32x4 k[NT][4]; f32x4 v[4], wg[4], dc[4], a[4], rd[ROWS ? NT : 1]; float cd; };
   // a chunk's operands: q tiles (lane: token r16 of tile j, 4 dims), k (lane: dim r16, tokens 4g ..), v, factors, the wave's score columns.
   // Tokens past the end re-read the last one: their weight is 0 and their numerators are not stored.
   auto fetch = [&](uint32_t ch, Ops& x) {
     const uint32_t t0 = ch * 64;
 #pragma unroll
     for (int j = 0; j < 4; j++) {
-      const uint32_t t = t0 + j * 16 + r16, ro = (t < M ? t : M - 1) * s.ldcat + qo;
+      const uint32_t t = t0 + j * 16 + r16, ro = (t < M ? t : M - 1) * s.ldqk + qo;
 #pragma unroll
-      for (int i = 0; i < NT; i++) x.q[i][j] = row4<VEC>(b.cat, ro + i * 16);
+      for (int i = 0; i < NT; i++) x.q[i][j] = row4<VEC>(b.qk, ro + i * 16);
 #pragma unroll
       for (int e = 0; e < 4; e++) {
-        const uint32_t ts = t0 + j * 16 + g * 4 + e, tsc = ts < M ? ts : M - 1, so = tsc * s.ldcat;
-        x.v[j][e] = row1(b.cat, so + vo);   // (columns past vdim: computed, never stored)
-        x.wg[j][e] = row1(wgt, ts);   // (0 behind the block's last token)
-        x.dc[j][e] = row1(dec, tsc);
+        const uint32_t ts = t0 + j * 16 + g * 4 + e, tsc = ts < M ? ts : M - 1;
+        x.v[j][e] = row1(b.cat, tsc * s.ldcat + vo);   // (columns past vdim: computed, never stored)
+        if constexpr (!ROWS) {
+          x.wg[j][e] = row1(wgt, ts);   // (0 behind the block's last token)
+          x.dc[j][e] = row1(dec, tsc);
+        }
 #pragma unroll
-        for (int i = 0; i < NT; i++) x.k[i][j][e] = row1(b.cat, so + ko + i * 16);
+        for (int i = 0; i < NT; i++) x.k[i][j][e] = row1(b.qk, (ROWS ? ts : tsc) * s.ldqk + ko + i * 16);   // (ROWS: zeros behind the last token)
       }
       x.a[j] = *reinterpret_cast<const f32x4*>(b.a + ((size_t)ch * s.heads + h) * 4096 + (j * 16 + r16) * 64 + (w & 3) * 16 + g * 4);
     }
-    x.cd = cdec[ch];
+    if constexpr (ROWS) {
+#pragma unroll
+      for (int i = 0; i < NT; i++) x.rd[i] = row4<VEC>(b.rowdec, (ch * s.heads + h) * s.dim + dbase + g * 4 + i * 16);
+    } else {
+      x.cd = cdec[ch];
+    }
   };
   auto chunk = [&](uint32_t ch, const Ops& x) {
     const uint32_t t0 = ch * 64;
@@ -311,16 +318,19 @@ __global__ void __launch_bounds__(NW * 64, 1) mlstm_state_kernel(const MlstmShap
     }
 #pragma unroll
     for (int j = 0; j < 4; j++) {
-      o[j] *= x.dc[j];
+      if constexpr (!ROWS) o[j] *= x.dc[j];
       if (w < 4) o[j] = Frag<float>::mma(x.a[j], vw, o[j]);   // (scores of later keys are stored as zeros)
       part[ch & 1][w][j][lane] = o[j];
     }
     // the state at the chunk's end
 #pragma unroll
-    for (int i = 0; i < NT; i++) S[i] *= x.cd;
+    for (int i = 0; i < NT; i++) {
+      if constexpr (ROWS) S[i] *= x.rd[i];
+      else S[i] *= x.cd;
+    }
 #pragma unroll
     for (int j = 0; j < 4; j++) {
-      const f32x4 wv = x.v[j] * x.wg[j];
+      const f32x4 wv = ROWS ? x.v[j] : x.v[j] * x.wg[j];
 #pragma unroll
       for (int i = 0; i < NT; i++) S[i] = Frag<float>::mma(x.k[i][j], wv, S[i]);
     }
@@ -379,25 +389,34 @@ hipError_t mlstm_block_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t 
     }
     return hipSuccess;
   }
-  const dim3 gs((s.vdim + 15) / 16, s.heads), t(256);
+  const dim3 t(256);
   hipLaunchKernelGGL(mlstm_gates_kernel, dim3(s.heads), dim3(1024), 0, st, s, b, pos0, M);
   const bool vec = (s.dim & 3) == 0 && (s.ldcat & 3) == 0 && (s.off_q & 3) == 0 && (s.off_k & 3) == 0;
   const dim3 gq((M + 63) / 64, s.heads);
   if (vec) hipLaunchKernelGGL(mlstm_scores_kernel<true>, gq, t, 0, st, s, b, M);
   else hipLaunchKernelGGL(mlstm_scores_kernel<false>, gq, t, 0, st, s, b, M);
   hipLaunchKernelGGL(mlstm_n_kernel, dim3((s.dim + 255) / 256, s.heads), t, 0, st, s, b, pos0, M);
+  return mlstm_state_launch(s, b, pos0, M, st);
+}
+
+template <bool VEC, bool ROWS>
+static hipError_t mlstm_state_go(const MlstmShape& s, const MlstmBufs& b, uint32_t pos0, uint32_t M, hipStream_t st) {
   const uint32_t nt = (s.dim + 63) / 64;
-#define LGH_STATE(N, W, P)                                                                                      \
-  do {                                                                                                          \
-    if (vec) hipLaunchKernelGGL((mlstm_state_kernel<N, W, P, true>), gs, dim3(W * 64), 0, st, s, b, pos0, M);   \
-    else hipLaunchKernelGGL((mlstm_state_kernel<N, W, P, false>), gs, dim3(W * 64), 0, st, s, b, pos0, M);      \
-  } while (0)
+  const dim3 gs((s.vdim + 15) / 16, s.heads);
+#define LGH_STATE(N, W, P) hipLaunchKernelGGL((mlstm_state_kernel<N, W, P, VEC, ROWS>), gs, dim3(W * 64), 0, st, s, b, pos0, M)
   if (nt <= 1) LGH_STATE(1, 4, true);
   else if (nt <= 2) LGH_STATE(2, 4, true);
   else if (nt <= 4) LGH_STATE(4, 4, true);
   else LGH_STATE(4, 8, false);
 #undef LGH_STATE
   return hipGetLastError();
+}
+
+hipError_t mlstm_state_launch(const MlstmShape& s, const MlstmBufs& b, uint32_t pos0, uint32_t M, hipStream_t st) {
+  if (M == 0 || M > b.Mcap || b.Mcap % 64 || s.dim > kMlstmBlockDim || !b.qk || s.lds < s.vdim) return hipErrorInvalidValue;
+  const bool vec = (s.dim & 3) == 0 && (s.ldqk & 3) == 0 && (s.off_q & 3) == 0 && (s.off_k & 3) == 0;
+  if (b.rowdec) return vec ? mlstm_state_go<true, true>(s, b, pos0, M, st) : mlstm_state_go<false, true>(s, b, pos0, M, st);
+  return vec ? mlstm_state_go<true, false>(s, b, pos0, M, st) : mlstm_state_go<false, false>(s, b, pos0, M, st);
 }
 
 // ------------------------------------------------------------------------------------------------

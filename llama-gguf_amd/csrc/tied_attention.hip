@@ -58,24 +58,6 @@ __host__ __device__ constexpr uint32_t tied_lanes(uint32_t dp, uint32_t el) {
 constexpr uint32_t kTiedBatch = 4;   // key rows a lane has in flight
 __host__ __device__ constexpr uint32_t tied_round(uint32_t lanes) { return 4 * kTiedBatch * (64 / lanes); }   // keys of a workgroup per round
 
-// sum over `N` neighbouring lanes, every one of them gets it
-template <uint32_t N> __device__ __forceinline__ float lanes_sum(float v) {
-  v += dpp_f<0xB1>(v); v += dpp_f<0x4E>(v); v += dpp_f<0x141>(v);
-  if constexpr (N >= 16) v += dpp_f<0x140>(v);
-  if constexpr (N >= 32) v += __shfl_xor(v, 16, 64);
-  if constexpr (N >= 64) v += __shfl_xor(v, 32, 64);
-  return v;
-}
-
-template <class T, int PER> __device__ __forceinline__ void unpack_row(const u32x4& w, float* f) {
-  if constexpr (sizeof(T) == 2) {
-    f[0] = bf_lo(w.x); f[1] = bf_hi(w.x); f[2] = bf_lo(w.y); f[3] = bf_hi(w.y);
-    f[4] = bf_lo(w.z); f[5] = bf_hi(w.z); f[6] = bf_lo(w.w); f[7] = bf_hi(w.w);
-  } else {
-    f[0] = __uint_as_float(w.x); f[1] = __uint_as_float(w.y); f[2] = __uint_as_float(w.z); f[3] = __uint_as_float(w.w);
-  }
-}
-
 // PER values of a head's row from d0 on, 0 behind its end; vec: rows start and end at multiples of 4
 template <int PER> __device__ __forceinline__ void row_chunk(const float* p, uint32_t d0, uint32_t dim, bool vec, float* o) {
   if (vec) {

@@ -72,6 +72,49 @@ def _tied_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
             raise ConfigError(f"{where}: a window of {layer.window} positions")
 
 
+def _rotation(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    rot = mx.get("rot")
+    if rot:
+        layer.rot_dims, layer.rot_base = int(_need(rot, "dims", where)), float(_need(rot, "base", where))
+        if layer.rot_dims % 2 or layer.rot_dims > layer.dim:
+            raise ConfigError(f"{where}: {layer.rot_dims} rotated values of {layer.dim}")
+
+
+def _gated_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_GATED_ATTENTION
+    _sizes(layer, mx, where, heads="heads", kv_heads="kv_heads", dim="dim", vdim="vdim")
+    if not layer.kv_heads or layer.heads % layer.kv_heads:
+        raise ConfigError(f"{where}: {layer.heads} heads do not divide into {layer.kv_heads} key heads")
+    layer.scale = float(_need(mx, "scale", where))
+    _rotation(layer, mx, where)
+    mask = mx.get("mask")
+    if mask:
+        layer.chunk = int(_need(mask, "size", where))
+        if layer.chunk < 1:
+            raise ConfigError(f"{where}: chunks of {layer.chunk} positions")
+
+
+def _gla(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_GLA
+    _sizes(layer, mx, where, gla_heads="heads", gla_dim="dim", gla_vdim="vdim")
+    layer.gla_tau = float(_need(mx, "tau", where))
+
+
+def _parallel(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    _gated_attention(layer, _need(mx, "left", where), where + " left")
+    _gla(layer, _need(mx, "right", where), where + " right")
+    layer.mixer = hb.MIXER_PARALLEL
+    layer.left_scale, layer.right_scale = float(_need(mx, "left_scale", where)), float(_need(mx, "right_scale", where))
+
+
+def _rglru(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_GLRU
+    width, layer.heads, layer.taps = (int(_need(mx, k, where)) for k in ("width", "blocks", "conv"))
+    if layer.heads < 1 or width % layer.heads or layer.taps < 1:
+        raise ConfigError(f"{where}: {width} channels, {layer.heads} blocks, {layer.taps} taps")
+    layer.dim = layer.vdim = width // layer.heads
+
+
 def _dense(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
     layer.ff_kind, layer.ff = hb.FF_GEGLU, int(_need(mlp, "ff", where))
 
@@ -84,8 +127,23 @@ def _moe(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
         layer.shared_ff = int(_need(mlp["shared"], "ff", where))
 
 
-MIXERS = {"latent_attention": _latent_attention, "mlstm": _mlstm, "attention": _tied_attention}
-FEED_FORWARDS = {"dense": _dense, "moe": _moe}
+def _grouped_moe(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
+    """Clamped experts, chosen by corrected softmax scores among the best groups; router outputs without tensors hand the input back."""
+    _moe(layer, mlp, where)
+    layer.router_form, layer.expert_form = hb.ROUTER_SOFTMAX_GROUPS, hb.EXPERT_CLAMPED
+    layer.expert_limit = float(_need(mlp["expert"], "limit", where))
+    router = mlp["router"]
+    groups = router.get("groups") or {"count": 1, "keep": 1}
+    layer.groups, layer.keep_groups = int(_need(groups, "count", where)), int(_need(groups, "keep", where))
+    layer.identity = int(router.get("identity") or 0)
+    n = layer.experts + layer.identity
+    if layer.groups < 1 or n % layer.groups or not 1 <= layer.keep_groups <= layer.groups or layer.keep_groups * (n // layer.groups) < layer.top:
+        raise ConfigError(f"{where}: {n} router outputs, {layer.groups} groups of which {layer.keep_groups} stay open, {layer.top} per token")
+
+
+MIXERS = {"latent_attention": _latent_attention, "mlstm": _mlstm, "attention": _tied_attention, "gated_attention": _gated_attention, "gla": _gla,
+          "parallel": _parallel, "rglru": _rglru}
+FEED_FORWARDS = {"dense": _dense, "moe": _moe, "grouped_moe": _grouped_moe}
 
 
 @dataclass
@@ -99,6 +157,8 @@ class LayeredConfig:
     bigram: Optional[Tuple[int, int, int]] = None      # buckets, factor of the previous token, factor of the token
     residual: int = hb.RESIDUAL_POST_LN
     conv_taps: int = 0
+    tied_head: bool = False                            # the output projection is the embedding table
+    logit_scale: float = 1.0
 
     @property
     def num_layers(self) -> int:
@@ -110,6 +170,7 @@ class LayeredConfig:
         d.width, d.vocab_size, d.num_layers = self.hidden_size, self.vocab_size, self.num_layers
         d.norm_eps, d.residual_mult = self.norm_eps, self.residual_mult
         d.residual, d.conv_taps = self.residual, self.conv_taps
+        d.tied_head, d.logit_scale = int(self.tied_head), self.logit_scale
         if self.bigram:
             d.bigram_buckets, d.bigram_mul_prev, d.bigram_mul_cur = self.bigram
         return d
@@ -130,6 +191,50 @@ class LayeredConfig:
             yield from self._norm_shapes(f"{p}norm{which}b")
         if self.conv_taps:
             yield f"{p}canon{which}", (self.hidden_size, self.conv_taps)
+
+    def resolve(self, shape_of) -> "LayeredConfig":
+        """Sizes that only a tensor's shape tells; shape_of(name) -> shape or None."""
+        for i, l in enumerate(self.layers):
+            if l.mixer in (hb.MIXER_GLA, hb.MIXER_PARALLEL):
+                name = f"l{i}.mix.{'right.' if l.mixer == hb.MIXER_PARALLEL else ''}a1"
+                shape = shape_of(name)
+                if shape is None or len(shape) != 2 or shape[0] < 1:
+                    raise ConfigError(f"tensor '{name}': shape {shape} does not tell the decay's inner size")
+                l.gla_rank = int(shape[0])
+        return self
+
+    def _gated_shapes(self, p: str, l) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        W = self.hidden_size
+        for n, rows in (("q", l.heads * l.dim), ("k", l.kv_heads * l.dim), ("v", l.kv_heads * l.vdim)):
+            yield p + n, (rows, W)
+            yield p + n + ".b", (rows,)
+        yield p + "q.norm", (l.dim,)
+        yield p + "k.norm", (l.dim,)
+        yield p + "g", (l.heads * l.vdim, W)
+        yield p + "o", (W, l.heads * l.vdim)
+
+    def _gla_shapes(self, p: str, l) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        W, hd, vd = self.hidden_size, l.gla_heads * l.gla_dim, l.gla_heads * l.gla_vdim
+        for n, rows in (("q", hd), ("k", hd), ("v", vd), ("g", vd)):
+            yield p + n, (rows, W)
+        yield p + "o", (W, vd)
+        yield p + "norm", (l.gla_vdim,)
+        yield p + "a1", (l.gla_rank, W)
+        yield p + "a2", (hd, l.gla_rank)
+        yield p + "a2.b", (hd,)
+
+    def _rglru_shapes(self, p: str, l) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        W, n = self.hidden_size, l.heads * l.dim
+        for b in ("y", "x"):
+            yield p + b, (n, W)
+            yield p + b + ".b", (n,)
+        yield p + "conv", (n, l.taps)
+        yield p + "conv.b", (n,)
+        for g in ("ra", "ri"):
+            yield p + g, (l.heads, l.dim, l.dim)
+            yield p + g + ".b", (l.heads, l.dim)
+        yield p + "lam", (n,)
+        yield p + "o", (W, n)
 
     def tensor_shapes(self) -> Iterator[Tuple[str, Tuple[int, ...]]]:
         """(name, shape) of every tensor the model needs, [out, in]."""
@@ -154,6 +259,15 @@ class LayeredConfig:
                     yield p + "mix." + n + ".norm", (rows,)
                 yield p + "mix.temp", (l.heads,)
                 yield p + "mix.sink", (l.heads,)
+            elif l.mixer == hb.MIXER_GATED_ATTENTION:
+                yield from self._gated_shapes(p + "mix.", l)
+            elif l.mixer == hb.MIXER_GLA:
+                yield from self._gla_shapes(p + "mix.", l)
+            elif l.mixer == hb.MIXER_PARALLEL:
+                yield from self._gated_shapes(p + "mix.left.", l)
+                yield from self._gla_shapes(p + "mix.right.", l)
+            elif l.mixer == hb.MIXER_GLRU:
+                yield from self._rglru_shapes(p + "mix.", l)
             else:
                 yield p + "mix.q", (l.heads * l.dim, W)
                 yield p + "mix.k", (l.heads * l.dim, W)
@@ -163,11 +277,14 @@ class LayeredConfig:
                 for g in ("i", "f"):
                     yield p + "mix." + g, (l.heads, W)
                     yield p + "mix." + g + ".b", (l.heads,)
-            yield p + "mix.o", (W, vd)
+            if l.mixer in (hb.MIXER_LATENT_ATTENTION, hb.MIXER_TIED_ATTENTION, hb.MIXER_MLSTM):
+                yield p + "mix.o", (W, vd)
             if l.ff_kind:
                 yield from self._sublayer_shapes(p, 2)
             if l.ff_kind == hb.FF_MOE:
-                yield p + "mlp.router", (l.experts, W)
+                yield p + "mlp.router", (l.experts + l.identity, W)
+                if l.router_form == hb.ROUTER_SOFTMAX_GROUPS:
+                    yield p + "mlp.correction", (l.experts + l.identity,)
                 for e in range(l.experts):
                     yield from ff(f"{p}mlp.e{e}.", l.ff)
                 if l.shared_ff:
@@ -175,7 +292,8 @@ class LayeredConfig:
             elif l.ff_kind:
                 yield from ff(p + "mlp.", l.ff)
         yield from self._norm_shapes("final.norm")
-        yield "head", (self.vocab_size, W)
+        if not self.tied_head:
+            yield "head", (self.vocab_size, W)
 
 
 def _zamelix(cfg: dict) -> LayeredConfig:
@@ -204,8 +322,21 @@ def _pubopel(cfg: dict) -> LayeredConfig:
     return out
 
 
-def _layers(out: LayeredConfig, cfg: dict, where: str) -> None:
-    """The 'layers' list: a mixer and an optional feed-forward each."""
+def _sumevik(cfg: dict) -> LayeredConfig:
+    """Gated linear recurrences, and gated chunked attention beside gated linear attention, in any order; dense feed-forwards or grouped mixtures;
+    RMS norms in front of the sublayers; the embedding table as output projection."""
+    where = "Sumevik"
+    out = LayeredConfig(where, int(_need(cfg, "width", where)), int(_need(cfg, "vocab", where)),
+                        float(_need(_need(cfg, "norm", where), "eps", where)), 1.0, residual=hb.RESIDUAL_PRE_RMS, tied_head=True)
+    out.logit_scale = float(_need(cfg, "logit_scale", where))
+    if not out.logit_scale:
+        raise ConfigError(f"{where}: logit_scale is 0")
+    _layers(out, cfg, where, dict(FEED_FORWARDS, moe=_grouped_moe))
+    return out
+
+
+def _layers(out: LayeredConfig, cfg: dict, where: str, feed_forwards: dict = FEED_FORWARDS) -> None:
+    """The 'layers' list: a mixer and an optional feed-forward each; feed_forwards: what a design calls its own."""
     for i, entry in enumerate(_need(cfg, "layers", where)):
         at = f"{where} layer {i}"
         layer = hb.LayerDesc()
@@ -216,13 +347,13 @@ def _layers(out: LayeredConfig, cfg: dict, where: str) -> None:
         MIXERS[kind](layer, _need(entry, "mixer", at), at)
         mlp = entry.get("mlp")
         if mlp:
-            if _need(mlp, "kind", at) not in FEED_FORWARDS:
+            if _need(mlp, "kind", at) not in feed_forwards:
                 raise ConfigError(f"{at}: unknown feed-forward '{mlp['kind']}'")
-            FEED_FORWARDS[mlp["kind"]](layer, mlp, at)
+            feed_forwards[mlp["kind"]](layer, mlp, at)
         out.layers.append(layer)
 
 
-ARCHITECTURES = {"Zamelix": _zamelix, "Pubopel": _pubopel}      # config.json "architecture" -> parser
+ARCHITECTURES = {"Zamelix": _zamelix, "Pubopel": _pubopel, "Sumevik": _sumevik}      # config.json "architecture" -> parser
 
 
 def parse_config(cfg: dict) -> LayeredConfig:
@@ -244,6 +375,10 @@ class SafetensorsFile:
             self.header = json.loads(f.read(n))
         self.header.pop("__metadata__", None)
         self._data = np.memmap(path, dtype=np.uint8, mode="r", offset=8 + n) if size > 8 + n else np.zeros(0, np.uint8)
+
+    def shape(self, name: str) -> Optional[Tuple[int, ...]]:
+        h = self.header.get(name)
+        return None if h is None else tuple(h["shape"])
 
     def get(self, name: str, shape: Tuple[int, ...]) -> Tuple[int, np.ndarray]:
         """(ggml type, bytes) of a tensor, checked against the shape the model needs."""
@@ -269,7 +404,8 @@ class LayeredModel:
     def from_dir(cls, path: str) -> "LayeredModel":
         with open(os.path.join(path, "config.json")) as f:
             cfg = parse_config(json.load(f))
-        return cls(cfg, SafetensorsFile(os.path.join(path, "model.safetensors")))
+        source = SafetensorsFile(os.path.join(path, "model.safetensors"))
+        return cls(cfg.resolve(source.shape), source)
 
     def tensors(self):
         for name, shape in self.config.tensor_shapes():
