@@ -123,7 +123,8 @@ def parse_args():
     ap.add_argument("--fake-stage", action="store_true",
                     help="CPU rehearsal of the N>1 launcher and hop protocol: gloo + pipeline.FakeStage, no GPU, no engine (not a measurement)")
     ap.add_argument("--layered", default="", metavar="SIZE[,SIZE]",
-                    help="models described layer by layer (w*: latent attention + matrix memory; p*: windowed tied attention + mixtures) beside the "
+                    help="models described layer by layer (w*: latent attention + matrix memory; p*: windowed tied attention + mixtures; s*: linear recurrences + "
+                         "gated attention beside gated linear attention) beside the "
                          "Llama-style model of equal width, depth and feed-forward, random weights: " + ", ".join(LAYERED_SIZES) + " or all; not the headline metric")
     ap.add_argument("--layered-only", choices=("both", "layered", "closest"), default="both", help="with --layered: run one side (for a profiler)")
     ap.add_argument("--layered-context", type=int, default=2048, help="with --layered: prompt length")
@@ -148,6 +149,16 @@ LAYERED_SIZES = {
                    closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),   # (the closest model takes prompts of this one token by token)
     "p8192": dict(design="Pubopel", width=8192, ff=8192, vocab=32000, layers=2, heads=64, kv_heads=8, dim=128, window=4096, experts=8, top=2, shared=8192,
                   closest=dict(num_heads=64, num_kv_heads=8, head_dim=128)),
+    # gated linear recurrences and gated attention beside gated linear attention in turn, dense feed-forwards or grouped mixtures with identity experts
+    "s2048": dict(design="Sumevik", width=2048, ff=5632, vocab=32000, layers=8, heads=16, kv_heads=4, dim=128, vdim=128, chunk=8192, blocks=8, gheads=8, gdim=128,
+                  gvdim=256, rank=16, closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),
+    "s4096": dict(design="Sumevik", width=4096, ff=14336, vocab=128256, layers=8, heads=32, kv_heads=8, dim=128, vdim=128, chunk=8192, blocks=16, gheads=16, gdim=128,
+                  gvdim=256, rank=16, closest=dict(num_heads=32, num_kv_heads=8, head_dim=128)),
+    "s4096m": dict(design="Sumevik", width=4096, ff=4096, vocab=32000, layers=4, heads=32, kv_heads=8, dim=128, vdim=128, chunk=8192, blocks=16, gheads=16, gdim=128,
+                   gvdim=256, rank=16, experts=8, top=2, identity=4, groups=4, keep=3, closest=dict(num_heads=32, num_kv_heads=8, head_dim=128)),
+    "s2048e": dict(design="Sumevik", width=2048, ff=768, vocab=32000, layers=8, heads=16, kv_heads=4, dim=128, vdim=128, chunk=1024, blocks=8, gheads=8, gdim=128,
+                   gvdim=256, rank=16, experts=64, top=6, identity=16, groups=8, keep=4,
+                   closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),   # (the closest model takes prompts of this one token by token)
 }
 
 
@@ -167,6 +178,18 @@ class RandomBf16:
 
 
 def layered_config(sz):
+    if sz.get("design") == "Sumevik":
+        W = sz["width"]
+        mlp = {"kind": "dense", "ff": sz["ff"]} if "experts" not in sz else {
+            "kind": "moe", "expert": {"ff": sz["ff"], "limit": 7.0},
+            "router": {"experts": sz["experts"], "top": sz["top"], "identity": sz["identity"], "groups": {"count": sz["groups"], "keep": sz["keep"]}}}
+        rec = {"type": "rglru", "mlp": mlp, "mixer": {"width": W, "blocks": sz["blocks"], "conv": 4}}
+        par = {"type": "parallel", "mlp": mlp, "mixer": {
+            "left": {"heads": sz["heads"], "kv_heads": sz["kv_heads"], "dim": sz["dim"], "vdim": sz["vdim"], "scale": sz["dim"] ** -0.5, "mask": {"size": sz["chunk"]},
+                     "rot": {"base": 10000.0, "dims": sz["dim"] // 2}},
+            "right": {"heads": sz["gheads"], "dim": sz["gdim"], "vdim": sz["gvdim"], "tau": 16.0}, "left_scale": 1.0, "right_scale": 1.0}}
+        return {"architecture": "Sumevik", "width": W, "vocab": sz["vocab"], "norm": {"eps": 1e-6}, "logit_scale": 1.0,
+                "layers": [par if i % 2 else rec for i in range(sz["layers"])]}
     if sz.get("design") == "Pubopel":
         layer = {"type": "attention", "mlp": {"kind": "moe", "expert": {"ff": sz["ff"]}, "router": {"experts": sz["experts"], "top": sz["top"]}, "shared": {"ff": sz["shared"]}},
                  "mixer": {"heads": sz["heads"], "kv_heads": sz["kv_heads"], "dim": sz["dim"], "vdim": sz["dim"], "scale": sz["dim"] ** -0.5, "softcap": 30.0,
@@ -226,7 +249,7 @@ def run_layered(args, pkg):
         prompt = prompt_tokens(n, sz["vocab"])
         cap = n + steps * (args.reps + 1) + 64
         if args.layered_only != "closest":
-            cfg = pkg.layered_model.parse_config(layered_config(sz))
+            cfg = pkg.layered_model.parse_config(layered_config(sz)).resolve(lambda name: (sz["rank"], sz["width"]))
             eng = pkg.HipGpuInference.from_layered(pkg.LayeredModel(cfg, RandomBf16()), cap)
             r["layered"] = layered_measure(eng, prompt, steps, args.reps)
             eng.close()

@@ -73,57 +73,53 @@ __device__ __forceinline__ void gattn_split(const GattnShape& s, const GattnBufs
     }
   };
   fetch(rb);
-  // a head's row of this token: normed, rotated
-  const f32x2* cs = reinterpret_cast<const f32x2*>(b.cs) + (size_t)pos * (s.rot_n / 2);
-  auto head_row = [&](const float* p, const float* nw, float (*o)[PER]) {
-    float ss = 0.0f, nf[C][PER];
+  // a head's row of this token: normed, rotated.  Everything the rows need is requested before the first of them is used.
+  const bool owner = OWN && re == rounds, kvec = (s.dim & 3) == 0, vvec = (s.vdim & 3) == 0;
+  float q[HQ][C][PER], ok[C][PER], ov[C][PER], nq[C][PER], nk[C][PER];
+  f32x2 cs[C][PER / 2];
+#pragma unroll
+  for (int c = 0; c < C; c++) {
+    row_chunk<PER>(b.qn, d0[c], s.dim, kvec, nq[c]);
+#pragma unroll
+    for (int h = 0; h < HQ; h++) row_chunk<PER>(cat + s.off_q + (size_t)(h0 + ((uint32_t)h < hn ? h : 0)) * s.dim, d0[c], s.dim, kvec, q[h][c]);
+#pragma unroll
+    for (int e = 0; e < PER / 2; e++) {
+      const uint32_t d = d0[c] + 2 * e;
+      cs[c][e].x = 1.0f; cs[c][e].y = 0.0f;
+      if (d < s.rot_n) cs[c][e] = reinterpret_cast<const f32x2*>(b.cs)[(size_t)pos * (s.rot_n / 2) + d / 2];
+    }
+    if (owner) {
+      row_chunk<PER>(b.kn, d0[c], s.dim, kvec, nk[c]);
+      row_chunk<PER>(cat + s.off_k + (size_t)g * s.dim, d0[c], s.dim, kvec, ok[c]);
+      row_chunk<PER>(cat + s.off_v + (size_t)g * s.vdim, d0[c], s.vdim, vvec, ov[c]);
+    }
+  }
+  auto head_row = [&](float (*o)[PER], const float (*nf)[PER], float f) {
+    float ss = 0.0f;
 #pragma unroll
     for (int c = 0; c < C; c++)
 #pragma unroll
-      for (int e = 0; e < PER; e++) {
-        const uint32_t d = d0[c] + e, dc = d < s.dim ? d : 0;
-        const float v = p[dc];
-        nf[c][e] = nw[dc];
-        o[c][e] = d < s.dim ? v : 0.0f;
-        ss = __builtin_fmaf(o[c][e], o[c][e], ss);
-      }
-    const float inv = 1.0f / __builtin_sqrtf(lanes_sum<LPK>(ss) / (float)s.dim + s.eps);
+      for (int e = 0; e < PER; e++) ss = __builtin_fmaf(o[c][e], o[c][e], ss);
+    const float inv = f / __builtin_sqrtf(lanes_sum<LPK>(ss) / (float)s.dim + s.eps);
 #pragma unroll
     for (int c = 0; c < C; c++)
 #pragma unroll
       for (int e = 0; e < PER; e += 2) {
-        const uint32_t d = d0[c] + e;
-        float u = o[c][e] * inv * nf[c][e], v = o[c][e + 1] * inv * nf[c][e + 1];
-        if (d + 1 < s.rot_n) {
-          const f32x2 r = rotate2(u, v, cs[d / 2]);
-          u = r.x; v = r.y;
-        }
-        o[c][e] = u; o[c][e + 1] = v;
+        const f32x2 r = rotate2(o[c][e] * inv * nf[c][e], o[c][e + 1] * inv * nf[c][e + 1], cs[c][e / 2]);
+        o[c][e] = r.x; o[c][e + 1] = r.y;
       }
   };
-  float q[HQ][C][PER], ok[C][PER], ov[C][PER];
-  const float f = s.scale * kGattnLog2e;
 #pragma unroll
-  for (int h = 0; h < HQ; h++) {
-    head_row(cat + s.off_q + (size_t)(h0 + ((uint32_t)h < hn ? h : 0)) * s.dim, b.qn, q[h]);
-#pragma unroll
-    for (int c = 0; c < C; c++)
-#pragma unroll
-      for (int e = 0; e < PER; e++) q[h][c][e] *= f;
-  }
-  const bool owner = OWN && re == rounds;
+  for (int h = 0; h < HQ; h++) head_row(q[h], nq, s.scale * kGattnLog2e);
   if (owner) {
-    head_row(cat + s.off_k + (size_t)g * s.dim, b.kn, ok);
-    const float* vp = cat + s.off_v + (size_t)g * s.vdim;
+    head_row(ok, nk, 1.0f);
 #pragma unroll
     for (int c = 0; c < C; c++) {
       T rk[PER], rv[PER];
 #pragma unroll
       for (int e = 0; e < PER; e++) {
-        const uint32_t d = d0[c] + e;
-        const float v = vp[d < s.vdim ? d : 0];
         rk[e] = to_act<T>(ok[c][e]);
-        rv[e] = to_act<T>(d < s.vdim ? v : 0.0f);
+        rv[e] = to_act<T>(ov[c][e]);
         ok[c][e] = (float)rk[e];
         ov[c][e] = (float)rv[e];
       }
@@ -426,8 +422,10 @@ hipError_t gattn_merge_launch(const GattnShape& s, const GattnBufs& b, const Gla
 }
 
 // ------------------------------------------------------------------------------------------------
-// a block's cache rows and queries; a workgroup per token, a wave per head
+// a block's cache rows and queries; grid (tokens, groups of kPrepHeads heads), a wave per head
 // ------------------------------------------------------------------------------------------------
+constexpr uint32_t kPrepHeads = 8;
+
 template <class T>
 __global__ void __launch_bounds__(256) gattn_prep_kernel(const GattnShape s, const GattnBufs b, uint32_t pos0) {
   const uint32_t t = blockIdx.x, pos = pos0 + t, lane = threadIdx.x & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
@@ -439,7 +437,8 @@ __global__ void __launch_bounds__(256) gattn_prep_kernel(const GattnShape s, con
     __builtin_memcpy(__builtin_assume_aligned(p, sizeof(o)), o, sizeof(o));
   };
   const uint32_t nh = s.heads + s.kv_heads;
-  for (uint32_t i = b.q ? w : s.heads + w; i < nh; i += 4) {
+  const uint32_t i0 = (b.q ? 0 : s.heads) + blockIdx.y * kPrepHeads, i1 = i0 + kPrepHeads < nh ? i0 + kPrepHeads : nh;
+  for (uint32_t i = i0 + w; i < i1; i += 4) {
     const bool key = i >= s.heads;
     const uint32_t h = key ? i - s.heads : i;
     const float* p = cat + (key ? s.off_k : s.off_q) + (size_t)h * s.dim;
@@ -467,14 +466,15 @@ __global__ void __launch_bounds__(256) gattn_prep_kernel(const GattnShape s, con
       if (d < s.dp) store2(o + d, v.x * f, v.y * f);
     }
   }
-  for (uint32_t i = threadIdx.x; i < s.kv_heads * s.vdim; i += 256)
+  for (uint32_t i = blockIdx.y * 256 + threadIdx.x; i < s.kv_heads * s.vdim; i += 256 * gridDim.y)
     reinterpret_cast<T*>(b.vc)[((size_t)(i / s.vdim) * s.rows + pos) * s.vp + i % s.vdim] = to_act<T>(cat[s.off_v + i]);
 }
 
 hipError_t gattn_prep_launch(const GattnShape& s, const GattnBufs& b, uint32_t pos0, uint32_t M, bool f32, hipStream_t st) {
   if (!gattn_ok(s) || M == 0 || (b.q && M > b.Mcap) || pos0 + M > s.rows || (s.rot_n && !b.cs)) return hipErrorInvalidValue;
-  if (f32) hipLaunchKernelGGL((gattn_prep_kernel<float>), dim3(M), dim3(256), 0, st, s, b, pos0);
-  else hipLaunchKernelGGL((gattn_prep_kernel<__bf16>), dim3(M), dim3(256), 0, st, s, b, pos0);
+  const dim3 grid(M, ((b.q ? s.heads : 0) + s.kv_heads + kPrepHeads - 1) / kPrepHeads);
+  if (f32) hipLaunchKernelGGL((gattn_prep_kernel<float>), grid, dim3(256), 0, st, s, b, pos0);
+  else hipLaunchKernelGGL((gattn_prep_kernel<__bf16>), grid, dim3(256), 0, st, s, b, pos0);
   return hipGetLastError();
 }
 

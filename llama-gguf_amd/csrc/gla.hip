@@ -1,7 +1,7 @@
 // gla.hip — gated linear attention of layered.h, all of it in 32-bit: S_t = diag(alpha_t) S_(t-1) + k_t v_t^T per head, o_t = S_t^T q_t, every
 // key channel with a decay of its own, alpha = sigmoid(z)^(1 / tau).
 //
-// Blocks of tokens, 64 at a time.  With b_t the running sum of log alpha within the chunk (b_e at its last token):
+// Blocks of tokens, 64 at a time.  With b_t the running sum of log alpha (in units of log2) within the chunk (b_e at its last token):
 //   o_t = S_p^T (exp(b_t) q_t) + sum_(s<=t) A_ts v_s,   A_ts = sum_d q_td k_sd exp(b_td - b_sd)
 //   S_e = diag(exp(b_e)) S_p + sum_s (exp(b_e - b_s) k_s) v_s^T
 // The state's part is the matrix memory's chunk kernel (mlstm.hip) on queries and keys that carry their decays.  A is formed 16 x 16 tokens at a
@@ -34,7 +34,7 @@ __global__ void __launch_bounds__(256) gla_chunk_kernel(const GlaShape s, const 
   __shared__ float a1s[64][kRankTile];
   const uint32_t ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6));
   const uint32_t r16 = lane & 15, g = lane >> 4, t0 = ch * 64, HD = s.heads * s.dim;
-  const float scale = 1.0f / __builtin_sqrtf((float)s.dim);
+  const float scale = 1.0f / __builtin_sqrtf((float)s.dim), rtau = 1.4426950408889634f / s.tau;
   f32x4 acc[3];                                // scores of group w's tokens with the groups before it
   float dg[4] = {0.0f, 0.0f, 0.0f, 0.0f};      // ... within the group: query r16, keys 4g ..
 #pragma unroll
@@ -75,7 +75,7 @@ __global__ void __launch_bounds__(256) gla_chunk_kernel(const GlaShape s, const 
 #pragma unroll
     for (int i = 0; i < 16; i++) {
       const bool ok = t0 + w * 16 + i < M && d < s.dim;
-      run += ok ? gla_log_decay(z[i] + zb, s.tau) : 0.0f;
+      run += ok ? gla_log2_decay(z[i] + zb, rtau) : 0.0f;
       z[i] = run;
       q[i] = ok ? q[i] * scale : 0.0f;
       k[i] = ok ? k[i] : 0.0f;
@@ -95,10 +95,10 @@ __global__ void __launch_bounds__(256) gla_chunk_kernel(const GlaShape s, const 
 #pragma unroll
       for (int i = 0; i < 16; i++) {           // (rows behind the block's last token: zeros)
         float* o = b.qk + (size_t)(t0 + w * 16 + i) * 2 * HD + row;
-        o[0] = q[i] * expf(before + z[i]);
-        o[HD] = k[i] * expf(after + (run - z[i]));
+        o[0] = q[i] * __builtin_amdgcn_exp2f(before + z[i]);
+        o[HD] = k[i] * __builtin_amdgcn_exp2f(after + (run - z[i]));
       }
-      if (w == 0) b.dec[(size_t)ch * HD + row] = expf(run + after);
+      if (w == 0) b.dec[(size_t)ch * HD + row] = __builtin_amdgcn_exp2f(run + after);
     }
     // scores with the groups before: queries relative to the start of group w
 #pragma unroll
@@ -107,7 +107,7 @@ __global__ void __launch_bounds__(256) gla_chunk_kernel(const GlaShape s, const 
       f32x4 qf = *reinterpret_cast<const f32x4*>(&qs[w * 16 + r16][e0]);
       const f32x4 bq = *reinterpret_cast<const f32x4*>(&bs[w * 16 + r16][e0]);
 #pragma unroll
-      for (int e = 0; e < 4; e++) qf[e] *= expf(bq[e]);
+      for (int e = 0; e < 4; e++) qf[e] *= __builtin_amdgcn_exp2f(bq[e]);
       f32x4 mid = (f32x4)(0.0f);               // groups between
 #pragma unroll
       for (int j = 2; j >= 0; j--) {
@@ -115,7 +115,7 @@ __global__ void __launch_bounds__(256) gla_chunk_kernel(const GlaShape s, const 
         f32x4 kf = *reinterpret_cast<const f32x4*>(&ks[j * 16 + r16][e0]);
         const f32x4 bk = *reinterpret_cast<const f32x4*>(&bs[j * 16 + r16][e0]), tj = *reinterpret_cast<const f32x4*>(&tot[j][e0]);
 #pragma unroll
-        for (int e = 0; e < 4; e++) kf[e] *= expf(mid[e] + (tj[e] - bk[e]));
+        for (int e = 0; e < 4; e++) kf[e] *= __builtin_amdgcn_exp2f(mid[e] + (tj[e] - bk[e]));
         acc[j] = Frag<float>::mma(qf, kf, acc[j]);
         mid += tj;
       }
@@ -128,7 +128,7 @@ __global__ void __launch_bounds__(256) gla_chunk_kernel(const GlaShape s, const 
         const uint32_t key = w * 16 + g * 4 + i;
         const f32x4 kv = *reinterpret_cast<const f32x4*>(&ks[key][e0]), bk = *reinterpret_cast<const f32x4*>(&bs[key][e0]);
 #pragma unroll
-        for (int e = 0; e < 4; e++) dg[i] = __builtin_fmaf(qv[e] * kv[e], expf(fminf(bq[e] - bk[e], 0.0f)), dg[i]);
+        for (int e = 0; e < 4; e++) dg[i] = __builtin_fmaf(qv[e] * kv[e], __builtin_amdgcn_exp2f(fminf(bq[e] - bk[e], 0.0f)), dg[i]);
       }
     }
   }

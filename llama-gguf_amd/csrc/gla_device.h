@@ -5,8 +5,8 @@
 
 namespace lgh {
 
-// z of key channel d (all heads counted through) -> log of its decay
-__device__ __forceinline__ float gla_log_decay(float z, float tau) { return log_sigmoid_f(z) / tau; }
+// z of a key channel -> log2 of its decay; rtau: log2(e) / tau
+__device__ __forceinline__ float gla_log2_decay(float z, float rtau) { return log_sigmoid_f(z) * rtau; }
 
 // One token: a workgroup owns 16 columns (block cb) of head h's state, 4 lanes x 4 columns, 64 rows at a time
 __device__ __forceinline__ void gla_step(const GlaShape& s, const GlaBufs& b, uint32_t pos, uint32_t cb, uint32_t h) {
@@ -41,15 +41,27 @@ __device__ __forceinline__ void gla_step(const GlaShape& s, const GlaBufs& b, ui
       const uint32_t d = d0 + tid, dc = d < s.dim ? d : s.dim - 1;
       const uint16_t* w = b.a2 + ((size_t)h * s.dim + dc) * s.a2_ld;
       float z = b.a2b[(size_t)h * s.dim + dc];
-      for (uint32_t r = 0; r < s.rank; r += 8) {   // (rows of a2 end in zeros)
-        const u32x4 p = *reinterpret_cast<const u32x4*>(w + r);
-        float f[8];
-        unpack_row<__bf16, 8>(p, f);
+      for (uint32_t r0 = 0; r0 < s.rank; r0 += 32) {   // (rows of a2 end in zeros, the segment of a1 at a multiple of 16)
+        u32x4 p[4];
+        f32x4 a[8];
 #pragma unroll
-        for (uint32_t e = 0; e < 8; e++) z = __builtin_fmaf(f[e], a1[r + e < s.rank ? r + e : 0], z);
+        for (uint32_t j = 0; j < 4; j++) {
+          const uint32_t r = r0 + j * 8 < s.rank ? r0 + j * 8 : 0;
+          p[j] = *reinterpret_cast<const u32x4*>(w + r);
+          a[2 * j] = *reinterpret_cast<const f32x4*>(a1 + r);
+          a[2 * j + 1] = *reinterpret_cast<const f32x4*>(a1 + r + 4);
+        }
+#pragma unroll
+        for (uint32_t j = 0; j < 4; j++) {
+          if (r0 + j * 8 >= s.rank) break;
+          float f[8];
+          unpack_row<__bf16, 8>(p[j], f);
+#pragma unroll
+          for (uint32_t e = 0; e < 8; e++) z = __builtin_fmaf(f[e], a[2 * j + e / 4][e & 3], z);
+        }
       }
       if (d0) __syncthreads();
-      al[tid] = expf(gla_log_decay(z, s.tau));
+      al[tid] = __builtin_amdgcn_exp2f(gla_log2_decay(z, 1.4426950408889634f / s.tau));
       __syncthreads();
     }
 #pragma unroll

@@ -17,10 +17,17 @@ constexpr uint32_t kGlruTile = 64, kGlruLd = kGlruTile + 4, kGlruLdB = kGlruTile
 // decay and input factor of a channel from its two gates' pre-activations
 struct GlruStep { float a, x; };
 __device__ __forceinline__ GlruStep glru_coef(float rz, float iz, float sp, float u) {
-  const float la = kGlruRate * sigmoid_f(rz) * sp;
+  const float la = kGlruRate * sigmoid_hw(rz) * sp, y = 2.0f * la;
   GlruStep o;
-  o.a = expf(la);
-  o.x = __builtin_sqrtf(-expm1f(2.0f * la)) * sigmoid_f(iz) * u;
+  o.a = exp_hw(la);
+  // 1 - exp(y): its series where the difference would cancel (next term below 1e-9 of the value), else from a
+  float p = __builtin_fmaf(y, 1.0f / 5040.0f, 1.0f / 720.0f);
+  p = __builtin_fmaf(y, p, 1.0f / 120.0f);
+  p = __builtin_fmaf(y, p, 1.0f / 24.0f);
+  p = __builtin_fmaf(y, p, 1.0f / 6.0f);
+  p = __builtin_fmaf(y, p, 0.5f);
+  p = __builtin_fmaf(y, p, 1.0f);
+  o.x = __builtin_amdgcn_sqrtf(y > -0.25f ? -y * p : __builtin_fmaf(-o.a, o.a, 1.0f)) * sigmoid_hw(iz) * u;
   return o;
 }
 
@@ -79,7 +86,7 @@ __global__ void __launch_bounds__(256) glru_step_kernel(const GlruShape s, const
     const float S = __builtin_fmaf(c.a, pos ? S0 : 0.0f, c.x);   // at position 0 whatever is stored belongs to another sequence
     b.S[ch] = S;
     b.hist[(size_t)((uint32_t)pos % s.taps) * s.width + ch] = xv;
-    out[ch] = S * gelu_tanh_f(yv);
+    out[ch] = S * gelu_tanh_hw(yv);
   }
 }
 
@@ -116,12 +123,11 @@ __device__ __forceinline__ float glru_x(const GlruShape& s, const GlruBufs& b, u
 }
 
 template <class T>
-__global__ void __launch_bounds__(256) glru_gates_kernel(const GlruShape s, const GlruBufs b, uint32_t pos0, uint32_t M) {
+__global__ void __launch_bounds__(256, 3) glru_gates_kernel(const GlruShape s, const GlruBufs b, uint32_t pos0, uint32_t M) {
   constexpr bool BF = sizeof(T) == 2;
-  // the columns' u, as the products' operand: f32, or three bf16 terms; later the tile's factors and inputs
-  constexpr size_t kOp = BF ? 3 * kGlruTile * kGlruLdB * 2 : kGlruTile * kGlruLd * 4, kFac = 2 * kGlruTile * kGlruLd * 4;
-  __shared__ __attribute__((aligned(16))) uint8_t mem[kOp > kFac ? kOp : kFac];
-  __shared__ __attribute__((aligned(16))) float own[kGlruTile][kGlruLd];   // u of the workgroup's own channels
+  // the columns' u, as the products' operand: f32, or three bf16 terms; later the tile's factors
+  __shared__ __attribute__((aligned(16))) uint8_t mem[BF ? 3 * kGlruTile * kGlruLdB * 2 : kGlruTile * kGlruLd * 4];
+  __shared__ __attribute__((aligned(16))) float own[kGlruTile][kGlruLd];   // u of the workgroup's own channels; later the tile's inputs, each in place of its u
   __shared__ float part[4][kGlruTile][2];
   const uint32_t tid = threadIdx.x, lane = tid & 63, w = (uint32_t)__builtin_amdgcn_readfirstlane((int)(tid >> 6)), r16 = lane & 15, g = lane >> 4;
   const uint32_t tiles = (s.bs + 63) / 64, blk = blockIdx.y / tiles, rt = blockIdx.y % tiles, t0 = blockIdx.x * kGlruTile, cb = blk * s.bs;
@@ -131,20 +137,27 @@ __global__ void __launch_bounds__(256) glru_gates_kernel(const GlruShape s, cons
   f32x4 ar[4], ai[4];
 #pragma unroll
   for (int j = 0; j < 4; j++) { ar[j] = (f32x4)(0.0f); ai[j] = (f32x4)(0.0f); }
-  for (uint32_t kc = 0; kc < s.gate_kp / 64; kc++) {
+  const int tw = (int)(t0 + w * 16);
+  // u of 16 tokens of channel 64 kc + lane
+  auto load_u = [&](uint32_t kc, float* u) {
     const uint32_t c = kc * 64 + lane, cc = cb + (c < s.bs ? c : s.bs - 1);
-    const int tw = (int)(t0 + w * 16);
-    float u[16];
     if (s.taps <= 4) {                          // a window of inputs in registers
       float x[19], f[4];
       const float bias = b.conv_b[cc];
 #pragma unroll
       for (int i = 0; i < 4; i++) f[i] = (int)s.taps - 1 - i >= 0 ? b.conv[(size_t)cc * s.taps + (s.taps - 1 - i)] : 0.0f;   // f[i]: i positions back
+      if (tw > 0) {
+        const float* p = b.cat + (size_t)(tw - 3) * s.ldcat + s.off_x + cc;
+        if (tw + 16 <= (int)M) {
 #pragma unroll
-      for (int i = 0; i < 19; i++) {
-        const int t = tw + i - 3, tc = t < (int)M ? t : (int)M - 1;
-        if (t0 > 0 || w > 0) x[i] = b.cat[(size_t)tc * s.ldcat + s.off_x + cc];
-        else x[i] = i >= 3 || (int)s.taps > 3 - i ? glru_x(s, b, pos0, tc, cc) : 0.0f;
+          for (int i = 0; i < 19; i++) x[i] = p[(size_t)i * s.ldcat];
+        } else {
+#pragma unroll
+          for (int i = 0; i < 19; i++) x[i] = b.cat[(size_t)(tw + i - 3 < (int)M ? tw + i - 3 : (int)M - 1) * s.ldcat + s.off_x + cc];
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < 19; i++) x[i] = i >= 3 || (int)s.taps > 3 - i ? glru_x(s, b, pos0, i - 3 < (int)M ? i - 3 : (int)M - 1, cc) : 0.0f;
       }
 #pragma unroll
       for (int i = 0; i < 16; i++) u[i] = __builtin_fmaf(f[0], x[i + 3], __builtin_fmaf(f[1], x[i + 2], __builtin_fmaf(f[2], x[i + 1], __builtin_fmaf(f[3], x[i], bias))));
@@ -160,10 +173,28 @@ __global__ void __launch_bounds__(256) glru_gates_kernel(const GlruShape s, cons
         }
       }
     }
+  };
+  constexpr int NQ = 64 / Frag<T>::KU;
+  struct Wf { u32x4 r[BF ? NQ : 1], i[BF ? NQ : 1]; u32x2 r2[BF ? 1 : NQ], i2[BF ? 1 : NQ]; };   // weights of 64 columns: f32 products take 4 values a unit
+  auto load_w = [&](uint32_t kc, Wf& o) {
+#pragma unroll
+    for (int q = 0; q < NQ; q++) {
+      const uint32_t k = kc * 64 + q * Frag<T>::KU;
+      if constexpr (BF) { o.r[q] = *reinterpret_cast<const u32x4*>(wr + k); o.i[q] = *reinterpret_cast<const u32x4*>(wi + k); }
+      else { o.r2[q] = *reinterpret_cast<const u32x2*>(wr + k); o.i2[q] = *reinterpret_cast<const u32x2*>(wi + k); }
+    }
+  };
+  float u[16];
+  Wf wf;
+  load_w(0, wf);
+  load_u(0, u);
+  const uint32_t chunks = s.gate_kp / 64;
+  for (uint32_t kc = 0; kc < chunks; kc++) {
+    const bool in = kc * 64 + lane < s.bs;
     __syncthreads();                            // the operand before is used up
 #pragma unroll
     for (int i = 0; i < 16; i++) {
-      const float v = c < s.bs ? u[i] : 0.0f;
+      const float v = in ? u[i] : 0.0f;
       const uint32_t t = w * 16 + i;
       if (kc == rt) own[t][lane] = v;
       if constexpr (BF) {
@@ -179,17 +210,17 @@ __global__ void __launch_bounds__(256) glru_gates_kernel(const GlruShape s, cons
       }
     }
     __syncthreads();
+    const Wf cw = wf;
+    if (kc + 1 < chunks) { load_w(kc + 1, wf); load_u(kc + 1, u); }
 #pragma unroll
-    for (int q = 0; q < 64 / Frag<T>::KU; q++) {
+    for (int q = 0; q < NQ; q++) {
       typename Frag<T>::V fr, fi;
-      const uint32_t k = kc * 64 + q * Frag<T>::KU;
       if constexpr (BF) {
-        fr = *reinterpret_cast<const bf16x8*>(wr + k);
-        fi = *reinterpret_cast<const bf16x8*>(wi + k);
+        fr = __builtin_bit_cast(bf16x8, cw.r[q]);
+        fi = __builtin_bit_cast(bf16x8, cw.i[q]);
       } else {
-        const u32x2 hr = *reinterpret_cast<const u32x2*>(wr + k), hi = *reinterpret_cast<const u32x2*>(wi + k);
-        fr.x = bf_lo(hr.x); fr.y = bf_hi(hr.x); fr.z = bf_lo(hr.y); fr.w = bf_hi(hr.y);
-        fi.x = bf_lo(hi.x); fi.y = bf_hi(hi.x); fi.z = bf_lo(hi.y); fi.w = bf_hi(hi.y);
+        fr.x = bf_lo(cw.r2[q].x); fr.y = bf_hi(cw.r2[q].x); fr.z = bf_lo(cw.r2[q].y); fr.w = bf_hi(cw.r2[q].y);
+        fi.x = bf_lo(cw.i2[q].x); fi.y = bf_hi(cw.i2[q].x); fi.z = bf_lo(cw.i2[q].y); fi.w = bf_hi(cw.i2[q].y);
       }
 #pragma unroll
       for (int j = 0; j < 4; j++) {
@@ -210,7 +241,7 @@ __global__ void __launch_bounds__(256) glru_gates_kernel(const GlruShape s, cons
   }
   __syncthreads();
   float* fa = reinterpret_cast<float*>(mem);
-  float* fx = fa + kGlruTile * kGlruLd;
+  float* fx = &own[0][0];
   // lane: channels 4g .. 4g + 3 of the wave's tile, token r16 of token tile j
   const uint32_t cl = w * 16 + g * 4;           // within the 64
   float sp[4], rb[4], ib[4];
@@ -300,7 +331,7 @@ __global__ void __launch_bounds__(256) glru_scan_kernel(const GlruShape s, const
   for (int i = 0; i < 16; i++) {
     const uint32_t t = t0 + w * 16 + i;
     S = __builtin_fmaf(a[i], S, x[i]);
-    if (live && t < M) out[(size_t)t * ldo + c] = to_act<T>(S * gelu_tanh_f(y[i]));
+    if (live && t < M) out[(size_t)t * ldo + c] = to_act<T>(S * gelu_tanh_hw(y[i]));
   }
   if (tile + 1 == gridDim.y && live) {          // what the sequence keeps
     if (w == 3) b.S[c] = S;

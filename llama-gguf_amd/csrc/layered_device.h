@@ -45,6 +45,11 @@ __device__ __forceinline__ float tanh_f(float x) {
   return fabsf(x) < 0.25f ? tanh_series(x) : far;
 }
 
+// exp and sigmoid from the hardware's exp2 and reciprocal (1 ulp each, and the argument's rounding), gelu in its sigmoid form
+__device__ __forceinline__ float exp_hw(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
+__device__ __forceinline__ float sigmoid_hw(float z) { return __builtin_amdgcn_rcpf(1.0f + exp_hw(-z)); }
+__device__ __forceinline__ float gelu_tanh_hw(float z) { return z * sigmoid_hw(1.5957691216057308f * __builtin_fmaf(0.044715f * z * z, z, z)); }
+
 // what is not a number ranks last, so that every place is taken
 __device__ __forceinline__ float rank_key(float z) { return z == z ? z : -INFINITY; }
 
@@ -185,6 +190,24 @@ template <class T, int PER> __device__ __forceinline__ void unpack_row(const u32
     f[4] = bf_lo(w.z); f[5] = bf_hi(w.z); f[6] = bf_lo(w.w); f[7] = bf_hi(w.w);
   } else {
     f[0] = __uint_as_float(w.x); f[1] = __uint_as_float(w.y); f[2] = __uint_as_float(w.z); f[3] = __uint_as_float(w.w);
+  }
+}
+
+// PER values of a head's row from d0 on, 0 behind its end; vec: rows start and end at multiples of 4
+template <int PER> __device__ __forceinline__ void row_chunk(const float* p, uint32_t d0, uint32_t dim, bool vec, float* o) {
+  if (vec) {
+#pragma unroll
+    for (int i = 0; i < PER; i += 4) {
+      const f32x4 v = *reinterpret_cast<const f32x4*>(p + (d0 + i < dim ? d0 + i : 0));
+#pragma unroll
+      for (int e = 0; e < 4; e++) o[i + e] = d0 + i < dim ? v[e] : 0.0f;
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < PER; e++) {
+      const float v = p[d0 + e < dim ? d0 + e : 0];
+      o[e] = d0 + e < dim ? v : 0.0f;
+    }
   }
 }
 

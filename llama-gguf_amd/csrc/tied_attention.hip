@@ -58,23 +58,6 @@ __host__ __device__ constexpr uint32_t tied_lanes(uint32_t dp, uint32_t el) {
 constexpr uint32_t kTiedBatch = 4;   // key rows a lane has in flight
 __host__ __device__ constexpr uint32_t tied_round(uint32_t lanes) { return 4 * kTiedBatch * (64 / lanes); }   // keys of a workgroup per round
 
-// PER values of a head's row from d0 on, 0 behind its end; vec: rows start and end at multiples of 4
-template <int PER> __device__ __forceinline__ void row_chunk(const float* p, uint32_t d0, uint32_t dim, bool vec, float* o) {
-  if (vec) {
-#pragma unroll
-    for (int i = 0; i < PER; i += 4) {
-      const f32x4 v = *reinterpret_cast<const f32x4*>(p + (d0 + i < dim ? d0 + i : 0));
-#pragma unroll
-      for (int e = 0; e < 4; e++) o[i + e] = d0 + i < dim ? v[e] : 0.0f;
-    }
-  } else {
-#pragma unroll
-    for (int e = 0; e < PER; e++) {
-      const float v = p[d0 + e < dim ? d0 + e : 0];
-      o[e] = d0 + e < dim ? v : 0.0f;
-    }
-  }
-}
 // a thread's share (of 256) of the sum of n squares; its first 16 values requested by `squares_fetch`
 struct Squares { f32x4 v[4]; };
 __device__ __forceinline__ void squares_fetch(const float* p, uint32_t n, uint32_t i0, Squares& o) {

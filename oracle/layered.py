@@ -295,7 +295,8 @@ def route_groups(z, correction, router):
     s = np.exp(z - z.max())
     s = s / s.sum()
     c = s + correction
-    n, keep = router["groups"]["count"], router["groups"]["keep"]
+    groups = router.get("groups") or {"count": 1, "keep": 1}
+    n, keep = groups["count"], groups["keep"]
     size = len(z) // n
     best = sorted(range(n), key=lambda g: (-c[g * size:(g + 1) * size].max(), g))[:keep]
     open_ = [e for e in range(len(z)) if e // size in best]
@@ -320,7 +321,7 @@ MIXERS = {"latent_attention": latent_attention, "mlstm": mlstm, "attention": tie
 def feed_forward(x, w, mlp):
     if mlp["kind"] != "moe":
         return dense_ff(x, w)
-    return grouped_moe_ff(x, w, mlp) if "groups" in mlp["router"] else moe_ff(x, w, mlp)
+    return grouped_moe_ff(x, w, mlp) if "limit" in mlp["expert"] else moe_ff(x, w, mlp)
 
 
 def forward_pre_norm(cfg, weights, tokens, layers_out=None):

@@ -46,6 +46,51 @@ def sandwich(layers, width=88, vocab=150, eps=1e-5, taps=3):
     return {"architecture": "Pubopel", "width": width, "vocab": vocab, "norm": {"eps": eps}, "canon": {"taps": taps}, "layers": layers}
 
 
+def rglru(width=96, blocks=3, taps=4, mlp=None):
+    return {"type": "rglru", "mixer": {"width": width, "blocks": blocks, "conv": taps}, "mlp": mlp}
+
+
+def gated(heads=6, kv_heads=2, dim=20, vdim=28, chunk=40, rot=8, base=10000.0, scale=None, mlp=None):
+    """Attention with gated values; chunk 0: no chunks, rot 0: nothing is rotated."""
+    mx = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale or dim ** -0.5}
+    if chunk:
+        mx["mask"] = {"size": chunk}
+    if rot:
+        mx["rot"] = {"base": base, "dims": rot}
+    return {"type": "gated_attention", "mixer": mx, "mlp": mlp}
+
+
+def gla(heads=3, dim=24, vdim=20, tau=16.0, rank=12, mlp=None):
+    """rank is told by a tensor's shape, not by the configuration: the tests keep it beside the layer."""
+    return {"type": "gla", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "tau": tau}, "mlp": mlp, "rank": rank}
+
+
+def parallel(left=None, right=None, scales=(0.8, 1.3), mlp=None):
+    left, right = left or gated(), right or gla()
+    return {"type": "parallel", "mixer": {"left": left["mixer"], "right": right["mixer"], "left_scale": scales[0], "right_scale": scales[1]}, "mlp": mlp, "rank": right["rank"]}
+
+
+def dense(ff=72):
+    return {"kind": "dense", "ff": ff}
+
+
+def grouped(experts=9, identity=3, top=3, ff=40, groups=(4, 2), limit=1.1):
+    router = {"experts": experts, "top": top, "identity": identity}
+    if groups:
+        router["groups"] = {"count": groups[0], "keep": groups[1]}
+    return {"kind": "moe", "expert": {"ff": ff, "limit": limit}, "router": router}
+
+
+def prenorm(layers, width=88, vocab=150, eps=1e-6, logit_scale=1.7):
+    return {"architecture": "Sumevik", "width": width, "vocab": vocab, "norm": {"eps": eps}, "logit_scale": logit_scale, "layers": layers}
+
+
+def parse(pkg, cfg):
+    def shape_of(name):
+        return cfg["layers"][int(name[1:].split(".")[0])].get("rank"), cfg["width"]
+    return pkg.layered_model.parse_config(cfg).resolve(shape_of)
+
+
 def bf16(x):
     """Round to bf16 (nearest even), as f32."""
     u = np.ascontiguousarray(x, np.float32).view(np.uint32)
@@ -59,7 +104,22 @@ class Weights(dict):
         super().__init__()
         rng = np.random.default_rng(seed)
         for name, shape in parsed.tensor_shapes():
-            if name.endswith(".alpha"):
+            last = name.split(".")[-1]
+            if getattr(parsed, "residual", 0) == 2 and last in ("norm1", "norm2") or getattr(parsed, "tied_head", False) and name == "final.norm":
+                v = 0.2 * rng.standard_normal(shape)           # stored around zero
+            elif last == "lam":
+                v = -5.0 + 1.5 * rng.standard_normal(shape)    # a state that lasts
+            elif last == "conv":
+                v = 0.5 * rng.standard_normal(shape)
+            elif last == "correction":
+                v = 0.1 * rng.standard_normal(shape)
+            elif name.endswith(".a2.b"):
+                v = 2.0 + rng.standard_normal(shape)
+            elif len(shape) == 3:
+                v = rng.standard_normal(shape) / np.sqrt(shape[-1])
+            elif last == "b":
+                v = (3.0 if name.endswith(".f.b") else 0.0) + (1.0 if name.endswith(".f.b") else 0.5) * rng.standard_normal(shape)
+            elif name.endswith(".alpha"):
                 v = np.asarray(0.4 + 0.4 * rng.random())
             elif name.endswith(".temp"):
                 v = 1.0 + 0.3 * rng.standard_normal(shape)
@@ -106,6 +166,27 @@ def clear_calls(W, cfg, seed=77):
     return W
 
 
+def clear_calls_prenorm(W, cfg, seed=77):
+    """The same where sublayers add to the stream: nothing is added to the channels that carry the ranking (an identity expert scales them all)."""
+    moes = [lay["mlp"]["router"] for lay in cfg["layers"] if lay["mlp"] and lay["mlp"]["kind"] == "moe"]
+    if not moes:
+        return W
+    E = max(r["experts"] + r.get("identity", 0) for r in moes)
+    rng = np.random.default_rng(seed)
+    for t in range(cfg["vocab"]):
+        W["embed"][t, :E] = bf16((rng.permutation(E) - (E - 1) / 2) * (6.0 / E))
+    for name, v in W.items():
+        if name.endswith((".o", ".down")):
+            v[:E] = 0.0
+    for i, lay in enumerate(cfg["layers"]):
+        if lay["mlp"] and lay["mlp"]["kind"] == "moe":
+            W[f"l{i}.norm2"][:E] = 0.0
+            n = W[f"l{i}.mlp.router"].shape[0]
+            W[f"l{i}.mlp.router"][:] = 2.0 * np.eye(n, cfg["width"])
+            W[f"l{i}.mlp.correction"][:] = bf16(0.003 * rng.standard_normal(n))
+    return W
+
+
 def write_dir(path, cfg, weights):
     """config.json + model.safetensors as a checkpoint folder holds them."""
     head, blobs, at = {}, [], 0
@@ -137,7 +218,7 @@ DTYPES = ("f32", "bf16")
 
 
 def make(pkg, cfg, dtype, max_seq=256, seed=0, weights=None, **kw):
-    parsed = pkg.layered_model.parse_config(cfg)
+    parsed = parse(pkg, cfg)
     W = weights if weights is not None else Weights(parsed, seed)
     hb = pkg.hip_backend
     eng = pkg.HipGpuInference.from_layered(pkg.LayeredModel(parsed, W), max_seq, compute=hb.COMPUTE_F32 if dtype == "f32" else hb.COMPUTE_BF16, **kw)

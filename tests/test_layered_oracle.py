@@ -205,11 +205,11 @@ def test_bench_sizes_are_models_the_registry_takes(pkg):
     import bench
     for name, sz in bench.LAYERED_SIZES.items():
         cfg = bench.layered_config(sz)
-        p = pkg.layered_model.parse_config(cfg)
-        assert p.num_layers == sz["layers"] and {l.mixer for l in p.layers} == ({3} if name[0] == "p" else {1, 2}), name
+        p = pkg.layered_model.parse_config(cfg).resolve(lambda _: (16, sz["width"]))
+        assert p.num_layers == sz["layers"] and {l.mixer for l in p.layers} == {"p": {3}, "w": {1, 2}, "s": {6, 7}}[name[0]], name
         shapes = dict(p.tensor_shapes())
         t, data = bench.RandomBf16().get("l0.mix.o", (8, 16))
-        assert t == 30 and data.size == 128 and shapes["head"] == (sz["vocab"], sz["width"])
+        assert t == 30 and data.size == 128 and shapes["embed" if p.tied_head else "head"] == (sz["vocab"], sz["width"])
 
 
 # ---- the Pubopel design ----
@@ -329,3 +329,177 @@ def test_create_refuses_unusable_experts_and_heads(pkg):
     assert status(lc.sandwich([lc.tied(heads=1, kv_heads=1, dim=300)])) == "Unsupported"
     assert status(lc.sandwich([lc.tied(mlp=lc.moe(experts=1, top=1, ff=8, shared=40000))], width=4, vocab=8)) == "Unsupported"
     assert status(lc.sandwich([lc.tied()], taps=65)) == "Unsupported"
+
+
+# ---- the Sumevik design ----
+def _random(shapes, seed):
+    rng = np.random.default_rng(seed)
+    return {k: rng.standard_normal(s) for k, s in shapes.items()}, rng
+
+
+def test_linear_recurrence_equals_its_explicit_sum():
+    rng = np.random.default_rng(11)
+    a, x = rng.random((12, 5)), rng.standard_normal((12, 5))
+    S = lo.linear_recurrence(a, x)
+    for t in range(12):
+        assert np.allclose(S[t], sum(np.prod(a[s + 1: t + 1], axis=0) * x[s] for s in range(t + 1)))
+
+
+def test_gated_recurrence_step_by_step():
+    """One channel block at a time with plain loops: gates, decay, convolution with nothing before the first token."""
+    T, W, n, nb, taps = 7, 9, 6, 2, 3
+    s = n // nb
+    w, rng = _random({"y": (n, W), "y.b": (n,), "x": (n, W), "x.b": (n,), "conv": (n, taps), "conv.b": (n,), "ra": (nb, s, s), "ra.b": (nb, s), "ri": (nb, s, s), "ri.b": (nb, s),
+                      "lam": (n,), "o": (W, n)}, 12)
+    h = rng.standard_normal((T, W))
+    got = lo.rglru(h, w, {"width": n, "blocks": nb, "conv": taps}, 1e-6)
+    x = h @ w["x"].T + w["x.b"]
+    S, out = np.zeros(n), []
+    for t in range(T):
+        u = np.array([w["conv.b"][c] + sum(w["conv"][c, taps - 1 - j] * x[t - j, c] for j in range(taps) if t >= j) for c in range(n)])
+        for c in range(n):
+            k = c // s
+            r = 1 / (1 + math.exp(-(w["ra"][k, c % s] @ u[k * s:(k + 1) * s] + w["ra.b"][k, c % s])))
+            i = 1 / (1 + math.exp(-(w["ri"][k, c % s] @ u[k * s:(k + 1) * s] + w["ri.b"][k, c % s])))
+            a = math.exp(-8 * r * math.log1p(math.exp(w["lam"][c])))
+            S[c] = a * S[c] + math.sqrt(1 - a * a) * i * u[c]
+        out.append(w["o"] @ (S * lo.gelu_tanh(w["y"] @ h[t] + w["y.b"])))
+    assert np.allclose(got, out)
+
+
+def test_chunks_are_counted_from_the_start():
+    assert lo.chunk_keys(7, 4) == [4, 5, 6, 7] and lo.chunk_keys(8, 4) == [8] and lo.chunk_keys(3, 0) == [0, 1, 2, 3] and lo.chunk_keys(5, 1) == [5]
+
+
+def test_gated_attention_equals_an_explicit_matrix_form():
+    T, Wd, H, G, d, dv, size = 11, 17, 4, 2, 6, 5, 4
+    mx = lc.gated(heads=H, kv_heads=G, dim=d, vdim=dv, chunk=size, rot=4, base=50.0, scale=0.7)["mixer"]
+    w, rng = _random({"q": (H * d, Wd), "q.b": (H * d,), "k": (G * d, Wd), "k.b": (G * d,), "v": (G * dv, Wd), "v.b": (G * dv,), "q.norm": (d,), "k.norm": (d,), "g": (H * dv, Wd),
+                      "o": (Wd, H * dv)}, 13)
+    h = rng.standard_normal((T, Wd))
+    n = lambda x, g: x / np.sqrt((x * x).mean(-1, keepdims=True) + 1e-6) * g
+    q = n((h @ w["q"].T + w["q.b"]).reshape(T, H, d), w["q.norm"])
+    k = np.repeat(n((h @ w["k"].T + w["k.b"]).reshape(T, G, d), w["k.norm"]), H // G, axis=1)
+    v = np.repeat((h @ w["v"].T + w["v.b"]).reshape(T, G, dv), H // G, axis=1)
+    turn = np.exp(1j * np.arange(T)[:, None, None] * 50.0 ** (-np.arange(2) / 2.0))          # neighbouring pairs as complex numbers
+    rot = lambda x: np.concatenate([np.stack([((x[..., 0:4:2] + 1j * x[..., 1:4:2]) * turn).real, ((x[..., 0:4:2] + 1j * x[..., 1:4:2]) * turn).imag], -1).reshape(T, H, 4), x[..., 4:]], -1)
+    s = np.einsum("ihd,jhd->hij", rot(q), rot(k)) * 0.7
+    i = np.arange(T)
+    s[:, (i[None] > i[:, None]) | (i[None] // size != i[:, None] // size)] = -np.inf
+    e = np.exp(s)
+    out = np.einsum("hij,jhd->ihd", e / e.sum(-1, keepdims=True), v).reshape(T, -1) / (1 + np.exp(-(h @ w["g"].T)))
+    assert np.allclose(lo.gated_attention(h, w, mx, 1e-6), out @ w["o"].T)
+
+
+def test_gated_linear_attention_equals_its_explicit_sum():
+    T, Wd, H, d, dv, rank = 8, 10, 2, 4, 3, 2
+    w, rng = _random({"q": (H * d, Wd), "k": (H * d, Wd), "v": (H * dv, Wd), "g": (H * dv, Wd), "o": (Wd, H * dv), "norm": (dv,), "a1": (rank, Wd), "a2": (H * d, rank), "a2.b": (H * d,)}, 14)
+    h = rng.standard_normal((T, Wd))
+    z = (h @ w["a1"].T @ w["a2"].T + w["a2.b"]).reshape(T, H, d)
+    alpha = (1 / (1 + np.exp(-z))) ** (1 / 5.0)
+    q, k, v = ((h @ w[n].T).reshape(T, H, -1) for n in "qkv")
+    out = np.zeros((T, H, dv))
+    for t in range(T):
+        for n in range(H):
+            for s in range(t + 1):
+                out[t, n] += (q[t, n] / 2.0 * np.prod(alpha[s + 1: t + 1, n], axis=0)) @ k[s, n] * v[s, n]
+    out = out / np.sqrt((out * out).mean(-1, keepdims=True) + 1e-6) * w["norm"]
+    g = h @ w["g"].T
+    assert np.allclose(lo.gated_linear_attention(h, w, {"heads": H, "dim": d, "vdim": dv, "tau": 5.0}, 1e-6), (out.reshape(T, -1) * g / (1 + np.exp(-g))) @ w["o"].T)
+
+
+def test_routing_by_groups():
+    s = np.array([0.30, 0.02, 0.25, 0.03, 0.05, 0.35])
+    route = lambda c, n, keep, top: lo.route_groups(np.log(s), np.array(c), {"groups": {"count": n, "keep": keep}, "top": top})
+    assert [e for e, _ in route([0] * 6, 3, 3, 2)] == [5, 0] and [e for e, _ in route([0] * 6, 3, 1, 2)] == [5, 4]       # the second best lies in a closed group
+    assert [e for e, _ in route([-9.0, -9.0, -9.0, -9.0, -8.5, -8.0], 3, 2, 3)] == [5, 4, 0]                              # all negative: closed ones stay out
+    (a, wa), (b, wb) = route([0, 0, 0, 5.0, 0, 0], 2, 2, 2)
+    assert (a, b) == (3, 5) and wa == pytest.approx(0.03 / 0.38) and wb == pytest.approx(0.35 / 0.38)                     # weights without the correction
+
+
+def test_identity_experts_and_clamped_experts():
+    w, rng = _random({"router": (3, 6), "correction": (3,), "e0.gate": (4, 6), "e0.up": (4, 6), "e0.down": (6, 4)}, 15)
+    mlp = {"kind": "moe", "expert": {"ff": 4, "limit": 0.6}, "router": {"experts": 1, "identity": 2, "top": 3, "groups": {"count": 3, "keep": 3}}}
+    x = rng.standard_normal((2, 6))
+    for t in range(2):
+        e = np.exp(w["router"] @ x[t])
+        e /= e.sum()
+        g, u = np.minimum(w["e0.gate"] @ x[t], 0.6), np.clip(w["e0.up"] @ x[t], -0.6, 0.6)
+        assert np.allclose(lo.feed_forward(x, w, mlp)[t], (e[1] + e[2]) * x[t] + e[0] * (w["e0.down"] @ (g / (1 + np.exp(-1.702 * g)) * (u + 1))))
+
+
+def test_a_sumevik_sequence_does_not_see_its_future(pkg):
+    cfg = lc.prenorm([lc.rglru(mlp=lc.grouped()), lc.parallel(mlp=lc.dense())])
+    W = lc.Weights(lc.parse(pkg, cfg))
+    t = lc.tokens(14, cfg["vocab"])
+    assert np.allclose(lo.forward(cfg, W, t)[:9], lo.forward(cfg, W, t[:9]))
+
+
+def test_parse_sumevik_reads_every_size_and_constant(pkg):
+    hb = pkg.hip_backend
+    cfg = lc.prenorm([lc.rglru(width=90, blocks=5, taps=3, mlp=lc.grouped(10, 2, 3, 19, (6, 2), 0.7)),
+                      lc.parallel(lc.gated(9, 3, 18, 7, 21, 6, 77.0, 0.3), lc.gla(2, 11, 13, 4.0, 5), (0.3, 0.6), lc.dense(31)), lc.rglru()], eps=3e-6, logit_scale=0.25)
+    p = lc.parse(pkg, cfg)
+    a, b, c = p.layers
+    assert (a.mixer, a.heads, a.dim, a.vdim, a.taps) == (hb.MIXER_GLRU, 5, 18, 18, 3)
+    assert (a.ff_kind, a.ff, a.experts, a.identity, a.top, a.groups, a.keep_groups, a.expert_limit) == (hb.FF_MOE, 19, 10, 2, 3, 6, 2, 0.7)
+    assert (a.router_form, a.expert_form, a.shared_ff) == (hb.ROUTER_SOFTMAX_GROUPS, hb.EXPERT_CLAMPED, 0)
+    assert (b.mixer, b.heads, b.kv_heads, b.dim, b.vdim, b.chunk, b.rot_dims, b.rot_base, b.scale) == (hb.MIXER_PARALLEL, 9, 3, 18, 7, 21, 6, 77.0, 0.3)
+    assert (b.gla_heads, b.gla_dim, b.gla_vdim, b.gla_tau, b.gla_rank, b.left_scale, b.right_scale, b.ff_kind, b.ff) == (2, 11, 13, 4.0, 5, 0.3, 0.6, hb.FF_GEGLU, 31)
+    assert c.ff_kind == hb.FF_NONE
+    d = p.desc()
+    assert (d.width, d.vocab_size, d.norm_eps, d.residual_mult, d.residual, d.conv_taps, d.tied_head, d.logit_scale) == (88, 150, 3e-6, 1.0, hb.RESIDUAL_PRE_RMS, 0, 1, 0.25)
+    s = dict(p.tensor_shapes())
+    assert s["l0.mix.ra"] == (5, 18, 18) and s["l0.mix.ri.b"] == (5, 18) and s["l0.mix.conv"] == (90, 3) and s["l0.mlp.router"] == (12, 88) and s["l0.mlp.correction"] == (12,)
+    assert s["l0.mlp.e9.down"] == (88, 19) and "l0.mlp.e10.down" not in s and s["l1.mix.left.v.b"] == (21,) and s["l1.mix.left.q.norm"] == (18,) and s["l1.mix.right.a2"] == (22, 5)
+    assert s["l1.mix.right.norm"] == (13,) and s["l1.mix.left.o"] == (88, 63) and "head" not in s and "l2.norm2" not in s and "l1.mix.o" not in s
+    # the parts of a mixture that another design leaves out
+    q = pkg.layered_model.parse_config(lc.prenorm([lc.rglru(mlp={"kind": "moe", "expert": {"ff": 8, "limit": 1.0}, "router": {"experts": 4, "top": 2}})]))
+    assert (q.layers[0].groups, q.layers[0].keep_groups, q.layers[0].identity) == (1, 1, 0)
+
+
+@pytest.mark.parametrize("break_it", [
+    lambda c: c.pop("logit_scale"), lambda c: c["norm"].pop("eps"), lambda c: c["layers"][0]["mixer"].update(blocks=7), lambda c: c["layers"][0]["mixer"].update(conv=0),
+    lambda c: c["layers"][0]["mixer"].pop("width"), lambda c: c["layers"][1]["mixer"].pop("left_scale"), lambda c: c["layers"][1]["mixer"]["left"].update(kv_heads=4),
+    lambda c: c["layers"][1]["mixer"]["left"]["rot"].update(dims=7), lambda c: c["layers"][1]["mixer"]["left"]["rot"].update(dims=40),
+    lambda c: c["layers"][1]["mixer"]["left"]["mask"].update(size=0), lambda c: c["layers"][1]["mixer"]["right"].pop("tau"), lambda c: c["layers"][1].update(rank=0),
+    lambda c: c["layers"][0]["mlp"]["expert"].pop("limit"), lambda c: c["layers"][0]["mlp"]["router"]["groups"].update(count=5),
+    lambda c: c["layers"][0]["mlp"]["router"]["groups"].update(keep=5), lambda c: c["layers"][0]["mlp"]["router"].update(top=7)])
+def test_unusable_sumevik_configurations_are_refused(pkg, break_it):
+    c = lc.prenorm([lc.rglru(mlp=lc.grouped()), lc.parallel()])
+    lc.parse(pkg, c)
+    break_it(c)
+    with pytest.raises(pkg.layered_model.ConfigError):
+        lc.parse(pkg, c)
+
+
+def test_a_size_that_only_a_tensor_tells(pkg, tmp_path):
+    cfg = lc.prenorm([lc.rglru(), lc.parallel(right=lc.gla(rank=7), mlp=lc.grouped())])
+    W = lc.Weights(lc.parse(pkg, cfg))
+    lc.write_dir(tmp_path, cfg, W)
+    m = pkg.LayeredModel.from_dir(str(tmp_path))
+    assert m.config.layers[1].gla_rank == 7 and {t[0]: t[2] for t in m.tensors()}["l0.mix.ra"] == (32, 32, 3)
+    del W["l1.mix.right.a1"]
+    lc.write_dir(tmp_path, cfg, W)
+    with pytest.raises(pkg.layered_model.ConfigError, match="right.a1"):
+        pkg.LayeredModel.from_dir(str(tmp_path))
+
+
+def test_create_refuses_unusable_recurrences_and_routers(pkg):
+    hb = pkg.hip_backend
+
+    def status(cfg, **change):
+        p = lc.parse(pkg, cfg)
+        for k, v in change.items():
+            setattr(p.layers[0], k, v)
+        with pytest.raises(pkg.BackendError) as ei:
+            hb.HipGpuInference.from_layered(pkg.LayeredModel(p, {}), 16)
+        return ei.value.variant
+    assert status(lc.prenorm([lc.rglru(taps=65)])) == "Unsupported"
+    assert status(lc.prenorm([lc.rglru()]), vdim=31) == "InvalidArgument"
+    assert status(lc.prenorm([lc.gated(heads=1, kv_heads=1, dim=520)])) == "Unsupported"
+    assert status(lc.prenorm([lc.gla()]), gla_tau=0.0) == "InvalidArgument"
+    assert status(lc.prenorm([lc.rglru(mlp=lc.grouped())]), groups=5) == "InvalidArgument"
+    assert status(lc.prenorm([lc.rglru(mlp=lc.grouped())]), router_form=7) == "Unsupported"
+    assert status(lc.prenorm([lc.rglru(mlp=lc.grouped(600, 8, 2, 8, None))])) == "Unsupported"
+    assert status(lc.config([lc.mem(ff=0) | {"mlp": None}]), ff_kind=2, ff=8, experts=2, top=1, router_form=1, expert_form=1, groups=1, keep_groups=1, identity=1) == "Unsupported"
