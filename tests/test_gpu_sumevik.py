@@ -38,7 +38,7 @@ CASES = {
     "recurrence, nineteen taps": dict(layers=[lc.rglru(taps=19)]),
     "recurrence, one block": dict(layers=[lc.rglru(width=130, blocks=1)]),
     "recurrence, blocks of one": dict(layers=[lc.rglru(width=11, blocks=11)]),
-    "recurrence, blocks of 64": dict(layers=[lc.rglru(width=256, blocks=4)]),
+    "recurrence, blocks of 64": dict(layers=[lc.rglru(width=320, blocks=5)]),
     "recurrence, blocks of 65": dict(layers=[lc.rglru(width=195, blocks=3)]),
     "recurrence, blocks of 320": dict(layers=[lc.rglru(width=640, blocks=2)]),
     "recurrence, blocks of 18": dict(layers=[lc.rglru(width=90, blocks=5)]),
@@ -416,7 +416,7 @@ def test_hidden_state_and_refusals(pkg, gpu):
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_bench_like_sizes(pkg, gpu, dtype):
     """Sizes a real layer has, against the oracle: 128-wide heads, groups of four, diagonal blocks of 256, states of 128 x 256, experts of several hundred."""
-    cfg = lc.prenorm([lc.rglru(width=1024, blocks=4, mlp=lc.grouped(12, 4, 4, 320, (4, 2), 5.0)),
+    cfg = lc.prenorm([lc.rglru(width=1024, blocks=4, mlp=lc.grouped(14, 4, 3, 320, (6, 2), 5.0)),
                       lc.parallel(lc.gated(8, 2, 128, 128, 150, 64), lc.gla(3, 128, 256, rank=16), (1.0, 0.7), lc.dense(700))], width=1024, vocab=300)
     eng, W = engine(pkg, cfg, dtype, max_seq=320)
     toks = lc.tokens(280, cfg["vocab"], 71)
