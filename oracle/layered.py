@@ -67,6 +67,19 @@ def rotate_pairs(x, positions, rot):
     return out
 
 
+def rotate_halves(x, positions, rot):
+    """x [T, ..., d]: value i of the first rot.dims paired with value i + dims / 2."""
+    f, mag = rope_frequencies(rot)
+    n = int(rot["dims"])
+    out = np.array(x, dtype=F)
+    ang = np.asarray(positions, dtype=F).reshape((-1,) + (1,) * (x.ndim - 1)) * f
+    c, s = np.cos(ang) * mag, np.sin(ang) * mag
+    u, v = x[..., : n // 2], x[..., n // 2: n]
+    out[..., : n // 2] = u * c - v * s
+    out[..., n // 2: n] = v * c + u * s
+    return out
+
+
 def latent_attention(h, w, mx, eps):
     """h [T, width] -> [T, width]; w: the layer's mixer tensors by short name."""
     T, H, d, r, dv, kr = len(h), mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"], mx["kv_rank"]
@@ -108,6 +121,86 @@ def mlstm(h, w, mx, eps):
             out[t, n] = (S.T @ q[t, n]) / (max(abs(nv @ q[t, n]), math.exp(-m)) + 1e-6)
     out = rms(out, eps).reshape(T, H * dv) * w["norm"] * sigmoid(h @ w["g"].T)
     return out @ w["o"].T
+
+
+def query_latent(h, w, eps):
+    """Queries through a latent of their own, which is normed between its two projections."""
+    return (rms(h @ w["dq"].T, eps) * w["dq.norm"]) @ w["uq"].T
+
+
+def windowed_latent_attention(h, w, mx, eps):
+    """Attention over a shared latent whose queries have a latent too; the last `size` positions are visible; halves rotated; every value gated."""
+    T, H, d, r, dv, kr = len(h), mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"], mx["kv_rank"]
+    pos = np.arange(T)
+    q = query_latent(h, w, eps).reshape(T, H, d + r)
+    dkv = h @ w["dkv"].T
+    c = rms(dkv[:, :kr], eps) * w["dkv.norm"]
+    turn = lambda x: rotate_halves(x, pos, mx["rot"]) if mx.get("rot") else x
+    k_rot, q_rot = turn(dkv[:, kr:]), turn(q[..., d:])
+    k = (c @ w["uk"].T).reshape(T, H, d)
+    v = (c @ w["uv"].T).reshape(T, H, dv)
+    out = np.zeros((T, H, dv), dtype=F)
+    for i in range(T):
+        seen = visible_keys(i, mx.get("mask"))
+        for n in range(H):
+            s = (k[seen, n] @ q[i, n, :d] + k_rot[seen] @ q_rot[i, n]) * mx["scale"]
+            p = np.exp(s - s.max())
+            out[i, n] = (p / p.sum()) @ v[seen, n]
+    return (out.reshape(T, H * dv) * sigmoid(h @ w["g"].T)) @ w["o"].T
+
+
+def grouped_keys_values(h, w, mx):
+    """What a grouped attention layer caches: rotated keys [T, G, d] and values [T, G, dv]."""
+    T, G = len(h), mx["kv_heads"]
+    k, v = linear(h, w, "k").reshape(T, G, mx["dim"]), linear(h, w, "v").reshape(T, G, mx["vdim"])
+    return (rotate_pairs(k, np.arange(T), mx["rot"]) if mx.get("rot") else k), v
+
+
+def grouped_attention(h, w, mx, kv):
+    """Grouped attention on given keys and values (its own or another layer's): rotated queries, a window, one more in the softmax's denominator."""
+    T, H, G = len(h), mx["heads"], mx["kv_heads"]
+    k, v = kv
+    q = linear(h, w, "q").reshape(T, H, mx["dim"])
+    if mx.get("rot"):
+        q = rotate_pairs(q, np.arange(T), mx["rot"])
+    out = np.zeros((T, H, mx["vdim"]), dtype=F)
+    for i in range(T):
+        seen = visible_keys(i, mx.get("mask"))
+        for n in range(H):
+            g = n // (H // G)
+            out[i, n] = sink_softmax((k[seen, g] @ q[i, n]) * mx["scale"], 0.0) @ v[seen, g]
+    return linear(out.reshape(T, -1), w, "o")
+
+
+def unit(x):
+    """Vectors of length one along the last axis."""
+    return x / np.sqrt(np.sum(x * x, axis=-1, keepdims=True) + 1e-6)
+
+
+def delta_rule(h, w, mx, eps):
+    """A matrix state per head that decays as a whole and is corrected towards each value, one token after the other."""
+    T, H, G, d, dv = len(h), mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+    short = lambda name: silu(causal_conv(h @ w[name].T, w[name + ".conv"]))
+    q = unit(short("q").reshape(T, G, d)) * d ** -0.5
+    k = unit(short("k").reshape(T, G, d))
+    v = short("v").reshape(T, H, dv)
+    beta = sigmoid(h @ w["b"].T)
+    g = np.exp(-np.exp(w["A_log"]) * softplus(h @ w["a"].T + w["dt_bias"]))
+    out = np.zeros((T, H, dv), dtype=F)
+    for n in range(H):
+        S = np.zeros((d, dv), dtype=F)
+        m = n // (H // G)
+        for t in range(T):
+            S = g[t, n] * S
+            u = beta[t, n] * (v[t, n] - S.T @ k[t, m])
+            S = S + np.outer(k[t, m], u)
+            out[t, n] = S.T @ q[t, m]
+    o = rms(out, eps) * w["norm"]
+    return (o.reshape(T, H * dv) * silu(h @ w["g"].T)) @ w["o"].T
+
+
+def squared_relu_ff(x, w):
+    return (np.maximum(x @ w["up"].T, 0.0) ** 2) @ w["down"].T
 
 
 def visible_keys(i, mask):
@@ -362,10 +455,38 @@ def forward_sandwich(cfg, weights, tokens, layers_out=None):
     return norm(x, "final.norm") @ W["head"].T
 
 
+def forward_sandwich_ln(cfg, weights, tokens, layers_out=None):
+    """Layer norms before and after every sublayer, whose result is scaled channel by channel; layers may read another layer's keys and values;
+    logits are squashed."""
+    W = {k: np.asarray(v, dtype=F) for k, v in weights.items()}
+    eps = cfg["norm"]["eps"]
+    norm = lambda v, name: layer_norm(v, W[name], eps)
+    x = W["embed"][list(tokens)]
+    kvs = {}
+    for i, lay in enumerate(cfg["layers"]):
+        p, mx = f"l{i}.", lay["mixer"]
+        sub = lambda g: {k[len(p + g):]: v for k, v in W.items() if k.startswith(p + g)}
+        h, w = norm(x, p + "norm1"), sub("mix.")
+        if lay["type"] == "attention":
+            src = mx.get("kv_from")
+            kvs[i] = grouped_keys_values(h, w, mx) if src is None else kvs[src]
+            y = grouped_attention(h, w, mx, kvs[i])
+        else:
+            y = {"latent_attention": windowed_latent_attention, "delta": delta_rule}[lay["type"]](h, w, mx, eps)
+        x = x + norm(y, p + "norm1b") * W[p + "ls1"]
+        if lay["mlp"]:
+            x = x + norm(squared_relu_ff(norm(x, p + "norm2"), sub("mlp.")), p + "norm2b") * W[p + "ls2"]
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return soft_cap(norm(x, "final.norm") @ W["head"].T, cfg["logit_softcap"])
+
+
 def forward(cfg, weights, tokens, layers_out=None):
     """Logits [T, vocab] of a whole sequence; layers_out (a list) receives the residual stream after every layer."""
     if "canon" in cfg:
         return forward_sandwich(cfg, weights, tokens, layers_out)
+    if "logit_softcap" in cfg:
+        return forward_sandwich_ln(cfg, weights, tokens, layers_out)
     if "logit_scale" in cfg:
         return forward_pre_norm(cfg, weights, tokens, layers_out)
     W = {k: np.asarray(v, dtype=F) for k, v in weights.items()}
