@@ -170,7 +170,8 @@ enum {
   LGH_SYM_GATTN = 25,      /* lgh::gattn_* : attention with gated values; gated linear attention where it runs beside it */
   LGH_SYM_GLA = 26,        /* lgh::gla_* : gated linear attention */
   LGH_SYM_GLRU = 27,       /* lgh::glru_* : gated linear recurrence per channel */
-  LGH_SYM_COUNT = 28
+  LGH_SYM_DELTA = 28,      /* lgh::delta_* : gated delta rule */
+  LGH_SYM_COUNT = 29
 };
 
 typedef struct lgh_stats {
@@ -282,6 +283,7 @@ int lgh_eval(lgh_ctx* ctx, const uint32_t* tokens, size_t n, const uint32_t* wan
  *   LGH_RESIDUAL_SANDWICH_DYT  h = dyt(x); h += conv(h); x += residual_mult * dyt'(sublayer(h)), where dyt(x) = tanh(alpha x) * w + b and
  *                              conv is a causal convolution over conv_taps positions, one filter per channel (0 taps: none)
  *   LGH_RESIDUAL_PRE_RMS       x += residual_mult * sublayer(rms_norm(x) * (1 + w))
+ *   LGH_RESIDUAL_SANDWICH_LN   x += residual_mult * (layer_norm'(sublayer(layer_norm(x))) * ls), layer norms with a weight, ls one factor per channel
  * No reference counterpart.  The context is driven by the entry points above (GpuInference, lgh_eval, lgh_decode_greedy, ...; the
  * cache rows and recurrent states are the context's).  Weights are bf16 and stay bf16 in HBM; tensors are uploaded by their
  * checkpoint names (`embed`, `bigram`, `l0.mix.q`, `l0.mlp.gate`, `l0.mlp.e0.gate`, `l0.norm1`, `l0.norm1.alpha`, `l0.canon1`, `final.norm`,
@@ -292,10 +294,16 @@ enum { LGH_MIXER_LATENT_ATTENTION = 1, LGH_MIXER_MLSTM = 2,
        LGH_MIXER_GATED_ATTENTION = 4,                  /* grouped heads, biases, norms per head, rotation, chunks; the output gated value by value */
        LGH_MIXER_GLA = 5,                              /* gated linear attention: a matrix state whose rows decay each at its own rate */
        LGH_MIXER_PARALLEL = 6,                         /* left_scale * gated attention + right_scale * gated linear attention, same input */
-       LGH_MIXER_GLRU = 7 };                           /* gated linear recurrence per channel behind a short convolution, times a gelu branch */
-enum { LGH_RESIDUAL_POST_LN = 0, LGH_RESIDUAL_SANDWICH_DYT = 1, LGH_RESIDUAL_PRE_RMS = 2 };
+       LGH_MIXER_GLRU = 7,                             /* gated linear recurrence per channel behind a short convolution, times a gelu branch */
+       LGH_MIXER_GROUPED_ATTENTION = 8,                /* grouped heads with values of their own, biases, rotation; window, sink, another layer's keys */
+       LGH_MIXER_DELTA = 9 };                          /* gated delta rule: a matrix state that decays as a whole and is corrected towards each value */
+enum { LGH_RESIDUAL_POST_LN = 0, LGH_RESIDUAL_SANDWICH_DYT = 1, LGH_RESIDUAL_PRE_RMS = 2, LGH_RESIDUAL_SANDWICH_LN = 3 };
 enum { LGH_FF_NONE = 0, LGH_FF_GEGLU = 1 };            /* down(gelu_tanh(gate x) * (up x)) */
 enum { LGH_FF_MOE = 2 };                               /* routed experts down(silu(gate x) * (up x)), sigmoid scores; optionally a shared one */
+enum { LGH_FF_RELU2 = 3 };                             /* down(relu(up x)^2) */
+enum { LGH_ROT_PAIRS = 0,                              /* rotation of neighbouring pairs (2i, 2i + 1) */
+       LGH_ROT_HALVES = 1 };                           /* ... of pairs (i, i + rot_dims / 2); latent attention */
+enum { LGH_GATE_HEADS = 0, LGH_GATE_VALUES = 1 };      /* latent attention: one output gate per head, or one per value */
 /* how a mixture's experts are chosen and weighted: sigmoid scores, the score multiplies the expert's input; or softmax scores, the choice by
  * score + correction among the best groups of neighbours, the chosen scores divided by their sum multiply the experts' outputs */
 enum { LGH_ROUTER_SIGMOID = 0, LGH_ROUTER_SOFTMAX_GROUPS = 1 };
@@ -307,18 +315,22 @@ typedef struct lgh_layer_desc {
   uint32_t mixer;                    /* LGH_MIXER_* */
   uint32_t heads, dim, vdim;         /* query / key size per head (latent attention: the unrotated part), value size per head */
   uint32_t kv_rank, rot_dim;         /* latent attention: latent size, rotated query / key part */
-  uint32_t rot_dims;                 /* leading values of the rotated part that are rotated (neighbouring pairs) */
+  uint32_t rot_dims;                 /* leading values of the rotated part that are rotated (pairs as rot_form says) */
   uint32_t ff_kind, ff;              /* LGH_FF_*, feed-forward size (mixture: of one expert) */
-  uint32_t kv_heads;                 /* tied, gated attention: key heads; query head h uses h / (heads / kv_heads) */
-  uint32_t window, keep_first;       /* tied attention: position i sees j <= i with i - j < window (0: no limit) or j < keep_first */
+  uint32_t kv_heads;                 /* tied, gated, grouped attention, delta rule: key heads; query (value) head h uses h / (heads / kv_heads) */
+  uint32_t window, keep_first;       /* tied, grouped, latent attention: position i sees j <= i with i - j < window (0: no limit); tied: or j < keep_first */
   uint32_t experts, top;             /* mixture: experts, and how many a token uses */
   uint32_t shared_ff;                /* mixture: size of the expert every token uses (0: none) */
   uint32_t router_form, expert_form; /* mixture: LGH_ROUTER_*, LGH_EXPERT_* */
   uint32_t groups, keep_groups;      /* LGH_ROUTER_SOFTMAX_GROUPS: groups of neighbours, and how many of them stay open */
   uint32_t identity;                 /* LGH_ROUTER_SOFTMAX_GROUPS: further router outputs behind the experts whose expert is its input */
   uint32_t chunk;                    /* gated attention: position i sees j <= i of the same chunk of this many positions (0: one chunk) */
-  uint32_t taps;                     /* linear recurrence: positions of its convolution; heads = diagonal blocks, dim = vdim = their size */
+  uint32_t taps;                     /* linear recurrence, delta rule: positions of the convolution; linear recurrence: heads = diagonal blocks, dim = vdim = their size */
   uint32_t gla_heads, gla_dim, gla_vdim, gla_rank;   /* gated linear attention; gla_rank: inner size of the decay's projection */
+  uint32_t q_rank;                   /* latent attention: size of the queries' own latent (tensors dq, dq.norm, uq; 0: they are projected directly, tensor q) */
+  uint32_t rot_form, gate_form;      /* latent attention: LGH_ROT_*, LGH_GATE_* */
+  uint32_t sink_one;                 /* grouped attention: 1: the softmax's denominator has one more term, exp(0) */
+  uint32_t kv_from;                  /* grouped attention: 1 + the earlier layer whose keys and values this one reads (0: its own) */
   double scale;                      /* attention: factor on the scores */
   double rot_base;
   double yarn_factor, yarn_original, yarn_fast, yarn_slow;   /* yarn_factor 0: plain frequencies */
@@ -342,6 +354,7 @@ typedef struct lgh_layered_desc {
   uint32_t tied_head;                /* 1: the output projection is the embedding table (no tensor `head`) */
   uint32_t reserved;
   double logit_scale;                /* factor on the logits (0: 1) */
+  double logit_cap;                  /* logits = cap * tanh(logits / cap) (0: none) */
 } lgh_layered_desc;
 int lgh_create_layered(const lgh_layered_desc* desc, const lgh_layer_desc* layers, lgh_ctx** out);
 /* Residual stream after every layer, for parity tests: switched on, the next lgh_eval portions (block path) keep it;

@@ -1,12 +1,14 @@
-// gated_attention.hip — grouped softmax attention of layered.h with values of their own size: queries and keys are RMS-normed per head and rotated
-// (neighbouring pairs) before they are used or cached, position i sees the keys of its own chunk (counted from the sequence's start) up to itself,
-// and the heads' outputs are gated value by value.  Scores, softmax and sums are in 32-bit, in units of log2.
+// gated_attention.hip — grouped softmax attention of layered.h with values of their own size: queries and keys are (RMS-normed per head and) rotated
+// (neighbouring pairs) before they are used or cached, position i sees the keys of its own chunk (counted from the sequence's start) and of its window
+// up to itself, the softmax may have a sink (one more term exp(0), which has no value), and the heads' outputs may be gated value by value.  Scores,
+// softmax and sums are in 32-bit, in units of log2.
 //
 //   decode and short portions: a workgroup = one key head (up to 4 of its query heads) x one share of the visible keys; a lane holds 16-byte
 //     pieces of a few keys' and values' rows, for the score and for the weighted sum.  In decode the same launch steps the gated linear attention
 //     that reads the same input (further workgroups), and the merge of the shares reads it out.
 //   prompt portions: causal flash attention in transposed form (S^T = K Q^T, O^T = V^T P^T), key and value tiles through LDS; only the tiles
-//     from the first query's chunk on.
+//     from the first query's first visible key on.
+// A layer may read another layer's caches: it has queries only, and its launches come after the ones that fill them.
 #include <algorithm>
 
 #include "gla_device.h"
@@ -16,7 +18,11 @@ namespace lgh {
 constexpr float kGattnNeg = -1e30f, kGattnLog2e = 1.4426950408889634f;
 constexpr uint32_t kGattnMaxSplits = 128, kGattnBatch = 4;
 
-__host__ __device__ __forceinline__ uint32_t chunk_start(const GattnShape& s, uint32_t i) { return i / s.chunk * s.chunk; }
+// the first key that position i sees; never falls with i
+__host__ __device__ __forceinline__ uint32_t key_start(const GattnShape& s, uint32_t i) {
+  const uint32_t c = i / s.chunk * s.chunk, w = i >= s.window ? i - s.window + 1 : 0;
+  return c > w ? c : w;
+}
 
 // lanes that share a row: 16 bytes each, of the wider of key and value
 __host__ __device__ constexpr uint32_t gattn_lanes(uint32_t bytes) { return bytes <= 128 ? 8 : bytes <= 256 ? 16 : bytes <= 512 ? 32 : 64; }
@@ -43,7 +49,7 @@ __device__ __forceinline__ void gattn_split(const GattnShape& s, const GattnBufs
   const uint32_t tid = threadIdx.x, lane = tid & 63, w = tid >> 6, grp = lane / LPK, sub = lane % LPK;
   const uint32_t gq = s.heads / s.kv_heads, chunks = (gq + HQ - 1) / HQ, g = hy / chunks, h0 = g * gq + (hy % chunks) * HQ;
   const uint32_t hn = (g + 1) * gq - h0 < (uint32_t)HQ ? (g + 1) * gq - h0 : (uint32_t)HQ;
-  const uint32_t lo = chunk_start(s, pos), total = pos + 1 - lo;
+  const uint32_t lo = key_start(s, pos), total = pos + 1 - lo;
   constexpr uint32_t KR = gattn_round(LPK);
   const uint32_t rounds = (total + KR - 1) / KR, per = (rounds + n_splits - 1) / n_splits;
   const uint32_t rb = sp * per, re = rb + per < rounds ? rb + per : rounds;
@@ -74,12 +80,12 @@ __device__ __forceinline__ void gattn_split(const GattnShape& s, const GattnBufs
   };
   fetch(rb);
   // a head's row of this token: normed, rotated.  Everything the rows need is requested before the first of them is used.
-  const bool owner = OWN && re == rounds, kvec = (s.dim & 3) == 0, vvec = (s.vdim & 3) == 0;
+  const bool owner = OWN && re == rounds, kvec = (s.dim & 3) == 0, vvec = (s.vdim & 3) == 0, normed = b.qn != nullptr;
   float q[HQ][C][PER], ok[C][PER], ov[C][PER], nq[C][PER], nk[C][PER];
   f32x2 cs[C][PER / 2];
 #pragma unroll
   for (int c = 0; c < C; c++) {
-    row_chunk<PER>(b.qn, d0[c], s.dim, kvec, nq[c]);
+    if (normed) row_chunk<PER>(b.qn, d0[c], s.dim, kvec, nq[c]);
 #pragma unroll
     for (int h = 0; h < HQ; h++) row_chunk<PER>(cat + s.off_q + (size_t)(h0 + ((uint32_t)h < hn ? h : 0)) * s.dim, d0[c], s.dim, kvec, q[h][c]);
 #pragma unroll
@@ -89,23 +95,29 @@ __device__ __forceinline__ void gattn_split(const GattnShape& s, const GattnBufs
       if (d < s.rot_n) cs[c][e] = reinterpret_cast<const f32x2*>(b.cs)[(size_t)pos * (s.rot_n / 2) + d / 2];
     }
     if (owner) {
-      row_chunk<PER>(b.kn, d0[c], s.dim, kvec, nk[c]);
+      if (normed) row_chunk<PER>(b.kn, d0[c], s.dim, kvec, nk[c]);
       row_chunk<PER>(cat + s.off_k + (size_t)g * s.dim, d0[c], s.dim, kvec, ok[c]);
       row_chunk<PER>(cat + s.off_v + (size_t)g * s.vdim, d0[c], s.vdim, vvec, ov[c]);
     }
   }
   auto head_row = [&](float (*o)[PER], const float (*nf)[PER], float f) {
-    float ss = 0.0f;
+    if (normed) {
+      float ss = 0.0f;
 #pragma unroll
-    for (int c = 0; c < C; c++)
+      for (int c = 0; c < C; c++)
 #pragma unroll
-      for (int e = 0; e < PER; e++) ss = __builtin_fmaf(o[c][e], o[c][e], ss);
-    const float inv = f / __builtin_sqrtf(lanes_sum<LPK>(ss) / (float)s.dim + s.eps);
+        for (int e = 0; e < PER; e++) ss = __builtin_fmaf(o[c][e], o[c][e], ss);
+      const float inv = 1.0f / __builtin_sqrtf(lanes_sum<LPK>(ss) / (float)s.dim + s.eps);
+#pragma unroll
+      for (int c = 0; c < C; c++)
+#pragma unroll
+        for (int e = 0; e < PER; e++) o[c][e] *= inv * nf[c][e];
+    }
 #pragma unroll
     for (int c = 0; c < C; c++)
 #pragma unroll
       for (int e = 0; e < PER; e += 2) {
-        const f32x2 r = rotate2(o[c][e] * inv * nf[c][e], o[c][e + 1] * inv * nf[c][e + 1], cs[c][e / 2]);
+        const f32x2 r = rotate2(o[c][e] * f, o[c][e + 1] * f, cs[c][e / 2]);
         o[c][e] = r.x; o[c][e + 1] = r.y;
       }
   };
@@ -271,7 +283,7 @@ __global__ void __launch_bounds__(256) gattn_attn_kernel(const GattnShape s, con
 
 static bool gattn_ok(const GattnShape& s) {
   return s.heads && s.kv_heads && s.heads % s.kv_heads == 0 && s.dim && s.dim <= s.dp && s.dp % 64 == 0 && s.dp <= kGattnMaxDim && s.vdim && s.vdim <= s.vp &&
-         s.vp % 64 == 0 && s.vp <= kGattnMaxDim && s.chunk && s.rows % 64 == 0 && s.rot_n <= s.dim && s.rot_n % 2 == 0;
+         s.vp % 64 == 0 && s.vp <= kGattnMaxDim && s.chunk && s.window && s.rows % 64 == 0 && s.rot_n <= s.dim && s.rot_n % 2 == 0;
 }
 
 template <class T, uint32_t LPK, int HQ, int C>
@@ -297,7 +309,7 @@ static hipError_t gattn_attn_pick(const GattnShape& s, const GattnBufs& b, const
 hipError_t gattn_attn_launch(const GattnShape& s, const GattnBufs& b, const GlaShape* gs, const GlaBufs* gb, const int* pos_ptr, uint32_t pos0, uint32_t M, bool own,
                              uint32_t n_splits, bool f32, hipStream_t st) {
   if (!gattn_ok(s) || M == 0 || M > kGattnShort || (own && M != 1) || (gs && (!gb || !own)) || n_splits == 0 || n_splits > kGattnMaxSplits ||
-      (!pos_ptr && pos0 + M > s.rows) || (s.rot_n && !b.cs))
+      (!pos_ptr && pos0 + M > s.rows) || (s.rot_n && !b.cs) || (own && b.shared) || !b.qn != !b.kn)
     return hipErrorInvalidValue;
   const uint32_t bytes = gattn_row_bytes(s, f32);
 #define LGH_GATTN_CASE(L, N) \
@@ -317,7 +329,7 @@ hipError_t gattn_attn_launch(const GattnShape& s, const GattnBufs& b, const GlaS
 // shares of the keys that fill the chip; not more than there are rounds of keys
 uint32_t gattn_splits(const GattnShape& s, uint32_t max_seq, uint32_t M, bool f32, uint32_t forced) {
   const uint32_t bytes = gattn_row_bytes(s, f32), gq = s.heads / s.kv_heads, hq = gq <= 2 ? gq : bytes > 1024 ? 2 : 4, wgs = s.kv_heads * ((gq + hq - 1) / hq) * M;
-  const uint32_t kr = gattn_round(gattn_lanes(bytes)), rounds = (std::min(max_seq, s.chunk) + kr - 1) / kr;
+  const uint32_t kr = gattn_round(gattn_lanes(bytes)), rounds = (std::min(std::min(max_seq, s.chunk), s.window) + kr - 1) / kr;
   const uint32_t want = forced ? forced : std::max(1u, 512 / wgs);
   return std::min(std::min(want, kGattnMaxSplits), std::max(rounds, 1u));
 }
@@ -342,7 +354,7 @@ __global__ void __launch_bounds__(256) gattn_merge_kernel(const GattnShape s, co
     return;
   }
   const uint32_t pos = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + t;
-  const uint32_t total = pos + 1 - chunk_start(s, pos), rounds = (total + kr - 1) / kr, per = (rounds + n_splits - 1) / n_splits, act = (rounds + per - 1) / per;
+  const uint32_t total = pos + 1 - key_start(s, pos), rounds = (total + kr - 1) / kr, per = (rounds + n_splits - 1) / n_splits, act = (rounds + per - 1) / per;
   const size_t rows = (size_t)M * s.heads, r = (size_t)t * s.heads + h;
   // (what the inactive shares hold is not used: the loads need no position)
   f32x2 ml[2];
@@ -367,13 +379,13 @@ __global__ void __launch_bounds__(256) gattn_merge_kernel(const GattnShape s, co
 #pragma unroll
     for (int i = 0; i < F; i++) first[i] = load(grp + i * groups < n_splits ? grp + i * groups : n_splits - 1, c0);
 #pragma unroll
-    for (int j = 0; j < V; j++) { gt.v[j] = cat[s.off_g + (size_t)h * s.vdim + c0 + j]; v.v[j] = 0.0f; }
+    for (int j = 0; j < V; j++) { gt.v[j] = s.gated ? cat[s.off_g + (size_t)h * s.vdim + c0 + j] : 0.0f; v.v[j] = 0.0f; }
     if (base == 0 && tid < 64) {
       const float m0 = lane < act ? ml[0].x : kGattnNeg, m1 = lane + 64 < act ? ml[1].x : kGattnNeg;
-      const float mm = wave_max(fmaxf(m0, m1));
+      const float mm = fmaxf(wave_max(fmaxf(m0, m1)), s.sink ? 0.0f : kGattnNeg);
       const float f0 = __builtin_amdgcn_exp2f(m0 - mm), f1 = __builtin_amdgcn_exp2f(m1 - mm);
       const float l0 = lane < act ? f0 * ml[0].y : 0.0f, l1 = lane + 64 < act ? f1 * ml[1].y : 0.0f;
-      const float tot = wave_sum(l0 + l1);
+      const float tot = wave_sum(l0 + l1) + (s.sink ? __builtin_amdgcn_exp2f(-mm) : 0.0f);
       wgt[lane] = f0 / tot; wgt[lane + 64] = f1 / tot;
     }
     __syncthreads();
@@ -398,7 +410,7 @@ __global__ void __launch_bounds__(256) gattn_merge_kernel(const GattnShape s, co
 #pragma unroll
         for (int j = 0; j < V; j++) v.v[j] += part[tid + k * cols].v[j];
 #pragma unroll
-      for (int j = 0; j < V; j++) out[(size_t)h * s.vdim + c0 + j] = to_act<O>(v.v[j] * sigmoid_f(gt.v[j]) * s.out_scale);
+      for (int j = 0; j < V; j++) out[(size_t)h * s.vdim + c0 + j] = to_act<O>(v.v[j] * (s.gated ? sigmoid_f(gt.v[j]) : 1.0f) * s.out_scale);
     }
     __syncthreads();
   }
@@ -436,7 +448,8 @@ __global__ void __launch_bounds__(256) gattn_prep_kernel(const GattnShape s, con
     T o[2] = {to_act<T>(u), to_act<T>(v)};
     __builtin_memcpy(__builtin_assume_aligned(p, sizeof(o)), o, sizeof(o));
   };
-  const uint32_t nh = s.heads + s.kv_heads;
+  const uint32_t nh = s.heads + (b.shared ? 0 : s.kv_heads);
+  const bool normed = b.qn != nullptr;
   const uint32_t i0 = (b.q ? 0 : s.heads) + blockIdx.y * kPrepHeads, i1 = i0 + kPrepHeads < nh ? i0 + kPrepHeads : nh;
   for (uint32_t i = i0 + w; i < i1; i += 4) {
     const bool key = i >= s.heads;
@@ -448,16 +461,17 @@ __global__ void __launch_bounds__(256) gattn_prep_kernel(const GattnShape s, con
 #pragma unroll
     for (uint32_t j = 0; j < NP; j++) {
       const uint32_t d = j * 128 + lane * 2;
-      x[j] = n[j] = (f32x2)(0.0f);
+      x[j] = (f32x2)(0.0f);
+      n[j] = (f32x2)(1.0f);
       r[j].x = 1.0f; r[j].y = 0.0f;
       if (j * 128 < s.dim) {
-        if (d < s.dim) { x[j].x = p[d]; n[j].x = nw[d]; }
-        if (d + 1 < s.dim) { x[j].y = p[d + 1]; n[j].y = nw[d + 1]; }
+        if (d < s.dim) { x[j].x = p[d]; if (normed) n[j].x = nw[d]; }
+        if (d + 1 < s.dim) { x[j].y = p[d + 1]; if (normed) n[j].y = nw[d + 1]; }
         if (d + 1 < s.rot_n) r[j] = cs[d / 2];
       }
       ss = __builtin_fmaf(x[j].x, x[j].x, __builtin_fmaf(x[j].y, x[j].y, ss));
     }
-    const float inv = 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)s.dim + s.eps), f = key ? 1.0f : s.scale * kGattnLog2e;
+    const float inv = normed ? 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)s.dim + s.eps) : 1.0f, f = key ? 1.0f : s.scale * kGattnLog2e;
     T* o = key ? reinterpret_cast<T*>(b.kc) + ((size_t)h * s.rows + pos) * s.dp : reinterpret_cast<T*>(b.q) + ((size_t)h * b.Mcap + t) * s.dp;
 #pragma unroll
     for (uint32_t j = 0; j < NP; j++) {
@@ -466,13 +480,15 @@ __global__ void __launch_bounds__(256) gattn_prep_kernel(const GattnShape s, con
       if (d < s.dp) store2(o + d, v.x * f, v.y * f);
     }
   }
+  if (b.shared) return;
   for (uint32_t i = blockIdx.y * 256 + threadIdx.x; i < s.kv_heads * s.vdim; i += 256 * gridDim.y)
     reinterpret_cast<T*>(b.vc)[((size_t)(i / s.vdim) * s.rows + pos) * s.vp + i % s.vdim] = to_act<T>(cat[s.off_v + i]);
 }
 
 hipError_t gattn_prep_launch(const GattnShape& s, const GattnBufs& b, uint32_t pos0, uint32_t M, bool f32, hipStream_t st) {
-  if (!gattn_ok(s) || M == 0 || (b.q && M > b.Mcap) || pos0 + M > s.rows || (s.rot_n && !b.cs)) return hipErrorInvalidValue;
-  const dim3 grid(M, ((b.q ? s.heads : 0) + s.kv_heads + kPrepHeads - 1) / kPrepHeads);
+  if (!gattn_ok(s) || M == 0 || (b.q && M > b.Mcap) || pos0 + M > s.rows || (s.rot_n && !b.cs) || !b.qn != !b.kn) return hipErrorInvalidValue;
+  if (b.shared && !b.q) return hipSuccess;
+  const dim3 grid(M, ((b.q ? s.heads : 0) + (b.shared ? 0 : s.kv_heads) + kPrepHeads - 1) / kPrepHeads);
   if (f32) hipLaunchKernelGGL((gattn_prep_kernel<float>), grid, dim3(256), 0, st, s, b, pos0);
   else hipLaunchKernelGGL((gattn_prep_kernel<__bf16>), grid, dim3(256), 0, st, s, b, pos0);
   return hipGetLastError();
@@ -499,7 +515,7 @@ __global__ void __launch_bounds__(256, (gattn_wgs<T, DQ, DV>())) gattn_flash_ker
   // the longest rows first, and of the second half of the grid the shortest first (workgroups i and i + half share a CU when all are resident)
   const uint32_t h = blockIdx.x % s.heads, qi = blockIdx.x / s.heads, hi = (nqb + 1) / 2, qb = qi < hi ? nqb - 1 - qi : qi - hi, v0 = blockIdx.y * DV;
   const uint32_t q0 = qb * 64 * QT, qw = q0 + w * 16 * QT, qlast = q0 + 64 * QT - 1 < M - 1 ? q0 + 64 * QT - 1 : M - 1;
-  const uint32_t tw = chunk_start(s, pos0 + q0) / KT, tiles = (pos0 + qlast) / KT + 1 - tw;
+  const uint32_t tw = key_start(s, pos0 + q0) / KT, tiles = (pos0 + qlast) / KT + 1 - tw;
   const uint32_t kh = h / (s.heads / s.kv_heads);
   const T* K = reinterpret_cast<const T*>(b.kc) + (size_t)kh * s.rows * DQ;
   const T* Vc = reinterpret_cast<const T*>(b.vc) + (size_t)kh * s.rows * s.vp + v0;
@@ -527,16 +543,17 @@ __global__ void __launch_bounds__(256, (gattn_wgs<T, DQ, DV>())) gattn_flash_ker
   }
   f32x4 o[ND][QT];
   float mx[QT], l[QT];
-  uint32_t ci[QT];                                              // where the chunk of this lane's query starts
+  uint32_t ci[QT];                                              // the first key that this lane's query sees
 #pragma unroll
   for (int t = 0; t < QT; t++) {
-    mx[t] = kGattnNeg; l[t] = 0.0f;
-    ci[t] = chunk_start(s, pos0 + qw + t * 16 + r16);
+    mx[t] = s.sink ? 0.0f : kGattnNeg;                          // the sink: a first key of score 0 and no value
+    l[t] = s.sink && g == 0 ? 1.0f : 0.0f;
+    ci[t] = key_start(s, pos0 + qw + t * 16 + r16);
 #pragma unroll
     for (int i = 0; i < ND; i++) o[i][t] = (f32x4)(0.0f);
   }
   const uint32_t iw0 = pos0 + qw, iw1 = iw0 + 16 * QT - 1;      // this wave's queries
-  const uint32_t c0 = chunk_start(s, iw0), c1 = chunk_start(s, iw1);
+  const uint32_t c0 = key_start(s, iw0), c1 = key_start(s, iw1);
   wait_vm(0);
   __syncthreads();
   for (uint32_t it = 0; it < tiles; it++) {
@@ -652,15 +669,16 @@ __global__ void __launch_bounds__(256, (gattn_wgs<T, DQ, DV>())) gattn_flash_ker
       const uint32_t v = v0 + d * 16 + g * 4;
       if (v >= s.vdim) continue;
       if (vec) {
-        const f32x4 z = *reinterpret_cast<const f32x4*>(gt + v);
+        f32x4 z = (f32x4)(0.0f);
+        if (s.gated) z = *reinterpret_cast<const f32x4*>(gt + v);
         T r[4];
 #pragma unroll
-        for (int e = 0; e < 4; e++) r[e] = to_act<T>(o[d][t][e] * fac * sigmoid_f(z[e]));
+        for (int e = 0; e < 4; e++) r[e] = to_act<T>(o[d][t][e] * fac * (s.gated ? sigmoid_f(z[e]) : 1.0f));
         __builtin_memcpy(__builtin_assume_aligned(dst + v, sizeof(r)), r, sizeof(r));
       } else {
 #pragma unroll
         for (int e = 0; e < 4; e++)
-          if (v + e < s.vdim) dst[v + e] = to_act<T>(o[d][t][e] * fac * sigmoid_f(gt[v + e]));
+          if (v + e < s.vdim) dst[v + e] = to_act<T>(o[d][t][e] * fac * (s.gated ? sigmoid_f(gt[v + e]) : 1.0f));
       }
     }
   }

@@ -92,12 +92,7 @@ __device__ __forceinline__ void gla_step(const GlaShape& s, const GlaBufs& b, ui
 
 // a wave: head h's output of one token (num, its row of cat), normed and gated -> o [vdim]
 template <class O> __device__ __forceinline__ void gla_read_out(const GlaShape& s, const float* norm, const float* num, const float* cat, uint32_t h, O* o) {
-  const uint32_t lane = threadIdx.x & 63;
-  const float* gate = cat + s.off_g + (size_t)h * s.vdim;
-  float ss = 0.0f;
-  for (uint32_t j = lane; j < s.vdim; j += 64) ss = __builtin_fmaf(num[j], num[j], ss);
-  const float r = s.out_scale / __builtin_sqrtf(wave_sum(ss) / (float)s.vdim + s.eps);
-  for (uint32_t j = lane; j < s.vdim; j += 64) o[j] = to_act<O>(num[j] * r * norm[j] * silu_f(gate[j]));
+  head_read_out<O>(num, norm, cat + s.off_g + (size_t)h * s.vdim, s.vdim, s.eps, s.out_scale, o);
 }
 
 }  // namespace lgh

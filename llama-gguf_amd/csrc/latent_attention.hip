@@ -13,14 +13,19 @@
 
 namespace lgh {
 
-constexpr float kNegHuge = -1e30f, kLog2e = 1.4426950408889634f;
+constexpr float kNegHuge = -1e30f, kNegRef = -1e25f, kLog2e = 1.4426950408889634f;
 
-// token t of a block -> rotated pair i of src
-__device__ __forceinline__ void rot_pair(const float* src, const float* cs, uint32_t i, float& a, float& b) {
-  const float u = src[2 * i], v = src[2 * i + 1], c = cs[2 * i], s = cs[2 * i + 1];
-  a = u * c - v * s;
-  b = v * c + u * s;
+// value i (below rot_n) of a rotated part
+__device__ __forceinline__ float rot_value(const LatentShape& s, const float* src, const float* cs, uint32_t i) {
+  const uint32_t half = s.rot_n / 2, p = s.halves ? (i < half ? i : i - half) : i >> 1;   // its pair
+  const bool second = s.halves ? i >= half : i & 1;
+  const float u = src[s.halves ? p : 2 * p], v = src[s.halves ? p + half : 2 * p + 1], c = cs[2 * p], n = cs[2 * p + 1];
+  return second ? v * c + u * n : u * c - v * n;
 }
+
+// the first key that position i sees; never falls with i
+__host__ __device__ __forceinline__ uint32_t lat_key_start(uint32_t window, uint32_t i) { return i >= window ? i - window + 1 : 0; }
+uint32_t latent_key_start(const LatentShape& s, uint32_t i) { return lat_key_start(s.window, i); }
 
 // cache row of token t: RMS norm of the latent, rotation of the shared key part.  One workgroup.
 template <class T>
@@ -33,7 +38,7 @@ __device__ __forceinline__ void latent_cache_row(const LatentShape& s, const Lat
   const float* cs = b.cs + (size_t)pos * s.rot_n;
   for (uint32_t i = threadIdx.x; i < s.rot_dim; i += 256) {
     float v = dkv[s.rank + i];
-    if (i < s.rot_n) { float p0, p1; rot_pair(dkv + s.rank, cs, i >> 1, p0, p1); v = (i & 1) ? p1 : p0; }
+    if (i < s.rot_n) v = rot_value(s, dkv + s.rank, cs, i);
     row[s.rank + i] = to_act<T>(v);
   }
 }
@@ -50,7 +55,7 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(const LatentShape s, c
     if (blockIdx.x == 0) latent_cache_row<T>(s, b, cat + s.off_dkv, pos, red);
     return;
   }
-  const float* q = cat + s.off_q + (size_t)h * (s.dim + s.rot_dim);
+  const float* q = b.q + (size_t)t * s.ldq + (size_t)h * (s.dim + s.rot_dim);
   T* qa = reinterpret_cast<T*>(b.qa) + ((size_t)t * s.heads + h) * s.ldc;
   for (uint32_t i = tid; i < s.dimp; i += 256) qn[i] = i < s.dim ? q[i] : 0.0f;
   __syncthreads();
@@ -77,14 +82,14 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(const LatentShape s, c
     const float* cs = b.cs + (size_t)pos * s.rot_n;
     for (uint32_t i = tid; i < s.ldc - s.rank; i += 256) {
       float v = i < s.rot_dim ? q[s.dim + i] : 0.0f;
-      if (i < s.rot_n) { float p0, p1; rot_pair(q + s.dim, cs, i >> 1, p0, p1); v = (i & 1) ? p1 : p0; }
+      if (i < s.rot_n) v = rot_value(s, q + s.dim, cs, i);
       qa[s.rank + i] = to_act<T>(v);
     }
   }
 }
 
 hipError_t latent_prep_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, bool f32, hipStream_t st) {
-  if (s.dimp % 8 || s.ldc < s.rank + s.rot_dim || s.rot_n > s.rot_dim || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
+  if (s.dimp % 8 || s.ldc < s.rank + s.rot_dim || s.rot_n > s.rot_dim || !b.q || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
   const dim3 grid((s.rank + 63) / 64, s.heads + 1, M);
   if (f32) hipLaunchKernelGGL(latent_prep_kernel<float>, grid, dim3(256), s.dimp * 4, st, s, b, pos_ptr, pos0);
   else hipLaunchKernelGGL(latent_prep_kernel<__bf16>, grid, dim3(256), s.dimp * 4, st, s, b, pos_ptr, pos0);
@@ -116,9 +121,9 @@ __global__ void __launch_bounds__(256 * lat_teams<T>()) latent_attn_kernel(const
   const uint32_t r16 = lane & 15, g = lane >> 4;
   const uint32_t rows = M * s.heads, row0 = blockIdx.y * 16, sp = blockIdx.x, col0 = blockIdx.z * (NCT * 64);   // (a split's row tiles on one XCD when the splits are a multiple of 8)
   const uint32_t p0 = pos_ptr ? (uint32_t)*pos_ptr : pos0;
-  const uint32_t kv = p0 + M;                                   // keys 0 .. kv - 1
-  const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles + n_splits - 1) / n_splits;
-  const uint32_t tb = sp * per, te = tb + per < tiles ? tb + per : tiles;
+  const uint32_t kv = p0 + M, tile0 = lat_key_start(s.window, p0) / KT;   // keys up to kv - 1, from the first token's first visible one on
+  const uint32_t tiles = (kv + KT - 1) / KT, per = (tiles - tile0 + n_splits - 1) / n_splits;
+  const uint32_t tb = tile0 + sp * per, te = tb + per < tiles ? tb + per : tiles;
   if (tb >= te) return;                                         // (the merge skips the same splits)
   const uint32_t ld = s.ldc, cpr = ld / PER, nu = cpr / 4;      // 16-byte chunks (a multiple of 8) and units of a row
   T* Cs = reinterpret_cast<T*>(smem) + (q_alias ? 0 : 16 * ld); // [team][nbuf][KT][ld]
@@ -149,7 +154,7 @@ __global__ void __launch_bounds__(256 * lat_teams<T>()) latent_attn_kernel(const
   const uint32_t t_first = tb + team;
   for (uint32_t i = 0; i < ahead && t_first + i * TM < te; i++) stage(t_first + i * TM, i);
   const uint32_t row = row0 + r16 < rows ? row0 + r16 : rows - 1;   // this lane's (token, head) row
-  const uint32_t lim = p0 + row / s.heads + 1;                  // keys it sees
+  const uint32_t lim = p0 + row / s.heads + 1, low = lat_key_start(s.window, lim - 1);   // keys it sees: low .. lim - 1
   // bf16: scores in units of log2 (one v_exp per weight); f32: natural, with the library exponential
   const float scl = BF ? s.scale * kLog2e : s.scale;
   auto ex = [](float x) { return BF ? __builtin_amdgcn_exp2f(x) : expf(x); };
@@ -210,7 +215,7 @@ __global__ void __launch_bounds__(256 * lat_teams<T>()) latent_attn_kernel(const
     for (int n = 0; n < 2; n++)
 #pragma unroll
       for (int e = 0; e < 4; e++) {
-        const float v = k0 + n * 16 + g * 4 + e < lim ? sa[n][e] * scl : kNegHuge;
+        const float v = k0 + n * 16 + g * 4 + e - low < lim - low ? sa[n][e] * scl : kNegHuge;
         sa[n][e] = v;
         m1 = fmaxf(m1, v);
       }
@@ -222,7 +227,7 @@ __global__ void __launch_bounds__(256 * lat_teams<T>()) latent_attn_kernel(const
     for (int n = 0; n < 2; n++)
 #pragma unroll
       for (int e = 0; e < 4; e++) {
-        const float p = k0 + n * 16 + g * 4 + e < lim ? ex(sa[n][e] - m1) : 0.0f;
+        const float p = k0 + n * 16 + g * 4 + e - low < lim - low ? ex(sa[n][e] - m1) : 0.0f;
         sa[n][e] = p;
         sum += p;
       }
@@ -323,7 +328,7 @@ static hipError_t latent_attn_go(const LatentShape& s, const LatentBufs& b, cons
 hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, bool f32,
                               hipStream_t st) {
   const LatentPlan pl = latent_plan(s, f32);
-  if (!pl.bytes || s.ldc % 64 || n_splits == 0 || n_splits > kLatMaxSplits || M == 0 || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
+  if (!pl.bytes || s.window == 0 || s.ldc % 64 || n_splits == 0 || n_splits > kLatMaxSplits || M == 0 || (uint64_t)M * s.heads > kLatAbsorbRows) return hipErrorInvalidValue;
   const uint32_t nct = (s.rank + 63) / 64;
 #define LGH_LAT_CASE(N) return f32 ? latent_attn_go<float, N>(s, b, pos_ptr, pos0, M, n_splits, pl, zs, st) : latent_attn_go<__bf16, N>(s, b, pos_ptr, pos0, M, n_splits, pl, zs, st)
   uint32_t zs = 1;
@@ -347,8 +352,8 @@ __global__ void __launch_bounds__(512) latent_out_kernel(const LatentShape s, co
   extern __shared__ __attribute__((aligned(16))) float lat[];   // [rankp], with room for the merge's thread groups
   __shared__ float wgt[kLatMaxSplits];
   const uint32_t tid = threadIdx.x, r = blockIdx.y, t = r / s.heads, h = r % s.heads, rows = M * s.heads;
-  const uint32_t kv = (pos_ptr ? (uint32_t)*pos_ptr : pos0) + M;
-  const uint32_t tiles = (kv + kLatKeys - 1) / kLatKeys, per = (tiles + n_splits - 1) / n_splits, act = (tiles + per - 1) / per;
+  const uint32_t p0 = pos_ptr ? (uint32_t)*pos_ptr : pos0, kv = p0 + M;
+  const uint32_t tiles = (kv + kLatKeys - 1) / kLatKeys - lat_key_start(s.window, p0) / kLatKeys, per = (tiles + n_splits - 1) / n_splits, act = (tiles + per - 1) / per;
   const uint32_t lane = tid & 63, w = tid >> 6;
   static_assert(kLatMaxSplits == 128, "two splits per lane");
   float mi[2], li[2];
@@ -411,7 +416,13 @@ __global__ void __launch_bounds__(512) latent_out_kernel(const LatentShape s, co
     if (tid < quads) acc4[tid] = v;
     __syncthreads();
   }
-  const float gate = sigmoid_f(b.cat[(size_t)t * s.ldcat + s.off_g + h]);
+  const float* gates = b.cat + (size_t)t * s.ldcat + s.off_g;
+  float gate[4];
+#pragma unroll
+  for (int it = 0; it < 4; it++) {
+    const uint32_t v = blockIdx.x * 32 + it * 8 + w;
+    gate[it] = gates[s.gate_values ? h * s.vdim + (v < s.vdim ? v : 0) : h];
+  }
 #pragma unroll
   for (int it = 0; it < 4; it++) {
     const uint32_t v = blockIdx.x * 32 + it * 8 + w;
@@ -427,7 +438,7 @@ __global__ void __launch_bounds__(512) latent_out_kernel(const LatentShape s, co
       acc = __builtin_fmaf(bf_lo(wv.w), x1.z, acc); acc = __builtin_fmaf(bf_hi(wv.w), x1.w, acc);
     }
     acc = wave_sum_to_lane63(acc);
-    if (lane == 63) out[(size_t)t * ldo + h * s.vdim + v] = to_act<O>(acc * gate);
+    if (lane == 63) out[(size_t)t * ldo + h * s.vdim + v] = to_act<O>(acc * sigmoid_f(gate[it]));
   }
 }
 
@@ -463,18 +474,14 @@ __global__ void __launch_bounds__(256) latent_flash_prep_kernel(const LatentShap
   const uint32_t hd = s.dim + s.rot_dim;
   for (uint32_t i = threadIdx.x; i < s.heads * dq; i += 256) {
     const uint32_t h = i / dq, j = i % dq;
-    const float* src = cat + s.off_q + (size_t)h * hd;
+    const float* src = b.q + (size_t)t * s.ldq + (size_t)h * hd;
     float v = j < hd ? src[j] : 0.0f;
-    if (j >= s.dim && j - s.dim < s.rot_n) {
-      float p0, p1;
-      rot_pair(src + s.dim, cs, (j - s.dim) >> 1, p0, p1);
-      v = ((j - s.dim) & 1) ? p1 : p0;
-    }
+    if (j >= s.dim && j - s.dim < s.rot_n) v = rot_value(s, src + s.dim, cs, j - s.dim);
     q[((size_t)h * Mcap + t) * dq + j] = to_act<T>(v);
   }
 }
 
-// the shared rotated key part of every cached position, beside each head's own key; grid (positions)
+// the shared rotated key part of every cached position (cache: from the first one on), beside each head's own key; grid (positions)
 template <class T>
 __global__ void __launch_bounds__(256) latent_rot_spread_kernel(const LatentShape s, const T* __restrict__ cache, T* __restrict__ k, uint32_t dq, uint64_t Tcap) {
   const uint32_t t = blockIdx.x;
@@ -485,13 +492,14 @@ __global__ void __launch_bounds__(256) latent_rot_spread_kernel(const LatentShap
 }
 
 hipError_t latent_flash_prep_launch(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, bool f32, hipStream_t st) {
-  if (M == 0 || M > f.Mcap || pos0 + M > f.Tcap) return hipErrorInvalidValue;
+  if (M == 0 || M > f.Mcap || f.base % 64 || f.base > pos0 || pos0 - f.base + M > f.Tcap || f.base > lat_key_start(s.window, pos0) || !b.q) return hipErrorInvalidValue;
+  const uint32_t n = pos0 - f.base + M;
   if (f32) {
     hipLaunchKernelGGL(latent_flash_prep_kernel<float>, dim3(M), dim3(256), 0, st, s, b, (float*)f.q, f.dq, f.Mcap, pos0);
-    if (s.rot_dim) hipLaunchKernelGGL(latent_rot_spread_kernel<float>, dim3(pos0 + M), dim3(256), 0, st, s, (const float*)b.cache, (float*)f.k, f.dq, f.Tcap);
+    if (s.rot_dim) hipLaunchKernelGGL(latent_rot_spread_kernel<float>, dim3(n), dim3(256), 0, st, s, (const float*)b.cache + (size_t)f.base * s.ldc, (float*)f.k, f.dq, f.Tcap);
   } else {
     hipLaunchKernelGGL(latent_flash_prep_kernel<__bf16>, dim3(M), dim3(256), 0, st, s, b, (__bf16*)f.q, f.dq, f.Mcap, pos0);
-    if (s.rot_dim) hipLaunchKernelGGL(latent_rot_spread_kernel<__bf16>, dim3(pos0 + M), dim3(256), 0, st, s, (const __bf16*)b.cache, (__bf16*)f.k, f.dq, f.Tcap);
+    if (s.rot_dim) hipLaunchKernelGGL(latent_rot_spread_kernel<__bf16>, dim3(n), dim3(256), 0, st, s, (const __bf16*)b.cache + (size_t)f.base * s.ldc, (__bf16*)f.k, f.dq, f.Tcap);
   }
   return hipGetLastError();
 }
@@ -516,7 +524,7 @@ __global__ void __launch_bounds__(256, (flash_wgs<T, DQ, DV>())) latent_flash_ke
   const uint32_t h = blockIdx.x % s.heads, qi = blockIdx.x / s.heads, hi = (nqb + 1) / 2, qb = qi < hi ? nqb - 1 - qi : qi - hi;
   const uint32_t q0 = qb * 64 * QT, qw = q0 + w * 16 * QT;
   const uint32_t qlast = q0 + 64 * QT - 1 < M - 1 ? q0 + 64 * QT - 1 : M - 1;
-  const uint32_t tiles = (pos0 + qlast + KT) / KT;   // keys 0 .. pos0 + qlast
+  const uint32_t tw = lat_key_start(s.window, pos0 + q0) / KT, tiles = (pos0 + qlast + KT) / KT;   // keys up to pos0 + qlast (positions count from f.base)
   const T* K = reinterpret_cast<const T*>(f.k) + (size_t)h * f.Tcap * DQ;
   const T* V = reinterpret_cast<const T*>(f.vt) + (size_t)h * f.dvp * f.Tcap;
   auto stage = [&](uint32_t tl, uint32_t buf) {
@@ -532,7 +540,7 @@ __global__ void __launch_bounds__(256, (flash_wgs<T, DQ, DV>())) latent_flash_ke
       lds_dma16(V + (size_t)row * f.Tcap + (size_t)tl * KT + ch * (16 / sizeof(T)), base + kK + (i * 4 + w) * 1024);
     }
   };
-  stage(0, 0);
+  stage(tw, 0);
   typename Frag<T>::V qf[QT][NU];
 #pragma unroll
   for (int t = 0; t < QT; t++) {
@@ -545,7 +553,7 @@ __global__ void __launch_bounds__(256, (flash_wgs<T, DQ, DV>())) latent_flash_ke
   float mx[QT], l[QT];
 #pragma unroll
   for (int t = 0; t < QT; t++) {
-    mx[t] = kNegHuge; l[t] = 0.0f;
+    mx[t] = kNegRef; l[t] = 0.0f;   // (far above a masked score: a query that has seen nothing yet weighs masked keys with 0)
 #pragma unroll
     for (int i = 0; i < ND; i++) o[i][t] = (f32x4)(0.0f);
   }
@@ -553,8 +561,9 @@ __global__ void __launch_bounds__(256, (flash_wgs<T, DQ, DV>())) latent_flash_ke
   const float sc = BF ? s.scale * kLog2e : s.scale;
   __builtin_amdgcn_s_waitcnt(0x0F70);   // vmcnt(0)
   __syncthreads();
-  for (uint32_t tl = 0; tl < tiles; tl++) {
-    const uint32_t cur = tl & 1, k0 = tl * KT;
+  const uint32_t low1 = lat_key_start(s.window, pos0 + qw + 16 * QT - 1);   // (wave-uniform) every query of this wave sees all keys from here to pos0 + qw
+  for (uint32_t tl = tw; tl < tiles; tl++) {
+    const uint32_t cur = (tl - tw) & 1, k0 = tl * KT;
     if (tl + 1 < tiles) stage(tl + 1, cur ^ 1);
     const uint8_t* kb = smem + cur * kBuf;
     const uint8_t* vb = kb + kK;
@@ -572,15 +581,15 @@ __global__ void __launch_bounds__(256, (flash_wgs<T, DQ, DV>())) latent_flash_ke
 #pragma unroll
         for (int t = 0; t < QT; t++) sa[n][t] = Frag<T>::mma(kf, qf[t][u], sa[n][t]);
       }
-    if (k0 + KT > pos0 + qw + 1) {   // wave-uniform: some key may lie behind some query
+    if (k0 + KT > pos0 + qw + 1 || k0 < low1) {   // wave-uniform: some key may lie behind some query, or before its window
       asm volatile("");              // (kept a branch: most tiles have no masks to apply)
 #pragma unroll
       for (int t = 0; t < QT; t++) {
-        const uint32_t lim = pos0 + qw + t * 16 + r16;   // last visible key
+        const uint32_t lim = pos0 + qw + t * 16 + r16, low = lat_key_start(s.window, lim);   // first and last visible key
 #pragma unroll
         for (int n = 0; n < NK; n++)
 #pragma unroll
-          for (int e = 0; e < 4; e++) sa[n][t][e] = k0 + n * 16 + g * 4 + e > lim ? kNegHuge : sa[n][t][e];
+          for (int e = 0; e < 4; e++) sa[n][t][e] = k0 + n * 16 + g * 4 + e - low > lim - low ? kNegHuge : sa[n][t][e];
       }
     }
 #pragma unroll
@@ -594,7 +603,7 @@ __global__ void __launch_bounds__(256, (flash_wgs<T, DQ, DV>())) latent_flash_ke
       m1 = fmaxf(m1, __shfl_xor(m1, 32, 64));
       const float off = -m1 * sc;
       auto weight = [&](float v) { const float x = __builtin_fmaf(v, sc, off); return BF ? __builtin_amdgcn_exp2f(x) : expf((v - m1) * sc); };
-      const float a = weight(mx[t]);
+      const float a = BF ? __builtin_amdgcn_exp2f((mx[t] - m1) * sc) : expf((mx[t] - m1) * sc);
       float sum = 0.0f;
 #pragma unroll
       for (int n = 0; n < NK; n++)
@@ -648,14 +657,15 @@ __global__ void __launch_bounds__(256, (flash_wgs<T, DQ, DV>())) latent_flash_ke
     lt += __shfl_xor(lt, 32, 64);
     const uint32_t m = qw + t * 16 + r16;
     if (m >= M) continue;
-    const float fac = sigmoid_f(b.cat[(size_t)m * s.ldcat + s.off_g + h]) / lt;
+    const float* gates = b.cat + (size_t)m * s.ldcat + s.off_g;
+    const float fac = (s.gate_values ? 1.0f : sigmoid_f(gates[h])) / lt;
     T* dst = out + (size_t)m * ldo + h * s.vdim;
 #pragma unroll
     for (int i = 0; i < ND; i++)
 #pragma unroll
       for (int e = 0; e < 4; e++) {
         const uint32_t v = i * 16 + g * 4 + e;
-        if (v < s.vdim) dst[v] = to_act<T>(o[i][t][e] * fac);
+        if (v < s.vdim) dst[v] = to_act<T>(o[i][t][e] * fac * (s.gate_values ? sigmoid_f(gates[h * s.vdim + v]) : 1.0f));
       }
   }
 }
@@ -685,7 +695,9 @@ static hipError_t latent_flash_pick(const LatentShape& s, const LatentBufs& b, c
 hipError_t latent_flash_launch(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, bool f32, void* out, uint32_t ldo,
                                hipStream_t st) {
   const uint64_t KT = f32 ? 32 : 64;
-  if (M == 0 || M > f.Mcap || f.Tcap % 64 || (pos0 + M + KT - 1) / KT * KT > f.Tcap) return hipErrorInvalidValue;   // whole key tiles are read
+  if (M == 0 || M > f.Mcap || f.Tcap % 64 || f.base > pos0 || s.window == 0) return hipErrorInvalidValue;
+  pos0 -= f.base;
+  if ((pos0 + M + KT - 1) / KT * KT > f.Tcap) return hipErrorInvalidValue;   // whole key tiles are read
   return f32 ? latent_flash_pick<float>(s, b, f, pos0, M, out, ldo, st) : latent_flash_pick<__bf16>(s, b, f, pos0, M, out, ldo, st);
 }
 

@@ -43,7 +43,9 @@ enum LinPro : int {
   LP_RESID = 1,   // x + mult * layer_norm(y) * nw, also written to xout (the new residual stream)
   LP_HEAD = 2,    // layer_norm of the same sum, times nw2 (final norm in front of the output projection)
   LP_MLSTM = 3,   // matrix-memory read-out: numerators / denominators, per-head RMS norm, norm weight, sigmoid gate
-  LP_PRE = 4,     // v = x + mult * y (y may be absent), also written to xout; rms_norm(v) * (1 + nw2) * in_scale, also written to hout
+  LP_PRE = 4,     // v = x + mult * y (y may be absent), also written to xout; rms_norm(v) * (nw_add + nw2) * in_scale, also written to hout
+  LP_SANDWICH = 5,// v = x + mult * layer_norm(y) * nw (y may be absent), also written to xout; layer_norm(v) * nw2
+  LP_READ = 6,    // read-out of a matrix state: per-head RMS norm, one norm weight [vdim] for all heads, silu gate
 };
 // Which weights its rows come from
 enum LinSrc : int {
@@ -52,7 +54,8 @@ enum LinSrc : int {
   LS_EXPERTS = 2,  // the top experts of `logits` (every workgroup ranks them), their gate | up pairs; the input is weighted by the expert's score
   LS_MOE_DOWN = 3, // input [shared | expert | expert ..]: a row is a row of w (shared, absent: kps = 0) followed by the same row of every chosen expert
 };
-enum LinAct : uint32_t { LA_GELU = 0, LA_SILU = 1, LA_CLAMPED = 2 };   // act(gate) * up; LA_CLAMPED: clamped_glu_f
+enum LinAct : uint32_t { LA_GELU = 0, LA_SILU = 1, LA_CLAMPED = 2,     // act(gate) * up; LA_CLAMPED: clamped_glu_f
+                        LA_RELU2 = 3 };                                  // unpaired rows: relu(v)^2
 // how a token's experts are chosen (LGH_ROUTER_*)
 struct RouteForm {
   uint32_t form = LGH_ROUTER_SIGMOID;
@@ -70,10 +73,12 @@ struct LinMv {
   const float* nw2;
   float* xout;
   float eps, mult, in_scale;
+  float nw_add;                // LP_PRE
+  float cap;                   // unpaired rows: cap * tanh(v / cap) (0: none)
   const float* bias;           // [n], unpaired rows (NULL: none)
   float* hout;                 // LP_PRE: the input vector (NULL: not kept)
   float limit;                 // LA_CLAMPED
-  const float* num;            // LP_MLSTM: [heads][ldo] numerators, column vdim = n . q, column vdim + 1 = exp(-m)
+  const float* num;            // LP_READ: [heads][ldo]; LP_MLSTM: [heads][ldo] numerators, column vdim = n . q, column vdim + 1 = exp(-m)
   const float* gate;
   uint32_t heads, vdim, ldo;
   const uint16_t* w2;          // LS_TWO: second matrix; LS_EXPERTS / LS_MOE_DOWN: the experts, one below the other
@@ -103,6 +108,7 @@ enum LinEpi : int {
   LE_HEADS = 3,   // activation type, row n = head * hd + j of token m at out[(head * tcap + m) * ldo + j]
   LE_HEADS_T = 4, // activation type, transposed per head: out[(head * hrows + j) * ldo + m]
   LE_SWIGLU = 5,  // paired weights: silu(gate) * up as activation type [M][ldo]
+  LE_RELU2 = 7,   // activation type, relu(v)^2
   LE_CLAMPED = 6, // grouped rows, paired weights: scale * clamped_glu_f(gate, up) as activation type [M][ldo]
 };
 // rows grouped by expert: row tile i takes rows tile_row[i] .. of the group tile_e[i] (-1: no tile), which ends at seg[group + 1]; that
@@ -123,6 +129,7 @@ struct LinGemm {
   uint32_t hd, hrows;          // LE_HEADS / LE_HEADS_T
   uint64_t tcap;
   const float* bias;           // LE_F32: [n] (NULL: none)
+  float cap;                   // LE_F32: cap * tanh(v / cap) (0: none)
   LinGroup grp;
 };
 hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st);
@@ -192,6 +199,18 @@ struct PreBlock {
   float eps, mult;
 };
 hipError_t pre_block_launch(const PreBlock& a, bool f32, hipStream_t st);
+// LGH_RESIDUAL_SANDWICH_LN over a block: x += mult * layer_norm(y) * pw (y NULL: not yet); layer_norm(x) * nw -> xa (nw NULL: not wanted)
+struct LnBlock {
+  float* x;
+  const float *y, *pw, *nw;
+  void* xa;
+  uint32_t ldy, ldx, width, M;
+  float eps, mult;
+};
+hipError_t ln_block_launch(const LnBlock& a, bool f32, hipStream_t st);
+// rms_norm of n columns of every row * w, as activations (columns n .. ldx are not touched)
+hipError_t rms_cols_launch(const float* x, uint32_t ld, const float* w, float eps, uint32_t n, uint32_t M, void* xa, uint32_t ldx, bool f32, hipStream_t st);
+hipError_t vec_mul_launch(float* x, const float* y, uint32_t n, hipStream_t st);   // x *= y
 // decode without a consumer: xout = x + mult * y
 hipError_t resid_add_launch(const float* x, const float* y, float mult, uint32_t width, float* xout, hipStream_t st);
 hipError_t final_rms_rows_launch(const float* x, const int* rows, uint32_t n_rows, const float* w, float eps, float scale, uint32_t width, void* xa, uint32_t ldx,
@@ -265,18 +284,20 @@ hipError_t gla_block_launch(const GlaShape& s, const GlaBufs& b, uint32_t pos0, 
 // per-head RMS norm, norm weight, silu gate, out_scale -> columns of out
 hipError_t gla_out_launch(const GlaShape& s, const GlaBufs& b, uint32_t M, void* out, uint32_t ldo, bool f32, hipStream_t st);
 
-// ---- gated_attention.hip: grouped heads with values of their own ----
+// ---- gated_attention.hip: grouped heads with values of their own; norms, gate, chunks, window and sink as the layer has them ----
 struct GattnShape {
   uint32_t heads, kv_heads, dim, vdim, dp, vp;   // dp, vp: row strides of the caches, multiples of 64
   uint32_t off_q, off_k, off_v, off_g, ldcat;
-  uint32_t chunk;                      // i sees j <= i with j / chunk == i / chunk
+  uint32_t chunk, window;              // i sees j <= i with j / chunk == i / chunk and i - j < window
+  uint32_t gated, sink;                // 0 or 1: outputs times sigmoid(cat + off_g); the softmax's denominator has one more term, exp(0)
   uint32_t rot_n;                      // leading values of a head that are rotated
   uint64_t rows;                       // cache rows per key head, multiple of 64
   float scale, eps, out_scale;
 };
 struct GattnBufs {
   const float* cat;                    // [M][ldcat]
-  const float *qn, *kn, *cs;           // norm weights [dim]; [max_seq][rot_n / 2][2]
+  const float *qn, *kn, *cs;           // norm weights [dim] (NULL: queries and keys are not normed); [max_seq][rot_n / 2][2]
+  bool shared;                         // the keys and values are another layer's: nothing is written to the caches
   void *kc, *vc;                       // [kv_heads][rows][dp | vp]: keys normed and rotated, values
   void* q;                             // blocks: [heads][Mcap][dp]
   uint32_t Mcap;
@@ -293,6 +314,34 @@ hipError_t gattn_merge_launch(const GattnShape& s, const GattnBufs& b, const Gla
                               uint32_t M, uint32_t n_splits, bool f32, void* out, uint32_t ldo, bool out_f32, hipStream_t st);
 hipError_t gattn_prep_launch(const GattnShape& s, const GattnBufs& b, uint32_t pos0, uint32_t M, bool f32, hipStream_t st);
 hipError_t gattn_flash_launch(const GattnShape& s, const GattnBufs& b, uint32_t pos0, uint32_t M, bool f32, void* out, uint32_t ldo, hipStream_t st);
+
+// ---- delta.hip: gated delta rule, S_t = g_t S_(t-1) + k_t u_t^T with u_t = beta_t (v_t - g_t S_(t-1)^T k_t) per head, out S_t^T q_t ----
+struct DeltaShape {
+  uint32_t heads, kv_heads, dim, vdim, taps;
+  uint32_t dk, lv;                     // dim, vdim up to 16: row strides of queries and keys; of the state [head][dk][lv], values and outputs
+  uint32_t off_q, off_k, off_v, off_g, off_b, off_a, ldcat;
+  uint32_t cols;                       // leading columns of cat that pass the convolution (queries, keys, values)
+  float eps;
+};
+struct DeltaBufs {
+  const float* cat;                    // [M][ldcat]
+  const float* conv;                   // [cols][taps], the last tap at the token itself
+  const float *a_log, *dt, *norm;      // [heads], [heads], [vdim]
+  float* S;
+  float* hist;                         // [taps][cols]: the convolution's input at position p lies in row p % taps
+  float* num;                          // [M][heads][lv] outputs before their norm; blocks: whole chunks of 64 tokens
+  // blocks, whole chunks of 64 tokens (zeros behind the last token and in the padding)
+  float *q, *k;                        // [Mcap][kv_heads][dk] unit queries (times dim^-1/2) and keys
+  float *v, *u;                        // [Mcap][heads][lv] values; what a chunk writes from an empty state
+  float *w, *p;                        // [Mcap][heads][dk] what the state before the chunk takes off u; what it adds to the outputs
+  float *wge, *cd;                     // [heads][Mcap] decay from a token to its chunk's end; [heads][Mcap / 64] a chunk's decay
+  uint32_t Mcap;
+};
+constexpr uint32_t kDeltaBlockDim = 512;     // larger heads take blocks token by token
+hipError_t delta_step_launch(const DeltaShape& s, const DeltaBufs& b, const int* pos_ptr, uint32_t pos0, hipStream_t st);
+hipError_t delta_block_launch(const DeltaShape& s, const DeltaBufs& b, uint32_t pos0, uint32_t M, hipStream_t st);
+// read-out of a block (per-head RMS norm, norm weight, silu gate), and what the sequence keeps of the convolution's inputs
+hipError_t delta_out_launch(const DeltaShape& s, const DeltaBufs& b, uint32_t pos0, uint32_t M, void* out, uint32_t ldo, bool f32, hipStream_t st);
 
 // ---- glru.hip: S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t per channel ----
 struct GlruShape {
@@ -319,11 +368,15 @@ struct LatentShape {
   uint32_t heads, dim, rot_dim, rot_n, vdim, rank;
   uint32_t ldc;                // elements of a cache row: [latent rank | rotated key part rot_dim | zeros], multiple of 64
   uint32_t dimp, rankp;        // row strides of the transposed key expansion [head][rank][dimp] and the value expansion [head * vdim][rankp]
-  uint32_t off_q, off_dkv, off_g, ldcat;   // where a token's projections lie in its row of the fused product
+  uint32_t off_q, off_dkv, off_g, ldcat;   // where a token's projections lie in its row of the fused product (off_q: queries, or their latent)
+  uint32_t ldq;                // row stride of the queries
+  uint32_t window;             // i sees j <= i with i - j < window
+  uint32_t halves, gate_values;   // 0 or 1: pairs (i, i + rot_n / 2) instead of (2i, 2i + 1); a gate per value instead of per head
   float scale, eps;
 };
 struct LatentBufs {
   const float* cat;            // [M][ldcat]
+  const float* q;              // [M][ldq]: queries, head by head [dim | rot_dim]
   const float* dkv_norm;       // [rank]
   const float* cs;             // [max_seq][rot_n / 2][2]
   const uint16_t *uk_t, *uv;
@@ -340,14 +393,16 @@ hipError_t latent_attn_launch(const LatentShape& s, const LatentBufs& b, const i
 // merges the splits, expands the latent to the value and applies the head gate -> out [M][ldo] (f32 vector in decode, activations otherwise)
 hipError_t latent_out_launch(const LatentShape& s, const LatentBufs& b, const int* pos_ptr, uint32_t pos0, uint32_t M, uint32_t n_splits, void* out, uint32_t ldo, bool out_f32, hipStream_t st);
 bool latent_fits(const LatentShape& s, bool f32);   // the absorbed kernel's tiles fit LDS
-// expanded path (long prompts): keys and values per head
+// expanded path (long prompts): keys and values per head, from position `base` on
 struct LatentFlash {
   void* q;                     // [heads][Mcap][dq]
   void* k;                     // [heads][Tcap][dq]
   void* vt;                    // [heads][dvp][Tcap]
   uint32_t dq, dvp, Mcap;
+  uint32_t base;               // a multiple of 64, no position before it is visible
   uint64_t Tcap;
 };
+uint32_t latent_key_start(const LatentShape& s, uint32_t i);   // the first key that position i sees
 bool latent_flash_shape(const LatentShape& s, uint32_t* dq, uint32_t* dvp);
 hipError_t latent_flash_prep_launch(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, bool f32, hipStream_t st);
 hipError_t latent_flash_launch(const LatentShape& s, const LatentBufs& b, const LatentFlash& f, uint32_t pos0, uint32_t M, bool f32, void* out,

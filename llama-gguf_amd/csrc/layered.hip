@@ -8,14 +8,18 @@
 //   tied attention     fused q | k product -> split attention (norms of q and k in its prologue, cache row written) -> merge -> output product
 //   gated attention    fused q | k | v | gate product -> split attention (norms and rotation in its prologue, cache rows written) -> merge + gate ->
 //                      output product; a gated linear attention beside it steps and is read out in the same launches, one output product for both
+//   grouped attention  the same without norms and gate; a layer that reads another layer's cache rows projects queries only
+//   latent attention with a query latent: fused query latent | latent | gate product -> query product (the latent's norm in its prologue) -> as above
+//   delta rule         fused q | k | v | gate, step and decay product -> convolution and state step -> output product (read-out norm and gate in its prologue)
 //   linear recurrence  fused y | x product -> convolution, gates and recurrence step -> output product
-//   feed-forward       gate | up product with gelu * in its epilogue -> down product
+//   feed-forward       gate | up product with gelu * in its epilogue (or up product with the squared relu) -> down product
 //   mixture            shared gate | up + router product -> the chosen experts' gate | up (every workgroup ranks the scores) -> one down
 //                      product over [shared | experts]
 // With norms in front of the sublayers (LGH_RESIDUAL_PRE_RMS) the prologue of the product that reads the stream updates and norms it.
+// With layer norms on both sides (LGH_RESIDUAL_SANDWICH_LN) it norms the sublayer's output, updates the stream and norms that.
 // With squashing norms (LGH_RESIDUAL_SANDWICH_DYT) everything between two sublayers is per channel: it rides in the EPILOGUE of the
 // product that finishes a channel, and no norm is computed more than once.
-// A sequence's state: the cache rows, the matrix memories with their running maxima, the linear recurrences, the convolutions' last inputs, and the last token
+// A sequence's state: the cache rows, the matrix states (and running maxima), the linear recurrences, the convolutions' last inputs, and the last token
 // (pair embedding), kept as a token history by position; a position of 0 makes every kernel ignore what is stored, so lgh_reset stays O(1).
 #include <algorithm>
 #include <cmath>
@@ -44,6 +48,10 @@ struct LayeredLayer {
   GattnShape gs{};
   GlaShape as{};
   GlruShape rs{};
+  DeltaShape des{};
+  LinW uq;                                 // latent attention: the queries' second projection
+  float *dq_norm = nullptr, *a_log = nullptr, *dt = nullptr, *out_bias = nullptr;
+  float *post1 = nullptr, *post2 = nullptr, *ls1 = nullptr, *ls2 = nullptr;   // LGH_RESIDUAL_SANDWICH_LN: norms behind the sublayers (times ls, from finalize on)
   LinW a2, gates;                          // linear attention: the decay's second factor; linear recurrence: its gates' diagonal blocks
   float *in_bias = nullptr, *a2b = nullptr, *gnorm = nullptr, *conv = nullptr, *conv_b = nullptr, *rb = nullptr, *ib = nullptr, *lam = nullptr, *correction = nullptr;
   float *rS = nullptr, *rhist = nullptr;
@@ -59,7 +67,9 @@ struct LayeredLayer {
   bool latent() const { return d.mixer == LGH_MIXER_LATENT_ATTENTION; }
   bool mlstm() const { return d.mixer == LGH_MIXER_MLSTM; }
   bool tied() const { return d.mixer == LGH_MIXER_TIED_ATTENTION; }
-  bool gattn() const { return d.mixer == LGH_MIXER_GATED_ATTENTION || d.mixer == LGH_MIXER_PARALLEL; }
+  bool grouped() const { return d.mixer == LGH_MIXER_GROUPED_ATTENTION; }
+  bool gattn() const { return d.mixer == LGH_MIXER_GATED_ATTENTION || d.mixer == LGH_MIXER_PARALLEL || grouped(); }
+  bool delta() const { return d.mixer == LGH_MIXER_DELTA; }
   bool gla() const { return d.mixer == LGH_MIXER_GLA || d.mixer == LGH_MIXER_PARALLEL; }
   bool glru() const { return d.mixer == LGH_MIXER_GLRU; }
   bool rotated() const { return latent() || gattn(); }
@@ -107,6 +117,7 @@ struct LayeredModel {
   std::vector<LayeredSub> subs;
   LayeredNorm final_dyt;
   float *h = nullptr, *hist = nullptr, *tails = nullptr;   // a sublayer's input (decode); the convolutions' histories and a block's last inputs
+  bool ln2() const { return d.residual == LGH_RESIDUAL_SANDWICH_LN; }
   bool dyt() const { return d.residual == LGH_RESIDUAL_SANDWICH_DYT; }
   bool pre() const { return d.residual == LGH_RESIDUAL_PRE_RMS; }
   size_t hist_floats() const { return d.conv_taps > 1 ? (size_t)n_sub * (d.conv_taps - 1) * d.width : 0; }
@@ -125,6 +136,8 @@ struct LayeredModel {
   // decode
   float *x[2] = {nullptr, nullptr}, *y = nullptr, *cat = nullptr, *ao = nullptr, *act = nullptr, *num = nullptr, *part_ml = nullptr, *part_acc = nullptr;
   void* qa = nullptr;
+  float* lq = nullptr;                     // latent attention with a query latent: a token's queries
+  uint32_t max_lq = 0, max_qrank = 0;
   uint32_t max_cat = 0, max_ao = 0, max_act = 0, max_num = 0;
   // blocks
   bool blk_ready = false;
@@ -137,6 +150,10 @@ struct LayeredModel {
   float *bdec = nullptr, *bwgt = nullptr, *bcdec = nullptr, *bnk = nullptr;
   void *bxa = nullptr, *bao = nullptr, *bact = nullptr, *bla = nullptr;
   int *btok = nullptr, *brows = nullptr;
+  float* blq = nullptr;                    // queries made from their latent
+  void* blqa = nullptr;                    // that latent, normed
+  uint32_t max_dqk = 0, max_dw = 0, max_dv = 0, max_dheads = 0;   // delta rules: kv_heads * dk, heads * dk, heads * lv, heads
+  float *bdq = nullptr, *bdk = nullptr, *bdv = nullptr, *bdu = nullptr, *bdw = nullptr, *bdp = nullptr, *bdwge = nullptr, *bdcd = nullptr;
   // expanded attention (grown with the context)
   LatentFlash fl{};
   size_t fl_q_bytes = 0, fl_k_bytes = 0, fl_v_bytes = 0;
@@ -172,14 +189,16 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
   if (up(d.width, 64) > 32768) { why = "width above 32768"; return LGH_UNSUPPORTED; }
   if (d.tied_head > 1 || !std::isfinite(d.logit_scale)) { why = "output projection"; return LGH_INVALID_ARGUMENT; }
   if (d.logit_scale != 0.0 && d.logit_scale != 1.0 && d.residual != LGH_RESIDUAL_PRE_RMS) { why = "a factor on the logits"; return LGH_UNSUPPORTED; }
-  if (d.residual > LGH_RESIDUAL_PRE_RMS) { why = "unknown residual form"; return LGH_UNSUPPORTED; }
+  if (!(d.logit_cap >= 0.0) || !std::isfinite(d.logit_cap)) { why = "a cap of the logits"; return LGH_INVALID_ARGUMENT; }
+  if (d.residual > LGH_RESIDUAL_SANDWICH_LN) { why = "unknown residual form"; return LGH_UNSUPPORTED; }
   if (d.conv_taps > kMaxConvTaps || (d.conv_taps && d.residual != LGH_RESIDUAL_SANDWICH_DYT)) { why = "convolution taps"; return LGH_UNSUPPORTED; }
   for (uint32_t i = 0; i < d.num_layers; i++) {
     const lgh_layer_desc& l = L[i];
     const std::string at = "layer " + std::to_string(i) + ": ";
     if (l.struct_size != sizeof(lgh_layer_desc)) { why = at + "descriptor size"; return LGH_INVALID_ARGUMENT; }
     if (l.mixer != LGH_MIXER_GLA && (!l.heads || !l.dim || !l.vdim)) { why = at + "a mixer dimension is zero"; return LGH_INVALID_ARGUMENT; }
-    if (l.ff_kind > LGH_FF_MOE || (l.ff_kind && !l.ff)) { why = at + "feed-forward"; return LGH_INVALID_ARGUMENT; }
+    if (l.ff_kind > LGH_FF_RELU2 || (l.ff_kind && !l.ff)) { why = at + "feed-forward"; return LGH_INVALID_ARGUMENT; }
+    if (l.ff_kind == LGH_FF_MOE && d.residual == LGH_RESIDUAL_SANDWICH_LN) { why = at + "mixtures between layer norms"; return LGH_UNSUPPORTED; }
     if (l.ff_kind == LGH_FF_MOE) {
       if (l.router_form > LGH_ROUTER_SOFTMAX_GROUPS || l.expert_form > LGH_EXPERT_CLAMPED) { why = at + "router or expert form"; return LGH_UNSUPPORTED; }
       const bool grp = l.router_form == LGH_ROUTER_SOFTMAX_GROUPS;
@@ -195,11 +214,13 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
       if (l.experts > kMaxExperts || l.top > kMaxTop) { why = at + "more than " + std::to_string(kMaxExperts) + " experts or " + std::to_string(kMaxTop) + " per token"; return LGH_UNSUPPORTED; }
       if ((uint64_t)up(l.shared_ff, 64) + (uint64_t)l.top * up(l.ff, 64) > kLinMvMaxK) { why = at + "a token's experts together above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
     } else if (l.ff_kind && up(l.ff, 64) > kLinMvMaxK) { why = at + "feed-forward above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
-    const bool ga = l.mixer == LGH_MIXER_GATED_ATTENTION || l.mixer == LGH_MIXER_PARALLEL, la = l.mixer == LGH_MIXER_GLA || l.mixer == LGH_MIXER_PARALLEL;
+    const bool gr = l.mixer == LGH_MIXER_GROUPED_ATTENTION, ga = l.mixer == LGH_MIXER_GATED_ATTENTION || l.mixer == LGH_MIXER_PARALLEL || gr, la = l.mixer == LGH_MIXER_GLA || l.mixer == LGH_MIXER_PARALLEL;
     if ((uint64_t)(l.mixer == LGH_MIXER_GLA ? 0 : up(l.heads * l.vdim, 64)) + (la ? up(l.gla_heads * l.gla_vdim, 64) : 0) > kLinMvMaxK) { why = at + "heads * vdim above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
     if (l.mixer == LGH_MIXER_LATENT_ATTENTION) {
       if (!l.kv_rank || l.rot_dims > l.rot_dim || l.rot_dims % 2) { why = at + "latent attention sizes"; return LGH_INVALID_ARGUMENT; }
       if (l.rot_dims && !(l.rot_base > 0.0)) { why = at + "rotation base"; return LGH_INVALID_ARGUMENT; }
+      if (l.rot_form > LGH_ROT_HALVES || l.gate_form > LGH_GATE_VALUES) { why = at + "rotation or gate form"; return LGH_UNSUPPORTED; }
+      if (up(l.q_rank, 64) > kLinMvMaxK) { why = at + "query latent above " + std::to_string(kLinMvMaxK); return LGH_UNSUPPORTED; }
       LatentShape s{};
       s.rank = l.kv_rank;
       s.ldc = up(l.kv_rank + l.rot_dim, 64);
@@ -210,10 +231,22 @@ static int layered_check(const lgh_layered_desc& d, const lgh_layer_desc* L, std
     } else if (ga || la) {
       if (ga) {
         if (!l.kv_heads || l.heads % l.kv_heads || l.rot_dims > l.dim || l.rot_dims % 2 || (l.rot_dims && !(l.rot_base > 0.0))) { why = at + "gated attention sizes"; return LGH_INVALID_ARGUMENT; }
+        if (l.sink_one > 1 || ((l.sink_one || l.kv_from) && !gr)) { why = at + "a sink or shared keys need grouped attention"; return LGH_UNSUPPORTED; }
+        if (l.kv_from) {
+          const lgh_layer_desc& o = L[l.kv_from <= i ? l.kv_from - 1 : i];
+          if (l.kv_from > i || o.mixer != l.mixer || o.kv_from || o.kv_heads != l.kv_heads || o.heads != l.heads || o.dim != l.dim || o.vdim != l.vdim) {
+            why = at + "no such keys and values in layer " + std::to_string(l.kv_from - 1);
+            return LGH_INVALID_ARGUMENT;
+          }
+        }
         if (up(l.dim, 64) > kGattnMaxDim || up(l.vdim, 64) > kGattnMaxDim) { why = at + "heads above " + std::to_string(kGattnMaxDim); return LGH_UNSUPPORTED; }
       }
       if (la && (!l.gla_heads || !l.gla_dim || !l.gla_vdim || !l.gla_rank || !(l.gla_tau > 0.0))) { why = at + "linear attention sizes"; return LGH_INVALID_ARGUMENT; }
       if (!std::isfinite(l.left_scale) || !std::isfinite(l.right_scale)) { why = at + "scales of the two sides"; return LGH_INVALID_ARGUMENT; }
+    } else if (l.mixer == LGH_MIXER_DELTA) {
+      if (!l.kv_heads || l.heads % l.kv_heads || !l.taps) { why = at + "delta rule sizes"; return LGH_INVALID_ARGUMENT; }
+      if (l.taps > kMaxRecTaps) { why = at + "convolution taps"; return LGH_UNSUPPORTED; }
+      if (up(l.dim, 16) > 16384 || 2 * l.kv_heads + l.heads > 65535) { why = at + "delta rule heads"; return LGH_UNSUPPORTED; }
     } else if (l.mixer == LGH_MIXER_GLRU) {
       if (l.vdim != l.dim || !l.taps) { why = at + "linear recurrence sizes"; return LGH_INVALID_ARGUMENT; }
       if (l.taps > kMaxRecTaps) { why = at + "convolution taps"; return LGH_UNSUPPORTED; }
@@ -255,8 +288,12 @@ static void add_dyt(LayeredModel& m, const std::string& nm, LayeredNorm& n) {
   add_vec(m, nm + ".alpha", &n.alpha, 1);
 }
 // the norms around a sublayer ("1": mixer, "2": feed-forward)
-static void add_sub(LayeredModel& m, const std::string& p, const char* which, float** post_ln) {
+static void add_sub(LayeredModel& m, const std::string& p, const char* which, float** post_ln, float** post, float** ls) {
   m.n_sub++;
+  if (m.ln2()) {
+    add_vec(m, p + "norm" + which + "b", post, m.d.width);
+    add_vec(m, p + "ls" + which, ls, m.d.width);
+  }
   if (!m.dyt()) { add_vec(m, p + "norm" + which, post_ln, m.d.width); return; }
   m.subs.emplace_back();                   // (never grows beyond what was reserved: the slots keep addresses)
   LayeredSub& s = m.subs.back();
@@ -281,7 +318,7 @@ static void layered_plan(LayeredModel& m) {
     LayeredLayer& L = m.layers[i];
     const lgh_layer_desc& l = L.d;
     const std::string p = "l" + std::to_string(i) + ".";
-    add_sub(m, p, "1", &L.norm1);
+    add_sub(m, p, "1", &L.norm1, &L.post1, &L.ls1);
     L.in.k = W; L.in.kp = up(W, 64);
     const uint32_t vd = l.mixer == LGH_MIXER_GLA ? 0 : l.heads * l.vdim;
     auto in_seg = [&](const char* nm, uint32_t rows) { const uint32_t at = seg(L.in, rows); add_mat(m, p + "mix." + nm, &L.in, at, rows, W); return at; };
@@ -292,11 +329,22 @@ static void layered_plan(LayeredModel& m) {
       s.dimp = up(l.dim, 8);
       s.rankp = up(l.kv_rank, 64);
       s.scale = (float)l.scale; s.eps = (float)d.norm_eps;
-      s.off_q = in_seg("q", l.heads * (l.dim + l.rot_dim));
+      s.window = l.window ? l.window : 0xFFFFFFFFu;
+      s.halves = l.rot_form == LGH_ROT_HALVES; s.gate_values = l.gate_form == LGH_GATE_VALUES;
+      const uint32_t qrows = l.heads * (l.dim + l.rot_dim);
+      s.off_q = in_seg(l.q_rank ? "dq" : "q", l.q_rank ? l.q_rank : qrows);
       s.off_dkv = in_seg("dkv", l.kv_rank + l.rot_dim);
-      s.off_g = in_seg("g", l.heads);
+      s.off_g = in_seg("g", s.gate_values ? vd : l.heads);
       L.in.n = up(L.in.n, 16);
-      s.ldcat = L.in.n;
+      s.ldcat = s.ldq = L.in.n;
+      if (l.q_rank) {
+        whole(L.uq, qrows, l.q_rank);
+        add_mat(m, p + "mix.uq", &L.uq, 0, qrows, l.q_rank);
+        add_vec(m, p + "mix.dq.norm", &L.dq_norm, l.q_rank);
+        s.ldq = up(qrows, 4);
+        m.max_lq = std::max(m.max_lq, s.ldq);
+        m.max_qrank = std::max(m.max_qrank, L.uq.kp);
+      }
       add_vec(m, p + "mix.dkv.norm", &L.dkv_norm, l.kv_rank);
       whole(L.uk, l.heads * l.dim, l.kv_rank);
       whole(L.uv, vd, l.kv_rank);
@@ -324,6 +372,32 @@ static void layered_plan(LayeredModel& m) {
         m.max_tied_acc = std::max(m.max_tied_acc, rows * l.dim);
       }
       m.max_tied_q = std::max(m.max_tied_q, l.heads * s.dp);
+    } else if (L.delta()) {
+      DeltaShape& s = L.des;
+      s.heads = l.heads; s.kv_heads = l.kv_heads; s.dim = l.dim; s.vdim = l.vdim; s.taps = l.taps; s.dk = up(l.dim, 16); s.lv = up(l.vdim, 16);
+      s.eps = (float)d.norm_eps;
+      const uint32_t qk = l.kv_heads * l.dim;
+      s.off_q = in_seg("q", qk);
+      s.off_k = in_seg("k", qk);
+      s.off_v = in_seg("v", vd);
+      s.cols = s.off_v + vd;
+      s.off_g = in_seg("g", vd);
+      s.off_b = in_seg("b", l.heads);
+      s.off_a = in_seg("a", l.heads);
+      L.in.n = up(L.in.n, 16);
+      s.ldcat = L.in.n;
+      add_bias(m, p + "mix.q.conv", &L.conv, s.off_q * l.taps, qk * l.taps, s.cols * l.taps);
+      add_bias(m, p + "mix.k.conv", &L.conv, s.off_k * l.taps, qk * l.taps, s.cols * l.taps);
+      add_bias(m, p + "mix.v.conv", &L.conv, s.off_v * l.taps, vd * l.taps, s.cols * l.taps);
+      add_vec(m, p + "mix.A_log", &L.a_log, l.heads);
+      add_vec(m, p + "mix.dt_bias", &L.dt, l.heads);
+      add_vec(m, p + "mix.norm", &L.gnorm, l.vdim);
+      m.recurrent = true;
+      m.max_num = std::max(m.max_num, l.heads * s.lv);
+      m.max_dqk = std::max(m.max_dqk, l.kv_heads * s.dk);
+      m.max_dw = std::max(m.max_dw, l.heads * s.dk);
+      m.max_dv = std::max(m.max_dv, l.heads * s.lv);
+      m.max_dheads = std::max(m.max_dheads, l.heads);
     } else if (L.glru()) {
       GlruShape& s = L.rs;
       s.width = vd; s.blocks = l.heads; s.bs = l.dim; s.taps = l.taps;
@@ -354,15 +428,22 @@ static void layered_plan(LayeredModel& m) {
       if (L.gattn()) {
         GattnShape& s = L.gs;
         s.heads = l.heads; s.kv_heads = l.kv_heads; s.dim = l.dim; s.vdim = l.vdim; s.dp = up(l.dim, 64); s.vp = up(l.vdim, 64);
-        s.chunk = l.chunk ? l.chunk : 0xFFFFFFFFu; s.rot_n = l.rot_dims;
+        s.chunk = l.chunk ? l.chunk : 0xFFFFFFFFu; s.window = L.grouped() && l.window ? l.window : 0xFFFFFFFFu; s.rot_n = l.rot_dims;
+        s.gated = !L.grouped(); s.sink = l.sink_one;
         s.rows = up(d.max_seq_len, 64);
         s.scale = (float)l.scale; s.eps = (float)d.norm_eps; s.out_scale = par ? (float)l.left_scale : 1.0f;
         s.off_q = in_seg((left + "q").c_str(), l.heads * l.dim);
-        s.off_k = in_seg((left + "k").c_str(), l.kv_heads * l.dim);
-        s.off_v = in_seg((left + "v").c_str(), l.kv_heads * l.vdim);
-        s.off_g = in_seg((left + "g").c_str(), vd);
-        add_vec(m, pl + "q.norm", &L.qn, l.dim);
-        add_vec(m, pl + "k.norm", &L.kn, l.dim);
+        if (!l.kv_from) {
+          s.off_k = in_seg((left + "k").c_str(), l.kv_heads * l.dim);
+          s.off_v = in_seg((left + "v").c_str(), l.kv_heads * l.vdim);
+        }
+        if (s.gated) {
+          s.off_g = in_seg((left + "g").c_str(), vd);
+          add_vec(m, pl + "q.norm", &L.qn, l.dim);
+          add_vec(m, pl + "k.norm", &L.kn, l.dim);
+        } else {
+          add_vec(m, pl + "o.b", &L.out_bias, W);
+        }
         L.splits = gattn_splits(s, d.max_seq_len, 1, m.f32, m.forced_splits);
         for (uint32_t t = 1; t <= kGattnShort; t++) {
           const size_t rows = (size_t)t * l.heads * gattn_splits(s, d.max_seq_len, t, m.f32, m.forced_splits);
@@ -394,8 +475,10 @@ static void layered_plan(LayeredModel& m) {
       L.gs.ldcat = L.as.ldcat = L.in.n;
       if (L.gattn()) {
         add_bias(m, pl + "q.b", &L.in_bias, L.gs.off_q, l.heads * l.dim, L.in.n);
-        add_bias(m, pl + "k.b", &L.in_bias, L.gs.off_k, l.kv_heads * l.dim, L.in.n);
-        add_bias(m, pl + "v.b", &L.in_bias, L.gs.off_v, l.kv_heads * l.vdim, L.in.n);
+        if (!l.kv_from) {
+          add_bias(m, pl + "k.b", &L.in_bias, L.gs.off_k, l.kv_heads * l.dim, L.in.n);
+          add_bias(m, pl + "v.b", &L.in_bias, L.gs.off_v, l.kv_heads * l.vdim, L.in.n);
+        }
       }
       // both sides' output projections side by side: one product
       L.gla_col = up(vd, 64);
@@ -432,7 +515,7 @@ static void layered_plan(LayeredModel& m) {
     }
     m.max_ao = std::max(m.max_ao, L.out.kp);
     if (L.moe()) {
-      add_sub(m, p, "2", &L.norm2);
+      add_sub(m, p, "2", &L.norm2, &L.post2, &L.ls2);
       whole(L.router, l.experts + l.identity, W);
       add_mat(m, p + "mlp.router", &L.router, 0, L.router.n, W);
       if (l.router_form == LGH_ROUTER_SOFTMAX_GROUPS) add_vec(m, p + "mlp.correction", &L.correction, L.router.n);
@@ -460,11 +543,16 @@ static void layered_plan(LayeredModel& m) {
       m.max_top = std::max(m.max_top, l.top);
       m.max_pair_act = std::max(m.max_pair_act, l.top * L.edown.kp);
     } else if (l.ff_kind) {
-      add_sub(m, p, "2", &L.norm2);
-      whole(L.gu, 2 * up(l.ff, 16), W);
-      L.gu.paired = true;
-      add_mat(m, p + "mlp.gate", &L.gu, 0, l.ff, W, 1);
-      add_mat(m, p + "mlp.up", &L.gu, 0, l.ff, W, 2);
+      add_sub(m, p, "2", &L.norm2, &L.post2, &L.ls2);
+      if (l.ff_kind == LGH_FF_RELU2) {
+        whole(L.gu, l.ff, W);
+        add_mat(m, p + "mlp.up", &L.gu, 0, l.ff, W);
+      } else {
+        whole(L.gu, 2 * up(l.ff, 16), W);
+        L.gu.paired = true;
+        add_mat(m, p + "mlp.gate", &L.gu, 0, l.ff, W, 1);
+        add_mat(m, p + "mlp.up", &L.gu, 0, l.ff, W, 2);
+      }
       whole(L.down, W, l.ff);
       add_mat(m, p + "mlp.down", &L.down, 0, W, l.ff);
       m.max_act = std::max(m.max_act, L.down.kp);
@@ -616,7 +704,13 @@ int layered_finalize(lgh_ctx* c) {
         if (!cs.empty()) L_TRY(c, LGH_OPERATION_FAILED, hipMemcpy(L.cs, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
       }
     }
-    if (L.latent()) {
+    if (L.d.kv_from) {                     // an earlier layer's cache rows
+      L.cache = m.layers[L.d.kv_from - 1].cache;
+      L.vcache = m.layers[L.d.kv_from - 1].vcache;
+    } else if (L.delta()) {
+      if ((rc = zeroed(c, (void**)&L.S, (size_t)L.des.heads * L.des.dk * L.des.lv * 4, &c->stats.kv_bytes))) return rc;
+      if ((rc = zeroed(c, (void**)&L.rhist, (size_t)L.des.taps * L.des.cols * 4, &c->stats.kv_bytes))) return rc;
+    } else if (L.latent()) {
       if ((rc = zeroed(c, &L.cache, (size_t)d.max_seq_len * L.ls.ldc * m.el(), &c->stats.kv_bytes))) return rc;
       max_rows = std::max(max_rows, L.ls.heads); max_rank = std::max(max_rank, L.ls.rank); max_ldc = std::max(max_ldc, L.ls.ldc);
     } else if (L.tied()) {
@@ -646,7 +740,7 @@ int layered_finalize(lgh_ctx* c) {
   struct { void** p; size_t n; } bufs[] = {
       {(void**)&m.x[0], (size_t)d.width * 4}, {(void**)&m.x[1], (size_t)d.width * 4}, {(void**)&m.y, (size_t)up(d.width, 16) * 4},
       {(void**)&m.cat, (size_t)m.max_cat * 4}, {(void**)&m.ao, (size_t)m.max_ao * 4}, {(void**)&m.act, (size_t)m.max_act * 4},
-      {(void**)&m.num, (size_t)m.max_num * 4}, {(void**)&m.qa, rows * max_ldc * m.el()},
+      {(void**)&m.num, (size_t)m.max_num * 4}, {(void**)&m.qa, rows * max_ldc * m.el()}, {(void**)&m.lq, (size_t)m.max_lq * 4},
       {(void**)&m.part_ml, std::max(rows * m.n_splits, m.max_tied_rows) * 2 * 4}, {(void**)&m.part_acc, std::max(rows * m.n_splits * max_rank, m.max_tied_acc) * 4},
       {(void**)&m.selw, (size_t)m.max_top * 4},
       {(void**)&m.tokens, (size_t)d.max_seq_len * 4}, {(void**)&m.h, m.dyt() || m.pre() ? (size_t)up(d.width, 16) * 4 : 0}, {(void**)&m.hist, m.hist_floats() * 4},
@@ -655,6 +749,11 @@ int layered_finalize(lgh_ctx* c) {
   };
   for (auto& b : bufs)
     if ((rc = zeroed(c, b.p, b.n, sb))) return rc;
+  if (m.ln2())                             // a sublayer's scale per channel goes into the weight of the norm in front of it
+    for (LayeredLayer& L : m.layers) {
+      L_TRY(c, LGH_OPERATION_FAILED, vec_mul_launch(L.post1, L.ls1, d.width, c->stream));
+      if (L.d.ff_kind) L_TRY(c, LGH_OPERATION_FAILED, vec_mul_launch(L.post2, L.ls2, d.width, c->stream));
+    }
   // where the residual stream ends up: every sublayer's update swaps the two vectors; channel by channel it stays in place
   c->hidden = m.dyt() ? m.x[0] : m.x[m.n_sub & 1];
   L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(c->stream));
@@ -668,10 +767,19 @@ static EmbedArgs embed_args(const LayeredModel& m) {
   return a;
 }
 
-static LatentBufs latent_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat) {
+// q: the queries where they are made from their latent
+static LatentBufs latent_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat, const float* q) {
   LatentBufs b{};
-  b.cat = cat; b.dkv_norm = L.dkv_norm; b.cs = L.cs; b.uk_t = L.uk_t; b.uv = L.uv.w; b.cache = L.cache; b.qa = m.qa;
+  b.cat = cat; b.q = L.d.q_rank ? q : cat + L.ls.off_q; b.dkv_norm = L.dkv_norm; b.cs = L.cs; b.uk_t = L.uk_t; b.uv = L.uv.w; b.cache = L.cache; b.qa = m.qa;
   b.part_ml = m.part_ml; b.part_acc = m.part_acc;
+  return b;
+}
+// shares of the visible keys: no more than a window has tiles
+static uint32_t latent_splits(const LayeredModel& m, const LayeredLayer& L) { return std::min(m.n_splits, L.ls.window / 32 + 2); }
+static DeltaBufs delta_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat, float* num) {
+  DeltaBufs b{};
+  b.cat = cat; b.conv = L.conv; b.a_log = L.a_log; b.dt = L.dt; b.norm = L.gnorm; b.S = L.S; b.hist = L.rhist; b.num = num;
+  b.q = m.bdq; b.k = m.bdk; b.v = m.bdv; b.u = m.bdu; b.w = m.bdw; b.p = m.bdp; b.wge = m.bdwge; b.cd = m.bdcd; b.Mcap = up(m.blk, 64);
   return b;
 }
 static MlstmBufs mlstm_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat, float* num) {
@@ -683,7 +791,7 @@ static MlstmBufs mlstm_bufs(const LayeredModel& m, const LayeredLayer& L, const 
 }
 static GattnBufs gattn_bufs(const LayeredModel& m, const LayeredLayer& L, const float* cat) {
   GattnBufs b{};
-  b.cat = cat; b.qn = L.qn; b.kn = L.kn; b.cs = L.cs; b.kc = L.cache; b.vc = L.vcache;
+  b.cat = cat; b.qn = L.qn; b.kn = L.kn; b.cs = L.cs; b.kc = L.cache; b.vc = L.vcache; b.shared = L.d.kv_from != 0;
   b.part_ml = m.part_ml; b.part_acc = m.part_acc;
   return b;
 }
@@ -739,11 +847,12 @@ static uint64_t mixer_bytes(const lgh_ctx* c, const LayeredLayer& L) {
   if (L.glru()) return L.gates.bytes() + (uint64_t)L.rs.width * (L.rs.taps * 2 + 7) * 4;
   if (L.gattn() || L.gla()) {
     uint64_t b = 0;
-    if (L.gattn()) b += (uint64_t)(c->pos + 1 - c->pos / L.gs.chunk * L.gs.chunk) * L.gs.kv_heads * (L.gs.dim + L.gs.vdim) * c->lm->el();
+    if (L.gattn()) b += std::min<uint64_t>(c->pos + 1 - c->pos / L.gs.chunk * L.gs.chunk, L.gs.window) * L.gs.kv_heads * (L.gs.dim + L.gs.vdim) * c->lm->el();
     if (L.gla()) b += (uint64_t)L.as.heads * L.as.dim * L.as.vdim * 8 + L.a2.bytes();
     return b;
   }
-  if (L.latent()) return (uint64_t)(c->pos + 1) * (L.ls.rank + L.ls.rot_dim) * c->lm->el();
+  if (L.delta()) return (uint64_t)L.des.heads * L.des.dim * L.des.vdim * 8 + (uint64_t)L.des.cols * (L.des.taps * 2 + 1) * 4;
+  if (L.latent()) return std::min<uint64_t>(c->pos + 1, L.ls.window) * (L.ls.rank + L.ls.rot_dim) * c->lm->el();
   return (uint64_t)L.ms.heads * L.ms.dim * (L.ms.vdim + 1) * 8;   // state read and written
 }
 
@@ -773,7 +882,17 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
   auto read = [&](LinMv& a, const float* pre, const float* nw2 = nullptr) -> int {
     a.x = m.dyt() ? m.h : m.x[cur];
     int pro = LP_COPY;
+    if (m.ln2()) {
+      a.nw2 = nw2 ? nw2 : pre; a.eps = (float)m.d.norm_eps; a.mult = (float)m.d.residual_mult;
+      if (pend) {
+        a.y = m.y; a.nw = pend; a.xout = m.x[cur ^ 1];
+        cur ^= 1;
+        pend = nullptr;
+      }
+      return LP_SANDWICH;
+    }
     if (m.pre()) {
+      a.nw_add = 1.0f;
       a.nw2 = nw2 ? nw2 : pre; a.eps = (float)m.d.norm_eps; a.mult = (float)m.d.residual_mult; a.in_scale = nw2 && m.d.logit_scale != 0.0 ? (float)m.d.logit_scale : 1.0f;
       if (pend) {
         a.y = m.y; a.xout = m.x[cur ^ 1];
@@ -790,44 +909,51 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
     }
     return pro;
   };
-  auto mv_x = [&](int cls, const LinW& W, float* out, const float* pre, const float* nw2 = nullptr, const float* bias = nullptr) {
+  auto mv_x = [&](int cls, const LinW& W, float* out, const float* pre, const float* nw2 = nullptr, const float* bias = nullptr, uint32_t act = 0, float cap = 0.0f) {
     LinMv a{};
-    a.bias = bias;
+    a.bias = bias; a.act = act; a.cap = cap;
     const int pro = read(a, pre, nw2);
     return mv(cls, W, out, a, pro);
   };
   for (LayeredLayer& L : m.layers) {
+    float *after1 = m.ln2() ? L.post1 : L.norm1, *after2 = m.ln2() ? L.post2 : L.norm2;   // the norm that the sublayer's output waits for
     if ((rc = mv_x(LGH_K_QKV, L.in, m.cat, L.norm1, nullptr, L.in_bias))) return rc;
     if (L.latent()) {
-      const LatentBufs b = latent_bufs(m, L, m.cat);
+      const LatentBufs b = latent_bufs(m, L, m.cat, m.lq);
+      const uint32_t splits = latent_splits(m, L);
+      if (L.d.q_rank) {
+        LinMv q{};
+        q.x = m.cat + L.ls.off_q; q.nw2 = L.dq_norm; q.eps = L.ls.eps; q.in_scale = 1.0f;
+        if ((rc = mv(LGH_K_QKV, L.uq, m.lq, q, LP_PRE))) return rc;
+      }
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, (uint64_t)L.ls.heads * L.ls.rank * L.ls.dim * 2, [&] { return latent_prep_launch(L.ls, b, pos, 0, 1, m.f32, st); }))) return rc;
-      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, mixer_bytes(c, L), [&] { return latent_attn_launch(L.ls, b, pos, 0, 1, m.n_splits, m.f32, st); }))) return rc;
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, mixer_bytes(c, L), [&] { return latent_attn_launch(L.ls, b, pos, 0, 1, splits, m.f32, st); }))) return rc;
       if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_LATENT, L.uv.bytes(), [&] {
-             return latent_out_launch(L.ls, b, pos, 0, 1, m.n_splits, m.ao, 0, true, st);
+             return latent_out_launch(L.ls, b, pos, 0, 1, splits, m.ao, 0, true, st);
            })))
         return rc;
       LinMv a{};
       a.x = m.ao;
-      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, after1))) return rc;
     } else if (L.tied()) {
       const TiedBufs b = tied_bufs(m, L, m.cat);
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_TIED, mixer_bytes(c, L), [&] { return tied_attn_launch(L.ts, b, pos, 0, 1, true, L.splits, m.f32, st); }))) return rc;
       if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_TIED, 0, [&] { return tied_merge_launch(L.ts, b, pos, 0, 1, L.splits, m.f32, m.ao, 0, true, st); }))) return rc;
       LinMv a{};
       a.x = m.ao;
-      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, after1))) return rc;
     } else if (L.glru()) {
       const GlruBufs b = glru_bufs(m, L, m.cat);
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GLRU, mixer_bytes(c, L), [&] { return glru_step_launch(L.rs, b, pos, m.ao, st); }))) return rc;
       LinMv a{};
       a.x = m.ao;
-      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, after1))) return rc;
     } else if (L.gattn() || L.gla()) {
       const GattnBufs b = gattn_bufs(m, L, m.cat);
       const GlaBufs g = gla_bufs(m, L, m.cat, m.num);
       const GlaShape* as = L.gla() ? &L.as : nullptr;
       if (L.gattn()) {
-        if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GATTN, mixer_bytes(c, L), [&] { return gattn_attn_launch(L.gs, b, as, &g, pos, 0, 1, true, L.splits, m.f32, st); }))) return rc;
+        if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_GATTN, mixer_bytes(c, L), [&] { return gattn_attn_launch(L.gs, b, as, &g, pos, 0, 1, !b.shared, L.splits, m.f32, st); }))) return rc;
         if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_GATTN, 0, [&] {
                return gattn_merge_launch(L.gs, b, as, &g, L.gla_col, pos, 0, 1, L.splits, m.f32, m.ao, 0, true, st);
              })))
@@ -837,14 +963,20 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
         if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_GLA, 0, [&] { return gla_out_launch(L.as, g, 1, m.ao, L.out.kp, true, st); }))) return rc;
       }
       LinMv a{};
-      a.x = m.ao;
-      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, L.norm1))) return rc;
+      a.x = m.ao; a.bias = L.out_bias;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_COPY, after1))) return rc;
+    } else if (L.delta()) {
+      const DeltaBufs b = delta_bufs(m, L, m.cat, m.num);
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_DELTA, mixer_bytes(c, L), [&] { return delta_step_launch(L.des, b, pos, 0, st); }))) return rc;
+      LinMv a{};
+      a.num = m.num; a.nw = L.gnorm; a.gate = m.cat + L.des.off_g; a.heads = L.des.heads; a.vdim = L.des.vdim; a.ldo = L.des.lv; a.eps = L.des.eps;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_READ, after1))) return rc;
     } else {
       const MlstmBufs b = mlstm_bufs(m, L, m.cat, m.num);
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_MLSTM, mixer_bytes(c, L), [&] { return mlstm_step_launch(L.ms, b, pos, st); }))) return rc;
       LinMv a{};
       a.num = m.num; a.nw = L.mnorm; a.gate = m.cat + L.ms.off_g; a.heads = L.ms.heads; a.vdim = L.ms.vdim; a.ldo = L.ms.ldo; a.eps = L.ms.eps;
-      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_MLSTM, L.norm1))) return rc;
+      if ((rc = mv_end(LGH_K_WO, L.out, a, LP_MLSTM, after1))) return rc;
     }
     if (L.moe()) {
       const RouteForm route = L.route();
@@ -865,13 +997,13 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
       o.experts = L.d.experts; o.selw = m.selw; o.id_x = route.identity ? m.h : nullptr;
       o.w2 = L.edown.w; o.top = L.d.top; o.sel = m.sel; o.stride = (uint64_t)L.edown_rows * L.edown.kp; o.kpe = L.edown.kp;
       if (m.dyt()) o.post = post_update(c, sub++);
-      else pend = L.norm2;
+      else pend = after2;
       if ((rc = run_k(c, LGH_K_DOWN, LGH_SYM_LINEAR, L.down.bytes() + L.edown.bytes() / L.d.experts * L.d.top, [&] { return lin_mv_launch(LP_COPY, o, st, LS_MOE_DOWN); }))) return rc;
     } else if (L.d.ff_kind) {
-      if ((rc = mv_x(LGH_K_GATEUP, L.gu, m.act, L.norm2))) return rc;
+      if ((rc = mv_x(LGH_K_GATEUP, L.gu, m.act, L.norm2, nullptr, nullptr, L.d.ff_kind == LGH_FF_RELU2 ? LA_RELU2 : LA_GELU))) return rc;
       LinMv a{};
       a.x = m.act;
-      if ((rc = mv_end(LGH_K_DOWN, L.down, a, LP_COPY, L.norm2))) return rc;
+      if ((rc = mv_end(LGH_K_DOWN, L.down, a, LP_COPY, after2))) return rc;
     }
   }
   if (mode == MODE_PREFILL && m.dyt()) return LGH_OK;
@@ -881,7 +1013,7 @@ int layered_enqueue_token(lgh_ctx* c, int mode) {
     return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
       return resid_norm_out_launch(m.x[cur], m.y, pend, (float)m.d.norm_eps, (float)m.d.residual_mult, m.d.width, m.x[cur ^ 1], st);
     });
-  if ((rc = mv_x(LGH_K_OUTPUT, m.head, c->logits, nullptr, m.final_norm))) return rc;
+  if ((rc = mv_x(LGH_K_OUTPUT, m.head, c->logits, nullptr, m.final_norm, nullptr, 0, (float)m.d.logit_cap))) return rc;
   if (mode == MODE_GREEDY)
     return run_k(c, LGH_K_ARGMAX, LGH_SYM_ARGMAX, (uint64_t)m.d.vocab_size * 4, [&] {
       return argmax_launch(c->logits, m.d.vocab_size, c->amax_v, c->amax_i, c->state, c->tok_log, st);
@@ -894,7 +1026,8 @@ uint64_t layered_step_bytes(const lgh_ctx* c) {
   uint64_t b = (uint64_t)m.d.width * (m.bigram ? 4 : 2) + m.head.bytes() + (uint64_t)m.d.vocab_size * 4 + m.d.width * 4;
   for (const LayeredLayer& L : m.layers) {
     b += L.in.bytes() + L.out.bytes() + mixer_bytes(c, L) + (uint64_t)m.d.width * 4;
-    if (L.latent()) b += L.uk.bytes() + L.uv.bytes();
+    if (L.latent()) b += L.uk.bytes() + L.uv.bytes() + L.uq.bytes();
+    if (m.ln2()) b += (uint64_t)m.d.width * (L.d.ff_kind ? 8 : 4);
     if (L.d.ff_kind) b += L.gu.bytes() + L.down.bytes() + (uint64_t)m.d.width * 4;
     if (L.moe()) b += L.router.bytes() + (L.egu.bytes() + L.edown.bytes()) / L.d.experts * L.d.top;
   }
@@ -918,7 +1051,10 @@ static int block_ensure(lgh_ctx* c) {
   struct { void** p; size_t n; } bufs[] = {
       {(void**)&m.bx, B * d.width * 4}, {&m.bxa, B * up(d.width, 64) * el}, {(void**)&m.by, B * up(d.width, 4) * 4},
       {(void**)&m.bcat, (B * m.max_cat + kMlstmRowSlack) * 4}, {&m.bao, B * m.max_ao * el}, {&m.bact, B * m.max_act * el},
-      {(void**)&m.bnum, B * m.max_num * 4}, {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * Bc * 8}, {(void**)&m.bmx, heads * Bc * 8},
+      {(void**)&m.bnum, Bc * m.max_num * 4}, {(void**)&m.blq, B * m.max_lq * 4}, {&m.blqa, B * m.max_qrank * el},
+      {(void**)&m.bdq, Bc * m.max_dqk * 4}, {(void**)&m.bdk, Bc * m.max_dqk * 4}, {(void**)&m.bdv, Bc * m.max_dv * 4}, {(void**)&m.bdu, Bc * m.max_dv * 4},
+      {(void**)&m.bdw, Bc * m.max_dw * 4}, {(void**)&m.bdp, Bc * m.max_dw * 4}, {(void**)&m.bdwge, Bc * m.max_dheads * 4}, {(void**)&m.bdcd, chunks * m.max_dheads * 4},
+      {(void**)&m.ba, chunks * heads * 4096 * 4}, {(void**)&m.bu, heads * Bc * 8}, {(void**)&m.bmx, heads * Bc * 8},
       {(void**)&m.bdec, heads * Bc * 4}, {(void**)&m.bwgt, heads * Bc * 4}, {(void**)&m.bcdec, heads * chunks * 4}, {(void**)&m.bnk, chunks * hdim * 4},
       {(void**)&m.brec, B * m.max_rec * 2 * 4}, {(void**)&m.brsum, (chunks * 2 + 1) * m.max_rec * 4},
       {(void**)&m.bqk, m.max_gla ? (Bc * m.max_gla * 2 + kMlstmRowSlack) * 4 : 0}, {(void**)&m.bgdec, m.max_gla ? (chunks * m.max_gla + kMlstmRowSlack) * 4 : 0},
@@ -938,9 +1074,9 @@ static int block_ensure(lgh_ctx* c) {
   return LGH_OK;
 }
 
-static int block_gemm(lgh_ctx* c, int cls, const LinW& W, int epi, const void* x, uint32_t ldx, void* out, uint32_t ldo, uint32_t M, const float* bias = nullptr) {
+static int block_gemm(lgh_ctx* c, int cls, const LinW& W, int epi, const void* x, uint32_t ldx, void* out, uint32_t ldo, uint32_t M, const float* bias = nullptr, float cap = 0.0f) {
   LinGemm g{};
-  g.bias = bias;
+  g.bias = bias; g.cap = cap;
   g.w = W.w; g.x = x; g.out = out; g.n = W.n; g.np = W.np(); g.kp = W.kp; g.ldx = ldx; g.ldo = ldo; g.M = M;
   return run_k(c, cls, LGH_SYM_LINEAR, W.bytes(), [&] { return lin_gemm_launch(epi, c->lm->f32, g, c->stream); });
 }
@@ -966,17 +1102,25 @@ static int block_latent(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) 
   hipStream_t st = c->stream;
   int rc;
   LatentFlash& f = m.fl;
-  if (M >= kExpandTokens && pos0 <= 64 * M && latent_flash_shape(L.ls, &f.dq, &f.dvp)) {
-    const uint32_t kv = pos0 + M, H = L.ls.heads;
+  if (L.d.q_rank) {
+    if ((rc = run_k(c, LGH_K_QKV, LGH_SYM_OTHER, 0, [&] {
+           return rms_cols_launch(m.bcat + L.ls.off_q, L.ls.ldcat, L.dq_norm, L.ls.eps, L.d.q_rank, M, m.blqa, L.uq.kp, m.f32, st);
+         })))
+      return rc;
+    if ((rc = block_gemm(c, LGH_K_QKV, L.uq, LE_F32, m.blqa, L.uq.kp, m.blq, L.ls.ldq, M))) return rc;
+  }
+  f.base = latent_key_start(L.ls, pos0) / 64 * 64;
+  if (M >= kExpandTokens && pos0 - f.base <= 64 * M && latent_flash_shape(L.ls, &f.dq, &f.dvp)) {
+    const uint32_t kv = pos0 - f.base + M, H = L.ls.heads;   // positions from the first visible tile on
     f.Mcap = m.blk;
     f.Tcap = up(kv, 1024);
     if ((rc = grow(c, &f.q, &m.fl_q_bytes, (size_t)H * f.Mcap * f.dq * m.el())) || (rc = grow(c, &f.k, &m.fl_k_bytes, (size_t)H * f.Tcap * f.dq * m.el())) ||
         (rc = grow(c, &f.vt, &m.fl_v_bytes, (size_t)H * f.dvp * f.Tcap * m.el())))
       return rc;
-    const LatentBufs b = latent_bufs(m, L, m.bcat);
+    const LatentBufs b = latent_bufs(m, L, m.bcat, m.blq);
     if ((rc = run_k(c, LGH_K_EXPAND, LGH_SYM_LATENT, 0, [&] { return latent_flash_prep_launch(L.ls, b, f, pos0, M, m.f32, st); }))) return rc;
     LinGemm g{};
-    g.x = L.cache; g.ldx = L.ls.ldc; g.M = kv;
+    g.x = (const uint8_t*)L.cache + (size_t)f.base * L.ls.ldc * m.el(); g.ldx = L.ls.ldc; g.M = kv;
     g.w = L.uk.w; g.n = L.uk.n; g.np = L.uk.np(); g.kp = L.uk.kp; g.out = f.k; g.ldo = f.dq; g.hd = L.ls.dim; g.tcap = f.Tcap;
     if ((rc = run_k(c, LGH_K_EXPAND, LGH_SYM_LINEAR, L.uk.bytes(), [&] { return lin_gemm_launch(LE_HEADS, m.f32, g, st); }))) return rc;
     g.w = L.uv.w; g.n = L.uv.n; g.np = L.uv.np(); g.kp = L.uv.kp; g.out = f.vt; g.ldo = (uint32_t)f.Tcap; g.hd = L.ls.vdim; g.hrows = f.dvp;
@@ -988,7 +1132,7 @@ static int block_latent(lgh_ctx* c, LayeredLayer& L, uint32_t pos0, uint32_t M) 
   for (uint32_t t = 0; t < M; t += step) {
     const uint32_t n = std::min(step, M - t), p = pos0 + t;
     const uint32_t splits = std::max(1u, std::min(m.n_splits, 512u / ((n * L.ls.heads + 15) / 16)));
-    const LatentBufs b = latent_bufs(m, L, m.bcat + (size_t)t * L.ls.ldcat);
+    const LatentBufs b = latent_bufs(m, L, m.bcat + (size_t)t * L.ls.ldcat, m.blq + (L.d.q_rank ? (size_t)t * L.ls.ldq : 0));
     if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, 0, [&] { return latent_prep_launch(L.ls, b, nullptr, p, n, m.f32, st); }))) return rc;
     if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_LATENT, 0, [&] { return latent_attn_launch(L.ls, b, nullptr, p, n, splits, m.f32, st); }))) return rc;
     if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_LATENT, 0, [&] {
@@ -1115,9 +1259,18 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
     return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, (uint64_t)M * d.width * 14, [&] { return pre_block_launch(b, m.f32, st); });
   };
   if (m.pre() && (rc = resid_pre(m.layers[0].norm1, true, nullptr))) return rc;
+  // LGH_RESIDUAL_SANDWICH_LN: the sublayer's output through the norm behind it (NULL: there is no output yet), then the next sublayer's norm
+  auto resid_ln = [&](const float* post, const float* nw) {
+    LnBlock b{};
+    b.x = m.bx; b.width = d.width; b.M = M; b.mult = mult; b.eps = eps; b.nw = nw; b.xa = m.bxa; b.ldx = ldx;
+    if (post) { b.y = m.by; b.ldy = ldy; b.pw = post; }
+    return run_k(c, LGH_K_MISC, LGH_SYM_OTHER, (uint64_t)M * d.width * 14, [&] { return ln_block_launch(b, m.f32, st); });
+  };
+  if (m.ln2() && (rc = resid_ln(nullptr, m.layers[0].norm1))) return rc;
   const float* next = nullptr;             // the norm in front of the sublayer that follows
   auto resid = [&](const float* nw, const LayeredLayer* moe = nullptr) -> int {
     if (m.pre()) return resid_pre(next, false, moe);
+    if (m.ln2()) return resid_ln(nw, next);
     if (m.dyt()) return resid_dyt(false, moe);
     if (moe && (rc = run_k(c, LGH_K_MISC, LGH_SYM_OTHER, 0, [&] {
                   return pair_sum_launch(m.by, ldy, m.bpair, ldy, m.bslot, moe->d.top, d.width, M, moe->d.shared_ff != 0, st);
@@ -1133,6 +1286,10 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
     if ((rc = block_gemm(c, LGH_K_QKV, L.in, LE_F32, m.bxa, ldx, m.bcat, L.in.n, M, L.in_bias))) return rc;
     if (L.latent()) {
       if ((rc = block_latent(c, L, pos0, M))) return rc;
+    } else if (L.delta()) {
+      const DeltaBufs b = delta_bufs(m, L, m.bcat, m.bnum);
+      if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_DELTA, 0, [&] { return delta_block_launch(L.des, b, pos0, M, st); }))) return rc;
+      if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_DELTA, 0, [&] { return delta_out_launch(L.des, b, pos0, M, m.bao, L.out.kp, m.f32, st); }))) return rc;
     } else if (L.tied()) {
       if ((rc = block_tied(c, L, pos0, M))) return rc;
     } else if (L.glru()) {
@@ -1145,17 +1302,17 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
       if ((rc = run_k(c, LGH_K_ATTN, LGH_SYM_MLSTM, 0, [&] { return mlstm_block_launch(L.ms, b, pos0, M, st); }))) return rc;
       if ((rc = run_k(c, LGH_K_ATTN_COMBINE, LGH_SYM_MLSTM, 0, [&] { return mlstm_out_launch(L.ms, b, M, m.bao, L.out.kp, m.f32, st); }))) return rc;
     }
-    if ((rc = block_gemm(c, LGH_K_WO, L.out, LE_F32, m.bao, L.out.kp, m.by, ldy, M))) return rc;
+    if ((rc = block_gemm(c, LGH_K_WO, L.out, LE_F32, m.bao, L.out.kp, m.by, ldy, M, L.out_bias))) return rc;
     next = L.d.ff_kind ? L.norm2 : after;
-    if ((rc = resid(L.norm1))) return rc;
+    if ((rc = resid(m.ln2() ? L.post1 : L.norm1))) return rc;
     next = after;
     if (L.moe()) {
       if ((rc = block_moe(c, L, ldx, ldy, M))) return rc;
       if ((rc = resid(L.norm2, &L))) return rc;
     } else if (L.d.ff_kind) {
-      if ((rc = block_gemm(c, LGH_K_GATEUP, L.gu, LE_GEGLU, m.bxa, ldx, m.bact, L.down.kp, M))) return rc;
+      if ((rc = block_gemm(c, LGH_K_GATEUP, L.gu, L.d.ff_kind == LGH_FF_RELU2 ? LE_RELU2 : LE_GEGLU, m.bxa, ldx, m.bact, L.down.kp, M))) return rc;
       if ((rc = block_gemm(c, LGH_K_DOWN, L.down, LE_F32, m.bact, L.down.kp, m.by, ldy, M))) return rc;
-      if ((rc = resid(L.norm2))) return rc;
+      if ((rc = resid(m.ln2() ? L.post2 : L.norm2))) return rc;
     }
     if (m.tap && m.tap_tokens == M)
       L_TRY(c, LGH_OPERATION_FAILED, hipMemcpyAsync(m.tap_buf + (size_t)li * M * d.width, xs, (size_t)M * d.width * 4, hipMemcpyDeviceToDevice, st));
@@ -1175,7 +1332,7 @@ static int block_pass(lgh_ctx* c, const uint32_t* tokens, uint32_t M, const uint
                           : final_norm_rows_launch(xs, m.brows, n, m.final_norm, eps, d.width, m.bla, ldx, m.f32, st);
          })))
       return rc;
-    if ((rc = block_gemm(c, LGH_K_OUTPUT, m.head, LE_F32, m.bla, ldx, m.blogits, ldl, n))) return rc;
+    if ((rc = block_gemm(c, LGH_K_OUTPUT, m.head, LE_F32, m.bla, ldx, m.blogits, ldl, n, nullptr, (float)d.logit_cap))) return rc;
     L_TRY(c, LGH_OPERATION_FAILED, hipMemcpy2DAsync(logits_out + (size_t)w * d.vocab_size, (size_t)d.vocab_size * 4, m.blogits, (size_t)ldl * 4,
                                                     (size_t)d.vocab_size * 4, n, hipMemcpyDeviceToHost, st));
     L_TRY(c, LGH_OPERATION_FAILED, hipStreamSynchronize(st));

@@ -183,6 +183,8 @@ template <uint32_t N> __device__ __forceinline__ float lanes_sum(float v) {
   return v;
 }
 
+template <class T> __device__ __forceinline__ T to_act(float v) { return (T)v; }
+
 // 16 bytes of a cache row as floats
 template <class T, int PER> __device__ __forceinline__ void unpack_row(const u32x4& w, float* f) {
   if constexpr (sizeof(T) == 2) {
@@ -223,6 +225,15 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
   return t;
 }
 
+// a wave: one head's output of a token, RMS-normed (w [vdim]) and silu-gated, times f -> o [vdim]
+template <class O> __device__ __forceinline__ void head_read_out(const float* num, const float* w, const float* gate, uint32_t vdim, float eps, float f, O* o) {
+  const uint32_t lane = threadIdx.x & 63;
+  float ss = 0.0f;
+  for (uint32_t j = lane; j < vdim; j += 64) ss = __builtin_fmaf(num[j], num[j], ss);
+  const float r = f / __builtin_sqrtf(wave_sum(ss) / (float)vdim + eps);
+  for (uint32_t j = lane; j < vdim; j += 64) o[j] = to_act<O>(num[j] * r * w[j] * silu_f(gate[j]));
+}
+
 // A matrix-core "unit": 16 bytes of the k axis per lane.  bf16: one v_mfma_f32_16x16x32_bf16 over 32 k (lane group g holds k = 8g ..
 // 8g + 7).  f32: four v_mfma_f32_16x16x4_f32 over 16 k, the j-th one over k = {j, 4 + j, 8 + j, 12 + j} (lane group g holds
 // k = 4g .. 4g + 3).  Both operands use the same assignment, so the sum runs over every k once.
@@ -245,8 +256,6 @@ template <> struct Frag<float> {
     return c;
   }
 };
-
-template <class T> __device__ __forceinline__ T to_act(float v) { return (T)v; }
 
 // value fragment from a tile of keys (rows of `ld` elements, 16-byte chunks stored at chunk ^ (row & 7)); k slots (lane group g, j):
 // bf16: keys 4g + j of the tile's first 16 rows (j < 4) and of its second 16 (j >= 4); f32: keys 4g + j of rows 16 n ..; column c0 + r16.

@@ -412,6 +412,116 @@ hipError_t pre_block_launch(const PreBlock& a, bool f32, hipStream_t st) {
   return f32 ? pre_block_go<float, 1>(a, st) : pre_block_go<__bf16, 1>(a, st);
 }
 
+// ------------------------------------------------------------------------------------------------
+// LGH_RESIDUAL_SANDWICH_LN over a block: a workgroup per token, the row in LDS (every thread its own channels)
+// ------------------------------------------------------------------------------------------------
+template <int V> __device__ __forceinline__ void ln_stats(const float* row, uint32_t width, float eps, float* red, float& mean, float& inv) {
+  float s = 0.0f, q = 0.0f;
+  for (uint32_t c = threadIdx.x * V; c < width; c += 256 * V) {
+    const VecF<V> v = load_vec<V>(row + c);
+#pragma unroll
+    for (int i = 0; i < V; i++) s += v.v[i];
+  }
+  mean = block_sum(s, red) / (float)width;
+  for (uint32_t c = threadIdx.x * V; c < width; c += 256 * V) {
+    const VecF<V> v = load_vec<V>(row + c);
+#pragma unroll
+    for (int i = 0; i < V; i++) { const float d = v.v[i] - mean; q = __builtin_fmaf(d, d, q); }
+  }
+  inv = 1.0f / __builtin_sqrtf(block_sum(q, red) / (float)width + eps);
+}
+
+template <class T, int V>
+__global__ void __launch_bounds__(256) ln_block_kernel(const LnBlock a) {
+  extern __shared__ __attribute__((aligned(16))) float row[];
+  __shared__ float red[16];
+  const uint32_t t = blockIdx.x;
+  float* x = a.x + (size_t)t * a.width;
+  float mean, inv;
+  if (a.y) {
+    const float* y = a.y + (size_t)t * a.ldy;
+    for (uint32_t c = threadIdx.x * V; c < a.width; c += 256 * V) store_vec<V>(row + c, load_vec<V>(y + c));
+    ln_stats<V>(row, a.width, a.eps, red, mean, inv);
+    for (uint32_t c = threadIdx.x * V; c < a.width; c += 256 * V) {
+      VecF<V> v = load_vec<V>(x + c);
+      const VecF<V> z = load_vec<V>(row + c), w = load_vec<V>(a.pw + c);
+#pragma unroll
+      for (int i = 0; i < V; i++) v.v[i] = __builtin_fmaf(a.mult, (z.v[i] - mean) * inv * w.v[i], v.v[i]);
+      store_vec<V>(row + c, v);
+      store_vec<V>(x + c, v);
+    }
+  } else {
+    for (uint32_t c = threadIdx.x * V; c < a.width; c += 256 * V) store_vec<V>(row + c, load_vec<V>(x + c));
+  }
+  if (!a.nw) return;
+  ln_stats<V>(row, a.width, a.eps, red, mean, inv);
+  T* xa = reinterpret_cast<T*>(a.xa) + (size_t)t * a.ldx;
+  for (uint32_t c = threadIdx.x * V; c < a.width; c += 256 * V) {
+    const VecF<V> v = load_vec<V>(row + c), w = load_vec<V>(a.nw + c);
+    T o[V];
+#pragma unroll
+    for (int i = 0; i < V; i++) o[i] = to_act<T>((v.v[i] - mean) * inv * w.v[i]);
+    __builtin_memcpy(__builtin_assume_aligned(xa + c, sizeof(o)), o, sizeof(o));
+  }
+}
+
+template <class T, int V>
+static hipError_t ln_block_go(const LnBlock& a, hipStream_t st) {
+  static bool opted[64] = {};
+  if (hipError_t e = lds_opt_in(reinterpret_cast<const void*>(&ln_block_kernel<T, V>), kNormMaxWidth * 4, opted); e != hipSuccess) return e;
+  hipLaunchKernelGGL((ln_block_kernel<T, V>), dim3(a.M), dim3(256), (size_t)a.width * 4, st, a);
+  return hipGetLastError();
+}
+
+hipError_t ln_block_launch(const LnBlock& a, bool f32, hipStream_t st) {
+  if (!a.x || a.M == 0 || a.width == 0 || a.width > kNormMaxWidth || (a.y && (!a.pw || a.ldy < a.width)) || (a.nw && (!a.xa || a.ldx < a.width)) || (!a.y && !a.nw)) return hipErrorInvalidValue;
+  const bool v4 = a.width % 4 == 0 && (!a.y || a.ldy % 4 == 0) && a.ldx % 4 == 0;
+  if (v4) return f32 ? ln_block_go<float, 4>(a, st) : ln_block_go<__bf16, 4>(a, st);
+  return f32 ? ln_block_go<float, 1>(a, st) : ln_block_go<__bf16, 1>(a, st);
+}
+
+// a wave per row
+template <class T>
+__global__ void __launch_bounds__(256) rms_cols_kernel(const float* __restrict__ x, uint32_t ld, const float* __restrict__ w, float eps, uint32_t n, uint32_t M, T* __restrict__ xa,
+                                                       uint32_t ldx) {
+  const uint32_t t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (t >= M) return;
+  const float* r = x + (size_t)t * ld;
+  constexpr uint32_t U = 8;   // values of a lane kept between the two passes
+  float v[U], q = 0.0f;
+#pragma unroll
+  for (uint32_t u = 0; u < U; u++) {
+    const uint32_t c = lane + u * 64;
+    v[u] = c < n ? r[c] : 0.0f;
+    q = __builtin_fmaf(v[u], v[u], q);
+  }
+  for (uint32_t c = lane + U * 64; c < n; c += 64) q = __builtin_fmaf(r[c], r[c], q);
+  const float inv = 1.0f / __builtin_sqrtf(wave_sum(q) / (float)n + eps);
+#pragma unroll
+  for (uint32_t u = 0; u < U; u++) {
+    const uint32_t c = lane + u * 64;
+    if (c < n) xa[(size_t)t * ldx + c] = to_act<T>(v[u] * inv * w[c]);
+  }
+  for (uint32_t c = lane + U * 64; c < n; c += 64) xa[(size_t)t * ldx + c] = to_act<T>(r[c] * inv * w[c]);
+}
+
+hipError_t rms_cols_launch(const float* x, uint32_t ld, const float* w, float eps, uint32_t n, uint32_t M, void* xa, uint32_t ldx, bool f32, hipStream_t st) {
+  if (!x || !w || !xa || n == 0 || M == 0 || ldx < n || ld < n) return hipErrorInvalidValue;
+  if (f32) hipLaunchKernelGGL(rms_cols_kernel<float>, dim3((M + 3) / 4), dim3(256), 0, st, x, ld, w, eps, n, M, (float*)xa, ldx);
+  else hipLaunchKernelGGL(rms_cols_kernel<__bf16>, dim3((M + 3) / 4), dim3(256), 0, st, x, ld, w, eps, n, M, (__bf16*)xa, ldx);
+  return hipGetLastError();
+}
+
+__global__ void __launch_bounds__(256) vec_mul_kernel(float* __restrict__ x, const float* __restrict__ y, uint32_t n) {
+  const uint32_t i = blockIdx.x * 256 + threadIdx.x;
+  if (i < n) x[i] *= y[i];
+}
+
+hipError_t vec_mul_launch(float* x, const float* y, uint32_t n, hipStream_t st) {
+  hipLaunchKernelGGL(vec_mul_kernel, dim3((n + 255) / 256), dim3(256), 0, st, x, y, n);
+  return hipGetLastError();
+}
+
 __global__ void __launch_bounds__(256) conv_store_kernel(const float* __restrict__ tails, float* __restrict__ hists, uint32_t back, uint32_t width, uint32_t last) {
   const uint32_t c = blockIdx.x * 256 + threadIdx.x, i = blockIdx.y, k = blockIdx.z;
   if (c < width) hists[((size_t)k * back + (last - i) % back) * width + c] = tails[((size_t)k * back + i) * width + c];

@@ -93,6 +93,21 @@ __device__ __forceinline__ void mv_acc(const MvW& o, f32x4 x0, f32x4 x1, float* 
     acc[r] = s;
   }
 }
+// what becomes of an unpaired row's sum
+__device__ __forceinline__ float mv_row_out(const LinMv& a, float v) {
+  if (a.act == LA_RELU2) { const float r = fmaxf(v, 0.0f); return r * r; }
+  return a.cap > 0.0f ? a.cap * tanh_f(v / a.cap) : v;
+}
+// sum over the workgroup, one barrier; red: 16 floats of LDS that nothing else uses
+__device__ __forceinline__ float mv_block_sum(float v, float* red) {
+  v = wave_sum(v);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  f32x4 t = *reinterpret_cast<const f32x4*>(red);
+#pragma unroll
+  for (int i = 4; i < 16; i += 4) t += *reinterpret_cast<const f32x4*>(red + i);
+  return (t.x + t.y) + (t.z + t.w);
+}
 __device__ __forceinline__ float mv_glu(const LinMv& a, float gate, float up) {
   if (a.act == LA_CLAMPED) return clamped_glu_f(gate, up, a.limit);
   return (a.act == LA_SILU ? silu_f(gate) : gelu_tanh_f(gate)) * up;
@@ -103,7 +118,7 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
   constexpr bool MOE = SRC == LS_EXPERTS || SRC == LS_MOE_DOWN;
   extern __shared__ __attribute__((aligned(16))) float xs[];   // [kp]
   __shared__ float red[2][16][kMvR];
-  __shared__ float bred[16];
+  __shared__ __attribute__((aligned(16))) float bred[PRO == LP_SANDWICH ? 64 : 16];
   __shared__ __attribute__((aligned(16))) float zs[SRC == LS_EXPERTS ? kMaxExperts : 4];
   __shared__ __attribute__((aligned(16))) float zc[SRC == LS_EXPERTS ? 2 * kMaxRouted : 4];   // choice scores, groups
   __shared__ float id_w;
@@ -160,10 +175,67 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
       for (uint32_t u = 0; u < U; u++) {
         const uint32_t i = i0 + u * kMvThreads;
         if (i >= a.k) break;
-        const float h = xs[i] * inv * (1.0f + (i0 == tid ? nw[u] : a.nw2[i]));
+        const float h = xs[i] * inv * (a.nw_add + (i0 == tid ? nw[u] : a.nw2[i]));
         xs[i] = h;
         if (a.hout && blockIdx.x == 0) a.hout[i] = h;
       }
+  } else if (PRO == LP_SANDWICH) {
+    constexpr uint32_t U = 4;   // channels a thread has in flight, with everything they need
+    float v[U], y[U], w1[U], w2[U];
+#pragma unroll
+    for (uint32_t u = 0; u < U; u++) {
+      const uint32_t i = tid + u * kMvThreads, ic = i < a.k ? i : a.k - 1;
+      v[u] = a.x[ic];
+      w2[u] = a.nw2[ic];
+      if (a.y) { y[u] = a.y[ic]; w1[u] = a.nw[ic]; }
+    }
+    const float n = 1.0f / (float)a.k;
+    auto each = [&](auto f) {   // (thread, channel, its place among the first)
+      for (uint32_t i0 = tid; i0 < a.k; i0 += U * kMvThreads)
+#pragma unroll
+        for (uint32_t u = 0; u < U; u++)
+          if (i0 + u * kMvThreads < a.k) f(i0 + u * kMvThreads, u, i0 == tid);
+    };
+    if (a.y) {
+      float s = 0.0f, q = 0.0f;
+      each([&](uint32_t i, uint32_t u, bool first) { const float z = first ? y[u] : a.y[i]; xs[i] = z; s += z; });
+      const float mean = mv_block_sum(s, bred) * n;
+      each([&](uint32_t i, uint32_t, bool) { const float d = xs[i] - mean; q = __builtin_fmaf(d, d, q); });
+      const float inv = 1.0f / __builtin_sqrtf(mv_block_sum(q, bred + 16) * n + a.eps);
+      each([&](uint32_t i, uint32_t u, bool first) {
+        const float z = __builtin_fmaf(a.mult, (xs[i] - mean) * inv * (first ? w1[u] : a.nw[i]), first ? v[u] : a.x[i]);
+        xs[i] = z;
+        if (blockIdx.x == 0) a.xout[i] = z;
+      });
+    } else {
+      each([&](uint32_t i, uint32_t u, bool first) { xs[i] = first ? v[u] : a.x[i]; });
+    }
+    float s = 0.0f, q = 0.0f;
+    each([&](uint32_t i, uint32_t, bool) { s += xs[i]; });
+    const float mean = mv_block_sum(s, bred + 32) * n;
+    each([&](uint32_t i, uint32_t, bool) { const float d = xs[i] - mean; q = __builtin_fmaf(d, d, q); });
+    const float inv = 1.0f / __builtin_sqrtf(mv_block_sum(q, bred + 48) * n + a.eps);
+    each([&](uint32_t i, uint32_t u, bool first) { xs[i] = (xs[i] - mean) * inv * (first ? w2[u] : a.nw2[i]); });
+  } else if (PRO == LP_READ) {
+    for (uint32_t h = wave; h < a.heads; h += 16) {
+      const float* num = a.num + (size_t)h * a.ldo;
+      const float* gt = a.gate + h * a.vdim;
+      float v[4], w[4], z[4], ss = 0.0f;
+#pragma unroll
+      for (int j = 0; j < 4; j++) {   // everything a lane needs of the first 256 values requested at once
+        const uint32_t e = lane + j * 64, ec = e < a.vdim ? e : 0;
+        v[j] = num[ec]; w[j] = a.nw[ec]; z[j] = gt[ec];
+        ss = __builtin_fmaf(e < a.vdim ? v[j] : 0.0f, v[j], ss);
+      }
+      for (uint32_t e = lane + 256; e < a.vdim; e += 64) ss = __builtin_fmaf(num[e], num[e], ss);
+      const float r = 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        const uint32_t e = lane + j * 64;
+        if (e < a.vdim) xs[h * a.vdim + e] = v[j] * r * w[j] * silu_f(z[j]);
+      }
+      for (uint32_t e = lane + 256; e < a.vdim; e += 64) xs[h * a.vdim + e] = num[e] * r * a.nw[e] * silu_f(gt[e]);
+    }
   } else if (PRO == LP_RESID || PRO == LP_HEAD) {
     for (uint32_t i = tid; i < a.k; i += kMvThreads) xs[i] = a.y[i];
     ln_lds(xs, a.k, a.nw, a.eps, bred);
@@ -291,7 +363,7 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
             float v = acc[r];
             if (a.bias) v += a.bias[n];
             if (SRC == LS_MOE_DOWN && a.id_x) v = __builtin_fmaf(id_w, a.id_x[n], v);
-            a.out[n] = v;
+            a.out[n] = SRC == LS_PLAIN ? mv_row_out(a, v) : v;
           }
       } else {
 #pragma unroll
@@ -334,7 +406,7 @@ bool route_ok(const RouteForm& f, uint32_t outputs, uint32_t top) {
 }
 
 hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st, int src) {
-  if (a.bias && (a.paired || a.post.xout)) return hipErrorInvalidValue;
+  if ((a.bias && (a.paired || a.post.xout)) || ((a.act == LA_RELU2 || a.cap > 0.0f) && (a.paired || a.post.xout || src != LS_PLAIN))) return hipErrorInvalidValue;
   if ((a.n && src != LS_EXPERTS && !a.w && !(src == LS_MOE_DOWN && a.kps == 0)) || (a.n && !a.out && !a.post.xout) || (a.n == 0 && src != LS_TWO) || a.kp % 64 ||
       a.kp > kLinMvMaxK || a.k > a.kp || (a.paired && a.n % 32))
     return hipErrorInvalidValue;
@@ -356,6 +428,9 @@ hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st, int src) {
     case LP_RESID: return a.x && a.y && a.nw && a.xout ? lin_mv_go<LP_RESID>(a, src, st) : hipErrorInvalidValue;
     case LP_HEAD: return a.x && a.y && a.nw && a.nw2 && a.xout && src == LS_PLAIN && !a.post.xout ? lin_mv_run<LP_HEAD, LS_PLAIN, false>(a, st) : hipErrorInvalidValue;
     case LP_PRE: return a.x && a.nw2 && (!a.y || a.xout) ? lin_mv_go<LP_PRE>(a, src, st) : hipErrorInvalidValue;
+    case LP_SANDWICH: return a.x && a.nw2 && (!a.y || (a.nw && a.xout)) && src == LS_PLAIN && !a.post.xout ? lin_mv_run<LP_SANDWICH, LS_PLAIN, false>(a, st) : hipErrorInvalidValue;
+    case LP_READ:
+      return a.num && a.nw && a.gate && a.heads * a.vdim == a.k && src == LS_PLAIN && !a.post.xout ? lin_mv_run<LP_READ, LS_PLAIN, false>(a, st) : hipErrorInvalidValue;
     case LP_MLSTM:
       return a.num && a.nw && a.gate && a.heads * a.vdim == a.k && src == LS_PLAIN ? lin_mv_post<LP_MLSTM, LS_PLAIN>(a, st) : hipErrorInvalidValue;
   }
@@ -500,10 +575,23 @@ __global__ void __launch_bounds__(256) lin_gemm_kernel(const LinGemm a, uint32_t
 #pragma unroll
             for (int e = 0; e < 4; e++) acc[i][j][e] += a.bias[nb + e < a.n ? nb + e : a.n - 1];
           }
+          if (a.cap > 0.0f) {
+#pragma unroll
+            for (int e = 0; e < 4; e++) acc[i][j][e] = a.cap * tanh_f(acc[i][j][e] / a.cap);
+          }
           if (nb + 4 <= a.n && (a.ldo & 3) == 0) *reinterpret_cast<f32x4*>(o) = acc[i][j];
           else
             for (int e = 0; e < 4; e++)
               if (nb + e < a.n) o[e] = acc[i][j][e];
+        } else if constexpr (EPI == LE_RELU2) {
+          T* o = reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + nb;
+          T r[4];
+#pragma unroll
+          for (int e = 0; e < 4; e++) { const float v = fmaxf(acc[i][j][e], 0.0f); r[e] = to_act<T>(v * v); }
+          if (nb + 4 <= a.n) __builtin_memcpy(__builtin_assume_aligned(o, sizeof(r)), r, sizeof(r));   // (rows are multiples of 64)
+          else
+            for (int e = 0; e < 4; e++)
+              if (nb + e < a.n) o[e] = r[e];
         } else if constexpr (EPI == LE_ACT) {
           T* o = reinterpret_cast<T*>(a.out) + (size_t)m * a.ldo + nb;
 #pragma unroll
@@ -567,6 +655,7 @@ static hipError_t lin_gemm_group(const LinGemm& a, hipStream_t st) {
 hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st) {
   const uint32_t el = f32 ? 4 : 2;
   if (!a.w || !a.x || !a.out || a.n == 0 || a.M == 0 || a.kp % 64 || a.ldx < a.kp || (a.ldx * el) % 16 || a.np % 16 || a.n > a.np) return hipErrorInvalidValue;
+  if ((epi == LE_RELU2 && a.ldo % 64) || (a.cap > 0.0f && (epi != LE_F32 || a.grp.tiles))) return hipErrorInvalidValue;
   if ((epi == LE_GEGLU || epi == LE_SWIGLU || epi == LE_CLAMPED) && a.n % 32) return hipErrorInvalidValue;
   if (a.grp.tiles) {
     if (!a.grp.seg || !a.grp.tile_e || !a.grp.tile_row || ((epi == LE_SWIGLU || epi == LE_CLAMPED) && !a.grp.scale)) return hipErrorInvalidValue;
@@ -585,6 +674,7 @@ hipError_t lin_gemm_launch(int epi, bool f32, const LinGemm& a, hipStream_t st) 
     LGH_GEMM_CASE(LE_HEADS)
     LGH_GEMM_CASE(LE_HEADS_T)
     LGH_GEMM_CASE(LE_SWIGLU)
+    LGH_GEMM_CASE(LE_RELU2)
   }
 #undef LGH_GEMM_CASE
   return hipErrorInvalidValue;

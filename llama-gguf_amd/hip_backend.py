@@ -42,14 +42,14 @@ ABI_SYMBOLS = (
 
 K_NAMES = ("embed", "qkv", "attn", "attn_combine", "wo", "gate_up", "down", "router", "output", "argmax", "misc", "token", "expand", "experts")
 K_COUNT = 16
-SYM_COUNT = 28
+SYM_COUNT = 29
 # kernel symbols as rocprofv3 prints them (LGH_SYM_* order)
 SYM_NAMES = ("lgh::mv_kernel<1u, 1024>", "lgh::mv_kernel<8u, 1024>", "lgh::mv_kernel<16u, 1024>",
              "lgh::mv_kernel<2u, 768>", "lgh::mv_kernel<4u, 512>", "lgh::mv_kernel<5u, 512>", "lgh::mv_kernel<6u, 512>",
              "lgh::mv_kernel<31u, 512>", "lgh::f32_matvec_kernel", "lgh::attn_partial_kernel", "lgh::attn_combine_kernel",
              "lgh::embed_kernel", "lgh::argmax_stage1+2", "lgh::moe_router_kernel", "other", "lgh::mvq_kernel<1u>", "lgh::mvq_kernel<2u>", "lgh::mvq_kernel<3u>", "lgh::mvq_kernel<4u>",
              "lgh::mvq_kernel<8u>", "unused", "lgh::lin_mv / lin_gemm", "lgh::latent_*", "lgh::mlstm_*", "lgh::tied_*", "lgh::gattn_*", "lgh::gla_*",
-             "lgh::glru_*")
+             "lgh::glru_*", "lgh::delta_*")
 FLAG_NO_GRAPH = 1
 FLAG_EXACT_PREFILL = 4   # forward_batch feeds tokens one by one (f32 throughout) instead of the batched f16 GEMM path
 KV_F32, KV_INT8, KV_FP8_E4M3, KV_FP8_E5M2 = 0, 1, 2, 3   # lgh_model_desc.kv_cache_type: f32, or QuantizedKVCache's formats (kv_quantized.rs; no CLI flag reaches them)
@@ -85,7 +85,8 @@ class LayerDesc(C.Structure):
     """lgh_layer_desc: one layer of a model described layer by layer."""
     _fields_ = ([(n, C.c_uint32) for n in ("struct_size", "mixer", "heads", "dim", "vdim", "kv_rank", "rot_dim", "rot_dims", "ff_kind", "ff",
                                          "kv_heads", "window", "keep_first", "experts", "top", "shared_ff", "router_form", "expert_form", "groups",
-                                         "keep_groups", "identity", "chunk", "taps", "gla_heads", "gla_dim", "gla_vdim", "gla_rank")]
+                                         "keep_groups", "identity", "chunk", "taps", "gla_heads", "gla_dim", "gla_vdim", "gla_rank", "q_rank", "rot_form",
+                                         "gate_form", "sink_one", "kv_from")]
                 + [(n, C.c_double) for n in ("scale", "rot_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow", "gate_cap", "score_cap",
                                             "expert_limit", "gla_tau", "left_scale", "right_scale")])
 
@@ -95,12 +96,15 @@ class LayeredDesc(C.Structure):
     _fields_ = ([(n, C.c_uint32) for n in ("struct_size", "width", "vocab_size", "num_layers", "max_seq_len", "compute")]
                 + [("device_id", C.c_int32), ("flags", C.c_uint32), ("bigram_buckets", C.c_uint32), ("bigram_mul_prev", C.c_uint64),
                    ("bigram_mul_cur", C.c_uint64), ("norm_eps", C.c_double), ("residual_mult", C.c_double), ("residual", C.c_uint32), ("conv_taps", C.c_uint32),
-                   ("tied_head", C.c_uint32), ("reserved", C.c_uint32), ("logit_scale", C.c_double)])
+                   ("tied_head", C.c_uint32), ("reserved", C.c_uint32), ("logit_scale", C.c_double), ("logit_cap", C.c_double)])
 
 
 MIXER_LATENT_ATTENTION, MIXER_MLSTM, MIXER_TIED_ATTENTION, MIXER_GATED_ATTENTION, MIXER_GLA, MIXER_PARALLEL, MIXER_GLRU = 1, 2, 3, 4, 5, 6, 7   # LGH_MIXER_*
-FF_NONE, FF_GEGLU, FF_MOE = 0, 1, 2             # LGH_FF_*
-RESIDUAL_POST_LN, RESIDUAL_SANDWICH_DYT, RESIDUAL_PRE_RMS = 0, 1, 2     # LGH_RESIDUAL_*
+MIXER_GROUPED_ATTENTION, MIXER_DELTA = 8, 9
+FF_NONE, FF_GEGLU, FF_MOE, FF_RELU2 = 0, 1, 2, 3   # LGH_FF_*
+RESIDUAL_POST_LN, RESIDUAL_SANDWICH_DYT, RESIDUAL_PRE_RMS, RESIDUAL_SANDWICH_LN = 0, 1, 2, 3     # LGH_RESIDUAL_*
+ROT_PAIRS, ROT_HALVES = 0, 1                    # LGH_ROT_*
+GATE_HEADS, GATE_VALUES = 0, 1                  # LGH_GATE_*
 ROUTER_SIGMOID, ROUTER_SOFTMAX_GROUPS = 0, 1    # LGH_ROUTER_*
 EXPERT_SWIGLU, EXPERT_CLAMPED = 0, 1            # LGH_EXPERT_*
 COMPUTE_BF16, COMPUTE_F32 = 0, 1                # LGH_COMPUTE_*

@@ -35,18 +35,75 @@ def _sizes(layer: hb.LayerDesc, mixer: dict, where: str, **fields) -> None:
         setattr(layer, name, int(_need(mixer, key, where)))
 
 
-def _latent_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
-    layer.mixer = hb.MIXER_LATENT_ATTENTION
-    _sizes(layer, mx, where, heads="heads", dim="dim", vdim="vdim", kv_rank="kv_rank", rot_dim="rot_dim")
-    layer.scale = float(_need(mx, "scale", where))
+def _rotation(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    """Leading values of a head (of its rotated part) that are rotated, with the frequencies' scaling; without an entry nothing is."""
     rot = mx.get("rot")
     if not rot:
-        return                                     # nothing is rotated
+        return
     layer.rot_dims, layer.rot_base = int(_need(rot, "dims", where)), float(_need(rot, "base", where))
     sc = rot.get("scaling")
     if sc:
         for f in ("factor", "original", "fast", "slow"):
             setattr(layer, "yarn_" + f, float(_need(sc, f, where)))
+        if layer.yarn_factor <= 0.0:
+            raise ConfigError(f"{where}: a scaling of {layer.yarn_factor}")
+
+
+def _rotated_of(layer: hb.LayerDesc, size: int, where: str) -> None:
+    if layer.rot_dims % 2 or layer.rot_dims > size:
+        raise ConfigError(f"{where}: {layer.rot_dims} rotated values of {size}")
+
+
+def _window(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    """The last positions that a position sees; without an entry all of them."""
+    mask = mx.get("mask")
+    if mask:
+        layer.window = int(_need(mask, "size", where))
+        if layer.window < 1:
+            raise ConfigError(f"{where}: a window of {layer.window} positions")
+
+
+def _head_groups(layer: hb.LayerDesc, where: str) -> None:
+    if layer.kv_heads < 1 or layer.heads % layer.kv_heads:
+        raise ConfigError(f"{where}: {layer.heads} heads do not divide into {layer.kv_heads} key heads")
+
+
+def _latent_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_LATENT_ATTENTION
+    _sizes(layer, mx, where, heads="heads", dim="dim", vdim="vdim", kv_rank="kv_rank", rot_dim="rot_dim")
+    layer.scale = float(_need(mx, "scale", where))
+    _rotation(layer, mx, where)
+
+
+def _windowed_latent_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    """Queries through a latent of their own, halves rotated, a window, every value gated."""
+    _latent_attention(layer, mx, where)
+    _sizes(layer, mx, where, q_rank="q_rank")
+    if layer.q_rank < 1:
+        raise ConfigError(f"{where}: a query latent of {layer.q_rank}")
+    _rotated_of(layer, layer.rot_dim, where)
+    layer.rot_form, layer.gate_form = hb.ROT_HALVES, hb.GATE_VALUES
+    _window(layer, mx, where)
+
+
+def _grouped_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_GROUPED_ATTENTION
+    _sizes(layer, mx, where, heads="heads", kv_heads="kv_heads", dim="dim", vdim="vdim")
+    _head_groups(layer, where)
+    layer.scale, layer.sink_one = float(_need(mx, "scale", where)), 1
+    _rotation(layer, mx, where)
+    _rotated_of(layer, layer.dim, where)
+    _window(layer, mx, where)
+    if mx.get("kv_from") is not None:
+        layer.kv_from = int(mx["kv_from"]) + 1
+
+
+def _delta(layer: hb.LayerDesc, mx: dict, where: str) -> None:
+    layer.mixer = hb.MIXER_DELTA
+    _sizes(layer, mx, where, heads="heads", kv_heads="kv_heads", dim="dim", vdim="vdim", taps="conv")
+    _head_groups(layer, where)
+    if layer.taps < 1:
+        raise ConfigError(f"{where}: a convolution of {layer.taps} taps")
 
 
 def _mlstm(layer: hb.LayerDesc, mx: dict, where: str) -> None:
@@ -61,32 +118,21 @@ def _tied_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
     layer.vdim = int(mx.get("vdim") or layer.dim)
     if layer.vdim != layer.dim:
         raise ConfigError(f"{where}: values are keys, 'vdim' {layer.vdim} differs from 'dim' {layer.dim}")
-    if not layer.kv_heads or layer.heads % layer.kv_heads:
-        raise ConfigError(f"{where}: {layer.heads} heads do not divide into {layer.kv_heads} key heads")
+    _head_groups(layer, where)
     layer.scale = float(_need(mx, "scale", where))
     layer.score_cap = float(mx.get("softcap") or 0.0)
-    mask = mx.get("mask")
-    if mask:
-        layer.window, layer.keep_first = int(_need(mask, "size", where)), int(mask.get("keep_first") or 0)
-        if layer.window < 1:
-            raise ConfigError(f"{where}: a window of {layer.window} positions")
-
-
-def _rotation(layer: hb.LayerDesc, mx: dict, where: str) -> None:
-    rot = mx.get("rot")
-    if rot:
-        layer.rot_dims, layer.rot_base = int(_need(rot, "dims", where)), float(_need(rot, "base", where))
-        if layer.rot_dims % 2 or layer.rot_dims > layer.dim:
-            raise ConfigError(f"{where}: {layer.rot_dims} rotated values of {layer.dim}")
+    _window(layer, mx, where)
+    if mx.get("mask"):
+        layer.keep_first = int(mx["mask"].get("keep_first") or 0)
 
 
 def _gated_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
     layer.mixer = hb.MIXER_GATED_ATTENTION
     _sizes(layer, mx, where, heads="heads", kv_heads="kv_heads", dim="dim", vdim="vdim")
-    if not layer.kv_heads or layer.heads % layer.kv_heads:
-        raise ConfigError(f"{where}: {layer.heads} heads do not divide into {layer.kv_heads} key heads")
+    _head_groups(layer, where)
     layer.scale = float(_need(mx, "scale", where))
     _rotation(layer, mx, where)
+    _rotated_of(layer, layer.dim, where)
     mask = mx.get("mask")
     if mask:
         layer.chunk = int(_need(mask, "size", where))
@@ -119,6 +165,10 @@ def _dense(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
     layer.ff_kind, layer.ff = hb.FF_GEGLU, int(_need(mlp, "ff", where))
 
 
+def _squared_relu(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
+    layer.ff_kind, layer.ff = hb.FF_RELU2, int(_need(mlp, "ff", where))
+
+
 def _moe(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
     layer.ff_kind, layer.ff = hb.FF_MOE, int(_need(_need(mlp, "expert", where), "ff", where))
     router = _need(mlp, "router", where)
@@ -142,8 +192,9 @@ def _grouped_moe(layer: hb.LayerDesc, mlp: dict, where: str) -> None:
 
 
 MIXERS = {"latent_attention": _latent_attention, "mlstm": _mlstm, "attention": _tied_attention, "gated_attention": _gated_attention, "gla": _gla,
-          "parallel": _parallel, "rglru": _rglru}
-FEED_FORWARDS = {"dense": _dense, "moe": _moe, "grouped_moe": _grouped_moe}
+          "parallel": _parallel, "rglru": _rglru, "grouped_attention": _grouped_attention, "windowed_latent_attention": _windowed_latent_attention,
+          "delta": _delta}
+FEED_FORWARDS = {"dense": _dense, "moe": _moe, "grouped_moe": _grouped_moe, "squared_relu": _squared_relu}
 
 
 @dataclass
@@ -159,6 +210,7 @@ class LayeredConfig:
     conv_taps: int = 0
     tied_head: bool = False                            # the output projection is the embedding table
     logit_scale: float = 1.0
+    logit_cap: float = 0.0                             # logits = cap * tanh(logits / cap); 0: none
 
     @property
     def num_layers(self) -> int:
@@ -170,7 +222,7 @@ class LayeredConfig:
         d.width, d.vocab_size, d.num_layers = self.hidden_size, self.vocab_size, self.num_layers
         d.norm_eps, d.residual_mult = self.norm_eps, self.residual_mult
         d.residual, d.conv_taps = self.residual, self.conv_taps
-        d.tied_head, d.logit_scale = int(self.tied_head), self.logit_scale
+        d.tied_head, d.logit_scale, d.logit_cap = int(self.tied_head), self.logit_scale, self.logit_cap
         if self.bigram:
             d.bigram_buckets, d.bigram_mul_prev, d.bigram_mul_cur = self.bigram
         return d
@@ -189,6 +241,9 @@ class LayeredConfig:
         yield from self._norm_shapes(f"{p}norm{which}")
         if self.residual == hb.RESIDUAL_SANDWICH_DYT:
             yield from self._norm_shapes(f"{p}norm{which}b")
+        if self.residual == hb.RESIDUAL_SANDWICH_LN:
+            yield f"{p}norm{which}b", (self.hidden_size,)
+            yield f"{p}ls{which}", (self.hidden_size,)
         if self.conv_taps:
             yield f"{p}canon{which}", (self.hidden_size, self.conv_taps)
 
@@ -236,6 +291,42 @@ class LayeredConfig:
         yield p + "lam", (n,)
         yield p + "o", (W, n)
 
+    def _latent_shapes(self, p: str, l) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        W, rows, vd = self.hidden_size, l.heads * (l.dim + l.rot_dim), l.heads * l.vdim
+        if l.q_rank:
+            yield p + "dq", (l.q_rank, W)
+            yield p + "dq.norm", (l.q_rank,)
+            yield p + "uq", (rows, l.q_rank)
+        else:
+            yield p + "q", (rows, W)
+        yield p + "dkv", (l.kv_rank + l.rot_dim, W)
+        yield p + "dkv.norm", (l.kv_rank,)
+        yield p + "uk", (l.heads * l.dim, l.kv_rank)
+        yield p + "uv", (vd, l.kv_rank)
+        yield p + "g", (vd if l.gate_form == hb.GATE_VALUES else l.heads, W)
+        yield p + "o", (W, vd)
+
+    def _grouped_shapes(self, p: str, l) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        W = self.hidden_size
+        for n, rows in (("q", l.heads * l.dim), ("k", l.kv_heads * l.dim), ("v", l.kv_heads * l.vdim)):
+            if n == "q" or not l.kv_from:
+                yield p + n, (rows, W)
+                yield p + n + ".b", (rows,)
+        yield p + "o", (W, l.heads * l.vdim)
+        yield p + "o.b", (W,)
+
+    def _delta_shapes(self, p: str, l) -> Iterator[Tuple[str, Tuple[int, ...]]]:
+        W, vd = self.hidden_size, l.heads * l.vdim
+        for n, rows in (("q", l.kv_heads * l.dim), ("k", l.kv_heads * l.dim), ("v", vd)):
+            yield p + n, (rows, W)
+            yield p + n + ".conv", (rows, l.taps)
+        for n, rows in (("b", l.heads), ("a", l.heads), ("g", vd)):
+            yield p + n, (rows, W)
+        yield p + "A_log", (l.heads,)
+        yield p + "dt_bias", (l.heads,)
+        yield p + "norm", (l.vdim,)
+        yield p + "o", (W, vd)
+
     def tensor_shapes(self) -> Iterator[Tuple[str, Tuple[int, ...]]]:
         """(name, shape) of every tensor the model needs, [out, in]."""
         W = self.hidden_size
@@ -247,12 +338,11 @@ class LayeredConfig:
             p, vd = f"l{i}.", l.heads * l.vdim
             yield from self._sublayer_shapes(p, 1)
             if l.mixer == hb.MIXER_LATENT_ATTENTION:
-                yield p + "mix.q", (l.heads * (l.dim + l.rot_dim), W)
-                yield p + "mix.dkv", (l.kv_rank + l.rot_dim, W)
-                yield p + "mix.dkv.norm", (l.kv_rank,)
-                yield p + "mix.uk", (l.heads * l.dim, l.kv_rank)
-                yield p + "mix.uv", (vd, l.kv_rank)
-                yield p + "mix.g", (l.heads, W)
+                yield from self._latent_shapes(p + "mix.", l)
+            elif l.mixer == hb.MIXER_GROUPED_ATTENTION:
+                yield from self._grouped_shapes(p + "mix.", l)
+            elif l.mixer == hb.MIXER_DELTA:
+                yield from self._delta_shapes(p + "mix.", l)
             elif l.mixer == hb.MIXER_TIED_ATTENTION:
                 for n, rows in (("q", vd), ("k", l.kv_heads * l.dim)):
                     yield p + "mix." + n, (rows, W)
@@ -277,7 +367,7 @@ class LayeredConfig:
                 for g in ("i", "f"):
                     yield p + "mix." + g, (l.heads, W)
                     yield p + "mix." + g + ".b", (l.heads,)
-            if l.mixer in (hb.MIXER_LATENT_ATTENTION, hb.MIXER_TIED_ATTENTION, hb.MIXER_MLSTM):
+            if l.mixer in (hb.MIXER_TIED_ATTENTION, hb.MIXER_MLSTM):
                 yield p + "mix.o", (W, vd)
             if l.ff_kind:
                 yield from self._sublayer_shapes(p, 2)
@@ -289,6 +379,9 @@ class LayeredConfig:
                     yield from ff(f"{p}mlp.e{e}.", l.ff)
                 if l.shared_ff:
                     yield from ff(p + "mlp.shared.", l.shared_ff)
+            elif l.ff_kind == hb.FF_RELU2:
+                yield p + "mlp.up", (l.ff, W)
+                yield p + "mlp.down", (W, l.ff)
             elif l.ff_kind:
                 yield from ff(p + "mlp.", l.ff)
         yield from self._norm_shapes("final.norm")
@@ -335,16 +428,35 @@ def _sumevik(cfg: dict) -> LayeredConfig:
     return out
 
 
-def _layers(out: LayeredConfig, cfg: dict, where: str, feed_forwards: dict = FEED_FORWARDS) -> None:
-    """The 'layers' list: a mixer and an optional feed-forward each; feed_forwards: what a design calls its own."""
+def _tarudra(cfg: dict) -> LayeredConfig:
+    """Windowed grouped attention (some layers on another layer's keys and values), windowed latent attention with query latents and gated delta rules,
+    in any order; squared-relu feed-forwards; layer norms before and after every sublayer with a scale per channel; squashed logits."""
+    where = "Tarudra"
+    out = LayeredConfig(where, int(_need(cfg, "width", where)), int(_need(cfg, "vocab", where)),
+                        float(_need(_need(cfg, "norm", where), "eps", where)), 1.0, residual=hb.RESIDUAL_SANDWICH_LN)
+    out.logit_cap = float(_need(cfg, "logit_softcap", where))
+    if not out.logit_cap > 0.0:
+        raise ConfigError(f"{where}: logits capped at {out.logit_cap}")
+    _layers(out, cfg, where, dict(FEED_FORWARDS, dense=_squared_relu), dict(MIXERS, attention=_grouped_attention, latent_attention=_windowed_latent_attention))
+    for i, l in enumerate(out.layers):
+        src = out.layers[l.kv_from - 1] if 0 < l.kv_from <= i else None
+        if l.kv_from and (src is None or src.mixer != l.mixer or src.kv_from):
+            raise ConfigError(f"{where} layer {i}: no keys and values in layer {l.kv_from - 1}")
+        if src and any(getattr(l, f) != getattr(src, f) for f in ("heads", "kv_heads", "dim", "vdim", "rot_dims", "rot_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow")):
+            raise ConfigError(f"{where} layer {i}: sizes or rotation differ from layer {l.kv_from - 1}, whose keys it reads")
+    return out
+
+
+def _layers(out: LayeredConfig, cfg: dict, where: str, feed_forwards: dict = FEED_FORWARDS, mixers: dict = MIXERS) -> None:
+    """The 'layers' list: a mixer and an optional feed-forward each; feed_forwards, mixers: what a design calls its own."""
     for i, entry in enumerate(_need(cfg, "layers", where)):
         at = f"{where} layer {i}"
         layer = hb.LayerDesc()
         layer.struct_size = hb.C.sizeof(hb.LayerDesc)
         kind = _need(entry, "type", at)
-        if kind not in MIXERS:
+        if kind not in mixers:
             raise ConfigError(f"{at}: unknown mixer '{kind}'")
-        MIXERS[kind](layer, _need(entry, "mixer", at), at)
+        mixers[kind](layer, _need(entry, "mixer", at), at)
         mlp = entry.get("mlp")
         if mlp:
             if _need(mlp, "kind", at) not in feed_forwards:
@@ -353,7 +465,7 @@ def _layers(out: LayeredConfig, cfg: dict, where: str, feed_forwards: dict = FEE
         out.layers.append(layer)
 
 
-ARCHITECTURES = {"Zamelix": _zamelix, "Pubopel": _pubopel, "Sumevik": _sumevik}      # config.json "architecture" -> parser
+ARCHITECTURES = {"Zamelix": _zamelix, "Pubopel": _pubopel, "Sumevik": _sumevik, "Tarudra": _tarudra}      # config.json "architecture" -> parser
 
 
 def parse_config(cfg: dict) -> LayeredConfig:
