@@ -124,7 +124,7 @@ def parse_args():
                     help="CPU rehearsal of the N>1 launcher and hop protocol: gloo + pipeline.FakeStage, no GPU, no engine (not a measurement)")
     ap.add_argument("--layered", default="", metavar="SIZE[,SIZE]",
                     help="models described layer by layer (w*: latent attention + matrix memory; p*: windowed tied attention + mixtures; s*: linear recurrences + "
-                         "gated attention beside gated linear attention) beside the "
+                         "gated attention beside gated linear attention; t*: grouped attention, half of it on shared keys, latent attention, delta rules) beside the "
                          "Llama-style model of equal width, depth and feed-forward, random weights: " + ", ".join(LAYERED_SIZES) + " or all; not the headline metric")
     ap.add_argument("--layered-only", choices=("both", "layered", "closest"), default="both", help="with --layered: run one side (for a profiler)")
     ap.add_argument("--layered-context", type=int, default=2048, help="with --layered: prompt length")
@@ -159,11 +159,20 @@ LAYERED_SIZES = {
     "s2048e": dict(design="Sumevik", width=2048, ff=768, vocab=32000, layers=8, heads=16, kv_heads=4, dim=128, vdim=128, chunk=1024, blocks=8, gheads=8, gdim=128,
                    gvdim=256, rank=16, experts=64, top=6, identity=16, groups=8, keep=4,
                    closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),   # (the closest model takes prompts of this one token by token)
+    # grouped attention, delta rule, grouped attention on the first one's keys, latent attention with a query latent, in turn; squared-relu feed-forwards
+    "t2048": dict(design="Tarudra", width=2048, ff=5632, vocab=32000, layers=8, heads=16, kv_heads=4, dim=128, vdim=128, window=8192, dheads=16, dkv=8, ddim=128, dvdim=128,
+                  lheads=16, rot=64, rank=512, q_rank=768, closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),
+    "t2048w": dict(design="Tarudra", width=2048, ff=5632, vocab=32000, layers=8, heads=16, kv_heads=4, dim=128, vdim=128, window=1024, dheads=8, dkv=4, ddim=256, dvdim=256,
+                   lheads=16, rot=64, rank=512, q_rank=768, closest=dict(num_heads=32, num_kv_heads=4, head_dim=64)),
+    "t4096": dict(design="Tarudra", width=4096, ff=14336, vocab=128256, layers=8, heads=32, kv_heads=8, dim=128, vdim=128, window=8192, dheads=32, dkv=16, ddim=128, dvdim=128,
+                  lheads=32, rot=64, rank=512, q_rank=1536, closest=dict(num_heads=32, num_kv_heads=8, head_dim=128)),
+    "t8192": dict(design="Tarudra", width=8192, ff=28672, vocab=32000, layers=4, heads=64, kv_heads=8, dim=128, vdim=128, window=8192, dheads=64, dkv=16, ddim=128, dvdim=128,
+                  lheads=64, rot=64, rank=512, q_rank=1536, closest=dict(num_heads=64, num_kv_heads=8, head_dim=128)),
 }
 
 
 class RandomBf16:
-    """Random weights for a layered model: slices of one random block, scaled by 1 / sqrt(in); norm weights and temperatures 1."""
+    """Random weights for a layered model: slices of one random block, scaled by 1 / sqrt(in); norm weights, temperatures and channel scales 1."""
 
     def __init__(self, seed=1):
         self.block, self.scaled = np.random.default_rng(seed).standard_normal(1 << 22, dtype=np.float32), {}
@@ -171,13 +180,23 @@ class RandomBf16:
     def get(self, name, shape):
         n = int(np.prod(shape))
         if len(shape) <= 1:
-            return 0, np.full(n, 0.5 if not shape else 1.0 if "norm" in name.rsplit(".", 1)[-1] or name.endswith("temp") else 0.0, np.float32)
+            return 0, np.full(n, 0.5 if not shape else 1.0 if "norm" in name.rsplit(".", 1)[-1] or name.endswith(("temp", ".ls1", ".ls2")) else 0.0, np.float32)
         if shape[1] not in self.scaled:
             self.scaled[shape[1]] = ((self.block * np.float32(1.0 / np.sqrt(shape[1]))).view(np.uint32) >> 16).astype(np.uint16)
         return 30, np.resize(np.roll(self.scaled[shape[1]], len(name) * 7919), n)
 
 
 def layered_config(sz):
+    if sz.get("design") == "Tarudra":
+        mlp, mask = {"kind": "dense", "ff": sz["ff"]}, {"size": sz["window"]}
+        grouped = {"heads": sz["heads"], "kv_heads": sz["kv_heads"], "dim": sz["dim"], "vdim": sz["vdim"], "scale": sz["dim"] ** -0.5, "mask": mask,
+                   "rot": {"base": 10000.0, "dims": sz["dim"], "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+        delta = {"heads": sz["dheads"], "kv_heads": sz["dkv"], "dim": sz["ddim"], "vdim": sz["dvdim"], "conv": 4}
+        latent = {"heads": sz["lheads"], "dim": sz["dim"], "rot_dim": sz["rot"], "vdim": sz["vdim"], "kv_rank": sz["rank"], "q_rank": sz["q_rank"],
+                  "scale": (sz["dim"] + sz["rot"]) ** -0.5, "mask": mask, "rot": {"base": 10000.0, "dims": sz["rot"]}}
+        kinds = [("attention", lambda i: grouped), ("delta", lambda i: delta), ("attention", lambda i: dict(grouped, kv_from=i - 2)), ("latent_attention", lambda i: latent)]
+        return {"architecture": "Tarudra", "width": sz["width"], "vocab": sz["vocab"], "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+                "layers": [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1](i), "mlp": mlp} for i in range(sz["layers"])]}
     if sz.get("design") == "Sumevik":
         W = sz["width"]
         mlp = {"kind": "dense", "ff": sz["ff"]} if "experts" not in sz else {
@@ -249,7 +268,7 @@ def run_layered(args, pkg):
         prompt = prompt_tokens(n, sz["vocab"])
         cap = n + steps * (args.reps + 1) + 64
         if args.layered_only != "closest":
-            cfg = pkg.layered_model.parse_config(layered_config(sz)).resolve(lambda name: (sz["rank"], sz["width"]))
+            cfg = pkg.layered_model.parse_config(layered_config(sz)).resolve(lambda name: (sz.get("rank"), sz["width"]))
             eng = pkg.HipGpuInference.from_layered(pkg.LayeredModel(cfg, RandomBf16()), cap)
             r["layered"] = layered_measure(eng, prompt, steps, args.reps)
             eng.close()

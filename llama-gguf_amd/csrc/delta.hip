@@ -82,7 +82,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(const DeltaShape s, con
     }
     vs[tid - 192] = v;
   }
-  ssq = wave_sum(ssq); ssk = wave_sum(ssk); sqk = wave_sum(sqk);
+  ssq = wave_total(ssq); ssk = wave_total(ssk); sqk = wave_total(sqk);
   if (lane == 0) { sums[0][wv] = ssq; sums[1][wv] = ssk; sums[2][wv] = sqk; }
   __syncthreads();
   auto tot = [&](int i) { return (sums[i][0] + sums[i][1]) + (sums[i][2] + sums[i][3]); };
@@ -211,7 +211,7 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(const DeltaShape s, con
         float ss = 0.0f;
 #pragma unroll
         for (int n = 0; n < NC; n++) ss = __builtin_fmaf(x[n][i], x[n][i], ss);
-        f = 1.0f / __builtin_sqrtf(wave_sum(ss) + 1e-6f);
+        f = 1.0f / __builtin_sqrtf(wave_total(ss) + 1e-6f);
         if (kind == 0) f /= __builtin_sqrtf((float)s.dim);
       }
 #pragma unroll

@@ -174,6 +174,11 @@ __device__ __forceinline__ void post_finish(const PostUpdate& a, const PostIn& r
   post_input(a, r, c, p, v, nalpha);
 }
 
+// sum over the wave without the LDS crossbar, every lane gets it
+__device__ __forceinline__ float wave_total(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, wave_sum_to_lane63(v)), 63));
+}
+
 // sum over `N` neighbouring lanes, every one of them gets it
 template <uint32_t N> __device__ __forceinline__ float lanes_sum(float v) {
   v += dpp_f<0xB1>(v); v += dpp_f<0x4E>(v); v += dpp_f<0x141>(v);

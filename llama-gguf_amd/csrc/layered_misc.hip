@@ -480,35 +480,51 @@ hipError_t ln_block_launch(const LnBlock& a, bool f32, hipStream_t st) {
   return f32 ? ln_block_go<float, 1>(a, st) : ln_block_go<__bf16, 1>(a, st);
 }
 
-// a wave per row
-template <class T>
+// a wave per row, V values at a time
+template <class T, int V>
 __global__ void __launch_bounds__(256) rms_cols_kernel(const float* __restrict__ x, uint32_t ld, const float* __restrict__ w, float eps, uint32_t n, uint32_t M, T* __restrict__ xa,
                                                        uint32_t ldx) {
   const uint32_t t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= M) return;
   const float* r = x + (size_t)t * ld;
-  constexpr uint32_t U = 8;   // values of a lane kept between the two passes
-  float v[U], q = 0.0f;
+  T* o = xa + (size_t)t * ldx;
+  constexpr uint32_t U = 8, S = 64 * V;   // loads of a lane kept between the two passes
+  VecF<V> v[U];
+  float q = 0.0f;
 #pragma unroll
   for (uint32_t u = 0; u < U; u++) {
-    const uint32_t c = lane + u * 64;
-    v[u] = c < n ? r[c] : 0.0f;
-    q = __builtin_fmaf(v[u], v[u], q);
+    const uint32_t c = lane * V + u * S;
+    v[u] = load_vec<V>(r + (c < n ? c : 0));
+#pragma unroll
+    for (int i = 0; i < V; i++) q = c < n ? __builtin_fmaf(v[u].v[i], v[u].v[i], q) : q;
   }
-  for (uint32_t c = lane + U * 64; c < n; c += 64) q = __builtin_fmaf(r[c], r[c], q);
+  for (uint32_t c = lane * V + U * S; c < n; c += S) {
+    const VecF<V> z = load_vec<V>(r + c);
+#pragma unroll
+    for (int i = 0; i < V; i++) q = __builtin_fmaf(z.v[i], z.v[i], q);
+  }
   const float inv = 1.0f / __builtin_sqrtf(wave_sum(q) / (float)n + eps);
+  auto put = [&](uint32_t c, const VecF<V>& z) {
+    const VecF<V> wt = load_vec<V>(w + c);
+    T d[V];
 #pragma unroll
-  for (uint32_t u = 0; u < U; u++) {
-    const uint32_t c = lane + u * 64;
-    if (c < n) xa[(size_t)t * ldx + c] = to_act<T>(v[u] * inv * w[c]);
-  }
-  for (uint32_t c = lane + U * 64; c < n; c += 64) xa[(size_t)t * ldx + c] = to_act<T>(r[c] * inv * w[c]);
+    for (int i = 0; i < V; i++) d[i] = to_act<T>(z.v[i] * inv * wt.v[i]);
+    __builtin_memcpy(__builtin_assume_aligned(o + c, sizeof(d)), d, sizeof(d));
+  };
+#pragma unroll
+  for (uint32_t u = 0; u < U; u++)
+    if (lane * V + u * S < n) put(lane * V + u * S, v[u]);
+  for (uint32_t c = lane * V + U * S; c < n; c += S) put(c, load_vec<V>(r + c));
 }
 
 hipError_t rms_cols_launch(const float* x, uint32_t ld, const float* w, float eps, uint32_t n, uint32_t M, void* xa, uint32_t ldx, bool f32, hipStream_t st) {
   if (!x || !w || !xa || n == 0 || M == 0 || ldx < n || ld < n) return hipErrorInvalidValue;
-  if (f32) hipLaunchKernelGGL(rms_cols_kernel<float>, dim3((M + 3) / 4), dim3(256), 0, st, x, ld, w, eps, n, M, (float*)xa, ldx);
-  else hipLaunchKernelGGL(rms_cols_kernel<__bf16>, dim3((M + 3) / 4), dim3(256), 0, st, x, ld, w, eps, n, M, (__bf16*)xa, ldx);
+  const dim3 grid((M + 3) / 4), th(256);
+  const bool v4 = n % 4 == 0 && ld % 4 == 0 && ldx % 4 == 0 && (uintptr_t)x % 16 == 0;
+  if (f32 && v4) hipLaunchKernelGGL((rms_cols_kernel<float, 4>), grid, th, 0, st, x, ld, w, eps, n, M, (float*)xa, ldx);
+  else if (f32) hipLaunchKernelGGL((rms_cols_kernel<float, 1>), grid, th, 0, st, x, ld, w, eps, n, M, (float*)xa, ldx);
+  else if (v4) hipLaunchKernelGGL((rms_cols_kernel<__bf16, 4>), grid, th, 0, st, x, ld, w, eps, n, M, (__bf16*)xa, ldx);
+  else hipLaunchKernelGGL((rms_cols_kernel<__bf16, 1>), grid, th, 0, st, x, ld, w, eps, n, M, (__bf16*)xa, ldx);
   return hipGetLastError();
 }
 

@@ -113,12 +113,46 @@ __device__ __forceinline__ float mv_glu(const LinMv& a, float gate, float up) {
   return (a.act == LA_SILU ? silu_f(gate) : gelu_tanh_f(gate)) * up;
 }
 
+// mean and 1 / sqrt(variance + eps) of the workgroup's K values, U per thread (channel tid + u * kMvThreads), with one barrier: every wave takes its own
+// mean and squared deviations, which are then put together.  st: [3][16] floats of LDS that nothing else uses
+template <int U> __device__ __forceinline__ void mv_layer_stats(const float* v, uint32_t K, float eps, float (*st)[16], float& mean, float& inv) {
+  const uint32_t wave = threadIdx.x >> 6;
+  float n = 0.0f, s = 0.0f, q = 0.0f;
+#pragma unroll
+  for (int u = 0; u < U; u++) {
+    const uint32_t c0 = wave * 64 + u * kMvThreads;
+    n += (float)(c0 < K ? (K - c0 < 64 ? K - c0 : 64u) : 0u);
+    s += threadIdx.x + u * kMvThreads < K ? v[u] : 0.0f;
+  }
+  const float mw = wave_total(s) / fmaxf(n, 1.0f);
+#pragma unroll
+  for (int u = 0; u < U; u++) { const float d = v[u] - mw; q = threadIdx.x + u * kMvThreads < K ? __builtin_fmaf(d, d, q) : q; }
+  q = wave_total(q);
+  if ((threadIdx.x & 63) == 0) { st[0][wave] = n; st[1][wave] = mw; st[2][wave] = q; }
+  __syncthreads();
+  f32x4 nn[4], mm[4], t = (f32x4)(0.0f);
+#pragma unroll
+  for (int i = 0; i < 4; i++) {
+    nn[i] = *reinterpret_cast<const f32x4*>(&st[0][i * 4]);
+    mm[i] = *reinterpret_cast<const f32x4*>(&st[1][i * 4]);
+    t += nn[i] * mm[i];
+  }
+  const float rk = 1.0f / (float)K;
+  mean = ((t.x + t.y) + (t.z + t.w)) * rk;
+  t = (f32x4)(0.0f);
+#pragma unroll
+  for (int i = 0; i < 4; i++) { const f32x4 d = mm[i] - mean; t += *reinterpret_cast<const f32x4*>(&st[2][i * 4]) + nn[i] * d * d; }
+  inv = 1.0f / __builtin_sqrtf(((t.x + t.y) + (t.z + t.w)) * rk + eps);
+}
+
+// PRO: LinPro; LP_SANDWICH + 256 U: up to U values per thread, in registers
 template <int PRO, int SRC, bool POST>
 __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint32_t n_groups, uint32_t ks, uint32_t g1) {
   constexpr bool MOE = SRC == LS_EXPERTS || SRC == LS_MOE_DOWN;
   extern __shared__ __attribute__((aligned(16))) float xs[];   // [kp]
   __shared__ float red[2][16][kMvR];
   __shared__ __attribute__((aligned(16))) float bred[PRO == LP_SANDWICH ? 64 : 16];
+  __shared__ __attribute__((aligned(16))) float lst[PRO > 255 ? 2 : 1][3][16];
   __shared__ __attribute__((aligned(16))) float zs[SRC == LS_EXPERTS ? kMaxExperts : 4];
   __shared__ __attribute__((aligned(16))) float zc[SRC == LS_EXPERTS ? 2 * kMaxRouted : 4];   // choice scores, groups
   __shared__ float id_w;
@@ -179,6 +213,31 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
         xs[i] = h;
         if (a.hout && blockIdx.x == 0) a.hout[i] = h;
       }
+  } else if constexpr (PRO > 255) {
+    constexpr int U = PRO >> 8;
+    float v[U], y[U], w1[U], w2[U], mean, inv;
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      const uint32_t i = tid + u * kMvThreads, ic = i < a.k ? i : a.k - 1;
+      if (a.y) { y[u] = a.y[ic]; if (U <= 4) w1[u] = a.nw[ic]; }
+      v[u] = a.x[ic];
+      if (U <= 4) w2[u] = a.nw2[ic];   // (more of them do not fit the registers)
+    }
+    if (a.y) {
+      mv_layer_stats<U>(y, a.k, a.eps, lst[0], mean, inv);
+#pragma unroll
+      for (int u = 0; u < U; u++) {
+        const uint32_t i = tid + u * kMvThreads;
+        v[u] = __builtin_fmaf(a.mult, (y[u] - mean) * inv * (U <= 4 ? w1[u] : a.nw[i < a.k ? i : a.k - 1]), v[u]);
+        if (blockIdx.x == 0 && i < a.k) a.xout[i] = v[u];
+      }
+    }
+    mv_layer_stats<U>(v, a.k, a.eps, lst[1], mean, inv);
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      const uint32_t i = tid + u * kMvThreads;
+      if (i < a.k) xs[i] = (v[u] - mean) * inv * (U <= 4 ? w2[u] : a.nw2[i]);
+    }
   } else if (PRO == LP_SANDWICH) {
     constexpr uint32_t U = 4;   // channels a thread has in flight, with everything they need
     float v[U], y[U], w1[U], w2[U];
@@ -228,7 +287,7 @@ __global__ void __launch_bounds__(kMvThreads) lin_mv_kernel(const LinMv a, uint3
         ss = __builtin_fmaf(e < a.vdim ? v[j] : 0.0f, v[j], ss);
       }
       for (uint32_t e = lane + 256; e < a.vdim; e += 64) ss = __builtin_fmaf(num[e], num[e], ss);
-      const float r = 1.0f / __builtin_sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+      const float r = 1.0f / __builtin_sqrtf(wave_total(ss) / (float)a.vdim + a.eps);
 #pragma unroll
       for (int j = 0; j < 4; j++) {
         const uint32_t e = lane + j * 64;
@@ -428,7 +487,13 @@ hipError_t lin_mv_launch(int pro, const LinMv& a, hipStream_t st, int src) {
     case LP_RESID: return a.x && a.y && a.nw && a.xout ? lin_mv_go<LP_RESID>(a, src, st) : hipErrorInvalidValue;
     case LP_HEAD: return a.x && a.y && a.nw && a.nw2 && a.xout && src == LS_PLAIN && !a.post.xout ? lin_mv_run<LP_HEAD, LS_PLAIN, false>(a, st) : hipErrorInvalidValue;
     case LP_PRE: return a.x && a.nw2 && (!a.y || a.xout) ? lin_mv_go<LP_PRE>(a, src, st) : hipErrorInvalidValue;
-    case LP_SANDWICH: return a.x && a.nw2 && (!a.y || (a.nw && a.xout)) && src == LS_PLAIN && !a.post.xout ? lin_mv_run<LP_SANDWICH, LS_PLAIN, false>(a, st) : hipErrorInvalidValue;
+    case LP_SANDWICH:
+      if (!a.x || !a.nw2 || (a.y && (!a.nw || !a.xout)) || src != LS_PLAIN || a.post.xout) return hipErrorInvalidValue;
+      if (a.k <= 1 * kMvThreads) return lin_mv_run<LP_SANDWICH + 256 * 1, LS_PLAIN, false>(a, st);
+      if (a.k <= 2 * kMvThreads) return lin_mv_run<LP_SANDWICH + 256 * 2, LS_PLAIN, false>(a, st);
+      if (a.k <= 4 * kMvThreads) return lin_mv_run<LP_SANDWICH + 256 * 4, LS_PLAIN, false>(a, st);
+      if (a.k <= 8 * kMvThreads) return lin_mv_run<LP_SANDWICH + 256 * 8, LS_PLAIN, false>(a, st);
+      return lin_mv_run<LP_SANDWICH, LS_PLAIN, false>(a, st);
     case LP_READ:
       return a.num && a.nw && a.gate && a.heads * a.vdim == a.k && src == LS_PLAIN && !a.post.xout ? lin_mv_run<LP_READ, LS_PLAIN, false>(a, st) : hipErrorInvalidValue;
     case LP_MLSTM:

@@ -57,7 +57,7 @@ def _rotated_of(layer: hb.LayerDesc, size: int, where: str) -> None:
 def _window(layer: hb.LayerDesc, mx: dict, where: str) -> None:
     """The last positions that a position sees; without an entry all of them."""
     mask = mx.get("mask")
-    if mask:
+    if mask is not None:
         layer.window = int(_need(mask, "size", where))
         if layer.window < 1:
             raise ConfigError(f"{where}: a window of {layer.window} positions")
@@ -96,6 +96,8 @@ def _grouped_attention(layer: hb.LayerDesc, mx: dict, where: str) -> None:
     _window(layer, mx, where)
     if mx.get("kv_from") is not None:
         layer.kv_from = int(mx["kv_from"]) + 1
+        if layer.kv_from < 1:
+            raise ConfigError(f"{where}: keys and values of layer {mx['kv_from']}")
 
 
 def _delta(layer: hb.LayerDesc, mx: dict, where: str) -> None:

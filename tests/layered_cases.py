@@ -85,6 +85,35 @@ def prenorm(layers, width=88, vocab=150, eps=1e-6, logit_scale=1.7):
     return {"architecture": "Sumevik", "width": width, "vocab": vocab, "norm": {"eps": eps}, "logit_scale": logit_scale, "layers": layers}
 
 
+def grouped_attn(heads=6, kv_heads=2, dim=24, vdim=20, window=40, rot=8, base=10000.0, scaling=None, scale=None, source=None, mlp=None):
+    """Grouped attention with a sink; window 0: no mask, rot 0: nothing is rotated; source: the layer whose keys and values it reads."""
+    mx = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale or dim ** -0.5}
+    if window:
+        mx["mask"] = {"size": window}
+    if rot:
+        mx["rot"] = dict({"base": base, "dims": rot}, **({"scaling": scaling} if scaling else {}))
+    if source is not None:
+        mx["kv_from"] = source
+    return {"type": "attention", "mixer": mx, "mlp": mlp}
+
+
+def latent2(heads=3, dim=24, rot=8, vdim=20, rank=40, q_rank=28, window=40, scale=None, base=10000.0, dims=None, scaling=None, rotate=True, mlp=None):
+    """Latent attention with a query latent and a gate per value; window 0: no mask."""
+    lay = attn(heads, dim, rot, vdim, rank, scale, base, dims, scaling, 0, rotate)
+    lay["mixer"]["q_rank"] = q_rank
+    if window:
+        lay["mixer"]["mask"] = {"size": window}
+    return dict(lay, mlp=mlp)
+
+
+def delta(heads=4, kv_heads=2, dim=24, vdim=20, taps=4, mlp=None):
+    return {"type": "delta", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": taps}, "mlp": mlp}
+
+
+def sandwich_ln(layers, width=88, vocab=150, eps=1e-5, cap=2.5):
+    return {"architecture": "Tarudra", "width": width, "vocab": vocab, "norm": {"eps": eps}, "logit_softcap": cap, "layers": layers}
+
+
 def parse(pkg, cfg):
     def shape_of(name):
         return cfg["layers"][int(name[1:].split(".")[0])].get("rank"), cfg["width"]
@@ -107,6 +136,10 @@ class Weights(dict):
             last = name.split(".")[-1]
             if getattr(parsed, "residual", 0) == 2 and last in ("norm1", "norm2") or getattr(parsed, "tied_head", False) and name == "final.norm":
                 v = 0.2 * rng.standard_normal(shape)           # stored around zero
+            elif last in ("ls1", "ls2"):
+                v = 0.7 + 0.2 * rng.standard_normal(shape)
+            elif last == "dt_bias":
+                v = -4.0 + 1.5 * rng.standard_normal(shape)    # a state that lasts
             elif last == "lam":
                 v = -5.0 + 1.5 * rng.standard_normal(shape)    # a state that lasts
             elif last == "conv":
@@ -117,7 +150,7 @@ class Weights(dict):
                 v = 2.0 + rng.standard_normal(shape)
             elif len(shape) == 3:
                 v = rng.standard_normal(shape) / np.sqrt(shape[-1])
-            elif last == "b":
+            elif last == "b" and not name.endswith("mix.b"):
                 v = (3.0 if name.endswith(".f.b") else 0.0) + (1.0 if name.endswith(".f.b") else 0.5) * rng.standard_normal(shape)
             elif name.endswith(".alpha"):
                 v = np.asarray(0.4 + 0.4 * rng.random())
@@ -127,7 +160,7 @@ class Weights(dict):
                 v = rng.standard_normal(shape)
             elif "canon" in name:
                 v = 0.4 * rng.standard_normal(shape)
-            elif "norm" in name.split(".")[-1] or name.endswith(("norm1", "norm2")):
+            elif "norm" in last or name.endswith(("norm1", "norm2")):
                 v = 1.0 + 0.2 * rng.standard_normal(shape)
             elif name.endswith(".f.b"):
                 v = 3.0 + rng.standard_normal(shape)          # a memory that lasts

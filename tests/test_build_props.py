@@ -33,7 +33,7 @@ def _usage(src):
 def test_no_kernel_uses_scratch_or_spills_vgprs():
     for src in ("matvec_mfma.hip", "matvec_batch.hip", "prefill.hip", "attention.hip", "attention_tq.hip", "misc.hip", "dequant.hip",
                 "linear_bf16.hip", "latent_attention.hip", "tied_attention.hip", "gated_attention.hip", "moe_route.hip", "mlstm.hip",
-                "gla.hip", "glru.hip", "layered_misc.hip"):
+                "gla.hip", "glru.hip", "delta.hip", "layered_misc.hip"):
         usage = _usage(src)
         assert usage, f"no kernels found in {src}"
         for fn, u in usage.items():

@@ -206,7 +206,7 @@ def test_bench_sizes_are_models_the_registry_takes(pkg):
     for name, sz in bench.LAYERED_SIZES.items():
         cfg = bench.layered_config(sz)
         p = pkg.layered_model.parse_config(cfg).resolve(lambda _: (16, sz["width"]))
-        assert p.num_layers == sz["layers"] and {l.mixer for l in p.layers} == {"p": {3}, "w": {1, 2}, "s": {6, 7}}[name[0]], name
+        assert p.num_layers == sz["layers"] and {l.mixer for l in p.layers} == {"p": {3}, "w": {1, 2}, "s": {6, 7}, "t": {1, 8, 9}}[name[0]], name
         shapes = dict(p.tensor_shapes())
         t, data = bench.RandomBf16().get("l0.mix.o", (8, 16))
         assert t == 30 and data.size == 128 and shapes["embed" if p.tied_head else "head"] == (sz["vocab"], sz["width"])
@@ -503,3 +503,170 @@ def test_create_refuses_unusable_recurrences_and_routers(pkg):
     assert status(lc.prenorm([lc.rglru(mlp=lc.grouped())]), router_form=7) == "Unsupported"
     assert status(lc.prenorm([lc.rglru(mlp=lc.grouped(600, 8, 2, 8, None))])) == "Unsupported"
     assert status(lc.config([lc.mem(ff=0) | {"mlp": None}]), ff_kind=2, ff=8, experts=2, top=1, router_form=1, expert_form=1, groups=1, keep_groups=1, identity=1) == "Unsupported"
+
+
+# ---- the Tarudra design ----
+def test_halves_turn_as_complex_numbers():
+    rng = np.random.default_rng(21)
+    x, rot = rng.standard_normal((5, 2, 9)), {"dims": 6, "base": 30.0}
+    got = lo.rotate_halves(x, np.arange(5), rot)
+    z = (x[..., :3] + 1j * x[..., 3:6]) * np.exp(1j * np.arange(5)[:, None, None] * 30.0 ** (-np.arange(3) / 3.0))
+    assert np.allclose(got[..., :3], z.real) and np.allclose(got[..., 3:6], z.imag) and np.array_equal(got[..., 6:], x[..., 6:])
+    assert np.allclose(lo.rotate_pairs(x[..., [0, 3, 1, 4, 2, 5]], np.arange(5), rot)[..., 0::2], z.real)       # the same rotation, other neighbours
+
+
+def test_grouped_attention_equals_an_explicit_matrix_form():
+    T, Wd, H, G, d, dv, size = 11, 17, 4, 2, 6, 5, 4
+    mx = lc.grouped_attn(H, G, d, dv, size, 4, 50.0, scale=0.7)["mixer"]
+    w, rng = _random({"q": (H * d, Wd), "q.b": (H * d,), "k": (G * d, Wd), "k.b": (G * d,), "v": (G * dv, Wd), "v.b": (G * dv,), "o": (Wd, H * dv), "o.b": (Wd,)}, 22)
+    h, other = rng.standard_normal((T, Wd)), rng.standard_normal((T, Wd))
+    turn = np.exp(1j * np.arange(T)[:, None, None] * 50.0 ** (-np.arange(2) / 2.0))
+
+    def rot(x):
+        z = (x[..., 0:4:2] + 1j * x[..., 1:4:2]) * turn
+        return np.concatenate([np.stack([z.real, z.imag], -1).reshape(T, x.shape[1], 4), x[..., 4:]], -1)
+    for src in (h, other):                       # its own keys and values, and another layer's
+        k = np.repeat(rot((src @ w["k"].T + w["k.b"]).reshape(T, G, d)), H // G, axis=1)
+        v = np.repeat((src @ w["v"].T + w["v.b"]).reshape(T, G, dv), H // G, axis=1)
+        s = np.einsum("ihd,jhd->hij", rot((h @ w["q"].T + w["q.b"]).reshape(T, H, d)), k) * 0.7
+        i = np.arange(T)
+        e = np.where((i[None] <= i[:, None]) & (i[:, None] - i[None] < size), np.exp(s), 0.0)
+        out = np.einsum("hij,jhd->ihd", e / (1.0 + e.sum(-1, keepdims=True)), v).reshape(T, -1)
+        assert np.allclose(lo.grouped_attention(h, w, mx, lo.grouped_keys_values(src, w, mx)), out @ w["o"].T + w["o.b"])
+
+
+def test_windowed_latent_attention_equals_an_explicit_matrix_form():
+    T, Wd, H, d, r, dv, kr, qr, size = 10, 13, 3, 4, 4, 5, 6, 7, 3
+    mx = lc.latent2(H, d, r, dv, kr, qr, size, 0.6, 40.0)["mixer"]
+    w, rng = _random({"dq": (qr, Wd), "dq.norm": (qr,), "uq": (H * (d + r), qr), "dkv": (kr + r, Wd), "dkv.norm": (kr,), "uk": (H * d, kr), "uv": (H * dv, kr), "g": (H * dv, Wd),
+                      "o": (Wd, H * dv)}, 23)
+    h = rng.standard_normal((T, Wd))
+    n = lambda x, g: x / np.sqrt((x * x).mean(-1, keepdims=True) + 1e-6) * g
+    q = (n(h @ w["dq"].T, w["dq.norm"]) @ w["uq"].T).reshape(T, H, d + r)
+    c, kr_part = n(h @ w["dkv"][:kr].T, w["dkv.norm"]), h @ w["dkv"][kr:].T
+    turn = np.exp(1j * np.arange(T)[:, None] * 40.0 ** (-np.arange(2) / 2.0))
+    rot = lambda x: (x[..., :2] + 1j * x[..., 2:]) * (turn if x.ndim == 2 else turn[:, None])
+    s = np.einsum("ihd,jhd->hij", q[..., :d], (c @ w["uk"].T).reshape(T, H, d)) + np.einsum("ihd,jd->hij", rot(q[..., d:]), rot(kr_part).conj()).real
+    i = np.arange(T)
+    e = np.where((i[None] <= i[:, None]) & (i[:, None] - i[None] < size), np.exp(0.6 * s), 0.0)
+    out = np.einsum("hij,jhd->ihd", e / e.sum(-1, keepdims=True), (c @ w["uv"].T).reshape(T, H, dv)).reshape(T, -1) / (1 + np.exp(-(h @ w["g"].T)))
+    assert np.allclose(lo.windowed_latent_attention(h, w, mx, 1e-6), out @ w["o"].T)
+
+
+def test_delta_rule_equals_one_linear_system():
+    """The written rows solve (I + L) U = B V for the whole sequence; outputs are decayed scores times them."""
+    T, Wd, H, G, d, dv, taps = 9, 12, 4, 2, 5, 3, 3
+    w, rng = _random({"q": (G * d, Wd), "k": (G * d, Wd), "v": (H * dv, Wd), "q.conv": (G * d, taps), "k.conv": (G * d, taps), "v.conv": (H * dv, taps), "b": (H, Wd), "a": (H, Wd),
+                      "A_log": (H,), "dt_bias": (H,), "norm": (dv,), "g": (H * dv, Wd), "o": (Wd, H * dv)}, 24)
+    h = rng.standard_normal((T, Wd))
+
+    def short(n):
+        x = np.concatenate([np.zeros((taps - 1, w[n].shape[0])), h @ w[n].T])
+        y = sum(x[j:j + T] * w[n + ".conv"][:, j] for j in range(taps))
+        return y / (1 + np.exp(-y))
+    unit = lambda x: x / np.sqrt((x * x).sum(-1, keepdims=True) + 1e-6)
+    q, k, v = unit(short("q").reshape(T, G, d)) / math.sqrt(d), unit(short("k").reshape(T, G, d)), short("v").reshape(T, H, dv)
+    beta = 1 / (1 + np.exp(-(h @ w["b"].T)))
+    ld = np.cumsum(-np.exp(w["A_log"]) * np.log1p(np.exp(h @ w["a"].T + w["dt_bias"])), axis=0)
+    out = np.zeros((T, H, dv))
+    for n in range(H):
+        dec = np.tril(np.exp(np.minimum(ld[:, None, n] - ld[None, :, n], 0.0)))
+        kn, qn = k[:, n // 2], q[:, n // 2]
+        U = np.linalg.solve(np.eye(T) + beta[:, n, None] * np.tril(dec * (kn @ kn.T), -1), beta[:, n, None] * v[:, n])
+        out[:, n] = (dec * (qn @ kn.T)) @ U
+    out = out / np.sqrt((out * out).mean(-1, keepdims=True) + 1e-5) * w["norm"]
+    g = h @ w["g"].T
+    mx = {"heads": H, "kv_heads": G, "dim": d, "vdim": dv}
+    assert np.allclose(lo.delta_rule(h, w, mx, 1e-5), (out.reshape(T, -1) * g / (1 + np.exp(-g))) @ w["o"].T)
+
+
+def test_squared_relu_and_capped_logits(pkg):
+    w, rng = _random({"up": (5, 4), "down": (4, 5)}, 25)
+    x = rng.standard_normal((3, 4))
+    z = x @ w["up"].T
+    assert np.allclose(lo.squared_relu_ff(x, w), np.where(z > 0, z * z, 0) @ w["down"].T)
+    cfg = lc.sandwich_ln([lc.grouped_attn()], cap=0.7)
+    W = lc.Weights(lc.parse(pkg, cfg))
+    o = lo.forward(cfg, W, lc.tokens(5, cfg["vocab"]))
+    wide = lo.forward(dict(cfg, logit_softcap=1e9), W, lc.tokens(5, cfg["vocab"]))
+    assert np.abs(o).max() < 0.7 and np.allclose(o, 0.7 * np.tanh(wide / 0.7))
+
+
+def test_a_tarudra_sequence_does_not_see_its_future(pkg):
+    cfg = lc.sandwich_ln([lc.grouped_attn(window=4, mlp=lc.dense()), lc.delta(), lc.latent2(window=5), lc.grouped_attn(window=6, source=0)])
+    W = lc.Weights(lc.parse(pkg, cfg))
+    t = lc.tokens(14, cfg["vocab"])
+    assert np.allclose(lo.forward(cfg, W, t)[:9], lo.forward(cfg, W, t[:9]))
+
+
+def test_a_reader_sees_the_cache_of_its_source(pkg):
+    """The source's keys and values decide, not the reader's input; the reader's window is its own."""
+    cfg = lc.sandwich_ln([lc.grouped_attn(window=2), lc.grouped_attn(window=5, source=0)])
+    W = lc.Weights(lc.parse(pkg, cfg))
+    assert "l1.mix.k" not in W and "l1.mix.v.b" not in W and "l1.mix.o.b" in W
+    t = lc.tokens(9, cfg["vocab"])
+    base = lo.forward(cfg, W, t)[-1]
+    for far, seen in ((4, True), (3, False)):              # the last token is 8: its widest window is 4 .. 8
+        u = list(t)
+        u[far] = (u[far] + 1) % cfg["vocab"]
+        assert np.allclose(lo.forward(cfg, W, u)[-1], base) != seen
+
+
+def test_parse_tarudra_reads_every_size_and_constant(pkg):
+    hb = pkg.hip_backend
+    cfg = lc.sandwich_ln([lc.grouped_attn(9, 3, 18, 7, 21, 6, 77.0, dict(factor=3.0, original=50, fast=9.0, slow=2.0), 0.3, mlp=lc.dense(31)), lc.delta(6, 2, 11, 13, 3),
+                          lc.grouped_attn(9, 3, 18, 7, 40, 6, 77.0, dict(factor=3.0, original=50, fast=9.0, slow=2.0), 0.2, source=0), lc.latent2(5, 12, 6, 9, 17, 23, 33, 0.4, 88.0, 4, mlp=lc.dense(8)),
+                          lc.latent2(window=0, rotate=False), lc.grouped_attn(window=0, rot=0)], eps=3e-6, cap=12.5)
+    p = pkg.layered_model.parse_config(cfg)
+    a, b, c, e, f, g = p.layers
+    assert (a.mixer, a.heads, a.kv_heads, a.dim, a.vdim, a.window, a.rot_dims, a.rot_base, a.scale, a.sink_one, a.kv_from) == (hb.MIXER_GROUPED_ATTENTION, 9, 3, 18, 7, 21, 6, 77.0, 0.3, 1, 0)
+    assert (a.yarn_factor, a.yarn_original, a.yarn_fast, a.yarn_slow, a.ff_kind, a.ff) == (3.0, 50.0, 9.0, 2.0, hb.FF_RELU2, 31)
+    assert (b.mixer, b.heads, b.kv_heads, b.dim, b.vdim, b.taps, b.ff_kind) == (hb.MIXER_DELTA, 6, 2, 11, 13, 3, hb.FF_NONE)
+    assert (c.kv_from, c.window, c.scale) == (1, 40, 0.2)
+    assert (e.mixer, e.heads, e.dim, e.rot_dim, e.vdim, e.kv_rank, e.q_rank, e.window, e.scale, e.rot_base, e.rot_dims) == (hb.MIXER_LATENT_ATTENTION, 5, 12, 6, 9, 17, 23, 33, 0.4, 88.0, 4)
+    assert (e.rot_form, e.gate_form, e.yarn_factor) == (hb.ROT_HALVES, hb.GATE_VALUES, 0.0) and (f.window, f.rot_dims, g.window, g.rot_dims) == (0, 0, 0, 0)
+    d = p.desc()
+    assert (d.width, d.vocab_size, d.norm_eps, d.residual_mult, d.residual, d.tied_head, d.logit_cap) == (88, 150, 3e-6, 1.0, hb.RESIDUAL_SANDWICH_LN, 0, 12.5)
+    s = dict(p.tensor_shapes())
+    assert s["l0.mix.v.b"] == (21,) and s["l0.mix.o"] == (88, 63) and s["l0.mix.o.b"] == (88,) and s["l0.mlp.up"] == (31, 88) and "l0.mlp.gate" not in s and s["l0.ls2"] == (88,)
+    assert s["l1.mix.v.conv"] == (78, 3) and s["l1.mix.q"] == (22, 88) and s["l1.mix.b"] == (6, 88) and s["l1.mix.dt_bias"] == (6,) and s["l1.mix.norm"] == (13,) and "l1.ls2" not in s
+    assert "l2.mix.k" not in s and s["l2.mix.q"] == (162, 88) and s["l3.mix.uq"] == (90, 23) and s["l3.mix.dkv"] == (23, 88) and s["l3.mix.g"] == (45, 88) and s["l3.norm2b"] == (88,)
+    assert "l3.mix.q" not in s and "head" in s
+
+
+@pytest.mark.parametrize("break_it", [
+    lambda c: c.pop("logit_softcap"), lambda c: c.update(logit_softcap=0.0), lambda c: c["norm"].pop("eps"), lambda c: c["layers"][0]["mixer"].pop("kv_heads"),
+    lambda c: c["layers"][0]["mixer"].update(kv_heads=4), lambda c: c["layers"][0]["mixer"].pop("scale"), lambda c: c["layers"][0]["mixer"]["mask"].update(size=0),
+    lambda c: c["layers"][0]["mixer"]["rot"].update(dims=7), lambda c: c["layers"][0]["mixer"]["rot"].update(dims=40), lambda c: c["layers"][0]["mixer"]["rot"].update(scaling={"factor": 2.0}),
+    lambda c: c["layers"][1]["mixer"].pop("conv"), lambda c: c["layers"][1]["mixer"].update(conv=0), lambda c: c["layers"][1]["mixer"].update(kv_heads=3),
+    lambda c: c["layers"][2]["mixer"].update(kv_from=1), lambda c: c["layers"][2]["mixer"].update(kv_from=2), lambda c: c["layers"][2]["mixer"].update(kv_from=3),
+    lambda c: c["layers"][2]["mixer"].update(kv_from=-1), lambda c: c["layers"][2]["mixer"].update(dim=30), lambda c: c["layers"][2]["mixer"]["rot"].update(base=5.0),
+    lambda c: c["layers"][3]["mixer"].pop("q_rank"), lambda c: c["layers"][3]["mixer"].update(q_rank=0), lambda c: c["layers"][3]["mixer"]["rot"].update(dims=10),
+    lambda c: c["layers"][3]["mixer"]["mask"].pop("size"), lambda c: c["layers"][0].update(type="mamba"), lambda c: c["layers"][0]["mlp"].update(kind="moe")])
+def test_unusable_tarudra_configurations_are_refused(pkg, break_it):
+    c = lc.sandwich_ln([lc.grouped_attn(mlp=lc.dense()), lc.delta(), lc.grouped_attn(source=0), lc.latent2()])
+    pkg.layered_model.parse_config(c)
+    break_it(c)
+    with pytest.raises(pkg.layered_model.ConfigError):
+        pkg.layered_model.parse_config(c)
+
+
+def test_create_refuses_unusable_delta_rules_and_shared_keys(pkg):
+    hb, parse = pkg.hip_backend, pkg.layered_model.parse_config
+
+    def status(cfg, layer=0, **change):
+        p = parse(cfg)
+        for k, v in change.items():
+            setattr(p.layers[layer], k, v)
+        with pytest.raises(pkg.BackendError) as ei:
+            hb.HipGpuInference.from_layered(pkg.LayeredModel(p, {}), 16)
+        return ei.value.variant
+    two = lc.sandwich_ln([lc.grouped_attn(), lc.grouped_attn(source=0)])
+    assert status(lc.sandwich_ln([lc.delta(taps=65)])) == "Unsupported"
+    assert status(lc.sandwich_ln([lc.delta()]), kv_heads=3) == "InvalidArgument"
+    assert status(lc.sandwich_ln([lc.delta()]), taps=0) == "InvalidArgument"
+    assert status(lc.sandwich_ln([lc.grouped_attn(heads=1, kv_heads=1, dim=520)])) == "Unsupported"
+    assert status(two, 1, kv_from=2) == "InvalidArgument" and status(two, 1, kv_from=9) == "InvalidArgument" and status(two, 1, dim=16) == "InvalidArgument"
+    assert status(lc.prenorm([lc.gated()]), sink_one=1) == "Unsupported" and status(lc.prenorm([lc.gated(), lc.gated()]), 1, kv_from=1) == "Unsupported"
+    assert status(lc.sandwich_ln([lc.latent2()]), rot_form=2) == "Unsupported" and status(lc.sandwich_ln([lc.latent2()]), gate_form=2) == "Unsupported"
+    assert status(lc.sandwich_ln([lc.grouped_attn(mlp=lc.dense())]), ff_kind=2, experts=2, top=1) == "Unsupported"
