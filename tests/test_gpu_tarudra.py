@@ -46,7 +46,7 @@ CASES = {
     "shared keys, narrower window": dict(layers=TWO(window=11)),
     "shared keys, no window": dict(layers=TWO(window=0)),
     "shared keys, other scale": dict(layers=TWO(scale=0.7)),
-    "shared keys, two readers": dict(layers=[D(), G(heads=4, kv_heads=4, dim=64, vdim=48), G(4, 4, 64, 48, source=1), L(), G(4, 4, 64, 48, window=5, source=1)]),
+    "shared keys, two readers": dict(layers=[D(), G(heads=4, kv_heads=4, dim=64, vdim=40), G(4, 4, 64, 40, source=1), L(), G(4, 4, 64, 40, window=5, source=1)]),
     "latent": dict(layers=[L()]),
     "latent, no window": dict(layers=[L(window=0)]),
     "latent, no rotation": dict(layers=[L(rotate=False)]),
