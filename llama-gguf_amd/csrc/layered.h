@@ -1,6 +1,6 @@
 // layered.h — models whose layers are described one by one (lgh_layer_desc: a mixer and an optional feed-forward), on the engine's own
 // context, step function and graphs (internal).  Kernels: linear_bf16.hip (matrix products), latent_attention.hip, tied_attention.hip,
-// gated_attention.hip, mlstm.hip, gla.hip, glru.hip, moe_route.hip (routing of the experts), layered_misc.hip (embedding, norms, residual updates); layered.hip assembles them.
+// gated_attention.hip, mlstm.hip, gla.hip, glru.hip, delta.hip, moe_route.hip (routing of the experts), layered_misc.hip (embedding, norms, residual updates); layered.hip assembles them.
 #pragma once
 
 #include "common.h"
